@@ -18,6 +18,9 @@ LIB = PKG / "libmi355llama.so"
 OBJ_DIR = PKG / "csrc" / "_obj"
 SOURCES = ["generic.hip", "gemv.hip", "int8.hip", "int8_gemm.hip", "attention.hip", "engine.hip", "gptq.hip", "fused_step.hip", "fused_step_ring.hip", "fused_step_wide.hip", "tp_comm.hip", "gemm.hip", "flash_prefill.hip", "sample.hip"]
 ARCH = "gfx950"
+# hipcc -O3 turns ordinary float code into packed-f32 instructions, some forms of which have given wrong results on these
+# machines; the host pass says it does not know the feature, which is harmless
+NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _hipcc() -> str:
@@ -38,7 +41,7 @@ def build(force: bool = False, verbose: bool = True) -> Path:
     hipcc = _hipcc()
     OBJ_DIR.mkdir(exist_ok=True)
     headers = [CSRC / "common.h", CSRC / "fused_step_common.h", CSRC / "gemm_fuse.h", PKG.parent / "include" / "mi355_llama.h"]
-    flags = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function"]
+    flags = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", *NO_PACKED_F32]
 
     def compile_one(name: str):
         src = CSRC / name

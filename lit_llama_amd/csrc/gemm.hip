@@ -725,7 +725,7 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
             }
         };
         auto apply = [&]() {  // end of a group: tabc = this group's pairs, tabn = the next group's
-            // two FMAs per output element, issued as v_pk_fma_f32 on register pairs (the VALU, not the matrix pipe, bounds
+            // two FMAs per output element on register pairs (the VALU, not the matrix pipe, bounds
             // the grouped kernel: 64-token blocks halve the MFMAs a weight conversion is amortised over)
             f32x2 ds[kTPW][2], szp[kTPW][2];
 #pragma unroll

@@ -69,6 +69,11 @@ constexpr size_t kSplitBudget = (size_t)32 << 20;
 constexpr int kMaxSplit = 8;
 
 // ---- 1. rows: f16 operand, absmax over the sub-threshold entries, outlier column mask
+__global__ void i8_clear_mask_kernel(unsigned* mask, int n) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) mask[i] = 0u;
+}
+
 __global__ __launch_bounds__(256) void i8_stage_kernel(const void* x, int x_dtype, int64_t ldx, const void* norm_scale,
                                                        int norm_dtype, float eps, float threshold, int K, int Kp, f16_t* xh,
                                                        float* sca, unsigned* mask) {
@@ -519,7 +524,9 @@ extern "C" int mi355_linear_int8_gemm(const mi355_int8_args* a, void* workspace,
                (size_t)2 * ksplit * a->M * ldp * 4 <= kSplitBudget)
             ksplit *= 2;
     }
-    MI355_HIP(hipMemsetAsync(mask, 0, (size_t)kp / 8, s));
+    // (a kernel, not hipMemsetAsync: a caller may capture this launch, and memset nodes have replayed wrongly)
+    hipLaunchKernelGGL(i8_clear_mask_kernel, dim3((kp / 32 + 255) / 256), dim3(256), 0, s, mask, kp / 32);
+    MI355_LAUNCH_CHECK();
     hipLaunchKernelGGL(i8_stage_kernel, dim3(a->M), dim3(256), 0, s, a->x, a->x_dtype, a->ldx, a->norm_scale, a->norm_dtype, a->eps,
                        a->threshold, a->K, kp, xh, sca, mask);
     MI355_LAUNCH_CHECK();

@@ -13,6 +13,9 @@
 //
 // Buffers are fine-grained (uncached) device memory shared through HIP IPC; stores / loads are system-scope relaxed
 // atomics (sc0 sc1).  Every spin is bounded by wall-clock time; a time-out raises the abort word.
+#include <mutex>
+#include <vector>
+
 #include "common.h"
 
 namespace {
@@ -147,9 +150,40 @@ extern "C" size_t mi355_tp_comm_bytes(int world, int slot_floats) {
     return (size_t)3 * world * slot_floats * sizeof(u64);  // two parity planes for the all-reduces + the arg-max plane
 }
 
+// Uncached memory a kernel has read must stay mapped until the process ends (ordinary allocations placed over a freed range
+// have read stale values), so a freed buffer goes to a list and serves the next request of its device and size.
+namespace {
+struct ParkedBuffer {
+    void* p;
+    size_t bytes;
+    int device;
+    bool parked;
+};
+std::mutex g_buffers_lock;
+std::vector<ParkedBuffer> g_buffers;
+}  // namespace
+
 extern "C" int mi355_tp_buffer_alloc(size_t bytes, void** out) {
     MI355_CHECK_ARG(out != nullptr && bytes > 0, MI355_E_ARG, "tp_buffer_alloc: bad argument");
     void* p = nullptr;
+    int device = 0;
+    MI355_HIP(hipGetDevice(&device));
+    {
+        std::lock_guard<std::mutex> lock(g_buffers_lock);
+        for (ParkedBuffer& b : g_buffers)
+            if (b.parked && b.bytes == bytes && b.device == device) {
+                b.parked = false;
+                p = b.p;
+                break;
+            }
+    }
+    if (p != nullptr) {
+        MI355_HIP(hipDeviceSynchronize());  // (work of the previous owner)
+        MI355_HIP(hipMemset(p, 0, bytes));
+        MI355_HIP(hipDeviceSynchronize());
+        *out = p;
+        return 0;
+    }
     // fine-grained (uncached) device memory: what a peer writes over xGMI must be seen by a kernel that is already
     // running here (coarse-grained allocations are only coherent at kernel boundaries)
     hipError_t e = hipExtMallocWithFlags(&p, bytes, hipDeviceMallocUncached);
@@ -161,13 +195,24 @@ extern "C" int mi355_tp_buffer_alloc(size_t bytes, void** out) {
                     hipGetErrorString(e));
     MI355_HIP(hipMemset(p, 0, bytes));
     MI355_HIP(hipDeviceSynchronize());
+    {
+        std::lock_guard<std::mutex> lock(g_buffers_lock);
+        g_buffers.push_back({p, bytes, device, false});
+    }
     *out = p;
     return 0;
 }
 
 extern "C" int mi355_tp_buffer_free(void* p) {
-    if (p != nullptr) MI355_HIP(hipFree(p));
-    return 0;
+    if (p == nullptr) return 0;
+    std::lock_guard<std::mutex> lock(g_buffers_lock);
+    for (ParkedBuffer& b : g_buffers)
+        if (b.p == p && !b.parked) {
+            b.parked = true;
+            return 0;
+        }
+    mi355_set_error("tp_buffer_free: not a live buffer of mi355_tp_buffer_alloc");
+    return MI355_E_ARG;
 }
 
 extern "C" int mi355_ipc_export(void* dev_ptr, void* handle64) {
