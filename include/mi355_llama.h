@@ -35,6 +35,8 @@ enum { MI355_E_ARG = -1, MI355_E_SHAPE = -2, MI355_E_DTYPE = -3, MI355_E_STATE =
 enum { MI355_W_Q4 = 0, MI355_W_BF16 = 1, MI355_W_I8 = 2 };
 /* epilogues of the fast linear */
 enum { MI355_EPI_STORE = 0, MI355_EPI_ACCUM = 1, MI355_EPI_SWIGLU = 2 };
+/* bits of mi355_linear_args.flags: STORE writes max(y, 0)^2 */
+enum { MI355_LF_RELU2 = 1 };
 
 typedef void* mi355_stream_t; /* hipStream_t */
 
@@ -122,14 +124,14 @@ typedef struct mi355_linear_args {
     int32_t waves;      /* waves per workgroup (split of K) */
     int32_t grid;       /* workgroups (persistent loop over tiles) */
     int32_t prefetch;   /* accepted, ignored: one ring depth per format (4 units Q4, 2 units bf16) */
-    int32_t flags;      /* reserved, pass 0 (a retired tuning knob) */
+    int32_t flags;      /* MI355_LF_* bits, or 0 */
     /* activations given as split-attention partial records instead of x (x may be NULL): the prologue combines
      * them (K = attn_heads * attn_hs); layout as written by mi355_attention with n_split = attn_splits.  M = 1 */
     const float* attn_partials;
     int32_t attn_splits;
     int32_t attn_heads;
     int32_t attn_hs;
-    int32_t reserved1;
+    float alpha;        /* factor of the product, in front of the epilogue; 0 is read as 1 */
     /* optional profiling aid: uint64 [grid][8] wall-clock stamps (100 MHz) written by wave 0 of every workgroup:
      * 0 entry, 1 ring issued, 2 activations staged, 3 first tile's loop done, 4 first epilogue done, 5 exit */
     uint64_t* debug_stamps;
@@ -611,6 +613,151 @@ int mi355_tp_argmax(const mi355_tp_comm* c, const float* logits_local, int v_loc
 /* sizeof() of the ABI structs, for binding self-checks: 0 linear_args, 1 attn_args, 2 int8_args, 3 weight,
  * 4 layer, 5 model, 6 fused_step_args, 7 tp_comm; -1 for an unknown index */
 int mi355_sizeof(int which);
+
+/* ------------------------------------------------------------------------------------------
+ * Layered hybrid models: window attention, gated delta rule, gated linear attention.
+ *
+ * A step works on the packed rows of a batch: sequence s owns rows row0[s] .. row0[s] + count[s] - 1, its first row sits at
+ * position pos[s], and what it carries from step to step lies in slot slot[s] of every layer's cache / state.
+ * ---------------------------------------------------------------------------------------- */
+typedef struct mi355_seq_batch {
+    int32_t rows;          /* rows of the step */
+    int32_t seqs;
+    int32_t max_count;     /* largest count[] (1: a decode step) */
+    int32_t reserved0;
+    const int32_t* row0;   /* device [seqs] */
+    const int32_t* count;  /* device [seqs] */
+    const int32_t* slot;   /* device [seqs] */
+    const int32_t* pos;    /* device [seqs] */
+} mi355_seq_batch;
+
+/* Causal attention over a sliding window with grouped key / value heads, partial interleaved rotation and a sigmoid gate per
+ * head.  Row i of a sequence sees rows j with 0 <= i - j < window.  The cache of a slot is a ring of `ring` rows per key head
+ * (position p in row p % ring; ring >= window or >= the longest sequence). */
+typedef struct mi355_window_attn_args {
+    void* proj;            /* [rows, ld]: q, k, v, gate columns; q and k are rotated IN PLACE by a prompt step */
+    int64_t ld;
+    int32_t dtype;         /* of proj, rings and y: F32 or BF16 */
+    int32_t heads, kv_heads, dim, vdim;
+    int32_t off_q, off_k, off_v, off_g; /* first columns; off_g < 0: no gate */
+    float scale;
+    int32_t window, ring;
+    int32_t rot_dims;      /* 0: no rotation */
+    const double* inv_freq; /* device [rot_dims / 2]: pair (2i, 2i + 1) turns by position * inv_freq[i] */
+    void* kring;           /* [slots][kv_heads][ring][dim] */
+    void* vring;           /* [slots][kv_heads][ring][vdim] */
+    void* y;               /* [rows, ldy], head h at column h * vdim */
+    int64_t ldy;
+    float* partials;       /* scratch of a split decode step, or NULL */
+    uint64_t partials_bytes;
+    int32_t path;          /* 0: by shape; 1: one workgroup per row; 2: matrix-core tiles (bf16 prompts) */
+    int32_t reserved0;
+} mi355_window_attn_args;
+
+int mi355_window_attention(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
+
+/* Linear recurrences over a state S [dim, vdim] per head, kept in f32 [slots][heads][dim][vdim]:
+ *   kind MI355_REC_DELTA  gated delta rule: short causal convolutions + SiLU on q, k, v; unit q, k; S = g S, u = beta (v - S^T k),
+ *                         S += k u^T, o = S^T q with g = exp(-exp(A_log) softplus(a + dt_bias)), beta = sigmoid(b)
+ *   kind MI355_REC_GLA    S = diag(alpha) S + k v^T, o = S^T q with alpha = sigmoid(a2 a1 + a2_bias)^(1 / tau) per key channel
+ * then per head o / rms(o) * head_norm * silu(g). */
+enum { MI355_REC_DELTA = 0, MI355_REC_GLA = 1 };
+typedef struct mi355_recurrent_args {
+    int32_t kind;
+    int32_t dtype;         /* of proj, conv_ring and y */
+    const void* proj;      /* [rows, ld] */
+    int64_t ld;
+    int32_t heads, kv_heads, dim, vdim;
+    int32_t off_q, off_k, off_v, off_g, off_a, off_b; /* off_a: DELTA decay input [heads], GLA low-rank input [rank]; off_b: DELTA only */
+    float q_scale;         /* dim^-1/2 */
+    float eps;             /* of the output norm */
+    int32_t taps;          /* DELTA: convolution taps */
+    int32_t rank;          /* GLA */
+    float inv_tau;         /* GLA */
+    float unit_eps;        /* DELTA */
+    const float* conv_q;   /* [kv_heads * dim][taps], last tap = the current row */
+    const float* conv_k;
+    const float* conv_v;   /* [heads * vdim][taps] */
+    const float* a_log;    /* [heads] */
+    const float* dt_bias;  /* [heads] */
+    const float* a2;       /* [heads * dim][rank] */
+    const float* a2_bias;  /* [heads * dim] */
+    const float* head_norm; /* [vdim] */
+    float* state;          /* [slots][heads][dim][vdim] */
+    void* conv_ring;       /* [slots][taps][2 * kv_heads * dim + heads * vdim]: raw q | k | v inputs, position p in row p % taps */
+    void* y;               /* [rows, ldy], head h at column h * vdim */
+    int64_t ldy;
+    float* scratch;        /* chunked prompt steps, or NULL */
+    uint64_t scratch_bytes;
+    int32_t path;          /* 0: by shape; 1: row by row; 2: chunks */
+    int32_t reserved0;
+} mi355_recurrent_args;
+
+int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
+/* scratch bytes a chunked prompt step of `rows` rows in `seqs` sequences takes; 0: the shape runs row by row */
+size_t mi355_recurrent_scratch_bytes(int kind, int rows, int seqs, int heads, int kv_heads, int dim, int vdim);
+
+/* A weight of a hybrid model: BF16 stream (mi355_bf16_repack, R = 1) of a bf16 model, row-major f32 of an f32 model */
+typedef struct mi355_proj {
+    const void* w;
+    int32_t N, K;
+} mi355_proj;
+
+enum { MI355_MIX_ATTENTION = 0, MI355_MIX_DELTA = 1, MI355_MIX_GLA = 2 };
+/* one RUN of a layer (a looped layer appears once per pass: same weights, its own cache / state) */
+typedef struct mi355_hybrid_layer {
+    int32_t mixer;         /* MI355_MIX_* */
+    int32_t mlp;           /* != 0: a squared-ReLU feed-forward follows */
+    const void* norm1;     /* [width] of norm_dtype */
+    const void* norm2;
+    mi355_proj in;         /* every projection that reads the normalised row, stacked */
+    mi355_proj out;        /* heads * vdim -> width */
+    mi355_proj up, down;
+    mi355_window_attn_args attn;   /* as the mixer's kernels take them; proj / y / scratch are filled in per step */
+    mi355_recurrent_args rec;
+} mi355_hybrid_layer;
+
+typedef struct mi355_hybrid_model {
+    int32_t n_runs;
+    int32_t dtype;         /* F32 or BF16: weights, projections, caches */
+    int32_t norm_dtype;
+    int32_t width;
+    int32_t ldx;           /* row pitch of x (width padded to 16; the padding stays zero) */
+    int32_t vocab;
+    int32_t max_rows;      /* rows the scratch buffers hold */
+    int32_t ld_logits;
+    float eps;
+    float residual_mult;
+    const void* embed;     /* [vocab, width] of dtype */
+    const void* final_norm;
+    mi355_proj head;
+    const mi355_hybrid_layer* layers;
+    float* x;              /* [max_rows, ldx] residual stream */
+    float* xw;             /* [max_rows, ldx] rows whose logits are wanted */
+    float* xn;             /* [max_rows, ldx] f32 models: normalised rows */
+    void* proj;            /* [max_rows, widest in.N] of dtype */
+    void* att;             /* [max_rows, widest out.K padded to 16] of dtype */
+    void* hid;             /* [max_rows, widest up.N] of dtype */
+    float* tmp;            /* [max_rows, ldx] f32 models: a product in front of its residual */
+    int64_t ld_att;
+    void* gemm_ws;
+    uint64_t gemm_ws_bytes;
+    float* partials;
+    uint64_t partials_bytes;
+    float* rec_scratch;
+    uint64_t rec_scratch_bytes;
+} mi355_hybrid_model;
+
+/* embedding, every layer run, and the logits (f32 [n_want, ld_logits]) of the rows want[0 .. n_want) (device; NULL: all rows).
+ * run_end < n_runs stops behind that many runs without logits (x holds the residual stream). */
+int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq_batch* b, const int32_t* tokens, const int32_t* want,
+                         int n_want, float* logits, int run_end, mi355_stream_t stream);
+/* zero the state of `n` slots (device list) in every recurrent run */
+int mi355_hybrid_reset_slots(const mi355_hybrid_model* m, const int32_t* slots, int n, mi355_stream_t stream);
+/* greedy end of a decode step, one row per sequence: next[b] = tokens[b] = argmax(logits[b]), out[b * ld_out + pos[b] + 1] = it
+ * (out may be NULL), pos[b] += 1 */
+int mi355_argmax_advance_rows(const float* logits, int64_t ld, int vocab, int seqs, int32_t* next, int32_t* tokens, int32_t* pos,
+                              int32_t* out, int64_t ld_out, mi355_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -15,8 +15,12 @@ from pathlib import Path
 PKG = Path(__file__).resolve().parent
 CSRC = PKG / "csrc"
 LIB = PKG / "libmi355llama.so"
+CORE_LIB = PKG / "libmi355core.so"
 OBJ_DIR = PKG / "csrc" / "_obj"
-SOURCES = ["generic.hip", "gemv.hip", "int8.hip", "int8_gemm.hip", "attention.hip", "engine.hip", "gptq.hip", "fused_step.hip", "fused_step_ring.hip", "fused_step_wide.hip", "tp_comm.hip", "gemm.hip", "flash_prefill.hip", "sample.hip"]
+# what a layered hybrid model runs on; linked alone into CORE_LIB where only such a model is served
+CORE_SOURCES = ["generic.hip", "gemv.hip", "gemm.hip", "sample.hip", "graph.hip", "window_attention.hip", "recurrent.hip", "hybrid.hip"]
+SOURCES = CORE_SOURCES + ["int8.hip", "int8_gemm.hip", "attention.hip", "engine.hip", "gptq.hip", "fused_step.hip", "fused_step_ring.hip",
+                          "fused_step_wide.hip", "tp_comm.hip", "flash_prefill.hip"]
 ARCH = "gfx950"
 # hipcc -O3 turns ordinary float code into packed-f32 instructions, some forms of which have given wrong results on these
 # machines; the host pass says it does not know the feature, which is harmless
@@ -37,7 +41,13 @@ def _stale(target: Path, deps) -> bool:
     return any(Path(d).stat().st_mtime > t for d in deps)
 
 
-def build(force: bool = False, verbose: bool = True) -> Path:
+def build_core(force: bool = False, verbose: bool = True) -> Path:
+    """The part of the library that a layered hybrid model needs (a fresh checkout that serves one compiles no more)."""
+    return build(force, verbose, CORE_SOURCES, CORE_LIB)
+
+
+def build(force: bool = False, verbose: bool = True, sources=None, lib: Path = LIB) -> Path:
+    sources = SOURCES if sources is None else sources
     hipcc = _hipcc()
     OBJ_DIR.mkdir(exist_ok=True)
     headers = [CSRC / "common.h", CSRC / "fused_step_common.h", CSRC / "gemm_fuse.h", PKG.parent / "include" / "mi355_llama.h"]
@@ -67,20 +77,20 @@ def build(force: bool = False, verbose: bool = True) -> Path:
             compiled.append(name)
         return out
 
-    with ThreadPoolExecutor(max_workers=min(len(SOURCES), os.cpu_count() or 4)) as ex:
-        objs = list(ex.map(compile_tracked, SOURCES))
-    relink = force or _stale(LIB, objs)
+    with ThreadPoolExecutor(max_workers=min(len(sources), os.cpu_count() or 4)) as ex:
+        objs = list(ex.map(compile_tracked, sources))
+    relink = force or _stale(lib, objs)
     if verbose:  # say what this call did: an up-to-date tree compiles nothing, and the caller should see that
-        print(f"[build] {len(SOURCES)} sources for {ARCH}: compiled {sorted(compiled) if compiled else 'none (objects up to date)'}; "
-              f"{'linking' if relink else 'library up to date:'} {LIB}", file=sys.stderr)
+        print(f"[build] {len(sources)} sources for {ARCH}: compiled {sorted(compiled) if compiled else 'none (objects up to date)'}; "
+              f"{'linking' if relink else 'library up to date:'} {lib}", file=sys.stderr)
     if relink:
-        cmd = [hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", str(LIB), *map(str, objs)]
+        cmd = [hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", str(lib), *map(str, objs)]
         if verbose:
             print(" ".join(cmd), file=sys.stderr)
         r = subprocess.run(cmd, capture_output=True, text=True)
         if r.returncode != 0:
             raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
-    return LIB
+    return lib
 
 
 if __name__ == "__main__":

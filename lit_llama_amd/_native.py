@@ -14,10 +14,12 @@ import torch
 
 _PKG = Path(__file__).resolve().parent
 LIB_PATH = _PKG / "libmi355llama.so"
+CORE_LIB_PATH = _PKG / "libmi355core.so"  # the part a layered hybrid model needs (_build.build_core)
 
 F32, BF16, F16 = 0, 1, 2
 W_Q4, W_BF16, W_I8 = 0, 1, 2
 EPI_STORE, EPI_ACCUM, EPI_SWIGLU = 0, 1, 2
+LF_RELU2 = 1
 
 _DTYPE_CODE = {torch.float32: F32, torch.bfloat16: BF16, torch.float16: F16}
 
@@ -38,7 +40,7 @@ class LinearArgs(C.Structure):
         ("y", c_void_p), ("y_dtype", c_int32), ("group_cols", c_int32), ("ldy", c_int64),
         ("waves", c_int32), ("grid", c_int32), ("prefetch", c_int32), ("flags", c_int32),
         ("attn_partials", c_void_p), ("attn_splits", c_int32), ("attn_heads", c_int32), ("attn_hs", c_int32),
-        ("reserved1", c_int32), ("debug_stamps", c_void_p),
+        ("alpha", c_float), ("debug_stamps", c_void_p),
     ]
 
 
@@ -138,6 +140,61 @@ class TpComm(C.Structure):
     ]
 
 
+class SeqBatch(C.Structure):
+    _fields_ = [
+        ("rows", c_int32), ("seqs", c_int32), ("max_count", c_int32), ("reserved0", c_int32),
+        ("row0", c_void_p), ("count", c_void_p), ("slot", c_void_p), ("pos", c_void_p),
+    ]
+
+
+class WindowAttnArgs(C.Structure):
+    _fields_ = [
+        ("proj", c_void_p), ("ld", c_int64), ("dtype", c_int32),
+        ("heads", c_int32), ("kv_heads", c_int32), ("dim", c_int32), ("vdim", c_int32),
+        ("off_q", c_int32), ("off_k", c_int32), ("off_v", c_int32), ("off_g", c_int32),
+        ("scale", c_float), ("window", c_int32), ("ring", c_int32), ("rot_dims", c_int32), ("inv_freq", c_void_p),
+        ("kring", c_void_p), ("vring", c_void_p), ("y", c_void_p), ("ldy", c_int64),
+        ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("path", c_int32), ("reserved0", c_int32),
+    ]
+
+
+class RecurrentArgs(C.Structure):
+    _fields_ = [
+        ("kind", c_int32), ("dtype", c_int32), ("proj", c_void_p), ("ld", c_int64),
+        ("heads", c_int32), ("kv_heads", c_int32), ("dim", c_int32), ("vdim", c_int32),
+        ("off_q", c_int32), ("off_k", c_int32), ("off_v", c_int32), ("off_g", c_int32), ("off_a", c_int32), ("off_b", c_int32),
+        ("q_scale", c_float), ("eps", c_float), ("taps", c_int32), ("rank", c_int32), ("inv_tau", c_float), ("unit_eps", c_float),
+        ("conv_q", c_void_p), ("conv_k", c_void_p), ("conv_v", c_void_p), ("a_log", c_void_p), ("dt_bias", c_void_p),
+        ("a2", c_void_p), ("a2_bias", c_void_p), ("head_norm", c_void_p), ("state", c_void_p), ("conv_ring", c_void_p),
+        ("y", c_void_p), ("ldy", c_int64), ("scratch", c_void_p), ("scratch_bytes", C.c_uint64),
+        ("path", c_int32), ("reserved0", c_int32),
+    ]
+
+
+class Proj(C.Structure):
+    _fields_ = [("w", c_void_p), ("N", c_int32), ("K", c_int32)]
+
+
+class HybridLayer(C.Structure):
+    _fields_ = [
+        ("mixer", c_int32), ("mlp", c_int32), ("norm1", c_void_p), ("norm2", c_void_p),
+        ("in", Proj), ("out", Proj), ("up", Proj), ("down", Proj),
+        ("attn", WindowAttnArgs), ("rec", RecurrentArgs),
+    ]
+
+
+class HybridModel(C.Structure):
+    _fields_ = [
+        ("n_runs", c_int32), ("dtype", c_int32), ("norm_dtype", c_int32), ("width", c_int32),
+        ("ldx", c_int32), ("vocab", c_int32), ("max_rows", c_int32), ("ld_logits", c_int32),
+        ("eps", c_float), ("residual_mult", c_float),
+        ("embed", c_void_p), ("final_norm", c_void_p), ("head", Proj), ("layers", C.POINTER(HybridLayer)),
+        ("x", c_void_p), ("xw", c_void_p), ("xn", c_void_p), ("proj", c_void_p), ("att", c_void_p), ("hid", c_void_p),
+        ("tmp", c_void_p), ("ld_att", c_int64), ("gemm_ws", c_void_p), ("gemm_ws_bytes", C.c_uint64),
+        ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("rec_scratch", c_void_p), ("rec_scratch_bytes", C.c_uint64),
+    ]
+
+
 # name -> (restype, argtypes); must list every function declared in include/mi355_llama.h
 PROTOTYPES = {
     "mi355_version": (c_int, []),
@@ -203,12 +260,19 @@ PROTOTYPES = {
     "mi355_sizeof": (c_int, [c_int]),
     "mi355_linear_max_rows": (c_int, [c_int, c_int, c_int, c_int]),
     "mi355_debug_time_next_launch": (c_int, [c_void_p, c_void_p]),
+    "mi355_window_attention": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
+    "mi355_recurrent": (c_int, [C.POINTER(RecurrentArgs), C.POINTER(SeqBatch), c_void_p]),
+    "mi355_recurrent_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mi355_hybrid_forward": (c_int, [C.POINTER(HybridModel), C.POINTER(SeqBatch), c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p]),
+    "mi355_hybrid_reset_slots": (c_int, [C.POINTER(HybridModel), c_void_p, c_int, c_void_p]),
+    "mi355_argmax_advance_rows": (c_int, [c_void_p, c_int64, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_void_p]),
     "mi355_gptq_row_params": (c_int, [c_void_p, c_int64, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p]),
     "mi355_gptq_block": (c_int, [c_void_p, c_int64, c_int, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_int64,
                                  c_int64, c_int, c_void_p, c_void_p, c_void_p, c_int64, c_void_p]),
 }
 
-ABI_STRUCTS = [LinearArgs, AttnArgs, Int8Args, Weight, Layer, Model, FusedStepArgs, TpComm]
+ABI_STRUCTS = [LinearArgs, AttnArgs, Int8Args, Weight, Layer, Model, FusedStepArgs, TpComm,
+               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel]
 
 _lib: Optional[C.CDLL] = None
 
@@ -225,27 +289,36 @@ def lib() -> C.CDLL:
     global _lib
     if _lib is None:
         path = Path(os.environ.get("MI355_LLAMA_LIB", LIB_PATH))
+        if not path.exists() and CORE_LIB_PATH.exists():
+            path = CORE_LIB_PATH  # (a call outside the core then fails on its missing symbol)
         if not path.exists():
             raise NativeError(
                 f"{path} not found: build it with `python -c 'import __graft_entry__ as g; g.build()'` "
                 "(hipcc --offload-arch=gfx950).  There is no CPU fallback for the hot path."
             )
-        _preload_hip_runtime()
-        try:
-            handle = C.CDLL(str(path))
-        except OSError as e:  # pragma: no cover
-            raise NativeError(f"cannot load {path}: {e}") from e
-        for name, (res, args) in PROTOTYPES.items():
-            fn = getattr(handle, name)  # AttributeError if the .so is stale
-            fn.restype = res
-            fn.argtypes = args
-        if handle.mi355_version() != 1:
-            raise NativeError("libmi355llama ABI version mismatch; rebuild")
-        for i, st in enumerate(ABI_STRUCTS):
-            if handle.mi355_sizeof(i) != C.sizeof(st):
-                raise NativeError(f"ABI struct {st.__name__}: C sizeof {handle.mi355_sizeof(i)} != ctypes {C.sizeof(st)}")
-        _lib = handle
+        _lib = _bind(path)
     return _lib
+
+
+def _bind(path: Path) -> C.CDLL:
+    _preload_hip_runtime()
+    try:
+        handle = C.CDLL(str(path))
+    except OSError as e:  # pragma: no cover
+        raise NativeError(f"cannot load {path}: {e}") from e
+    core_only = path.name == CORE_LIB_PATH.name
+    for name, (res, args) in PROTOTYPES.items():
+        if core_only and not hasattr(handle, name):
+            continue
+        fn = getattr(handle, name)  # AttributeError if the .so is stale
+        fn.restype = res
+        fn.argtypes = args
+    if handle.mi355_version() != 1:
+        raise NativeError("libmi355llama ABI version mismatch; rebuild")
+    for i, st in enumerate(ABI_STRUCTS):
+        if handle.mi355_sizeof(i) != C.sizeof(st):
+            raise NativeError(f"ABI struct {st.__name__}: C sizeof {handle.mi355_sizeof(i)} != ctypes {C.sizeof(st)}")
+    return handle
 
 
 E_ARG, E_SHAPE, E_DTYPE, E_STATE = -1, -2, -3, -4  # include/mi355_llama.h MI355_E_*

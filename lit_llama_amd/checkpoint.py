@@ -17,6 +17,7 @@ Host-side plumbing only (file parsing, no arithmetic): nothing here runs on the 
 """
 from __future__ import annotations
 
+import json
 import pickle
 import struct
 import sys
@@ -256,9 +257,62 @@ def _rebuild_from_type(func, new_type, args, state):
     return ret
 
 
+class _Safetensors:
+    """`lazy_load` of a safetensors file: {name: LazyTensor} in file order.  Layout: u64 little-endian header length, that many bytes of
+    JSON (name -> dtype, shape, [begin, end) behind the header), then the bytes; nothing of the file is executed."""
+
+    _DTYPES = {"F64": torch.float64, "F32": torch.float32, "F16": torch.float16, "BF16": torch.bfloat16, "I64": torch.int64,
+               "I32": torch.int32, "I16": torch.int16, "I8": torch.int8, "U8": torch.uint8, "BOOL": torch.bool}
+
+    def __init__(self, fn):
+        self.path = Path(fn)
+        self.bytes_mapped = 0
+        size = self.path.stat().st_size
+        with open(self.path, "rb") as f:
+            n = struct.unpack("<Q", f.read(8))[0]
+            if 8 + n > size:
+                raise ValueError(f"{self.path}: header of {n} bytes in a file of {size}")
+            header = json.loads(f.read(n))
+        self._ranges: Dict[str, Tuple[int, int]] = {}
+        self.sd = OrderedDict()
+        for name, e in header.items():
+            if name == "__metadata__":
+                continue
+            dtype, shape, (lo, hi) = self._DTYPES[e["dtype"]], tuple(e["shape"]), e["data_offsets"]
+            numel, stride = 1, []
+            for d in reversed(shape):
+                stride.insert(0, numel)
+                numel *= d
+            if hi - lo != numel * torch.empty((), dtype=dtype).element_size() or 8 + n + hi > size:
+                raise ValueError(f"{self.path}: bad extent of {name}")
+            self._ranges[name] = (8 + n + lo, hi - lo)
+            self.sd[name] = LazyTensor(_StorageRef(self, name, dtype, numel), 0, shape, tuple(stride))
+
+    def _map(self, key: str, byte_off: int, nbytes: int) -> np.ndarray:
+        start, size = self._ranges[key]
+        if byte_off < 0 or byte_off + nbytes > size:
+            raise ValueError(f"tensor range [{byte_off}, {byte_off + nbytes}) outside {key} ({size} B)")
+        self.bytes_mapped += nbytes
+        if nbytes == 0:
+            return np.empty((0,), dtype=np.uint8)
+        return np.memmap(self.path, dtype=np.uint8, mode="r", offset=start + byte_off, shape=(nbytes,))
+
+    def __enter__(self) -> Any:
+        return self.sd
+
+    def __exit__(self, exc_type, exc_val, exc_tb):
+        return False
+
+
 class lazy_load:
     """Context manager over a `torch.save` checkpoint; yields the unpickled object with LazyTensor leaves.
-    `bytes_mapped` counts the bytes handed out so far (what was actually read from the file)."""
+    `bytes_mapped` counts the bytes handed out so far (what was actually read from the file).  A path that ends in .safetensors is
+    read as such a file (_Safetensors: same interface)."""
+
+    def __new__(cls, fn):
+        if Path(fn).suffix == ".safetensors":
+            return _Safetensors(fn)
+        return super().__new__(cls)
 
     def __init__(self, fn):
         self.path = Path(fn)

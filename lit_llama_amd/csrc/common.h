@@ -169,6 +169,12 @@ __device__ __forceinline__ float group_sum(float v, int lpr) {
     return v;
 }
 
+// max(v, 0)^2
+__device__ __forceinline__ float relu2_f32(float v) {
+    const float r = fmaxf(v, 0.f);
+    return r * r;
+}
+
 // silu(a) * b in f32 (F.silu: a * sigmoid(a))
 __device__ __forceinline__ float swiglu_f32(float a, float b) { return (a / (1.0f + expf(-a))) * b; }
 

@@ -108,6 +108,7 @@ struct GemmParams {
     // by splitk_reduce_kernel; sx then holds [M][ksplit] per-slice operand sums
     int ksplit;
     float* part;
+    int relu2;             // STORE: max(y, 0)^2
     // grouped scales (GRP kernels): gtab[group 0..n_groups][r][tab_ld rows] = bf16 scale | bf16 zero << 16 (row n_groups
     // is all zero), sxt[group][M] = operand sums per group; upg = 128-column units per group (groups of >= 128 columns)
     const uint32_t* gtab;
@@ -164,11 +165,11 @@ __device__ __forceinline__ float ldsz(const void* p, int i, int dtype) {
     return dtype == MI355_F32 ? ((const float*)p)[i] : bf16_to_f32(((const bf16_t*)p)[i]);
 }
 
-// one row per workgroup: xb = bf16(norm_scale * x), rinv = rsqrt(mean(x^2) + eps) (1 without norm), sx[m][s] = sum of xb over
+// one row per workgroup: xb = bf16(norm_scale * x), rinv = alpha rsqrt(mean(x^2) + eps) (alpha without norm), sx[m][s] = sum of xb over
 // K-slice s (ksplit = 1: the whole row)
 __global__ __launch_bounds__(256) void stage_rows_kernel(const void* x, int x_dtype, int64_t ldx, const void* norm_scale,
                                                          int norm_dtype, float eps, int K, int Kp, bf16_t* xb, int64_t ldxb,
-                                                         float* rinv, float* sx, int ksplit) {
+                                                         float* rinv, float* sx, int ksplit, float alpha) {
     __shared__ float red[32];
     const int m = blockIdx.x;
     const int units = Kp >> 7;
@@ -193,7 +194,7 @@ __global__ __launch_bounds__(256) void stage_rows_kernel(const void* x, int x_dt
         if (threadIdx.x == 0) sx[(int64_t)m * ksplit + s] = tot;
     }
     const float tss = block_sum(ss, red);
-    if (threadIdx.x == 0) rinv[m] = norm_scale != nullptr ? rsqrtf(tss / (float)K + eps) : 1.0f;
+    if (threadIdx.x == 0) rinv[m] = norm_scale != nullptr ? rsqrtf(tss / (float)K + eps) * alpha : alpha;
 }
 
 // grouped scales: as stage_rows_kernel, but sxt[grp][m] = sum of xb over the group's input columns.  A wave per group
@@ -252,7 +253,7 @@ __global__ __launch_bounds__(256) void group_table_kernel(const bf16_t* s0, cons
 // y[m][n] (+)= sum over the K-slices, in slice order (deterministic)
 template <int EPI>
 __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, int ksplit, int M, int N, void* y, int y_dtype,
-                                                            int64_t ldy) {
+                                                            int64_t ldy, int relu2) {
     const int64_t n4 = N >> 2;
     for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < (int64_t)M * n4; i += (int64_t)gridDim.x * blockDim.x) {
         const int m = (int)(i / n4), n = (int)(i - (int64_t)m * n4) * 4;
@@ -273,6 +274,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, i
             float* dst = (float*)y + (int64_t)m * ldy + n;
             if constexpr (EPI == MI355_EPI_ACCUM) o = *(const f32x4*)dst;
             for (int s = 0; s < ksplit; ++s) o += *(const f32x4*)(part + ((int64_t)s * M + m) * N + n);
+            if (EPI == MI355_EPI_STORE && relu2) o = f32x4{relu2_f32(o[0]), relu2_f32(o[1]), relu2_f32(o[2]), relu2_f32(o[3])};
             *(f32x4*)dst = o;
         } else {
             bf16_t* dst = (bf16_t*)y + (int64_t)m * ldy + n;
@@ -281,6 +283,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, i
                 for (int r = 0; r < 4; ++r) o[r] = bf16_to_f32(dst[r]);
             }
             for (int s = 0; s < ksplit; ++s) o += *(const f32x4*)(part + ((int64_t)s * M + m) * N + n);
+            if (EPI == MI355_EPI_STORE && relu2) o = f32x4{relu2_f32(o[0]), relu2_f32(o[1]), relu2_f32(o[2]), relu2_f32(o[3])};
             u32x2 pk;
             pk[0] = (uint32_t)bf16_hw(o[0]) | ((uint32_t)bf16_hw(o[1]) << 16);
             pk[1] = (uint32_t)bf16_hw(o[2]) | ((uint32_t)bf16_hw(o[3]) << 16);
@@ -901,6 +904,7 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
                     float* dst = (float*)p.y + (int64_t)m * p.ldy + n;
                     f32x4 o = {v[t][0], v[t][1], v[t][2], v[t][3]};
                     if constexpr (EPI == MI355_EPI_ACCUM) o += *(const f32x4*)dst;
+                    if (!FUSE && EPI == MI355_EPI_STORE && p.relu2) o = f32x4{relu2_f32(o[0]), relu2_f32(o[1]), relu2_f32(o[2]), relu2_f32(o[3])};
                     *(f32x4*)dst = o;
                     if constexpr (FUSE && EPI == MI355_EPI_ACCUM) {
                         if (emit) {  // the next linear's operand: bf16(norm scale * x), as stage_rows_kernel rounds it
@@ -921,6 +925,10 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
                     if constexpr (EPI == MI355_EPI_ACCUM) {
 #pragma unroll
                         for (int r = 0; r < 4; ++r) o[r] += bf16_to_f32(dst[r]);
+                    }
+                    if (!FUSE && EPI == MI355_EPI_STORE && p.relu2) {
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) o[r] = relu2_f32(o[r]);
                     }
                     u32x2 pk;
                     pk[0] = (uint32_t)bf16_hw(o[0]) | ((uint32_t)bf16_hw(o[1]) << 16);
@@ -1006,7 +1014,7 @@ int launch_gemm_w(const GemmParams& p, hipStream_t s) {  // p.n_tiles: 16-row ti
     if (q.ksplit > 1) {
         const int64_t n = (int64_t)p.M * (p.N >> 2);
         const int grid = (int)((n + 255) / 256 < 2048 ? (n + 255) / 256 : 2048);
-        hipLaunchKernelGGL(splitk_reduce_kernel<EPI>, dim3(grid), dim3(256), 0, s, q.part, q.ksplit, p.M, p.N, p.y, p.y_dtype, p.ldy);
+        hipLaunchKernelGGL(splitk_reduce_kernel<EPI>, dim3(grid), dim3(256), 0, s, q.part, q.ksplit, p.M, p.N, p.y, p.y_dtype, p.ldy, p.relu2);
         MI355_LAUNCH_CHECK();
     }
     return 0;
@@ -1252,7 +1260,7 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
         p.tab_ld = tab_ld;
     } else if (!f_in) {
         hipLaunchKernelGGL(stage_rows_kernel, dim3(a->M), dim3(256), 0, s, a->x, a->x_dtype, a->ldx, a->norm_scale, a->norm_dtype,
-                           a->eps, a->K, kp, xb, (int64_t)kp, rinv, sx, ksplit);
+                           a->eps, a->K, kp, xb, (int64_t)kp, rinv, sx, ksplit, a->alpha == 0.f ? 1.f : a->alpha);
         MI355_LAUNCH_CHECK();
     }
     p.w = (const uint8_t*)a->w;
@@ -1271,6 +1279,9 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
     p.zeros = a->zeros;
     p.scales2 = a->scales2;
     p.zeros2 = a->zeros2;
+    p.relu2 = (a->flags & MI355_LF_RELU2) ? 1 : 0;
+    MI355_CHECK_ARG(!p.relu2 || (a->epi == MI355_EPI_STORE && !fused), MI355_E_ARG, "linear_gemm: RELU2 belongs to the plain STORE epilogue");
+    MI355_CHECK_ARG(!(grouped || f_in) || a->alpha == 0.f || a->alpha == 1.f, MI355_E_ARG, "linear_gemm: alpha needs the staging pass of per-row scales");
     p.y = a->y;
     p.ldy = a->ldy;
     p.M = a->M;

@@ -64,6 +64,8 @@ struct GemvParams {
     unsigned long long* dbg;  // optional wall-clock stamps [grid][8]
     float eps;
     // grouped scales (GRP kernels): scales / zeros are [N, n_groups] bf16, one pair per 32 << gq_shift input columns
+    float alpha;    // factor of the product
+    int relu2;      // STORE: max(y, 0)^2
     int n_groups, gq_shift;
     float inv_ng;  // 1 / n_groups (element index -> row without an integer division)
 };
@@ -394,6 +396,7 @@ __device__ __forceinline__ void tile_epilogue(const GemvParams& p, const char* p
                 float out = v[r];
                 if (p.bias != nullptr) out += cvt2(o.bias[r] >> o.sh_sz[r], p.sz_dtype);
                 if (EPI == MI355_EPI_ACCUM) out += cvt2(o.old[r] >> o.sh_y[r], p.y_dtype);
+                if (EPI == MI355_EPI_STORE && p.relu2) out = relu2_f32(out);
                 st2(p.y, (int64_t)e_col * p.ldy + n, p.y_dtype, out);
             }
         }
@@ -575,11 +578,11 @@ __global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const 
     __syncthreads();
     MI355_STAMP(2);
 
-    float rinv = 1.f;
+    float rinv = p.alpha;
     if (p.norm_scale != nullptr && e_owner) {
         float ss = 0.f;
         for (int w = 0; w < W; ++w) ss += wss[w * 16 + e_col];
-        rinv = rsqrtf(ss / (float)p.K + p.eps);
+        rinv = rsqrtf(ss / (float)p.K + p.eps) * p.alpha;
     }
 
     f32x4 acc[R], acc1 = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -1193,6 +1196,9 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
     p.epi = a->epi;
     p.xs_stride = (p.units + 1) * kUnitK * 2 + 16;  // + one all-zero unit (idle ring steps read it)
     p.eps = a->eps;
+    p.alpha = a->alpha == 0.f ? 1.f : a->alpha;
+    p.relu2 = (a->flags & MI355_LF_RELU2) ? 1 : 0;
+    MI355_CHECK_ARG(!p.relu2 || a->epi == MI355_EPI_STORE, MI355_E_ARG, "linear_fast: RELU2 belongs to the STORE epilogue");
     int waves = a->waves > 0 ? a->waves : 8;
     if (waves > 16) waves = 16;
     if ((a->fmt != MI355_W_Q4 || (a->group_cols > 0 && a->group_cols < a->K)) && waves > 8) waves = 8;  // see kMaxThreads

@@ -30,6 +30,12 @@ extern "C" int mi355_sizeof(int which) {
         case 5: return (int)sizeof(mi355_model);
         case 6: return (int)sizeof(mi355_fused_step_args);
         case 7: return (int)sizeof(mi355_tp_comm);
+        case 8: return (int)sizeof(mi355_seq_batch);
+        case 9: return (int)sizeof(mi355_window_attn_args);
+        case 10: return (int)sizeof(mi355_recurrent_args);
+        case 11: return (int)sizeof(mi355_proj);
+        case 12: return (int)sizeof(mi355_hybrid_layer);
+        case 13: return (int)sizeof(mi355_hybrid_model);
         default: return -1;
     }
 }

@@ -1,0 +1,189 @@
+// The forward pass of a layered hybrid model (mi355_hybrid_forward): a host-side walk over the layer runs that enqueues this library's
+// linears (gemv.hip for up to 16 rows, gemm.hip above, the exact f32 kernel for f32 models) and mixers (window_attention.hip,
+// recurrent.hip).  RMSNorm rides in the consuming linear and the residual sum in the producing one; the residual stream is f32.
+#include "common.h"
+
+namespace {
+
+// one row per workgroup; columns width .. ldx - 1 are zero
+__global__ __launch_bounds__(256) void embed_rows_kernel(const int32_t* tokens, const void* wte, int dtype, float* x, int width, int ldx,
+                                                         int vocab) {
+    const int m = blockIdx.x;
+    const int tok = min(max(tokens[m], 0), vocab - 1);
+    for (int k = threadIdx.x; k < ldx; k += 256) x[(int64_t)m * ldx + k] = k < width ? ld_as_f32(wte, (int64_t)tok * width + k, dtype) : 0.f;
+}
+
+__global__ __launch_bounds__(256) void gather_rows_kernel(const float* x, const int32_t* want, float* xw, int ldx) {
+    const int64_t src = (int64_t)want[blockIdx.x] * ldx, dst = (int64_t)blockIdx.x * ldx;
+    for (int k = threadIdx.x; k < ldx; k += 256) xw[dst + k] = x[src + k];
+}
+
+__global__ __launch_bounds__(256) void relu2_kernel(float* h, int64_t n) {
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) h[i] = relu2_f32(h[i]);
+}
+
+// x += alpha * t over rows of the same pitch
+__global__ __launch_bounds__(256) void residual_kernel(float* x, const float* t, float alpha, int64_t n) {
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) x[i] += alpha * t[i];
+}
+
+// grid (seqs, parts)
+__global__ __launch_bounds__(256) void zero_slots_kernel(const int32_t* slots, float* state, int64_t per_slot) {
+    float* s = state + (int64_t)slots[blockIdx.x] * per_slot;
+    for (int64_t i = (int64_t)blockIdx.y * 256 + threadIdx.x; i < per_slot; i += (int64_t)gridDim.y * 256) s[i] = 0.f;
+}
+
+__global__ __launch_bounds__(1024) void argmax_advance_rows_kernel(const float* logits, int64_t ld, int vocab, int32_t* next, int32_t* tokens,
+                                                                   int32_t* pos, int32_t* out, int64_t ld_out) {
+    const int b = blockIdx.x;
+    const int best = block_argmax_first(logits + (int64_t)b * ld, vocab);
+    if (threadIdx.x == 0) {
+        const int p = pos[b];
+        if (next != nullptr) next[b] = best;
+        tokens[b] = best;
+        if (out != nullptr) out[(int64_t)b * ld_out + p + 1] = best;
+        pos[b] = p + 1;
+    }
+}
+
+int ew_blocks(int64_t n) {
+    const int64_t b = (n + 255) / 256;
+    return (int)(b > 4096 ? 4096 : b);
+}
+
+enum { kStore = 0, kRelu2 = 1, kResidual = 2 };
+
+// y[M, N] (+)= alpha * W norm(x).  x f32 with `norm`, or dtype without
+int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int64_t ldx, const void* norm, int what, void* y, int64_t ldy,
+           int y_dtype, int M, hipStream_t s) {
+    if (m->dtype == MI355_F32) {
+        const float* in = (const float*)x;
+        int64_t ld_in = ldx;
+        if (norm != nullptr) {
+            if (int rc = mi355_rmsnorm(x, ldx, norm, m->norm_dtype, m->eps, m->xn, m->ldx, M, w.K, MI355_F32, MI355_F32, s)) return rc;
+            in = m->xn;
+            ld_in = m->ldx;
+        }
+        void* dst = what == kResidual ? (void*)m->tmp : y;
+        const int64_t ld_dst = what == kResidual ? m->ldx : ldy;
+        if (int rc = mi355_linear_dense(in, ld_in, w.w, nullptr, dst, ld_dst, M, w.N, w.K, MI355_F32, s)) return rc;
+        if (what == kRelu2) {  // (ldy = w.N: rows without gaps)
+            hipLaunchKernelGGL(relu2_kernel, dim3(ew_blocks((int64_t)M * ldy)), dim3(256), 0, s, (float*)y, (int64_t)M * ldy);
+            MI355_LAUNCH_CHECK();
+        } else if (what == kResidual) {  // (N = ldx = ldy)
+            hipLaunchKernelGGL(residual_kernel, dim3(ew_blocks((int64_t)M * m->ldx)), dim3(256), 0, s, (float*)y, m->tmp, m->residual_mult,
+                               (int64_t)M * m->ldx);
+            MI355_LAUNCH_CHECK();
+        }
+        return 0;
+    }
+    mi355_linear_args a;
+    memset(&a, 0, sizeof(a));
+    a.fmt = MI355_W_BF16;
+    a.R = 1;
+    a.w = w.w;
+    a.N = w.N;
+    a.K = w.K;
+    a.x_dtype = norm != nullptr ? MI355_F32 : MI355_BF16;
+    a.ldx = ldx;
+    a.norm_scale = norm;
+    a.norm_dtype = m->norm_dtype;
+    a.eps = m->eps;
+    a.epi = what == kResidual ? MI355_EPI_ACCUM : MI355_EPI_STORE;
+    a.flags = what == kRelu2 ? MI355_LF_RELU2 : 0;
+    a.alpha = what == kResidual ? m->residual_mult : 1.f;
+    a.y_dtype = y_dtype;
+    a.ldy = ldy;
+    const int most = mi355_linear_max_rows(MI355_W_BF16, w.K, 1, 0);
+    if (M > 16 || most < 1) {
+        a.x = x;
+        a.y = y;
+        a.M = M;
+        return mi355_linear_gemm(&a, m->gemm_ws, (size_t)m->gemm_ws_bytes, s);
+    }
+    for (int m0 = 0; m0 < M; m0 += most) {
+        a.M = M - m0 < most ? M - m0 : most;
+        a.x = (const char*)x + (int64_t)m0 * ldx * dtype_size(a.x_dtype);
+        a.y = (char*)y + (int64_t)m0 * ldy * dtype_size(y_dtype);
+        if (int rc = mi355_linear_fast(&a, s)) return rc;
+    }
+    return 0;
+}
+
+}  // namespace
+
+extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq_batch* b, const int32_t* tokens, const int32_t* want,
+                                    int n_want, float* logits, int run_end, mi355_stream_t stream) {
+    MI355_CHECK_ARG(m && b && tokens && m->layers && m->x && m->proj && m->att && m->embed, MI355_E_ARG, "hybrid_forward: null argument");
+    MI355_CHECK_ARG(m->dtype == MI355_BF16 || (m->dtype == MI355_F32 && m->xn && m->tmp), MI355_E_DTYPE, "hybrid_forward: bad dtype");
+    const int M = b->rows;
+    MI355_CHECK_ARG(M > 0 && M <= m->max_rows && n_want >= 0 && (want != nullptr ? n_want <= m->max_rows : n_want == 0 || n_want == M),
+                    MI355_E_SHAPE, "hybrid_forward: %d rows (of %d), %d wanted", M, m->max_rows, n_want);
+    MI355_CHECK_ARG(b->max_count > 1 || b->rows == b->seqs, MI355_E_SHAPE, "hybrid_forward: a decode step has one row per sequence");
+    MI355_CHECK_ARG(m->residual_mult != 0.f, MI355_E_ARG, "hybrid_forward: residual_mult is 0");
+    MI355_CHECK_ARG(n_want == 0 || run_end < m->n_runs || (logits && m->final_norm), MI355_E_ARG, "hybrid_forward: nowhere to write logits");
+    hipStream_t s = (hipStream_t)stream;
+    hipLaunchKernelGGL(embed_rows_kernel, dim3(M), dim3(256), 0, s, tokens, m->embed, m->dtype, m->x, m->width, m->ldx, m->vocab);
+    MI355_LAUNCH_CHECK();
+    const int runs = run_end < m->n_runs ? run_end : m->n_runs;
+    for (int r = 0; r < runs; ++r) {
+        const mi355_hybrid_layer& l = m->layers[r];
+        const int64_t ldp = l.in.N;
+        if (int rc = linear(m, l.in, m->x, m->ldx, l.norm1, kStore, m->proj, ldp, m->dtype, M, s)) return rc;
+        if (l.mixer == MI355_MIX_ATTENTION) {
+            mi355_window_attn_args a = l.attn;
+            a.proj = m->proj;
+            a.ld = ldp;
+            a.dtype = m->dtype;
+            a.y = m->att;
+            a.ldy = m->ld_att;
+            a.partials = m->partials;
+            a.partials_bytes = m->partials_bytes;
+            if (int rc = mi355_window_attention(&a, b, stream)) return rc;
+        } else {
+            mi355_recurrent_args a = l.rec;
+            a.proj = m->proj;
+            a.ld = ldp;
+            a.dtype = m->dtype;
+            a.y = m->att;
+            a.ldy = m->ld_att;
+            a.scratch = m->rec_scratch;
+            a.scratch_bytes = m->rec_scratch_bytes;
+            if (int rc = mi355_recurrent(&a, b, stream)) return rc;
+        }
+        if (int rc = linear(m, l.out, m->att, m->ld_att, nullptr, kResidual, m->x, m->ldx, MI355_F32, M, s)) return rc;
+        if (l.mlp) {
+            if (int rc = linear(m, l.up, m->x, m->ldx, l.norm2, kRelu2, m->hid, l.up.N, m->dtype, M, s)) return rc;
+            if (int rc = linear(m, l.down, m->hid, l.up.N, nullptr, kResidual, m->x, m->ldx, MI355_F32, M, s)) return rc;
+        }
+    }
+    if (run_end < m->n_runs || n_want == 0) return 0;
+    const float* xh = m->x;
+    if (want != nullptr) {
+        hipLaunchKernelGGL(gather_rows_kernel, dim3(n_want), dim3(256), 0, s, m->x, want, m->xw, m->ldx);
+        MI355_LAUNCH_CHECK();
+        xh = m->xw;
+    }
+    return linear(m, m->head, xh, m->ldx, m->final_norm, kStore, logits, m->ld_logits, MI355_F32, n_want, s);
+}
+
+extern "C" int mi355_hybrid_reset_slots(const mi355_hybrid_model* m, const int32_t* slots, int n, mi355_stream_t stream) {
+    MI355_CHECK_ARG(m && slots && n > 0 && m->layers, MI355_E_ARG, "hybrid_reset_slots: bad argument");
+    for (int r = 0; r < m->n_runs; ++r) {
+        const mi355_hybrid_layer& l = m->layers[r];
+        if (l.mixer == MI355_MIX_ATTENTION) continue;  // (a ring row is written before it can be seen)
+        const int64_t per = (int64_t)l.rec.heads * l.rec.dim * l.rec.vdim;
+        hipLaunchKernelGGL(zero_slots_kernel, dim3(n, per > 65536 ? 64 : 4), dim3(256), 0, (hipStream_t)stream, slots, l.rec.state, per);
+        MI355_LAUNCH_CHECK();
+    }
+    return 0;
+}
+
+extern "C" int mi355_argmax_advance_rows(const float* logits, int64_t ld, int vocab, int seqs, int32_t* next, int32_t* tokens, int32_t* pos,
+                                         int32_t* out, int64_t ld_out, mi355_stream_t stream) {
+    MI355_CHECK_ARG(logits && tokens && pos && vocab > 0 && seqs > 0, MI355_E_ARG, "argmax_advance_rows: bad argument");
+    hipLaunchKernelGGL(argmax_advance_rows_kernel, dim3(seqs), dim3(1024), 0, (hipStream_t)stream, logits, ld, vocab, next, tokens, pos, out,
+                       ld_out);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}

@@ -700,6 +700,10 @@ class DecodeEngine:
         return None
 
     # ---- bookkeeping ---------------------------------------------------------------------------------
+    @property
+    def n_logits(self) -> int:
+        return int(self.m.lm_head.N)
+
     def weight_stream_bytes(self) -> int:
         return sum(p.stream_bytes for p in self.packed)
 

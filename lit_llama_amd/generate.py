@@ -114,7 +114,7 @@ def _generate_sampled(model, eng, idx, max_new_tokens, max_seq_length, temperatu
         eng.out_tokens[:T].copy_(idx.to(torch.int32))
         eng.prefill(idx, 0, all_logits=False, argmax=False)  # logits of the last prompt token in row 0
         eng.set_step(idx[-1:], 1, T - 1)                      # position slot = T - 1: the draw lands at out_tokens[T]
-        row = eng.logits[0, : eng.m.lm_head.N]
+        row = eng.logits[0, : eng.n_logits]
         kw = dict(out_tokens=eng.out_tokens, tokens=eng.tokens, advance=True)
         ops.sample(row, temperature, top_k, uniforms, eng.pos, eng.next_token, **kw)
         done = 1

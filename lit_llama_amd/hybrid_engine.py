@@ -1,0 +1,475 @@
+"""Native engine of a layered hybrid model: descriptors, slots of state, steps over packed batches.
+
+`step(entries)` is the one way tokens get in: every entry is a slot, the position its first new token has and the tokens; rows of all
+entries are packed without padding and run through `mi355_hybrid_forward` once (a step with more rows than the scratch holds is cut).
+A decode step (one token per entry) is replayed as a hipGraph per batch size.  `generate()` drives the engine through the same
+attributes and methods as `engine.DecodeEngine` (`_ensure_cache`, `prefill`, `set_step`, `run_step`, ...).
+"""
+from __future__ import annotations
+
+import ctypes as C
+import os
+from typing import Dict, List, NamedTuple, Optional, Sequence
+
+import torch
+
+from . import _native as nat
+from . import ops
+from ._native import HybridLayer, HybridModel, Proj, SeqBatch, check, lib, ptr
+from .hybrid import PROJECTIONS, HybridLM
+from .state import SlotManager, grown
+
+MIX = {"attention": 0, "delta": 1, "gla": 2}
+REC_DELTA, REC_GLA = 0, 1
+
+
+class Entry(NamedTuple):
+    """New tokens of one sequence: `want` = the places among them whose logits are asked for."""
+
+    slot: int
+    pos: int
+    tokens: Sequence[int]
+    want: Sequence[int]
+
+
+def _pad16(n: int) -> int:
+    return (n + 15) // 16 * 16
+
+
+class HybridEngine:
+    supports_batches = True
+
+    def __init__(self, model: HybridLM, *, max_rows: Optional[int] = None):
+        self.model, self.cfg, self.device = model, model.config, model.device
+        self.dtype = model.dtype
+        self.max_rows = max_rows or int(os.environ.get("MI355_HYBRID_ROWS", "4096"))
+        self.use_graph = os.environ.get("MI355_HYBRID_GRAPH", "1") != "0"
+        self.stream = torch.cuda.Stream(self.device)
+        self._keep: List[torch.Tensor] = []
+        self._graphs: Dict[tuple, C.c_void_p] = {}
+        self._warm: set = set()
+        self.max_len = 0            # longest sequence the rings are sized for
+        with torch.cuda.device(self.device), torch.cuda.stream(self.stream):
+            self.stream.wait_stream(torch.cuda.default_stream(self.device))
+            self._pack()
+            self._scratch()
+        self.slots = SlotManager(self._grow)
+        self._single: Optional[int] = None  # generate()'s slot
+        self.stream.synchronize()
+
+    # ---- weights ---------------------------------------------------------------------------------------
+    def _proj(self, w: torch.Tensor) -> Proj:
+        """A weight [N, K] with its rows padded to a multiple of 16 (zero rows: the padding columns of every buffer stay zero)."""
+        N, K = w.shape
+        n = _pad16(N)
+        if n != N:
+            w = torch.cat([w, w.new_zeros((n - N, K))])
+        if self.dtype == torch.bfloat16:
+            w = ops.repack_bf16(w, None, 1)
+        else:
+            w = w.contiguous()
+        self._keep.append(w)
+        self.weight_bytes += w.numel() * w.element_size()
+        return Proj(ptr(w), n, K)
+
+    def _f32(self, t: torch.Tensor) -> int:
+        t = t.detach().float().contiguous()
+        self._keep.append(t)
+        return ptr(t)
+
+    def _pack(self) -> None:
+        cfg, T = self.cfg, self.model.tensors
+        self.weight_bytes = 0
+        self.norm_dtype = nat.dtype_code(self.dtype)
+        layers = []
+        for i, spec in enumerate(cfg.layers):
+            m, p = spec.mixer, f"l{i}."
+            x = p + "mix."
+            L = HybridLayer()
+            L.mixer, L.mlp = MIX[m.type], 1 if spec.ff else 0
+            L.norm1 = ptr(T[p + "norm1"])
+            # one stacked projection, every piece padded to 16 columns
+            off, parts = {}, []
+            for name in PROJECTIONS[m.type]:
+                w = T[x + name]
+                off[name] = sum(q.shape[0] for q in parts)
+                pad = _pad16(w.shape[0]) - w.shape[0]
+                parts.append(torch.cat([w, w.new_zeros((pad, w.shape[1]))]) if pad else w)
+            setattr(L, "in", self._proj(torch.cat(parts)))
+            L.out = self._proj(T[x + "o"])
+            if spec.ff:
+                L.norm2 = ptr(T[p + "norm2"])
+                L.up, L.down = self._proj(T[p + "mlp.up"]), self._proj(T[p + "mlp.down"])
+            if m.type == "attention":
+                a = L.attn
+                a.heads, a.kv_heads, a.dim, a.vdim = m.heads, m.kv_heads, m.dim, m.vdim
+                a.off_q, a.off_k, a.off_v, a.off_g = off["q"], off["k"], off["v"], off["g"]
+                a.scale, a.window, a.rot_dims = m.scale, m.window, m.rot_dims
+                if m.rot_dims:
+                    f = torch.tensor([m.rot_base ** (-2.0 * j / m.rot_dims) for j in range(m.rot_dims // 2)], dtype=torch.float64,
+                                     device=self.device)
+                    self._keep.append(f)
+                    a.inv_freq = ptr(f)
+            else:
+                r = L.rec
+                r.kind = REC_DELTA if m.type == "delta" else REC_GLA
+                r.heads, r.kv_heads, r.dim, r.vdim = m.heads, m.kv_heads, m.dim, m.vdim
+                r.off_q, r.off_k, r.off_v, r.off_g = off["q"], off["k"], off["v"], off["g"]
+                r.q_scale, r.eps, r.unit_eps = m.dim ** -0.5, cfg.eps, 1e-6
+                r.head_norm = self._f32(T[x + "norm"])
+                if m.type == "delta":
+                    r.off_a, r.off_b, r.taps = off["a"], off["b"], m.taps
+                    r.conv_q, r.conv_k, r.conv_v = (self._f32(T[x + n + ".conv"]) for n in "qkv")
+                    r.a_log, r.dt_bias = self._f32(T[x + "A_log"]), self._f32(T[x + "dt_bias"])
+                else:
+                    r.off_a, r.rank, r.inv_tau = off["a1"], T[x + "a1"].shape[0], 1.0 / m.tau
+                    r.a2, r.a2_bias = self._f32(T[x + "a2"]), self._f32(T[x + "a2.b"])
+            layers.append(L)
+        runs = cfg.runs()
+        self.run_layers = runs
+        self.layers = (HybridLayer * max(1, len(runs)))()
+        for r, i in enumerate(runs):
+            C.memmove(C.byref(self.layers[r]), C.byref(layers[i]), C.sizeof(HybridLayer))
+        M = self.m = HybridModel()
+        M.n_runs, M.dtype, M.norm_dtype = len(runs), nat.dtype_code(self.dtype), self.norm_dtype
+        M.width, M.ldx, M.vocab, M.max_rows = cfg.width, _pad16(cfg.width), cfg.vocab_size, self.max_rows
+        M.eps, M.residual_mult = cfg.eps, cfg.residual_mult
+        M.embed, M.final_norm = ptr(T["embed"]), ptr(T["final.norm"])
+        M.head = self._proj(T["head"])
+        M.ld_logits = M.head.N
+        M.layers = self.layers
+        self.n_logits = cfg.vocab_size
+
+    def _buf(self, n: int, dtype: torch.dtype) -> torch.Tensor:
+        t = torch.zeros(max(1, n), dtype=dtype, device=self.device)
+        self._keep.append(t)
+        return t
+
+    def _scratch(self) -> None:
+        M, R, cfg = self.m, self.max_rows, self.cfg
+        ls = list(self.layers)[: M.n_runs]
+        self.x = self._buf(R * M.ldx, torch.float32)
+        M.x, M.xw = ptr(self.x), ptr(self._buf(R * M.ldx, torch.float32))
+        M.ld_att = max([_pad16(l.out.K) for l in ls], default=16)
+        M.proj = ptr(self._buf(R * max([getattr(l, "in").N for l in ls], default=16), self.dtype))
+        M.att = ptr(self._buf(R * M.ld_att, self.dtype))
+        M.hid = ptr(self._buf(R * max([l.up.N for l in ls], default=16), self.dtype))
+        if self.dtype == torch.float32:
+            M.xn, M.tmp = ptr(self._buf(R * M.ldx, torch.float32)), ptr(self._buf(R * M.ldx, torch.float32))
+        else:
+            K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down)])
+            n = int(lib().mi355_linear_gemm_workspace_bytes(R, K))
+            M.gemm_ws, M.gemm_ws_bytes = ptr(self._buf(n, torch.uint8)), n
+        # a split attention step keeps one record per (row, head, split); one split takes none
+        n = max([512 * (l.attn.vdim + 2) * max(8, l.attn.heads // l.attn.kv_heads) for l in ls if l.mixer == 0], default=0)
+        M.partials, M.partials_bytes = ptr(self._buf(n, torch.float32)), n * 4
+        n = max([int(lib().mi355_recurrent_scratch_bytes(l.rec.kind, R, min(R, 1024), l.rec.heads, l.rec.kv_heads, l.rec.dim, l.rec.vdim))
+                 for l in ls if l.mixer != 0], default=0)
+        M.rec_scratch, M.rec_scratch_bytes = ptr(self._buf(n, torch.uint8)), n
+        self.logits_buf = self._buf(self.max_logits_rows * M.ld_logits, torch.float32).view(self.max_logits_rows, M.ld_logits)
+        # the step's integers: tokens | row0 | count | slot | pos | want, one upload
+        self.meta = torch.zeros((6, R), dtype=torch.int32, device=self.device)
+        self.meta_host = torch.zeros((6, R), dtype=torch.int32, pin_memory=True)
+        self._meta_sent = torch.cuda.Event()
+        self._meta_sent.record(self.stream)
+
+    @property
+    def max_logits_rows(self) -> int:
+        return min(self.max_rows, max(256, (1 << 28) // max(1, self.m.ld_logits)))
+
+    # ---- slots -----------------------------------------------------------------------------------------
+    def ensure(self, n_slots: int, max_len: int) -> None:
+        """Room for `n_slots` live sequences of at most `max_len` tokens."""
+        if max_len > self.max_len:
+            self._set_len(max_len)
+        with torch.cuda.stream(self.stream):
+            self.slots.reserve(n_slots)
+
+    def _set_len(self, n: int) -> None:
+        """Rings hold min(window, longest sequence) rows.  Growing them re-lays the rings, so no sequence may be live unless every ring
+        already spans its window."""
+        need = any(l.mixer == 0 and self._ring(l, n) != self._ring(l, self.max_len) for l in list(self.layers)[: self.m.n_runs])
+        if need and self.max_len and self.slots.live:
+            raise nat.NativeError(f"hybrid engine: sequences are live at cache length {self.max_len}; {n} needs a larger one")
+        self.max_len = n
+        if need and self.slots.capacity:
+            self.pools = [None] * self.m.n_runs
+            with torch.cuda.stream(self.stream):
+                self._grow(self.slots.capacity)
+
+    @staticmethod
+    def _ring(l: HybridLayer, max_len: int) -> int:
+        return min(l.attn.window, max(1, max_len))
+
+    def _grow(self, n: int) -> None:
+        self._destroy_graphs()  # captured launches hold the old addresses
+        if not hasattr(self, "pools"):
+            self.pools = [None] * self.m.n_runs
+        dev = self.device
+        for r in range(self.m.n_runs):
+            l, old = self.layers[r], self.pools[r] or (None, None)
+            if l.mixer == 0:
+                a = l.attn
+                a.ring = self._ring(l, self.max_len or 1)
+                k = grown(old[0], (n, a.kv_heads, a.ring, a.dim), self.dtype, dev)
+                v = grown(old[1], (n, a.kv_heads, a.ring, a.vdim), self.dtype, dev)
+                a.kring, a.vring = ptr(k), ptr(v)
+                self.pools[r] = (k, v)
+            else:
+                e = l.rec
+                st = grown(old[0], (n, e.heads, e.dim, e.vdim), torch.float32, dev)
+                cv = None
+                if e.kind == REC_DELTA:
+                    cv = grown(old[1], (n, e.taps, 2 * e.kv_heads * e.dim + e.heads * e.vdim), self.dtype, dev)
+                    e.conv_ring = ptr(cv)
+                e.state = ptr(st)
+                self.pools[r] = (st, cv)
+
+    def state_bytes(self) -> int:
+        """Bytes of cache and state per slot."""
+        return sum(t.numel() * t.element_size() for p in self.pools for t in p if t is not None) // max(1, self.slots.capacity)
+
+    def acquire(self) -> int:
+        """A slot for a new sequence, its recurrent state zeroed."""
+        with torch.cuda.stream(self.stream):
+            slot = self.slots.acquire()
+            self._reset([slot])
+        return slot
+
+    def release(self, slot: int) -> None:
+        self.slots.release(slot)
+
+    def _reset(self, slots: List[int]) -> None:
+        t = torch.tensor(slots, dtype=torch.int32).to(self.device)
+        check(lib().mi355_hybrid_reset_slots(C.byref(self.m), ptr(t), len(slots), self.stream.cuda_stream), "mi355_hybrid_reset_slots")
+        self.stream.synchronize()  # (`t` may go)
+
+    # ---- steps -----------------------------------------------------------------------------------------
+    def _batch(self, rows: int, seqs: int, max_count: int) -> SeqBatch:
+        b = SeqBatch()
+        b.rows, b.seqs, b.max_count = rows, seqs, max_count
+        b.row0, b.count, b.slot, b.pos = (ptr(self.meta[i]) for i in (1, 2, 3, 4))
+        return b
+
+    def _upload(self, entries: Sequence[Entry]) -> tuple:
+        """Packs a step's integers and sends them; returns (batch, wanted rows)."""
+        h = self.meta_host
+        self._meta_sent.synchronize()  # the previous upload has left the pinned buffer
+        rows, n_want, most = 0, 0, 0
+        for s, e in enumerate(entries):
+            n = len(e.tokens)
+            h[0, rows:rows + n] = torch.as_tensor(e.tokens, dtype=torch.int32)
+            h[1, s], h[2, s], h[3, s], h[4, s] = rows, n, e.slot, e.pos
+            if len(e.want):
+                h[5, n_want:n_want + len(e.want)] = torch.as_tensor(e.want, dtype=torch.int32) + rows
+                n_want += len(e.want)
+            rows += n
+            most = max(most, n)
+        self.meta.copy_(h, non_blocking=True)
+        self._meta_sent.record(self.stream)
+        return self._batch(rows, len(entries), most), n_want
+
+    def _cut(self, entries: Sequence[Entry]) -> List[List[Entry]]:
+        """Sub-steps of at most max_rows rows and max_logits_rows wanted rows; a long portion continues in the next one."""
+        subs, cur, room, wants = [], [], self.max_rows, self.max_logits_rows
+        for e in entries:
+            if e.pos + len(e.tokens) > self.max_len:
+                raise nat.NativeError(f"hybrid engine: position {e.pos + len(e.tokens) - 1} is outside the cache of {self.max_len}")
+            if min(e.tokens, default=0) < 0 or max(e.tokens, default=0) >= self.cfg.vocab_size:
+                raise nat.NativeError(f"hybrid engine: token outside the vocabulary of {self.cfg.vocab_size}")
+            at, want = 0, sorted(e.want)
+            if list(e.want) != want:
+                raise nat.NativeError("hybrid engine: wanted places must ascend")
+            while at < len(e.tokens):
+                if room == 0 or wants == 0:
+                    subs.append(cur)
+                    cur, room, wants = [], self.max_rows, self.max_logits_rows
+                n = min(room, len(e.tokens) - at)
+                inside = [k for k in want if at <= k < at + n]
+                if len(inside) > wants:  # stop behind the last row whose logits still fit
+                    inside = inside[:wants]
+                    n = inside[-1] + 1 - at
+                cur.append(Entry(e.slot, e.pos + at, e.tokens[at:at + n], [k - at for k in inside]))
+                at, room, wants = at + n, room - n, wants - len(inside)
+                if at < len(e.tokens):  # one sequence has one entry per sub-step
+                    subs.append(cur)
+                    cur, room, wants = [], self.max_rows, self.max_logits_rows
+        if cur:
+            subs.append(cur)
+        return subs
+
+    def step(self, entries: Sequence[Entry]) -> torch.Tensor:
+        """Runs the new tokens of every entry; returns the wanted logits [n, vocab] f32 in the order of entries and places (a buffer of
+        this engine when one sub-step was enough: valid until the next step).  Work is queued on the current stream's behalf."""
+        entries = [e for e in entries if len(e.tokens)]
+        cur = torch.cuda.current_stream(self.device)
+        self.stream.wait_stream(cur)
+        outs = []
+        with torch.cuda.device(self.device), torch.cuda.stream(self.stream):
+            subs = self._cut(entries)
+            for sub in subs:
+                b, n_want = self._upload(sub)
+                self._run(b, n_want)
+                if n_want:
+                    out = self.logits_buf[:n_want, : self.n_logits]
+                    outs.append(out if len(subs) == 1 else out.clone())
+            res = outs[0] if len(outs) == 1 else torch.cat(outs) if outs else self.logits_buf[:0, : self.n_logits]
+        cur.wait_stream(self.stream)
+        return res
+
+    def _launch(self, b: SeqBatch, n_want: int, all_rows: bool, run_end: int = 1 << 30) -> None:
+        check(lib().mi355_hybrid_forward(C.byref(self.m), C.byref(b), ptr(self.meta[0]), None if all_rows else ptr(self.meta[5]), n_want,
+                                         ptr(self.logits_buf), min(run_end, self.m.n_runs), self.stream.cuda_stream), "mi355_hybrid_forward")
+
+    def _run(self, b: SeqBatch, n_want: int) -> None:
+        decode = b.max_count == 1 and (n_want == b.rows or n_want == 0)
+        if not decode:
+            self._launch(b, n_want, False)
+        else:
+            self._replay(("step", b.rows, n_want), lambda: self._launch(b, n_want, n_want > 0))
+
+    def _replay(self, key: tuple, enqueue) -> None:
+        """The launches of `enqueue` as a graph of their own per key.  The first time they run as they are (launchers set kernel attributes
+        lazily, which a capture must not see; a recurrent step cannot be repeated), the second time they are captured, then replayed."""
+        s = self.stream.cuda_stream
+        if not self.use_graph or key not in self._warm:
+            enqueue()
+            self._warm.add(key)
+            return
+        g = self._graphs.get(key)
+        if g is None:
+            check(lib().mi355_graph_begin(s), "mi355_graph_begin")
+            handle = C.c_void_p()
+            try:
+                enqueue()
+            finally:
+                rc = lib().mi355_graph_end(s, C.byref(handle))
+            check(rc, "mi355_graph_end")
+            g = self._graphs[key] = handle
+        check(lib().mi355_graph_launch(g, s), "mi355_graph_launch")
+
+    def _destroy_graphs(self) -> None:
+        if self._graphs:
+            self.stream.synchronize()
+        for g in self._graphs.values():
+            lib().mi355_graph_destroy(g)
+        self._graphs = {}
+
+    def __del__(self):
+        try:
+            self._destroy_graphs()
+        except Exception:
+            pass
+
+    def residual_after(self, entries: Sequence[Entry], run_end: int) -> torch.Tensor:
+        """The residual stream [rows, width] behind the first `run_end` layer runs of a step (it advances the state like a step)."""
+        with torch.cuda.device(self.device), torch.cuda.stream(self.stream):
+            b, _ = self._upload(entries)
+            self._launch(b, 0, False, run_end)
+        self.stream.synchronize()
+        return self.x.view(self.max_rows, self.m.ldx)[: b.rows, : self.cfg.width].clone()
+
+    # ---- model(idx, max_seq_length, input_pos) ---------------------------------------------------------
+    def forward_no_cache(self, idx: torch.Tensor) -> torch.Tensor:
+        B, T = idx.shape
+        self.ensure(self.slots.live + B, max(self.max_len, T))
+        slots = [self.acquire() for _ in range(B)]
+        rows = idx.tolist()
+        out = self.step([Entry(s, 0, r, range(T)) for s, r in zip(slots, rows)]).clone().view(B, T, -1)
+        for s in slots:
+            self.release(s)
+        return out
+
+    def forward(self, idx: torch.Tensor, max_seq_length: int, input_pos: torch.Tensor) -> torch.Tensor:
+        T = idx.shape[1]
+        pos0 = getattr(input_pos, "_mi355_pos0", None)
+        if pos0 is None:
+            pos0 = int(input_pos[0])
+        if pos0 == 0 or self._single is None:
+            self._ensure_cache(max_seq_length)
+        if pos0 != self._next:
+            raise nat.NativeError(f"a recurrent model continues its sequence at position {self._next}, not {pos0} (reset_cache() starts over)")
+        out = self.step([Entry(self._single, pos0, idx.reshape(-1).tolist(), range(T))]).clone()
+        self._next = pos0 + T
+        return out.view(1, T, -1)
+
+    # ---- generate()'s interface (engine.DecodeEngine's) ------------------------------------------------
+    def reset_cache(self) -> None:
+        if self._single is not None:
+            self.release(self._single)
+            self._single = None
+
+    def _ensure_cache(self, S: int) -> None:
+        """A fresh sequence of at most S tokens in the slot that generate() owns."""
+        self.reset_cache()
+        self.ensure(self.slots.live + 1, max(S, self.max_len))
+        self._single, self._next = self.acquire(), 0
+        if getattr(self, "out_tokens", None) is None or self.out_tokens.numel() < S + 1:
+            self.out_tokens = torch.zeros(S + 1, dtype=torch.int32, device=self.device)
+            self._destroy_graphs()
+        self.next_token = getattr(self, "next_token", None)
+        if self.next_token is None:
+            self.next_token = torch.zeros(1, dtype=torch.int32, device=self.device)
+
+    @property
+    def tokens(self) -> torch.Tensor:
+        return self.meta[0]
+
+    @property
+    def pos(self) -> torch.Tensor:
+        return self.meta[4]
+
+    @property
+    def logits(self) -> torch.Tensor:
+        return self.logits_buf
+
+    def clear_status(self) -> None:
+        pass
+
+    def status_due(self) -> bool:
+        return False  # (no step of this engine leaves a state to be read back)
+
+    def check_status(self) -> Optional[int]:
+        return None
+
+    def _advance(self) -> None:
+        check(lib().mi355_argmax_advance_rows(ptr(self.logits_buf), self.m.ld_logits, self.n_logits, 1, ptr(self.next_token),
+                                              ptr(self.meta[0]), ptr(self.meta[4]), ptr(self.out_tokens), self.out_tokens.numel(),
+                                              self.stream.cuda_stream), "mi355_argmax_advance_rows")
+
+    def prefill(self, idx: torch.Tensor, pos0: int, *, all_logits: bool, argmax: bool = False) -> Optional[torch.Tensor]:
+        toks = idx.reshape(-1).tolist()
+        T = len(toks)
+        subs = self._cut([Entry(self._single, pos0, toks, range(T) if all_logits else [T - 1])])
+        out = []
+        for sub in subs:
+            b, n = self._upload(sub)
+            self._launch(b, n, False)
+            if all_logits and n:
+                out.append(self.logits_buf[:n, : self.n_logits].clone())
+        self._next = pos0 + T
+        if argmax:  # the draw of position T - 1: out_tokens[T]
+            self.set_step(idx.reshape(-1)[-1:], 1, pos0 + T - 1)
+            self._advance()
+        return torch.cat(out) if all_logits else None
+
+    def set_step(self, idx: Optional[torch.Tensor], T: int, pos0: int, from_next: bool = False) -> None:
+        """One-token entry state of generate()'s slot (host-known token or the last draw)."""
+        self.meta[0, :1].copy_((self.next_token if from_next else idx.reshape(-1)[:1]).to(torch.int32))
+        h = torch.tensor([[0], [1], [self._single], [pos0]], dtype=torch.int32)
+        self.meta[1:5, :1].copy_(h.to(self.device))
+
+    def embed_step(self) -> None:
+        pass  # (the step starts at its token)
+
+    def run_step(self, argmax) -> None:
+        """One decode step at the token / position on the device; argmax 3: the greedy draw becomes the next step's token."""
+        b = self._batch(1, 1, 1)
+
+        def enqueue():
+            self._launch(b, 1, True)
+            if int(argmax) & 1:
+                self._advance()
+
+        self._replay(("single", int(argmax)), enqueue)
+        self._next += 1
