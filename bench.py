@@ -68,6 +68,12 @@ def parse():
     ap.add_argument("--tp-model", default="65B")
     ap.add_argument("--tp-steps", type=int, default=48)
     ap.add_argument("--tp-comm", default="native", choices=["native", "rccl"])
+    ap.add_argument("--hybrid", default=None, metavar="WIDTH[,WIDTH]",
+                    help="instead of the headline workload: prompt and decode rates of a layered hybrid model (Sekulorn design) of these "
+                         "widths beside an unquantised LLaMA of the same width and layer count (random weights)")
+    ap.add_argument("--hybrid-layers", type=int, default=8)
+    ap.add_argument("--hybrid-batches", default="1,16,64")
+    ap.add_argument("--hybrid-only", default="both", choices=["both", "hybrid", "llama"], help="(profiling) one side of --hybrid")
     ap.add_argument("--tune", default=None, help="JSON dict of per-linear launch tuning (engine.DecodeEngine tune)")
     return ap.parse_args()
 
@@ -460,6 +466,98 @@ def spawn_command(n: int, argv):
             "--master-port", str(port), os.path.abspath(__file__), *argv]
 
 
+def _timed(stream, fn, reps: int) -> float:
+    """Seconds per call of `fn` (device time of `reps` calls queued on `stream`), median of three."""
+    fn()
+    out = []
+    for _ in range(3):
+        a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        torch.cuda.synchronize()
+        a.record(stream)
+        for _ in range(reps):
+            fn()
+        b.record(stream)
+        torch.cuda.synchronize()
+        out.append(a.elapsed_time(b) / 1e3 / reps)
+    return sorted(out)[1]
+
+
+def hybrid_bench(args, dev) -> dict:
+    """--hybrid: prompt pass and decode steps of the hybrid model and of an unquantised LLaMA of equal width and depth."""
+    from lit_llama_amd import synth
+    from lit_llama_amd.hybrid import HybridConfig, HybridLM
+    from lit_llama_amd.hybrid_engine import Entry
+    from lit_llama_amd.model import LLaMA, LLaMAConfig
+    from lit_llama_amd.utils import EmptyInitOnDevice
+
+    T, steps, S = 2048, args.steps if args.steps != 256 else 32, 4096
+    batches = [int(x) for x in args.hybrid_batches.split(",")]
+    g = torch.Generator().manual_seed(7)
+    res = []
+    for width in (int(w) for w in args.hybrid.split(",")):
+        row = {"width": width, "layers": args.hybrid_layers, "prompt": T}
+        if args.hybrid_only != "llama":
+            conf = synth.hybrid_bench_config(width, args.hybrid_layers)
+            model = HybridLM(HybridConfig.from_dict(conf), device=dev)
+            model.load_state_dict(synth.make_hybrid_state_dict(conf, device=dev))
+            eng = model.engine()
+            eng.ensure(max(batches), S)
+            prompt = torch.randint(0, conf["vocab"], (T,), generator=g).tolist()
+            slots = [eng.acquire() for _ in range(max(batches))]
+            for s_ in slots:  # every sequence at position T: decode steps see full windows
+                eng.step([Entry(s_, 0, prompt, [])])
+            with torch.cuda.stream(eng.stream):
+                sec = _timed(eng.stream, lambda: eng.step([Entry(slots[0], 0, prompt, [T - 1])]), 4)
+            h = {"prefill_ms": round(sec * 1e3, 3), "prefill_tokens_per_s": round(T / sec, 1), "weight_bytes": eng.weight_bytes,
+                 "state_bytes_per_sequence": eng.state_bytes(), "decode": {}}
+            for B in batches:
+                at = [T]
+
+                def one():
+                    eng.step([Entry(s_, at[0], prompt[:1], [0]) for s_ in slots[:B]])
+                    at[0] += 1
+
+                one()
+                with torch.cuda.stream(eng.stream):
+                    b, n = eng._upload([Entry(s_, at[0], prompt[:1], [0]) for s_ in slots[:B]])
+                    # device time of the step itself: the same batch replayed (positions stay, the work of a step does not depend on them)
+                    sec = _timed(eng.stream, lambda: eng._run(b, n), steps)
+                weights = eng.weight_bytes / sec
+                h["decode"][str(B)] = {"us_per_step": round(sec * 1e6, 1), "tokens_per_s": round(B / sec, 1),
+                                       "weight_bytes_frac_of_8TBps": round(weights / 8e12, 4)}
+            row["hybrid"] = h
+            del model, eng
+            torch.cuda.empty_cache()
+        if args.hybrid_only != "hybrid":
+            cfg = LLaMAConfig(n_layer=args.hybrid_layers, n_head=width // 128, n_embd=width, block_size=S)
+            with EmptyInitOnDevice(device=dev, dtype=torch.bfloat16):
+                llama = LLaMA(cfg)
+            with torch.no_grad():
+                for p in llama.parameters():
+                    p.normal_(0.0, p.shape[-1] ** -0.5) if p.dim() > 1 else p.fill_(1.0)
+            eng = llama.engine()
+            assert eng is not None, llama._engine_failed
+            idx = torch.randint(0, 32000, (T,), generator=g).to(dev)
+            with torch.cuda.stream(eng.stream):
+                eng._ensure_cache(S)
+                sec = _timed(eng.stream, lambda: eng.prefill(idx, 0, all_logits=False), 4)
+                h = {"prefill_ms": round(sec * 1e3, 3), "prefill_tokens_per_s": round(T / sec, 1), "weight_bytes": eng.weight_stream_bytes()}
+
+                def one_llama():
+                    eng.set_step(idx[:1], 1, T)
+                    eng.run_step(False)
+
+                sec = _timed(eng.stream, one_llama, steps)
+                h["decode"] = {"1": {"us_per_step": round(sec * 1e6, 1), "tokens_per_s": round(1 / sec, 1),
+                                     "weight_bytes_frac_of_8TBps": round(eng.weight_stream_bytes() / sec / 8e12, 4),
+                                     "persistent_step": bool(eng.fused is not None and eng.fused_ready())}}
+            row["llama"] = h
+            del llama, eng
+            torch.cuda.empty_cache()
+        res.append(row)
+    return {"hybrid_bench": res, "dtype": "bf16", "data": "synthetic", "steps": steps}
+
+
 def main():
     args = parse()
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
@@ -519,6 +617,9 @@ def main():
         raise SystemExit("bench.py needs an MI355X (no GPU visible); there is no CPU fallback for the hot path")
     dev = torch.device("cuda", local_rank)
     torch.cuda.set_device(dev)
+    if args.hybrid:
+        print(json.dumps(hybrid_bench(args, dev)))
+        return
     dist = None
     if world > 1:
         import torch.distributed as dist

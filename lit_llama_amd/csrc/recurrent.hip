@@ -2,55 +2,13 @@
 //
 //   rec_rows_kernel       one workgroup per (head, sequence) walks its rows one by one with the state in registers: decode steps
 //                         (convolution, gates, state update, output norm and gate in ONE launch) and short portions
+//   (longer portions: recurrent_chunks.hip)
 //   conv_ring_kernel      behind a portion of several rows: its last taps - 1 inputs enter the convolution's ring
 //
 // Everything that enters the recurrence is f32, whatever the dtype of the projections.
-#include "common.h"
+#include "recurrent.h"
 
 namespace {
-
-constexpr int kMaxRank = 256;
-
-__device__ __forceinline__ float silu_f32(float v) { return v / (1.0f + expf(-v)); }
-__device__ __forceinline__ float sigmoid_f32(float v) { return 1.0f / (1.0f + expf(-v)); }
-__device__ __forceinline__ float softplus_f32(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
-
-template <typename T>
-__device__ __forceinline__ float to_f32(T v);
-template <>
-__device__ __forceinline__ float to_f32<float>(float v) { return v; }
-template <>
-__device__ __forceinline__ float to_f32<bf16_t>(bf16_t v) { return bf16_to_f32(v); }
-template <typename T>
-__device__ __forceinline__ T from_f32(float v);
-template <>
-__device__ __forceinline__ float from_f32<float>(float v) { return v; }
-template <>
-__device__ __forceinline__ bf16_t from_f32<bf16_t>(float v) { return f32_to_bf16(v); }
-
-struct RecParams {
-    mi355_recurrent_args a;
-    mi355_seq_batch b;
-    int parts, slices;  // row kernel: row parts of the state, 64-column slices
-};
-
-// one convolution output: channel c of the q | k | v inputs (`off` = its column in proj, `cr` = its column in the ring), row i of the
-// portion that starts at position pos0
-template <typename T>
-__device__ __forceinline__ float conv_at(const mi355_recurrent_args& a, const T* rows, const T* ring, int ring_ld, int off, int cr,
-                                         const float* w, int i, int pos0) {
-    float v = 0.f;
-    for (int j = 0; j < a.taps; ++j) {  // j rows back
-        const int r = i - j;
-        float x = 0.f;
-        if (r >= 0)
-            x = to_f32<T>(rows[(int64_t)r * a.ld + off]);
-        else if (pos0 + r >= 0)
-            x = to_f32<T>(ring[(int64_t)((pos0 + r) % a.taps) * ring_ld + cr]);
-        v += w[a.taps - 1 - j] * x;
-    }
-    return silu_f32(v);
-}
 
 // state S [dim][vdim] of one (slot, head): column 64 * slice + lane, rows part * RMAX + r in registers
 template <typename T, int KIND, int RMAX>
@@ -237,8 +195,15 @@ int run_rows(RecParams p, hipStream_t s) {
 
 template <typename T>
 int run(const RecParams& p, hipStream_t s) {
-    if (int rc = p.a.kind == MI355_REC_DELTA ? run_rows<T, MI355_REC_DELTA>(p, s) : run_rows<T, MI355_REC_GLA>(p, s)) return rc;
-    if (p.a.kind == MI355_REC_DELTA && p.b.max_count > 1) {
+    const bool fit = mi355_recurrent_chunks_fit(p.a, p.b);
+    MI355_CHECK_ARG(p.a.path != 2 || fit, MI355_E_SHAPE, "recurrent: chunks take states of up to 256 x 256 and their scratch");
+    const bool chunks = p.a.path == 2 || (p.a.path == 0 && fit && p.b.max_count > 8);
+    if (chunks) {
+        if (int rc = mi355_recurrent_chunks(p, s)) return rc;
+    } else if (int rc = p.a.kind == MI355_REC_DELTA ? run_rows<T, MI355_REC_DELTA>(p, s) : run_rows<T, MI355_REC_GLA>(p, s)) {
+        return rc;
+    }
+    if (p.a.kind == MI355_REC_DELTA && (chunks || p.b.max_count > 1)) {
         hipLaunchKernelGGL(conv_ring_kernel<T>, dim3(p.a.taps < p.b.max_count ? p.a.taps : p.b.max_count, p.b.seqs), dim3(256), 0, s, p);
         MI355_LAUNCH_CHECK();
     }
@@ -246,11 +211,6 @@ int run(const RecParams& p, hipStream_t s) {
 }
 
 }  // namespace
-
-extern "C" size_t mi355_recurrent_scratch_bytes(int kind, int rows, int seqs, int heads, int kv_heads, int dim, int vdim) {
-    (void)kind, (void)rows, (void)seqs, (void)heads, (void)kv_heads, (void)dim, (void)vdim;
-    return 0;
-}
 
 extern "C" int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_batch* b, mi355_stream_t stream) {
     MI355_CHECK_ARG(a && b && a->proj && a->state && a->y && a->head_norm, MI355_E_ARG, "recurrent: null argument");

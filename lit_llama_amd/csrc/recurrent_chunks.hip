@@ -1,0 +1,716 @@
+// Prompt steps of the linear recurrences in chunks of 64 rows, on the f32 matrix cores (v_mfma_f32_16x16x4_f32: operands, products and
+// sums are f32, as the recurrence asks).
+//
+// With G_i = sum of the log decays of a chunk up to row i, S_0 the state in front of the chunk and U the rows written into it:
+//
+//   delta  (I + A) U = diag(beta) (V - diag(e^G) K S_0),   A_ij = beta_i e^(G_i - G_j) k_i . k_j  (j < i)
+//          O = diag(e^G) Q S_0 + P U,                      P_ij = e^(G_i - G_j) q_i . k_j         (j <= i)
+//          S = e^(G_end) S_0 + K^T diag(e^(G_end - G)) U
+//   gla    U = V,  e^(G_i - G_j) acts per key channel inside the products,  O = (Q e^G) S_0 + P V,  S = diag(e^(G_end)) S_0 + (K e^(G_end - G))^T V
+//
+// Every exponent is <= 0.  Launches of a step (each over all chunks at once but the scan):
+//   delta_qk_kernel    convolutions, unit norms; Q, K^T, K K^T, Q K^T per key head
+//   delta_head_kernel  decays, T = (I + A)^-1 by 16 x 16 blocks, U0 = T diag(beta) V, W = T diag(beta e^G) K, P per head
+//   gla_prep_kernel    decays, Q e^G, (K e^(G_end - G))^T, P (off-diagonal 16 x 16 blocks anchored at the row block's first row), V^T
+//   scan_kernel        one workgroup per (sequence, head, 16 columns): U = U0 - W S_0, S; the state in accumulator registers
+//   chunk_out_kernel   O, output norm, gate
+//
+// Matrix operand layouts: A row-major and B column-major in memory with the contraction index contiguous; of every 16 of it lane group g
+// (lane >> 4) takes 4g .. 4g + 3 with one 16-B load, one element per MFMA.
+#include "recurrent.h"
+
+namespace {
+
+constexpr int kC = 64;        // rows of a chunk
+constexpr int kP = kC + 4;    // pitch of [..][64] matrices in LDS
+constexpr int kX = 20;        // pitch of [..][16] ones
+
+__device__ __forceinline__ f32x4 mfma4(f32x4 a, f32x4 b, f32x4 c) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], c, 0, 0, 0);
+    return c;
+}
+__device__ __forceinline__ f32x4 zero4() { return f32x4{0.f, 0.f, 0.f, 0.f}; }
+
+// ---------------------------------------------------------------- scratch, per packed chunk (padded sizes DP, VP: multiples of 16)
+struct Scratch {
+    float* q;     // [NC][GQ][64][DP]        delta: unit q * q_scale; gla: q e^G * q_scale
+    float* kt;    // [NC][GQ][DP][64]        delta: unit k; gla: k e^(G_end - G)
+    float* kk;    // [NC][G][64][64]         delta: k_i . k_j
+    float* qk;    // [NC][G][64][64]         delta: q_i . k_j
+    float* P;     // [NC][H][64][64]
+    float* W;     // [NC][H][64][DP]         delta
+    float* ut;    // [NC][H][VP][64]         U^T (delta: U0^T until the scan)
+    float* st;    // [NC][H][VP][DP]         S_0^T
+    float* gam;   // [NC][H][DP]             e^(G_end) (delta: element 0)
+    float* eg;    // [NC][H][64]             delta: e^G
+    float* ed;    // [NC][H][64]             delta: e^(G_end - G)
+};
+
+struct ChunkParams {
+    RecParams r;
+    Scratch s;
+    int seq0;     // first sequence of this group
+    int GQ, DP, VP;
+};
+
+__device__ __forceinline__ int chunk_base(const ChunkParams& p, int seq) {
+    return p.r.b.row0[seq] / kC + seq - (p.r.b.row0[p.seq0] / kC + p.seq0);
+}
+
+// ------------------------------------------------------------------------------------ delta: q, k per key head
+// grid (chunks, kv_heads, seqs), 256 threads.  LDS: k, q [64][DP + 4]
+template <typename T>
+__global__ __launch_bounds__(256) void delta_qk_kernel(const ChunkParams p) {
+    const mi355_recurrent_args& a = p.r.a;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    const int seq = p.seq0 + blockIdx.z, kvh = blockIdx.y, t0 = blockIdx.x * kC;
+    const int cnt = p.r.b.count[seq];
+    if (t0 >= cnt) return;
+    const int DP = p.DP, ld = DP + 4, dim = a.dim;
+    float* k = sm;
+    float* q = sm + kC * ld;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int pos0 = p.r.b.pos[seq];
+    const T* rows = (const T*)a.proj + (int64_t)p.r.b.row0[seq] * a.ld;
+    const int ring_ld = 2 * a.kv_heads * dim + a.heads * a.vdim;
+    const T* ring = (const T*)a.conv_ring + (int64_t)p.r.b.slot[seq] * a.taps * ring_ld;
+    for (int i = tid; i < kC * DP; i += 256) {
+        const int t = i / DP, d = i - t * DP;
+        float qv = 0.f, kv = 0.f;
+        if (d < dim && t0 + t < cnt) {
+            const int c = kvh * dim + d;
+            qv = conv_at<T>(a, rows, ring, ring_ld, a.off_q + c, c, a.conv_q + (int64_t)c * a.taps, t0 + t, pos0);
+            kv = conv_at<T>(a, rows, ring, ring_ld, a.off_k + c, a.kv_heads * dim + c, a.conv_k + (int64_t)c * a.taps, t0 + t, pos0);
+        }
+        q[t * ld + d] = qv;
+        k[t * ld + d] = kv;
+    }
+    __syncthreads();
+    for (int t = wave; t < kC; t += 4) {  // unit vectors: a wave per row
+        float sq = 0.f, sk = 0.f;
+        for (int d = lane; d < dim; d += 64) {
+            sq += q[t * ld + d] * q[t * ld + d];
+            sk += k[t * ld + d] * k[t * ld + d];
+        }
+        sq = group_sum(sq, 64);
+        sk = group_sum(sk, 64);
+        const float iq = a.q_scale / sqrtf(sq + a.unit_eps), ik = 1.0f / sqrtf(sk + a.unit_eps);
+        for (int d = lane; d < dim; d += 64) {
+            q[t * ld + d] *= iq;
+            k[t * ld + d] *= ik;
+        }
+    }
+    __syncthreads();
+    const int64_t gi = (int64_t)(chunk_base(p, seq) + blockIdx.x) * p.GQ + kvh;
+    float* oq = p.s.q + gi * kC * DP;
+    float* okt = p.s.kt + gi * DP * kC;
+    for (int i = tid; i < kC * DP / 4; i += 256) {
+        const int t = i / (DP / 4), d = (i - t * (DP / 4)) * 4;
+        *(f32x4*)(oq + t * DP + d) = *(const f32x4*)(q + t * ld + d);
+    }
+    for (int i = tid; i < kC * DP / 4; i += 256) {
+        const int d = i / (kC / 4), t = (i - d * (kC / 4)) * 4;
+        *(f32x4*)(okt + d * kC + t) = f32x4{k[t * ld + d], k[(t + 1) * ld + d], k[(t + 2) * ld + d], k[(t + 3) * ld + d]};
+    }
+    // wave w: rows 16 w .. 16 w + 15 of K K^T and Q K^T, column blocks up to its own
+    const int c16 = lane & 15, g = lane >> 4;
+    float* okk = p.s.kk + gi * kC * kC;
+    float* oqk = p.s.qk + gi * kC * kC;
+    for (int cb = 0; cb <= wave; ++cb) {
+        f32x4 akk = zero4(), aqk = zero4();
+        for (int d = 4 * g; d < DP; d += 16) {
+            const f32x4 b = *(const f32x4*)(k + (cb * 16 + c16) * ld + d);
+            akk = mfma4(*(const f32x4*)(k + (wave * 16 + c16) * ld + d), b, akk);
+            aqk = mfma4(*(const f32x4*)(q + (wave * 16 + c16) * ld + d), b, aqk);
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            okk[(wave * 16 + 4 * g + r) * kC + cb * 16 + c16] = akk[r];
+            oqk[(wave * 16 + 4 * g + r) * kC + cb * 16 + c16] = aqk[r];
+        }
+    }
+}
+
+// ------------------------------------------------------------------------------------ delta: per head
+// grid (chunks, heads, seqs), 256 threads.  LDS: A, T [64][kP], X [64][kX], vt [VP][kP]
+template <typename T>
+__global__ __launch_bounds__(256) void delta_head_kernel(const ChunkParams p) {
+    const mi355_recurrent_args& a = p.r.a;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    __shared__ double gcum[kC];
+    __shared__ float beta[kC], bg[kC];
+    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, t0 = blockIdx.x * kC;
+    const int cnt = p.r.b.count[seq];
+    if (t0 >= cnt) return;
+    const int DP = p.DP, VP = p.VP;
+    float* A = sm;
+    float* Ti = A + kC * kP;
+    float* X = Ti + kC * kP;
+    float* vt = X + kC * kX;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c16 = lane & 15, g = lane >> 4;
+    const int kvh = head / (a.heads / a.kv_heads);
+    const int pos0 = p.r.b.pos[seq];
+    const T* rows = (const T*)a.proj + (int64_t)p.r.b.row0[seq] * a.ld;
+    const int ring_ld = 2 * a.kv_heads * a.dim + a.heads * a.vdim;
+    const T* ring = (const T*)a.conv_ring + (int64_t)p.r.b.slot[seq] * a.taps * ring_ld;
+    const int64_t ci = chunk_base(p, seq) + blockIdx.x;
+    const int64_t gi = ci * p.GQ + kvh, hi = ci * a.heads + head;
+
+    if (tid < kC) {
+        float lg = 0.f, b = 0.f;
+        if (t0 + tid < cnt) {
+            const T* row = rows + (int64_t)(t0 + tid) * a.ld;
+            lg = -expf(a.a_log[head]) * softplus_f32(to_f32<T>(row[a.off_a + head]) + a.dt_bias[head]);
+            b = sigmoid_f32(to_f32<T>(row[a.off_b + head]));
+        }
+        // inclusive sum over the wave; f64, so that differences of far sums keep f32 accuracy
+        double s = lg;
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const double v = __shfl_up(s, o, 64);
+            if (lane >= o) s += v;
+        }
+        gcum[tid] = s;
+        beta[tid] = b;
+        const double end = __shfl(s, 63, 64);
+        const float eg = expf((float)s);
+        bg[tid] = b * eg;
+        p.s.eg[hi * kC + tid] = eg;
+        p.s.ed[hi * kC + tid] = expf((float)(end - s));
+        if (tid == 63) p.s.gam[hi * DP] = expf((float)end);
+    }
+    // V^T with the convolution (beta rides on it below)
+    for (int i = tid; i < kC * VP; i += 256) {
+        const int t = i / VP, d = i - t * VP;
+        float v = 0.f;
+        if (d < a.vdim && t0 + t < cnt) {
+            const int c = head * a.vdim + d;
+            v = conv_at<T>(a, rows, ring, ring_ld, a.off_v + c, 2 * a.kv_heads * a.dim + c, a.conv_v + (int64_t)c * a.taps, t0 + t, pos0);
+        }
+        vt[d * kP + t] = v;
+    }
+    __syncthreads();
+    const float* kk = p.s.kk + gi * kC * kC;
+    const float* qk = p.s.qk + gi * kC * kC;
+    float* oP = p.s.P + hi * kC * kC;
+    for (int i = tid; i < kC * kC; i += 256) {
+        const int r = i >> 6, c = i & 63;
+        float e = 0.f, x = 0.f, y = 0.f;
+        if (c <= r) {
+            e = expf((float)(gcum[r] - gcum[c]));
+            y = e * qk[i];
+            if (c < r) x = beta[r] * e * kk[i];
+        }
+        A[r * kP + c] = x;
+        Ti[r * kP + c] = 0.f;
+        oP[i] = y;
+    }
+    for (int i = tid; i < kC * VP; i += 256) {
+        const int d = i / kC, t = i - d * kC;
+        vt[d * kP + t] *= beta[t];
+    }
+    __syncthreads();
+    // ---- diagonal blocks of T: thread (block, column), forward substitution in registers
+    if (tid < 64) {
+        const int b0 = (tid >> 4) * 16, c = tid & 15;
+        float x[16];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            float s = i == c ? 1.f : 0.f;
+#pragma unroll
+            for (int j = 0; j < i; ++j) s -= A[(b0 + i) * kP + b0 + j] * x[j];
+            x[i] = i < c ? 0.f : s;
+        }
+#pragma unroll
+        for (int i = 0; i < 16; ++i) Ti[(b0 + i) * kP + b0 + c] = x[i];
+    }
+    __syncthreads();
+    // ---- below the diagonal, distance by distance: T_ij = -T_ii sum_{j <= k < i} A_ik T_kj; wave j takes column block j.
+    // X holds the transposed sum (the B operand of the second product); T_kj is read as B from row-major T
+    for (int dist = 1; dist < 4; ++dist) {
+        const int jb = wave, ib = jb + dist;
+        if (ib < 4) {
+            f32x4 s = zero4();
+            for (int kb = jb; kb < ib; ++kb) {
+                const f32x4 av = *(const f32x4*)(A + (ib * 16 + c16) * kP + kb * 16 + 4 * g);
+                f32x4 bv;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) bv[j] = Ti[(kb * 16 + 4 * g + j) * kP + jb * 16 + c16];
+                s = mfma4(av, bv, s);
+            }
+            // D: rows 4 g + r, column c16 -> X[column][row]
+            *(f32x4*)(X + (jb * 16 + c16) * kX + 4 * g) = s;
+        }
+        __syncthreads();
+        if (ib < 4) {
+            const f32x4 av = *(const f32x4*)(Ti + (ib * 16 + c16) * kP + ib * 16 + 4 * g);
+            const f32x4 bv = *(const f32x4*)(X + (jb * 16 + c16) * kX + 4 * g);
+            const f32x4 t = mfma4(av, bv, zero4());
+#pragma unroll
+            for (int r = 0; r < 4; ++r) Ti[(ib * 16 + 4 * g + r) * kP + jb * 16 + c16] = -t[r];
+        }
+        __syncthreads();
+    }
+    // ---- U0^T and W: wave w holds rows 16 w .. 16 w + 15 (T is lower triangular: columns up to 16 w + 15)
+    f32x4 ta[4];
+#pragma unroll
+    for (int kb = 0; kb < 4; ++kb) ta[kb] = *(const f32x4*)(Ti + (wave * 16 + c16) * kP + kb * 16 + 4 * g);
+    float* out = p.s.ut + hi * VP * kC;
+    for (int nb = 0; nb < VP / 16; ++nb) {
+        f32x4 acc = zero4();
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb)
+            if (kb <= wave) acc = mfma4(ta[kb], *(const f32x4*)(vt + (nb * 16 + c16) * kP + kb * 16 + 4 * g), acc);
+        *(f32x4*)(out + (nb * 16 + c16) * kC + wave * 16 + 4 * g) = acc;
+    }
+    const float* kt = p.s.kt + gi * DP * kC;
+    float* oW = p.s.W + hi * kC * DP;
+    f32x4 bgv[4];
+#pragma unroll
+    for (int kb = 0; kb < 4; ++kb) bgv[kb] = *(const f32x4*)(bg + kb * 16 + 4 * g);
+    for (int nb = 0; nb < DP / 16; ++nb) {
+        f32x4 acc = zero4();
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb)
+            if (kb <= wave) acc = mfma4(ta[kb], *(const f32x4*)(kt + (nb * 16 + c16) * kC + kb * 16 + 4 * g) * bgv[kb], acc);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) oW[(wave * 16 + 4 * g + r) * DP + nb * 16 + c16] = acc[r];
+    }
+}
+
+// ------------------------------------------------------------------------------------ gla: per head
+// grid (chunks, heads, seqs), 256 threads; key channels in slices of 64.  LDS: q, k, G [64 rows][68], low-rank rows [64][rank], sums
+constexpr int kCh = 64;
+template <typename T>
+__global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
+    const mi355_recurrent_args& a = p.r.a;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, t0 = blockIdx.x * kC;
+    const int cnt = p.r.b.count[seq];
+    if (t0 >= cnt) return;
+    const int DP = p.DP, VP = p.VP, dim = a.dim, rank = a.rank;
+    float* q = sm;
+    float* k = q + kC * kP;
+    float* G = k + kC * kP;
+    float* seg = G + kC * kP;       // [4][64]
+    float* lr = seg + 4 * kCh;      // [64][rank]
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c16 = lane & 15, g = lane >> 4;
+    const T* rows = (const T*)a.proj + (int64_t)(p.r.b.row0[seq] + t0) * a.ld;
+    const int n = min(kC, cnt - t0);
+    const int64_t hi = (int64_t)(chunk_base(p, seq) + blockIdx.x) * a.heads + head;
+    for (int i = tid; i < kC * rank; i += 256) {
+        const int t = i / rank, r = i - t * rank;
+        lr[i] = t < n ? to_f32<T>(rows[(int64_t)t * a.ld + a.off_a + r]) : 0.f;
+    }
+    float* oq = p.s.q + hi * kC * DP;
+    float* okt = p.s.kt + hi * DP * kC;
+    f32x4 off[4];                    // wave w: P blocks (w, 0 .. w - 1)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) off[i] = zero4();
+    float dg[4] = {0.f, 0.f, 0.f, 0.f};  // wave w: rows 4 rr + g of diagonal block w, column c16
+    for (int c0 = 0; c0 < DP; c0 += kCh) {
+        __syncthreads();
+        // ---- decays: thread = (channel, 16-row block)
+        {
+            const int c = tid & 63, sb = tid >> 6, ch = c0 + c;
+            const bool ok = ch < dim;
+            float s = 0.f;
+            const float* w = a.a2 + (int64_t)(head * dim + (ok ? ch : 0)) * rank;
+            const float bias = ok ? a.a2_bias[head * dim + ch] : 0.f;
+            for (int t = sb * 16; t < sb * 16 + 16; ++t) {
+                float la = 0.f, qv = 0.f, kv = 0.f;
+                if (ok && t < n) {
+                    float z = bias;
+                    for (int r = 0; r < rank; ++r) z += w[r] * lr[t * rank + r];
+                    la = -softplus_f32(-z) * a.inv_tau;
+                    qv = to_f32<T>(rows[(int64_t)t * a.ld + a.off_q + head * dim + ch]) * a.q_scale;
+                    kv = to_f32<T>(rows[(int64_t)t * a.ld + a.off_k + head * dim + ch]);
+                }
+                s += la;
+                G[t * kP + c] = s;   // sums from the block's first row on
+                q[t * kP + c] = qv;
+                k[t * kP + c] = kv;
+            }
+            seg[sb * kCh + c] = s;
+        }
+        __syncthreads();
+        // ---- diagonal blocks: wave = block, lane group g and c16 = column j, rows 4 rr + g
+#pragma unroll
+        for (int rr = 0; rr < 4; ++rr) {
+            const int i = wave * 16 + rr * 4 + g, j = wave * 16 + c16;
+            if (j <= i) {
+                float s = 0.f;
+                for (int c = 0; c < kCh; c += 4) {
+                    const f32x4 qi = *(const f32x4*)(q + i * kP + c), kj = *(const f32x4*)(k + j * kP + c);
+                    const f32x4 gi = *(const f32x4*)(G + i * kP + c), gj = *(const f32x4*)(G + j * kP + c);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) s += qi[e] * kj[e] * expf(gi[e] - gj[e]);
+                }
+                dg[rr] += s;
+            }
+        }
+        // ---- off-diagonal blocks (I, J): q_i e^(G_i - start of I) against k_j e^(start of I - G_j)
+        for (int J = 0; J < wave; ++J)
+            for (int cb = 0; cb < kCh; cb += 16) {
+                const int c = cb + 4 * g;
+                const int i = wave * 16 + c16, j = J * 16 + c16;
+                f32x4 gap = *(const f32x4*)(seg + J * kCh + c) - *(const f32x4*)(G + j * kP + c);  // from j to the end of block J
+                for (int m = J + 1; m < wave; ++m) gap += *(const f32x4*)(seg + m * kCh + c);
+                f32x4 av = *(const f32x4*)(q + i * kP + c), bv = *(const f32x4*)(k + j * kP + c);
+                const f32x4 gi = *(const f32x4*)(G + i * kP + c);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    av[e] *= expf(gi[e]);
+                    bv[e] *= expf(gap[e]);
+                }
+#pragma unroll
+                for (int b = 0; b < 3; ++b)  // (constant register index)
+                    if (b == J) off[b] = mfma4(av, bv, off[b]);
+            }
+        // ---- q e^G and (k e^(G_end - G))^T of the slice
+        const int nch = min(kCh, DP - c0);
+        for (int i = tid; i < kC * nch; i += 256) {
+            const int t = i / nch, c = i - t * nch, sb = t >> 4;
+            float before = 0.f;
+            for (int m = 0; m < sb; ++m) before += seg[m * kCh + c];
+            oq[t * DP + c0 + c] = q[t * kP + c] * expf(before + G[t * kP + c]);
+        }
+        for (int i = tid; i < kC * nch; i += 256) {
+            const int c = i >> 6, t = i & 63, sb = t >> 4;
+            float rest = seg[sb * kCh + c] - G[t * kP + c];
+            for (int m = sb + 1; m < 4; ++m) rest += seg[m * kCh + c];
+            okt[(c0 + c) * kC + t] = k[t * kP + c] * expf(rest);
+        }
+        if (tid < nch) p.s.gam[hi * DP + c0 + tid] = expf(seg[tid] + seg[kCh + tid] + seg[2 * kCh + tid] + seg[3 * kCh + tid]);
+    }
+    float* oP = p.s.P + hi * kC * kC;
+#pragma unroll
+    for (int rr = 0; rr < 4; ++rr) oP[(wave * 16 + rr * 4 + g) * kC + wave * 16 + c16] = dg[rr];
+#pragma unroll
+    for (int J = 0; J < 3; ++J)
+        if (J < wave) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) oP[(wave * 16 + 4 * g + r) * kC + J * 16 + c16] = off[J][r];
+        }
+    for (int i = lane; i < 16 * (3 - wave) * 16; i += 64) {  // above the diagonal: zeros
+        const int w = (3 - wave) * 16, r = i / w;
+        oP[(wave * 16 + r) * kC + (wave + 1) * 16 + (i - r * w)] = 0.f;
+    }
+    float* out = p.s.ut + hi * VP * kC;
+    for (int i = tid; i < kC * VP; i += 256) {
+        const int d = i >> 6, t = i & 63;
+        out[i] = d < a.vdim && t < n ? to_f32<T>(rows[(int64_t)t * a.ld + a.off_v + head * a.vdim + d]) : 0.f;
+    }
+}
+
+// ------------------------------------------------------------------------------------ the serial part
+// grid (VP / 16, heads, seqs), 256 threads; NT = 16-row tiles of the state per wave (DP <= 64 NT)
+template <int KIND, int NT>
+__global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
+    const mi355_recurrent_args& a = p.r.a;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, n0 = blockIdx.x * 16;
+    const int DP = p.DP, VP = p.VP, ls = DP + 4;
+    float* sl = sm;            // [16][DP + 4]: S_0 columns
+    float* ul = sm + 16 * ls;  // [16][kP]: U columns, weighted by e^(G_end - G)
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c16 = lane & 15, g = lane >> 4;
+    const int n_chunks = (p.r.b.count[seq] + kC - 1) / kC;
+    const int kvh = KIND == MI355_REC_DELTA ? head / (a.heads / a.kv_heads) : head;
+    float* state = a.state + ((int64_t)p.r.b.slot[seq] * a.heads + head) * a.dim * a.vdim;
+    const int64_t cb = chunk_base(p, seq);
+    const int n_tiles = DP / 16;
+    const bool col_ok = n0 + c16 < a.vdim;
+
+    f32x4 S[NT];
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int i = (wave + 4 * t) * 16 + 4 * g + r;
+            S[t][r] = (col_ok && i < a.dim) ? state[(int64_t)i * a.vdim + n0 + c16] : 0.f;
+        }
+    // a chunk's operands of this wave, requested one chunk ahead
+    f32x4 wr[4 * NT], kr[NT][4], ur, dr, gr[NT], vr[4];
+    auto load = [&](int ch) {
+        const int64_t hi = (cb + ch) * a.heads + head, gi = (cb + ch) * p.GQ + kvh;
+        const float* kt = p.s.kt + gi * DP * kC;
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int row = (wave + 4 * t) * 16 + c16;
+#pragma unroll
+            for (int b = 0; b < 4; ++b) kr[t][b] = wave + 4 * t < n_tiles ? *(const f32x4*)(kt + row * kC + b * 16 + 4 * g) : zero4();
+        }
+        const float* ut = p.s.ut + hi * VP * kC + (int64_t)(n0 + c16) * kC;
+        if constexpr (KIND == MI355_REC_DELTA) {
+            const float* W = p.s.W + hi * kC * DP + (int64_t)(wave * 16 + c16) * DP;
+#pragma unroll
+            for (int b = 0; b < 4 * NT; ++b) wr[b] = b < n_tiles ? *(const f32x4*)(W + b * 16 + 4 * g) : zero4();
+            ur = *(const f32x4*)(ut + wave * 16 + 4 * g);
+            dr = *(const f32x4*)(p.s.ed + hi * kC + wave * 16 + 4 * g);
+            const float gm = p.s.gam[hi * DP];
+            gr[0] = f32x4{gm, gm, gm, gm};
+        } else {
+#pragma unroll
+            for (int b = 0; b < 4; ++b) vr[b] = *(const f32x4*)(ut + b * 16 + 4 * g);
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+                gr[t] = wave + 4 * t < n_tiles ? *(const f32x4*)(p.s.gam + hi * DP + (wave + 4 * t) * 16 + 4 * g) : zero4();
+        }
+    };
+    load(0);
+    for (int ch = 0; ch < n_chunks; ++ch) {
+        const int64_t hi = (cb + ch) * a.heads + head;
+        float* st = p.s.st + hi * VP * DP + (int64_t)(n0 + c16) * DP;
+        // S_0: to the output kernel, and to LDS as the B operand of W S_0
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+            if (wave + 4 * t < n_tiles) {
+                const int i = (wave + 4 * t) * 16 + 4 * g;
+                *(f32x4*)(st + i) = S[t];
+                if constexpr (KIND == MI355_REC_DELTA) *(f32x4*)(sl + c16 * ls + i) = S[t];
+            }
+        if constexpr (KIND == MI355_REC_DELTA) {
+            __syncthreads();
+            f32x4 u = zero4(), u2 = zero4();
+#pragma unroll
+            for (int b = 0; b < 4 * NT; ++b)
+                if (b < n_tiles) {
+                    const f32x4 sv = *(const f32x4*)(sl + c16 * ls + b * 16 + 4 * g);
+                    if (b & 1) u2 = mfma4(wr[b], sv, u2);
+                    else u = mfma4(wr[b], sv, u);
+                }
+            u = ur - (u + u2);
+            *(f32x4*)(p.s.ut + hi * VP * kC + (int64_t)(n0 + c16) * kC + wave * 16 + 4 * g) = u;
+            *(f32x4*)(ul + c16 * kP + wave * 16 + 4 * g) = u * dr;
+            __syncthreads();
+#pragma unroll
+            for (int b = 0; b < 4; ++b) vr[b] = *(const f32x4*)(ul + c16 * kP + b * 16 + 4 * g);
+        }
+        f32x4 kc[NT][4], vc[4];
+#pragma unroll
+        for (int b = 0; b < 4; ++b) vc[b] = vr[b];
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            S[t] *= gr[KIND == MI355_REC_DELTA ? 0 : t];
+#pragma unroll
+            for (int b = 0; b < 4; ++b) kc[t][b] = kr[t][b];
+        }
+        if (ch + 1 < n_chunks) load(ch + 1);
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+            for (int t = 0; t < NT; ++t) S[t] = mfma4(kc[t][b], vc[b], S[t]);
+    }
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int i = (wave + 4 * t) * 16 + 4 * g + r;
+            if (col_ok && i < a.dim) state[(int64_t)i * a.vdim + n0 + c16] = S[t][r];
+        }
+}
+
+// ------------------------------------------------------------------------------------ outputs
+// grid (chunks, heads, seqs), 256 threads: wave w takes the 16-column tiles w, w + 4, ...; NV = tiles per wave (VP <= 64 NV)
+template <typename T, int KIND, int NV>
+__global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
+    const mi355_recurrent_args& a = p.r.a;
+    __shared__ float ssq[4][kC];
+    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, t0 = blockIdx.x * kC;
+    const int cnt = p.r.b.count[seq];
+    if (t0 >= cnt) return;
+    const int DP = p.DP, VP = p.VP;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int c16 = lane & 15, g = lane >> 4;
+    const int kvh = KIND == MI355_REC_DELTA ? head / (a.heads / a.kv_heads) : head;
+    const int64_t ci = chunk_base(p, seq) + blockIdx.x, hi = ci * a.heads + head;
+    const float* q = p.s.q + (ci * p.GQ + kvh) * kC * DP;
+    const float* st = p.s.st + hi * VP * DP;
+    const float* P = p.s.P + hi * kC * kC;
+    const float* ut = p.s.ut + hi * VP * kC;
+    const int n_tiles = VP / 16;
+    f32x4 o[4][NV];
+#pragma unroll
+    for (int rb = 0; rb < 4; ++rb)
+#pragma unroll
+        for (int v = 0; v < NV; ++v) o[rb][v] = zero4();
+    for (int d = 4 * g; d < DP; d += 16) {
+        f32x4 b[NV];
+#pragma unroll
+        for (int v = 0; v < NV; ++v) b[v] = wave + 4 * v < n_tiles ? *(const f32x4*)(st + (int64_t)((wave + 4 * v) * 16 + c16) * DP + d) : zero4();
+#pragma unroll
+        for (int rb = 0; rb < 4; ++rb) {
+            const f32x4 qv = *(const f32x4*)(q + (rb * 16 + c16) * DP + d);
+#pragma unroll
+            for (int v = 0; v < NV; ++v) o[rb][v] = mfma4(qv, b[v], o[rb][v]);
+        }
+    }
+    if constexpr (KIND == MI355_REC_DELTA) {
+#pragma unroll
+        for (int rb = 0; rb < 4; ++rb) {
+            const f32x4 e = *(const f32x4*)(p.s.eg + hi * kC + rb * 16 + 4 * g);
+#pragma unroll
+            for (int v = 0; v < NV; ++v) o[rb][v] *= e;
+        }
+    }
+#pragma unroll
+    for (int kb = 0; kb < 4; ++kb) {
+        f32x4 b[NV];
+#pragma unroll
+        for (int v = 0; v < NV; ++v)
+            b[v] = wave + 4 * v < n_tiles ? *(const f32x4*)(ut + (int64_t)((wave + 4 * v) * 16 + c16) * kC + kb * 16 + 4 * g) : zero4();
+#pragma unroll
+        for (int rb = kb; rb < 4; ++rb) {
+            const f32x4 pv = *(const f32x4*)(P + (rb * 16 + c16) * kC + kb * 16 + 4 * g);
+#pragma unroll
+            for (int v = 0; v < NV; ++v) o[rb][v] = mfma4(pv, b[v], o[rb][v]);
+        }
+    }
+    // ---- output norm over the head's columns, gate
+#pragma unroll
+    for (int rb = 0; rb < 4; ++rb)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            float s = 0.f;
+#pragma unroll
+            for (int v = 0; v < NV; ++v) s += o[rb][v][r] * o[rb][v][r];
+            s = group_sum(s, 16);
+            if (c16 == 0) ssq[wave][rb * 16 + 4 * g + r] = s;
+        }
+    __syncthreads();
+    const T* rows = (const T*)a.proj + (int64_t)(p.r.b.row0[seq] + t0) * a.ld;
+    T* y = (T*)a.y + (int64_t)(p.r.b.row0[seq] + t0) * a.ldy;
+#pragma unroll
+    for (int rb = 0; rb < 4; ++rb)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int t = rb * 16 + 4 * g + r;
+            if (t0 + t >= cnt) continue;
+            const float rinv = 1.0f / sqrtf((ssq[0][t] + ssq[1][t] + ssq[2][t] + ssq[3][t]) / (float)a.vdim + a.eps);
+#pragma unroll
+            for (int v = 0; v < NV; ++v) {
+                const int n = (wave + 4 * v) * 16 + c16;
+                if (n >= a.vdim) continue;
+                const float gate = silu_f32(to_f32<T>(rows[(int64_t)t * a.ld + a.off_g + head * a.vdim + n]));
+                y[(int64_t)t * a.ldy + head * a.vdim + n] = from_f32<T>(o[rb][v][r] * rinv * a.head_norm[n] * gate);
+            }
+        }
+}
+
+inline int pad16(int n) { return (n + 15) / 16 * 16; }
+
+// floats per packed chunk
+size_t chunk_floats(int kind, int heads, int kv_heads, int dim, int vdim) {
+    const size_t DP = pad16(dim), VP = pad16(vdim), H = heads, G = kind == MI355_REC_DELTA ? kv_heads : heads;
+    size_t n = 2 * G * kC * DP + H * kC * kC + H * VP * kC + H * VP * DP + H * DP;
+    if (kind == MI355_REC_DELTA) n += 2 * G * kC * kC + H * kC * DP + 2 * H * kC;
+    return n;
+}
+
+template <typename K>
+int set_lds(K kernel, size_t bytes) {
+    if (bytes > 64 * 1024) {
+        const hipError_t e = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
+        MI355_CHECK_ARG(e == hipSuccess, (int)e, "recurrent: hipFuncSetAttribute(%zu) failed: %s", bytes, hipGetErrorString(e));
+    }
+    return 0;
+}
+
+template <int KIND>
+int launch_scan(const ChunkParams& p, int seqs, hipStream_t s) {
+    const dim3 grid(p.VP / 16, p.r.a.heads, seqs);
+    const size_t lds = ((size_t)16 * (p.DP + 4) + 16 * kP) * 4;
+    if (p.DP <= 64) hipLaunchKernelGGL((scan_kernel<KIND, 1>), grid, dim3(256), lds, s, p);
+    else if (p.DP <= 128) hipLaunchKernelGGL((scan_kernel<KIND, 2>), grid, dim3(256), lds, s, p);
+    else hipLaunchKernelGGL((scan_kernel<KIND, 4>), grid, dim3(256), lds, s, p);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+
+template <typename T, int KIND>
+int launch_out(const ChunkParams& p, dim3 grid, hipStream_t s) {
+    if (p.VP <= 64) hipLaunchKernelGGL((chunk_out_kernel<T, KIND, 1>), grid, dim3(256), 0, s, p);
+    else if (p.VP <= 128) hipLaunchKernelGGL((chunk_out_kernel<T, KIND, 2>), grid, dim3(256), 0, s, p);
+    else hipLaunchKernelGGL((chunk_out_kernel<T, KIND, 4>), grid, dim3(256), 0, s, p);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+
+template <typename T>
+int run_group(const ChunkParams& p, int seqs, hipStream_t s) {
+    const mi355_recurrent_args& a = p.r.a;
+    const int chunks = (p.r.b.max_count + kC - 1) / kC;
+    const dim3 heads(chunks, a.heads, seqs);
+    if (a.kind == MI355_REC_DELTA) {
+        const size_t lds1 = (size_t)2 * kC * (p.DP + 4) * 4;
+        if (int rc = set_lds(delta_qk_kernel<T>, lds1)) return rc;
+        hipLaunchKernelGGL(delta_qk_kernel<T>, dim3(chunks, a.kv_heads, seqs), dim3(256), lds1, s, p);
+        MI355_LAUNCH_CHECK();
+        const size_t lds2 = ((size_t)2 * kC * kP + (size_t)kC * kX + (size_t)p.VP * kP) * 4;
+        if (int rc = set_lds(delta_head_kernel<T>, lds2)) return rc;
+        hipLaunchKernelGGL(delta_head_kernel<T>, heads, dim3(256), lds2, s, p);
+        MI355_LAUNCH_CHECK();
+        if (int rc = launch_scan<MI355_REC_DELTA>(p, seqs, s)) return rc;
+        return launch_out<T, MI355_REC_DELTA>(p, heads, s);
+    }
+    const size_t lds = ((size_t)3 * kC * kP + 4 * kCh + (size_t)kC * a.rank) * 4;
+    if (int rc = set_lds(gla_prep_kernel<T>, lds)) return rc;
+    hipLaunchKernelGGL(gla_prep_kernel<T>, heads, dim3(256), lds, s, p);
+    MI355_LAUNCH_CHECK();
+    if (int rc = launch_scan<MI355_REC_GLA>(p, seqs, s)) return rc;
+    return launch_out<T, MI355_REC_GLA>(p, heads, s);
+}
+
+}  // namespace
+
+bool mi355_recurrent_chunks_fit(const mi355_recurrent_args& a, const mi355_seq_batch& b) {
+    if (a.dim > 256 || a.vdim > 256 || a.scratch == nullptr) return false;
+    return a.scratch_bytes / (chunk_floats(a.kind, a.heads, a.kv_heads, a.dim, a.vdim) * 4) >= (uint64_t)b.rows / kC + 1;
+}
+
+int mi355_recurrent_chunks(const RecParams& r, hipStream_t s) {
+    const mi355_recurrent_args& a = r.a;
+    ChunkParams p;
+    p.r = r;
+    p.DP = pad16(a.dim);
+    p.VP = pad16(a.vdim);
+    p.GQ = a.kind == MI355_REC_DELTA ? a.kv_heads : a.heads;
+    const size_t per = chunk_floats(a.kind, a.heads, a.kv_heads, a.dim, a.vdim);
+    // packed chunks of n sequences: at most rows / 64 + n (chunk_base)
+    const size_t cap = a.scratch_bytes / (per * 4);
+    const size_t most = cap - (size_t)r.b.rows / kC;  // >= 1 (mi355_recurrent_chunks_fit)
+    const size_t H = a.heads, G = p.GQ, DP = p.DP, VP = p.VP;
+    float* f = a.scratch;
+    auto take = [&](size_t n) {
+        float* q = f;
+        f += n * cap;
+        return q;
+    };
+    const bool delta = a.kind == MI355_REC_DELTA;
+    p.s.q = take(G * kC * DP);
+    p.s.kt = take(G * kC * DP);
+    p.s.kk = delta ? take(G * kC * kC) : nullptr;
+    p.s.qk = delta ? take(G * kC * kC) : nullptr;
+    p.s.P = take(H * kC * kC);
+    p.s.W = delta ? take(H * kC * DP) : nullptr;
+    p.s.ut = take(H * VP * kC);
+    p.s.st = take(H * VP * DP);
+    p.s.gam = take(H * DP);
+    p.s.eg = delta ? take(H * kC) : nullptr;
+    p.s.ed = delta ? take(H * kC) : nullptr;
+    for (int s0 = 0; s0 < r.b.seqs; s0 += (int)most) {
+        const int n = (size_t)(r.b.seqs - s0) < most ? r.b.seqs - s0 : (int)most;
+        p.seq0 = s0;
+        if (int rc = a.dtype == MI355_F32 ? run_group<float>(p, n, s) : run_group<bf16_t>(p, n, s)) return rc;
+    }
+    return 0;
+}
+
+extern "C" size_t mi355_recurrent_scratch_bytes(int kind, int rows, int seqs, int heads, int kv_heads, int dim, int vdim) {
+    if (rows < 1 || seqs < 1 || heads < 1 || kv_heads < 1 || dim < 1 || vdim < 1 || dim > 256 || vdim > 256) return 0;
+    return chunk_floats(kind, heads, kv_heads, dim, vdim) * 4 * ((size_t)rows / kC + seqs);
+}

@@ -331,6 +331,271 @@ __global__ __launch_bounds__(256) void ring_write_kernel(const WinParams p) {
     }
 }
 
+// ------------------------------------------------------------------------------------ matrix-core tiles (bf16 prompt steps)
+// One workgroup: 128 queries of one head, four waves of 32.  Keys in steps of 64: S^T = K Q^T and O^T += V^T P^T on 32x32x16 MFMAs, so a
+// lane holds scores and outputs of ONE query (its column).  A key step's K tile [64][D] (16-B columns XOR-swizzled by the key) and V tile
+// (transposed to [D][64 keys], the runs of four keys permuted to the order in which a lane's score registers hold them) are loaded into
+// registers while the step before is multiplied; keys of earlier portions come from the ring, the rest from the step's own rows.
+constexpr int kBQ = 128, kBK = 64;
+constexpr int kVtRow = 2 * kBK + 16;  // bytes per row of the transposed V tile
+
+__device__ __forceinline__ uint32_t pack_bf16x2(float a, float b) {
+    const bf16x2_t v = {(__bf16)a, (__bf16)b};
+    return __builtin_bit_cast(uint32_t, v);
+}
+__device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
+
+template <int D>  // both head sizes padded to D (a multiple of 32)
+constexpr int tiles_lds() { return 2 * (kBK * D * 2 + D * kVtRow); }
+
+template <int D>
+__global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(const WinParams p) {
+    const mi355_window_attn_args& a = p.a;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    constexpr int kCols = D / 8;                       // 16-B columns of a key row
+    constexpr int kKItems = kBK * kCols / 256;         // K chunks per thread
+    constexpr int kVItems = (16 * kCols + 255) / 256;  // V items per thread: (run of 4 keys, column)
+    constexpr int kKTile = kBK * D * 2, kVTile = D * kVtRow;
+    constexpr int kSwz = kCols < 16 ? kCols - 1 : 15;
+    const int seq = blockIdx.z;
+    const int cnt = p.b.count[seq];
+    // an XCD (block index mod 8) takes the query blocks of neighbouring heads: their key head stays in its L2
+    const int q_blocks = (p.b.max_count + kBQ - 1) / kBQ;
+    const int id = (blockIdx.x & 7) * (gridDim.x >> 3) + (blockIdx.x >> 3);  // (the grid is a multiple of 8)
+    if (id >= q_blocks * a.heads) return;
+    const int h = id / q_blocks, qb = q_blocks - 1 - id % q_blocks;
+    if (qb * kBQ >= cnt) return;
+    const int kvh = h / (a.heads / a.kv_heads);
+    const int row0 = p.b.row0[seq], pos0 = p.b.pos[seq];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int hh = lane >> 5, c = lane & 31;
+    const int qi = qb * kBQ + wave * 32 + c;
+    const bool q_ok = qi < cnt;
+    const int q_row = q_ok ? qi : cnt - 1;
+    const int q_pos = pos0 + q_row;
+    const bf16_t* proj = (const bf16_t*)a.proj;
+    const int q_first = pos0 + qb * kBQ, q_last = pos0 + min(qb * kBQ + kBQ, cnt) - 1;
+    const int kb0 = max(0, q_first - a.window + 1) / kBK, kb1 = q_last / kBK + 1;
+    // the wave's own range, for the masks
+    const int w_first = min(pos0 + qb * kBQ + wave * 32, pos0 + cnt - 1), w_last = min(w_first + 31, pos0 + cnt - 1);
+
+    // ---- Q^T operands: q[16 ks + 8 hh .. + 8), rotated, scaled to the exp2 domain, rounded once
+    bf16x8 bq[D / 16];
+    {
+        const bf16_t* src = proj + (int64_t)(row0 + q_row) * a.ld + a.off_q + (int64_t)h * a.dim;
+        const float qs = a.scale * 1.44269504088896340736f;
+#pragma unroll
+        for (int ks = 0; ks < D / 16; ++ks) {
+            const int d0 = 16 * ks + 8 * hh;
+            u32x4 o = {0u, 0u, 0u, 0u};
+            if (d0 < a.dim) {  // (dim % 8 == 0)
+                float v[8];
+                load_vec<bf16_t, 8>(src + d0, v);
+#pragma unroll
+                for (int e = 0; e < 8; e += 2) {
+                    float u = v[e], w = v[e + 1];
+                    if (d0 + e < a.rot_dims) {
+                        float cs, sn;
+                        pair_cos_sin(q_pos, a.inv_freq[(d0 + e) >> 1], cs, sn);
+                        const float r = u * cs - w * sn;
+                        w = w * cs + u * sn;
+                        u = r;
+                    }
+                    o[e >> 1] = pack_bf16x2(u * qs, w * qs);
+                }
+            }
+            bq[ks] = __builtin_bit_cast(bf16x8, o);
+        }
+    }
+    const int64_t slot_head = (int64_t)p.b.slot[seq] * a.kv_heads + kvh;
+    const bf16_t* kring = (const bf16_t*)a.kring + slot_head * a.ring * a.dim;
+    const bf16_t* vring = (const bf16_t*)a.vring + slot_head * a.ring * a.vdim;
+    const bf16_t* kcur = proj + (int64_t)row0 * a.ld + a.off_k + (int64_t)kvh * a.dim;
+    const bf16_t* vcur = proj + (int64_t)row0 * a.ld + a.off_v + (int64_t)kvh * a.vdim;
+    const int p_last = pos0 + cnt - 1;
+    u32x4 kreg[kKItems], vreg[kVItems][4];
+    const u32x4 zero4 = {0u, 0u, 0u, 0u};
+    auto load_tile = [&](int kb) {
+#pragma unroll
+        for (int i = 0; i < kKItems; ++i) {
+            const int it = i * 256 + threadIdx.x, key = it / kCols, col = it % kCols;
+            const int kp = kb * kBK + key;
+            kreg[i] = zero4;
+            if (col * 8 < a.dim && kp <= p_last) {
+                const bf16_t* src = kp >= pos0 ? kcur + (int64_t)(kp - pos0) * a.ld : kring + (int64_t)(kp % a.ring) * a.dim;
+                kreg[i] = *(const u32x4*)(src + col * 8);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < kVItems; ++i) {
+            const int it = i * 256 + threadIdx.x, run = it & 15, col = it >> 4;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int kp = kb * kBK + run * 4 + r;
+                vreg[i][r] = zero4;
+                if (col < kCols && col * 8 < a.vdim && kp <= p_last) {
+                    const bf16_t* src = kp >= pos0 ? vcur + (int64_t)(kp - pos0) * a.ld : vring + (int64_t)(kp % a.ring) * a.vdim;
+                    vreg[i][r] = *(const u32x4*)(src + col * 8);
+                }
+            }
+        }
+    };
+    auto store_tile = [&](int buf) {
+        char* kt = smem + buf * kKTile;
+        char* vt = smem + 2 * kKTile + buf * kVTile;
+#pragma unroll
+        for (int i = 0; i < kKItems; ++i) {
+            const int it = i * 256 + threadIdx.x, key = it / kCols, col = it % kCols;
+            *(u32x4*)(kt + key * (D * 2) + ((col ^ (key & kSwz)) << 4)) = kreg[i];
+        }
+#pragma unroll
+        for (int i = 0; i < kVItems; ++i) {
+            const int it = i * 256 + threadIdx.x, run = it & 15, col = it >> 4;
+            if (col >= kCols) continue;
+            const int G = run >> 2, r = run & 3;
+            const int pbyte = (G * 16 + 4 * ((r & 1) * 2 + (r >> 1))) * 2;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const int dw = e >> 1;
+                u32x2 o;
+                if (e & 1) {
+                    o[0] = __builtin_amdgcn_perm(vreg[i][1][dw], vreg[i][0][dw], 0x07060302u);
+                    o[1] = __builtin_amdgcn_perm(vreg[i][3][dw], vreg[i][2][dw], 0x07060302u);
+                } else {
+                    o[0] = __builtin_amdgcn_perm(vreg[i][1][dw], vreg[i][0][dw], 0x05040100u);
+                    o[1] = __builtin_amdgcn_perm(vreg[i][3][dw], vreg[i][2][dw], 0x05040100u);
+                }
+                *(u32x2*)(vt + (col * 8 + e) * kVtRow + pbyte) = o;
+            }
+        }
+    };
+    f32x16 acc[D / 32];
+#pragma unroll
+    for (int dt = 0; dt < D / 32; ++dt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) acc[dt][i] = 0.f;
+    float m_run = -1.0e30f, l_run = 0.f;
+
+    load_tile(kb0);
+    store_tile(0);
+    __syncthreads();
+    for (int kb = kb0; kb < kb1; ++kb) {
+        const int buf = (kb - kb0) & 1;
+        if (kb + 1 < kb1) load_tile(kb + 1);
+        const char* kt = smem + buf * kKTile;
+        const char* vt = smem + 2 * kKTile + buf * kVTile;
+        // a wave none of whose queries sees this step leaves it out (it still stages the next tile)
+        const bool seen = kb * kBK <= w_last && kb * kBK + kBK - 1 > w_first - a.window;
+        if (seen) {
+            f32x16 st[2];
+#pragma unroll
+            for (int t2 = 0; t2 < 2; ++t2)
+#pragma unroll
+                for (int i = 0; i < 16; ++i) st[t2][i] = 0.f;
+#pragma unroll
+            for (int ks = 0; ks < D / 16; ++ks)
+#pragma unroll
+                for (int t2 = 0; t2 < 2; ++t2) {
+                    const int key = t2 * 32 + c;
+                    const bf16x8 ka = *(const bf16x8*)(kt + key * (D * 2) + (((2 * ks + hh) ^ (key & kSwz)) << 4));
+                    st[t2] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka, bq[ks], st[t2], 0, 0, 0);
+                }
+            if (kb * kBK + kBK - 1 > w_first || kb * kBK <= w_last - a.window) {  // wave-uniform: the step touches an edge
+#pragma unroll
+                for (int t2 = 0; t2 < 2; ++t2)
+#pragma unroll
+                    for (int i = 0; i < 16; ++i) {
+                        const int kp = kb * kBK + t2 * 32 + (i & 3) + 8 * (i >> 2) + 4 * hh;
+                        st[t2][i] = (kp <= q_pos && kp > q_pos - a.window) ? st[t2][i] : -1.0e30f;
+                    }
+            }
+            float m_blk = -1.0e30f;
+#pragma unroll
+            for (int t2 = 0; t2 < 2; ++t2)
+#pragma unroll
+                for (int i = 0; i < 16; ++i) m_blk = fmaxf(m_blk, st[t2][i]);
+            m_blk = fmaxf(m_blk, lane_xor32(m_blk));
+            // the reference maximum moves only when it is exceeded by 2^8 (exp2 domain): few steps rescale the outputs.  (A query whose
+            // first keys are all masked sums ones at m = -1e30; its first visible key moves m and wipes them out with exp2(-1e30) = 0.)
+            const bool move = m_blk > m_run + 8.0f;
+            if (__any(move)) {
+                const float m_new = move ? m_blk : m_run;
+                const float corr = exp2_fast(m_run - m_new);
+                l_run *= corr;
+                m_run = m_new;
+#pragma unroll
+                for (int dt = 0; dt < D / 32; ++dt)
+#pragma unroll
+                    for (int i = 0; i < 16; ++i) acc[dt][i] *= corr;
+            }
+            u32x4 pb[2][2];
+            float psum = 0.f;
+#pragma unroll
+            for (int t2 = 0; t2 < 2; ++t2)
+#pragma unroll
+                for (int i = 0; i < 8; ++i) {
+                    const float p0 = exp2_fast(st[t2][2 * i] - m_run), p1 = exp2_fast(st[t2][2 * i + 1] - m_run);
+                    psum += p0 + p1;
+                    pb[t2][i >> 2][i & 3] = pack_bf16x2(p0, p1);
+                }
+            l_run += psum;
+#pragma unroll
+            for (int sg = 0; sg < 4; ++sg) {
+                const bf16x8 pf = __builtin_bit_cast(bf16x8, pb[sg >> 1][sg & 1]);
+#pragma unroll
+                for (int dt = 0; dt < D / 32; ++dt) {
+                    const bf16x8 va = *(const bf16x8*)(vt + (dt * 32 + c) * kVtRow + sg * 32 + hh * 16);
+                    acc[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(va, pf, acc[dt], 0, 0, 0);
+                }
+            }
+        }
+        if (kb + 1 < kb1) store_tile(buf ^ 1);
+        __syncthreads();
+    }
+    const float l = l_run + lane_xor32(l_run);
+    if (q_ok) {
+        float inv = 1.0f / l;
+        if (a.off_g >= 0) inv /= 1.0f + expf(-bf16_to_f32(proj[(int64_t)(row0 + q_row) * a.ld + a.off_g + h]));
+        bf16_t* y = (bf16_t*)a.y + (int64_t)(row0 + q_row) * a.ldy + (int64_t)h * a.vdim;
+#pragma unroll
+        for (int dt = 0; dt < D / 32; ++dt)
+#pragma unroll
+            for (int g = 0; g < 4; ++g) {
+                const int d = dt * 32 + 8 * g + 4 * hh;
+                if (d < a.vdim) {  // (vdim % 8 == 0)
+                    u32x2 o;
+                    o[0] = pack_bf16x2(acc[dt][4 * g] * inv, acc[dt][4 * g + 1] * inv);
+                    o[1] = pack_bf16x2(acc[dt][4 * g + 2] * inv, acc[dt][4 * g + 3] * inv);
+                    *(u32x2*)(y + d) = o;
+                }
+            }
+    }
+}
+
+template <int D>
+int launch_tiles(const WinParams& p, hipStream_t s) {
+    static hipError_t e = hipFuncSetAttribute((const void*)window_tiles_kernel<D>, hipFuncAttributeMaxDynamicSharedMemorySize, tiles_lds<D>());
+    MI355_CHECK_ARG(e == hipSuccess, (int)e, "window_attention: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
+    const int q_blocks = (p.b.max_count + kBQ - 1) / kBQ;
+    hipLaunchKernelGGL(window_tiles_kernel<D>, dim3((q_blocks * p.a.heads + 7) / 8 * 8, 1, p.b.seqs), dim3(256), tiles_lds<D>(), s, p);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+
+bool tiles_fit(const mi355_window_attn_args& a) {
+    return a.dtype == MI355_BF16 && a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 256 && a.vdim <= 256 && a.ld % 8 == 0 && a.ldy % 4 == 0 &&
+           a.off_q % 8 == 0 && a.off_k % 8 == 0 && a.off_v % 8 == 0 && (uintptr_t)a.proj % 16 == 0 && (uintptr_t)a.kring % 16 == 0 &&
+           (uintptr_t)a.vring % 16 == 0 && (uintptr_t)a.y % 8 == 0;
+}
+
+int run_tiles(const WinParams& p, hipStream_t s) {
+    const int d = p.a.dim > p.a.vdim ? p.a.dim : p.a.vdim;
+    if (d <= 32) return launch_tiles<32>(p, s);
+    if (d <= 64) return launch_tiles<64>(p, s);
+    if (d <= 128) return launch_tiles<128>(p, s);
+    return launch_tiles<256>(p, s);
+}
+
 template <typename T, int HT, int VE>
 int launch_rows(const WinParams& p, int rows, hipStream_t s) {
     const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + (size_t)HT * kKeys + (size_t)kRowThreads * VE + 3 * HT) * 4;
@@ -390,7 +655,14 @@ int run(WinParams p, hipStream_t s) {
         MI355_LAUNCH_CHECK();
     }
     p.n_split = 1;
-    if (int rc = run_rows<T>(p, s)) return rc;
+    // (a handful of rows per sequence would leave most of a 128-query tile empty)
+    const bool tiles = a.path == 2 || (a.path == 0 && p.b.max_count > 8);
+    if (tiles && tiles_fit(a)) {
+        if (int rc = run_tiles(p, s)) return rc;
+    } else {
+        MI355_CHECK_ARG(a.path != 2, MI355_E_SHAPE, "window_attention: the tile kernel takes bf16 heads of up to 256, multiples of 8");
+        if (int rc = run_rows<T>(p, s)) return rc;
+    }
     hipLaunchKernelGGL(ring_write_kernel<T>, dim3(p.b.max_count < a.ring ? p.b.max_count : a.ring, p.b.seqs), dim3(256), 0, s, p);
     MI355_LAUNCH_CHECK();
     return 0;

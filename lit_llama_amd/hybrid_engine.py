@@ -163,7 +163,7 @@ class HybridEngine:
         # a split attention step keeps one record per (row, head, split); one split takes none
         n = max([512 * (l.attn.vdim + 2) * max(8, l.attn.heads // l.attn.kv_heads) for l in ls if l.mixer == 0], default=0)
         M.partials, M.partials_bytes = ptr(self._buf(n, torch.float32)), n * 4
-        n = max([int(lib().mi355_recurrent_scratch_bytes(l.rec.kind, R, min(R, 1024), l.rec.heads, l.rec.kv_heads, l.rec.dim, l.rec.vdim))
+        n = max([int(lib().mi355_recurrent_scratch_bytes(l.rec.kind, R, 64, l.rec.heads, l.rec.kv_heads, l.rec.dim, l.rec.vdim))
                  for l in ls if l.mixer != 0], default=0)
         M.rec_scratch, M.rec_scratch_bytes = ptr(self._buf(n, torch.uint8)), n
         self.logits_buf = self._buf(self.max_logits_rows * M.ld_logits, torch.float32).view(self.max_logits_rows, M.ld_logits)

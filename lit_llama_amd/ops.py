@@ -603,3 +603,71 @@ def gptq_block(W1: torch.Tensor, Hinv1: torch.Tensor, scale: torch.Tensor, zero:
                                  scale.stride(0), 1 if per_col else 0, int(maxq), ptr(Q1), ptr(E1), ptr(L1), count,
                                  stream_ptr()), "mi355_gptq_block")
     return Q1, E1, L1
+
+
+# ------------------------------------------------------------------------------------------ layered hybrid models
+class PackedBatch:
+    """The packed rows of a step: counts, slots and first positions of its sequences (mi355_seq_batch)."""
+
+    def __init__(self, counts, slots, pos, device):
+        row0 = [sum(counts[:i]) for i in range(len(counts))]
+        self.meta = torch.tensor([row0, list(counts), list(slots), list(pos)], dtype=torch.int32, device=device)
+        self.rows = sum(counts)
+        b = self.c = nat.SeqBatch()
+        b.rows, b.seqs, b.max_count = self.rows, len(counts), max(counts)
+        b.row0, b.count, b.slot, b.pos = (ptr(self.meta[i]) for i in range(4))
+
+
+def window_attention(proj: torch.Tensor, batch: PackedBatch, kring: torch.Tensor, vring: torch.Tensor, *, heads: int, scale: float, window: int,
+                     off_q: int, off_k: int, off_v: int, off_g: int = -1, inv_freq: Optional[torch.Tensor] = None, path: int = 0,
+                     partials: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """mi355_window_attention: proj [rows, ld] (k rotated in place by prompt steps), rings [slots, kv_heads, ring, dim | vdim] (written)."""
+    require_gpu(proj, "window_attention")
+    _, G, ring, dim = kring.shape
+    vdim = vring.shape[3]
+    assert proj.dim() == 2 and proj.is_contiguous() and kring.is_contiguous() and vring.is_contiguous() and vring.shape[:3] == kring.shape[:3]
+    assert proj.shape[0] == batch.rows and proj.dtype == kring.dtype == vring.dtype
+    assert off_q + heads * dim <= proj.shape[1] and off_k + G * dim <= proj.shape[1] and off_v + G * vdim <= proj.shape[1]
+    y = torch.zeros((batch.rows, heads * vdim), dtype=proj.dtype, device=proj.device)
+    a = nat.WindowAttnArgs()
+    a.proj, a.ld, a.dtype = ptr(proj), proj.shape[1], dtype_code(proj.dtype)
+    a.heads, a.kv_heads, a.dim, a.vdim = heads, G, dim, vdim
+    a.off_q, a.off_k, a.off_v, a.off_g = off_q, off_k, off_v, off_g
+    a.scale, a.window, a.ring, a.path = scale, window, ring, path
+    if inv_freq is not None:
+        assert inv_freq.dtype == torch.float64
+        a.rot_dims, a.inv_freq = 2 * inv_freq.numel(), ptr(inv_freq)
+    a.kring, a.vring, a.y, a.ldy = ptr(kring), ptr(vring), ptr(y), y.shape[1]
+    if partials is not None:
+        a.partials, a.partials_bytes = ptr(partials), partials.numel() * partials.element_size()
+    check(lib().mi355_window_attention(C.byref(a), C.byref(batch.c), stream_ptr()), "mi355_window_attention")
+    return y
+
+
+def recurrent(kind: str, proj: torch.Tensor, batch: PackedBatch, state: torch.Tensor, *, off: dict, kv_heads: int, head_norm: torch.Tensor,
+              eps: float, conv_ring: Optional[torch.Tensor] = None, conv=None, a_log=None, dt_bias=None, a2=None, a2_bias=None,
+              tau: float = 1.0, path: int = 0) -> torch.Tensor:
+    """mi355_recurrent: `kind` delta | gla, state [slots, heads, dim, vdim] f32 (updated), `off`: first columns of q, k, v, g, a (and b);
+    `conv`: the (q, k, v) taps of the delta rule, f32 [channels, taps]."""
+    require_gpu(proj, "recurrent")
+    _, H, dim, vdim = state.shape
+    y = torch.zeros((batch.rows, H * vdim), dtype=proj.dtype, device=proj.device)
+    r = nat.RecurrentArgs()
+    r.kind, r.dtype = (0 if kind == "delta" else 1), dtype_code(proj.dtype)
+    r.proj, r.ld = ptr(proj), proj.shape[1]
+    r.heads, r.kv_heads, r.dim, r.vdim = H, kv_heads, dim, vdim
+    r.off_q, r.off_k, r.off_v, r.off_g, r.off_a = (off[n] for n in "qkvga")
+    r.q_scale, r.eps, r.unit_eps, r.path = dim ** -0.5, eps, 1e-6, path
+    r.head_norm, r.state, r.y, r.ldy = ptr(head_norm), ptr(state), ptr(y), y.shape[1]
+    if kind == "delta":
+        assert conv_ring.dtype == proj.dtype and conv_ring.shape[2] == 2 * kv_heads * dim + H * vdim
+        r.off_b, r.taps = off["b"], conv[0].shape[1]
+        r.conv_q, r.conv_k, r.conv_v = (ptr(t) for t in conv)
+        r.a_log, r.dt_bias, r.conv_ring = ptr(a_log), ptr(dt_bias), ptr(conv_ring)
+    else:
+        r.rank, r.inv_tau, r.a2, r.a2_bias = a2.shape[1], 1.0 / tau, ptr(a2), ptr(a2_bias)
+    need = int(lib().mi355_recurrent_scratch_bytes(r.kind, batch.rows, batch.c.seqs, H, kv_heads, dim, vdim))
+    scratch = torch.empty(max(need, 4), dtype=torch.uint8, device=proj.device)
+    r.scratch, r.scratch_bytes = ptr(scratch), need
+    check(lib().mi355_recurrent(C.byref(r), C.byref(batch.c), stream_ptr()), "mi355_recurrent")
+    return y

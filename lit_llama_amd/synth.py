@@ -286,3 +286,48 @@ def fill_tp_shard_random_int4(model, seed: int, rank: int, zero: float = 7.5, ga
                 sc = (7.2 / 15.0) * (gain / 2.2) * K_full**-0.5 * (1.0 + 0.1 * torch.rand((N, 1), generator=g, device=dev))
                 mod.scales.copy_(sc.to(mod.scales.dtype))
                 mod.zeros.fill_(zero)  # (zero-mean weights: see fill_model_random_int4)
+
+
+# ---------------------------------------------------------------------------------------- layered hybrid models
+def hybrid_bench_config(width: int, n_layer: int, vocab: int = 32000, window: int = 2048) -> dict:
+    """A hybrid configuration with the parameter count per layer of a LLaMA of the same width: attention | gla | attention | delta layers in
+    turn, heads of 128, every layer with a squared-ReLU feed-forward of 1.5 x the LLaMA's hidden size (two matrices instead of three)."""
+    heads = width // 128
+    hidden = LLaMAConfig(n_embd=width, n_head=heads).n_hidden
+    mixers = [
+        ("attention", {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "rot": {"base": 1e4, "dims": 128},
+                       "scale": 128 ** -0.5, "mask": {"size": window}}),
+        ("gla", {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0}),
+        ("attention", {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "rot": {"base": 1e4, "dims": 64},
+                       "scale": 128 ** -0.5, "mask": {"size": window // 2}}),
+        ("delta", {"heads": heads, "kv_heads": max(1, heads // 2), "dim": 128, "vdim": 128, "conv": 4}),
+    ]
+    layers = [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": hidden * 3 // 2}} for t, m in (mixers[i % 4] for i in range(n_layer))]
+    return {"architecture": "Sekulorn", "layers": layers, "loop": None, "norm": {"eps": 1e-5}, "residual_mult": 1.0, "vocab": vocab, "width": width}
+
+
+def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: torch.dtype = torch.bfloat16, rank: int = 16):
+    """Random weights of a hybrid configuration: unit-gain projections, decays around 0.9, so that far tokens still count."""
+    from .hybrid import HybridConfig, tensor_shapes
+
+    cfg = HybridConfig.from_dict(config)
+    gen = torch.Generator(device=device)
+    gen.manual_seed(seed)
+    ranks = {i: rank for i in range(len(cfg.layers))}
+    out = {}
+    for name, shape in tensor_shapes(cfg, ranks).items():
+        leaf = name.split(".", 1)[-1]
+        t = torch.randn(shape, generator=gen, device=device, dtype=torch.float32)
+        if leaf in ("norm1", "norm2", "norm") or leaf.endswith(".norm"):
+            t = 1.0 + 0.1 * t
+        elif leaf.endswith(".conv"):
+            t = t * 0.2
+            t[:, -1] += 0.7
+        elif leaf.endswith("A_log"):
+            t = t * 0.3 - 2.0
+        elif leaf.endswith(("dt_bias", "a2.b")):
+            t = t * 0.5 + (2.0 if leaf.endswith("a2.b") else 0.0)
+        elif name != "embed":
+            t = t * shape[-1] ** -0.5
+        out[name] = t.to(dtype)
+    return out
