@@ -109,6 +109,7 @@ struct GemmParams {
     int ksplit;
     float* part;
     int relu2;             // STORE: max(y, 0)^2
+    float alpha;           // factor of the product where rinv is NULL (an operand that needed no staging)
     // grouped scales (GRP kernels): gtab[group 0..n_groups][r][tab_ld rows] = bf16 scale | bf16 zero << 16 (row n_groups
     // is all zero), sxt[group][M] = operand sums per group; upg = 128-column units per group (groups of >= 128 columns)
     const uint32_t* gtab;
@@ -825,8 +826,8 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
             ri = fr[tt * 16 + c];
             sxm = fr[BM + tt * 16 + c];
         } else {
-            sxm = GRP ? 0.f : p.sx[(int64_t)m * p.ksplit + ks];
-            ri = p.rinv[m];
+            sxm = (GRP || FMT == MI355_W_BF16) ? 0.f : p.sx[(int64_t)m * p.ksplit + ks];  // (BF16 weights have no zero point)
+            ri = p.rinv != nullptr ? p.rinv[m] : p.alpha;
         }
         float v[kTPW][4];
 #pragma unroll
@@ -1236,6 +1237,9 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
     }
     float* part = (float*)((char*)workspace + (size_t)a->M * kp * 2 + (size_t)a->M * 4 * (1 + kMaxSplit) + 256);
     part = (float*)(((uintptr_t)part + 15) & ~(uintptr_t)15);
+    // a bf16 operand in front of BF16 weights, whole units of it and no norm: multiplied where it lies
+    const bool direct = !fused && !q4 && a->norm_scale == nullptr && a->x_dtype == MI355_BF16 && a->K % 128 == 0 && a->ldx % 8 == 0 &&
+                        (uintptr_t)a->x % 16 == 0;
     GemmParams p;
     memset(&p, 0, sizeof(p));
     if (grouped) {
@@ -1258,7 +1262,7 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
         p.gq_shift = gq_shift;
         p.upg = a->group_cols >= 128 ? a->group_cols / 128 : 1;
         p.tab_ld = tab_ld;
-    } else if (!f_in) {
+    } else if (!f_in && !direct) {
         hipLaunchKernelGGL(stage_rows_kernel, dim3(a->M), dim3(256), 0, s, a->x, a->x_dtype, a->ldx, a->norm_scale, a->norm_dtype,
                            a->eps, a->K, kp, xb, (int64_t)kp, rinv, sx, ksplit, a->alpha == 0.f ? 1.f : a->alpha);
         MI355_LAUNCH_CHECK();
@@ -1269,11 +1273,12 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
         MI355_CHECK_ARG(wb > 0 && wb < 0xFFFFFFF0ull, MI355_E_SHAPE, "linear_gemm: weight stream of %zu B", wb);
         p.w_bytes = (unsigned)wb;
     }
-    MI355_CHECK_ARG((size_t)a->M * (f_in ? (size_t)a->ldx : (size_t)kp) * 2 < 0xFFFFFFF0ull, MI355_E_SHAPE,
+    MI355_CHECK_ARG((size_t)a->M * (f_in || direct ? (size_t)a->ldx : (size_t)kp) * 2 < 0xFFFFFFF0ull, MI355_E_SHAPE,
                     "linear_gemm: M x K too large for one launch");
-    p.xb = f_in ? (const bf16_t*)a->x : xb;
-    p.ldxb = f_in ? a->ldx : (int64_t)kp;
-    p.rinv = rinv;
+    p.xb = f_in || direct ? (const bf16_t*)a->x : xb;
+    p.ldxb = f_in || direct ? a->ldx : (int64_t)kp;
+    p.rinv = direct ? nullptr : rinv;
+    p.alpha = a->alpha == 0.f ? 1.f : a->alpha;
     p.sx = sx;
     p.scales = a->scales;
     p.zeros = a->zeros;

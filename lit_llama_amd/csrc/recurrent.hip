@@ -81,6 +81,7 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
             for (int d = tid; d < dim; d += nt) {
                 const int c = head * dim + d;
                 float z = a.a2_bias[c];
+#pragma unroll 8
                 for (int r = 0; r < a.rank; ++r) z += a.a2[(int64_t)c * a.rank + r] * lr[r];
                 al[d] = expf(-softplus_f32(-z) * a.inv_tau);
                 q[d] = to_f32<T>(row[a.off_q + c]) * a.q_scale;

@@ -75,16 +75,20 @@ __global__ __launch_bounds__(256) void delta_qk_kernel(const ChunkParams p) {
     const T* rows = (const T*)a.proj + (int64_t)p.r.b.row0[seq] * a.ld;
     const int ring_ld = 2 * a.kv_heads * dim + a.heads * a.vdim;
     const T* ring = (const T*)a.conv_ring + (int64_t)p.r.b.slot[seq] * a.taps * ring_ld;
-    for (int i = tid; i < kC * DP; i += 256) {
-        const int t = i / DP, d = i - t * DP;
-        float qv = 0.f, kv = 0.f;
-        if (d < dim && t0 + t < cnt) {
+    for (int i = tid; i < 8 * DP; i += 256) {  // (q or k, 16-row block, channel)
+        const int d = i % DP, blk = i / DP, t = (blk & 3) * 16, is_k = blk >> 2;
+        float y[16];
+        if (d < dim) {
             const int c = kvh * dim + d;
-            qv = conv_at<T>(a, rows, ring, ring_ld, a.off_q + c, c, a.conv_q + (int64_t)c * a.taps, t0 + t, pos0);
-            kv = conv_at<T>(a, rows, ring, ring_ld, a.off_k + c, a.kv_heads * dim + c, a.conv_k + (int64_t)c * a.taps, t0 + t, pos0);
+            conv_rows16<T>(a, rows, ring, ring_ld, (is_k ? a.off_k : a.off_q) + c, is_k * a.kv_heads * dim + c,
+                           (is_k ? a.conv_k : a.conv_q) + (int64_t)c * a.taps, t0 + t, cnt, pos0, y);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 16; ++e) y[e] = 0.f;
         }
-        q[t * ld + d] = qv;
-        k[t * ld + d] = kv;
+        float* dst = (is_k ? k : q) + t * ld + d;
+#pragma unroll
+        for (int e = 0; e < 16; ++e) dst[e * ld] = y[e];
     }
     __syncthreads();
     for (int t = wave; t < kC; t += 4) {  // unit vectors: a wave per row
@@ -182,30 +186,31 @@ __global__ __launch_bounds__(256) void delta_head_kernel(const ChunkParams p) {
         if (tid == 63) p.s.gam[hi * DP] = expf((float)end);
     }
     // V^T with the convolution (beta rides on it below)
-    for (int i = tid; i < kC * VP; i += 256) {
-        const int t = i / VP, d = i - t * VP;
-        float v = 0.f;
-        if (d < a.vdim && t0 + t < cnt) {
+    for (int i = tid; i < 4 * VP; i += 256) {
+        const int d = i % VP, t = (i / VP) * 16;
+        float y[16];
+        if (d < a.vdim) {
             const int c = head * a.vdim + d;
-            v = conv_at<T>(a, rows, ring, ring_ld, a.off_v + c, 2 * a.kv_heads * a.dim + c, a.conv_v + (int64_t)c * a.taps, t0 + t, pos0);
+            conv_rows16<T>(a, rows, ring, ring_ld, a.off_v + c, 2 * a.kv_heads * a.dim + c, a.conv_v + (int64_t)c * a.taps, t0 + t, cnt, pos0, y);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 16; ++e) y[e] = 0.f;
         }
-        vt[d * kP + t] = v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) *(f32x4*)(vt + d * kP + t + 4 * e) = f32x4{y[4 * e], y[4 * e + 1], y[4 * e + 2], y[4 * e + 3]};
     }
     __syncthreads();
     const float* kk = p.s.kk + gi * kC * kC;
     const float* qk = p.s.qk + gi * kC * kC;
     float* oP = p.s.P + hi * kC * kC;
-    for (int i = tid; i < kC * kC; i += 256) {
-        const int r = i >> 6, c = i & 63;
-        float e = 0.f, x = 0.f, y = 0.f;
-        if (c <= r) {
-            e = expf((float)(gcum[r] - gcum[c]));
-            y = e * qk[i];
-            if (c < r) x = beta[r] * e * kk[i];
-        }
-        A[r * kP + c] = x;
+#pragma unroll 8
+    for (int n = 0; n < kC * kC / 256; ++n) {
+        const int i = n * 256 + tid, r = i >> 6, c = i & 63;
+        const float qv = qk[i], kv = kk[i];  // (above the diagonal blocks: unwritten scratch, dropped below)
+        const float e = c <= r ? exp_f32((float)(gcum[r] - gcum[c])) : 0.f;
+        A[r * kP + c] = c < r ? beta[r] * e * kv : 0.f;
         Ti[r * kP + c] = 0.f;
-        oP[i] = y;
+        oP[i] = c <= r ? e * qv : 0.f;
     }
     for (int i = tid; i < kC * VP; i += 256) {
         const int d = i / kC, t = i - d * kC;
@@ -295,7 +300,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
     float* k = q + kC * kP;
     float* G = k + kC * kP;
     float* seg = G + kC * kP;       // [4][64]
-    float* lr = seg + 4 * kCh;      // [64][rank]
+    float* lr = seg + 4 * kCh;      // [rank][64]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c16 = lane & 15, g = lane >> 4;
     const T* rows = (const T*)a.proj + (int64_t)(p.r.b.row0[seq] + t0) * a.ld;
@@ -303,7 +308,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
     const int64_t hi = (int64_t)(chunk_base(p, seq) + blockIdx.x) * a.heads + head;
     for (int i = tid; i < kC * rank; i += 256) {
         const int t = i / rank, r = i - t * rank;
-        lr[i] = t < n ? to_f32<T>(rows[(int64_t)t * a.ld + a.off_a + r]) : 0.f;
+        lr[r * kC + t] = t < n ? to_f32<T>(rows[(int64_t)t * a.ld + a.off_a + r]) : 0.f;
     }
     float* oq = p.s.q + hi * kC * DP;
     float* okt = p.s.kt + hi * DP * kC;
@@ -317,39 +322,52 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
         {
             const int c = tid & 63, sb = tid >> 6, ch = c0 + c;
             const bool ok = ch < dim;
-            float s = 0.f;
+            float qv[16], kv[16], z[16];
+#pragma unroll
+            for (int e = 0; e < 16; ++e) {
+                const int t = sb * 16 + e;
+                const bool in = ok && t < n;
+                const T* row = rows + (int64_t)(in ? t : 0) * a.ld + head * dim + (ok ? ch : 0);
+                qv[e] = in ? to_f32<T>(row[a.off_q]) * a.q_scale : 0.f;
+                kv[e] = in ? to_f32<T>(row[a.off_k]) : 0.f;
+            }
             const float* w = a.a2 + (int64_t)(head * dim + (ok ? ch : 0)) * rank;
             const float bias = ok ? a.a2_bias[head * dim + ch] : 0.f;
-            for (int t = sb * 16; t < sb * 16 + 16; ++t) {
-                float la = 0.f, qv = 0.f, kv = 0.f;
-                if (ok && t < n) {
-                    float z = bias;
-                    for (int r = 0; r < rank; ++r) z += w[r] * lr[t * rank + r];
-                    la = -softplus_f32(-z) * a.inv_tau;
-                    qv = to_f32<T>(rows[(int64_t)t * a.ld + a.off_q + head * dim + ch]) * a.q_scale;
-                    kv = to_f32<T>(rows[(int64_t)t * a.ld + a.off_k + head * dim + ch]);
+#pragma unroll
+            for (int e = 0; e < 16; ++e) z[e] = bias;
+#pragma unroll 4
+            for (int r = 0; r < rank; ++r) {
+                const float wr = w[r];
+#pragma unroll
+                for (int e = 0; e < 16; e += 4) {
+                    const f32x4 l = *(const f32x4*)(lr + r * kC + sb * 16 + e);
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) z[e + j] += wr * l[j];
                 }
-                s += la;
+            }
+            float s = 0.f;
+#pragma unroll
+            for (int e = 0; e < 16; ++e) {
+                const int t = sb * 16 + e;
+                s += ok && t < n ? -softplus_f32(-z[e]) * a.inv_tau : 0.f;
                 G[t * kP + c] = s;   // sums from the block's first row on
-                q[t * kP + c] = qv;
-                k[t * kP + c] = kv;
+                q[t * kP + c] = qv[e];
+                k[t * kP + c] = kv[e];
             }
             seg[sb * kCh + c] = s;
         }
         __syncthreads();
         // ---- diagonal blocks: wave = block, lane group g and c16 = column j, rows 4 rr + g
+#pragma unroll 2
+        for (int c = 0; c < kCh; c += 4) {
+            const int j = wave * 16 + c16;
+            const f32x4 kj = *(const f32x4*)(k + j * kP + c), gj = *(const f32x4*)(G + j * kP + c);
 #pragma unroll
-        for (int rr = 0; rr < 4; ++rr) {
-            const int i = wave * 16 + rr * 4 + g, j = wave * 16 + c16;
-            if (j <= i) {
-                float s = 0.f;
-                for (int c = 0; c < kCh; c += 4) {
-                    const f32x4 qi = *(const f32x4*)(q + i * kP + c), kj = *(const f32x4*)(k + j * kP + c);
-                    const f32x4 gi = *(const f32x4*)(G + i * kP + c), gj = *(const f32x4*)(G + j * kP + c);
+            for (int rr = 0; rr < 4; ++rr) {
+                const int i = wave * 16 + rr * 4 + g;
+                const f32x4 qi = *(const f32x4*)(q + i * kP + c), gi = *(const f32x4*)(G + i * kP + c);
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) s += qi[e] * kj[e] * expf(gi[e] - gj[e]);
-                }
-                dg[rr] += s;
+                for (int e = 0; e < 4; ++e) dg[rr] += qi[e] * kj[e] * exp_f32(fminf(gi[e] - gj[e], 0.f));  // (j > i: dropped at the end)
             }
         }
         // ---- off-diagonal blocks (I, J): q_i e^(G_i - start of I) against k_j e^(start of I - G_j)
@@ -363,8 +381,8 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
                 const f32x4 gi = *(const f32x4*)(G + i * kP + c);
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    av[e] *= expf(gi[e]);
-                    bv[e] *= expf(gap[e]);
+                    av[e] *= exp_f32(gi[e]);
+                    bv[e] *= exp_f32(gap[e]);
                 }
 #pragma unroll
                 for (int b = 0; b < 3; ++b)  // (constant register index)
@@ -376,19 +394,19 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
             const int t = i / nch, c = i - t * nch, sb = t >> 4;
             float before = 0.f;
             for (int m = 0; m < sb; ++m) before += seg[m * kCh + c];
-            oq[t * DP + c0 + c] = q[t * kP + c] * expf(before + G[t * kP + c]);
+            oq[t * DP + c0 + c] = q[t * kP + c] * exp_f32(before + G[t * kP + c]);
         }
         for (int i = tid; i < kC * nch; i += 256) {
             const int c = i >> 6, t = i & 63, sb = t >> 4;
             float rest = seg[sb * kCh + c] - G[t * kP + c];
             for (int m = sb + 1; m < 4; ++m) rest += seg[m * kCh + c];
-            okt[(c0 + c) * kC + t] = k[t * kP + c] * expf(rest);
+            okt[(c0 + c) * kC + t] = k[t * kP + c] * exp_f32(rest);
         }
         if (tid < nch) p.s.gam[hi * DP + c0 + tid] = expf(seg[tid] + seg[kCh + tid] + seg[2 * kCh + tid] + seg[3 * kCh + tid]);
     }
     float* oP = p.s.P + hi * kC * kC;
 #pragma unroll
-    for (int rr = 0; rr < 4; ++rr) oP[(wave * 16 + rr * 4 + g) * kC + wave * 16 + c16] = dg[rr];
+    for (int rr = 0; rr < 4; ++rr) oP[(wave * 16 + rr * 4 + g) * kC + wave * 16 + c16] = c16 <= rr * 4 + g ? dg[rr] : 0.f;
 #pragma unroll
     for (int J = 0; J < 3; ++J)
         if (J < wave) {
@@ -407,13 +425,16 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
 }
 
 // ------------------------------------------------------------------------------------ the serial part
-// grid (VP / 16, heads, seqs), 256 threads; NT = 16-row tiles of the state per wave (DP <= 64 NT)
+// grid (8 * ceil(heads / 8) * VP / 16, seqs), 256 threads; NT = 16-row tiles of the state per wave (DP <= 64 NT).  The column slices of
+// a head run on one XCD (block index mod 8): its L2 then serves W and K^T to all of them
 template <int KIND, int NT>
 __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
     const mi355_recurrent_args& a = p.r.a;
     extern __shared__ __attribute__((aligned(16))) float sm[];
-    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, n0 = blockIdx.x * 16;
     const int DP = p.DP, VP = p.VP, ls = DP + 4;
+    const int slices = VP / 16, idx = blockIdx.x >> 3;
+    const int seq = p.seq0 + blockIdx.y, head = (blockIdx.x & 7) + 8 * (idx / slices), n0 = (idx % slices) * 16;
+    if (head >= a.heads) return;
     float* sl = sm;            // [16][DP + 4]: S_0 columns
     float* ul = sm + 16 * ls;  // [16][kP]: U columns, weighted by e^(G_end - G)
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -622,7 +643,7 @@ int set_lds(K kernel, size_t bytes) {
 
 template <int KIND>
 int launch_scan(const ChunkParams& p, int seqs, hipStream_t s) {
-    const dim3 grid(p.VP / 16, p.r.a.heads, seqs);
+    const dim3 grid((p.r.a.heads + 7) / 8 * 8 * (p.VP / 16), seqs);
     const size_t lds = ((size_t)16 * (p.DP + 4) + 16 * kP) * 4;
     if (p.DP <= 64) hipLaunchKernelGGL((scan_kernel<KIND, 1>), grid, dim3(256), lds, s, p);
     else if (p.DP <= 128) hipLaunchKernelGGL((scan_kernel<KIND, 2>), grid, dim3(256), lds, s, p);

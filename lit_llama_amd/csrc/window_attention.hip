@@ -18,6 +18,7 @@ typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2_t;
 
 constexpr int kRowThreads = 256;
 constexpr int kKeys = 256;        // keys per pass of the row kernel
+constexpr int kMaxSplit = 32;     // workgroups over the keys of one (row, key head) in a decode step
 constexpr double kInvTwoPi = 0.15915494309189533577;
 
 // turn of (u, v) by pos * inv_freq: the angle is reduced in f64, so far positions keep f32 accuracy
@@ -278,14 +279,22 @@ __global__ __launch_bounds__(128) void window_join_kernel(const WinParams p) {
     const int h = blockIdx.x, row = blockIdx.y;
     const float* rec = a.partials + ((int64_t)row * a.heads + h) * p.n_split * (a.vdim + 2);
     float m = -INFINITY;
+#pragma unroll 16
     for (int s = 0; s < p.n_split; ++s) m = fmaxf(m, rec[s * (a.vdim + 2)]);
+    __shared__ float wgt[kMaxSplit];
     float l = 0.f;
-    for (int s = 0; s < p.n_split; ++s) l += expf(rec[s * (a.vdim + 2)] - m) * rec[s * (a.vdim + 2) + 1];
+    for (int s = 0; s < p.n_split; ++s) {
+        const float e = expf(rec[s * (a.vdim + 2)] - m);
+        l += e * rec[s * (a.vdim + 2) + 1];
+        if ((int)threadIdx.x == s) wgt[s] = e;
+    }
+    __syncthreads();
     float gate = 1.f / l;
     if (a.off_g >= 0) gate /= 1.0f + expf(-to_f32<T>(((const T*)a.proj)[(int64_t)row * a.ld + a.off_g + h]));
     for (int d = threadIdx.x; d < a.vdim; d += blockDim.x) {
         float o = 0.f;
-        for (int s = 0; s < p.n_split; ++s) o += expf(rec[s * (a.vdim + 2)] - m) * rec[s * (a.vdim + 2) + 2 + d];
+#pragma unroll 16
+        for (int s = 0; s < p.n_split; ++s) o += wgt[s] * rec[s * (a.vdim + 2) + 2 + d];
         ((T*)a.y)[(int64_t)row * a.ldy + (int64_t)h * a.vdim + d] = from_f32<T>(o * gate);
     }
 }
@@ -639,6 +648,7 @@ int run(WinParams p, hipStream_t s) {
         const int groups = p.b.rows * a.kv_heads * ((per + ht - 1) / ht);
         int n = 512 / groups;
         n = n < a.ring / 64 ? n : a.ring / 64;
+        n = n < kMaxSplit ? n : kMaxSplit;
         const uint64_t rec = (uint64_t)p.b.rows * a.heads * (a.vdim + 2) * 4;
         if (a.partials == nullptr) n = 1;
         while (n > 1 && rec * n > a.partials_bytes) n /= 2;
