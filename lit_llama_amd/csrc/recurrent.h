@@ -6,9 +6,15 @@ constexpr int kMaxRank = 256;  // of the low-rank decay projection
 
 // e^v by the hardware's 2^x: one rounding of v log2(e) (relative error |v| 2^-24) and v_exp_f32's own
 __device__ __forceinline__ float exp_f32(float v) { return __builtin_amdgcn_exp2f(v * 1.44269504088896340736f); }
-__device__ __forceinline__ float silu_f32(float v) { return v / (1.0f + expf(-v)); }
-__device__ __forceinline__ float sigmoid_f32(float v) { return 1.0f / (1.0f + expf(-v)); }
-__device__ __forceinline__ float softplus_f32(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
+__device__ __forceinline__ float sigmoid_f32(float v) { return __builtin_amdgcn_rcpf(1.0f + exp_f32(-v)); }
+__device__ __forceinline__ float silu_f32(float v) { return v * sigmoid_f32(v); }
+// log(1 + u) for u in [0, 1]: log(w) u / (w - 1) with w = 1 + u rounded, whose error cancels in the quotient (Goldberg, "What Every Computer
+// Scientist Should Know About Floating-Point Arithmetic", 1991, theorem 4)
+__device__ __forceinline__ float log1p_unit(float u) {
+    const float w = 1.0f + u, d = w - 1.0f;
+    return d == 0.f ? u : __builtin_amdgcn_logf(w) * 0.69314718055994530942f * u * __builtin_amdgcn_rcpf(d);
+}
+__device__ __forceinline__ float softplus_f32(float v) { return fmaxf(v, 0.f) + log1p_unit(exp_f32(-fabsf(v))); }
 
 template <typename T>
 __device__ __forceinline__ float to_f32(T v);

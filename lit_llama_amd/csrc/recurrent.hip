@@ -49,8 +49,18 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
     for (int t = 0; t < cnt; ++t) {
         const T* row = rows + (int64_t)t * a.ld;
         // ---- the row's q, k (and decays) into LDS
+        // (what needs no LDS is requested here, in front of the barriers: one memory latency instead of one per use)
+        const bool out_ok = part == 0 && col_ok;
+        const float gate = out_ok ? silu_f32(to_f32<T>(row[a.off_g + head * vdim + col])) * a.head_norm[col] : 0.f;
         float g = 1.f, beta = 1.f, v = 0.f;
         if constexpr (KIND == MI355_REC_DELTA) {
+            const float dt = softplus_f32(to_f32<T>(row[a.off_a + head]) + a.dt_bias[head]);
+            g = expf(-expf(a.a_log[head]) * dt);
+            beta = sigmoid_f32(to_f32<T>(row[a.off_b + head]));
+            if (col_ok) {
+                const int c = head * vdim + col;
+                v = conv_at<T>(a, rows, ring, ring_ld, a.off_v + c, 2 * a.kv_heads * dim + c, a.conv_v + (int64_t)c * a.taps, t, pos0);
+            }
             float sq = 0.f, sk = 0.f;
             for (int d = tid; d < dim; d += nt) {
                 const int c = kvh * dim + d;
@@ -68,14 +78,8 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
                 q[d] *= iq;
                 k[d] *= ik;
             }
-            const float dt = softplus_f32(to_f32<T>(row[a.off_a + head]) + a.dt_bias[head]);
-            g = expf(-expf(a.a_log[head]) * dt);
-            beta = sigmoid_f32(to_f32<T>(row[a.off_b + head]));
-            if (col_ok) {
-                const int c = head * vdim + col;
-                v = conv_at<T>(a, rows, ring, ring_ld, a.off_v + c, 2 * a.kv_heads * dim + c, a.conv_v + (int64_t)c * a.taps, t, pos0);
-            }
         } else {
+            if (col_ok) v = to_f32<T>(row[a.off_v + head * vdim + col]);
             for (int r = tid; r < a.rank; r += nt) lr[r] = to_f32<T>(row[a.off_a + r]);
             __syncthreads();
             for (int d = tid; d < dim; d += nt) {
@@ -87,7 +91,6 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
                 q[d] = to_f32<T>(row[a.off_q + c]) * a.q_scale;
                 k[d] = to_f32<T>(row[a.off_k + c]);
             }
-            if (col_ok) v = to_f32<T>(row[a.off_v + head * vdim + col]);
         }
         __syncthreads();
         // ---- state update and read-out
@@ -124,11 +127,10 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
         // ---- output norm over vdim, gate (part 0 holds the columns)
         o = 0.f;
         for (int j = 0; j < p.parts; ++j) o += pb[j * cols + col];
-        const float ss = block_sum(part == 0 && col_ok ? o * o : 0.f, red);
-        if (part == 0 && col_ok) {
+        const float ss = block_sum(out_ok ? o * o : 0.f, red);
+        if (out_ok) {
             const float rinv = 1.0f / sqrtf(ss / (float)vdim + a.eps);
-            const float gate = silu_f32(to_f32<T>(row[a.off_g + head * vdim + col]));
-            ((T*)a.y)[(int64_t)(p.b.row0[seq] + t) * a.ldy + head * vdim + col] = from_f32<T>(o * rinv * a.head_norm[col] * gate);
+            ((T*)a.y)[(int64_t)(p.b.row0[seq] + t) * a.ldy + head * vdim + col] = from_f32<T>(o * rinv * gate);
         }
         __syncthreads();
     }

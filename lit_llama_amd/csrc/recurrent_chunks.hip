@@ -32,6 +32,11 @@ __device__ __forceinline__ f32x4 mfma4(f32x4 a, f32x4 b, f32x4 c) {
 }
 __device__ __forceinline__ f32x4 zero4() { return f32x4{0.f, 0.f, 0.f, 0.f}; }
 
+// a barrier for data in LDS: global requests stay in flight across it
+__device__ __forceinline__ void lds_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+}
+
 // ---------------------------------------------------------------- scratch, per packed chunk (padded sizes DP, VP: multiples of 16)
 struct Scratch {
     float* q;     // [NC][GQ][64][DP]        delta: unit q * q_scale; gla: q e^G * q_scale
@@ -56,6 +61,14 @@ struct ChunkParams {
 
 __device__ __forceinline__ int chunk_base(const ChunkParams& p, int seq) {
     return p.r.b.row0[seq] / kC + seq - (p.r.b.row0[p.seq0] / kC + p.seq0);
+}
+
+// launches over (chunk, head): grid (8 * ceil(heads / 8) * chunks, seqs), a head's chunks on one XCD (block index mod 8), as its scan
+__device__ __forceinline__ bool head_chunk(const ChunkParams& p, int& head, int& chunk) {
+    const int chunks = (p.r.b.max_count + kC - 1) / kC, idx = blockIdx.x >> 3;
+    head = (blockIdx.x & 7) + 8 * (idx / chunks);
+    chunk = idx % chunks;
+    return head < p.r.a.heads;
 }
 
 // ------------------------------------------------------------------------------------ delta: q, k per key head
@@ -137,14 +150,16 @@ __global__ __launch_bounds__(256) void delta_qk_kernel(const ChunkParams p) {
 }
 
 // ------------------------------------------------------------------------------------ delta: per head
-// grid (chunks, heads, seqs), 256 threads.  LDS: A, T [64][kP], X [64][kX], vt [VP][kP]
+// 256 threads.  LDS: A, T [64][kP], X [64][kX], vt [VP][kP]
 template <typename T>
 __global__ __launch_bounds__(256) void delta_head_kernel(const ChunkParams p) {
     const mi355_recurrent_args& a = p.r.a;
     extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ double gcum[kC];
     __shared__ float beta[kC], bg[kC];
-    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, t0 = blockIdx.x * kC;
+    int head, chunk;
+    if (!head_chunk(p, head, chunk)) return;
+    const int seq = p.seq0 + blockIdx.y, t0 = chunk * kC;
     const int cnt = p.r.b.count[seq];
     if (t0 >= cnt) return;
     const int DP = p.DP, VP = p.VP;
@@ -159,7 +174,7 @@ __global__ __launch_bounds__(256) void delta_head_kernel(const ChunkParams p) {
     const T* rows = (const T*)a.proj + (int64_t)p.r.b.row0[seq] * a.ld;
     const int ring_ld = 2 * a.kv_heads * a.dim + a.heads * a.vdim;
     const T* ring = (const T*)a.conv_ring + (int64_t)p.r.b.slot[seq] * a.taps * ring_ld;
-    const int64_t ci = chunk_base(p, seq) + blockIdx.x;
+    const int64_t ci = chunk_base(p, seq) + chunk;
     const int64_t gi = ci * p.GQ + kvh, hi = ci * a.heads + head;
 
     if (tid < kC) {
@@ -286,13 +301,15 @@ __global__ __launch_bounds__(256) void delta_head_kernel(const ChunkParams p) {
 }
 
 // ------------------------------------------------------------------------------------ gla: per head
-// grid (chunks, heads, seqs), 256 threads; key channels in slices of 64.  LDS: q, k, G [64 rows][68], low-rank rows [64][rank], sums
+// 256 threads; key channels in slices of 64.  LDS: q, k, G [64 rows][68], low-rank rows [64][rank], sums
 constexpr int kCh = 64;
 template <typename T>
 __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
     const mi355_recurrent_args& a = p.r.a;
     extern __shared__ __attribute__((aligned(16))) float sm[];
-    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, t0 = blockIdx.x * kC;
+    int head, chunk;
+    if (!head_chunk(p, head, chunk)) return;
+    const int seq = p.seq0 + blockIdx.y, t0 = chunk * kC;
     const int cnt = p.r.b.count[seq];
     if (t0 >= cnt) return;
     const int DP = p.DP, VP = p.VP, dim = a.dim, rank = a.rank;
@@ -305,7 +322,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
     const int c16 = lane & 15, g = lane >> 4;
     const T* rows = (const T*)a.proj + (int64_t)(p.r.b.row0[seq] + t0) * a.ld;
     const int n = min(kC, cnt - t0);
-    const int64_t hi = (int64_t)(chunk_base(p, seq) + blockIdx.x) * a.heads + head;
+    const int64_t hi = (int64_t)(chunk_base(p, seq) + chunk) * a.heads + head;
     for (int i = tid; i < kC * rank; i += 256) {
         const int t = i / rank, r = i - t * rank;
         lr[r * kC + t] = t < n ? to_f32<T>(rows[(int64_t)t * a.ld + a.off_a + r]) : 0.f;
@@ -390,17 +407,31 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
             }
         // ---- q e^G and (k e^(G_end - G))^T of the slice
         const int nch = min(kCh, DP - c0);
-        for (int i = tid; i < kC * nch; i += 256) {
-            const int t = i / nch, c = i - t * nch, sb = t >> 4;
+        {   // wave = 16-row block, lane = channel
+            const int c = lane;
             float before = 0.f;
-            for (int m = 0; m < sb; ++m) before += seg[m * kCh + c];
-            oq[t * DP + c0 + c] = q[t * kP + c] * exp_f32(before + G[t * kP + c]);
+            for (int m = 0; m < wave; ++m) before += seg[m * kCh + c];
+            if (c < nch) {
+#pragma unroll
+                for (int e = 0; e < 16; ++e) {
+                    const int t = wave * 16 + e;
+                    oq[t * DP + c0 + c] = q[t * kP + c] * exp_f32(before + G[t * kP + c]);
+                }
+            }
         }
-        for (int i = tid; i < kC * nch; i += 256) {
-            const int c = i >> 6, t = i & 63, sb = t >> 4;
-            float rest = seg[sb * kCh + c] - G[t * kP + c];
-            for (int m = sb + 1; m < 4; ++m) rest += seg[m * kCh + c];
-            okt[(c0 + c) * kC + t] = k[t * kP + c] * exp_f32(rest);
+        {   // thread = (4 rows, channel c4 + 16 e)
+            const int t = (tid & 15) * 4, sb = t >> 4;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int c = (tid >> 4) + 16 * e;
+                float rest = 0.f;
+#pragma unroll
+                for (int m = 0; m < 4; ++m) rest += m >= sb ? seg[m * kCh + c] : 0.f;
+                f32x4 o;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) o[j] = k[(t + j) * kP + c] * exp_f32(rest - G[(t + j) * kP + c]);
+                if (c < nch) *(f32x4*)(okt + (c0 + c) * kC + t) = o;
+            }
         }
         if (tid < nch) p.s.gam[hi * DP + c0 + tid] = expf(seg[tid] + seg[kCh + tid] + seg[2 * kCh + tid] + seg[3 * kCh + tid]);
     }
@@ -454,38 +485,40 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
             const int i = (wave + 4 * t) * 16 + 4 * g + r;
             S[t][r] = (col_ok && i < a.dim) ? state[(int64_t)i * a.vdim + n0 + c16] : 0.f;
         }
-    // a chunk's operands of this wave, requested one chunk ahead
-    f32x4 wr[4 * NT], kr[NT][4], ur, dr, gr[NT], vr[4];
-    auto load = [&](int ch) {
+    // a chunk's operands of this wave: two sets, the next chunk's requested when a chunk begins
+    struct Ops {
+        f32x4 w[KIND == MI355_REC_DELTA ? 4 * NT : 1], k[NT][4], u, d, g[NT], v[4];
+    };
+    auto load = [&](int ch, Ops& x) {
         const int64_t hi = (cb + ch) * a.heads + head, gi = (cb + ch) * p.GQ + kvh;
+        const float* ut = p.s.ut + hi * VP * kC + (int64_t)(n0 + c16) * kC;
+        if constexpr (KIND == MI355_REC_DELTA) {
+            const float* W = p.s.W + hi * kC * DP + (int64_t)(wave * 16 + c16) * DP;
+#pragma unroll
+            for (int b = 0; b < 4 * NT; ++b) x.w[b] = b < n_tiles ? *(const f32x4*)(W + b * 16 + 4 * g) : zero4();
+            x.u = *(const f32x4*)(ut + wave * 16 + 4 * g);
+            x.d = *(const f32x4*)(p.s.ed + hi * kC + wave * 16 + 4 * g);
+            const float gm = p.s.gam[hi * DP];
+            x.g[0] = f32x4{gm, gm, gm, gm};
+        } else {
+#pragma unroll
+            for (int b = 0; b < 4; ++b) x.v[b] = *(const f32x4*)(ut + b * 16 + 4 * g);
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+                x.g[t] = wave + 4 * t < n_tiles ? *(const f32x4*)(p.s.gam + hi * DP + (wave + 4 * t) * 16 + 4 * g) : zero4();
+        }
         const float* kt = p.s.kt + gi * DP * kC;
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
             const int row = (wave + 4 * t) * 16 + c16;
 #pragma unroll
-            for (int b = 0; b < 4; ++b) kr[t][b] = wave + 4 * t < n_tiles ? *(const f32x4*)(kt + row * kC + b * 16 + 4 * g) : zero4();
-        }
-        const float* ut = p.s.ut + hi * VP * kC + (int64_t)(n0 + c16) * kC;
-        if constexpr (KIND == MI355_REC_DELTA) {
-            const float* W = p.s.W + hi * kC * DP + (int64_t)(wave * 16 + c16) * DP;
-#pragma unroll
-            for (int b = 0; b < 4 * NT; ++b) wr[b] = b < n_tiles ? *(const f32x4*)(W + b * 16 + 4 * g) : zero4();
-            ur = *(const f32x4*)(ut + wave * 16 + 4 * g);
-            dr = *(const f32x4*)(p.s.ed + hi * kC + wave * 16 + 4 * g);
-            const float gm = p.s.gam[hi * DP];
-            gr[0] = f32x4{gm, gm, gm, gm};
-        } else {
-#pragma unroll
-            for (int b = 0; b < 4; ++b) vr[b] = *(const f32x4*)(ut + b * 16 + 4 * g);
-#pragma unroll
-            for (int t = 0; t < NT; ++t)
-                gr[t] = wave + 4 * t < n_tiles ? *(const f32x4*)(p.s.gam + hi * DP + (wave + 4 * t) * 16 + 4 * g) : zero4();
+            for (int b = 0; b < 4; ++b) x.k[t][b] = wave + 4 * t < n_tiles ? *(const f32x4*)(kt + row * kC + b * 16 + 4 * g) : zero4();
         }
     };
-    load(0);
-    for (int ch = 0; ch < n_chunks; ++ch) {
+    auto chunk = [&](int ch, Ops& x, Ops& next) {
         const int64_t hi = (cb + ch) * a.heads + head;
         float* st = p.s.st + hi * VP * DP + (int64_t)(n0 + c16) * DP;
+        if (ch + 1 < n_chunks) load(ch + 1, next);
         // S_0: to the output kernel, and to LDS as the B operand of W S_0
 #pragma unroll
         for (int t = 0; t < NT; ++t)
@@ -495,36 +528,34 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
                 if constexpr (KIND == MI355_REC_DELTA) *(f32x4*)(sl + c16 * ls + i) = S[t];
             }
         if constexpr (KIND == MI355_REC_DELTA) {
-            __syncthreads();
+            lds_barrier();
             f32x4 u = zero4(), u2 = zero4();
 #pragma unroll
             for (int b = 0; b < 4 * NT; ++b)
                 if (b < n_tiles) {
                     const f32x4 sv = *(const f32x4*)(sl + c16 * ls + b * 16 + 4 * g);
-                    if (b & 1) u2 = mfma4(wr[b], sv, u2);
-                    else u = mfma4(wr[b], sv, u);
+                    if (b & 1) u2 = mfma4(x.w[b], sv, u2);
+                    else u = mfma4(x.w[b], sv, u);
                 }
-            u = ur - (u + u2);
+            u = x.u - (u + u2);
             *(f32x4*)(p.s.ut + hi * VP * kC + (int64_t)(n0 + c16) * kC + wave * 16 + 4 * g) = u;
-            *(f32x4*)(ul + c16 * kP + wave * 16 + 4 * g) = u * dr;
-            __syncthreads();
+            *(f32x4*)(ul + c16 * kP + wave * 16 + 4 * g) = u * x.d;
+            lds_barrier();
 #pragma unroll
-            for (int b = 0; b < 4; ++b) vr[b] = *(const f32x4*)(ul + c16 * kP + b * 16 + 4 * g);
+            for (int b = 0; b < 4; ++b) x.v[b] = *(const f32x4*)(ul + c16 * kP + b * 16 + 4 * g);
         }
-        f32x4 kc[NT][4], vc[4];
 #pragma unroll
-        for (int b = 0; b < 4; ++b) vc[b] = vr[b];
-#pragma unroll
-        for (int t = 0; t < NT; ++t) {
-            S[t] *= gr[KIND == MI355_REC_DELTA ? 0 : t];
-#pragma unroll
-            for (int b = 0; b < 4; ++b) kc[t][b] = kr[t][b];
-        }
-        if (ch + 1 < n_chunks) load(ch + 1);
+        for (int t = 0; t < NT; ++t) S[t] *= x.g[KIND == MI355_REC_DELTA ? 0 : t];
 #pragma unroll
         for (int b = 0; b < 4; ++b)
 #pragma unroll
-            for (int t = 0; t < NT; ++t) S[t] = mfma4(kc[t][b], vc[b], S[t]);
+            for (int t = 0; t < NT; ++t) S[t] = mfma4(x.k[t][b], x.v[b], S[t]);
+    };
+    Ops xa, xb;
+    load(0, xa);
+    for (int ch = 0; ch < n_chunks; ch += 2) {
+        chunk(ch, xa, xb);
+        if (ch + 1 < n_chunks) chunk(ch + 1, xb, xa);
     }
 #pragma unroll
     for (int t = 0; t < NT; ++t)
@@ -536,19 +567,21 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
 }
 
 // ------------------------------------------------------------------------------------ outputs
-// grid (chunks, heads, seqs), 256 threads: wave w takes the 16-column tiles w, w + 4, ...; NV = tiles per wave (VP <= 64 NV)
+// 256 threads: wave w takes the 16-column tiles w, w + 4, ...; NV = tiles per wave (VP <= 64 NV)
 template <typename T, int KIND, int NV>
 __global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
     const mi355_recurrent_args& a = p.r.a;
     __shared__ float ssq[4][kC];
-    const int seq = p.seq0 + blockIdx.z, head = blockIdx.y, t0 = blockIdx.x * kC;
+    int head, chunk;
+    if (!head_chunk(p, head, chunk)) return;
+    const int seq = p.seq0 + blockIdx.y, t0 = chunk * kC;
     const int cnt = p.r.b.count[seq];
     if (t0 >= cnt) return;
     const int DP = p.DP, VP = p.VP;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int c16 = lane & 15, g = lane >> 4;
     const int kvh = KIND == MI355_REC_DELTA ? head / (a.heads / a.kv_heads) : head;
-    const int64_t ci = chunk_base(p, seq) + blockIdx.x, hi = ci * a.heads + head;
+    const int64_t ci = chunk_base(p, seq) + chunk, hi = ci * a.heads + head;
     const float* q = p.s.q + (ci * p.GQ + kvh) * kC * DP;
     const float* st = p.s.st + hi * VP * DP;
     const float* P = p.s.P + hi * kC * kC;
@@ -665,7 +698,7 @@ template <typename T>
 int run_group(const ChunkParams& p, int seqs, hipStream_t s) {
     const mi355_recurrent_args& a = p.r.a;
     const int chunks = (p.r.b.max_count + kC - 1) / kC;
-    const dim3 heads(chunks, a.heads, seqs);
+    const dim3 heads((a.heads + 7) / 8 * 8 * chunks, seqs);
     if (a.kind == MI355_REC_DELTA) {
         const size_t lds1 = (size_t)2 * kC * (p.DP + 4) * 4;
         if (int rc = set_lds(delta_qk_kernel<T>, lds1)) return rc;

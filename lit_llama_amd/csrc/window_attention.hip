@@ -155,41 +155,51 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
 
     for (int kb = k_begin; kb < k_end; kb += kKeys) {
         const int nk = min(kKeys, k_end - kb);
-        // ---- scores: 16 lanes per key
+        // ---- scores: 16 lanes per key, four keys per lane group in flight
         const int l16 = tid & 15;
-        for (int kk = tid >> 4; kk < kKeys; kk += kRowThreads / 16) {
-            if (kk - (tid >> 4) >= nk) break;  // (uniform per wave up to the DPP groups: whole 16-lane groups leave together)
-            const int kp = kb + min(kk, nk - 1);
-            float dot[HT];
+        for (int k4 = tid >> 4; k4 - (tid >> 4) < nk; k4 += 4 * (kRowThreads / 16)) {
+            float dot[4][HT];
+            const T* src[4];
 #pragma unroll
-            for (int h = 0; h < HT; ++h) dot[h] = 0.f;
-            if (p.fresh && kp == pos) {
-                for (int d = l16; d < dim; d += 16) {
-                    const float kv = kn[d];
+            for (int u = 0; u < 4; ++u) {
+                const int kp = kb + min(k4 + u * (kRowThreads / 16), nk - 1);
+                src[u] = (p.fresh && kp == pos) ? nullptr
+                         : kp >= pos0           ? proj + (int64_t)(row0 + kp - pos0) * a.ld + a.off_k + (int64_t)kvh * dim
+                                                : kring + (int64_t)(kp % a.ring) * dim;
 #pragma unroll
-                    for (int h = 0; h < HT; ++h)
-                        if (h < nh) dot[h] += kv * q[h * dim + d];
-                }
-            } else {
-                const T* src = kp >= pos0 ? proj + (int64_t)(row0 + kp - pos0) * a.ld + a.off_k + (int64_t)kvh * dim
-                                          : kring + (int64_t)(kp % a.ring) * dim;
-                for (int d = l16 * VE; d < dim; d += 16 * VE) {
-                    float kv[VE];
-                    load_vec<T, VE>(src + d, kv);
-#pragma unroll
-                    for (int h = 0; h < HT; ++h)
-                        if (h < nh) {
-#pragma unroll
-                            for (int e = 0; e < VE; ++e) dot[h] += kv[e] * q[h * dim + d + e];
-                        }
-                }
+                for (int h = 0; h < HT; ++h) dot[u][h] = 0.f;
             }
+            for (int d = l16 * VE; d < dim; d += 16 * VE) {
+                float kv[4][VE];
 #pragma unroll
-            for (int h = 0; h < HT; ++h) dot[h] = group_sum(dot[h], 16);
-            if (l16 == 0 && kk < nk) {
+                for (int u = 0; u < 4; ++u)
+                    if (src[u] != nullptr) {
+                        load_vec<T, VE>(src[u] + d, kv[u]);
+                    } else {
+#pragma unroll
+                        for (int e = 0; e < VE; ++e) kv[u][e] = kn[d + e];
+                    }
 #pragma unroll
                 for (int h = 0; h < HT; ++h)
-                    if (h < nh) sc[h * kKeys + kk] = dot[h];
+                    if (h < nh) {
+#pragma unroll
+                        for (int e = 0; e < VE; ++e) {
+                            const float qv = q[h * dim + d + e];
+#pragma unroll
+                            for (int u = 0; u < 4; ++u) dot[u][h] += kv[u][e] * qv;
+                        }
+                    }
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const int kk = k4 + u * (kRowThreads / 16);
+#pragma unroll
+                for (int h = 0; h < HT; ++h) dot[u][h] = group_sum(dot[u][h], 16);
+                if (l16 == 0 && kk < nk) {
+#pragma unroll
+                    for (int h = 0; h < HT; ++h)
+                        if (h < nh) sc[h * kKeys + kk] = dot[u][h];
+                }
             }
         }
         __syncthreads();
@@ -223,6 +233,7 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
 #pragma unroll
                 for (int e = 0; e < VE; ++e) acc[h][e] *= corr;
             }
+#pragma unroll 4
             for (int kk = kl; kk < nk; kk += n_kl) {
                 const int kp = kb + kk;
                 const T* src = kp >= pos0 ? proj + (int64_t)(row0 + kp - pos0) * a.ld + a.off_v + (int64_t)kvh * vdim
@@ -370,9 +381,12 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const int cnt = p.b.count[seq];
     // an XCD (block index mod 8) takes the query blocks of neighbouring heads: their key head stays in its L2
     const int q_blocks = (p.b.max_count + kBQ - 1) / kBQ;
-    const int id = (blockIdx.x & 7) * (gridDim.x >> 3) + (blockIdx.x >> 3);  // (the grid is a multiple of 8)
+    const int idx = blockIdx.x >> 3, id = (blockIdx.x & 7) * (gridDim.x >> 3) + idx;  // (the grid is a multiple of 8)
     if (id >= q_blocks * a.heads) return;
-    const int h = id / q_blocks, qb = q_blocks - 1 - id % q_blocks;
+    // Long query blocks first; every second group of 32 (the CUs of an XCD) runs the other way round, so that of two workgroups that
+    // share a CU one walks many keys and one few
+    const bool up = 32 % q_blocks == 0 && ((idx >> 5) & 1);
+    const int h = id / q_blocks, qb = up ? id % q_blocks : q_blocks - 1 - id % q_blocks;
     if (qb * kBQ >= cnt) return;
     const int kvh = h / (a.heads / a.kv_heads);
     const int row0 = p.b.row0[seq], pos0 = p.b.pos[seq];
