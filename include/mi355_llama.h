@@ -735,6 +735,7 @@ typedef struct mi355_hybrid_model {
     float* x;              /* [max_rows, ldx] residual stream */
     float* xw;             /* [max_rows, ldx] rows whose logits are wanted */
     float* xn;             /* [max_rows, ldx] f32 models: normalised rows */
+    uint16_t* xb;          /* [max_rows, ldx] bf16 models: normalised rows of a wide product */
     void* proj;            /* [max_rows, widest in.N] of dtype */
     void* att;             /* [max_rows, widest out.K padded to 16] of dtype */
     void* hid;             /* [max_rows, widest up.N] of dtype */

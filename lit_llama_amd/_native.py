@@ -189,7 +189,7 @@ class HybridModel(C.Structure):
         ("ldx", c_int32), ("vocab", c_int32), ("max_rows", c_int32), ("ld_logits", c_int32),
         ("eps", c_float), ("residual_mult", c_float),
         ("embed", c_void_p), ("final_norm", c_void_p), ("head", Proj), ("layers", C.POINTER(HybridLayer)),
-        ("x", c_void_p), ("xw", c_void_p), ("xn", c_void_p), ("proj", c_void_p), ("att", c_void_p), ("hid", c_void_p),
+        ("x", c_void_p), ("xw", c_void_p), ("xn", c_void_p), ("xb", c_void_p), ("proj", c_void_p), ("att", c_void_p), ("hid", c_void_p),
         ("tmp", c_void_p), ("ld_att", c_int64), ("gemm_ws", c_void_p), ("gemm_ws_bytes", C.c_uint64),
         ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("rec_scratch", c_void_p), ("rec_scratch_bytes", C.c_uint64),
     ]

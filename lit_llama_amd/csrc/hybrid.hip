@@ -1,5 +1,5 @@
 // The forward pass of a layered hybrid model (mi355_hybrid_forward): a host-side walk over the layer runs that enqueues this library's
-// linears (gemv.hip for up to 16 rows, gemm.hip above, the exact f32 kernel for f32 models) and mixers (window_attention.hip,
+// linears (gemv.hip for a few rows, gemm.hip above, the exact f32 kernel for f32 models) and mixers (window_attention.hip,
 // recurrent.hip).  RMSNorm rides in the consuming linear and the residual sum in the producing one; the residual stream is f32.
 #include "common.h"
 
@@ -16,6 +16,48 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(const int32_t* tokens, 
 __global__ __launch_bounds__(256) void gather_rows_kernel(const float* x, const int32_t* want, float* xw, int ldx) {
     const int64_t src = (int64_t)want[blockIdx.x] * ldx, dst = (int64_t)blockIdx.x * ldx;
     for (int k = threadIdx.x; k < ldx; k += 256) xw[dst + k] = x[src + k];
+}
+
+// xb[m] = bf16(norm(x[m]) * scale), one row per workgroup: the operand of a wide product, multiplied where it lies.  K % 128 == 0, so rows
+// are whole 16-B vectors
+__global__ __launch_bounds__(512) void norm_rows_kernel(const float* x, int64_t ldx, const void* scale, int scale_dtype, float eps, int K,
+                                                        bf16_t* xb) {
+    __shared__ float red[32];
+    const f32x4* row = (const f32x4*)(x + (int64_t)blockIdx.x * ldx);
+    constexpr int kHeld = 4;  // vectors a thread keeps between the two passes
+    f32x4 v[kHeld];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i) {
+        const int j = threadIdx.x + i * 512;
+        v[i] = j < K / 4 ? row[j] : f32x4{0.f, 0.f, 0.f, 0.f};
+        ss += (v[i][0] * v[i][0] + v[i][1] * v[i][1]) + (v[i][2] * v[i][2] + v[i][3] * v[i][3]);
+    }
+    for (int j = threadIdx.x + kHeld * 512; j < K / 4; j += 512) {
+        const f32x4 w = row[j];
+        ss += (w[0] * w[0] + w[1] * w[1]) + (w[2] * w[2] + w[3] * w[3]);
+    }
+    const float rinv = 1.0f / sqrtf(block_sum(ss, red) / (float)K + eps);
+    u32x2* out = (u32x2*)(xb + (int64_t)blockIdx.x * K);
+    typedef __attribute__((ext_vector_type(2))) __bf16 bf2;
+    auto put = [&](int j, f32x4 w) {
+        float s[4];
+        if (scale_dtype == MI355_BF16) {
+            const u32x2 r = ((const u32x2*)scale)[j];
+            s[0] = __uint_as_float(r[0] << 16), s[1] = __uint_as_float(r[0] & 0xffff0000u);
+            s[2] = __uint_as_float(r[1] << 16), s[3] = __uint_as_float(r[1] & 0xffff0000u);
+        } else {
+            for (int e = 0; e < 4; ++e) s[e] = ld_as_f32(scale, 4 * j + e, scale_dtype);
+        }
+        const bf2 a = {(__bf16)(w[0] * rinv * s[0]), (__bf16)(w[1] * rinv * s[1])}, b = {(__bf16)(w[2] * rinv * s[2]), (__bf16)(w[3] * rinv * s[3])};
+        out[j] = u32x2{__builtin_bit_cast(uint32_t, a), __builtin_bit_cast(uint32_t, b)};
+    };
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i) {
+        const int j = threadIdx.x + i * 512;
+        if (j < K / 4) put(j, v[i]);
+    }
+    for (int j = threadIdx.x + kHeld * 512; j < K / 4; j += 512) put(j, row[j]);
 }
 
 __global__ __launch_bounds__(256) void relu2_kernel(float* h, int64_t n) {
@@ -95,19 +137,28 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
     a.y_dtype = y_dtype;
     a.ldy = ldy;
     const int most = mi355_linear_max_rows(MI355_W_BF16, w.K, 1, 0);
-    if (M > 16 || most < 1) {
+    // The weight-streaming kernel up to 8 rows; from there on, and for operands that leave its LDS room for a few rows only, the tiled
+    // product (split over K, the operand read in place) moves the weights faster: 4096 x 16512 at 4 / 8 / 16 rows 57 / 118 / 251 us against
+    // 28 / 28 / 30, 16512 x 4096 with the norm at 8 / 16 rows 31 / 41 against 35 / 36
+    const bool wide = M > 8 || most < M || (M > 2 && norm == nullptr && w.K > 12288 && w.K % 128 == 0);
+    if (wide) {
         a.x = x;
         a.y = y;
         a.M = M;
+        if (norm != nullptr && w.K % 128 == 0 && ldx % 4 == 0) {
+            hipLaunchKernelGGL(norm_rows_kernel, dim3(M), dim3(512), 0, s, (const float*)x, ldx, norm, m->norm_dtype, m->eps, w.K, m->xb);
+            MI355_LAUNCH_CHECK();
+            a.x = m->xb;
+            a.x_dtype = MI355_BF16;
+            a.ldx = w.K;
+            a.norm_scale = nullptr;
+        }
         return mi355_linear_gemm(&a, m->gemm_ws, (size_t)m->gemm_ws_bytes, s);
     }
-    for (int m0 = 0; m0 < M; m0 += most) {
-        a.M = M - m0 < most ? M - m0 : most;
-        a.x = (const char*)x + (int64_t)m0 * ldx * dtype_size(a.x_dtype);
-        a.y = (char*)y + (int64_t)m0 * ldy * dtype_size(y_dtype);
-        if (int rc = mi355_linear_fast(&a, s)) return rc;
-    }
-    return 0;
+    a.x = x;
+    a.y = y;
+    a.M = M;
+    return mi355_linear_fast(&a, s);
 }
 
 }  // namespace
@@ -115,7 +166,7 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
 extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq_batch* b, const int32_t* tokens, const int32_t* want,
                                     int n_want, float* logits, int run_end, mi355_stream_t stream) {
     MI355_CHECK_ARG(m && b && tokens && m->layers && m->x && m->proj && m->att && m->embed, MI355_E_ARG, "hybrid_forward: null argument");
-    MI355_CHECK_ARG(m->dtype == MI355_BF16 || (m->dtype == MI355_F32 && m->xn && m->tmp), MI355_E_DTYPE, "hybrid_forward: bad dtype");
+    MI355_CHECK_ARG((m->dtype == MI355_BF16 && m->xb) || (m->dtype == MI355_F32 && m->xn && m->tmp), MI355_E_DTYPE, "hybrid_forward: bad dtype");
     const int M = b->rows;
     MI355_CHECK_ARG(M > 0 && M <= m->max_rows && n_want >= 0 && (want != nullptr ? n_want <= m->max_rows : n_want == 0 || n_want == M),
                     MI355_E_SHAPE, "hybrid_forward: %d rows (of %d), %d wanted", M, m->max_rows, n_want);

@@ -31,27 +31,35 @@ __device__ __forceinline__ bf16_t from_f32<bf16_t>(float v) { return f32_to_bf16
 
 constexpr int kTaps = 8;  // taps a thread keeps in registers; longer convolutions take the loops
 
+// where input row r of a portion lies (rows of earlier portions below 0: in the ring).  Always a readable address, `ok` = the row exists:
+// loads without branches, so that all of a thread's requests are in flight together
+template <typename T>
+__device__ __forceinline__ const T* conv_input(const mi355_recurrent_args& a, const T* rows, const T* ring, int ring_ld, int off, int cr, int r,
+                                               int pos0, bool& ok) {
+    ok = ok && pos0 + r >= 0;
+    const T* old = ring + (int64_t)((unsigned)(ok ? pos0 + r : 0) % (unsigned)a.taps) * ring_ld + cr;
+    return r >= 0 ? rows + (int64_t)r * a.ld + off : old;
+}
+
 // one convolution output: channel c of the q | k | v inputs (`off` = its column in proj, `cr` = its column in the ring), row i of the
 // portion that starts at position pos0
 template <typename T>
 __device__ __forceinline__ float conv_at(const mi355_recurrent_args& a, const T* rows, const T* ring, int ring_ld, int off, int cr,
                                          const float* w, int i, int pos0) {
-    auto input = [&](int r) {  // row r of the portion, rows of earlier portions below 0
-        if (r >= 0) return to_f32<T>(rows[(int64_t)r * a.ld + off]);
-        return pos0 + r >= 0 ? to_f32<T>(ring[(int64_t)((pos0 + r) % a.taps) * ring_ld + cr]) : 0.f;
-    };
     float v = 0.f;
-    if (a.taps <= kTaps) {
-        float x[kTaps], wj[kTaps];
+    for (int j0 = 0; j0 < a.taps; j0 += 4) {
+        T x[4];
+        float wj[4];
+        bool ok[4];
 #pragma unroll
-        for (int j = 0; j < kTaps; ++j) {
-            x[j] = j < a.taps ? input(i - j) : 0.f;
-            wj[j] = j < a.taps ? w[a.taps - 1 - j] : 0.f;
+        for (int j = 0; j < 4; ++j) {
+            ok[j] = j0 + j < a.taps;
+            const int back = ok[j] ? j0 + j : 0;
+            x[j] = *conv_input<T>(a, rows, ring, ring_ld, off, cr, i - back, pos0, ok[j]);
+            wj[j] = w[a.taps - 1 - back];
         }
 #pragma unroll
-        for (int j = 0; j < kTaps; ++j) v += wj[j] * x[j];
-    } else {
-        for (int j = 0; j < a.taps; ++j) v += w[a.taps - 1 - j] * input(i - j);
+        for (int j = 0; j < 4; ++j) v += ok[j] ? wj[j] * to_f32<T>(x[j]) : 0.f;
     }
     return silu_f32(v);
 }
@@ -65,20 +73,21 @@ __device__ __forceinline__ void conv_rows16(const mi355_recurrent_args& a, const
         for (int t = 0; t < 16; ++t) out[t] = i + t < n ? conv_at<T>(a, rows, ring, ring_ld, off, cr, w, i + t, pos0) : 0.f;
         return;
     }
+    T raw[16 + kTaps - 1];
     float x[16 + kTaps - 1], wj[kTaps];
+    bool ok[16 + kTaps - 1];
 #pragma unroll
     for (int e = 0; e < 16 + kTaps - 1; ++e) {
         const int r = i + e - (kTaps - 1);
-        x[e] = 0.f;
-        if (e > kTaps - 1 - a.taps && r < n) {
-            if (r >= 0)
-                x[e] = to_f32<T>(rows[(int64_t)r * a.ld + off]);
-            else if (pos0 + r >= 0)
-                x[e] = to_f32<T>(ring[(int64_t)((pos0 + r) % a.taps) * ring_ld + cr]);
-        }
+        ok[e] = e > kTaps - 1 - a.taps && r < n;
+        raw[e] = *conv_input<T>(a, rows, ring, ring_ld, off, cr, ok[e] ? r : 0, pos0, ok[e]);
     }
 #pragma unroll
-    for (int j = 0; j < kTaps; ++j) wj[j] = j < a.taps ? w[a.taps - 1 - j] : 0.f;
+    for (int j = 0; j < kTaps; ++j) wj[j] = w[j < a.taps ? a.taps - 1 - j : 0];
+#pragma unroll
+    for (int e = 0; e < 16 + kTaps - 1; ++e) x[e] = ok[e] ? to_f32<T>(raw[e]) : 0.f;
+#pragma unroll
+    for (int j = 0; j < kTaps; ++j) wj[j] = j < a.taps ? wj[j] : 0.f;
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
         float v = 0.f;

@@ -153,7 +153,7 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
     }
 }
 
-// grid (taps, seqs): the last rows of every portion
+// grid (taps, seqs, column parts): the last rows of every portion
 template <typename T>
 __global__ __launch_bounds__(256) void conv_ring_kernel(const RecParams p) {
     const mi355_recurrent_args& a = p.a;
@@ -162,7 +162,7 @@ __global__ __launch_bounds__(256) void conv_ring_kernel(const RecParams p) {
     const int nqk = a.kv_heads * a.dim, nv = a.heads * a.vdim, ring_ld = 2 * nqk + nv;
     const T* src = (const T*)a.proj + (int64_t)(p.b.row0[seq] + i) * a.ld;
     T* dst = (T*)a.conv_ring + ((int64_t)p.b.slot[seq] * a.taps + (p.b.pos[seq] + i) % a.taps) * ring_ld;
-    for (int c = threadIdx.x; c < ring_ld; c += 256)
+    for (int c = blockIdx.z * 256 + threadIdx.x; c < ring_ld; c += 256 * gridDim.z)
         dst[c] = c < nqk ? src[a.off_q + c] : c < 2 * nqk ? src[a.off_k + c - nqk] : src[a.off_v + c - 2 * nqk];
 }
 
@@ -207,7 +207,7 @@ int run(const RecParams& p, hipStream_t s) {
         return rc;
     }
     if (p.a.kind == MI355_REC_DELTA && (chunks || p.b.max_count > 1)) {
-        hipLaunchKernelGGL(conv_ring_kernel<T>, dim3(p.a.taps < p.b.max_count ? p.a.taps : p.b.max_count, p.b.seqs), dim3(256), 0, s, p);
+        hipLaunchKernelGGL(conv_ring_kernel<T>, dim3(p.a.taps < p.b.max_count ? p.a.taps : p.b.max_count, p.b.seqs, 16), dim3(256), 0, s, p);
         MI355_LAUNCH_CHECK();
     }
     return 0;

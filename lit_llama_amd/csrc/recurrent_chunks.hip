@@ -339,14 +339,13 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
         {
             const int c = tid & 63, sb = tid >> 6, ch = c0 + c;
             const bool ok = ch < dim;
-            float qv[16], kv[16], z[16];
+            T qv[16], kv[16];
+            float z[16];
 #pragma unroll
-            for (int e = 0; e < 16; ++e) {
-                const int t = sb * 16 + e;
-                const bool in = ok && t < n;
-                const T* row = rows + (int64_t)(in ? t : 0) * a.ld + head * dim + (ok ? ch : 0);
-                qv[e] = in ? to_f32<T>(row[a.off_q]) * a.q_scale : 0.f;
-                kv[e] = in ? to_f32<T>(row[a.off_k]) : 0.f;
+            for (int e = 0; e < 16; ++e) {  // (all requests first: no branches)
+                const T* row = rows + (int64_t)min(sb * 16 + e, n - 1) * a.ld + head * dim + (ok ? ch : 0);
+                qv[e] = row[a.off_q];
+                kv[e] = row[a.off_k];
             }
             const float* w = a.a2 + (int64_t)(head * dim + (ok ? ch : 0)) * rank;
             const float bias = ok ? a.a2_bias[head * dim + ch] : 0.f;
@@ -368,8 +367,8 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
                 const int t = sb * 16 + e;
                 s += ok && t < n ? -softplus_f32(-z[e]) * a.inv_tau : 0.f;
                 G[t * kP + c] = s;   // sums from the block's first row on
-                q[t * kP + c] = qv[e];
-                k[t * kP + c] = kv[e];
+                q[t * kP + c] = ok && t < n ? to_f32<T>(qv[e]) * a.q_scale : 0.f;
+                k[t * kP + c] = ok && t < n ? to_f32<T>(kv[e]) : 0.f;
             }
             seg[sb * kCh + c] = s;
         }
@@ -495,7 +494,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
         if constexpr (KIND == MI355_REC_DELTA) {
             const float* W = p.s.W + hi * kC * DP + (int64_t)(wave * 16 + c16) * DP;
 #pragma unroll
-            for (int b = 0; b < 4 * NT; ++b) x.w[b] = b < n_tiles ? *(const f32x4*)(W + b * 16 + 4 * g) : zero4();
+            for (int b = 0; b < 4 * NT; ++b) x.w[b] = *(const f32x4*)(W + min(b, n_tiles - 1) * 16 + 4 * g);
             x.u = *(const f32x4*)(ut + wave * 16 + 4 * g);
             x.d = *(const f32x4*)(p.s.ed + hi * kC + wave * 16 + 4 * g);
             const float gm = p.s.gam[hi * DP];
@@ -505,14 +504,14 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
             for (int b = 0; b < 4; ++b) x.v[b] = *(const f32x4*)(ut + b * 16 + 4 * g);
 #pragma unroll
             for (int t = 0; t < NT; ++t)
-                x.g[t] = wave + 4 * t < n_tiles ? *(const f32x4*)(p.s.gam + hi * DP + (wave + 4 * t) * 16 + 4 * g) : zero4();
+                x.g[t] = *(const f32x4*)(p.s.gam + hi * DP + min(wave + 4 * t, n_tiles - 1) * 16 + 4 * g);
         }
         const float* kt = p.s.kt + gi * DP * kC;
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
-            const int row = (wave + 4 * t) * 16 + c16;
+            const int row = min(wave + 4 * t, n_tiles - 1) * 16 + c16;  // (tiles past the state: a copy of the last one, never stored)
 #pragma unroll
-            for (int b = 0; b < 4; ++b) x.k[t][b] = wave + 4 * t < n_tiles ? *(const f32x4*)(kt + row * kC + b * 16 + 4 * g) : zero4();
+            for (int b = 0; b < 4; ++b) x.k[t][b] = *(const f32x4*)(kt + row * kC + b * 16 + 4 * g);
         }
     };
     auto chunk = [&](int ch, Ops& x, Ops& next) {

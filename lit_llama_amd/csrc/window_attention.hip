@@ -69,7 +69,7 @@ struct WinParams {
 // ------------------------------------------------------------------------------------ row kernel
 // HT query heads of one key head per workgroup, VE consecutive elements per load (8: 16-B loads of bf16; 1: any head size)
 template <typename T, int HT, int VE>
-__global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParams p) {
+__global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kernel(const WinParams p) {
     const mi355_window_attn_args& a = p.a;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     const int tid = threadIdx.x;
@@ -80,8 +80,8 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
     const int h0 = kvh * per + ht * HT;
     const int dim = a.dim, vdim = a.vdim;
     float* q = (float*)smem;                      // [HT][dim], scaled
-    float* kn = q + HT * dim;                     // [dim]: the row's own key, as the ring stores it
-    float* sc = kn + dim;                         // [HT][kKeys]
+    float* kn = q + (HT * dim + 3) / 4 * 4;                     // [dim]: the row's own key, as the ring stores it
+    float* sc = kn + (dim + 3) / 4 * 4;           // [kKeys][HT]
     float* red = sc + HT * kKeys;                 // [kRowThreads][VE]
     float* stat = red + kRowThreads * VE;         // [3][HT]: maximum, sum, correction
     __shared__ int s_seq;
@@ -98,6 +98,9 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
     const T* prow = proj + (int64_t)row * a.ld;
     const T* kring = (const T*)a.kring + ((int64_t)p.b.slot[seq] * a.kv_heads + kvh) * a.ring * dim;
     const T* vring = (const T*)a.vring + ((int64_t)p.b.slot[seq] * a.kv_heads + kvh) * a.ring * vdim;
+
+    const T* kcur = proj + (int64_t)row0 * a.ld + a.off_k + (int64_t)kvh * dim;
+    const T* vcur = proj + (int64_t)row0 * a.ld + a.off_v + (int64_t)kvh * vdim;
 
     const int lo = max(0, pos - a.window + 1);
     const int n_keys = pos - lo + 1;
@@ -155,6 +158,7 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
 
     for (int kb = k_begin; kb < k_end; kb += kKeys) {
         const int nk = min(kKeys, k_end - kb);
+        const unsigned slot0 = (unsigned)kb % (unsigned)a.ring;  // (nk <= ring: a pass wraps once at most)
         // ---- scores: 16 lanes per key, four keys per lane group in flight
         const int l16 = tid & 15;
         for (int k4 = tid >> 4; k4 - (tid >> 4) < nk; k4 += 4 * (kRowThreads / 16)) {
@@ -162,23 +166,16 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
             const T* src[4];
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
-                const int kp = kb + min(k4 + u * (kRowThreads / 16), nk - 1);
-                src[u] = (p.fresh && kp == pos) ? nullptr
-                         : kp >= pos0           ? proj + (int64_t)(row0 + kp - pos0) * a.ld + a.off_k + (int64_t)kvh * dim
-                                                : kring + (int64_t)(kp % a.ring) * dim;
+                const int kk = min(k4 + u * (kRowThreads / 16), nk - 1), kp = kb + kk;
+                const unsigned sl = slot0 + kk < (unsigned)a.ring ? slot0 + kk : slot0 + kk - a.ring;
+                src[u] = kp >= pos0 ? kcur + (unsigned)(kp - pos0) * (unsigned)a.ld : kring + sl * (unsigned)dim;
 #pragma unroll
                 for (int h = 0; h < HT; ++h) dot[u][h] = 0.f;
             }
             for (int d = l16 * VE; d < dim; d += 16 * VE) {
                 float kv[4][VE];
 #pragma unroll
-                for (int u = 0; u < 4; ++u)
-                    if (src[u] != nullptr) {
-                        load_vec<T, VE>(src[u] + d, kv[u]);
-                    } else {
-#pragma unroll
-                        for (int e = 0; e < VE; ++e) kv[u][e] = kn[d + e];
-                    }
+                for (int u = 0; u < 4; ++u) load_vec<T, VE>(src[u] + d, kv[u]);
 #pragma unroll
                 for (int h = 0; h < HT; ++h)
                     if (h < nh) {
@@ -195,25 +192,32 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
                 const int kk = k4 + u * (kRowThreads / 16);
 #pragma unroll
                 for (int h = 0; h < HT; ++h) dot[u][h] = group_sum(dot[u][h], 16);
-                if (l16 == 0 && kk < nk) {
+                if (l16 == 0 && kk < nk && !(p.fresh && kb + kk == pos)) {
 #pragma unroll
                     for (int h = 0; h < HT; ++h)
-                        if (h < nh) sc[h * kKeys + kk] = dot[u][h];
+                        if (h < nh) sc[kk * HT + h] = dot[u][h];
                 }
             }
+        }
+        if (p.fresh && kb + nk > pos && (tid >> 4) < nh) {  // the row's own key, rotated above: lane group h takes head h
+            const int h = tid >> 4;
+            float s = 0.f;
+            for (int d = l16; d < dim; d += 16) s += kn[d] * q[h * dim + d];
+            s = group_sum(s, 16);
+            if (l16 == 0) sc[(pos - kb) * HT + h] = s;
         }
         __syncthreads();
         // ---- running maximum and sum: one wave per head
         for (int h = tid >> 6; h < nh; h += kRowThreads / 64) {
             const int lane = tid & 63;
             float m = -INFINITY;
-            for (int kk = lane; kk < nk; kk += 64) m = fmaxf(m, sc[h * kKeys + kk]);
+            for (int kk = lane; kk < nk; kk += 64) m = fmaxf(m, sc[kk * HT + h]);
             m = wave_max(m);
             const float m_old = stat[h], m_new = fmaxf(m_old, m);
             float l = 0.f;
             for (int kk = lane; kk < nk; kk += 64) {
-                const float e = expf(sc[h * kKeys + kk] - m_new);
-                sc[h * kKeys + kk] = e;
+                const float e = expf(sc[kk * HT + h] - m_new);
+                sc[kk * HT + h] = e;
                 l += e;
             }
             l = wave_sum(l);
@@ -236,16 +240,17 @@ __global__ __launch_bounds__(kRowThreads) void window_rows_kernel(const WinParam
 #pragma unroll 4
             for (int kk = kl; kk < nk; kk += n_kl) {
                 const int kp = kb + kk;
-                const T* src = kp >= pos0 ? proj + (int64_t)(row0 + kp - pos0) * a.ld + a.off_v + (int64_t)kvh * vdim
-                                          : vring + (int64_t)(kp % a.ring) * vdim;
-                float v[VE];
+                const unsigned sl = slot0 + kk < (unsigned)a.ring ? slot0 + kk : slot0 + kk - a.ring;
+                const T* src = kp >= pos0 ? vcur + (unsigned)(kp - pos0) * (unsigned)a.ld : vring + sl * (unsigned)vdim;
+                float v[VE], w[HT];
+#pragma unroll
+                for (int h = 0; h < HT; ++h) w[h] = sc[kk * HT + h];
                 load_vec<T, VE>(src + col * VE, v);
 #pragma unroll
                 for (int h = 0; h < HT; ++h)
                     if (h < nh) {
-                        const float w = sc[h * kKeys + kk];
 #pragma unroll
-                        for (int e = 0; e < VE; ++e) acc[h][e] += w * v[e];
+                        for (int e = 0; e < VE; ++e) acc[h][e] += w[h] * v[e];
                     }
             }
         }
@@ -621,7 +626,7 @@ int run_tiles(const WinParams& p, hipStream_t s) {
 
 template <typename T, int HT, int VE>
 int launch_rows(const WinParams& p, int rows, hipStream_t s) {
-    const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + (size_t)HT * kKeys + (size_t)kRowThreads * VE + 3 * HT) * 4;
+    const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + 8 + (size_t)HT * kKeys + (size_t)kRowThreads * VE + 3 * HT) * 4;
     MI355_CHECK_ARG(lds <= 160 * 1024 - 64, MI355_E_SHAPE, "window_attention: head size %d does not fit LDS", p.a.dim);
     if (lds > 64 * 1024) {
         static hipError_t e = hipFuncSetAttribute((const void*)window_rows_kernel<T, HT, VE>, hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -660,7 +665,7 @@ int run(WinParams p, hipStream_t s) {
         // splits: enough workgroups for the chip, at least 64 keys each, as far as the scratch goes
         const int per = a.heads / a.kv_heads, ht = per >= 5 ? 8 : per >= 2 ? 4 : 1;
         const int groups = p.b.rows * a.kv_heads * ((per + ht - 1) / ht);
-        int n = 512 / groups;
+        int n = 2048 / groups;
         n = n < a.ring / 64 ? n : a.ring / 64;
         n = n < kMaxSplit ? n : kMaxSplit;
         const uint64_t rec = (uint64_t)p.b.rows * a.heads * (a.vdim + 2) * 4;
@@ -702,6 +707,9 @@ extern "C" int mi355_window_attention(const mi355_window_attn_args* a, const mi3
     MI355_CHECK_ARG(a->dtype == MI355_F32 || a->dtype == MI355_BF16, MI355_E_DTYPE, "window_attention: dtype must be f32 or bf16");
     MI355_CHECK_ARG(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim > 0 && a->vdim > 0, MI355_E_SHAPE,
                     "window_attention: bad heads %d / %d or sizes %d / %d", a->heads, a->kv_heads, a->dim, a->vdim);
+    MI355_CHECK_ARG((uint64_t)b->max_count * (uint64_t)a->ld < 0xFFFFFFFFull && (uint64_t)a->ring * (a->dim > a->vdim ? a->dim : a->vdim) < 0xFFFFFFFFull,
+                    MI355_E_SHAPE, "window_attention: %d rows of pitch %lld or a ring of %d rows exceed 32-bit offsets", b->max_count,
+                    (long long)a->ld, a->ring);
     MI355_CHECK_ARG(a->window > 0 && a->ring > 0 && a->rot_dims >= 0 && a->rot_dims % 2 == 0 && a->rot_dims <= a->dim &&
                         (a->rot_dims == 0 || a->inv_freq),
                     MI355_E_SHAPE, "window_attention: bad window %d, ring %d or rotation %d", a->window, a->ring, a->rot_dims);

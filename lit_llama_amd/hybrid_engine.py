@@ -160,6 +160,7 @@ class HybridEngine:
             K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down)])
             n = int(lib().mi355_linear_gemm_workspace_bytes(R, K))
             M.gemm_ws, M.gemm_ws_bytes = ptr(self._buf(n, torch.uint8)), n
+            M.xb = ptr(self._buf(R * M.ldx, torch.bfloat16))
         # a split attention step keeps one record per (row, head, split); one split takes none
         n = max([512 * (l.attn.vdim + 2) * max(8, l.attn.heads // l.attn.kv_heads) for l in ls if l.mixer == 0], default=0)
         M.partials, M.partials_bytes = ptr(self._buf(n, torch.float32)), n * 4
