@@ -368,6 +368,11 @@ __device__ __forceinline__ uint32_t pack_bf16x2(float a, float b) {
     const bf16x2_t v = {(__bf16)a, (__bf16)b};
     return __builtin_bit_cast(uint32_t, v);
 }
+__device__ __forceinline__ float max3f(float a, float b, float c) {
+    float r;
+    asm("v_max3_f32 %0, %1, %2, %3" : "=v"(r) : "v"(a), "v"(b), "v"(c));
+    return r;
+}
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 
 template <int D>  // both head sizes padded to D (a multiple of 32)
@@ -443,7 +448,36 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const int p_last = pos0 + cnt - 1;
     u32x4 kreg[kKItems], vreg[kVItems][4];
     const u32x4 zero4 = {0u, 0u, 0u, 0u};
+    const int t_key = threadIdx.x / kCols, t_col = threadIdx.x % kCols, t_run = threadIdx.x & 15, t_vcol = threadIdx.x >> 4;
+    const bool k_in = t_col * 8 < a.dim;
     auto load_tile = [&](int kb) {
+        if (kb * kBK >= pos0 && kb * kBK + kBK - 1 <= p_last) {  // all of the step's own rows: one multiply per thread
+            const unsigned ld = (unsigned)a.ld;
+            const unsigned ko = (unsigned)(kb * kBK + t_key - pos0) * ld + t_col * 8;
+#pragma unroll
+            for (int i = 0; i < kKItems; ++i) kreg[i] = *(const u32x4*)(kcur + (k_in ? ko + (unsigned)i * (256 / kCols) * ld : 0u));
+            const unsigned vo = (unsigned)(kb * kBK + t_run * 4 - pos0) * ld;
+#pragma unroll
+            for (int i = 0; i < kVItems; ++i) {
+                const int col = t_vcol + 16 * i;
+                const unsigned o = col * 8 < a.vdim ? vo + col * 8 : 0u;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) vreg[i][r] = *(const u32x4*)(vcur + (o + (unsigned)r * ld));
+            }
+            if (!k_in) {
+#pragma unroll
+                for (int i = 0; i < kKItems; ++i) kreg[i] = zero4;
+            }
+            if (D != a.vdim) {
+#pragma unroll
+                for (int i = 0; i < kVItems; ++i)
+                    if ((t_vcol + 16 * i) * 8 >= a.vdim) {
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) vreg[i][r] = zero4;
+                    }
+            }
+            return;
+        }
 #pragma unroll
         for (int i = 0; i < kKItems; ++i) {
             const int it = i * 256 + threadIdx.x, key = it / kCols, col = it % kCols;
@@ -537,12 +571,12 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                         st[t2][i] = (kp <= q_pos && kp > q_pos - a.window) ? st[t2][i] : -1.0e30f;
                     }
             }
-            float m_blk = -1.0e30f;
+            // (inline assembly gets no wait states behind the matrix instruction that wrote its operands: 20 here cover the longest)
+            asm volatile("s_nop 15\n\ts_nop 3" : "+v"(st[0]), "+v"(st[1]));
+            float m_blk = max3f(st[0][0], st[1][0], st[0][1]);  // (v_max3_f32: fmaxf() canonicalises every MFMA result first)
 #pragma unroll
-            for (int t2 = 0; t2 < 2; ++t2)
-#pragma unroll
-                for (int i = 0; i < 16; ++i) m_blk = fmaxf(m_blk, st[t2][i]);
-            m_blk = fmaxf(m_blk, lane_xor32(m_blk));
+            for (int i = 1; i < 16; ++i) m_blk = max3f(m_blk, st[1][i], i < 15 ? st[0][i + 1] : st[1][i]);
+            m_blk = max3f(m_blk, lane_xor32(m_blk), m_blk);
             // the reference maximum moves only when it is exceeded by 2^8 (exp2 domain): few steps rescale the outputs.  (A query whose
             // first keys are all masked sums ones at m = -1e30; its first visible key moves m and wipes them out with exp2(-1e30) = 0.)
             const bool move = m_blk > m_run + 8.0f;

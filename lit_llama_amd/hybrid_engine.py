@@ -190,6 +190,8 @@ class HybridEngine:
         """Rings hold min(window, longest sequence) rows.  Growing them re-lays the rings, so no sequence may be live unless every ring
         already spans its window."""
         need = any(l.mixer == 0 and self._ring(l, n) != self._ring(l, self.max_len) for l in list(self.layers)[: self.m.n_runs])
+        if need and self.slots.live == 1 and self._single is not None:
+            self.reset_cache()  # (what is live is a sequence that generate() or forward() left behind)
         if need and self.max_len and self.slots.live:
             raise nat.NativeError(f"hybrid engine: sequences are live at cache length {self.max_len}; {n} needs a larger one")
         self.max_len = n

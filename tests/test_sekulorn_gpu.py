@@ -174,6 +174,7 @@ def run_rec(dev, kind, p, off, w, H, G, dim, vdim, cuts, path=0, taps=4, slots=(
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("kind,H,G,dim,vdim,taps", [("delta", 4, 2, 24, 40, 4), ("delta", 3, 3, 64, 32, 2), ("delta", 2, 1, 130, 70, 5), ("delta", 2, 2, 16, 144, 1),
+                                                    ("delta", 1, 1, 33, 17, 9),
                                                     ("gla", 3, 3, 24, 40, 0), ("gla", 2, 2, 130, 70, 0), ("gla", 1, 1, 64, 128, 0)])
 def test_recurrences(dev, dtype, kind, H, G, dim, vdim, taps):
     T = 203
@@ -245,16 +246,16 @@ def test_model_layer_by_layer_and_logits(dev, name):
     eng.release(s)
 
 
-@pytest.mark.parametrize("dtype,tol", [(torch.float32, 1e-4), (torch.bfloat16, 0.12)])
-def test_portions_batches_slots_and_decoding(dev, dtype, tol):
+@pytest.mark.parametrize("name,dtype,tol", [("mixed", torch.float32, 1e-4), ("mixed", torch.bfloat16, 0.12), ("all looped", torch.bfloat16, 0.12)])
+def test_portions_batches_slots_and_decoding(dev, name, dtype, tol):
     """Unequal requests in one batch, cut differently, decoded together, their slots used again: the logits of each alone."""
     from lit_llama_amd.hybrid_engine import Entry
 
-    config = CONFIGS["mixed"]
+    config = CONFIGS[name]
     m, sd = build(config, dtype, dev)
     eng = m.engine()
     eng.ensure(4, 200)
-    seqs = [tokens_of(n, seed=n) for n in (150, 9, 64, 33)]
+    seqs = [tokens_of(n, config["vocab"], seed=n) for n in (150, 9, 64, 33)]
     refs = [O.forward(config, sd, s)[0] for s in seqs]
     for first in ((100, 2, 31, 32), (64, 8, 1, 3)):  # (the second time in the slots of the first)
         slots = [eng.acquire() for _ in seqs]
@@ -339,6 +340,10 @@ def test_greedy_generation_through_generate_and_the_scheduler(dev):
         assert y[:len(p)] == p and len(y) == len(p) + 12 and y[len(p):len(p) + len(r)] == r
     again = lit_llama_amd.generate(m, torch.tensor(prompts[0], device=dev), 12, top_k=1).tolist()
     assert again[len(prompts[0]):] == outs[0]
+    # a batch behind generate() that needs longer rings than its sequence
+    fresh, _ = build(config, torch.float32, dev)
+    lit_llama_amd.generate(fresh, torch.tensor([1, 2, 3], device=dev), 2, top_k=1)
+    assert generate_batch(fresh, prompts[:2], 12, top_k=1) == outs[:2]
     # eos ends a request early and the others go on
     eos = outs[0][4]
     cut = generate_batch(m, prompts, 12, top_k=1, eos_id=eos)
