@@ -18,7 +18,7 @@ typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2_t;
 
 constexpr int kRowThreads = 256;
 constexpr int kKeys = 256;        // keys per pass of the row kernel
-constexpr int kMaxSplit = 32;     // workgroups over the keys of one (row, key head) in a decode step
+constexpr int kMaxSplit = 32;     // (<= 64, a lane each) workgroups over the keys of one (row, key head) in a decode step
 constexpr double kInvTwoPi = 0.15915494309189533577;
 
 // turn of (u, v) by pos * inv_freq: the angle is reduced in f64, so far positions keep f32 accuracy
@@ -82,8 +82,8 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     float* q = (float*)smem;                      // [HT][dim], scaled
     float* kn = q + (HT * dim + 3) / 4 * 4;                     // [dim]: the row's own key, as the ring stores it
     float* sc = kn + (dim + 3) / 4 * 4;           // [kKeys][HT]
-    float* red = sc + HT * kKeys;                 // [kRowThreads][VE]
-    float* stat = red + kRowThreads * VE;         // [3][HT]: maximum, sum, correction
+    float* stat = sc + HT * kKeys;                // [3][HT]: maximum, sum, correction
+    float* red = stat + 4 * HT;                   // [key lanes][HT][columns]: at most kRowThreads HT VE
     __shared__ int s_seq;
 
     if (!p.fresh) {
@@ -257,34 +257,35 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
         __syncthreads();
     }
     // ---- sum over the key lanes, gate, store
-    for (int h = 0; h < HT; ++h) {
-        if (h >= nh) break;
-        if (kl < n_kl) {
+    auto put = [&](int h, int d, float o) {
+        if (p.n_split > 1) {
+            a.partials[(((int64_t)row * a.heads + h0 + h) * p.n_split + split) * (vdim + 2) + 2 + d] = o;
+        } else {
+            o /= stat[HT + h];
+            if (a.off_g >= 0) o *= 1.0f / (1.0f + expf(-to_f32<T>(prow[a.off_g + h0 + h])));
+            ((T*)a.y)[(int64_t)row * a.ldy + (int64_t)(h0 + h) * vdim + d] = from_f32<T>(o);
+        }
+    };
+    if (p.n_split > 1 && tid < nh) {
+        float* rec = a.partials + (((int64_t)row * a.heads + h0 + tid) * p.n_split + split) * (vdim + 2);
+        rec[0] = stat[tid];
+        rec[1] = stat[HT + tid];
+    }
+    // (every key lane's sums to LDS at once: code that runs once per launch is paid for by instruction fetches, so it is kept short)
+    const int cols = n_cols * VE;
+    if (kl < n_kl) {
 #pragma unroll
-            for (int hh = 0; hh < HT; ++hh)
-                if (hh == h) {
+        for (int h = 0; h < HT; ++h)
 #pragma unroll
-                    for (int e = 0; e < VE; ++e) red[(kl * n_cols + col) * VE + e] = acc[hh][e];
-                }
-        }
-        __syncthreads();
-        for (int d = tid; d < vdim; d += kRowThreads) {
-            float o = 0.f;
-            for (int k = 0; k < n_kl; ++k) o += red[k * n_cols * VE + d];
-            if (p.n_split > 1) {
-                a.partials[(((int64_t)row * a.heads + h0 + h) * p.n_split + split) * (vdim + 2) + 2 + d] = o;
-            } else {
-                o /= stat[HT + h];
-                if (a.off_g >= 0) o *= 1.0f / (1.0f + expf(-to_f32<T>(prow[a.off_g + h0 + h])));
-                ((T*)a.y)[(int64_t)row * a.ldy + (int64_t)(h0 + h) * vdim + d] = from_f32<T>(o);
-            }
-        }
-        if (p.n_split > 1 && tid == 0) {
-            float* rec = a.partials + (((int64_t)row * a.heads + h0 + h) * p.n_split + split) * (vdim + 2);
-            rec[0] = stat[h];
-            rec[1] = stat[HT + h];
-        }
-        __syncthreads();
+            for (int e = 0; e < VE; ++e) red[(kl * HT + h) * cols + col * VE + e] = acc[h][e];
+    }
+    __syncthreads();
+    for (int i = tid; i < nh * cols; i += kRowThreads) {
+        const int h = i / cols, d = i - h * cols;
+        float o = 0.f;
+#pragma unroll 4
+        for (int k = 0; k < n_kl; ++k) o += red[k * HT * cols + i];
+        if (d < vdim) put(h, d, o);
     }
 }
 
@@ -294,19 +295,16 @@ __global__ __launch_bounds__(128) void window_join_kernel(const WinParams p) {
     const mi355_window_attn_args& a = p.a;
     const int h = blockIdx.x, row = blockIdx.y;
     const float* rec = a.partials + ((int64_t)row * a.heads + h) * p.n_split * (a.vdim + 2);
-    float m = -INFINITY;
-#pragma unroll 16
-    for (int s = 0; s < p.n_split; ++s) m = fmaxf(m, rec[s * (a.vdim + 2)]);
     __shared__ float wgt[kMaxSplit];
-    float l = 0.f;
-    for (int s = 0; s < p.n_split; ++s) {
-        const float e = expf(rec[s * (a.vdim + 2)] - m);
-        l += e * rec[s * (a.vdim + 2) + 1];
-        if ((int)threadIdx.x == s) wgt[s] = e;
-    }
-    __syncthreads();
-    float gate = 1.f / l;
+    const int lane = threadIdx.x & 63;  // (every wave joins the maxima and sums: lane = split)
+    const bool in = lane < p.n_split;
+    const float ms = in ? rec[lane * (a.vdim + 2)] : -INFINITY, ls = in ? rec[lane * (a.vdim + 2) + 1] : 0.f;
+    const float m = wave_max(ms);
+    const float e = expf(ms - m);
+    if ((int)threadIdx.x < p.n_split) wgt[threadIdx.x] = e;
+    float gate = 1.f / group_sum(e * ls, 64);
     if (a.off_g >= 0) gate /= 1.0f + expf(-to_f32<T>(((const T*)a.proj)[(int64_t)row * a.ld + a.off_g + h]));
+    __syncthreads();
     for (int d = threadIdx.x; d < a.vdim; d += blockDim.x) {
         float o = 0.f;
 #pragma unroll 16
@@ -660,7 +658,8 @@ int run_tiles(const WinParams& p, hipStream_t s) {
 
 template <typename T, int HT, int VE>
 int launch_rows(const WinParams& p, int rows, hipStream_t s) {
-    const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + 8 + (size_t)HT * kKeys + (size_t)kRowThreads * VE + 3 * HT) * 4;
+    const size_t red = (size_t)kRowThreads * HT * VE;
+    const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + 8 + (size_t)HT * kKeys + 4 * HT + red) * 4;
     MI355_CHECK_ARG(lds <= 160 * 1024 - 64, MI355_E_SHAPE, "window_attention: head size %d does not fit LDS", p.a.dim);
     if (lds > 64 * 1024) {
         static hipError_t e = hipFuncSetAttribute((const void*)window_rows_kernel<T, HT, VE>, hipFuncAttributeMaxDynamicSharedMemorySize,

@@ -8,7 +8,9 @@ attributes and methods as `engine.DecodeEngine` (`_ensure_cache`, `prefill`, `se
 from __future__ import annotations
 
 import ctypes as C
+import gc
 import os
+import weakref
 from typing import Dict, List, NamedTuple, Optional, Sequence
 
 import torch
@@ -40,7 +42,8 @@ class HybridEngine:
     supports_batches = True
 
     def __init__(self, model: HybridLM, *, max_rows: Optional[int] = None):
-        self.model, self.cfg, self.device = model, model.config, model.device
+        # (the weights, not the model: the model owns its engine, and a cycle would leave both to the garbage collector)
+        self.weights, self.cfg, self.device = model.tensors, model.config, model.device
         self.dtype = model.dtype
         self.max_rows = max_rows or int(os.environ.get("MI355_HYBRID_ROWS", "4096"))
         self.use_graph = os.environ.get("MI355_HYBRID_GRAPH", "1") != "0"
@@ -53,7 +56,8 @@ class HybridEngine:
             self.stream.wait_stream(torch.cuda.default_stream(self.device))
             self._pack()
             self._scratch()
-        self.slots = SlotManager(self._grow)
+        grow = weakref.WeakMethod(self._grow)
+        self.slots = SlotManager(lambda n: grow()(n))
         self._single: Optional[int] = None  # generate()'s slot
         self.stream.synchronize()
 
@@ -78,7 +82,7 @@ class HybridEngine:
         return ptr(t)
 
     def _pack(self) -> None:
-        cfg, T = self.cfg, self.model.tensors
+        cfg, T = self.cfg, self.weights
         self.weight_bytes = 0
         self.norm_dtype = nat.dtype_code(self.dtype)
         layers = []
@@ -341,12 +345,19 @@ class HybridEngine:
             return
         g = self._graphs.get(key)
         if g is None:
-            check(lib().mi355_graph_begin(s), "mi355_graph_begin")
-            handle = C.c_void_p()
+            # a collection inside the capture may free another engine or a tensor: synchronizing calls, which end the capture
+            collecting = gc.isenabled()
+            gc.disable()
             try:
-                enqueue()
+                check(lib().mi355_graph_begin(s), "mi355_graph_begin")
+                handle = C.c_void_p()
+                try:
+                    enqueue()
+                finally:
+                    rc = lib().mi355_graph_end(s, C.byref(handle))
             finally:
-                rc = lib().mi355_graph_end(s, C.byref(handle))
+                if collecting:
+                    gc.enable()
             check(rc, "mi355_graph_end")
             g = self._graphs[key] = handle
         check(lib().mi355_graph_launch(g, s), "mi355_graph_launch")

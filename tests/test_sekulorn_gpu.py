@@ -367,6 +367,28 @@ def test_sampled_generation(dev):
     assert x == y and [len(o) for o in x] == [15, 15]
 
 
+def test_a_dropped_model_frees_its_engine_without_the_collector(dev):
+    import gc
+    import weakref
+
+    from lit_llama_amd.hybrid_engine import Entry
+
+    m, _ = build(CONFIGS["mixed"], torch.float32, dev)
+    eng = m.engine()
+    eng.ensure(1, 16)
+    s = eng.acquire()
+    for i in range(4):  # (a captured step included)
+        eng.step([Entry(s, i, [i], [0])])
+    alive = weakref.ref(eng)
+    gc.collect()
+    gc.disable()
+    try:
+        del eng, m
+        assert alive() is None
+    finally:
+        gc.enable()
+
+
 def test_long_decoding_matches_the_prompt_pass(dev):
     """Hundreds of decoded tokens (windows pass over them, graphs replayed, eager work in between) against one prompt pass."""
     from lit_llama_amd.hybrid_engine import Entry
