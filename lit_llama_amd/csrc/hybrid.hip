@@ -10,7 +10,23 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(const int32_t* tokens, 
                                                          int vocab) {
     const int m = blockIdx.x;
     const int tok = min(max(tokens[m], 0), vocab - 1);
-    for (int k = threadIdx.x; k < ldx; k += 256) x[(int64_t)m * ldx + k] = k < width ? ld_as_f32(wte, (int64_t)tok * width + k, dtype) : 0.f;
+    float* dst = x + (int64_t)m * ldx;
+    if (dtype == MI355_BF16 && width % 8 == 0) {  // (ldx is a multiple of 16)
+        const u32x4* src = (const u32x4*)((const bf16_t*)wte + (int64_t)tok * width);
+        for (int j = threadIdx.x; j < ldx / 8; j += 256) {
+            const u32x4 r = j < width / 8 ? src[j] : u32x4{0u, 0u, 0u, 0u};
+            f32x4 lo, hi;
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+                lo[2 * e] = __uint_as_float(r[e] << 16), lo[2 * e + 1] = __uint_as_float(r[e] & 0xffff0000u);
+                hi[2 * e] = __uint_as_float(r[2 + e] << 16), hi[2 * e + 1] = __uint_as_float(r[2 + e] & 0xffff0000u);
+            }
+            ((f32x4*)dst)[2 * j] = lo;
+            ((f32x4*)dst)[2 * j + 1] = hi;
+        }
+        return;
+    }
+    for (int k = threadIdx.x; k < ldx; k += 256) dst[k] = k < width ? ld_as_f32(wte, (int64_t)tok * width + k, dtype) : 0.f;
 }
 
 __global__ __launch_bounds__(256) void gather_rows_kernel(const float* x, const int32_t* want, float* xw, int ldx) {
