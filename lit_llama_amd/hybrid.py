@@ -46,11 +46,13 @@ def _only(d: dict, known: Tuple[str, ...], what: str) -> None:
 
 
 def _attention(m: dict) -> MixerSpec:
+    """No `rot`: no rotation; no `mask`: every earlier row is seen."""
     _only(m, ("heads", "kv_heads", "dim", "vdim", "rot", "scale", "mask"), "attention mixer")
-    _only(m["rot"], ("base", "dims"), "rotation")
-    _only(m["mask"], ("size",), "mask")
-    return MixerSpec("attention", m["heads"], m["kv_heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=int(m["mask"]["size"]),
-                     rot_dims=int(m["rot"]["dims"]), rot_base=float(m["rot"]["base"]))
+    rot, mask = m.get("rot") or {"base": 1.0, "dims": 0}, m.get("mask") or {"size": 1 << 30}
+    _only(rot, ("base", "dims"), "rotation")
+    _only(mask, ("size",), "mask")
+    return MixerSpec("attention", m["heads"], m["kv_heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=int(mask["size"]),
+                     rot_dims=int(rot["dims"]), rot_base=float(rot["base"]))
 
 
 def _delta(m: dict) -> MixerSpec:
@@ -147,7 +149,7 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
 class HybridLM(nn.Module):
     """Weights by checkpoint name (`model.tensors["l0.mix.q"]`), forward through the native engine.
 
-    `forward(idx, max_seq_length, input_pos)` is LLaMA.forward's contract for one sequence with a cache; batches go through
+    `forward(idx, max_seq_length, input_pos)` is LLaMA.forward's interface for one sequence with a cache; batches go through
     `engine().step` (batching.BatchScheduler)."""
 
     def __init__(self, config: HybridConfig, dtype: torch.dtype = torch.bfloat16, device="cuda"):

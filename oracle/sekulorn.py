@@ -106,8 +106,9 @@ def attention_mixer(w: Tensors, p: str, m: dict, h: torch.Tensor, eps: float) ->
     q = (h @ w[p + "q"].T).view(T, m["heads"], m["dim"])
     k = (h @ w[p + "k"].T).view(T, m["kv_heads"], m["dim"])
     v = (h @ w[p + "v"].T).view(T, m["kv_heads"], m["vdim"])
-    q, k = (rotate_pairs(t, m["rot"]["dims"], m["rot"]["base"]) for t in (q, k))
-    o = window_attention(q, k, v, m["scale"], m["mask"]["size"])
+    if m.get("rot"):
+        q, k = (rotate_pairs(t, m["rot"]["dims"], m["rot"]["base"]) for t in (q, k))
+    o = window_attention(q, k, v, m["scale"], m["mask"]["size"] if m.get("mask") else T)
     o = o * torch.sigmoid(h @ w[p + "g"].T)[:, :, None]
     return o.reshape(T, -1) @ w[p + "o"].T
 

@@ -222,6 +222,8 @@ def tokens_of(n, vocab=211, seed=0):
 CONFIGS = {
     "mixed": small_config(),
     "no loop, unit multiplier": small_config(loop=None, residual_mult=1.0),
+    "no rotation, no window": small_config(layers=[{"type": "attention", "mixer": {"heads": 3, "kv_heads": 1, "dim": 16, "vdim": 16, "scale": 0.25},
+                                                    "mlp": None}], loop=None, width=64),
     "all looped": small_config(loop={"start": 0, "stop": 4, "times": 2}, width=97, vocab=130),
 }
 
