@@ -10,7 +10,7 @@ src=fused_step_ring.hip
 if [ "$1" = "-s" ]; then src=$2; shift 2; fi
 mkdir -p lit_llama_amd/_variants /tmp/variants
 obj=/tmp/variants/${src%.hip}_$tag.o
-/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -Wall -Wno-unused-function "$@" -c lit_llama_amd/csrc/$src -o $obj
+/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -Wall -Wno-unused-function -Xclang -target-feature -Xclang -packed-fp32-ops "$@" -c lit_llama_amd/csrc/$src -o $obj
 objs=$(ls lit_llama_amd/csrc/_obj/*.o | grep -v "/$src.o")
 /opt/rocm/bin/hipcc --offload-arch=gfx950 -shared -fPIC -o lit_llama_amd/_variants/libmi355llama_$tag.so $objs $obj
 echo built lit_llama_amd/_variants/libmi355llama_$tag.so
