@@ -34,9 +34,10 @@ enum { MI355_E_ARG = -1, MI355_E_SHAPE = -2, MI355_E_DTYPE = -3, MI355_E_STATE =
 /* weight stream formats of the fast (MFMA, M<=16) linear */
 enum { MI355_W_Q4 = 0, MI355_W_BF16 = 1, MI355_W_I8 = 2 };
 /* epilogues of the fast linear */
-enum { MI355_EPI_STORE = 0, MI355_EPI_ACCUM = 1, MI355_EPI_SWIGLU = 2 };
-/* bits of mi355_linear_args.flags: STORE writes max(y, 0)^2 */
-enum { MI355_LF_RELU2 = 1 };
+/* (GEGLU: the pair stream with the tanh form of GELU instead of SiLU; BF16 streams only) */
+enum { MI355_EPI_STORE = 0, MI355_EPI_ACCUM = 1, MI355_EPI_SWIGLU = 2, MI355_EPI_GEGLU = 3 };
+/* bits of mi355_linear_args.flags: STORE writes max(y, 0)^2; the norm's scale is 1 + norm_scale */
+enum { MI355_LF_RELU2 = 1, MI355_LF_NORM_ONE = 2 };
 
 typedef void* mi355_stream_t; /* hipStream_t */
 
@@ -631,11 +632,16 @@ typedef struct mi355_seq_batch {
     const int32_t* pos;    /* device [seqs] */
 } mi355_seq_batch;
 
-/* Causal attention over a sliding window with grouped key / value heads, partial interleaved rotation and a sigmoid gate per
- * head.  Row i of a sequence sees rows j with 0 <= i - j < window.  The cache of a slot is a ring of `ring` rows per key head
- * (position p in row p % ring; ring >= window or >= the longest sequence). */
+/* Causal attention over a sliding window with grouped key / value heads, partial interleaved rotation and sigmoid gates.
+ * Row i of a sequence sees rows j <= i with i - j < window or j < keep.  The cache of a slot is, per key head, `kept` >= keep rows
+ * (positions below kept) and a ring of `ring` rows (position p in row kept + (p - kept) % ring; ring >= window or >= the longest
+ * sequence).
+ * role: a layer that LENDS its keys and values leaves a prompt step's prepared rows in kv_rows, and its cache rows are written
+ * by mi355_window_cache_write behind its last borrower; a layer that BORROWS has the lender's rings (and kept, ring, kv_rows) and
+ * no key / value columns.  Lender and borrowers may differ in window and keep: kept and ring cover all of them. */
+enum { MI355_KV_OWN = 0, MI355_KV_LENDS = 1, MI355_KV_BORROWS = 2 };
 typedef struct mi355_window_attn_args {
-    void* proj;            /* [rows, ld]: q, k, v, gate columns; q and k are rotated IN PLACE by a prompt step */
+    void* proj;            /* [rows, ld]: q, k, v, gate columns; a prompt step normalises and rotates k IN PLACE (role 0) */
     int64_t ld;
     int32_t dtype;         /* of proj, rings and y: F32 or BF16 */
     int32_t heads, kv_heads, dim, vdim;
@@ -644,17 +650,26 @@ typedef struct mi355_window_attn_args {
     int32_t window, ring;
     int32_t rot_dims;      /* 0: no rotation */
     const double* inv_freq; /* device [rot_dims / 2]: pair (2i, 2i + 1) turns by position * inv_freq[i] */
-    void* kring;           /* [slots][kv_heads][ring][dim] */
-    void* vring;           /* [slots][kv_heads][ring][vdim] */
+    void* kring;           /* [slots][kv_heads][kept + ring][dim] */
+    void* vring;           /* [slots][kv_heads][kept + ring][vdim] */
     void* y;               /* [rows, ldy], head h at column h * vdim */
     int64_t ldy;
     float* partials;       /* scratch of a split decode step, or NULL */
     uint64_t partials_bytes;
     int32_t path;          /* 0: by shape; 1: one workgroup per row; 2: matrix-core tiles (bf16 prompts) */
+    int32_t keep, kept;
+    int32_t gate_values;   /* 0: one gate column per head; 1: heads * vdim gate columns */
+    int32_t unit_qk;       /* != 0: q and k of a head are divided by their root mean square (unit_eps inside the root) */
+    float unit_eps;
+    const float* sink;     /* [heads]: exp(sink) joins the sum of every softmax, or NULL */
+    int32_t role;          /* MI355_KV_* */
     int32_t reserved0;
+    void* kv_rows;         /* [rows][kv_heads * dim | kv_heads * vdim] of dtype, lender and borrowers */
 } mi355_window_attn_args;
 
 int mi355_window_attention(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
+/* the cache rows of a lender's prompt step (nothing to do in a decode step) */
+int mi355_window_cache_write(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
 
 /* Linear recurrences over a state S [dim, vdim] per head, kept in f32 [slots][heads][dim][vdim]:
  *   kind MI355_REC_DELTA  gated delta rule: short causal convolutions + SiLU on q, k, v; unit q, k; S = g S, u = beta (v - S^T k),
@@ -697,6 +712,40 @@ int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_batch* b, mi3
 /* scratch bytes a chunked prompt step of `rows` rows in `seqs` sequences takes; 0: the shape runs row by row */
 size_t mi355_recurrent_scratch_bytes(int kind, int rows, int seqs, int heads, int kv_heads, int dim, int vdim);
 
+/* Mixture of experts behind an RMSNorm: x += alpha (sum over the `top` experts with the largest s_e = sigmoid(router_e . h) of
+ * s_e / (their sum + 1e-20) * scale * expert_e(h)  +  shared(h)),  expert(h) = down (silu(gate h) * (up h)).
+ * dtype BF16: streams (mi355_bf16_repack; gate and up a pair stream) in 16-bit products with f32 sums; F32: row-major f32.  The experts'
+ * weights lie one behind the other (f32: gate, up, next expert). */
+typedef struct mi355_experts_args {
+    int32_t dtype;
+    int32_t rows;
+    int32_t width;
+    int32_t experts, top;
+    int32_t ff;            /* of an expert */
+    int32_t ff_shared;     /* 0: no shared expert */
+    float scale;
+    const void* norm;      /* [width] of norm_dtype: the scale is norm_add + norm */
+    int32_t norm_dtype;
+    float norm_add;
+    float eps;
+    float alpha;
+    const void* router;    /* [experts, width] */
+    const void* up;
+    const void* down;
+    const void* shared_up;
+    const void* shared_down;
+    float* x;              /* [rows, ldx], ldx >= width padded to 16 (the padding stays zero) */
+    int64_t ldx;
+    void* scratch;         /* mi355_experts_scratch_bytes, 256-byte aligned */
+    uint64_t scratch_bytes;
+    int32_t path;          /* bf16; 0: by shape; 1: every row by itself; 2: sorted by expert */
+    int32_t reserved0;
+} mi355_experts_args;
+
+int mi355_experts(const mi355_experts_args* a, mi355_stream_t stream);
+/* scratch bytes of a step (dtype, rows, width, experts, top, ff, ff_shared are read) */
+size_t mi355_experts_scratch_bytes(const mi355_experts_args* a);
+
 /* A weight of a hybrid model: BF16 stream (mi355_bf16_repack, R = 1) of a bf16 model, row-major f32 of an f32 model */
 typedef struct mi355_proj {
     const void* w;
@@ -704,10 +753,13 @@ typedef struct mi355_proj {
 } mi355_proj;
 
 enum { MI355_MIX_ATTENTION = 0, MI355_MIX_DELTA = 1, MI355_MIX_GLA = 2 };
+/* feed-forwards: down relu(up h)^2; down (gelu_tanh(gate h) * (up h)), `up` the pair (BF16 pair stream, or f32 gate rows then up rows;
+ * up.N = the hidden size); mixture of experts */
+enum { MI355_MLP_NONE = 0, MI355_MLP_RELU2 = 1, MI355_MLP_GEGLU = 2, MI355_MLP_EXPERTS = 3 };
 /* one RUN of a layer (a looped layer appears once per pass: same weights, its own cache / state) */
 typedef struct mi355_hybrid_layer {
     int32_t mixer;         /* MI355_MIX_* */
-    int32_t mlp;           /* != 0: a squared-ReLU feed-forward follows */
+    int32_t mlp;           /* MI355_MLP_* */
     const void* norm1;     /* [width] of norm_dtype */
     const void* norm2;
     mi355_proj in;         /* every projection that reads the normalised row, stacked */
@@ -715,6 +767,9 @@ typedef struct mi355_hybrid_layer {
     mi355_proj up, down;
     mi355_window_attn_args attn;   /* as the mixer's kernels take them; proj / y / scratch are filled in per step */
     mi355_recurrent_args rec;
+    mi355_experts_args moe;        /* weights, sizes and scale */
+    int32_t kv_lender;     /* run whose cache this run's attention reads (role MI355_KV_BORROWS) */
+    int32_t kv_last;       /* of a lender: its last borrower's run */
 } mi355_hybrid_layer;
 
 typedef struct mi355_hybrid_model {
@@ -728,6 +783,8 @@ typedef struct mi355_hybrid_model {
     int32_t ld_logits;
     float eps;
     float residual_mult;
+    float norm_add;        /* the norms' scales are norm_add + their weights; 0, or 1 in bf16 models */
+    float logit_scale;
     const void* embed;     /* [vocab, width] of dtype */
     const void* final_norm;
     mi355_proj head;
@@ -738,7 +795,7 @@ typedef struct mi355_hybrid_model {
     uint16_t* xb;          /* [max_rows, ldx] bf16 models: normalised rows of a wide product */
     void* proj;            /* [max_rows, widest in.N] of dtype */
     void* att;             /* [max_rows, widest out.K padded to 16] of dtype */
-    void* hid;             /* [max_rows, widest up.N] of dtype */
+    void* hid;             /* [max_rows, widest up.N (f32 GEGLU: 3 up.N)] of dtype */
     float* tmp;            /* [max_rows, ldx] f32 models: a product in front of its residual */
     int64_t ld_att;
     void* gemm_ws;
@@ -747,6 +804,8 @@ typedef struct mi355_hybrid_model {
     uint64_t partials_bytes;
     float* rec_scratch;
     uint64_t rec_scratch_bytes;
+    void* moe_scratch;
+    uint64_t moe_scratch_bytes;
 } mi355_hybrid_model;
 
 /* embedding, every layer run, and the logits (f32 [n_want, ld_logits]) of the rows want[0 .. n_want) (device; NULL: all rows).

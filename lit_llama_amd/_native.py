@@ -18,8 +18,8 @@ CORE_LIB_PATH = _PKG / "libmi355core.so"  # the part a layered hybrid model need
 
 F32, BF16, F16 = 0, 1, 2
 W_Q4, W_BF16, W_I8 = 0, 1, 2
-EPI_STORE, EPI_ACCUM, EPI_SWIGLU = 0, 1, 2
-LF_RELU2 = 1
+EPI_STORE, EPI_ACCUM, EPI_SWIGLU, EPI_GEGLU = 0, 1, 2, 3
+LF_RELU2, LF_NORM_ONE = 1, 2
 
 _DTYPE_CODE = {torch.float32: F32, torch.bfloat16: BF16, torch.float16: F16}
 
@@ -154,7 +154,9 @@ class WindowAttnArgs(C.Structure):
         ("off_q", c_int32), ("off_k", c_int32), ("off_v", c_int32), ("off_g", c_int32),
         ("scale", c_float), ("window", c_int32), ("ring", c_int32), ("rot_dims", c_int32), ("inv_freq", c_void_p),
         ("kring", c_void_p), ("vring", c_void_p), ("y", c_void_p), ("ldy", c_int64),
-        ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("path", c_int32), ("reserved0", c_int32),
+        ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("path", c_int32),
+        ("keep", c_int32), ("kept", c_int32), ("gate_values", c_int32), ("unit_qk", c_int32), ("unit_eps", c_float), ("sink", c_void_p),
+        ("role", c_int32), ("reserved0", c_int32), ("kv_rows", c_void_p),
     ]
 
 
@@ -171,6 +173,16 @@ class RecurrentArgs(C.Structure):
     ]
 
 
+class ExpertsArgs(C.Structure):
+    _fields_ = [
+        ("dtype", c_int32), ("rows", c_int32), ("width", c_int32), ("experts", c_int32), ("top", c_int32),
+        ("ff", c_int32), ("ff_shared", c_int32), ("scale", c_float),
+        ("norm", c_void_p), ("norm_dtype", c_int32), ("norm_add", c_float), ("eps", c_float), ("alpha", c_float),
+        ("router", c_void_p), ("up", c_void_p), ("down", c_void_p), ("shared_up", c_void_p), ("shared_down", c_void_p),
+        ("x", c_void_p), ("ldx", c_int64), ("scratch", c_void_p), ("scratch_bytes", C.c_uint64), ("path", c_int32), ("reserved0", c_int32),
+    ]
+
+
 class Proj(C.Structure):
     _fields_ = [("w", c_void_p), ("N", c_int32), ("K", c_int32)]
 
@@ -179,7 +191,7 @@ class HybridLayer(C.Structure):
     _fields_ = [
         ("mixer", c_int32), ("mlp", c_int32), ("norm1", c_void_p), ("norm2", c_void_p),
         ("in", Proj), ("out", Proj), ("up", Proj), ("down", Proj),
-        ("attn", WindowAttnArgs), ("rec", RecurrentArgs),
+        ("attn", WindowAttnArgs), ("rec", RecurrentArgs), ("moe", ExpertsArgs), ("kv_lender", c_int32), ("kv_last", c_int32),
     ]
 
 
@@ -187,11 +199,12 @@ class HybridModel(C.Structure):
     _fields_ = [
         ("n_runs", c_int32), ("dtype", c_int32), ("norm_dtype", c_int32), ("width", c_int32),
         ("ldx", c_int32), ("vocab", c_int32), ("max_rows", c_int32), ("ld_logits", c_int32),
-        ("eps", c_float), ("residual_mult", c_float),
+        ("eps", c_float), ("residual_mult", c_float), ("norm_add", c_float), ("logit_scale", c_float),
         ("embed", c_void_p), ("final_norm", c_void_p), ("head", Proj), ("layers", C.POINTER(HybridLayer)),
         ("x", c_void_p), ("xw", c_void_p), ("xn", c_void_p), ("xb", c_void_p), ("proj", c_void_p), ("att", c_void_p), ("hid", c_void_p),
         ("tmp", c_void_p), ("ld_att", c_int64), ("gemm_ws", c_void_p), ("gemm_ws_bytes", C.c_uint64),
         ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("rec_scratch", c_void_p), ("rec_scratch_bytes", C.c_uint64),
+        ("moe_scratch", c_void_p), ("moe_scratch_bytes", C.c_uint64),
     ]
 
 
@@ -261,6 +274,9 @@ PROTOTYPES = {
     "mi355_linear_max_rows": (c_int, [c_int, c_int, c_int, c_int]),
     "mi355_debug_time_next_launch": (c_int, [c_void_p, c_void_p]),
     "mi355_window_attention": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
+    "mi355_window_cache_write": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
+    "mi355_experts": (c_int, [C.POINTER(ExpertsArgs), c_void_p]),
+    "mi355_experts_scratch_bytes": (c_size_t, [C.POINTER(ExpertsArgs)]),
     "mi355_recurrent": (c_int, [C.POINTER(RecurrentArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_recurrent_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
     "mi355_hybrid_forward": (c_int, [C.POINTER(HybridModel), C.POINTER(SeqBatch), c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p]),
@@ -272,7 +288,7 @@ PROTOTYPES = {
 }
 
 ABI_STRUCTS = [LinearArgs, AttnArgs, Int8Args, Weight, Layer, Model, FusedStepArgs, TpComm,
-               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel]
+               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel, ExpertsArgs]
 
 _lib: Optional[C.CDLL] = None
 

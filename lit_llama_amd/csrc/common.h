@@ -178,6 +178,19 @@ __device__ __forceinline__ float relu2_f32(float v) {
 // silu(a) * b in f32 (F.silu: a * sigmoid(a))
 __device__ __forceinline__ float swiglu_f32(float a, float b) { return (a / (1.0f + expf(-a))) * b; }
 
+// the tanh form of GELU: 0.5 z (1 + tanh(u)) = z sigmoid(2 u), u = sqrt(2 / pi) (z + 0.044715 z^3)
+__device__ __forceinline__ float gelu_tanh_f32(float z) {
+    const float u2 = 1.59576912160573071176f * (z + 0.044715f * z * z * z);
+    return z / (1.0f + expf(-u2));
+}
+
+// epilogues over a pair stream, and what they store
+constexpr bool is_pair_epi(int epi) { return epi == MI355_EPI_SWIGLU || epi == MI355_EPI_GEGLU; }
+template <int EPI>
+__device__ __forceinline__ float pair_act_f32(float a, float b) {
+    return EPI == MI355_EPI_GEGLU ? gelu_tanh_f32(a) * b : swiglu_f32(a, b);
+}
+
 // Block-wide index of the first maximum of logits[0..V) (lowest index wins ties, as torch.topk(.., 1) /
 // argmax do on the CPU oracle); every thread gets the result.  An all-NaN row gives 0.
 __device__ inline int block_argmax_first(const float* logits, int V) {

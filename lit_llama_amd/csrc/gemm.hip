@@ -34,9 +34,12 @@
 // profiles/r06_prefill_epilogue_cost.txt): v_cvt_pk_bf16_f32 rounds to nearest even exactly as f32_to_bf16 does (finite inputs),
 // v_exp_f32 / v_rcp_f32 are within 1 ulp of f32 — 2^-15 of the bf16 step the result is rounded to.
 __device__ __forceinline__ bf16_t bf16_hw(float f) { return __builtin_bit_cast(bf16_t, (__bf16)f); }
-__device__ __forceinline__ float swiglu_fast(float a, float b) {
+template <int EPI>
+__device__ __forceinline__ float pair_act_fast(float a, float b) {
     // silu(a) * b = a / (1 + 2^(-a log2 e)) * b; a -> -inf: 2^(+inf) = inf, rcp = 0; a -> +inf: rcp(1) = 1
-    return (a * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(a * -1.44269504088896340736f))) * b;
+    // gelu(a) in the tanh form = a / (1 + 2^(-2 u log2 e)), u = sqrt(2 / pi) (a + 0.044715 a^3)
+    const float t = EPI == MI355_EPI_GEGLU ? a * (1.59576912160573071176f + 0.07135481282792783f * (a * a)) : a;
+    return (a * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(t * -1.44269504088896340736f))) * b;
 }
 
 namespace {
@@ -170,7 +173,7 @@ __device__ __forceinline__ float ldsz(const void* p, int i, int dtype) {
 // K-slice s (ksplit = 1: the whole row)
 __global__ __launch_bounds__(256) void stage_rows_kernel(const void* x, int x_dtype, int64_t ldx, const void* norm_scale,
                                                          int norm_dtype, float eps, int K, int Kp, bf16_t* xb, int64_t ldxb,
-                                                         float* rinv, float* sx, int ksplit, float alpha) {
+                                                         float* rinv, float* sx, int ksplit, float alpha, float norm_add) {
     __shared__ float red[32];
     const int m = blockIdx.x;
     const int units = Kp >> 7;
@@ -184,7 +187,7 @@ __global__ __launch_bounds__(256) void stage_rows_kernel(const void* x, int x_dt
                 float v = ld_as_f32(x, (int64_t)m * ldx + k, x_dtype);
                 if (norm_scale != nullptr) {
                     ss += v * v;
-                    v *= ld_as_f32(norm_scale, k, norm_dtype);
+                    v *= norm_add + ld_as_f32(norm_scale, k, norm_dtype);
                 }
                 o = bf16_hw(v);
                 sum += bf16_to_f32(o);
@@ -259,7 +262,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, i
     for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < (int64_t)M * n4; i += (int64_t)gridDim.x * blockDim.x) {
         const int m = (int)(i / n4), n = (int)(i - (int64_t)m * n4) * 4;
         f32x4 o = {0.f, 0.f, 0.f, 0.f};
-        if constexpr (EPI == MI355_EPI_SWIGLU) {
+        if constexpr (is_pair_epi(EPI)) {
             f32x4 b = {0.f, 0.f, 0.f, 0.f};
             for (int s = 0; s < ksplit; ++s) {
                 const float* row = part + ((int64_t)s * M + m) * (2 * (int64_t)N);
@@ -268,8 +271,8 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, i
             }
             bf16_t* dst = (bf16_t*)y + (int64_t)m * ldy + n;
             u32x2 pk;
-            pk[0] = (uint32_t)bf16_hw(swiglu_fast(o[0], b[0])) | ((uint32_t)bf16_hw(swiglu_fast(o[1], b[1])) << 16);
-            pk[1] = (uint32_t)bf16_hw(swiglu_fast(o[2], b[2])) | ((uint32_t)bf16_hw(swiglu_fast(o[3], b[3])) << 16);
+            pk[0] = (uint32_t)bf16_hw(pair_act_fast<EPI>(o[0], b[0])) | ((uint32_t)bf16_hw(pair_act_fast<EPI>(o[1], b[1])) << 16);
+            pk[1] = (uint32_t)bf16_hw(pair_act_fast<EPI>(o[2], b[2])) | ((uint32_t)bf16_hw(pair_act_fast<EPI>(o[3], b[3])) << 16);
             *(u32x2*)dst = pk;
         } else if (y_dtype == MI355_F32) {
             float* dst = (float*)y + (int64_t)m * ldy + n;
@@ -305,7 +308,7 @@ __global__ __launch_bounds__(256) void splitk_fused_reduce_kernel(const GemmPara
     for (int64_t grp = ((int64_t)blockIdx.x * 256 + threadIdx.x) >> 5; grp < groups; grp += (int64_t)gridDim.x * 8) {
         const int m = (int)(grp / units_n), un = (int)(grp - (int64_t)m * units_n);
         const int n = un * 128 + l32 * 4;
-        if constexpr (EPI == MI355_EPI_SWIGLU) {
+        if constexpr (is_pair_epi(EPI)) {
             f32x4 a = {0.f, 0.f, 0.f, 0.f}, b = {0.f, 0.f, 0.f, 0.f};
             for (int sl = 0; sl < p.ksplit; ++sl) {
                 const float* row = p.part + ((int64_t)sl * p.M + m) * (2 * (int64_t)p.N);
@@ -314,7 +317,7 @@ __global__ __launch_bounds__(256) void splitk_fused_reduce_kernel(const GemmPara
             }
             bf16_t ob[4];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(swiglu_fast(a[r], b[r]));
+            for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(pair_act_fast<EPI>(a[r], b[r]));
             u32x2 pk;
             pk[0] = (uint32_t)ob[0] | ((uint32_t)ob[1] << 16);
             pk[1] = (uint32_t)ob[2] | ((uint32_t)ob[3] << 16);
@@ -850,7 +853,7 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
             }
             continue;
         }
-        if constexpr (EPI == MI355_EPI_SWIGLU) {
+        if constexpr (is_pair_epi(EPI)) {
 #pragma unroll
             for (int t = 0; t < kTPW; t += 2) {
                 const int n = tile[t] * 16 + 4 * g;
@@ -858,7 +861,7 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
                     bf16_t* dst = (bf16_t*)p.y + (int64_t)m * p.ldy + n;
                     bf16_t ob[4];
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(swiglu_fast(v[t][r], v[t + 1][r]));
+                    for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(pair_act_fast<EPI>(v[t][r], v[t + 1][r]));
                     u32x2 o;
                     o[0] = (uint32_t)ob[0] | ((uint32_t)ob[1] << 16);
                     o[1] = (uint32_t)ob[2] | ((uint32_t)ob[3] << 16);
@@ -1118,6 +1121,9 @@ int launch_gemm_grouped_epi(const GemmParams& p, int epi, hipStream_t s) {
 template <int FMT, bool FUSE>
 int launch_gemm_epi(const GemmParams& p, int epi, hipStream_t s) {
     if (epi == MI355_EPI_SWIGLU) return launch_gemm<MI355_EPI_SWIGLU, true, FMT, FUSE>(p, s);
+    if constexpr (FMT == MI355_W_BF16 && !FUSE) {
+        if (epi == MI355_EPI_GEGLU) return launch_gemm<MI355_EPI_GEGLU, true, FMT, FUSE>(p, s);
+    }
     if (epi == MI355_EPI_ACCUM) return launch_gemm<MI355_EPI_ACCUM, false, FMT, FUSE>(p, s);
     return launch_gemm<MI355_EPI_STORE, false, FMT, FUSE>(p, s);
 }
@@ -1170,8 +1176,11 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
     }
     MI355_CHECK_ARG(a->M >= 1 && a->N > 0 && a->K > 0, MI355_E_SHAPE, "linear_gemm: bad shape M=%d N=%d K=%d", a->M, a->N, a->K);
     MI355_CHECK_ARG(a->attn_partials == nullptr && a->bias == nullptr, MI355_E_ARG, "linear_gemm: no bias / attention prologue");
-    const bool swiglu = a->epi == MI355_EPI_SWIGLU;
-    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_SWIGLU, MI355_E_ARG, "linear_gemm: bad epi");
+    const bool swiglu = is_pair_epi(a->epi);
+    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_GEGLU, MI355_E_ARG, "linear_gemm: bad epi");
+    MI355_CHECK_ARG(a->epi != MI355_EPI_GEGLU || (!q4 && f == nullptr), MI355_E_ARG, "linear_gemm: GEGLU takes the BF16 pair stream");
+    MI355_CHECK_ARG(!(a->flags & MI355_LF_NORM_ONE) || !q4 || a->group_cols <= 0 || a->group_cols >= a->K, MI355_E_ARG,
+                    "linear_gemm: no 1 + scale norm in front of grouped scales");
     MI355_CHECK_ARG(swiglu ? (a->R == 2 && (!q4 || (a->scales2 && a->zeros2)) && a->y_dtype == MI355_BF16) : a->R == 1, MI355_E_ARG,
                     "linear_gemm: STORE / ACCUM take the R = 1 stream, SWIGLU the interleaved R = 2 stream with bf16 output");
     MI355_CHECK_ARG(a->N % 4 == 0 && a->ldy % 4 == 0, MI355_E_SHAPE, "linear_gemm: N and ldy must be multiples of 4");
@@ -1264,7 +1273,8 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
         p.tab_ld = tab_ld;
     } else if (!f_in && !direct) {
         hipLaunchKernelGGL(stage_rows_kernel, dim3(a->M), dim3(256), 0, s, a->x, a->x_dtype, a->ldx, a->norm_scale, a->norm_dtype,
-                           a->eps, a->K, kp, xb, (int64_t)kp, rinv, sx, ksplit, a->alpha == 0.f ? 1.f : a->alpha);
+                           a->eps, a->K, kp, xb, (int64_t)kp, rinv, sx, ksplit, a->alpha == 0.f ? 1.f : a->alpha,
+                           (a->flags & MI355_LF_NORM_ONE) ? 1.f : 0.f);
         MI355_LAUNCH_CHECK();
     }
     p.w = (const uint8_t*)a->w;

@@ -66,6 +66,7 @@ struct GemvParams {
     // grouped scales (GRP kernels): scales / zeros are [N, n_groups] bf16, one pair per 32 << gq_shift input columns
     float alpha;    // factor of the product
     int relu2;      // STORE: max(y, 0)^2
+    float norm_add; // the norm's scale is norm_add + norm_scale
     int n_groups, gq_shift;
     float inv_ng;  // 1 / n_groups (element index -> row without an integer division)
 };
@@ -136,7 +137,7 @@ struct Stager<0> {  // element loop, any dtype
             float v = ld2(p.x, base + k, p.x_dtype);
             if (norm) {
                 ss += v * v;
-                v = ld2(p.norm_scale, k, p.norm_dtype) * v;
+                v = (p.norm_add + ld2(p.norm_scale, k, p.norm_dtype)) * v;
             }
             row[k] = f32_to_bf16(v);
         }
@@ -175,8 +176,8 @@ struct StagerF32Norm {  // f32 row, bf16 norm scale, <= NC x 8 elements per thre
                     const float x0 = i < 2 ? xa[c][2 * i] : xb[c][2 * i - 4];
                     const float x1 = i < 2 ? xa[c][2 * i + 1] : xb[c][2 * i - 3];
                     ss += x0 * x0 + x1 * x1;
-                    const bf16_t a = f32_to_bf16(__uint_as_float(ns[c][i] << 16) * x0);
-                    const bf16_t b = f32_to_bf16(__uint_as_float(ns[c][i] & 0xffff0000u) * x1);
+                    const bf16_t a = f32_to_bf16((p.norm_add + __uint_as_float(ns[c][i] << 16)) * x0);
+                    const bf16_t b = f32_to_bf16((p.norm_add + __uint_as_float(ns[c][i] & 0xffff0000u)) * x1);
                     o[i] = (uint32_t)a | ((uint32_t)b << 16);
                 }
                 *(u32x4*)(row + v * 16) = o;
@@ -314,7 +315,7 @@ __device__ __forceinline__ float cvt2(uint32_t raw, int dtype) {
 template <int FMT, int R, int EPI, int GRP = 0>
 __device__ __forceinline__ void load_epi(const GemvParams& p, const EpiRsrc& er, int tile, int e_row, int e_col,
                                          bool e_owner, EpiOps<R>& o) {
-    constexpr bool sw = EPI == MI355_EPI_SWIGLU;
+    constexpr bool sw = is_pair_epi(EPI);
     const bool live = e_owner && tile < p.n_tiles;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
@@ -383,10 +384,10 @@ __device__ __forceinline__ void tile_epilogue(const GemvParams& p, const char* p
             s = cvt2(o.s[r] >> o.sh_sz[r], p.sz_dtype) * (s - (128.f + cvt2(o.z[r] >> o.sh_sz[r], p.sz_dtype)) * sx);
         v[r] = s * rinv;
     }
-    if constexpr (EPI == MI355_EPI_SWIGLU) {
+    if constexpr (is_pair_epi(EPI)) {
         if constexpr (R == 2) {
             const int n = tile * 16 + e_row;
-            if (n < p.N) st2(p.y, (int64_t)e_col * p.ldy + n, p.y_dtype, swiglu_f32(v[0], v[1]));
+            if (n < p.N) st2(p.y, (int64_t)e_col * p.ldy + n, p.y_dtype, pair_act_f32<EPI>(v[0], v[1]));
         }
     } else {
 #pragma unroll
@@ -513,7 +514,7 @@ __global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const 
     uint32_t gs[GRP ? R : 1][kGrpLoads], gz[GRP ? R : 1][kGrpLoads];
     auto grp_load = [&](int t) {
         if constexpr (GRP) {
-            constexpr bool sw = EPI == MI355_EPI_SWIGLU;
+            constexpr bool sw = is_pair_epi(EPI);
 #pragma unroll
             for (int r = 0; r < R; ++r) {
 #pragma unroll
@@ -532,7 +533,7 @@ __global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const 
     };
     auto grp_park = [&](int t, int b) {  // raw bits -> LDS block b; rows past N carry (0, 0): they multiply zeros
         if constexpr (GRP) {
-            constexpr bool sw = EPI == MI355_EPI_SWIGLU;
+            constexpr bool sw = is_pair_epi(EPI);
 #pragma unroll
             for (int r = 0; r < R; ++r) {
 #pragma unroll
@@ -1007,10 +1008,10 @@ int launch_gemv_epi(const GemvParams& p, int grid, int waves, size_t lds, hipStr
             if constexpr (EPI != MI355_EPI_ACCUM) return launch_gemv_v<FMT, R, P, EPI, 4, GRP>(p, grid, waves, lds, stream);
             break;
         case 2:
-            if constexpr (EPI != MI355_EPI_SWIGLU) return launch_gemv_v<FMT, R, P, EPI, 2, GRP>(p, grid, waves, lds, stream);
+            if constexpr (!is_pair_epi(EPI)) return launch_gemv_v<FMT, R, P, EPI, 2, GRP>(p, grid, waves, lds, stream);
             break;
         case 3:
-            if constexpr (EPI != MI355_EPI_SWIGLU) return launch_gemv_v<FMT, R, P, EPI, 3, GRP>(p, grid, waves, lds, stream);
+            if constexpr (!is_pair_epi(EPI)) return launch_gemv_v<FMT, R, P, EPI, 3, GRP>(p, grid, waves, lds, stream);
             break;
         default: break;
     }
@@ -1026,6 +1027,10 @@ int launch_gemv(const GemvParams& p, int grid, int waves, size_t lds, hipStream_
     switch (p.epi) {
         case MI355_EPI_STORE: return launch_gemv_epi<FMT, R, P, MI355_EPI_STORE, GRP>(p, grid, waves, lds, stream);
         case MI355_EPI_ACCUM: return launch_gemv_epi<FMT, R, P, MI355_EPI_ACCUM, GRP>(p, grid, waves, lds, stream);
+        case MI355_EPI_GEGLU:
+            if constexpr (R == 2 && FMT == MI355_W_BF16) return launch_gemv_epi<FMT, R, P, MI355_EPI_GEGLU, GRP>(p, grid, waves, lds, stream);
+            mi355_set_error("the GEGLU epilogue takes the BF16 pair stream");
+            return MI355_E_ARG;
         default:
             if constexpr (R == 2) return launch_gemv_epi<FMT, R, P, MI355_EPI_SWIGLU, GRP>(p, grid, waves, lds, stream);
             mi355_set_error("SwiGLU epilogue needs R == 2");
@@ -1151,13 +1156,13 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
     MI355_CHECK_ARG(a->w && (a->x || a->attn_partials) && a->y, MI355_E_ARG, "linear_fast: null w/x/y");
     if (a->attn_partials != nullptr) {
         MI355_CHECK_ARG(a->M == 1 && a->attn_splits >= 1 && a->attn_heads >= 1 && a->attn_hs % 8 == 0 && a->norm_scale == nullptr &&
-                            a->K == a->attn_heads * a->attn_hs && a->epi != MI355_EPI_SWIGLU,
+                            a->K == a->attn_heads * a->attn_hs && !is_pair_epi(a->epi),
                         MI355_E_ARG, "linear_fast: bad split-attention activation spec");
     }
     MI355_CHECK_ARG(a->M >= 1 && a->M <= kMaxM, MI355_E_SHAPE, "linear_fast: M=%d outside 1..%d", a->M, kMaxM);
     MI355_CHECK_ARG(a->K > 0 && a->N > 0, MI355_E_SHAPE, "linear_fast: N=%d K=%d must be positive", a->N, a->K);
-    const bool swiglu = a->epi == MI355_EPI_SWIGLU;
-    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_SWIGLU, MI355_E_ARG, "linear_fast: bad epi");
+    const bool swiglu = is_pair_epi(a->epi);
+    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_GEGLU, MI355_E_ARG, "linear_fast: bad epi");
     MI355_CHECK_ARG(!swiglu || a->R == 2, MI355_E_ARG, "linear_fast: SwiGLU epilogue needs the interleaved R=2 stream");
     const int rows_per_tile = swiglu ? 16 : 16 * a->R;
     if (a->fmt == MI355_W_Q4) {
@@ -1198,6 +1203,7 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
     p.eps = a->eps;
     p.alpha = a->alpha == 0.f ? 1.f : a->alpha;
     p.relu2 = (a->flags & MI355_LF_RELU2) ? 1 : 0;
+    p.norm_add = (a->flags & MI355_LF_NORM_ONE) ? 1.f : 0.f;
     MI355_CHECK_ARG(!p.relu2 || a->epi == MI355_EPI_STORE, MI355_E_ARG, "linear_fast: RELU2 belongs to the STORE epilogue");
     int waves = a->waves > 0 ? a->waves : 8;
     if (waves > 16) waves = 16;

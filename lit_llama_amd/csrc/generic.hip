@@ -36,6 +36,7 @@ extern "C" int mi355_sizeof(int which) {
         case 11: return (int)sizeof(mi355_proj);
         case 12: return (int)sizeof(mi355_hybrid_layer);
         case 13: return (int)sizeof(mi355_hybrid_model);
+        case 14: return (int)sizeof(mi355_experts_args);
         default: return -1;
     }
 }

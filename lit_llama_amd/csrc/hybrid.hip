@@ -1,6 +1,6 @@
 // The forward pass of a layered hybrid model (mi355_hybrid_forward): a host-side walk over the layer runs that enqueues this library's
-// linears (gemv.hip for a few rows, gemm.hip above, the exact f32 kernel for f32 models) and mixers (window_attention.hip,
-// recurrent.hip).  RMSNorm rides in the consuming linear and the residual sum in the producing one; the residual stream is f32.
+// linears (gemv.hip for a few rows, gemm.hip above, the exact f32 kernel for f32 models), mixers (window_attention.hip, recurrent.hip) and
+// experts (experts.hip).  RMSNorm rides in the consuming linear and the residual sum in the producing one; the residual stream is f32.
 #include "common.h"
 
 namespace {
@@ -37,7 +37,7 @@ __global__ __launch_bounds__(256) void gather_rows_kernel(const float* x, const 
 // xb[m] = bf16(norm(x[m]) * scale), one row per workgroup: the operand of a wide product, multiplied where it lies.  K % 128 == 0, so rows
 // are whole 16-B vectors
 __global__ __launch_bounds__(512) void norm_rows_kernel(const float* x, int64_t ldx, const void* scale, int scale_dtype, float eps, int K,
-                                                        bf16_t* xb) {
+                                                        float norm_add, bf16_t* xb) {
     __shared__ float red[32];
     const f32x4* row = (const f32x4*)(x + (int64_t)blockIdx.x * ldx);
     constexpr int kHeld = 4;  // vectors a thread keeps between the two passes
@@ -65,6 +65,7 @@ __global__ __launch_bounds__(512) void norm_rows_kernel(const float* x, int64_t 
         } else {
             for (int e = 0; e < 4; ++e) s[e] = ld_as_f32(scale, 4 * j + e, scale_dtype);
         }
+        for (int e = 0; e < 4; ++e) s[e] += norm_add;
         const bf2 a = {(__bf16)(w[0] * rinv * s[0]), (__bf16)(w[1] * rinv * s[1])}, b = {(__bf16)(w[2] * rinv * s[2]), (__bf16)(w[3] * rinv * s[3])};
         out[j] = u32x2{__builtin_bit_cast(uint32_t, a), __builtin_bit_cast(uint32_t, b)};
     };
@@ -78,6 +79,18 @@ __global__ __launch_bounds__(512) void norm_rows_kernel(const float* x, int64_t 
 
 __global__ __launch_bounds__(256) void relu2_kernel(float* h, int64_t n) {
     for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) h[i] = relu2_f32(h[i]);
+}
+
+// rows [gate | up] of 2 n values -> gelu_tanh(gate) * up
+__global__ __launch_bounds__(256) void geglu_kernel(const float* gu, float* h, int n, int64_t total) {
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
+        const int64_t m = i / n, k = i - m * n;
+        h[i] = gelu_tanh_f32(gu[m * 2 * n + k]) * gu[m * 2 * n + n + k];
+    }
+}
+
+__global__ __launch_bounds__(256) void scale_kernel(float* y, float f, int64_t n) {
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) y[i] *= f;
 }
 
 // x += alpha * t over rows of the same pitch
@@ -109,9 +122,9 @@ int ew_blocks(int64_t n) {
     return (int)(b > 4096 ? 4096 : b);
 }
 
-enum { kStore = 0, kRelu2 = 1, kResidual = 2 };
+enum { kStore = 0, kRelu2 = 1, kResidual = 2, kGeglu = 3, kLogits = 4 };
 
-// y[M, N] (+)= alpha * W norm(x).  x f32 with `norm`, or dtype without
+// y[M, N] (+)= alpha * W norm(x), or what a feed-forward makes of it; alpha: residual_mult (kResidual), logit_scale (kLogits), 1.  x f32 with `norm`, or dtype without
 int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int64_t ldx, const void* norm, int what, void* y, int64_t ldy,
            int y_dtype, int M, hipStream_t s) {
     if (m->dtype == MI355_F32) {
@@ -122,10 +135,17 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
             in = m->xn;
             ld_in = m->ldx;
         }
-        void* dst = what == kResidual ? (void*)m->tmp : y;
-        const int64_t ld_dst = what == kResidual ? m->ldx : ldy;
-        if (int rc = mi355_linear_dense(in, ld_in, w.w, nullptr, dst, ld_dst, M, w.N, w.K, MI355_F32, s)) return rc;
-        if (what == kRelu2) {  // (ldy = w.N: rows without gaps)
+        // (kGeglu: the products lie behind the M hidden rows)
+        void* dst = what == kResidual ? (void*)m->tmp : what == kGeglu ? (void*)((float*)y + (int64_t)M * ldy) : y;
+        const int64_t ld_dst = what == kResidual ? m->ldx : what == kGeglu ? 2 * ldy : ldy;
+        if (int rc = mi355_linear_dense(in, ld_in, w.w, nullptr, dst, ld_dst, M, what == kGeglu ? 2 * w.N : w.N, w.K, MI355_F32, s)) return rc;
+        if (what == kGeglu) {  // (ldy = w.N)
+            hipLaunchKernelGGL(geglu_kernel, dim3(ew_blocks((int64_t)M * ldy)), dim3(256), 0, s, (const float*)dst, (float*)y, w.N, (int64_t)M * ldy);
+            MI355_LAUNCH_CHECK();
+        } else if (what == kLogits && m->logit_scale != 1.f) {
+            hipLaunchKernelGGL(scale_kernel, dim3(ew_blocks((int64_t)M * ldy)), dim3(256), 0, s, (float*)y, m->logit_scale, (int64_t)M * ldy);
+            MI355_LAUNCH_CHECK();
+        } else if (what == kRelu2) {  // (ldy = w.N: rows without gaps)
             hipLaunchKernelGGL(relu2_kernel, dim3(ew_blocks((int64_t)M * ldy)), dim3(256), 0, s, (float*)y, (int64_t)M * ldy);
             MI355_LAUNCH_CHECK();
         } else if (what == kResidual) {  // (N = ldx = ldy)
@@ -138,7 +158,7 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
     mi355_linear_args a;
     memset(&a, 0, sizeof(a));
     a.fmt = MI355_W_BF16;
-    a.R = 1;
+    a.R = what == kGeglu ? 2 : 1;
     a.w = w.w;
     a.N = w.N;
     a.K = w.K;
@@ -147,12 +167,12 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
     a.norm_scale = norm;
     a.norm_dtype = m->norm_dtype;
     a.eps = m->eps;
-    a.epi = what == kResidual ? MI355_EPI_ACCUM : MI355_EPI_STORE;
-    a.flags = what == kRelu2 ? MI355_LF_RELU2 : 0;
-    a.alpha = what == kResidual ? m->residual_mult : 1.f;
+    a.epi = what == kResidual ? MI355_EPI_ACCUM : what == kGeglu ? MI355_EPI_GEGLU : MI355_EPI_STORE;
+    a.flags = (what == kRelu2 ? MI355_LF_RELU2 : 0) | (m->norm_add != 0.f ? MI355_LF_NORM_ONE : 0);
+    a.alpha = what == kResidual ? m->residual_mult : what == kLogits ? m->logit_scale : 1.f;
     a.y_dtype = y_dtype;
     a.ldy = ldy;
-    const int most = mi355_linear_max_rows(MI355_W_BF16, w.K, 1, 0);
+    const int most = mi355_linear_max_rows(MI355_W_BF16, w.K, a.R, 0);
     // The weight-streaming kernel up to 8 rows; from there on, and for operands that leave its LDS room for a few rows only, the tiled
     // product (split over K, the operand read in place) moves the weights faster: 4096 x 16512 at 4 / 8 / 16 rows 57 / 118 / 251 us against
     // 28 / 28 / 30, 16512 x 4096 with the norm at 8 / 16 rows 31 / 41 against 35 / 36
@@ -162,7 +182,7 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
         a.y = y;
         a.M = M;
         if (norm != nullptr && w.K % 128 == 0 && ldx % 4 == 0) {
-            hipLaunchKernelGGL(norm_rows_kernel, dim3(M), dim3(512), 0, s, (const float*)x, ldx, norm, m->norm_dtype, m->eps, w.K, m->xb);
+            hipLaunchKernelGGL(norm_rows_kernel, dim3(M), dim3(512), 0, s, (const float*)x, ldx, norm, m->norm_dtype, m->eps, w.K, m->norm_add, m->xb);
             MI355_LAUNCH_CHECK();
             a.x = m->xb;
             a.x_dtype = MI355_BF16;
@@ -187,7 +207,8 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
     MI355_CHECK_ARG(M > 0 && M <= m->max_rows && n_want >= 0 && (want != nullptr ? n_want <= m->max_rows : n_want == 0 || n_want == M),
                     MI355_E_SHAPE, "hybrid_forward: %d rows (of %d), %d wanted", M, m->max_rows, n_want);
     MI355_CHECK_ARG(b->max_count > 1 || b->rows == b->seqs, MI355_E_SHAPE, "hybrid_forward: a decode step has one row per sequence");
-    MI355_CHECK_ARG(m->residual_mult != 0.f, MI355_E_ARG, "hybrid_forward: residual_mult is 0");
+    MI355_CHECK_ARG(m->residual_mult != 0.f && m->logit_scale != 0.f, MI355_E_ARG, "hybrid_forward: residual_mult or logit_scale is 0");
+    MI355_CHECK_ARG(m->norm_add == 0.f || (m->norm_add == 1.f && m->dtype == MI355_BF16), MI355_E_ARG, "hybrid_forward: norm_add is 0, or 1 in bf16 models");
     MI355_CHECK_ARG(n_want == 0 || run_end < m->n_runs || (logits && m->final_norm), MI355_E_ARG, "hybrid_forward: nowhere to write logits");
     hipStream_t s = (hipStream_t)stream;
     hipLaunchKernelGGL(embed_rows_kernel, dim3(M), dim3(256), 0, s, tokens, m->embed, m->dtype, m->x, m->width, m->ldx, m->vocab);
@@ -207,6 +228,16 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
             a.partials = m->partials;
             a.partials_bytes = m->partials_bytes;
             if (int rc = mi355_window_attention(&a, b, stream)) return rc;
+            // a lender's cache rows: behind the last attention of this step that reads the rows they replace
+            const int lender = a.role == MI355_KV_BORROWS ? l.kv_lender : r;
+            if (a.role != MI355_KV_OWN && m->layers[lender].kv_last == r) {
+                a = m->layers[lender].attn;
+                a.proj = m->proj;
+                a.ld = ldp;
+                a.dtype = m->dtype;
+                a.y = m->att;
+                if (int rc = mi355_window_cache_write(&a, b, stream)) return rc;
+            }
         } else {
             mi355_recurrent_args a = l.rec;
             a.proj = m->proj;
@@ -219,8 +250,23 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
             if (int rc = mi355_recurrent(&a, b, stream)) return rc;
         }
         if (int rc = linear(m, l.out, m->att, m->ld_att, nullptr, kResidual, m->x, m->ldx, MI355_F32, M, s)) return rc;
-        if (l.mlp) {
-            if (int rc = linear(m, l.up, m->x, m->ldx, l.norm2, kRelu2, m->hid, l.up.N, m->dtype, M, s)) return rc;
+        if (l.mlp == MI355_MLP_EXPERTS) {
+            mi355_experts_args e = l.moe;
+            e.dtype = m->dtype;
+            e.rows = M;
+            e.norm = l.norm2;
+            e.norm_dtype = m->norm_dtype;
+            e.norm_add = m->norm_add;
+            e.eps = m->eps;
+            e.alpha = m->residual_mult;
+            e.x = m->x;
+            e.ldx = m->ldx;
+            e.scratch = m->moe_scratch;
+            e.scratch_bytes = m->moe_scratch_bytes;
+            if (int rc = mi355_experts(&e, stream)) return rc;
+        } else if (l.mlp != MI355_MLP_NONE) {
+            const int what = l.mlp == MI355_MLP_GEGLU ? kGeglu : kRelu2;
+            if (int rc = linear(m, l.up, m->x, m->ldx, l.norm2, what, m->hid, l.up.N, m->dtype, M, s)) return rc;
             if (int rc = linear(m, l.down, m->hid, l.up.N, nullptr, kResidual, m->x, m->ldx, MI355_F32, M, s)) return rc;
         }
     }
@@ -231,7 +277,7 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
         MI355_LAUNCH_CHECK();
         xh = m->xw;
     }
-    return linear(m, m->head, xh, m->ldx, m->final_norm, kStore, logits, m->ld_logits, MI355_F32, n_want, s);
+    return linear(m, m->head, xh, m->ldx, m->final_norm, kLogits, logits, m->ld_logits, MI355_F32, n_want, s);
 }
 
 extern "C" int mi355_hybrid_reset_slots(const mi355_hybrid_model* m, const int32_t* slots, int n, mi355_stream_t stream) {

@@ -1,12 +1,14 @@
 // Causal attention over a sliding window: grouped key / value heads, different key and value sizes, interleaved rotation of the first
-// rot_dims dimensions, one sigmoid gate per head.  A slot's cache is a ring of rows per key head.
+// rot_dims dimensions, queries and keys over their root mean square, first rows that stay visible, a sink in the softmax sum, sigmoid gates
+// per head or per value.  A slot's cache is, per key head, `kept` rows for the first positions and a ring for the others.  A layer lends
+// its keys and values to later ones, which read its cache (and, in a prompt step, its prepared rows).
 //
 //   window_rows_kernel    one workgroup per (row, key head, split of the keys): decode steps of any size (q and the row's own k are
-//                         rotated here, the ring row is written here: one launch per layer), f32 models, odd head sizes
+//                         normalised and rotated here, the cache row is written here: one launch per layer), f32 models, odd head sizes
 //   window_tiles_kernel   128 queries of one head per workgroup on the matrix cores (bf16 prompt steps)
-//   rotate_keys_kernel    prompt steps: k rows rotated in place, in front of either kernel
-//   ring_write_kernel     prompt steps: the last rows of every portion enter the ring, behind either kernel (which reads the rows of
-//                         earlier portions from it)
+//   prepare_keys_kernel   prompt steps: k rows normalised and rotated in front of either kernel, in place or (a lender's) to kv_rows
+//   ring_write_kernel     prompt steps: the first and the last rows of every portion enter the cache, behind either kernel (which reads
+//                         the rows of earlier portions from it) and, of a lender, behind its last borrower
 //
 // Scores, softmax and weighted values are f32 (the tiles multiply bf16 operands into f32 accumulators).
 #include "common.h"
@@ -20,6 +22,10 @@ constexpr int kRowThreads = 256;
 constexpr int kKeys = 256;        // keys per pass of the row kernel
 constexpr int kMaxSplit = 32;     // (<= 64, a lane each) workgroups over the keys of one (row, key head) in a decode step
 constexpr double kInvTwoPi = 0.15915494309189533577;
+
+// row of position p in a slot's cache
+__device__ __forceinline__ int cache_row(const mi355_window_attn_args& a, int p) { return p < a.kept ? p : a.kept + (p - a.kept) % a.ring; }
+__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 // turn of (u, v) by pos * inv_freq: the angle is reduced in f64, so far positions keep f32 accuracy
 __device__ __forceinline__ void pair_cos_sin(int pos, double inv_freq, float& c, float& s) {
@@ -63,7 +69,10 @@ __device__ __forceinline__ void load_vec(const T* p, float (&o)[N]) {
 struct WinParams {
     mi355_window_attn_args a;
     mi355_seq_batch b;
-    int n_split, head_tiles, fresh;  // fresh: a decode step (the row's own k is unrotated and not in the ring yet)
+    int n_split, head_tiles, fresh;  // fresh: a decode step
+    int own;                         // a decode step of a layer with keys of its own: the row's k is raw and not in the cache yet
+    const void *krows, *vrows;       // prepared keys and values of the step's rows, first key head
+    int64_t ld_rows;
 };
 
 // ------------------------------------------------------------------------------------ row kernel
@@ -85,6 +94,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     float* stat = sc + HT * kKeys;                // [3][HT]: maximum, sum, correction
     float* red = stat + 4 * HT;                   // [key lanes][HT][columns]: at most kRowThreads HT VE
     __shared__ int s_seq;
+    __shared__ float s_rms[HT + 1];               // 1 / root mean square of the queries and of the row's own key
 
     if (!p.fresh) {
         for (int s = tid; s < p.b.seqs; s += kRowThreads)
@@ -96,18 +106,44 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     const int pos = pos0 + (row - row0);
     const T* proj = (const T*)a.proj;
     const T* prow = proj + (int64_t)row * a.ld;
-    const T* kring = (const T*)a.kring + ((int64_t)p.b.slot[seq] * a.kv_heads + kvh) * a.ring * dim;
-    const T* vring = (const T*)a.vring + ((int64_t)p.b.slot[seq] * a.kv_heads + kvh) * a.ring * vdim;
+    const int64_t head_row = ((int64_t)p.b.slot[seq] * a.kv_heads + kvh) * (a.kept + a.ring);
+    T* kcache = (T*)a.kring + head_row * dim;
+    T* vcache = (T*)a.vring + head_row * vdim;
 
-    const T* kcur = proj + (int64_t)row0 * a.ld + a.off_k + (int64_t)kvh * dim;
-    const T* vcur = proj + (int64_t)row0 * a.ld + a.off_v + (int64_t)kvh * vdim;
+    const unsigned ldk = (unsigned)p.ld_rows;
+    const T* kcur = (const T*)p.krows + (int64_t)row0 * ldk + (int64_t)kvh * dim;
+    const T* vcur = (const T*)p.vrows + (int64_t)row0 * ldk + (int64_t)kvh * vdim;
+    const int cur0 = p.fresh && !p.own ? 0x7fffffff : pos0;  // positions from here on are rows of the step (a borrower's decode step: none)
 
-    const int lo = max(0, pos - a.window + 1);
-    const int n_keys = pos - lo + 1;
+    // the visible keys, in order: number g < n_first is position g, the others follow from position w0 on; the last is the row's own
+    const int n_first = min(a.keep, pos + 1);
+    const int w0 = max(pos - a.window + 1, n_first);
+    const int n_keys = n_first + pos - w0 + 1;
+    const int r0 = max(w0, a.kept);                               // first of them in the ring
+    const unsigned slot_r0 = (unsigned)(r0 - a.kept) % (unsigned)a.ring;  // (pos - r0 < ring: one wrap at most)
+    auto pos_of = [&](int g) { return g < n_first ? g : w0 + (g - n_first); };
+    auto row_of = [&](int kp) {
+        const unsigned s = slot_r0 + (unsigned)(kp - r0);
+        return kp < a.kept ? (unsigned)kp : (unsigned)a.kept + (s < (unsigned)a.ring ? s : s - a.ring);
+    };
     const int step = (n_keys + p.n_split - 1) / p.n_split;
-    const int k_begin = lo + split * step, k_end = min(pos + 1, k_begin + step);
-    const bool owner = k_begin <= pos && k_end == pos + 1;  // this split holds the row's own key
+    const int k_begin = split * step, k_end = min(n_keys, k_begin + step);
+    const bool owner = p.own && k_begin < n_keys && k_end == n_keys;  // this split holds the row's own key
 
+    if (a.unit_qk) {  // a wave per head (the last one: the key)
+        for (int h = tid >> 6; h <= HT; h += kRowThreads / 64) {
+            if (h < HT ? h >= nh : !owner) continue;
+            const T* src = h < HT ? prow + a.off_q + (int64_t)(h0 + h) * dim : prow + a.off_k + (int64_t)kvh * dim;
+            float ss = 0.f;
+            for (int d = tid & 63; d < dim; d += 64) {
+                const float v = to_f32<T>(src[d]);
+                ss += v * v;
+            }
+            ss = group_sum(ss, 64);
+            if ((tid & 63) == 0) s_rms[h] = 1.0f / sqrtf(ss / (float)dim + a.unit_eps);
+        }
+        __syncthreads();
+    }
     for (int i = tid; i < nh * dim; i += kRowThreads) {
         const int h = i / dim, d = i - h * dim;
         const T* src = prow + a.off_q + (int64_t)(h0 + h) * dim;
@@ -118,10 +154,10 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             const float w = to_f32<T>(src[d ^ 1]);
             v = (d & 1) ? v * c + w * s : v * c - w * s;
         }
-        q[h * dim + d] = v * a.scale;
+        q[h * dim + d] = v * (a.unit_qk ? a.scale * s_rms[h] : a.scale);
     }
-    if (p.fresh && owner) {
-        T* kw = (T*)a.kring + ((int64_t)p.b.slot[seq] * a.kv_heads + kvh) * a.ring * dim + (int64_t)(pos % a.ring) * dim;
+    if (owner) {
+        T* kw = kcache + (int64_t)row_of(pos) * dim;
         const T* src = prow + a.off_k + (int64_t)kvh * dim;
         for (int d = tid; d < dim; d += kRowThreads) {
             float v = to_f32<T>(src[d]);
@@ -131,19 +167,20 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
                 const float w = to_f32<T>(src[d ^ 1]);
                 v = (d & 1) ? v * c + w * s : v * c - w * s;
             }
-            const T r = from_f32<T>(v);
+            const T r = from_f32<T>(a.unit_qk ? v * s_rms[HT] : v);
             kn[d] = to_f32<T>(r);
             if (ht == 0) kw[d] = r;
         }
         if (ht == 0) {
-            T* vw = (T*)a.vring + ((int64_t)p.b.slot[seq] * a.kv_heads + kvh) * a.ring * vdim + (int64_t)(pos % a.ring) * vdim;
+            T* vw = vcache + (int64_t)row_of(pos) * vdim;
             const T* vs = prow + a.off_v + (int64_t)kvh * vdim;
             for (int d = tid; d < vdim; d += kRowThreads) vw[d] = vs[d];
         }
     }
-    if (tid < HT) {
-        stat[tid] = -INFINITY;
-        stat[HT + tid] = 0.f;
+    if (tid < HT) {  // the sink is a key without a value: a score of its own in the first split
+        const bool sink = a.sink != nullptr && split == 0 && tid < nh;
+        stat[tid] = sink ? a.sink[h0 + tid] : -INFINITY;
+        stat[HT + tid] = sink ? 1.f : 0.f;
     }
     __syncthreads();
 
@@ -158,7 +195,6 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
 
     for (int kb = k_begin; kb < k_end; kb += kKeys) {
         const int nk = min(kKeys, k_end - kb);
-        const unsigned slot0 = (unsigned)kb % (unsigned)a.ring;  // (nk <= ring: a pass wraps once at most)
         // ---- scores: 16 lanes per key, four keys per lane group in flight
         const int l16 = tid & 15;
         for (int k4 = tid >> 4; k4 - (tid >> 4) < nk; k4 += 4 * (kRowThreads / 16)) {
@@ -166,9 +202,8 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             const T* src[4];
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
-                const int kk = min(k4 + u * (kRowThreads / 16), nk - 1), kp = kb + kk;
-                const unsigned sl = slot0 + kk < (unsigned)a.ring ? slot0 + kk : slot0 + kk - a.ring;
-                src[u] = kp >= pos0 ? kcur + (unsigned)(kp - pos0) * (unsigned)a.ld : kring + sl * (unsigned)dim;
+                const int kk = min(k4 + u * (kRowThreads / 16), nk - 1), kp = pos_of(kb + kk);
+                src[u] = kp >= cur0 ? kcur + (unsigned)(kp - pos0) * ldk : kcache + row_of(kp) * (unsigned)dim;
 #pragma unroll
                 for (int h = 0; h < HT; ++h) dot[u][h] = 0.f;
             }
@@ -192,19 +227,19 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
                 const int kk = k4 + u * (kRowThreads / 16);
 #pragma unroll
                 for (int h = 0; h < HT; ++h) dot[u][h] = group_sum(dot[u][h], 16);
-                if (l16 == 0 && kk < nk && !(p.fresh && kb + kk == pos)) {
+                if (l16 == 0 && kk < nk && !(p.own && kb + kk == n_keys - 1)) {
 #pragma unroll
                     for (int h = 0; h < HT; ++h)
                         if (h < nh) sc[kk * HT + h] = dot[u][h];
                 }
             }
         }
-        if (p.fresh && kb + nk > pos && (tid >> 4) < nh) {  // the row's own key, rotated above: lane group h takes head h
+        if (p.own && kb + nk == n_keys && (tid >> 4) < nh) {  // the row's own key, prepared above: lane group h takes head h
             const int h = tid >> 4;
             float s = 0.f;
             for (int d = l16; d < dim; d += 16) s += kn[d] * q[h * dim + d];
             s = group_sum(s, 16);
-            if (l16 == 0) sc[(pos - kb) * HT + h] = s;
+            if (l16 == 0) sc[(n_keys - 1 - kb) * HT + h] = s;
         }
         __syncthreads();
         // ---- running maximum and sum: one wave per head
@@ -239,9 +274,8 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             }
 #pragma unroll 4
             for (int kk = kl; kk < nk; kk += n_kl) {
-                const int kp = kb + kk;
-                const unsigned sl = slot0 + kk < (unsigned)a.ring ? slot0 + kk : slot0 + kk - a.ring;
-                const T* src = kp >= pos0 ? vcur + (unsigned)(kp - pos0) * (unsigned)a.ld : vring + sl * (unsigned)vdim;
+                const int kp = pos_of(kb + kk);
+                const T* src = kp >= cur0 ? vcur + (unsigned)(kp - pos0) * ldk : vcache + row_of(kp) * (unsigned)vdim;
                 float v[VE], w[HT];
 #pragma unroll
                 for (int h = 0; h < HT; ++h) w[h] = sc[kk * HT + h];
@@ -262,7 +296,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             a.partials[(((int64_t)row * a.heads + h0 + h) * p.n_split + split) * (vdim + 2) + 2 + d] = o;
         } else {
             o /= stat[HT + h];
-            if (a.off_g >= 0) o *= 1.0f / (1.0f + expf(-to_f32<T>(prow[a.off_g + h0 + h])));
+            if (a.off_g >= 0) o *= sigmoid_f32(to_f32<T>(prow[a.off_g + (a.gate_values ? (h0 + h) * vdim + d : h0 + h)]));
             ((T*)a.y)[(int64_t)row * a.ldy + (int64_t)(h0 + h) * vdim + d] = from_f32<T>(o);
         }
     };
@@ -302,55 +336,77 @@ __global__ __launch_bounds__(128) void window_join_kernel(const WinParams p) {
     const float m = wave_max(ms);
     const float e = expf(ms - m);
     if ((int)threadIdx.x < p.n_split) wgt[threadIdx.x] = e;
+    const T* gates = (const T*)a.proj + (int64_t)row * a.ld + a.off_g;
     float gate = 1.f / group_sum(e * ls, 64);
-    if (a.off_g >= 0) gate /= 1.0f + expf(-to_f32<T>(((const T*)a.proj)[(int64_t)row * a.ld + a.off_g + h]));
+    if (a.off_g >= 0 && !a.gate_values) gate *= sigmoid_f32(to_f32<T>(gates[h]));
     __syncthreads();
     for (int d = threadIdx.x; d < a.vdim; d += blockDim.x) {
         float o = 0.f;
 #pragma unroll 16
         for (int s = 0; s < p.n_split; ++s) o += wgt[s] * rec[s * (a.vdim + 2) + 2 + d];
+        if (a.off_g >= 0 && a.gate_values) o *= sigmoid_f32(to_f32<T>(gates[h * a.vdim + d]));
         ((T*)a.y)[(int64_t)row * a.ldy + (int64_t)h * a.vdim + d] = from_f32<T>(o * gate);
     }
 }
 
-// ------------------------------------------------------------------------------------ prompt steps: rotation, ring
+// ------------------------------------------------------------------------------------ prompt steps: keys, cache
 // grid (ceil(max_count / 4), seqs), 256 threads: a wave per row
 template <typename T>
-__global__ __launch_bounds__(256) void rotate_keys_kernel(const WinParams p) {
+__global__ __launch_bounds__(256) void prepare_keys_kernel(const WinParams p) {
     const mi355_window_attn_args& a = p.a;
     const int seq = blockIdx.y, i = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (i >= p.b.count[seq]) return;
     const int pos = p.b.pos[seq] + i, half = a.rot_dims / 2;
-    T* k = (T*)a.proj + (int64_t)(p.b.row0[seq] + i) * a.ld + a.off_k;
-    for (int pi = lane; pi < half; pi += 64) {
-        float c, s;
-        pair_cos_sin(pos, a.inv_freq[pi], c, s);
-        for (int g = 0; g < a.kv_heads; ++g) {
-            T* kp = k + (int64_t)g * a.dim + 2 * pi;
-            const float u = to_f32<T>(kp[0]), v = to_f32<T>(kp[1]);
-            kp[0] = from_f32<T>(u * c - v * s);
-            kp[1] = from_f32<T>(v * c + u * s);
+    const int64_t row = p.b.row0[seq] + i;
+    const T* src = (const T*)a.proj + row * a.ld;
+    T* dst = (T*)p.krows + row * p.ld_rows;
+    const bool moved = a.role == MI355_KV_LENDS;
+    for (int g = 0; g < a.kv_heads; ++g) {
+        const T* k = src + a.off_k + (int64_t)g * a.dim;
+        T* o = dst + (int64_t)g * a.dim;
+        float rms = 1.f;
+        if (a.unit_qk) {
+            float ss = 0.f;
+            for (int d = lane; d < a.dim; d += 64) {
+                const float v = to_f32<T>(k[d]);
+                ss += v * v;
+            }
+            rms = 1.0f / sqrtf(group_sum(ss, 64) / (float)a.dim + a.unit_eps);
         }
+        for (int pi = lane; pi < half; pi += 64) {
+            float c, s;
+            pair_cos_sin(pos, a.inv_freq[pi], c, s);
+            const float u = to_f32<T>(k[2 * pi]) * rms, v = to_f32<T>(k[2 * pi + 1]) * rms;
+            o[2 * pi] = from_f32<T>(u * c - v * s);
+            o[2 * pi + 1] = from_f32<T>(v * c + u * s);
+        }
+        if (a.unit_qk || moved)
+            for (int d = a.rot_dims + lane; d < a.dim; d += 64) o[d] = from_f32<T>(to_f32<T>(k[d]) * rms);
+    }
+    if (moved) {
+        T* vo = (T*)p.vrows + row * p.ld_rows;
+        for (int j = lane; j < a.kv_heads * a.vdim; j += 64) vo[j] = src[a.off_v + j];
     }
 }
 
-// grid (min(max_count, ring), seqs): the last `ring` rows of every portion
+// grid (min(max_count, ring) + kept, seqs): the last `ring` rows of every portion, and those of positions below `kept`
 template <typename T>
-__global__ __launch_bounds__(256) void ring_write_kernel(const WinParams p) {
+__global__ __launch_bounds__(256) void ring_write_kernel(const WinParams p, int n_last) {
     const mi355_window_attn_args& a = p.a;
-    const int seq = blockIdx.y, cnt = p.b.count[seq];
-    const int i = cnt - 1 - (int)blockIdx.x;
-    if (i < 0) return;
-    const int slot_row = (p.b.pos[seq] + i) % a.ring;
-    const T* src = (const T*)a.proj + (int64_t)(p.b.row0[seq] + i) * a.ld;
+    const int seq = blockIdx.y, cnt = p.b.count[seq], pos0 = p.b.pos[seq];
+    const bool first = (int)blockIdx.x >= n_last;
+    const int i = first ? (int)blockIdx.x - n_last - pos0 : cnt - 1 - (int)blockIdx.x;
+    if (i < 0 || i >= cnt || (!first && pos0 + i < a.kept)) return;
+    const int64_t row = p.b.row0[seq] + i, to = cache_row(a, pos0 + i), rows = a.kept + a.ring;
+    const T *ks = (const T*)p.krows + row * p.ld_rows, *vs = (const T*)p.vrows + row * p.ld_rows;
     const int64_t base = (int64_t)p.b.slot[seq] * a.kv_heads;
     for (int j = threadIdx.x; j < a.kv_heads * a.dim; j += 256) {
         const int g = j / a.dim, d = j - g * a.dim;
-        ((T*)a.kring)[((base + g) * a.ring + slot_row) * a.dim + d] = src[a.off_k + j];
+        ((T*)a.kring)[((base + g) * rows + to) * a.dim + d] = ks[j];
     }
     for (int j = threadIdx.x; j < a.kv_heads * a.vdim; j += 256) {
         const int g = j / a.vdim, d = j - g * a.vdim;
-        ((T*)a.vring)[((base + g) * a.ring + slot_row) * a.vdim + d] = src[a.off_v + j];
+        ((T*)a.vring)[((base + g) * rows + to) * a.vdim + d] = vs[j];
     }
 }
 
@@ -406,7 +462,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const int q_pos = pos0 + q_row;
     const bf16_t* proj = (const bf16_t*)a.proj;
     const int q_first = pos0 + qb * kBQ, q_last = pos0 + min(qb * kBQ + kBQ, cnt) - 1;
+    // key steps: those of the first `keep` positions that lie in front of the window, then the window's
     const int kb0 = max(0, q_first - a.window + 1) / kBK, kb1 = q_last / kBK + 1;
+    const int n_first = min((a.keep + kBK - 1) / kBK, kb0), n_steps = n_first + kb1 - kb0;
     // the wave's own range, for the masks
     const int w_first = min(pos0 + qb * kBQ + wave * 32, pos0 + cnt - 1), w_last = min(w_first + 31, pos0 + cnt - 1);
 
@@ -414,7 +472,22 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     bf16x8 bq[D / 16];
     {
         const bf16_t* src = proj + (int64_t)(row0 + q_row) * a.ld + a.off_q + (int64_t)h * a.dim;
-        const float qs = a.scale * 1.44269504088896340736f;
+        float qs = a.scale * 1.44269504088896340736f;
+        if (a.unit_qk) {  // lanes c and c + 32 hold the row between them
+            float ss = 0.f;
+#pragma unroll
+            for (int ks = 0; ks < D / 16; ++ks) {
+                const int d0 = 16 * ks + 8 * hh;
+                if (d0 < a.dim) {
+                    float v[8];
+                    load_vec<bf16_t, 8>(src + d0, v);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+                }
+            }
+            ss += lane_xor32(ss);
+            qs /= sqrtf(ss / (float)a.dim + a.unit_eps);
+        }
 #pragma unroll
         for (int ks = 0; ks < D / 16; ++ks) {
             const int d0 = 16 * ks + 8 * hh;
@@ -439,10 +512,10 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
         }
     }
     const int64_t slot_head = (int64_t)p.b.slot[seq] * a.kv_heads + kvh;
-    const bf16_t* kring = (const bf16_t*)a.kring + slot_head * a.ring * a.dim;
-    const bf16_t* vring = (const bf16_t*)a.vring + slot_head * a.ring * a.vdim;
-    const bf16_t* kcur = proj + (int64_t)row0 * a.ld + a.off_k + (int64_t)kvh * a.dim;
-    const bf16_t* vcur = proj + (int64_t)row0 * a.ld + a.off_v + (int64_t)kvh * a.vdim;
+    const bf16_t* kcache = (const bf16_t*)a.kring + slot_head * (a.kept + a.ring) * a.dim;
+    const bf16_t* vcache = (const bf16_t*)a.vring + slot_head * (a.kept + a.ring) * a.vdim;
+    const bf16_t* kcur = (const bf16_t*)p.krows + (int64_t)row0 * p.ld_rows + (int64_t)kvh * a.dim;
+    const bf16_t* vcur = (const bf16_t*)p.vrows + (int64_t)row0 * p.ld_rows + (int64_t)kvh * a.vdim;
     const int p_last = pos0 + cnt - 1;
     u32x4 kreg[kKItems], vreg[kVItems][4];
     const u32x4 zero4 = {0u, 0u, 0u, 0u};
@@ -450,7 +523,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const bool k_in = t_col * 8 < a.dim;
     auto load_tile = [&](int kb) {
         if (kb * kBK >= pos0 && kb * kBK + kBK - 1 <= p_last) {  // all of the step's own rows: one multiply per thread
-            const unsigned ld = (unsigned)a.ld;
+            const unsigned ld = (unsigned)p.ld_rows;
             const unsigned ko = (unsigned)(kb * kBK + t_key - pos0) * ld + t_col * 8;
 #pragma unroll
             for (int i = 0; i < kKItems; ++i) kreg[i] = *(const u32x4*)(kcur + (k_in ? ko + (unsigned)i * (256 / kCols) * ld : 0u));
@@ -482,7 +555,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             const int kp = kb * kBK + key;
             kreg[i] = zero4;
             if (col * 8 < a.dim && kp <= p_last) {
-                const bf16_t* src = kp >= pos0 ? kcur + (int64_t)(kp - pos0) * a.ld : kring + (int64_t)(kp % a.ring) * a.dim;
+                const bf16_t* src = kp >= pos0 ? kcur + (int64_t)(kp - pos0) * p.ld_rows : kcache + (int64_t)cache_row(a, kp) * a.dim;
                 kreg[i] = *(const u32x4*)(src + col * 8);
             }
         }
@@ -494,7 +567,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                 const int kp = kb * kBK + run * 4 + r;
                 vreg[i][r] = zero4;
                 if (col < kCols && col * 8 < a.vdim && kp <= p_last) {
-                    const bf16_t* src = kp >= pos0 ? vcur + (int64_t)(kp - pos0) * a.ld : vring + (int64_t)(kp % a.ring) * a.vdim;
+                    const bf16_t* src = kp >= pos0 ? vcur + (int64_t)(kp - pos0) * p.ld_rows : vcache + (int64_t)cache_row(a, kp) * a.vdim;
                     vreg[i][r] = *(const u32x4*)(src + col * 8);
                 }
             }
@@ -535,17 +608,22 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
 #pragma unroll
         for (int i = 0; i < 16; ++i) acc[dt][i] = 0.f;
     float m_run = -1.0e30f, l_run = 0.f;
+    if (a.sink != nullptr) {  // a key without a value; one of the two lanes of a query counts it
+        m_run = a.sink[h] * 1.44269504088896340736f;
+        l_run = hh == 0 ? 1.f : 0.f;
+    }
+    auto step_of = [&](int it) { return it < n_first ? it : kb0 + (it - n_first); };
 
-    load_tile(kb0);
+    load_tile(step_of(0));
     store_tile(0);
     __syncthreads();
-    for (int kb = kb0; kb < kb1; ++kb) {
-        const int buf = (kb - kb0) & 1;
-        if (kb + 1 < kb1) load_tile(kb + 1);
+    for (int it = 0; it < n_steps; ++it) {
+        const int kb = step_of(it), buf = it & 1;
+        if (it + 1 < n_steps) load_tile(step_of(it + 1));
         const char* kt = smem + buf * kKTile;
         const char* vt = smem + 2 * kKTile + buf * kVTile;
         // a wave none of whose queries sees this step leaves it out (it still stages the next tile)
-        const bool seen = kb * kBK <= w_last && kb * kBK + kBK - 1 > w_first - a.window;
+        const bool seen = kb * kBK <= w_last && (kb * kBK + kBK - 1 > w_first - a.window || kb * kBK < a.keep);
         if (seen) {
             f32x16 st[2];
 #pragma unroll
@@ -566,7 +644,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
 #pragma unroll
                     for (int i = 0; i < 16; ++i) {
                         const int kp = kb * kBK + t2 * 32 + (i & 3) + 8 * (i >> 2) + 4 * hh;
-                        st[t2][i] = (kp <= q_pos && kp > q_pos - a.window) ? st[t2][i] : -1.0e30f;
+                        st[t2][i] = (kp <= q_pos && (kp > q_pos - a.window || kp < a.keep)) ? st[t2][i] : -1.0e30f;
                     }
             }
             // (inline assembly gets no wait states behind the matrix instruction that wrote its operands: 20 here cover the longest)
@@ -609,13 +687,15 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                 }
             }
         }
-        if (kb + 1 < kb1) store_tile(buf ^ 1);
+        if (it + 1 < n_steps) store_tile(buf ^ 1);
         __syncthreads();
     }
     const float l = l_run + lane_xor32(l_run);
     if (q_ok) {
         float inv = 1.0f / l;
-        if (a.off_g >= 0) inv /= 1.0f + expf(-bf16_to_f32(proj[(int64_t)(row0 + q_row) * a.ld + a.off_g + h]));
+        const bf16_t* gates = proj + (int64_t)(row0 + q_row) * a.ld + a.off_g;
+        if (a.off_g >= 0 && !a.gate_values) inv *= sigmoid_f32(bf16_to_f32(gates[h]));
+        const bool each = a.off_g >= 0 && a.gate_values;
         bf16_t* y = (bf16_t*)a.y + (int64_t)(row0 + q_row) * a.ldy + (int64_t)h * a.vdim;
 #pragma unroll
         for (int dt = 0; dt < D / 32; ++dt)
@@ -623,9 +703,17 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             for (int g = 0; g < 4; ++g) {
                 const int d = dt * 32 + 8 * g + 4 * hh;
                 if (d < a.vdim) {  // (vdim % 8 == 0)
+                    float r[4];
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) r[e] = acc[dt][4 * g + e] * inv;
+                    if (each) {
+                        const u32x2 z = *(const u32x2*)(gates + h * a.vdim + d);
+                        r[0] *= sigmoid_f32(__uint_as_float(z[0] << 16)), r[1] *= sigmoid_f32(__uint_as_float(z[0] & 0xffff0000u));
+                        r[2] *= sigmoid_f32(__uint_as_float(z[1] << 16)), r[3] *= sigmoid_f32(__uint_as_float(z[1] & 0xffff0000u));
+                    }
                     u32x2 o;
-                    o[0] = pack_bf16x2(acc[dt][4 * g] * inv, acc[dt][4 * g + 1] * inv);
-                    o[1] = pack_bf16x2(acc[dt][4 * g + 2] * inv, acc[dt][4 * g + 3] * inv);
+                    o[0] = pack_bf16x2(r[0], r[1]);
+                    o[1] = pack_bf16x2(r[2], r[3]);
                     *(u32x2*)(y + d) = o;
                 }
             }
@@ -642,10 +730,16 @@ int launch_tiles(const WinParams& p, hipStream_t s) {
     return 0;
 }
 
-bool tiles_fit(const mi355_window_attn_args& a) {
+// keys and values of the step's rows and of the cache can be read 16 bytes at a time
+bool rows_aligned(const WinParams& p) {
+    return p.ld_rows % 8 == 0 && (uintptr_t)p.krows % 16 == 0 && (uintptr_t)p.vrows % 16 == 0 && (uintptr_t)p.a.kring % 16 == 0 &&
+           (uintptr_t)p.a.vring % 16 == 0;
+}
+
+bool tiles_fit(const WinParams& p) {
+    const mi355_window_attn_args& a = p.a;
     return a.dtype == MI355_BF16 && a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 256 && a.vdim <= 256 && a.ld % 8 == 0 && a.ldy % 4 == 0 &&
-           a.off_q % 8 == 0 && a.off_k % 8 == 0 && a.off_v % 8 == 0 && (uintptr_t)a.proj % 16 == 0 && (uintptr_t)a.kring % 16 == 0 &&
-           (uintptr_t)a.vring % 16 == 0 && (uintptr_t)a.y % 8 == 0;
+           a.off_q % 8 == 0 && rows_aligned(p) && (!a.gate_values || a.off_g % 4 == 0) && (uintptr_t)a.proj % 16 == 0 && (uintptr_t)a.y % 8 == 0;
 }
 
 int run_tiles(const WinParams& p, hipStream_t s) {
@@ -675,8 +769,7 @@ template <typename T>
 int run_rows(WinParams p, hipStream_t s) {
     const mi355_window_attn_args& a = p.a;
     const int per = a.heads / a.kv_heads;
-    const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0 && a.ld % 8 == 0 && a.off_q % 8 == 0 && a.off_k % 8 == 0 && a.off_v % 8 == 0 &&
-                     (uintptr_t)a.proj % 16 == 0 && (uintptr_t)a.kring % 16 == 0 && (uintptr_t)a.vring % 16 == 0;
+    const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0 && rows_aligned(p);
     MI355_CHECK_ARG(vec ? a.vdim <= 8 * kRowThreads : a.vdim <= kRowThreads, MI355_E_SHAPE,
                     "window_attention: value size %d exceeds the row kernel's %d", a.vdim, vec ? 8 * kRowThreads : kRowThreads);
     const int HT = per >= 5 ? 8 : per >= 2 ? 4 : 1;
@@ -692,6 +785,14 @@ int run_rows(WinParams p, hipStream_t s) {
 }
 
 template <typename T>
+int run_cache_write(const WinParams& p, hipStream_t s) {
+    const int n_last = p.b.max_count < p.a.ring ? p.b.max_count : p.a.ring;
+    hipLaunchKernelGGL(ring_write_kernel<T>, dim3(n_last + p.a.kept, p.b.seqs), dim3(256), 0, s, p, n_last);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+
+template <typename T>
 int run(WinParams p, hipStream_t s) {
     const mi355_window_attn_args& a = p.a;
     if (p.fresh) {
@@ -699,7 +800,8 @@ int run(WinParams p, hipStream_t s) {
         const int per = a.heads / a.kv_heads, ht = per >= 5 ? 8 : per >= 2 ? 4 : 1;
         const int groups = p.b.rows * a.kv_heads * ((per + ht - 1) / ht);
         int n = 2048 / groups;
-        n = n < a.ring / 64 ? n : a.ring / 64;
+        const int most = (a.keep + (a.window < a.ring ? a.window : a.ring)) / 64;
+        n = n < most ? n : most;
         n = n < kMaxSplit ? n : kMaxSplit;
         const uint64_t rec = (uint64_t)p.b.rows * a.heads * (a.vdim + 2) * 4;
         if (a.partials == nullptr) n = 1;
@@ -712,27 +814,23 @@ int run(WinParams p, hipStream_t s) {
         }
         return 0;
     }
-    if (a.rot_dims > 0) {
-        hipLaunchKernelGGL(rotate_keys_kernel<T>, dim3((p.b.max_count + 3) / 4, p.b.seqs), dim3(256), 0, s, p);
+    if (a.role == MI355_KV_LENDS || (a.role == MI355_KV_OWN && (a.rot_dims > 0 || a.unit_qk))) {
+        hipLaunchKernelGGL(prepare_keys_kernel<T>, dim3((p.b.max_count + 3) / 4, p.b.seqs), dim3(256), 0, s, p);
         MI355_LAUNCH_CHECK();
     }
     p.n_split = 1;
     // (a handful of rows per sequence would leave most of a 128-query tile empty)
     const bool tiles = a.path == 2 || (a.path == 0 && p.b.max_count > 8);
-    if (tiles && tiles_fit(a)) {
+    if (tiles && tiles_fit(p)) {
         if (int rc = run_tiles(p, s)) return rc;
     } else {
         MI355_CHECK_ARG(a.path != 2, MI355_E_SHAPE, "window_attention: the tile kernel takes bf16 heads of up to 256, multiples of 8");
         if (int rc = run_rows<T>(p, s)) return rc;
     }
-    hipLaunchKernelGGL(ring_write_kernel<T>, dim3(p.b.max_count < a.ring ? p.b.max_count : a.ring, p.b.seqs), dim3(256), 0, s, p);
-    MI355_LAUNCH_CHECK();
-    return 0;
+    return a.role == MI355_KV_OWN ? run_cache_write<T>(p, s) : 0;
 }
 
-}  // namespace
-
-extern "C" int mi355_window_attention(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream) {
+int make_params(const mi355_window_attn_args* a, const mi355_seq_batch* b, WinParams& p) {
     MI355_CHECK_ARG(a && b && a->proj && a->kring && a->vring && a->y, MI355_E_ARG, "window_attention: null argument");
     MI355_CHECK_ARG(b->row0 && b->count && b->slot && b->pos, MI355_E_ARG, "window_attention: null batch");
     MI355_CHECK_ARG(b->rows > 0 && b->rows <= 65535 && b->seqs > 0 && b->seqs <= b->rows && b->max_count > 0, MI355_E_SHAPE,
@@ -740,16 +838,46 @@ extern "C" int mi355_window_attention(const mi355_window_attn_args* a, const mi3
     MI355_CHECK_ARG(a->dtype == MI355_F32 || a->dtype == MI355_BF16, MI355_E_DTYPE, "window_attention: dtype must be f32 or bf16");
     MI355_CHECK_ARG(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim > 0 && a->vdim > 0, MI355_E_SHAPE,
                     "window_attention: bad heads %d / %d or sizes %d / %d", a->heads, a->kv_heads, a->dim, a->vdim);
-    MI355_CHECK_ARG((uint64_t)b->max_count * (uint64_t)a->ld < 0xFFFFFFFFull && (uint64_t)a->ring * (a->dim > a->vdim ? a->dim : a->vdim) < 0xFFFFFFFFull,
-                    MI355_E_SHAPE, "window_attention: %d rows of pitch %lld or a ring of %d rows exceed 32-bit offsets", b->max_count,
-                    (long long)a->ld, a->ring);
     MI355_CHECK_ARG(a->window > 0 && a->ring > 0 && a->rot_dims >= 0 && a->rot_dims % 2 == 0 && a->rot_dims <= a->dim &&
                         (a->rot_dims == 0 || a->inv_freq),
                     MI355_E_SHAPE, "window_attention: bad window %d, ring %d or rotation %d", a->window, a->ring, a->rot_dims);
-    WinParams p;
+    MI355_CHECK_ARG(a->keep >= 0 && a->keep <= a->kept, MI355_E_SHAPE, "window_attention: %d first rows visible, %d cached", a->keep, a->kept);
+    MI355_CHECK_ARG(a->role >= MI355_KV_OWN && a->role <= MI355_KV_BORROWS && (a->role == MI355_KV_OWN || a->kv_rows), MI355_E_ARG,
+                    "window_attention: a lender and its borrowers share kv_rows");
     p.a = *a;
     p.b = *b;
     p.fresh = b->max_count == 1;
+    p.own = p.fresh && a->role != MI355_KV_BORROWS;
     p.n_split = p.head_tiles = 1;
+    const int size = dtype_size(a->dtype);
+    if (a->role == MI355_KV_OWN || p.own) {
+        p.krows = (const char*)a->proj + (int64_t)a->off_k * size;
+        p.vrows = (const char*)a->proj + (int64_t)a->off_v * size;
+        p.ld_rows = a->ld;
+    } else {
+        p.krows = a->kv_rows;
+        p.vrows = (const char*)a->kv_rows + (int64_t)a->kv_heads * a->dim * size;
+        p.ld_rows = (int64_t)a->kv_heads * (a->dim + a->vdim);
+    }
+    MI355_CHECK_ARG((uint64_t)b->max_count * (uint64_t)p.ld_rows < 0xFFFFFFFFull && (uint64_t)b->max_count * (uint64_t)a->ld < 0xFFFFFFFFull &&
+                        (uint64_t)(a->kept + (int64_t)a->ring) * (a->dim > a->vdim ? a->dim : a->vdim) < 0xFFFFFFFFull,
+                    MI355_E_SHAPE, "window_attention: %d rows of pitch %lld or a cache of %d + %d rows exceed 32-bit offsets", b->max_count,
+                    (long long)a->ld, a->kept, a->ring);
+    return 0;
+}
+
+}  // namespace
+
+extern "C" int mi355_window_attention(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream) {
+    WinParams p;
+    if (int rc = make_params(a, b, p)) return rc;
     return a->dtype == MI355_F32 ? run<float>(p, (hipStream_t)stream) : run<bf16_t>(p, (hipStream_t)stream);
+}
+
+extern "C" int mi355_window_cache_write(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream) {
+    WinParams p;
+    if (int rc = make_params(a, b, p)) return rc;
+    MI355_CHECK_ARG(a->role == MI355_KV_LENDS, MI355_E_ARG, "window_cache_write: the other layers write their cache themselves");
+    if (p.fresh) return 0;  // (a decode step wrote its rows with the lender's attention)
+    return a->dtype == MI355_F32 ? run_cache_write<float>(p, (hipStream_t)stream) : run_cache_write<bf16_t>(p, (hipStream_t)stream);
 }

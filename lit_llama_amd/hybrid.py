@@ -1,14 +1,15 @@
 """Layered hybrid decoders: a list of layers, each with its own mixer (window attention, gated delta rule, gated linear attention) and an
-optional feed-forward, some of them run several times in a row.
+optional feed-forward (squared ReLU, gated GELU, mixture of experts), some of them run several times in a row.
 
 `HybridConfig` reads a parsed config.json; `HybridLM` holds the weights under their checkpoint names and hands the arithmetic to
-`hybrid_engine.HybridEngine` (csrc/hybrid.hip and the kernels it calls).  The Sekulorn design is the family registered here; a mixer or a
-feed-forward of another design is an entry in MIXERS / MLPS and a kernel.
+`hybrid_engine.HybridEngine` (csrc/hybrid.hip and the kernels it calls).  A design is an entry in DESIGNS: which mixers and feed-forwards it
+has, how it reads them from its configuration, and what it does around them; a mixer or a feed-forward that none has yet is a spec and a
+kernel.
 """
 from __future__ import annotations
 
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional, Tuple
+from typing import Callable, Dict, List, Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -27,20 +28,39 @@ class MixerSpec:
     vdim: int                      # value size of a head
     scale: float = 1.0             # attention
     window: int = 0
+    keep: int = 0                  # first tokens that stay visible
     rot_dims: int = 0
     rot_base: float = 10000.0
+    unit_qk: bool = False          # q and k over their root mean square
+    sink: bool = False             # a learned term in every softmax sum
+    gate_values: bool = False      # a gate per value, not per head
+    kv_from: Optional[int] = None  # the layer whose keys and values are read
     taps: int = 0                  # delta: convolution taps
     tau: float = 1.0               # gla
 
 
 @dataclass
+class MlpSpec:
+    kind: str                      # relu2 | geglu | experts
+    ff: int                        # hidden size (of one expert)
+    experts: int = 0
+    top: int = 0
+    scale: float = 1.0             # the chosen experts' weights sum to this
+    ff_shared: int = 0             # of the expert that every token runs, 0: none
+
+
+@dataclass
 class LayerSpec:
     mixer: MixerSpec
-    ff: int = 0                    # width of the squared-ReLU feed-forward, 0: none
+    mlp: Optional[MlpSpec] = None
+
+    @property
+    def ff(self) -> int:
+        return self.mlp.ff if self.mlp is not None else 0
 
 
 def _only(d: dict, known: Tuple[str, ...], what: str) -> None:
-    extra = sorted(set(d) - set(known))
+    extra = sorted(k for k in set(d) - set(known) if d[k] is not None)
     if extra:
         raise ValueError(f"{what}: unknown configuration {extra}")
 
@@ -55,6 +75,17 @@ def _attention(m: dict) -> MixerSpec:
                      rot_dims=int(rot["dims"]), rot_base=float(rot["base"]))
 
 
+def _sink_attention(m: dict) -> MixerSpec:
+    """Attention without rotation: unit queries and keys, first tokens kept, sinks, a gate per value, keys and values of another layer."""
+    _only(m, ("heads", "kv_heads", "dim", "vdim", "scale", "mask", "kv_from"), "attention mixer")
+    mask = m.get("mask") or {"size": 1 << 30}
+    _only(mask, ("size", "keep_first"), "mask")
+    lender = m.get("kv_from")
+    return MixerSpec("attention", m["heads"], m["kv_heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=int(mask["size"]),
+                     keep=int(mask.get("keep_first") or 0), unit_qk=True, sink=True, gate_values=True,
+                     kv_from=None if lender is None else int(lender))
+
+
 def _delta(m: dict) -> MixerSpec:
     _only(m, ("heads", "kv_heads", "dim", "vdim", "conv"), "delta mixer")
     return MixerSpec("delta", m["heads"], m["kv_heads"], m["dim"], m["vdim"], taps=int(m["conv"]))
@@ -65,8 +96,40 @@ def _gla(m: dict) -> MixerSpec:
     return MixerSpec("gla", m["heads"], m["heads"], m["dim"], m["vdim"], tau=float(m["tau"]))
 
 
-MIXERS = {"attention": _attention, "delta": _delta, "gla": _gla}
-MLPS = ("dense",)
+def _plain(kind: str) -> Callable[[dict], MlpSpec]:
+    def read(d: dict) -> MlpSpec:
+        _only(d, ("kind", "ff"), "feed-forward")
+        return MlpSpec(kind, int(d["ff"]))
+
+    return read
+
+
+def _experts(d: dict) -> MlpSpec:
+    _only(d, ("kind", "expert", "router", "shared"), "feed-forward")
+    _only(d["expert"], ("ff",), "expert")
+    _only(d["router"], ("experts", "top", "scale"), "router")
+    shared = d.get("shared") or {"ff": 0}
+    _only(shared, ("ff",), "shared expert")
+    r = d["router"]
+    spec = MlpSpec("experts", int(d["expert"]["ff"]), int(r["experts"]), int(r["top"]), float(r.get("scale", 1.0)), int(shared["ff"]))
+    if not 1 <= spec.top <= spec.experts:
+        raise ValueError(f"router: {spec.top} of {spec.experts} experts")
+    return spec
+
+
+@dataclass(frozen=True)
+class Design:
+    mixers: Dict[str, Callable[[dict], MixerSpec]]
+    mlps: Dict[str, Callable[[dict], MlpSpec]]
+    keys: Tuple[str, ...]          # of the configuration, next to the common ones
+    norm_add: float = 0.0          # an RMSNorm's scale is norm_add + its weight
+    tied: bool = False             # the logits are products with the embedding table
+
+
+DESIGNS = {
+    "Sekulorn": Design({"attention": _attention, "delta": _delta, "gla": _gla}, {"dense": _plain("relu2")}, ("loop", "residual_mult")),
+    "Kovalorn": Design({"attention": _sink_attention}, {"dense": _plain("geglu"), "moe": _experts}, ("logit_scale",), norm_add=1.0, tied=True),
+}
 
 
 @dataclass
@@ -76,6 +139,7 @@ class HybridConfig:
     layers: List[LayerSpec]
     eps: float
     residual_mult: float = 1.0
+    logit_scale: float = 1.0
     loop: Tuple[int, int, int] = (0, 0, 1)  # layers start .. stop - 1 run `times` times in a row
     architecture: str = "Sekulorn"
     block_size: int = 1 << 24               # (positions are not tabulated: nothing limits a sequence but its cache)
@@ -83,21 +147,30 @@ class HybridConfig:
 
     @classmethod
     def from_dict(cls, d: dict) -> "HybridConfig":
+        name = d.get("architecture", "Sekulorn")
+        if name not in DESIGNS:
+            raise ValueError(f"unknown design {name!r} (known: {sorted(DESIGNS)})")
+        design = DESIGNS[name]
+        _only(d, ("architecture", "vocab", "width", "layers", "norm", *design.keys), "configuration")
         _only(d["norm"], ("eps",), "norm")
-        layers = []
+        layers: List[LayerSpec] = []
         for e in d["layers"]:
             _only(e, ("type", "mixer", "mlp"), "layer")
-            if e["type"] not in MIXERS:
-                raise ValueError(f"unknown mixer {e['type']!r} (known: {sorted(MIXERS)})")
+            if e["type"] not in design.mixers:
+                raise ValueError(f"unknown mixer {e['type']!r} (known: {sorted(design.mixers)})")
             mlp = e.get("mlp")
-            if mlp is not None:
-                _only(mlp, ("kind", "ff"), "feed-forward")
-                if mlp["kind"] not in MLPS:
-                    raise ValueError(f"unknown feed-forward {mlp['kind']!r} (known: {list(MLPS)})")
-            spec = MIXERS[e["type"]](e["mixer"])
+            if mlp is not None and mlp["kind"] not in design.mlps:
+                raise ValueError(f"unknown feed-forward {mlp['kind']!r} (known: {sorted(design.mlps)})")
+            spec = design.mixers[e["type"]](e["mixer"])
             if spec.heads % spec.kv_heads:
                 raise ValueError(f"{spec.heads} heads over {spec.kv_heads} key / value heads")
-            layers.append(LayerSpec(spec, int(mlp["ff"]) if mlp is not None else 0))
+            if spec.kv_from is not None:
+                own = layers[spec.kv_from].mixer if 0 <= spec.kv_from < len(layers) else None
+                if own is None or own.type != "attention" or own.kv_from is not None:
+                    raise ValueError(f"layer {len(layers)}: layer {spec.kv_from} in front of it has no keys of its own")
+                if (own.kv_heads, own.dim, own.vdim) != (spec.kv_heads, spec.dim, spec.vdim):
+                    raise ValueError(f"layer {len(layers)}: the keys and values of layer {spec.kv_from} have other sizes")
+            layers.append(LayerSpec(spec, design.mlps[mlp["kind"]](mlp) if mlp is not None else None))
         loop = d.get("loop")
         if loop is not None:
             _only(loop, ("start", "stop", "times"), "loop")
@@ -105,7 +178,11 @@ class HybridConfig:
             if not (0 <= span[0] <= span[1] <= len(layers) and span[2] >= 1):
                 raise ValueError(f"bad loop {span} over {len(layers)} layers")
         return cls(int(d["vocab"]), int(d["width"]), layers, float(d["norm"]["eps"]), float(d.get("residual_mult", 1.0)),
-                   span if loop is not None else (0, 0, 1), d.get("architecture", "Sekulorn"), raw=d)
+                   float(d.get("logit_scale", 1.0)), span if loop is not None else (0, 0, 1), name, raw=d)
+
+    @property
+    def design(self) -> Design:
+        return DESIGNS[self.architecture]
 
     @property
     def padded_vocab_size(self) -> int:
@@ -116,22 +193,44 @@ class HybridConfig:
         a, b, times = self.loop
         return [*range(a), *(list(range(a, b)) * times), *range(b, len(self.layers))]
 
+    def lenders(self) -> List[Optional[int]]:
+        """Per run, the run whose keys and values it reads (the last one of its lender so far), None: its own."""
+        last: Dict[int, int] = {}
+        out: List[Optional[int]] = []
+        for r, i in enumerate(self.runs()):
+            j = self.layers[i].mixer.kv_from
+            out.append(None if j is None else last[j])
+            last[i] = r
+        return out
 
-# the pieces of a mixer's stacked input projection, in the order of their columns
-PROJECTIONS = {"attention": ("q", "k", "v", "g"), "delta": ("q", "k", "v", "g", "a", "b"), "gla": ("q", "k", "v", "g", "a1")}
+
+def projections(m: MixerSpec) -> Tuple[str, ...]:
+    """The pieces of a mixer's stacked input projection, in the order of their columns."""
+    if m.type == "attention":
+        return ("q", "g") if m.kv_from is not None else ("q", "k", "v", "g")
+    return ("q", "k", "v", "g", "a", "b") if m.type == "delta" else ("q", "k", "v", "g", "a1")
 
 
 def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[int, ...]]:
     """name -> shape of every tensor of a checkpoint; rank[i]: the low-rank size of gla layer i (only its tensors know it)."""
     W = cfg.width
     out = {"embed": (cfg.vocab_size, W)}
+
+    def gated(p: str, ff: int) -> None:
+        out.update({p + "gate": (ff, W), p + "up": (ff, W), p + "down": (W, ff)})
+
     for i, l in enumerate(cfg.layers):
         p, m = f"l{i}.", l.mixer
         hv, gk = m.heads * m.vdim, m.kv_heads * m.dim
         out[p + "norm1"] = (W,)
         x = p + "mix."
         if m.type == "attention":
-            out.update({x + "q": (m.heads * m.dim, W), x + "k": (gk, W), x + "v": (m.kv_heads * m.vdim, W), x + "g": (m.heads, W)})
+            out[x + "q"] = (m.heads * m.dim, W)
+            if m.kv_from is None:
+                out.update({x + "k": (gk, W), x + "v": (m.kv_heads * m.vdim, W)})
+            if m.sink:
+                out[x + "sink"] = (m.heads,)
+            out[x + "g"] = (hv if m.gate_values else m.heads, W)
         else:
             out.update({x + "q": (gk, W), x + "k": (gk, W), x + "v": (hv, W), x + "g": (hv, W), x + "norm": (m.vdim,)})
         if m.type == "delta":
@@ -140,9 +239,22 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
         if m.type == "gla":
             out.update({x + "a1": (rank[i], W), x + "a2": (gk, rank[i]), x + "a2.b": (gk,)})
         out[x + "o"] = (W, hv)
-        if l.ff:
-            out.update({p + "norm2": (W,), p + "mlp.up": (l.ff, W), p + "mlp.down": (W, l.ff)})
-    out.update({"final.norm": (W,), "head": (cfg.vocab_size, W)})
+        f = l.mlp
+        if f is not None:
+            out[p + "norm2"] = (W,)
+            if f.kind == "relu2":
+                out.update({p + "mlp.up": (f.ff, W), p + "mlp.down": (W, f.ff)})
+            elif f.kind == "geglu":
+                gated(p + "mlp.", f.ff)
+            else:
+                out[p + "mlp.router"] = (f.experts, W)
+                for e in range(f.experts):
+                    gated(f"{p}mlp.e{e}.", f.ff)
+                if f.ff_shared:
+                    gated(p + "mlp.shared.", f.ff_shared)
+    out["final.norm"] = (W,)
+    if not cfg.design.tied:
+        out["head"] = (cfg.vocab_size, W)
     return out
 
 

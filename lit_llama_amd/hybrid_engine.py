@@ -17,11 +17,13 @@ import torch
 
 from . import _native as nat
 from . import ops
-from ._native import HybridLayer, HybridModel, Proj, SeqBatch, check, lib, ptr
-from .hybrid import PROJECTIONS, HybridLM
+from ._native import ExpertsArgs, HybridLayer, HybridModel, Proj, SeqBatch, check, lib, ptr
+from .hybrid import HybridLM, MlpSpec, projections
 from .state import SlotManager, grown
 
 MIX = {"attention": 0, "delta": 1, "gla": 2}
+MLP = {"relu2": 1, "geglu": 2, "experts": 3}
+KV_OWN, KV_LENDS, KV_BORROWS = 0, 1, 2
 REC_DELTA, REC_GLA = 0, 1
 
 
@@ -62,19 +64,42 @@ class HybridEngine:
         self.stream.synchronize()
 
     # ---- weights ---------------------------------------------------------------------------------------
-    def _proj(self, w: torch.Tensor) -> Proj:
+    def _own(self, w: torch.Tensor) -> int:
+        self._keep.append(w)
+        self.weight_bytes += w.numel() * w.element_size()
+        return ptr(w)
+
+    def _stream(self, w: torch.Tensor, pair: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """What the products read of a weight [N, K] or of a pair of them."""
+        if self.dtype == torch.bfloat16:
+            return ops.repack_bf16(w, pair, 1 if pair is None else 2)
+        return (w if pair is None else torch.cat([w, pair])).contiguous()
+
+    def _proj(self, w: torch.Tensor, pair: Optional[torch.Tensor] = None) -> Proj:
         """A weight [N, K] with its rows padded to a multiple of 16 (zero rows: the padding columns of every buffer stay zero)."""
         N, K = w.shape
         n = _pad16(N)
         if n != N:
-            w = torch.cat([w, w.new_zeros((n - N, K))])
-        if self.dtype == torch.bfloat16:
-            w = ops.repack_bf16(w, None, 1)
-        else:
-            w = w.contiguous()
-        self._keep.append(w)
-        self.weight_bytes += w.numel() * w.element_size()
-        return Proj(ptr(w), n, K)
+            w, pair = (t if t is None else torch.cat([t, t.new_zeros((n - N, K))]) for t in (w, pair))
+        return Proj(self._own(self._stream(w, pair)), n, K)
+
+    def _norm(self, name: str) -> int:
+        """A norm's weight; f32 models hold what is multiplied by, bf16 models the stored weight (their kernels add norm_add)."""
+        w = self.weights[name]
+        return ptr(w) if self.dtype == torch.bfloat16 or not self.cfg.design.norm_add else self._f32(w.float() + self.cfg.design.norm_add)
+
+    def _experts(self, p: str, f: MlpSpec) -> ExpertsArgs:
+        T, a = self.weights, ExpertsArgs()
+        a.dtype, a.width, a.experts, a.top = nat.dtype_code(self.dtype), self.cfg.width, f.experts, f.top
+        a.ff, a.ff_shared, a.scale = f.ff, f.ff_shared, f.scale
+        a.router = self._own(self._stream(T[p + "router"]))
+        up = [self._stream(T[f"{p}e{e}.gate"], T[f"{p}e{e}.up"]) for e in range(f.experts)]
+        a.up = self._own(torch.stack(up))
+        a.down = self._own(torch.stack([self._stream(T[f"{p}e{e}.down"]) for e in range(f.experts)]))
+        if f.ff_shared:
+            a.shared_up = self._own(self._stream(T[p + "shared.gate"], T[p + "shared.up"]))
+            a.shared_down = self._own(self._stream(T[p + "shared.down"]))
+        return a
 
     def _f32(self, t: torch.Tensor) -> int:
         t = t.detach().float().contiguous()
@@ -90,25 +115,32 @@ class HybridEngine:
             m, p = spec.mixer, f"l{i}."
             x = p + "mix."
             L = HybridLayer()
-            L.mixer, L.mlp = MIX[m.type], 1 if spec.ff else 0
-            L.norm1 = ptr(T[p + "norm1"])
+            L.mixer, L.mlp = MIX[m.type], MLP[spec.mlp.kind] if spec.mlp is not None else 0
+            L.norm1 = self._norm(p + "norm1")
             # one stacked projection, every piece padded to 16 columns
             off, parts = {}, []
-            for name in PROJECTIONS[m.type]:
+            for name in projections(m):
                 w = T[x + name]
                 off[name] = sum(q.shape[0] for q in parts)
                 pad = _pad16(w.shape[0]) - w.shape[0]
                 parts.append(torch.cat([w, w.new_zeros((pad, w.shape[1]))]) if pad else w)
             setattr(L, "in", self._proj(torch.cat(parts)))
             L.out = self._proj(T[x + "o"])
-            if spec.ff:
-                L.norm2 = ptr(T[p + "norm2"])
-                L.up, L.down = self._proj(T[p + "mlp.up"]), self._proj(T[p + "mlp.down"])
+            if spec.mlp is not None:
+                L.norm2 = self._norm(p + "norm2")
+                if spec.mlp.kind == "experts":
+                    L.moe = self._experts(p + "mlp.", spec.mlp)
+                else:
+                    L.up = self._proj(T[p + "mlp.gate"], T[p + "mlp.up"]) if spec.mlp.kind == "geglu" else self._proj(T[p + "mlp.up"])
+                    L.down = self._proj(T[p + "mlp.down"])
             if m.type == "attention":
                 a = L.attn
                 a.heads, a.kv_heads, a.dim, a.vdim = m.heads, m.kv_heads, m.dim, m.vdim
-                a.off_q, a.off_k, a.off_v, a.off_g = off["q"], off["k"], off["v"], off["g"]
-                a.scale, a.window, a.rot_dims = m.scale, m.window, m.rot_dims
+                a.off_q, a.off_k, a.off_v, a.off_g = off["q"], off.get("k", 0), off.get("v", 0), off["g"]
+                a.scale, a.window, a.rot_dims, a.keep = m.scale, m.window, m.rot_dims, m.keep
+                a.gate_values, a.unit_qk, a.unit_eps = int(m.gate_values), int(m.unit_qk), cfg.eps
+                if m.sink:
+                    a.sink = self._f32(T[x + "sink"])
                 if m.rot_dims:
                     f = torch.tensor([m.rot_base ** (-2.0 * j / m.rot_dims) for j in range(m.rot_dims // 2)], dtype=torch.float64,
                                      device=self.device)
@@ -134,12 +166,22 @@ class HybridEngine:
         self.layers = (HybridLayer * max(1, len(runs)))()
         for r, i in enumerate(runs):
             C.memmove(C.byref(self.layers[r]), C.byref(layers[i]), C.sizeof(HybridLayer))
+            self.layers[r].kv_lender = self.layers[r].kv_last = -1
+        # a lender's cache covers the windows and the first tokens of all that read it
+        self.lenders = cfg.lenders()
+        self.spans = [(l.attn.window, l.attn.keep) for l in self.layers[: len(runs)]]
+        for r, j in enumerate(self.lenders):
+            if j is not None:
+                self.layers[r].kv_lender, self.layers[j].kv_last = j, r
+                self.layers[r].attn.role, self.layers[j].attn.role = KV_BORROWS, KV_LENDS
+                self.spans[j] = tuple(map(max, self.spans[j], self.spans[r]))
         M = self.m = HybridModel()
         M.n_runs, M.dtype, M.norm_dtype = len(runs), nat.dtype_code(self.dtype), self.norm_dtype
         M.width, M.ldx, M.vocab, M.max_rows = cfg.width, _pad16(cfg.width), cfg.vocab_size, self.max_rows
-        M.eps, M.residual_mult = cfg.eps, cfg.residual_mult
-        M.embed, M.final_norm = ptr(T["embed"]), ptr(T["final.norm"])
-        M.head = self._proj(T["head"])
+        M.eps, M.residual_mult, M.logit_scale = cfg.eps, cfg.residual_mult, cfg.logit_scale
+        M.norm_add = cfg.design.norm_add if self.dtype == torch.bfloat16 else 0.0
+        M.embed, M.final_norm = ptr(T["embed"]), self._norm("final.norm")
+        M.head = self._proj(T["embed" if cfg.design.tied else "head"])
         M.ld_logits = M.head.N
         M.layers = self.layers
         self.n_logits = cfg.vocab_size
@@ -157,11 +199,12 @@ class HybridEngine:
         M.ld_att = max([_pad16(l.out.K) for l in ls], default=16)
         M.proj = ptr(self._buf(R * max([getattr(l, "in").N for l in ls], default=16), self.dtype))
         M.att = ptr(self._buf(R * M.ld_att, self.dtype))
-        M.hid = ptr(self._buf(R * max([l.up.N for l in ls], default=16), self.dtype))
+        f32 = self.dtype == torch.float32
+        M.hid = ptr(self._buf(R * max([l.up.N * (3 if f32 and l.mlp == MLP["geglu"] else 1) for l in ls], default=16), self.dtype))
         if self.dtype == torch.float32:
             M.xn, M.tmp = ptr(self._buf(R * M.ldx, torch.float32)), ptr(self._buf(R * M.ldx, torch.float32))
         else:
-            K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down)])
+            K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down)])  # (K = 0: not there)
             n = int(lib().mi355_linear_gemm_workspace_bytes(R, K))
             M.gemm_ws, M.gemm_ws_bytes = ptr(self._buf(n, torch.uint8)), n
             M.xb = ptr(self._buf(R * M.ldx, torch.bfloat16))
@@ -171,6 +214,20 @@ class HybridEngine:
         n = max([int(lib().mi355_recurrent_scratch_bytes(l.rec.kind, R, 64, l.rec.heads, l.rec.kv_heads, l.rec.dim, l.rec.vdim))
                  for l in ls if l.mixer != 0], default=0)
         M.rec_scratch, M.rec_scratch_bytes = ptr(self._buf(n, torch.uint8)), n
+        n = 0
+        for l in ls:
+            if l.mlp == MLP["experts"]:
+                a = ExpertsArgs.from_buffer_copy(l.moe)
+                a.rows = R
+                n = max(n, int(lib().mi355_experts_scratch_bytes(C.byref(a))))
+        M.moe_scratch, M.moe_scratch_bytes = ptr(self._buf(n, torch.uint8)), n
+        # prepared keys and values of a step's rows, one buffer per lender
+        for r, l in enumerate(ls):
+            if l.mixer == MIX["attention"] and l.attn.role == KV_LENDS:
+                self.layers[r].attn.kv_rows = ptr(self._buf(R * l.attn.kv_heads * (l.attn.dim + l.attn.vdim), self.dtype))
+        for r, j in enumerate(self.lenders):
+            if j is not None:
+                self.layers[r].attn.kv_rows = self.layers[j].attn.kv_rows
         self.logits_buf = self._buf(self.max_logits_rows * M.ld_logits, torch.float32).view(self.max_logits_rows, M.ld_logits)
         # the step's integers: tokens | row0 | count | slot | pos | want, one upload
         self.meta = torch.zeros((6, R), dtype=torch.int32, device=self.device)
@@ -191,9 +248,9 @@ class HybridEngine:
             self.slots.reserve(n_slots)
 
     def _set_len(self, n: int) -> None:
-        """Rings hold min(window, longest sequence) rows.  Growing them re-lays the rings, so no sequence may be live unless every ring
+        """Rings hold min(window, longest sequence) rows (behind the first tokens').  Growing them re-lays the rings, so no sequence may be live unless every ring
         already spans its window."""
-        need = any(l.mixer == 0 and self._ring(l, n) != self._ring(l, self.max_len) for l in list(self.layers)[: self.m.n_runs])
+        need = any(l.mixer == 0 and self._ring(r, n) != self._ring(r, self.max_len) for r, l in enumerate(list(self.layers)[: self.m.n_runs]))
         if need and self.slots.live == 1 and self._single is not None:
             self.reset_cache()  # (what is live is a sequence that generate() or forward() left behind)
         if need and self.max_len and self.slots.live:
@@ -204,9 +261,8 @@ class HybridEngine:
             with torch.cuda.stream(self.stream):
                 self._grow(self.slots.capacity)
 
-    @staticmethod
-    def _ring(l: HybridLayer, max_len: int) -> int:
-        return min(l.attn.window, max(1, max_len))
+    def _ring(self, r: int, max_len: int) -> int:
+        return min(self.spans[r][0], max(1, max_len))
 
     def _grow(self, n: int) -> None:
         self._destroy_graphs()  # captured launches hold the old addresses
@@ -216,10 +272,15 @@ class HybridEngine:
         for r in range(self.m.n_runs):
             l, old = self.layers[r], self.pools[r] or (None, None)
             if l.mixer == 0:
-                a = l.attn
-                a.ring = self._ring(l, self.max_len or 1)
-                k = grown(old[0], (n, a.kv_heads, a.ring, a.dim), self.dtype, dev)
-                v = grown(old[1], (n, a.kv_heads, a.ring, a.vdim), self.dtype, dev)
+                a, j = l.attn, self.lenders[r]
+                if j is not None:
+                    b = self.layers[j].attn
+                    a.ring, a.kept, a.kring, a.vring = b.ring, b.kept, b.kring, b.vring
+                    self.pools[r] = (None, None)
+                    continue
+                a.ring, a.kept = self._ring(r, self.max_len or 1), self.spans[r][1]
+                k = grown(old[0], (n, a.kv_heads, a.kept + a.ring, a.dim), self.dtype, dev)
+                v = grown(old[1], (n, a.kv_heads, a.kept + a.ring, a.vdim), self.dtype, dev)
                 a.kring, a.vring = ptr(k), ptr(v)
                 self.pools[r] = (k, v)
             else:

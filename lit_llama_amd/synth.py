@@ -319,7 +319,9 @@ def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: tor
         leaf = name.split(".", 1)[-1]
         t = torch.randn(shape, generator=gen, device=device, dtype=torch.float32)
         if leaf in ("norm1", "norm2", "norm") or leaf.endswith(".norm"):
-            t = 1.0 + 0.1 * t
+            t = 1.0 - cfg.design.norm_add + 0.1 * t
+        elif leaf.endswith("sink"):
+            t = t + 1.0
         elif leaf.endswith(".conv"):
             t = t * 0.2
             t[:, -1] += 0.7
