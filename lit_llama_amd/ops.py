@@ -620,14 +620,36 @@ class PackedBatch:
 
 def window_attention(proj: torch.Tensor, batch: PackedBatch, kring: torch.Tensor, vring: torch.Tensor, *, heads: int, scale: float, window: int,
                      off_q: int, off_k: int, off_v: int, off_g: int = -1, inv_freq: Optional[torch.Tensor] = None, path: int = 0,
-                     partials: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """mi355_window_attention: proj [rows, ld] (k rotated in place by prompt steps), rings [slots, kv_heads, ring, dim | vdim] (written)."""
+                     partials: Optional[torch.Tensor] = None, keep: int = 0, kept: int = 0, gate_values: bool = False,
+                     unit_eps: Optional[float] = None, sink: Optional[torch.Tensor] = None, role: str = "own",
+                     kv_rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """mi355_window_attention: proj [rows, ld] (k prepared in place by prompt steps), rings [slots, kv_heads, kept + ring, dim | vdim]
+    (written).  `unit_eps`: q and k over their root mean square.  `role` own | lends | borrows: a lender fills `kv_rows` in a prompt step and
+    its cache is written by `window_cache_write`; a borrower has neither key nor value columns."""
+    y, a = _window_args(proj, batch, kring, vring, heads, scale, window, off_q, off_k, off_v, off_g, inv_freq, path, partials, keep, kept,
+                        gate_values, unit_eps, sink, role, kv_rows)
+    check(lib().mi355_window_attention(C.byref(a), C.byref(batch.c), stream_ptr()), "mi355_window_attention")
+    return y
+
+
+def window_cache_write(batch: PackedBatch, kring: torch.Tensor, vring: torch.Tensor, kv_rows: torch.Tensor, kept: int = 0) -> None:
+    """mi355_window_cache_write: the rows a lender left in `kv_rows` enter its cache."""
+    _, a = _window_args(kv_rows, batch, kring, vring, kring.shape[1], 1.0, 1, 0, 0, 0, -1, None, 0, None, 0, kept, False, None, None, "lends", kv_rows)
+    check(lib().mi355_window_cache_write(C.byref(a), C.byref(batch.c), stream_ptr()), "mi355_window_cache_write")
+
+
+def _window_args(proj, batch, kring, vring, heads, scale, window, off_q, off_k, off_v, off_g, inv_freq, path, partials, keep, kept, gate_values,
+                 unit_eps, sink, role, kv_rows):
     require_gpu(proj, "window_attention")
     _, G, ring, dim = kring.shape
+    ring -= kept
     vdim = vring.shape[3]
     assert proj.dim() == 2 and proj.is_contiguous() and kring.is_contiguous() and vring.is_contiguous() and vring.shape[:3] == kring.shape[:3]
     assert proj.shape[0] == batch.rows and proj.dtype == kring.dtype == vring.dtype
-    assert off_q + heads * dim <= proj.shape[1] and off_k + G * dim <= proj.shape[1] and off_v + G * vdim <= proj.shape[1]
+    assert off_q + heads * dim <= proj.shape[1]
+    assert role != "own" or (off_k + G * dim <= proj.shape[1] and off_v + G * vdim <= proj.shape[1])
+    assert off_g < 0 or off_g + (heads * vdim if gate_values else heads) <= proj.shape[1]
+    assert kv_rows is None or (kv_rows.dtype == proj.dtype and kv_rows.is_contiguous() and kv_rows.numel() >= batch.rows * G * (dim + vdim))
     y = torch.zeros((batch.rows, heads * vdim), dtype=proj.dtype, device=proj.device)
     a = nat.WindowAttnArgs()
     a.proj, a.ld, a.dtype = ptr(proj), proj.shape[1], dtype_code(proj.dtype)
@@ -640,8 +662,43 @@ def window_attention(proj: torch.Tensor, batch: PackedBatch, kring: torch.Tensor
     a.kring, a.vring, a.y, a.ldy = ptr(kring), ptr(vring), ptr(y), y.shape[1]
     if partials is not None:
         a.partials, a.partials_bytes = ptr(partials), partials.numel() * partials.element_size()
-    check(lib().mi355_window_attention(C.byref(a), C.byref(batch.c), stream_ptr()), "mi355_window_attention")
-    return y
+    a.keep, a.kept, a.gate_values = keep, kept, int(gate_values)
+    if unit_eps is not None:
+        a.unit_qk, a.unit_eps = 1, unit_eps
+    if sink is not None:
+        assert sink.dtype == torch.float32 and sink.numel() == heads and sink.is_contiguous()
+        a.sink = ptr(sink)
+    a.role, a.kv_rows = ("own", "lends", "borrows").index(role), ptr(kv_rows)
+    return y, a
+
+
+def experts(x: torch.Tensor, norm: torch.Tensor, router: torch.Tensor, weights, shared=None, *, top: int, scale: float, eps: float,
+            norm_add: float = 0.0, alpha: float = 1.0, path: int = 0) -> torch.Tensor:
+    """mi355_experts: x [rows, width] f32 -> x + alpha (experts + shared expert of its RMSNorm).  `weights`: per expert (gate, up, down), `shared`
+    the same or None, all of one dtype (bf16, f32) like `norm` and `router`."""
+    require_gpu(x, "experts")
+    rows, W = x.shape
+    dt = router.dtype
+    ld = (W + 15) // 16 * 16
+    out = torch.zeros((rows, ld), dtype=torch.float32, device=x.device)
+    out[:, :W] = x
+    stream = (lambda w, w1=None: repack_bf16(w, w1, 1 if w1 is None else 2)) if dt == torch.bfloat16 else (
+        lambda w, w1=None: (w if w1 is None else torch.cat([w, w1])).contiguous())
+    keep = [norm.contiguous(), stream(router), torch.stack([stream(g, u) for g, u, _ in weights]), torch.stack([stream(d) for _, _, d in weights])]
+    a = nat.ExpertsArgs()
+    a.dtype, a.rows, a.width, a.experts, a.top = dtype_code(dt), rows, W, router.shape[0], top
+    a.ff, a.scale, a.eps, a.norm_add, a.alpha, a.path = weights[0][0].shape[0], scale, eps, norm_add, alpha, path
+    a.norm, a.norm_dtype = ptr(keep[0]), dtype_code(norm.dtype)
+    a.router, a.up, a.down = (ptr(t) for t in keep[1:4])
+    if shared is not None:
+        keep += [stream(shared[0], shared[1]), stream(shared[2])]
+        a.ff_shared, a.shared_up, a.shared_down = shared[0].shape[0], ptr(keep[4]), ptr(keep[5])
+    a.x, a.ldx = ptr(out), ld
+    n = int(lib().mi355_experts_scratch_bytes(C.byref(a)))
+    scratch = torch.full((n,), 255, dtype=torch.uint8, device=x.device)  # (NaNs in every format: nothing may read what no kernel wrote)
+    a.scratch, a.scratch_bytes = ptr(scratch), n
+    check(lib().mi355_experts(C.byref(a), stream_ptr()), "mi355_experts")
+    return out[:, :W]
 
 
 def recurrent(kind: str, proj: torch.Tensor, batch: PackedBatch, state: torch.Tensor, *, off: dict, kv_heads: int, head_norm: torch.Tensor,
