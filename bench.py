@@ -71,6 +71,8 @@ def parse():
     ap.add_argument("--hybrid", default=None, metavar="WIDTH[,WIDTH]",
                     help="instead of the headline workload: prompt and decode rates of a layered hybrid model (Sekulorn design) of these "
                          "widths beside an unquantised LLaMA of the same width and layer count (random weights)")
+    ap.add_argument("--hybrid-designs", default="Sekulorn", metavar="NAME[,NAME]",
+                    help="the designs of --hybrid (Sekulorn, Kovalorn: width, layers and weights that a token uses per layer are the same)")
     ap.add_argument("--hybrid-layers", type=int, default=8)
     ap.add_argument("--hybrid-batches", default="1,16,64")
     ap.add_argument("--hybrid-only", default="both", choices=["both", "hybrid", "llama"], help="(profiling) one side of --hybrid")
@@ -496,36 +498,37 @@ def hybrid_bench(args, dev) -> dict:
     res = []
     for width in (int(w) for w in args.hybrid.split(",")):
         row = {"width": width, "layers": args.hybrid_layers, "prompt": T}
-        if args.hybrid_only != "llama":
-            conf = synth.hybrid_bench_config(width, args.hybrid_layers)
+        for design in args.hybrid_designs.split(",") if args.hybrid_only != "llama" else ():
+            conf = synth.HYBRID_BENCH[design](width, args.hybrid_layers)
             model = HybridLM(HybridConfig.from_dict(conf), device=dev)
             model.load_state_dict(synth.make_hybrid_state_dict(conf, device=dev))
             eng = model.engine()
             eng.ensure(max(batches), S)
             prompt = torch.randint(0, conf["vocab"], (T,), generator=g).tolist()
             slots = [eng.acquire() for _ in range(max(batches))]
-            for s_ in slots:  # every sequence at position T: decode steps see full windows
-                eng.step([Entry(s_, 0, prompt, [])])
+            for i, s_ in enumerate(slots):  # every sequence at position T: decode steps see full windows (and tokens of their own)
+                eng.step([Entry(s_, 0, prompt[i:] + prompt[:i], [])])
             with torch.cuda.stream(eng.stream):
                 sec = _timed(eng.stream, lambda: eng.step([Entry(slots[0], 0, prompt, [T - 1])]), 4)
             h = {"prefill_ms": round(sec * 1e3, 3), "prefill_tokens_per_s": round(T / sec, 1), "weight_bytes": eng.weight_bytes,
+                 "weight_bytes_of_one_row": eng.weight_bytes_of(1),
                  "state_bytes_per_sequence": eng.state_bytes(), "decode": {}}
             for B in batches:
                 at = [T]
 
                 def one():
-                    eng.step([Entry(s_, at[0], prompt[:1], [0]) for s_ in slots[:B]])
+                    eng.step([Entry(s_, at[0], prompt[i:i + 1], [0]) for i, s_ in enumerate(slots[:B])])
                     at[0] += 1
 
                 one()
                 with torch.cuda.stream(eng.stream):
-                    b, n = eng._upload([Entry(s_, at[0], prompt[:1], [0]) for s_ in slots[:B]])
+                    b, n = eng._upload([Entry(s_, at[0], prompt[i:i + 1], [0]) for i, s_ in enumerate(slots[:B])])
                     # device time of the step itself: the same batch replayed (positions stay, the work of a step does not depend on them)
                     sec = _timed(eng.stream, lambda: eng._run(b, n), steps)
-                weights = eng.weight_bytes / sec
+                weights = eng.weight_bytes_of(B) / sec
                 h["decode"][str(B)] = {"us_per_step": round(sec * 1e6, 1), "tokens_per_s": round(B / sec, 1),
                                        "weight_bytes_frac_of_8TBps": round(weights / 8e12, 4)}
-            row["hybrid"] = h
+            row["hybrid" if design == "Sekulorn" else design] = h
             del model, eng
             torch.cuda.empty_cache()
         if args.hybrid_only != "hybrid":

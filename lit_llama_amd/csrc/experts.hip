@@ -1,7 +1,7 @@
 // Mixture of experts: sigmoid router over the normalised row, the `top` largest scores, their experts' gated feed-forwards (SiLU) summed by
 // weight, and an optional shared expert that every row runs; the sum joins the residual stream.
 //
-//   route_rows_kernel    RMSNorm, router and choice of 16 rows per workgroup (router weights bf16 on the matrix cores, f32 sums)
+//   route_rows_kernel    RMSNorm, router and choice of 1 to 16 rows per workgroup (router weights bf16 on the matrix cores, f32 sums)
 //   few rows (decode):   up_rows_kernel, down_rows_kernel: a workgroup per (row tile, chosen expert, row) / (row tile, row), every weight
 //                        piece read once per row that chose its expert; three launches in all
 //   many rows:           plan_kernel sorts the (row, choice) pairs by expert and cuts them into tiles; grouped_kernel multiplies a tile of up
@@ -15,7 +15,7 @@
 namespace {
 
 constexpr int kMaxExperts = 1024, kMaxTop = 64;
-constexpr int kFewRows = 8;   // rows up to which every (row, choice) pair reads its weights by itself
+constexpr int kFewRows = 2;   // rows up to which every (row, choice) pair reads its weights by itself
 constexpr int kTPW = 2;       // 16-row tile slots per wave of the grouped product
 
 __host__ __device__ __forceinline__ int pad_to(int n, int m) { return (n + m - 1) / m * m; }
@@ -49,125 +49,175 @@ struct Params {
 };
 
 // ------------------------------------------------------------------------------------ router
+// largest value of a wave, in every lane
+__device__ __forceinline__ float wave_top(float v) {
+    v = MI355_DPP_MAX(v, 0xB1);
+    v = MI355_DPP_MAX(v, 0x4E);
+    v = MI355_DPP_MAX(v, 0x141);
+    v = MI355_DPP_MAX(v, 0x140);
+    v = fmaxf(v, lane_xor16(v));
+    return fmaxf(v, lane_xor32(v));
+}
+
 // one wave: the `top` largest of z[0 .. E) (LDS, overwritten; lowest index first among equals), their sigmoids scaled to sum to `scale`
-__device__ void choose(float* z, int E, int top, float scale, int32_t* ids, float* weights) {
+__device__ __forceinline__ void choose(float* z, int E, int top, float scale, int32_t* ids, float* weights) {
     const int lane = threadIdx.x & 63;
     float best = -INFINITY;
-    int bi = 0x7fffffff;
+    int bi = lane < E ? lane : E - 1;  // (rows of NaNs)
     auto scan = [&] {
         best = -INFINITY;
-        bi = 0x7fffffff;
         for (int e = lane; e < E; e += 64) {
             const float v = z[e];
             if (v > best) best = v, bi = e;
         }
     };
     scan();
-    float mine = 0.f, total = 0.f;
+    float mine = -INFINITY;
     int my_id = 0;
     for (int k = 0; k < top; ++k) {
-        float v = best;
-        int i = bi;
-#pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float ov = __shfl_xor(v, o, 64);
-            const int oi = __shfl_xor(i, o, 64);
-            if (ov > v || (ov == v && oi < i)) v = ov, i = oi;
-        }
-        if (i >= E) i = 0;  // (rows of NaNs)
-        const float s = 1.0f / (1.0f + expf(-v));
-        total += s;
-        if (lane == k) mine = s, my_id = i;
+        const float v = wave_top(best);
+        unsigned long long at = __ballot(best == v);
+        if (at == 0) at = 1;
+        int i = __builtin_amdgcn_readlane(bi, __builtin_ctzll(at));
+        for (unsigned long long more = at & (at - 1); more != 0; more &= more - 1) i = min(i, __builtin_amdgcn_readlane(bi, __builtin_ctzll(more)));
+        if (lane == k) mine = v, my_id = i;
         if (lane == (i & 63)) {
             z[i] = -INFINITY;
             scan();
         }
     }
+    const float s = lane < top ? 1.0f / (1.0f + expf(-mine)) : 0.f;
+    const float total = group_sum(s, 64);
     if (lane < top) {
         ids[lane] = my_id;
-        weights[lane] = mine / (total + 1e-20f) * scale;
+        weights[lane] = s / (total + 1e-20f) * scale;
     }
 }
 
-// grid ceil(rows / 16), 512 threads.  LDS: partial logits [8 waves][tiles of a pass][256], logits [16][experts + 1]
-constexpr int kRouteTiles = 8;
+// grid ceil(rows / R), 512 threads; R = 1, 2, 4, 8, 16.  LDS: partial logits [8 waves][tiles of a pass][256], logits [R][experts + 1]
+constexpr int kRouteTiles = 2;
+template <int R>
 __global__ __launch_bounds__(512) void route_rows_kernel(const Params p) {
     const mi355_experts_args& a = p.a;
+    constexpr int kPer = R < 8 ? 8 / R : 1, kRows = R > 8 ? R / 8 : 1;  // waves per row, rows per wave
     extern __shared__ __attribute__((aligned(16))) char smem[];
+    __shared__ float sums[8];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int g = lane >> 4, c = lane & 15;
-    const int row0 = blockIdx.x * 16;
+    const int row0 = blockIdx.x * R;
     const int W = a.width, E = a.experts, tiles = (E + 15) / 16, pass = tiles < kRouteTiles ? tiles : kRouteTiles;
     float* part = (float*)smem;
     float* z = part + 8 * pass * 256;
+    // a wave's first router weights are requested ahead of the norm, the next unit's ahead of a unit's products (past the last tile or unit:
+    // the last one again, not used)
+    const int units = p.kp / 128;
+    const uint8_t* wr = (const uint8_t*)a.router + lane * 16;
+    auto wload = [&](int t, int u, int d) {
+        return *(const bf16x8*)(wr + ((int64_t)(min(t, tiles - 1) * units + min(u, units - 1)) * 4 + d) * 1024);
+    };
+    bf16x8 wn[kRouteTiles][4];
+#pragma unroll
+    for (int t = 0; t < kRouteTiles; ++t)
+#pragma unroll
+        for (int d = 0; d < 4; ++d) wn[t][d] = wload(t, wave, d);
 
-    for (int r = wave; r < 16; r += 8) {
-        const int row = row0 + r;
-        if (row >= a.rows) break;
-        const float* x = a.x + (int64_t)row * a.ldx;
+#pragma unroll
+    for (int i = 0; i < kRows; ++i) {
+        const int row = row0 + wave / kPer + 8 * i, share = wave % kPer;
+        const bool live = row < a.rows;
+        const float* x = a.x + (int64_t)(live ? row : row0) * a.ldx;
         bf16_t* o = p.xn + (int64_t)row * p.kp;
+        const bool vec = W % 4 == 0 && a.norm_dtype == MI355_BF16;
+        constexpr int kHeld = 16 / kPer, kStep = 64 * kPer;  // (rows of 4096; what lies behind is read twice)
+        f32x4 v[kHeld];
+        u32x2 n[kHeld];
         float ss = 0.f;
-        if (W % 4 == 0) {
-            for (int j = lane; j < W / 4; j += 64) {
-                const f32x4 v = ((const f32x4*)x)[j];
-                ss += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+        if (vec) {
+#pragma unroll
+            for (int h = 0; h < kHeld; ++h) {
+                const int j = min(share * 64 + lane + h * kStep, W / 4 - 1);
+                v[h] = ((const f32x4*)x)[j];
+                n[h] = ((const u32x2*)a.norm)[j];
+            }
+#pragma unroll
+            for (int h = 0; h < kHeld; ++h) {
+                const float q = (v[h][0] * v[h][0] + v[h][1] * v[h][1]) + (v[h][2] * v[h][2] + v[h][3] * v[h][3]);
+                ss += share * 64 + lane + h * kStep < W / 4 ? q : 0.f;
+            }
+            for (int j = share * 64 + lane + kHeld * kStep; j < W / 4; j += kStep) {
+                const f32x4 t = ((const f32x4*)x)[j];
+                ss += (t[0] * t[0] + t[1] * t[1]) + (t[2] * t[2] + t[3] * t[3]);
             }
         } else {
-            for (int k = lane; k < W; k += 64) ss += x[k] * x[k];
+            for (int k = share * 64 + lane; k < W; k += kStep) ss += x[k] * x[k];
         }
-        const float rinv = 1.0f / sqrtf(group_sum(ss, 64) / (float)W + a.eps);
-        if (W % 4 == 0 && a.norm_dtype == MI355_BF16) {
-            for (int j = lane; j < p.kp / 4; j += 64) {
-                u32x2 q = {0u, 0u};
-                if (j < W / 4) {
-                    const f32x4 v = ((const f32x4*)x)[j];
-                    const u32x2 n = ((const u32x2*)a.norm)[j];
-                    q[0] = pack2(v[0] * rinv * (a.norm_add + __uint_as_float(n[0] << 16)), v[1] * rinv * (a.norm_add + __uint_as_float(n[0] & 0xffff0000u)));
-                    q[1] = pack2(v[2] * rinv * (a.norm_add + __uint_as_float(n[1] << 16)), v[3] * rinv * (a.norm_add + __uint_as_float(n[1] & 0xffff0000u)));
-                }
-                ((u32x2*)o)[j] = q;
+        ss = group_sum(ss, 64);
+        if constexpr (kPer > 1) {
+            if (lane == 0) sums[wave] = ss;
+            __syncthreads();
+            ss = 0.f;
+#pragma unroll
+            for (int s = 0; s < kPer; ++s) ss += sums[wave / kPer * kPer + s];
+        }
+        const float rinv = 1.0f / sqrtf(ss / (float)W + a.eps);
+        if (live && vec) {
+            auto put = [&](int j, f32x4 t, u32x2 m) {
+                u32x2 q = {pack2(t[0] * rinv * (a.norm_add + __uint_as_float(m[0] << 16)), t[1] * rinv * (a.norm_add + __uint_as_float(m[0] & 0xffff0000u))),
+                           pack2(t[2] * rinv * (a.norm_add + __uint_as_float(m[1] << 16)), t[3] * rinv * (a.norm_add + __uint_as_float(m[1] & 0xffff0000u)))};
+                if (j >= W / 4) q = u32x2{0u, 0u};
+                if (j < p.kp / 4) ((u32x2*)o)[j] = q;
+            };
+#pragma unroll
+            for (int h = 0; h < kHeld; ++h) put(share * 64 + lane + h * kStep, v[h], n[h]);
+            for (int j = share * 64 + lane + kHeld * kStep; j < p.kp / 4; j += kStep) {
+                const int i4 = min(j, W / 4 - 1);
+                put(j, ((const f32x4*)x)[i4], ((const u32x2*)a.norm)[i4]);
             }
-        } else {
-            for (int k = lane; k < p.kp; k += 64) o[k] = k < W ? bf16_hw(x[k] * rinv * (a.norm_add + ld_as_f32(a.norm, k, a.norm_dtype))) : (bf16_t)0;
+        } else if (live) {
+            for (int k = share * 64 + lane; k < p.kp; k += kStep)
+                o[k] = k < W ? bf16_hw(x[k] * rinv * (a.norm_add + ld_as_f32(a.norm, k, a.norm_dtype))) : (bf16_t)0;
         }
     }
     __syncthreads();
-    const int units = p.kp / 128;
-    const int row = row0 + c < a.rows ? row0 + c : a.rows - 1;
+    const int row = min(row0 + c % R, a.rows - 1);
     const bf16_t* xr = p.xn + (int64_t)row * p.kp + 32 * g;
-    const uint8_t* wr = (const uint8_t*)a.router + lane * 16;
     for (int t0 = 0; t0 < tiles; t0 += pass) {
         f32x4 acc[kRouteTiles];
 #pragma unroll
         for (int t = 0; t < kRouteTiles; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
         for (int u = wave; u < units; u += 8) {
-            bf16x8 b[4];
+            bf16x8 b[4], w[kRouteTiles][4];
 #pragma unroll
             for (int d = 0; d < 4; ++d) b[d] = *(const bf16x8*)(xr + u * 128 + 8 * d);
 #pragma unroll
             for (int t = 0; t < kRouteTiles; ++t)
-                if (t < pass && t0 + t < tiles) {
 #pragma unroll
-                    for (int d = 0; d < 4; ++d) {
-                        const bf16x8 w = *(const bf16x8*)(wr + ((int64_t)((t0 + t) * units + u) * 4 + d) * 1024);
-                        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, b[d], acc[t], 0, 0, 0);
-                    }
-                }
+                for (int d = 0; d < 4; ++d) w[t][d] = wn[t][d];
+            const bool more = u + 8 < units;  // (else the next pass begins)
+#pragma unroll
+            for (int t = 0; t < kRouteTiles; ++t)
+#pragma unroll
+                for (int d = 0; d < 4; ++d) wn[t][d] = wload(more ? t0 + t : t0 + pass + t, more ? u + 8 : wave, d);
+#pragma unroll
+            for (int d = 0; d < 4; ++d)
+#pragma unroll
+                for (int t = 0; t < kRouteTiles; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[t][d], b[d], acc[t], 0, 0, 0);
         }
 #pragma unroll
         for (int t = 0; t < kRouteTiles; ++t)
             if (t < pass) *(f32x4*)(part + (wave * pass + t) * 256 + lane * 4) = acc[t];
         __syncthreads();
         for (int i = threadIdx.x; i < pass * 256; i += 512) {
+            const int l = (i & 255) >> 2, e = (t0 + (i >> 8)) * 16 + 4 * (l >> 4) + (i & 3);
+            if ((l & 15) >= R || e >= E) continue;
             float s = 0.f;
 #pragma unroll
             for (int w = 0; w < 8; ++w) s += part[w * pass * 256 + i];
-            const int l = (i & 255) >> 2, e = (t0 + (i >> 8)) * 16 + 4 * (l >> 4) + (i & 3);
-            if (e < E) z[(l & 15) * (E + 1) + e] = s;
+            z[(l & 15) * (E + 1) + e] = s;
         }
         __syncthreads();
     }
-    for (int r = wave; r < 16 && row0 + r < a.rows; r += 8)
+    for (int r = wave; r < R && row0 + r < a.rows; r += 8)
         choose(z + r * (E + 1), E, a.top, a.scale, p.ids + (int64_t)(row0 + r) * a.top, p.weights + (int64_t)(row0 + r) * a.top);
 }
 
@@ -601,6 +651,28 @@ int run_many(Params& p, hipStream_t s) {
     return 0;
 }
 
+template <int R>
+int launch_route(const Params& p, hipStream_t s) {
+    const mi355_experts_args& a = p.a;
+    const int tiles = (a.experts + 15) / 16, pass = tiles < kRouteTiles ? tiles : kRouteTiles;
+    const size_t lds = ((size_t)8 * pass * 256 + R * (a.experts + 1)) * 4;
+    static hipError_t e = hipFuncSetAttribute((const void*)route_rows_kernel<R>, hipFuncAttributeMaxDynamicSharedMemorySize, 144 * 1024);
+    MI355_CHECK_ARG(e == hipSuccess, (int)e, "experts: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
+    hipLaunchKernelGGL(route_rows_kernel<R>, dim3((a.rows + R - 1) / R), dim3(512), lds, s, p);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+
+// rows per workgroup: as few as give every CU one workgroup
+int run_route(const Params& p, hipStream_t s) {
+    const int rows = p.a.rows;
+    if (rows <= 256) return launch_route<1>(p, s);
+    if (rows <= 512) return launch_route<2>(p, s);
+    if (rows <= 1024) return launch_route<4>(p, s);
+    if (rows <= 2048) return launch_route<8>(p, s);
+    return launch_route<16>(p, s);
+}
+
 int run_few(const Params& p, hipStream_t s) {
     const mi355_experts_args& a = p.a;
     const int shared = a.ff_shared > 0, widest = p.fp > p.fsp ? p.fp : p.fsp;
@@ -660,11 +732,6 @@ extern "C" int mi355_experts(const mi355_experts_args* a, mi355_stream_t stream)
                         (int64_t)a->rows * p.kp * 2 < 0xFFFFFFF0ll && (int64_t)((a->ff_shared + 15) / 16) * p.kp * 64 < 0xFFFFFFF0ll &&
                         (int64_t)p.np * p.fsp * 2 < 0xFFFFFFF0ll,
                     MI355_E_SHAPE, "experts: an operand exceeds 4 GiB");
-    const int tiles = (a->experts + 15) / 16, pass = tiles < kRouteTiles ? tiles : kRouteTiles;
-    const size_t lds = ((size_t)8 * pass * 256 + 16 * (a->experts + 1)) * 4;
-    static hipError_t e = hipFuncSetAttribute((const void*)route_rows_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-    MI355_CHECK_ARG(e == hipSuccess, (int)e, "experts: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
-    hipLaunchKernelGGL(route_rows_kernel, dim3((a->rows + 15) / 16), dim3(512), lds, s, p);
-    MI355_LAUNCH_CHECK();
+    if (int rc = run_route(p, s)) return rc;
     return a->path == 1 || (a->path == 0 && a->rows <= kFewRows) ? run_few(p, s) : run_many(p, s);
 }

@@ -76,8 +76,9 @@ struct WinParams {
 };
 
 // ------------------------------------------------------------------------------------ row kernel
-// HT query heads of one key head per workgroup, VE consecutive elements per load (8: 16-B loads of bf16; 1: any head size)
-template <typename T, int HT, int VE>
+// HT query heads of one key head per workgroup, VE consecutive elements per load (8: 16-B loads of bf16; 1: any head size).  FRESH: a decode
+// step, whose keys all lie in the cache but a row's own
+template <typename T, int HT, int VE, bool FRESH>
 __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kernel(const WinParams p) {
     const mi355_window_attn_args& a = p.a;
     extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -94,14 +95,13 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     float* stat = sc + HT * kKeys;                // [3][HT]: maximum, sum, correction
     float* red = stat + 4 * HT;                   // [key lanes][HT][columns]: at most kRowThreads HT VE
     __shared__ int s_seq;
-    __shared__ float s_rms[HT + 1];               // 1 / root mean square of the queries and of the row's own key
 
-    if (!p.fresh) {
+    if constexpr (!FRESH) {
         for (int s = tid; s < p.b.seqs; s += kRowThreads)
             if (row >= p.b.row0[s] && row < p.b.row0[s] + p.b.count[s]) s_seq = s;
         __syncthreads();
     }
-    const int seq = p.fresh ? row : s_seq;
+    const int seq = FRESH ? row : s_seq;
     const int row0 = p.b.row0[seq], pos0 = p.b.pos[seq];
     const int pos = pos0 + (row - row0);
     const T* proj = (const T*)a.proj;
@@ -113,69 +113,76 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     const unsigned ldk = (unsigned)p.ld_rows;
     const T* kcur = (const T*)p.krows + (int64_t)row0 * ldk + (int64_t)kvh * dim;
     const T* vcur = (const T*)p.vrows + (int64_t)row0 * ldk + (int64_t)kvh * vdim;
-    const int cur0 = p.fresh && !p.own ? 0x7fffffff : pos0;  // positions from here on are rows of the step (a borrower's decode step: none)
 
-    // the visible keys, in order: number g < n_first is position g, the others follow from position w0 on; the last is the row's own
+    // The visible keys, in order: number g < n_first is position g, the others follow from position w0 on; the last is the row's own.
+    // Numbers from g_cur on are rows of the step (a prompt's), those before lie in the cache, in three runs: first positions, ring, ring
+    // behind its wrap
     const int n_first = min(a.keep, pos + 1);
     const int w0 = max(pos - a.window + 1, n_first);
     const int n_keys = n_first + pos - w0 + 1;
-    const int r0 = max(w0, a.kept);                               // first of them in the ring
-    const unsigned slot_r0 = (unsigned)(r0 - a.kept) % (unsigned)a.ring;  // (pos - r0 < ring: one wrap at most)
-    auto pos_of = [&](int g) { return g < n_first ? g : w0 + (g - n_first); };
-    auto row_of = [&](int kp) {
-        const unsigned s = slot_r0 + (unsigned)(kp - r0);
-        return kp < a.kept ? (unsigned)kp : (unsigned)a.kept + (s < (unsigned)a.ring ? s : s - a.ring);
-    };
+    const int w_shift = w0 - n_first;                              // position of number g >= n_first, minus g
+    const int w_row = w0 < a.kept ? w0 : a.kept + (w0 - a.kept) % a.ring;
+    const int row_shift = w_row - n_first;
+    const int g_wrap = w0 < a.kept ? 0x7fffffff : n_first + a.kept + a.ring - w_row;  // (the window is no longer than the ring: one wrap at most)
+    const int g_cur = pos0 < n_first ? pos0 : max(n_first, pos0 - w_shift);
+    auto row_of = [&](int g) { return (unsigned)(g < n_first ? g : g < g_wrap ? g + row_shift : g + row_shift - a.ring); };
+    auto step_row = [&](int g) { return (unsigned)((g < n_first ? g : g + w_shift) - pos0); };
     const int step = (n_keys + p.n_split - 1) / p.n_split;
     const int k_begin = split * step, k_end = min(n_keys, k_begin + step);
-    const bool owner = p.own && k_begin < n_keys && k_end == n_keys;  // this split holds the row's own key
+    const bool owner = FRESH && p.own && k_begin < n_keys && k_end == n_keys;  // this split holds the row's own key
 
-    if (a.unit_qk) {  // a wave per head (the last one: the key)
-        for (int h = tid >> 6; h <= HT; h += kRowThreads / 64) {
-            if (h < HT ? h >= nh : !owner) continue;
-            const T* src = h < HT ? prow + a.off_q + (int64_t)(h0 + h) * dim : prow + a.off_k + (int64_t)kvh * dim;
-            float ss = 0.f;
-            for (int d = tid & 63; d < dim; d += 64) {
-                const float v = to_f32<T>(src[d]);
-                ss += v * v;
-            }
-            ss = group_sum(ss, 64);
-            if ((tid & 63) == 0) s_rms[h] = 1.0f / sqrtf(ss / (float)dim + a.unit_eps);
+    // 32 lanes per head, a pair of values each: over the root mean square, rotated, scaled; a decode step's own key likewise (number nh)
+    T* kw = kcache + row_of(n_keys - 1) * (unsigned)dim;
+    const int pairs = (dim + 1) / 2;  // (an odd size: the last pair is one value)
+    for (int h = tid >> 5; h < nh + (owner ? 1 : 0); h += kRowThreads / 32) {
+        const int lane = tid & 31;
+        const bool key = h == nh;
+        const T* src = key ? prow + a.off_k + (int64_t)kvh * dim : prow + a.off_q + (int64_t)(h0 + h) * dim;
+        auto at = [&](int d) { return d < dim ? to_f32<T>(src[d]) : 0.f; };
+        constexpr int kHeld = 2;  // pairs of a lane that are loaded once
+        float v[kHeld][2], ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < kHeld; ++i)
+#pragma unroll
+            for (int e = 0; e < 2; ++e) v[i][e] = at(2 * (lane + 32 * i) + e);
+        float f = key ? 1.f : a.scale;
+        if (a.unit_qk) {
+#pragma unroll
+            for (int i = 0; i < kHeld; ++i) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1];
+            for (int d = 64 * kHeld + lane; d < dim; d += 32) ss += at(d) * at(d);
+            f /= sqrtf(group_sum(ss, 32) / (float)dim + a.unit_eps);
         }
-        __syncthreads();
-    }
-    for (int i = tid; i < nh * dim; i += kRowThreads) {
-        const int h = i / dim, d = i - h * dim;
-        const T* src = prow + a.off_q + (int64_t)(h0 + h) * dim;
-        float v = to_f32<T>(src[d]);
-        if (d < a.rot_dims) {
-            float c, s;
-            pair_cos_sin(pos, a.inv_freq[d >> 1], c, s);
-            const float w = to_f32<T>(src[d ^ 1]);
-            v = (d & 1) ? v * c + w * s : v * c - w * s;
-        }
-        q[h * dim + d] = v * (a.unit_qk ? a.scale * s_rms[h] : a.scale);
-    }
-    if (owner) {
-        T* kw = kcache + (int64_t)row_of(pos) * dim;
-        const T* src = prow + a.off_k + (int64_t)kvh * dim;
-        for (int d = tid; d < dim; d += kRowThreads) {
-            float v = to_f32<T>(src[d]);
-            if (d < a.rot_dims) {
+        auto put = [&](int pi, float u, float w) {
+            if (2 * pi < a.rot_dims) {
                 float c, s;
-                pair_cos_sin(pos, a.inv_freq[d >> 1], c, s);
-                const float w = to_f32<T>(src[d ^ 1]);
-                v = (d & 1) ? v * c + w * s : v * c - w * s;
+                pair_cos_sin(pos, a.inv_freq[pi], c, s);
+                const float r = u * c - w * s;
+                w = w * c + u * s;
+                u = r;
             }
-            const T r = from_f32<T>(a.unit_qk ? v * s_rms[HT] : v);
-            kn[d] = to_f32<T>(r);
-            if (ht == 0) kw[d] = r;
-        }
-        if (ht == 0) {
-            T* vw = vcache + (int64_t)row_of(pos) * vdim;
-            const T* vs = prow + a.off_v + (int64_t)kvh * vdim;
-            for (int d = tid; d < vdim; d += kRowThreads) vw[d] = vs[d];
-        }
+            u *= f, w *= f;
+            if (key) {
+                const T ru = from_f32<T>(u), rw = from_f32<T>(w);
+                kn[2 * pi] = to_f32<T>(ru);
+                if (ht == 0) kw[2 * pi] = ru;
+                if (2 * pi + 1 < dim) {
+                    kn[2 * pi + 1] = to_f32<T>(rw);
+                    if (ht == 0) kw[2 * pi + 1] = rw;
+                }
+            } else {
+                q[h * dim + 2 * pi] = u;
+                if (2 * pi + 1 < dim) q[h * dim + 2 * pi + 1] = w;
+            }
+        };
+#pragma unroll
+        for (int i = 0; i < kHeld; ++i)
+            if (lane + 32 * i < pairs) put(lane + 32 * i, v[i][0], v[i][1]);
+        for (int pi = lane + 32 * kHeld; pi < pairs; pi += 32) put(pi, at(2 * pi), at(2 * pi + 1));
+    }
+    if (owner && ht == 0) {
+        T* vw = vcache + row_of(n_keys - 1) * (unsigned)vdim;
+        const T* vs = prow + a.off_v + (int64_t)kvh * vdim;
+        for (int d = tid; d < vdim; d += kRowThreads) vw[d] = vs[d];
     }
     if (tid < HT) {  // the sink is a key without a value: a score of its own in the first split
         const bool sink = a.sink != nullptr && split == 0 && tid < nh;
@@ -202,8 +209,8 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             const T* src[4];
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
-                const int kk = min(k4 + u * (kRowThreads / 16), nk - 1), kp = pos_of(kb + kk);
-                src[u] = kp >= cur0 ? kcur + (unsigned)(kp - pos0) * ldk : kcache + row_of(kp) * (unsigned)dim;
+                const int g = kb + min(k4 + u * (kRowThreads / 16), nk - 1);
+                src[u] = !FRESH && g >= g_cur ? kcur + step_row(g) * ldk : kcache + row_of(g) * (unsigned)dim;
 #pragma unroll
                 for (int h = 0; h < HT; ++h) dot[u][h] = 0.f;
             }
@@ -227,14 +234,14 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
                 const int kk = k4 + u * (kRowThreads / 16);
 #pragma unroll
                 for (int h = 0; h < HT; ++h) dot[u][h] = group_sum(dot[u][h], 16);
-                if (l16 == 0 && kk < nk && !(p.own && kb + kk == n_keys - 1)) {
+                if (l16 == 0 && kk < nk && !(owner && kb + kk == n_keys - 1)) {
 #pragma unroll
                     for (int h = 0; h < HT; ++h)
                         if (h < nh) sc[kk * HT + h] = dot[u][h];
                 }
             }
         }
-        if (p.own && kb + nk == n_keys && (tid >> 4) < nh) {  // the row's own key, prepared above: lane group h takes head h
+        if (owner && kb + nk == n_keys && (tid >> 4) < nh) {  // the row's own key, prepared above: lane group h takes head h
             const int h = tid >> 4;
             float s = 0.f;
             for (int d = l16; d < dim; d += 16) s += kn[d] * q[h * dim + d];
@@ -272,10 +279,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
 #pragma unroll
                 for (int e = 0; e < VE; ++e) acc[h][e] *= corr;
             }
-#pragma unroll 4
-            for (int kk = kl; kk < nk; kk += n_kl) {
-                const int kp = pos_of(kb + kk);
-                const T* src = kp >= cur0 ? vcur + (unsigned)(kp - pos0) * ldk : vcache + row_of(kp) * (unsigned)vdim;
+            auto add = [&](int kk, const T* src) {
                 float v[VE], w[HT];
 #pragma unroll
                 for (int h = 0; h < HT; ++h) w[h] = sc[kk * HT + h];
@@ -286,6 +290,14 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
 #pragma unroll
                         for (int e = 0; e < VE; ++e) acc[h][e] += w[h] * v[e];
                     }
+            };
+            const int nv = owner && kb + nk == n_keys ? nk - 1 : nk;  // (the own value is not in the cache yet)
+            if (nv < nk && kl == 0) add(nk - 1, prow + a.off_v + (int64_t)kvh * vdim);
+#pragma unroll 4
+            for (int kk = kl; kk < nv; kk += n_kl) {
+                const int g = kb + kk;
+                const T* src = !FRESH && g >= g_cur ? vcur + step_row(g) * ldk : vcache + row_of(g) * (unsigned)vdim;
+                add(kk, src);
             }
         }
         __syncthreads();
@@ -339,59 +351,64 @@ __global__ __launch_bounds__(128) void window_join_kernel(const WinParams p) {
     const T* gates = (const T*)a.proj + (int64_t)row * a.ld + a.off_g;
     float gate = 1.f / group_sum(e * ls, 64);
     if (a.off_g >= 0 && !a.gate_values) gate *= sigmoid_f32(to_f32<T>(gates[h]));
+    float each = 0.f;  // (requested ahead of the records; the loop has one turn unless the values are many)
+    if (a.off_g >= 0 && a.gate_values && (int)threadIdx.x < a.vdim) each = to_f32<T>(gates[h * a.vdim + threadIdx.x]);
     __syncthreads();
     for (int d = threadIdx.x; d < a.vdim; d += blockDim.x) {
         float o = 0.f;
 #pragma unroll 16
         for (int s = 0; s < p.n_split; ++s) o += wgt[s] * rec[s * (a.vdim + 2) + 2 + d];
-        if (a.off_g >= 0 && a.gate_values) o *= sigmoid_f32(to_f32<T>(gates[h * a.vdim + d]));
+        if (a.off_g >= 0 && a.gate_values) o *= sigmoid_f32(d < (int)blockDim.x ? each : to_f32<T>(gates[h * a.vdim + d]));
         ((T*)a.y)[(int64_t)row * a.ldy + (int64_t)h * a.vdim + d] = from_f32<T>(o * gate);
     }
 }
 
 // ------------------------------------------------------------------------------------ prompt steps: keys, cache
-// grid (ceil(max_count / 4), seqs), 256 threads: a wave per row
+// grid (ceil(max_count * kv_heads / 4), seqs), 256 threads: a wave per (row, key head)
 template <typename T>
 __global__ __launch_bounds__(256) void prepare_keys_kernel(const WinParams p) {
     const mi355_window_attn_args& a = p.a;
-    const int seq = blockIdx.y, i = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    const int seq = blockIdx.y, it = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    const int i = it / a.kv_heads, g = it - i * a.kv_heads;
     if (i >= p.b.count[seq]) return;
     const int pos = p.b.pos[seq] + i, half = a.rot_dims / 2;
     const int64_t row = p.b.row0[seq] + i;
     const T* src = (const T*)a.proj + row * a.ld;
-    T* dst = (T*)p.krows + row * p.ld_rows;
     const bool moved = a.role == MI355_KV_LENDS;
-    for (int g = 0; g < a.kv_heads; ++g) {
-        const T* k = src + a.off_k + (int64_t)g * a.dim;
-        T* o = dst + (int64_t)g * a.dim;
-        float rms = 1.f;
-        if (a.unit_qk) {
-            float ss = 0.f;
-            for (int d = lane; d < a.dim; d += 64) {
-                const float v = to_f32<T>(k[d]);
-                ss += v * v;
-            }
-            rms = 1.0f / sqrtf(group_sum(ss, 64) / (float)a.dim + a.unit_eps);
+    const T *k = src + a.off_k + (int64_t)g * a.dim, *v = src + a.off_v + (int64_t)g * a.vdim;
+    T *o = (T*)p.krows + row * p.ld_rows + (int64_t)g * a.dim, *vo = (T*)p.vrows + row * p.ld_rows + (int64_t)g * a.vdim;
+    if (moved)
+        for (int d = lane; d < a.vdim; d += 64) vo[d] = v[d];
+    const int pairs = (a.dim + 1) / 2;  // (an odd size: the last pair is one value)
+    const int p0 = lane < pairs ? lane : pairs - 1;
+    const float k0 = to_f32<T>(k[2 * p0]), k1 = 2 * p0 + 1 < a.dim ? to_f32<T>(k[2 * p0 + 1]) : 0.f;
+    float rms = 1.f;
+    if (a.unit_qk) {
+        float ss = lane < pairs ? k0 * k0 + k1 * k1 : 0.f;
+        for (int d = 128 + lane; d < a.dim; d += 64) {
+            const float u = to_f32<T>(k[d]);
+            ss += u * u;
         }
-        for (int pi = lane; pi < half; pi += 64) {
+        rms = 1.0f / sqrtf(group_sum(ss, 64) / (float)a.dim + a.unit_eps);
+    }
+    for (int pi = lane; pi < pairs; pi += 64) {
+        const bool two = 2 * pi + 1 < a.dim;
+        float u = (pi == lane ? k0 : to_f32<T>(k[2 * pi])) * rms, w = (pi == lane ? k1 : two ? to_f32<T>(k[2 * pi + 1]) : 0.f) * rms;
+        if (pi < half) {
             float c, s;
             pair_cos_sin(pos, a.inv_freq[pi], c, s);
-            const float u = to_f32<T>(k[2 * pi]) * rms, v = to_f32<T>(k[2 * pi + 1]) * rms;
-            o[2 * pi] = from_f32<T>(u * c - v * s);
-            o[2 * pi + 1] = from_f32<T>(v * c + u * s);
+            const float r = u * c - w * s;
+            w = w * c + u * s;
+            u = r;
         }
-        if (a.unit_qk || moved)
-            for (int d = a.rot_dims + lane; d < a.dim; d += 64) o[d] = from_f32<T>(to_f32<T>(k[d]) * rms);
-    }
-    if (moved) {
-        T* vo = (T*)p.vrows + row * p.ld_rows;
-        for (int j = lane; j < a.kv_heads * a.vdim; j += 64) vo[j] = src[a.off_v + j];
+        o[2 * pi] = from_f32<T>(u);
+        if (two) o[2 * pi + 1] = from_f32<T>(w);
     }
 }
 
 // grid (min(max_count, ring) + kept, seqs): the last `ring` rows of every portion, and those of positions below `kept`
 template <typename T>
-__global__ __launch_bounds__(256) void ring_write_kernel(const WinParams p, int n_last) {
+__global__ __launch_bounds__(256) void ring_write_kernel(const WinParams p, int n_last, int vec) {
     const mi355_window_attn_args& a = p.a;
     const int seq = blockIdx.y, cnt = p.b.count[seq], pos0 = p.b.pos[seq];
     const bool first = (int)blockIdx.x >= n_last;
@@ -400,6 +417,17 @@ __global__ __launch_bounds__(256) void ring_write_kernel(const WinParams p, int 
     const int64_t row = p.b.row0[seq] + i, to = cache_row(a, pos0 + i), rows = a.kept + a.ring;
     const T *ks = (const T*)p.krows + row * p.ld_rows, *vs = (const T*)p.vrows + row * p.ld_rows;
     const int64_t base = (int64_t)p.b.slot[seq] * a.kv_heads;
+    if (vec) {  // 16 bytes at a time
+        constexpr int V = 16 / sizeof(T);
+        const int nk = a.kv_heads * a.dim / V, nv = a.kv_heads * a.vdim / V;
+        for (int j = threadIdx.x; j < nk + nv; j += 256) {
+            const bool val = j >= nk;
+            const int e = (val ? j - nk : j) * V, n = val ? a.vdim : a.dim, g = e / n;
+            T* dst = (T*)(val ? a.vring : a.kring) + ((base + g) * rows + to) * n + (e - g * n);
+            *(u32x4*)dst = *(const u32x4*)((val ? vs : ks) + e);
+        }
+        return;
+    }
     for (int j = threadIdx.x; j < a.kv_heads * a.dim; j += 256) {
         const int g = j / a.dim, d = j - g * a.dim;
         ((T*)a.kring)[((base + g) * rows + to) * a.dim + d] = ks[j];
@@ -426,6 +454,9 @@ __device__ __forceinline__ float max3f(float a, float b, float c) {
     float r;
     asm("v_max3_f32 %0, %1, %2, %3" : "=v"(r) : "v"(a), "v"(b), "v"(c));
     return r;
+}
+__device__ __forceinline__ float sigmoid_fast(float z) {  // (in front of a rounding to bf16)
+    return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.44269504088896340736f));
 }
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 
@@ -464,7 +495,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const int q_first = pos0 + qb * kBQ, q_last = pos0 + min(qb * kBQ + kBQ, cnt) - 1;
     // key steps: those of the first `keep` positions that lie in front of the window, then the window's
     const int kb0 = max(0, q_first - a.window + 1) / kBK, kb1 = q_last / kBK + 1;
-    const int n_first = min((a.keep + kBK - 1) / kBK, kb0), n_steps = n_first + kb1 - kb0;
+    const int n_first = min((a.keep + kBK - 1) / kBK, kb0);
     // the wave's own range, for the masks
     const int w_first = min(pos0 + qb * kBQ + wave * 32, pos0 + cnt - 1), w_last = min(w_first + 31, pos0 + cnt - 1);
 
@@ -612,14 +643,14 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
         m_run = a.sink[h] * 1.44269504088896340736f;
         l_run = hh == 0 ? 1.f : 0.f;
     }
-    auto step_of = [&](int it) { return it < n_first ? it : kb0 + (it - n_first); };
+    int kb = n_first > 0 ? 0 : kb0, buf = 0;
 
-    load_tile(step_of(0));
+    load_tile(kb);
     store_tile(0);
     __syncthreads();
-    for (int it = 0; it < n_steps; ++it) {
-        const int kb = step_of(it), buf = it & 1;
-        if (it + 1 < n_steps) load_tile(step_of(it + 1));
+    for (; kb < kb1; buf ^= 1) {
+        const int next = kb + 1 == n_first ? kb0 : kb + 1;
+        if (next < kb1) load_tile(next);
         const char* kt = smem + buf * kKTile;
         const char* vt = smem + 2 * kKTile + buf * kVTile;
         // a wave none of whose queries sees this step leaves it out (it still stages the next tile)
@@ -687,8 +718,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                 }
             }
         }
-        if (it + 1 < n_steps) store_tile(buf ^ 1);
+        if (next < kb1) store_tile(buf ^ 1);
         __syncthreads();
+        kb = next;
     }
     const float l = l_run + lane_xor32(l_run);
     if (q_ok) {
@@ -708,8 +740,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                     for (int e = 0; e < 4; ++e) r[e] = acc[dt][4 * g + e] * inv;
                     if (each) {
                         const u32x2 z = *(const u32x2*)(gates + h * a.vdim + d);
-                        r[0] *= sigmoid_f32(__uint_as_float(z[0] << 16)), r[1] *= sigmoid_f32(__uint_as_float(z[0] & 0xffff0000u));
-                        r[2] *= sigmoid_f32(__uint_as_float(z[1] << 16)), r[3] *= sigmoid_f32(__uint_as_float(z[1] & 0xffff0000u));
+#pragma unroll
+                        for (int e = 0; e < 4; ++e)
+                            r[e] *= sigmoid_fast((e & 1) ? __uint_as_float(z[e >> 1] & 0xffff0000u) : __uint_as_float(z[e >> 1] << 16));
                     }
                     u32x2 o;
                     o[0] = pack_bf16x2(r[0], r[1]);
@@ -750,19 +783,24 @@ int run_tiles(const WinParams& p, hipStream_t s) {
     return launch_tiles<256>(p, s);
 }
 
-template <typename T, int HT, int VE>
-int launch_rows(const WinParams& p, int rows, hipStream_t s) {
+template <typename T, int HT, int VE, bool FRESH>
+int launch_rows_step(const WinParams& p, int rows, hipStream_t s) {
     const size_t red = (size_t)kRowThreads * HT * VE;
     const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + 8 + (size_t)HT * kKeys + 4 * HT + red) * 4;
     MI355_CHECK_ARG(lds <= 160 * 1024 - 64, MI355_E_SHAPE, "window_attention: head size %d does not fit LDS", p.a.dim);
     if (lds > 64 * 1024) {
-        static hipError_t e = hipFuncSetAttribute((const void*)window_rows_kernel<T, HT, VE>, hipFuncAttributeMaxDynamicSharedMemorySize,
+        static hipError_t e = hipFuncSetAttribute((const void*)window_rows_kernel<T, HT, VE, FRESH>, hipFuncAttributeMaxDynamicSharedMemorySize,
                                                   160 * 1024 - 64);
         MI355_CHECK_ARG(e == hipSuccess, (int)e, "window_attention: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
     }
-    hipLaunchKernelGGL((window_rows_kernel<T, HT, VE>), dim3(p.n_split, p.a.kv_heads * p.head_tiles, rows), dim3(kRowThreads), lds, s, p);
+    hipLaunchKernelGGL((window_rows_kernel<T, HT, VE, FRESH>), dim3(p.n_split, p.a.kv_heads * p.head_tiles, rows), dim3(kRowThreads), lds, s, p);
     MI355_LAUNCH_CHECK();
     return 0;
+}
+
+template <typename T, int HT, int VE>
+int launch_rows(const WinParams& p, int rows, hipStream_t s) {
+    return p.fresh ? launch_rows_step<T, HT, VE, true>(p, rows, s) : launch_rows_step<T, HT, VE, false>(p, rows, s);
 }
 
 template <typename T>
@@ -787,7 +825,8 @@ int run_rows(WinParams p, hipStream_t s) {
 template <typename T>
 int run_cache_write(const WinParams& p, hipStream_t s) {
     const int n_last = p.b.max_count < p.a.ring ? p.b.max_count : p.a.ring;
-    hipLaunchKernelGGL(ring_write_kernel<T>, dim3(n_last + p.a.kept, p.b.seqs), dim3(256), 0, s, p, n_last);
+    hipLaunchKernelGGL(ring_write_kernel<T>, dim3(n_last + p.a.kept, p.b.seqs), dim3(256), 0, s, p, n_last,
+                       p.a.dim % 8 == 0 && p.a.vdim % 8 == 0 && rows_aligned(p));
     MI355_LAUNCH_CHECK();
     return 0;
 }
@@ -815,7 +854,7 @@ int run(WinParams p, hipStream_t s) {
         return 0;
     }
     if (a.role == MI355_KV_LENDS || (a.role == MI355_KV_OWN && (a.rot_dims > 0 || a.unit_qk))) {
-        hipLaunchKernelGGL(prepare_keys_kernel<T>, dim3((p.b.max_count + 3) / 4, p.b.seqs), dim3(256), 0, s, p);
+        hipLaunchKernelGGL(prepare_keys_kernel<T>, dim3((unsigned)(((int64_t)p.b.max_count * a.kv_heads + 3) / 4), p.b.seqs), dim3(256), 0, s, p);
         MI355_LAUNCH_CHECK();
     }
     p.n_split = 1;

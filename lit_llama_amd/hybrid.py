@@ -78,10 +78,10 @@ def _attention(m: dict) -> MixerSpec:
 def _sink_attention(m: dict) -> MixerSpec:
     """Attention without rotation: unit queries and keys, first tokens kept, sinks, a gate per value, keys and values of another layer."""
     _only(m, ("heads", "kv_heads", "dim", "vdim", "scale", "mask", "kv_from"), "attention mixer")
-    mask = m.get("mask") or {"size": 1 << 30}
+    mask = m.get("mask") or {}
     _only(mask, ("size", "keep_first"), "mask")
     lender = m.get("kv_from")
-    return MixerSpec("attention", m["heads"], m["kv_heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=int(mask["size"]),
+    return MixerSpec("attention", m["heads"], m["kv_heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=int(mask.get("size") or 1 << 30),
                      keep=int(mask.get("keep_first") or 0), unit_qk=True, sink=True, gate_values=True,
                      kv_from=None if lender is None else int(lender))
 

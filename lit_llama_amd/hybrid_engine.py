@@ -88,14 +88,17 @@ class HybridEngine:
         w = self.weights[name]
         return ptr(w) if self.dtype == torch.bfloat16 or not self.cfg.design.norm_add else self._f32(w.float() + self.cfg.design.norm_add)
 
-    def _experts(self, p: str, f: MlpSpec) -> ExpertsArgs:
+    def _experts(self, i: int, f: MlpSpec) -> ExpertsArgs:
+        p = f"l{i}.mlp."
         T, a = self.weights, ExpertsArgs()
         a.dtype, a.width, a.experts, a.top = nat.dtype_code(self.dtype), self.cfg.width, f.experts, f.top
         a.ff, a.ff_shared, a.scale = f.ff, f.ff_shared, f.scale
         a.router = self._own(self._stream(T[p + "router"]))
         up = [self._stream(T[f"{p}e{e}.gate"], T[f"{p}e{e}.up"]) for e in range(f.experts)]
+        before = self.weight_bytes
         a.up = self._own(torch.stack(up))
         a.down = self._own(torch.stack([self._stream(T[f"{p}e{e}.down"]) for e in range(f.experts)]))
+        self._expert_bytes[i] = (self.weight_bytes - before) / f.experts
         if f.ff_shared:
             a.shared_up = self._own(self._stream(T[p + "shared.gate"], T[p + "shared.up"]))
             a.shared_down = self._own(self._stream(T[p + "shared.down"]))
@@ -109,6 +112,7 @@ class HybridEngine:
     def _pack(self) -> None:
         cfg, T = self.cfg, self.weights
         self.weight_bytes = 0
+        self._expert_bytes: Dict[int, float] = {}
         self.norm_dtype = nat.dtype_code(self.dtype)
         layers = []
         for i, spec in enumerate(cfg.layers):
@@ -129,7 +133,7 @@ class HybridEngine:
             if spec.mlp is not None:
                 L.norm2 = self._norm(p + "norm2")
                 if spec.mlp.kind == "experts":
-                    L.moe = self._experts(p + "mlp.", spec.mlp)
+                    L.moe = self._experts(i, spec.mlp)
                 else:
                     L.up = self._proj(T[p + "mlp.gate"], T[p + "mlp.up"]) if spec.mlp.kind == "geglu" else self._proj(T[p + "mlp.up"])
                     L.down = self._proj(T[p + "mlp.down"])
@@ -296,6 +300,16 @@ class HybridEngine:
     def state_bytes(self) -> int:
         """Bytes of cache and state per slot."""
         return sum(t.numel() * t.element_size() for p in self.pools for t in p if t is not None) // max(1, self.slots.capacity)
+
+    def weight_bytes_of(self, rows: int) -> float:
+        """Bytes of weights that a step of `rows` rows reads, rows choosing their experts independently."""
+        total = float(self.weight_bytes)
+        for i, l in enumerate(self.cfg.layers):
+            f = l.mlp
+            if f is not None and f.kind == "experts":
+                used = f.experts * (1 - (1 - f.top / f.experts) ** rows)
+                total -= (f.experts - used) * self._expert_bytes[i]
+        return total
 
     def acquire(self) -> int:
         """A slot for a new sequence, its recurrent state zeroed."""

@@ -306,6 +306,26 @@ def hybrid_bench_config(width: int, n_layer: int, vocab: int = 32000, window: in
     return {"architecture": "Sekulorn", "layers": layers, "loop": None, "norm": {"eps": 1e-5}, "residual_mult": 1.0, "vocab": vocab, "width": width}
 
 
+def experts_bench_config(width: int, n_layer: int, vocab: int = 32000, window: int = 2048, experts: int = 32, top: int = 6) -> dict:
+    """A Kovalorn configuration whose tokens use about as many weights per layer as a LLaMA of the same width: one dense layer, then mixtures
+    of small experts (an eighth of the LLaMA's hidden size each, the shared one two eighths); every fourth layer lends its keys and values
+    to the three behind it."""
+    heads = width // 128
+    hidden = LLaMAConfig(n_embd=width, n_head=heads).n_hidden
+    ff = (hidden // 8 + 127) // 128 * 128
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "scale": 2.0, "top": top}, "shared": {"ff": 2 * ff}}
+    layers = []
+    for i in range(n_layer):
+        m = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+             "mask": {"size": window if i % 2 == 0 else window // 2, "keep_first": 4}}
+        layers.append({"type": "attention", "mixer": m if i % 4 == 0 else {**m, "kv_from": i - i % 4},
+                       "mlp": {"kind": "dense", "ff": hidden} if i == 0 else moe})
+    return {"architecture": "Kovalorn", "layers": layers, "norm": {"eps": 1e-5}, "logit_scale": 0.25, "vocab": vocab, "width": width}
+
+
+HYBRID_BENCH = {"Sekulorn": hybrid_bench_config, "Kovalorn": experts_bench_config}
+
+
 def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: torch.dtype = torch.bfloat16, rank: int = 16):
     """Random weights of a hybrid configuration: unit-gain projections, decays around 0.9, so that far tokens still count."""
     from .hybrid import HybridConfig, tensor_shapes
