@@ -35,7 +35,7 @@ enum { MI355_E_ARG = -1, MI355_E_SHAPE = -2, MI355_E_DTYPE = -3, MI355_E_STATE =
 enum { MI355_W_Q4 = 0, MI355_W_BF16 = 1, MI355_W_I8 = 2 };
 /* epilogues of the fast linear */
 /* (GEGLU: the pair stream with the tanh form of GELU instead of SiLU; BF16 streams only) */
-enum { MI355_EPI_STORE = 0, MI355_EPI_ACCUM = 1, MI355_EPI_SWIGLU = 2, MI355_EPI_GEGLU = 3 };
+enum { MI355_EPI_STORE = 0, MI355_EPI_ACCUM = 1, MI355_EPI_SWIGLU = 2, MI355_EPI_GEGLU = 3, MI355_EPI_CLAMPGLU = 4 };
 /* bits of mi355_linear_args.flags: STORE writes max(y, 0)^2; the norm's scale is 1 + norm_scale */
 enum { MI355_LF_RELU2 = 1, MI355_LF_NORM_ONE = 2 };
 
@@ -133,6 +133,10 @@ typedef struct mi355_linear_args {
     int32_t attn_heads;
     int32_t attn_hs;
     float alpha;        /* factor of the product, in front of the epilogue; 0 is read as 1 */
+    float limit;        /* CLAMPGLU: bound of both halves */
+    int32_t slice_rows; /* mi355_linear_gemm, BF16 STORE: != 0: output rows [i slice_rows, (i + 1) slice_rows) read the operand slice_stride i
+                         * elements behind x (whole row blocks: slice_rows % 256 == 0; bf16 operands of whole units) */
+    int64_t slice_stride;
     /* optional profiling aid: uint64 [grid][8] wall-clock stamps (100 MHz) written by wave 0 of every workgroup:
      * 0 entry, 1 ring issued, 2 activations staged, 3 first tile's loop done, 4 first epilogue done, 5 exit */
     uint64_t* debug_stamps;
@@ -625,7 +629,7 @@ typedef struct mi355_seq_batch {
     int32_t rows;          /* rows of the step */
     int32_t seqs;
     int32_t max_count;     /* largest count[] (1: a decode step) */
-    int32_t reserved0;
+    int32_t max_end;       /* prompt steps: largest pos[] + count[] (read by latent attention; 0: not known) */
     const int32_t* row0;   /* device [seqs] */
     const int32_t* count;  /* device [seqs] */
     const int32_t* slot;   /* device [seqs] */
@@ -638,8 +642,9 @@ typedef struct mi355_seq_batch {
  * sequence).
  * role: a layer that LENDS its keys and values leaves a prompt step's prepared rows in kv_rows, and its cache rows are written
  * by mi355_window_cache_write behind its last borrower; a layer that BORROWS has the lender's rings (and kept, ring, kv_rows) and
- * no key / value columns.  Lender and borrowers may differ in window and keep: kept and ring cover all of them. */
-enum { MI355_KV_OWN = 0, MI355_KV_LENDS = 1, MI355_KV_BORROWS = 2 };
+ * no key / value columns.  Lender and borrowers may differ in window and keep: kept and ring cover all of them.
+ * A layer with role MI355_KV_ROWS has no cache of its own kind: a prompt step finds the keys and values of every position in kv_rows. */
+enum { MI355_KV_OWN = 0, MI355_KV_LENDS = 1, MI355_KV_BORROWS = 2, MI355_KV_ROWS = 3 };
 typedef struct mi355_window_attn_args {
     void* proj;            /* [rows, ld]: q, k, v, gate columns; a prompt step normalises and rotates k IN PLACE (role 0) */
     int64_t ld;
@@ -663,8 +668,18 @@ typedef struct mi355_window_attn_args {
     float unit_eps;
     const float* sink;     /* [heads]: exp(sink) joins the sum of every softmax, or NULL */
     int32_t role;          /* MI355_KV_* */
-    int32_t reserved0;
+    int32_t chunked;       /* != 0: row i sees rows j <= i of its own chunk of `window` positions, counted from position 0 */
     void* kv_rows;         /* [rows][kv_heads * dim | kv_heads * vdim] of dtype, lender and borrowers */
+    const float* head_scale; /* [heads]: one more factor of a head's scores, or NULL */
+    const float* slope;    /* [heads]: slope * (i - j) is taken off a head's scores, or NULL */
+    int32_t unit_v;        /* != 0: values are divided by their root mean square (unit_eps), and cached so */
+    int32_t rot_at;        /* first rotated dimension of a head */
+    int64_t rows_per_seq;  /* role MI355_KV_ROWS: position p of sequence s is row s * rows_per_seq + p of kv_rows (pitch ld_rows) */
+    int64_t ld_rows;
+    int32_t off_v_rows;    /* MI355_KV_ROWS: first value column of kv_rows */
+    int32_t tail_dims;     /* MI355_KV_ROWS: the last tail_dims dimensions of every key are those of key_tail, the same for all heads */
+    const void* key_tail;  /* position p of slot t at t * tail_slot + p * ld_tail */
+    int64_t ld_tail, tail_slot;
 } mi355_window_attn_args;
 
 int mi355_window_attention(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
@@ -675,19 +690,20 @@ int mi355_window_cache_write(const mi355_window_attn_args* a, const mi355_seq_ba
  *   kind MI355_REC_DELTA  gated delta rule: short causal convolutions + SiLU on q, k, v; unit q, k; S = g S, u = beta (v - S^T k),
  *                         S += k u^T, o = S^T q with g = exp(-exp(A_log) softplus(a + dt_bias)), beta = sigmoid(b)
  *   kind MI355_REC_GLA    S = diag(alpha) S + k v^T, o = S^T q with alpha = sigmoid(a2 a1 + a2_bias)^(1 / tau) per key channel
+ *   kind MI355_REC_WKV    o = (S + diag(u) k v^T)^T q, then S = diag(w) S + k v^T with w = exp(-exp(a2 tanh(a1) + a2_bias)) per key channel
  * then per head o / rms(o) * head_norm * silu(g). */
-enum { MI355_REC_DELTA = 0, MI355_REC_GLA = 1 };
+enum { MI355_REC_DELTA = 0, MI355_REC_GLA = 1, MI355_REC_WKV = 2 };
 typedef struct mi355_recurrent_args {
     int32_t kind;
     int32_t dtype;         /* of proj, conv_ring and y */
     const void* proj;      /* [rows, ld] */
     int64_t ld;
     int32_t heads, kv_heads, dim, vdim;
-    int32_t off_q, off_k, off_v, off_g, off_a, off_b; /* off_a: DELTA decay input [heads], GLA low-rank input [rank]; off_b: DELTA only */
-    float q_scale;         /* dim^-1/2 */
+    int32_t off_q, off_k, off_v, off_g, off_a, off_b; /* off_a: DELTA decay input [heads], GLA / WKV low-rank input [rank]; off_b: DELTA only */
+    float q_scale;         /* factor of q */
     float eps;             /* of the output norm */
     int32_t taps;          /* DELTA: convolution taps */
-    int32_t rank;          /* GLA */
+    int32_t rank;          /* GLA, WKV */
     float inv_tau;         /* GLA */
     float unit_eps;        /* DELTA */
     const float* conv_q;   /* [kv_heads * dim][taps], last tap = the current row */
@@ -697,7 +713,7 @@ typedef struct mi355_recurrent_args {
     const float* dt_bias;  /* [heads] */
     const float* a2;       /* [heads * dim][rank] */
     const float* a2_bias;  /* [heads * dim] */
-    const float* head_norm; /* [vdim] */
+    const float* head_norm; /* [vdim], or head h's at h * norm_ld */
     float* state;          /* [slots][heads][dim][vdim] */
     void* conv_ring;       /* [slots][taps][2 * kv_heads * dim + heads * vdim]: raw q | k | v inputs, position p in row p % taps */
     void* y;               /* [rows, ldy], head h at column h * vdim */
@@ -705,12 +721,60 @@ typedef struct mi355_recurrent_args {
     float* scratch;        /* chunked prompt steps, or NULL */
     uint64_t scratch_bytes;
     int32_t path;          /* 0: by shape; 1: row by row; 2: chunks */
-    int32_t reserved0;
+    int32_t norm_ld;       /* 0: the heads share head_norm */
+    const float* bonus;    /* WKV: u [heads * dim] */
 } mi355_recurrent_args;
 
 int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
 /* scratch bytes a chunked prompt step of `rows` rows in `seqs` sequences takes; 0: the shape runs row by row */
 size_t mi355_recurrent_scratch_bytes(int kind, int rows, int seqs, int heads, int kv_heads, int dim, int vdim);
+
+/* A weight of a hybrid model: BF16 stream (mi355_bf16_repack, R = 1) of a bf16 model, row-major f32 of an f32 model */
+typedef struct mi355_proj {
+    const void* w;
+    int32_t N, K;
+} mi355_proj;
+
+/* Causal attention whose keys and values are products with one latent row per position: q = uq (c_q / rms(c_q) * q_norm), per head
+ * [dim | rot_dim rotated]; c = c / rms(c) * c_norm; k = [uk c | the rotated tail, shared by all heads], v = uv c; scores (q . k) * scale,
+ * exp(sink) joins the sum.  A slot's cache is one row [c | tail] per position.
+ * Decode steps and short portions run on the latents: q . uk c = (uk^T q) . c and sum of w v = uv (sum of w c).  Long portions of bf16
+ * models expand the keys and values of every position of their sequences (expand, kv_rows) and run on the tiles of mi355_window_attention. */
+typedef struct mi355_latent_args {
+    const void* proj;      /* [rows, ld]: c_q at off_q, [c | tail] at off_c */
+    int64_t ld;
+    int32_t dtype;         /* of proj, cache, y and the weights */
+    int32_t heads, dim, rot_dim, vdim;
+    int32_t q_rank, kv_rank;
+    int32_t off_q, off_c;
+    float scale, eps;
+    int32_t cache_rows;    /* positions a slot holds */
+    const float* q_norm;   /* [q_rank] */
+    const float* c_norm;   /* [kv_rank] */
+    const double* inv_freq; /* device [rot_dim / 2]: pair (2i, 2i + 1) turns by position * inv_freq[i] */
+    const float* sink;     /* [heads] */
+    mi355_proj uq;         /* [heads * (dim + rot_dim), q_rank] */
+    mi355_proj expand;     /* BF16: uk (rows padded to a multiple of 16), then uv, [.., kv_rank] */
+    const void* uk_t;      /* [heads][kv_rank][dim] row-major */
+    const void* uv;        /* [heads][vdim][kv_rank] row-major */
+    void* cache;           /* [slots][cache_rows][kv_rank + rot_dim] */
+    void* y;               /* [rows, ldy], head h at column h * vdim */
+    int64_t ldy;
+    void* cq;              /* [rows][q_rank padded to 128] of dtype */
+    void* q;               /* [rows][uq.N] */
+    void* qa;              /* [rows][heads][kv_rank + rot_dim] */
+    float* partials;       /* softmax records of the key splits */
+    uint64_t partials_bytes;
+    void* rows_c;          /* BF16: [expand_rows][kv_rank padded to 128] */
+    void* kv_rows;         /* BF16: [expand_rows][expand.N] */
+    int64_t expand_rows;   /* >= cache_rows for the tile path */
+    void* gemm_ws;
+    uint64_t gemm_ws_bytes;
+    int32_t path;          /* 0: by shape; 1: one workgroup per row and head; 2: matrix cores on the latents; 3: expanded tiles */
+    int32_t reserved0;
+} mi355_latent_args;
+
+int mi355_latent_attention(const mi355_latent_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
 
 /* Mixture of experts behind an RMSNorm: x += alpha (sum over the `top` experts with the largest s_e = sigmoid(router_e . h) of
  * s_e / (their sum + 1e-20) * scale * expert_e(h)  +  shared(h)),  expert(h) = down (silu(gate h) * (up h)).
@@ -746,16 +810,11 @@ int mi355_experts(const mi355_experts_args* a, mi355_stream_t stream);
 /* scratch bytes of a step (dtype, rows, width, experts, top, ff, ff_shared are read) */
 size_t mi355_experts_scratch_bytes(const mi355_experts_args* a);
 
-/* A weight of a hybrid model: BF16 stream (mi355_bf16_repack, R = 1) of a bf16 model, row-major f32 of an f32 model */
-typedef struct mi355_proj {
-    const void* w;
-    int32_t N, K;
-} mi355_proj;
 
-enum { MI355_MIX_ATTENTION = 0, MI355_MIX_DELTA = 1, MI355_MIX_GLA = 2 };
+enum { MI355_MIX_ATTENTION = 0, MI355_MIX_DELTA = 1, MI355_MIX_GLA = 2, MI355_MIX_WKV = 3, MI355_MIX_LATENT = 4 };
 /* feed-forwards: down relu(up h)^2; down (gelu_tanh(gate h) * (up h)), `up` the pair (BF16 pair stream, or f32 gate rows then up rows;
- * up.N = the hidden size); mixture of experts */
-enum { MI355_MLP_NONE = 0, MI355_MLP_RELU2 = 1, MI355_MLP_GEGLU = 2, MI355_MLP_EXPERTS = 3 };
+ * up.N = the hidden size); mixture of experts; down (g sigmoid(1.702 g) (u + 1)) with g = min(gate h, limit), u = clamp(up h, -limit, limit) */
+enum { MI355_MLP_NONE = 0, MI355_MLP_RELU2 = 1, MI355_MLP_GEGLU = 2, MI355_MLP_EXPERTS = 3, MI355_MLP_CLAMPGLU = 4 };
 /* one RUN of a layer (a looped layer appears once per pass: same weights, its own cache / state) */
 typedef struct mi355_hybrid_layer {
     int32_t mixer;         /* MI355_MIX_* */
@@ -770,6 +829,21 @@ typedef struct mi355_hybrid_layer {
     mi355_experts_args moe;        /* weights, sizes and scale */
     int32_t kv_lender;     /* run whose cache this run's attention reads (role MI355_KV_BORROWS) */
     int32_t kv_last;       /* of a lender: its last borrower's run */
+    mi355_latent_args latent;
+    /* A PARALLEL layer: x += mixer(h) + ff(h), h = norm1(x).  Mixer output and hidden row lie side by side in `cat` (bf16 models: pitch
+     * ld_cat a multiple of 128, what lies between and behind them stays zero), so that `out` is one product over both. */
+    int32_t parallel;
+    int32_t hid_at;        /* first hidden column of cat */
+    void* cat;             /* [max_rows, ld_cat] of dtype */
+    int64_t ld_cat;
+    float limit;           /* CLAMPGLU */
+    /* token shift (n_mix > 0): input column block i is the product of mix_w[i] with h + (h' - h) mu[i], h' the row before (0 in front of the first) */
+    int32_t n_mix;
+    const float* mu;       /* [n_mix][width] */
+    float* shift;          /* [slots][width]: h of a sequence's last row */
+    mi355_proj mix_w[5];
+    int32_t mix_at[5];     /* its first column of proj */
+    int32_t mix_stacked;   /* bf16: the first mix_stacked weights are one stream of equal parts, mix_w[0] */
 } mi355_hybrid_layer;
 
 typedef struct mi355_hybrid_model {
@@ -785,17 +859,20 @@ typedef struct mi355_hybrid_model {
     float residual_mult;
     float norm_add;        /* the norms' scales are norm_add + their weights; 0, or 1 in bf16 models */
     float logit_scale;
+    int32_t norm_groups;   /* parallel layers and the final norm in front of them: parts of a row that are normalised by themselves; 0: RMSNorm */
+    int32_t ld_n;          /* row pitch of xn and xb (width padded to 128) */
     const void* embed;     /* [vocab, width] of dtype */
     const void* final_norm;
     mi355_proj head;
     const mi355_hybrid_layer* layers;
     float* x;              /* [max_rows, ldx] residual stream */
     float* xw;             /* [max_rows, ldx] rows whose logits are wanted */
-    float* xn;             /* [max_rows, ldx] f32 models: normalised rows */
-    uint16_t* xb;          /* [max_rows, ldx] bf16 models: normalised rows of a wide product */
+    float* xn;             /* [max_rows, ld_n] f32 models: normalised rows */
+    uint16_t* xb;          /* [max_rows, ld_n] bf16 models: normalised rows of a wide product or of a parallel layer */
+    void* mix;             /* [5][max_rows][ld_n] of dtype: the shifted mixes of a parallel layer */
     void* proj;            /* [max_rows, widest in.N] of dtype */
     void* att;             /* [max_rows, widest out.K padded to 16] of dtype */
-    void* hid;             /* [max_rows, widest up.N (f32 GEGLU: 3 up.N)] of dtype */
+    void* hid;             /* [max_rows, widest up.N (f32 pairs: 3 up.N)] of dtype */
     float* tmp;            /* [max_rows, ldx] f32 models: a product in front of its residual */
     int64_t ld_att;
     void* gemm_ws;
@@ -812,7 +889,7 @@ typedef struct mi355_hybrid_model {
  * run_end < n_runs stops behind that many runs without logits (x holds the residual stream). */
 int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq_batch* b, const int32_t* tokens, const int32_t* want,
                          int n_want, float* logits, int run_end, mi355_stream_t stream);
-/* zero the state of `n` slots (device list) in every recurrent run */
+/* zero the state of `n` slots (device list) in every recurrent run and token shift */
 int mi355_hybrid_reset_slots(const mi355_hybrid_model* m, const int32_t* slots, int n, mi355_stream_t stream);
 /* greedy end of a decode step, one row per sequence: next[b] = tokens[b] = argmax(logits[b]), out[b * ld_out + pos[b] + 1] = it
  * (out may be NULL), pos[b] += 1 */

@@ -19,7 +19,7 @@ CORE_LIB = PKG / "libmi355core.so"
 OBJ_DIR = PKG / "csrc" / "_obj"
 # what a layered hybrid model runs on; linked alone into CORE_LIB where only such a model is served
 CORE_SOURCES = ["generic.hip", "gemv.hip", "gemm.hip", "sample.hip", "graph.hip", "window_attention.hip", "recurrent.hip",
-                "recurrent_chunks.hip", "experts.hip", "hybrid.hip"]
+                "recurrent_chunks.hip", "latent_attention.hip", "experts.hip", "hybrid.hip"]
 SOURCES = CORE_SOURCES + ["int8.hip", "int8_gemm.hip", "attention.hip", "engine.hip", "gptq.hip", "fused_step.hip", "fused_step_ring.hip",
                           "fused_step_wide.hip", "tp_comm.hip", "flash_prefill.hip"]
 ARCH = "gfx950"
@@ -51,7 +51,7 @@ def build(force: bool = False, verbose: bool = True, sources=None, lib: Path = L
     sources = SOURCES if sources is None else sources
     hipcc = _hipcc()
     OBJ_DIR.mkdir(exist_ok=True)
-    headers = [CSRC / "common.h", CSRC / "fused_step_common.h", CSRC / "gemm_fuse.h", CSRC / "recurrent.h", PKG.parent / "include" / "mi355_llama.h"]
+    headers = [CSRC / "common.h", CSRC / "fused_step_common.h", CSRC / "gemm_fuse.h", CSRC / "recurrent.h", CSRC / "product.h", PKG.parent / "include" / "mi355_llama.h"]
     flags = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", *NO_PACKED_F32]
 
     def compile_one(name: str):

@@ -18,7 +18,7 @@ CORE_LIB_PATH = _PKG / "libmi355core.so"  # the part a layered hybrid model need
 
 F32, BF16, F16 = 0, 1, 2
 W_Q4, W_BF16, W_I8 = 0, 1, 2
-EPI_STORE, EPI_ACCUM, EPI_SWIGLU, EPI_GEGLU = 0, 1, 2, 3
+EPI_STORE, EPI_ACCUM, EPI_SWIGLU, EPI_GEGLU, EPI_CLAMPGLU = 0, 1, 2, 3, 4
 LF_RELU2, LF_NORM_ONE = 1, 2
 
 _DTYPE_CODE = {torch.float32: F32, torch.bfloat16: BF16, torch.float16: F16}
@@ -40,7 +40,7 @@ class LinearArgs(C.Structure):
         ("y", c_void_p), ("y_dtype", c_int32), ("group_cols", c_int32), ("ldy", c_int64),
         ("waves", c_int32), ("grid", c_int32), ("prefetch", c_int32), ("flags", c_int32),
         ("attn_partials", c_void_p), ("attn_splits", c_int32), ("attn_heads", c_int32), ("attn_hs", c_int32),
-        ("alpha", c_float), ("debug_stamps", c_void_p),
+        ("alpha", c_float), ("limit", c_float), ("slice_rows", c_int32), ("slice_stride", c_int64), ("debug_stamps", c_void_p),
     ]
 
 
@@ -142,7 +142,7 @@ class TpComm(C.Structure):
 
 class SeqBatch(C.Structure):
     _fields_ = [
-        ("rows", c_int32), ("seqs", c_int32), ("max_count", c_int32), ("reserved0", c_int32),
+        ("rows", c_int32), ("seqs", c_int32), ("max_count", c_int32), ("max_end", c_int32),
         ("row0", c_void_p), ("count", c_void_p), ("slot", c_void_p), ("pos", c_void_p),
     ]
 
@@ -156,7 +156,9 @@ class WindowAttnArgs(C.Structure):
         ("kring", c_void_p), ("vring", c_void_p), ("y", c_void_p), ("ldy", c_int64),
         ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("path", c_int32),
         ("keep", c_int32), ("kept", c_int32), ("gate_values", c_int32), ("unit_qk", c_int32), ("unit_eps", c_float), ("sink", c_void_p),
-        ("role", c_int32), ("reserved0", c_int32), ("kv_rows", c_void_p),
+        ("role", c_int32), ("chunked", c_int32), ("kv_rows", c_void_p),
+        ("head_scale", c_void_p), ("slope", c_void_p), ("unit_v", c_int32), ("rot_at", c_int32), ("rows_per_seq", c_int64), ("ld_rows", c_int64),
+        ("off_v_rows", c_int32), ("tail_dims", c_int32), ("key_tail", c_void_p), ("ld_tail", c_int64), ("tail_slot", c_int64),
     ]
 
 
@@ -169,7 +171,7 @@ class RecurrentArgs(C.Structure):
         ("conv_q", c_void_p), ("conv_k", c_void_p), ("conv_v", c_void_p), ("a_log", c_void_p), ("dt_bias", c_void_p),
         ("a2", c_void_p), ("a2_bias", c_void_p), ("head_norm", c_void_p), ("state", c_void_p), ("conv_ring", c_void_p),
         ("y", c_void_p), ("ldy", c_int64), ("scratch", c_void_p), ("scratch_bytes", C.c_uint64),
-        ("path", c_int32), ("reserved0", c_int32),
+        ("path", c_int32), ("norm_ld", c_int32), ("bonus", c_void_p),
     ]
 
 
@@ -187,11 +189,25 @@ class Proj(C.Structure):
     _fields_ = [("w", c_void_p), ("N", c_int32), ("K", c_int32)]
 
 
+class LatentArgs(C.Structure):
+    _fields_ = [
+        ("proj", c_void_p), ("ld", c_int64), ("dtype", c_int32), ("heads", c_int32), ("dim", c_int32), ("rot_dim", c_int32), ("vdim", c_int32),
+        ("q_rank", c_int32), ("kv_rank", c_int32), ("off_q", c_int32), ("off_c", c_int32), ("scale", c_float), ("eps", c_float),
+        ("cache_rows", c_int32), ("q_norm", c_void_p), ("c_norm", c_void_p), ("inv_freq", c_void_p), ("sink", c_void_p),
+        ("uq", Proj), ("expand", Proj), ("uk_t", c_void_p), ("uv", c_void_p), ("cache", c_void_p), ("y", c_void_p), ("ldy", c_int64),
+        ("cq", c_void_p), ("q", c_void_p), ("qa", c_void_p), ("partials", c_void_p), ("partials_bytes", C.c_uint64),
+        ("rows_c", c_void_p), ("kv_rows", c_void_p), ("expand_rows", c_int64), ("gemm_ws", c_void_p), ("gemm_ws_bytes", C.c_uint64),
+        ("path", c_int32), ("reserved0", c_int32),
+    ]
+
+
 class HybridLayer(C.Structure):
     _fields_ = [
         ("mixer", c_int32), ("mlp", c_int32), ("norm1", c_void_p), ("norm2", c_void_p),
         ("in", Proj), ("out", Proj), ("up", Proj), ("down", Proj),
         ("attn", WindowAttnArgs), ("rec", RecurrentArgs), ("moe", ExpertsArgs), ("kv_lender", c_int32), ("kv_last", c_int32),
+        ("latent", LatentArgs), ("parallel", c_int32), ("hid_at", c_int32), ("cat", c_void_p), ("ld_cat", c_int64), ("limit", c_float),
+        ("n_mix", c_int32), ("mu", c_void_p), ("shift", c_void_p), ("mix_w", Proj * 5), ("mix_at", c_int32 * 5), ("mix_stacked", c_int32),
     ]
 
 
@@ -200,8 +216,9 @@ class HybridModel(C.Structure):
         ("n_runs", c_int32), ("dtype", c_int32), ("norm_dtype", c_int32), ("width", c_int32),
         ("ldx", c_int32), ("vocab", c_int32), ("max_rows", c_int32), ("ld_logits", c_int32),
         ("eps", c_float), ("residual_mult", c_float), ("norm_add", c_float), ("logit_scale", c_float),
+        ("norm_groups", c_int32), ("ld_n", c_int32),
         ("embed", c_void_p), ("final_norm", c_void_p), ("head", Proj), ("layers", C.POINTER(HybridLayer)),
-        ("x", c_void_p), ("xw", c_void_p), ("xn", c_void_p), ("xb", c_void_p), ("proj", c_void_p), ("att", c_void_p), ("hid", c_void_p),
+        ("x", c_void_p), ("xw", c_void_p), ("xn", c_void_p), ("xb", c_void_p), ("mix", c_void_p), ("proj", c_void_p), ("att", c_void_p), ("hid", c_void_p),
         ("tmp", c_void_p), ("ld_att", c_int64), ("gemm_ws", c_void_p), ("gemm_ws_bytes", C.c_uint64),
         ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("rec_scratch", c_void_p), ("rec_scratch_bytes", C.c_uint64),
         ("moe_scratch", c_void_p), ("moe_scratch_bytes", C.c_uint64),
@@ -275,6 +292,7 @@ PROTOTYPES = {
     "mi355_debug_time_next_launch": (c_int, [c_void_p, c_void_p]),
     "mi355_window_attention": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_window_cache_write": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
+    "mi355_latent_attention": (c_int, [C.POINTER(LatentArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_experts": (c_int, [C.POINTER(ExpertsArgs), c_void_p]),
     "mi355_experts_scratch_bytes": (c_size_t, [C.POINTER(ExpertsArgs)]),
     "mi355_recurrent": (c_int, [C.POINTER(RecurrentArgs), C.POINTER(SeqBatch), c_void_p]),
@@ -288,7 +306,7 @@ PROTOTYPES = {
 }
 
 ABI_STRUCTS = [LinearArgs, AttnArgs, Int8Args, Weight, Layer, Model, FusedStepArgs, TpComm,
-               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel, ExpertsArgs]
+               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel, ExpertsArgs, LatentArgs]
 
 _lib: Optional[C.CDLL] = None
 

@@ -185,9 +185,15 @@ __device__ __forceinline__ float gelu_tanh_f32(float z) {
 }
 
 // epilogues over a pair stream, and what they store
-constexpr bool is_pair_epi(int epi) { return epi == MI355_EPI_SWIGLU || epi == MI355_EPI_GEGLU; }
+constexpr bool is_pair_epi(int epi) { return epi == MI355_EPI_SWIGLU || epi == MI355_EPI_GEGLU || epi == MI355_EPI_CLAMPGLU; }
+// g sigmoid(1.702 g) (u + 1) of the clamped halves g = min(a, limit), u = clamp(b, -limit, limit)
+__device__ __forceinline__ float clampglu_f32(float a, float b, float limit) {
+    const float g = fminf(a, limit), u = fminf(fmaxf(b, -limit), limit);
+    return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
 template <int EPI>
-__device__ __forceinline__ float pair_act_f32(float a, float b) {
+__device__ __forceinline__ float pair_act_f32(float a, float b, float limit) {
+    if (EPI == MI355_EPI_CLAMPGLU) return clampglu_f32(a, b, limit);
     return EPI == MI355_EPI_GEGLU ? gelu_tanh_f32(a) * b : swiglu_f32(a, b);
 }
 

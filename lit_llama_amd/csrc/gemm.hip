@@ -35,7 +35,11 @@
 // v_exp_f32 / v_rcp_f32 are within 1 ulp of f32 — 2^-15 of the bf16 step the result is rounded to.
 __device__ __forceinline__ bf16_t bf16_hw(float f) { return __builtin_bit_cast(bf16_t, (__bf16)f); }
 template <int EPI>
-__device__ __forceinline__ float pair_act_fast(float a, float b) {
+__device__ __forceinline__ float pair_act_fast(float a, float b, float limit) {
+    if constexpr (EPI == MI355_EPI_CLAMPGLU) {
+        const float g = fminf(a, limit), u = fminf(fmaxf(b, -limit), limit);
+        return (g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(g * (-1.702f * 1.44269504088896340736f)))) * (u + 1.0f);
+    }
     // silu(a) * b = a / (1 + 2^(-a log2 e)) * b; a -> -inf: 2^(+inf) = inf, rcp = 0; a -> +inf: rcp(1) = 1
     // gelu(a) in the tanh form = a / (1 + 2^(-2 u log2 e)), u = sqrt(2 / pi) (a + 0.044715 a^3)
     const float t = EPI == MI355_EPI_GEGLU ? a * (1.59576912160573071176f + 0.07135481282792783f * (a * a)) : a;
@@ -113,6 +117,9 @@ struct GemmParams {
     float* part;
     int relu2;             // STORE: max(y, 0)^2
     float alpha;           // factor of the product where rinv is NULL (an operand that needed no staging)
+    float limit;           // CLAMPGLU
+    int slice_blocks;      // != 0: row blocks [i slice_blocks, (i + 1) slice_blocks) read the operand at xb + i slice_stride
+    int64_t slice_stride;
     // grouped scales (GRP kernels): gtab[group 0..n_groups][r][tab_ld rows] = bf16 scale | bf16 zero << 16 (row n_groups
     // is all zero), sxt[group][M] = operand sums per group; upg = 128-column units per group (groups of >= 128 columns)
     const uint32_t* gtab;
@@ -257,7 +264,7 @@ __global__ __launch_bounds__(256) void group_table_kernel(const bf16_t* s0, cons
 // y[m][n] (+)= sum over the K-slices, in slice order (deterministic)
 template <int EPI>
 __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, int ksplit, int M, int N, void* y, int y_dtype,
-                                                            int64_t ldy, int relu2) {
+                                                            int64_t ldy, int relu2, float limit) {
     const int64_t n4 = N >> 2;
     for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < (int64_t)M * n4; i += (int64_t)gridDim.x * blockDim.x) {
         const int m = (int)(i / n4), n = (int)(i - (int64_t)m * n4) * 4;
@@ -271,8 +278,8 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, i
             }
             bf16_t* dst = (bf16_t*)y + (int64_t)m * ldy + n;
             u32x2 pk;
-            pk[0] = (uint32_t)bf16_hw(pair_act_fast<EPI>(o[0], b[0])) | ((uint32_t)bf16_hw(pair_act_fast<EPI>(o[1], b[1])) << 16);
-            pk[1] = (uint32_t)bf16_hw(pair_act_fast<EPI>(o[2], b[2])) | ((uint32_t)bf16_hw(pair_act_fast<EPI>(o[3], b[3])) << 16);
+            pk[0] = (uint32_t)bf16_hw(pair_act_fast<EPI>(o[0], b[0], limit)) | ((uint32_t)bf16_hw(pair_act_fast<EPI>(o[1], b[1], limit)) << 16);
+            pk[1] = (uint32_t)bf16_hw(pair_act_fast<EPI>(o[2], b[2], limit)) | ((uint32_t)bf16_hw(pair_act_fast<EPI>(o[3], b[3], limit)) << 16);
             *(u32x2*)dst = pk;
         } else if (y_dtype == MI355_F32) {
             float* dst = (float*)y + (int64_t)m * ldy + n;
@@ -317,7 +324,7 @@ __global__ __launch_bounds__(256) void splitk_fused_reduce_kernel(const GemmPara
             }
             bf16_t ob[4];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(pair_act_fast<EPI>(a[r], b[r]));
+            for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(pair_act_fast<EPI>(a[r], b[r], p.limit));
             u32x2 pk;
             pk[0] = (uint32_t)ob[0] | ((uint32_t)ob[1] << 16);
             pk[1] = (uint32_t)ob[2] | ((uint32_t)ob[3] << 16);
@@ -444,7 +451,11 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
     const __amdgpu_buffer_rsrc_t rw = __builtin_amdgcn_make_buffer_rsrc((void*)p.w, 0, (int)p.w_bytes, 0x00020000);
     const __amdgpu_buffer_rsrc_t rw0 = __builtin_amdgcn_make_buffer_rsrc((void*)p.w, 0, 0, 0x00020000);
     const unsigned xbytes = (unsigned)((int64_t)p.M * p.ldxb * 2);
-    const __amdgpu_buffer_rsrc_t rx = __builtin_amdgcn_make_buffer_rsrc((void*)p.xb, 0, (int)xbytes, 0x00020000);
+    const bf16_t* xbase = p.xb;
+    if constexpr (EPI == MI355_EPI_STORE && FMT == MI355_W_BF16 && !FUSE) {
+        if (p.slice_blocks != 0) xbase += (int64_t)(nb / p.slice_blocks) * p.slice_stride;
+    }
+    const __amdgpu_buffer_rsrc_t rx = __builtin_amdgcn_make_buffer_rsrc((void*)xbase, 0, (int)xbytes, 0x00020000);
     const unsigned lane_off = lane * 16;
     auto wload = [&](int t, int u, u32x4 (&dst)[kWP]) {
         // past the last unit / tile the load goes through a zero-sized descriptor: the scalar offset operand of a raw
@@ -861,7 +872,7 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
                     bf16_t* dst = (bf16_t*)p.y + (int64_t)m * p.ldy + n;
                     bf16_t ob[4];
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(pair_act_fast<EPI>(v[t][r], v[t + 1][r]));
+                    for (int r = 0; r < 4; ++r) ob[r] = bf16_hw(pair_act_fast<EPI>(v[t][r], v[t + 1][r], p.limit));
                     u32x2 o;
                     o[0] = (uint32_t)ob[0] | ((uint32_t)ob[1] << 16);
                     o[1] = (uint32_t)ob[2] | ((uint32_t)ob[3] << 16);
@@ -995,6 +1006,7 @@ int launch_gemm_w(const GemmParams& p, hipStream_t s) {  // p.n_tiles: 16-row ti
     const int per_block = PAIR ? kSlots / 2 : kSlots;
     GemmParams q = p;
     q.n_blocks = (p.n_tiles + per_block - 1) / per_block;
+    q.slice_blocks = p.slice_blocks / (16 * per_block);  // (in: rows; a multiple of 256, which every block divides)
     q.total_blocks = q.n_blocks * ((p.M + BM - 1) / BM);
     q.per_xcd = (q.total_blocks * q.ksplit + 7) / 8;
     if constexpr (FUSE) {
@@ -1018,7 +1030,7 @@ int launch_gemm_w(const GemmParams& p, hipStream_t s) {  // p.n_tiles: 16-row ti
     if (q.ksplit > 1) {
         const int64_t n = (int64_t)p.M * (p.N >> 2);
         const int grid = (int)((n + 255) / 256 < 2048 ? (n + 255) / 256 : 2048);
-        hipLaunchKernelGGL(splitk_reduce_kernel<EPI>, dim3(grid), dim3(256), 0, s, q.part, q.ksplit, p.M, p.N, p.y, p.y_dtype, p.ldy, p.relu2);
+        hipLaunchKernelGGL(splitk_reduce_kernel<EPI>, dim3(grid), dim3(256), 0, s, q.part, q.ksplit, p.M, p.N, p.y, p.y_dtype, p.ldy, p.relu2, p.limit);
         MI355_LAUNCH_CHECK();
     }
     return 0;
@@ -1123,6 +1135,7 @@ int launch_gemm_epi(const GemmParams& p, int epi, hipStream_t s) {
     if (epi == MI355_EPI_SWIGLU) return launch_gemm<MI355_EPI_SWIGLU, true, FMT, FUSE>(p, s);
     if constexpr (FMT == MI355_W_BF16 && !FUSE) {
         if (epi == MI355_EPI_GEGLU) return launch_gemm<MI355_EPI_GEGLU, true, FMT, FUSE>(p, s);
+        if (epi == MI355_EPI_CLAMPGLU) return launch_gemm<MI355_EPI_CLAMPGLU, true, FMT, FUSE>(p, s);
     }
     if (epi == MI355_EPI_ACCUM) return launch_gemm<MI355_EPI_ACCUM, false, FMT, FUSE>(p, s);
     return launch_gemm<MI355_EPI_STORE, false, FMT, FUSE>(p, s);
@@ -1177,8 +1190,8 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
     MI355_CHECK_ARG(a->M >= 1 && a->N > 0 && a->K > 0, MI355_E_SHAPE, "linear_gemm: bad shape M=%d N=%d K=%d", a->M, a->N, a->K);
     MI355_CHECK_ARG(a->attn_partials == nullptr && a->bias == nullptr, MI355_E_ARG, "linear_gemm: no bias / attention prologue");
     const bool swiglu = is_pair_epi(a->epi);
-    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_GEGLU, MI355_E_ARG, "linear_gemm: bad epi");
-    MI355_CHECK_ARG(a->epi != MI355_EPI_GEGLU || (!q4 && f == nullptr), MI355_E_ARG, "linear_gemm: GEGLU takes the BF16 pair stream");
+    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_CLAMPGLU, MI355_E_ARG, "linear_gemm: bad epi");
+    MI355_CHECK_ARG((a->epi != MI355_EPI_GEGLU && a->epi != MI355_EPI_CLAMPGLU) || (!q4 && f == nullptr), MI355_E_ARG, "linear_gemm: GEGLU and CLAMPGLU take the BF16 pair stream");
     MI355_CHECK_ARG(!(a->flags & MI355_LF_NORM_ONE) || !q4 || a->group_cols <= 0 || a->group_cols >= a->K, MI355_E_ARG,
                     "linear_gemm: no 1 + scale norm in front of grouped scales");
     MI355_CHECK_ARG(swiglu ? (a->R == 2 && (!q4 || (a->scales2 && a->zeros2)) && a->y_dtype == MI355_BF16) : a->R == 1, MI355_E_ARG,
@@ -1289,6 +1302,12 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
     p.ldxb = f_in || direct ? a->ldx : (int64_t)kp;
     p.rinv = direct ? nullptr : rinv;
     p.alpha = a->alpha == 0.f ? 1.f : a->alpha;
+    p.limit = a->limit;
+    MI355_CHECK_ARG(a->slice_rows == 0 || (direct && a->epi == MI355_EPI_STORE && a->slice_rows > 0 && a->slice_rows % 256 == 0 &&
+                                           a->N % a->slice_rows == 0 && a->slice_stride % 8 == 0),
+                    MI355_E_ARG, "linear_gemm: operand slices take whole row blocks of a bf16 operand and the STORE epilogue");
+    p.slice_blocks = a->slice_rows;
+    p.slice_stride = a->slice_stride;
     p.sx = sx;
     p.scales = a->scales;
     p.zeros = a->zeros;

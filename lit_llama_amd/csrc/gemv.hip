@@ -65,6 +65,7 @@ struct GemvParams {
     float eps;
     // grouped scales (GRP kernels): scales / zeros are [N, n_groups] bf16, one pair per 32 << gq_shift input columns
     float alpha;    // factor of the product
+    float limit;    // CLAMPGLU
     int relu2;      // STORE: max(y, 0)^2
     float norm_add; // the norm's scale is norm_add + norm_scale
     int n_groups, gq_shift;
@@ -387,7 +388,7 @@ __device__ __forceinline__ void tile_epilogue(const GemvParams& p, const char* p
     if constexpr (is_pair_epi(EPI)) {
         if constexpr (R == 2) {
             const int n = tile * 16 + e_row;
-            if (n < p.N) st2(p.y, (int64_t)e_col * p.ldy + n, p.y_dtype, pair_act_f32<EPI>(v[0], v[1]));
+            if (n < p.N) st2(p.y, (int64_t)e_col * p.ldy + n, p.y_dtype, pair_act_f32<EPI>(v[0], v[1], p.limit));
         }
     } else {
 #pragma unroll
@@ -1008,7 +1009,7 @@ int launch_gemv_epi(const GemvParams& p, int grid, int waves, size_t lds, hipStr
             if constexpr (EPI != MI355_EPI_ACCUM) return launch_gemv_v<FMT, R, P, EPI, 4, GRP>(p, grid, waves, lds, stream);
             break;
         case 2:
-            if constexpr (!is_pair_epi(EPI)) return launch_gemv_v<FMT, R, P, EPI, 2, GRP>(p, grid, waves, lds, stream);
+            if constexpr (!is_pair_epi(EPI) || EPI == MI355_EPI_CLAMPGLU) return launch_gemv_v<FMT, R, P, EPI, 2, GRP>(p, grid, waves, lds, stream);
             break;
         case 3:
             if constexpr (!is_pair_epi(EPI)) return launch_gemv_v<FMT, R, P, EPI, 3, GRP>(p, grid, waves, lds, stream);
@@ -1030,6 +1031,10 @@ int launch_gemv(const GemvParams& p, int grid, int waves, size_t lds, hipStream_
         case MI355_EPI_GEGLU:
             if constexpr (R == 2 && FMT == MI355_W_BF16) return launch_gemv_epi<FMT, R, P, MI355_EPI_GEGLU, GRP>(p, grid, waves, lds, stream);
             mi355_set_error("the GEGLU epilogue takes the BF16 pair stream");
+            return MI355_E_ARG;
+        case MI355_EPI_CLAMPGLU:
+            if constexpr (R == 2 && FMT == MI355_W_BF16) return launch_gemv_epi<FMT, R, P, MI355_EPI_CLAMPGLU, GRP>(p, grid, waves, lds, stream);
+            mi355_set_error("the CLAMPGLU epilogue takes the BF16 pair stream");
             return MI355_E_ARG;
         default:
             if constexpr (R == 2) return launch_gemv_epi<FMT, R, P, MI355_EPI_SWIGLU, GRP>(p, grid, waves, lds, stream);
@@ -1162,7 +1167,8 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
     MI355_CHECK_ARG(a->M >= 1 && a->M <= kMaxM, MI355_E_SHAPE, "linear_fast: M=%d outside 1..%d", a->M, kMaxM);
     MI355_CHECK_ARG(a->K > 0 && a->N > 0, MI355_E_SHAPE, "linear_fast: N=%d K=%d must be positive", a->N, a->K);
     const bool swiglu = is_pair_epi(a->epi);
-    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_GEGLU, MI355_E_ARG, "linear_fast: bad epi");
+    MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_CLAMPGLU, MI355_E_ARG, "linear_fast: bad epi");
+    MI355_CHECK_ARG(a->slice_rows == 0, MI355_E_ARG, "linear_fast: operand slices belong to linear_gemm");
     MI355_CHECK_ARG(!swiglu || a->R == 2, MI355_E_ARG, "linear_fast: SwiGLU epilogue needs the interleaved R=2 stream");
     const int rows_per_tile = swiglu ? 16 : 16 * a->R;
     if (a->fmt == MI355_W_Q4) {
@@ -1202,6 +1208,7 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
     p.xs_stride = (p.units + 1) * kUnitK * 2 + 16;  // + one all-zero unit (idle ring steps read it)
     p.eps = a->eps;
     p.alpha = a->alpha == 0.f ? 1.f : a->alpha;
+    p.limit = a->limit;
     p.relu2 = (a->flags & MI355_LF_RELU2) ? 1 : 0;
     p.norm_add = (a->flags & MI355_LF_NORM_ONE) ? 1.f : 0.f;
     MI355_CHECK_ARG(!p.relu2 || a->epi == MI355_EPI_STORE, MI355_E_ARG, "linear_fast: RELU2 belongs to the STORE epilogue");

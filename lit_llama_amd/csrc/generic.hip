@@ -37,6 +37,7 @@ extern "C" int mi355_sizeof(int which) {
         case 12: return (int)sizeof(mi355_hybrid_layer);
         case 13: return (int)sizeof(mi355_hybrid_model);
         case 14: return (int)sizeof(mi355_experts_args);
+        case 15: return (int)sizeof(mi355_latent_args);
         default: return -1;
     }
 }

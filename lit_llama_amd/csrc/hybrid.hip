@@ -1,7 +1,9 @@
 // The forward pass of a layered hybrid model (mi355_hybrid_forward): a host-side walk over the layer runs that enqueues this library's
 // linears (gemv.hip for a few rows, gemm.hip above, the exact f32 kernel for f32 models), mixers (window_attention.hip, recurrent.hip) and
 // experts (experts.hip).  RMSNorm rides in the consuming linear and the residual sum in the producing one; the residual stream is f32.
-#include "common.h"
+// A parallel layer normalises its row once (by groups, with the token shift of its mixer), and its mixer's output and hidden row leave
+// through one product.
+#include "product.h"
 
 namespace {
 
@@ -75,6 +77,130 @@ __global__ __launch_bounds__(512) void norm_rows_kernel(const float* x, int64_t 
         if (j < K / 4) put(j, v[i]);
     }
     for (int j = threadIdx.x + kHeld * 512; j < K / 4; j += 512) put(j, row[j]);
+}
+
+// ---- parallel layers: h = norm(x) in groups, and the mixes h + (h' - h) mu of the token shift (h' = the row before)
+struct NormParams {
+    const float* x;
+    int64_t ldx;
+    const int32_t* want;    // rows of x, or NULL: row m
+    int width, groups, size, scale_dtype;
+    float eps;
+    const void* scale;
+    void* h;                // [rows, ldh]
+    int64_t ldh;
+    int n_mix;
+    const float* mu;        // [n_mix][width]
+    float* shift;           // [slots][width]
+    void* mix;              // [n_mix], mix_stride apart, as h
+    int64_t mix_stride;
+    mi355_seq_batch b;
+};
+
+template <typename T>
+__device__ __forceinline__ void put4(T* p, f32x4 v) {
+    if constexpr (sizeof(T) == 4) {
+        *(f32x4*)p = v;
+    } else {
+        typedef __attribute__((ext_vector_type(2))) __bf16 bf2;
+        const bf2 a = {(__bf16)v[0], (__bf16)v[1]}, b = {(__bf16)v[2], (__bf16)v[3]};
+        *(u32x2*)p = u32x2{__builtin_bit_cast(uint32_t, a), __builtin_bit_cast(uint32_t, b)};
+    }
+}
+
+// one row per workgroup; V elements per load (4: groups of whole vectors).  Dynamic LDS: 2 groups floats of 1 / rms + 2 max(8, groups) sums
+template <typename T, int V>
+__global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    __shared__ int s_seq;
+    const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int parts = p.groups < 8 ? 8 / p.groups : 1;      // waves per group
+    float* rinv = sm;                                       // [2][groups]
+    float* sums = sm + 2 * p.groups;                        // [2][groups * parts]
+    const float* row = p.x + (int64_t)(p.want != nullptr ? p.want[m] : m) * p.ldx;
+    // a second row: the one before, or, in the workgroup of a portion's first row, the portion's last one (it enters the state there)
+    const float* other = nullptr;
+    int seq = 0, i = 0, cnt = 0;
+    if (p.n_mix > 0) {
+        if (p.b.max_count == 1) {
+            seq = m;
+        } else {
+            for (int s = tid; s < p.b.seqs; s += 512)
+                if (m >= p.b.row0[s] && m < p.b.row0[s] + p.b.count[s]) s_seq = s;
+            __syncthreads();
+            seq = s_seq;
+        }
+        i = m - p.b.row0[seq], cnt = p.b.count[seq];
+        other = i > 0 ? row - p.ldx : cnt > 1 ? row + (int64_t)(cnt - 1) * p.ldx : nullptr;
+    }
+    const int seg = (p.size / V + parts - 1) / parts;       // vectors of a wave's part of a group
+    for (int q = wave; q < p.groups * parts; q += 8) {
+        const int gr = q / parts, v0 = (q - gr * parts) * seg, v1 = min(p.size / V, v0 + seg);
+        const int64_t at = (int64_t)gr * p.size;
+        float s0 = 0.f, s1 = 0.f;
+#pragma unroll 4
+        for (int v = v0 + lane; v < v1; v += 64) {
+            if constexpr (V == 4) {
+                const f32x4 a = *(const f32x4*)(row + at + 4 * v);
+                s0 += (a[0] * a[0] + a[1] * a[1]) + (a[2] * a[2] + a[3] * a[3]);
+                if (other != nullptr) {
+                    const f32x4 c = *(const f32x4*)(other + at + 4 * v);
+                    s1 += (c[0] * c[0] + c[1] * c[1]) + (c[2] * c[2] + c[3] * c[3]);
+                }
+            } else {
+                s0 += row[at + v] * row[at + v];
+                if (other != nullptr) s1 += other[at + v] * other[at + v];
+            }
+        }
+        s0 = group_sum(s0, 64);
+        s1 = group_sum(s1, 64);
+        if (lane == 0) sums[q] = s0, sums[p.groups * parts + q] = s1;
+    }
+    __syncthreads();
+    for (int q = tid; q < 2 * p.groups; q += 512) {
+        float s = 0.f;
+        for (int j = 0; j < parts; ++j) s += sums[q * parts + j];
+        rinv[q] = 1.0f / sqrtf(s / (float)p.size + p.eps);
+    }
+    __syncthreads();
+    T* h = (T*)p.h + (int64_t)m * p.ldh;
+    float* state = p.n_mix > 0 ? p.shift + (int64_t)p.b.slot[seq] * p.width : nullptr;
+    const bool first = p.n_mix > 0 && i == 0, begun = first && p.b.pos[seq] > 0;
+    for (int v = tid; v < p.width / V; v += 512) {
+        const int k = v * V, gr = k / p.size;
+        const float r0 = rinv[gr], r1 = rinv[p.groups + gr];
+        float sc[V], a[V], o[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+            sc[e] = ld_as_f32(p.scale, k + e, p.scale_dtype);
+            a[e] = row[k + e] * r0 * sc[e];
+            o[e] = other != nullptr ? other[k + e] * r1 * sc[e] : a[e];
+        }
+        if constexpr (V == 4) put4(h + k, f32x4{a[0], a[1], a[2], a[3]});
+        else st_from_f32(h, k, sizeof(T) == 4 ? MI355_F32 : MI355_BF16, a[0]);
+        if (p.n_mix == 0) continue;
+        float d[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+            const float before = !first ? o[e] : begun ? state[k + e] : 0.f;
+            if (first) state[k + e] = o[e];  // (the portion's last row; of one row, itself)
+            d[e] = before - a[e];
+        }
+        for (int s = 0; s < p.n_mix; ++s) {
+            T* x = (T*)p.mix + s * p.mix_stride + (int64_t)m * p.ldh + k;
+            const float* mu = p.mu + (int64_t)s * p.width + k;
+            if constexpr (V == 4) put4(x, f32x4{a[0] + d[0] * mu[0], a[1] + d[1] * mu[1], a[2] + d[2] * mu[2], a[3] + d[3] * mu[3]});
+            else st_from_f32(x, 0, sizeof(T) == 4 ? MI355_F32 : MI355_BF16, a[0] + d[0] * mu[0]);
+        }
+    }
+}
+
+// rows [gate | up] of 2 n values -> the clamped gated unit
+__global__ __launch_bounds__(256) void clampglu_kernel(const float* gu, float* h, int n, int64_t ldh, int64_t total, float limit) {
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
+        const int64_t m = i / n, k = i - m * n;
+        h[m * ldh + k] = clampglu_f32(gu[m * 2 * n + k], gu[m * 2 * n + n + k], limit);
+    }
 }
 
 __global__ __launch_bounds__(256) void relu2_kernel(float* h, int64_t n) {
@@ -197,7 +323,143 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
     return mi355_linear_fast(&a, s);
 }
 
+int norm_groups(const mi355_hybrid_model* m, const void* scale, const mi355_hybrid_layer* l, const mi355_seq_batch* b, const int32_t* want, int rows,
+                hipStream_t s) {
+    NormParams p;
+    memset(&p, 0, sizeof(p));
+    const bool f32 = m->dtype == MI355_F32;
+    p.x = m->x, p.ldx = m->ldx, p.want = want;
+    p.width = m->width, p.groups = m->norm_groups, p.size = m->width / m->norm_groups;
+    p.eps = m->eps, p.scale = scale, p.scale_dtype = m->norm_dtype;
+    p.h = f32 ? (void*)m->xn : (void*)m->xb, p.ldh = m->ld_n;
+    if (l != nullptr && l->n_mix > 0) {
+        p.n_mix = l->n_mix, p.mu = l->mu, p.shift = l->shift;
+        p.mix = m->mix, p.mix_stride = (int64_t)m->max_rows * m->ld_n;
+        p.b = *b;
+    }
+    const size_t lds = (size_t)(2 * p.groups + 2 * (p.groups < 8 ? 8 : p.groups)) * 4;
+    const bool vec = p.size % 4 == 0;
+    if (f32) {
+        if (vec) hipLaunchKernelGGL((norm_groups_kernel<float, 4>), dim3(rows), dim3(512), lds, s, p);
+        else hipLaunchKernelGGL((norm_groups_kernel<float, 1>), dim3(rows), dim3(512), lds, s, p);
+    } else {
+        if (vec) hipLaunchKernelGGL((norm_groups_kernel<bf16_t, 4>), dim3(rows), dim3(512), lds, s, p);
+        else hipLaunchKernelGGL((norm_groups_kernel<bf16_t, 1>), dim3(rows), dim3(512), lds, s, p);
+    }
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+
+mi355_product product_of(const mi355_hybrid_model* m, const void* x, int64_t ldx, int M, int epi, void* y, int64_t ldy, int y_dtype) {
+    mi355_product p;
+    memset(&p, 0, sizeof(p));
+    p.dtype = m->dtype;
+    p.x = x, p.ldx = ldx, p.M = M;
+    p.y = y, p.ldy = ldy, p.y_dtype = y_dtype, p.epi = epi;
+    p.alpha = 1.f;
+    p.ws = m->gemm_ws, p.ws_bytes = m->gemm_ws_bytes;
+    return p;
+}
+
+// the input projections of a parallel layer, out of its normalised rows and their mixes
+int parallel_in(const mi355_hybrid_model* m, const mi355_hybrid_layer& l, int M, hipStream_t s) {
+    const bool f32 = m->dtype == MI355_F32;
+    const int64_t ldp = l.in.N;
+    if (l.n_mix == 0) return mi355_product_run(product_of(m, f32 ? (void*)m->xn : (void*)m->xb, m->ld_n, M, MI355_EPI_STORE, m->proj, ldp, m->dtype), l.in, s);
+    const size_t size = dtype_size(m->dtype);
+    const int64_t stride = (int64_t)m->max_rows * m->ld_n;
+    int i = 0;
+    if (l.mix_stacked > 1) {  // parts of equal size, one stream
+        const mi355_proj& w = l.mix_w[0];
+        mi355_proj part = w;
+        part.N = w.N / l.mix_stacked;
+        if (mi355_product_wide(w, M, 1) && part.N % 256 == 0) {
+            mi355_product p = product_of(m, m->mix, m->ld_n, M, MI355_EPI_STORE, (char*)m->proj + l.mix_at[0] * size, ldp, m->dtype);
+            p.slice_rows = part.N, p.slice_stride = stride;
+            if (int rc = mi355_product_run(p, w, s)) return rc;
+            i = l.mix_stacked;
+        } else {
+            for (; i < l.mix_stacked; ++i) {
+                part.w = (const char*)w.w + (int64_t)i * part.N * ((w.K + 127) / 128 * 128) * size;
+                const mi355_product p = product_of(m, (const char*)m->mix + i * stride * size, m->ld_n, M, MI355_EPI_STORE,
+                                                   (char*)m->proj + l.mix_at[i] * size, ldp, m->dtype);
+                if (int rc = mi355_product_run(p, part, s)) return rc;
+            }
+        }
+    }
+    for (; i < l.n_mix; ++i) {
+        const mi355_product p = product_of(m, (const char*)m->mix + i * stride * size, m->ld_n, M, MI355_EPI_STORE,
+                                           (char*)m->proj + l.mix_at[i] * size, ldp, m->dtype);
+        if (int rc = mi355_product_run(p, l.mix_w[i], s)) return rc;
+    }
+    return 0;
+}
+
+// hidden row into `cat`, then x += out [mixer | hidden]
+int parallel_out(const mi355_hybrid_model* m, const mi355_hybrid_layer& l, int M, hipStream_t s) {
+    const bool f32 = m->dtype == MI355_F32;
+    if (l.mlp == MI355_MLP_CLAMPGLU) {
+        char* hid = (char*)l.cat + (int64_t)l.hid_at * dtype_size(m->dtype);
+        if (f32) {  // gate rows, then up rows
+            mi355_proj both = l.up;
+            both.N *= 2;
+            if (int rc = mi355_product_run(product_of(m, m->xn, m->ld_n, M, MI355_EPI_STORE, m->hid, both.N, MI355_F32), both, s)) return rc;
+            const int64_t n = (int64_t)M * l.up.N;
+            hipLaunchKernelGGL(clampglu_kernel, dim3(ew_blocks(n)), dim3(256), 0, s, (const float*)m->hid, (float*)hid, l.up.N, l.ld_cat, n, l.limit);
+            MI355_LAUNCH_CHECK();
+        } else {
+            mi355_product p = product_of(m, m->xb, m->ld_n, M, MI355_EPI_CLAMPGLU, hid, l.ld_cat, MI355_BF16);
+            p.limit = l.limit;
+            if (int rc = mi355_product_run(p, l.up, s)) return rc;
+        }
+    }
+    if (f32) {
+        if (int rc = mi355_product_run(product_of(m, l.cat, l.ld_cat, M, MI355_EPI_STORE, m->tmp, m->ldx, MI355_F32), l.out, s)) return rc;
+        const int64_t n = (int64_t)M * m->ldx;
+        hipLaunchKernelGGL(residual_kernel, dim3(ew_blocks(n)), dim3(256), 0, s, m->x, m->tmp, m->residual_mult, n);
+        MI355_LAUNCH_CHECK();
+        return 0;
+    }
+    mi355_product p = product_of(m, l.cat, l.ld_cat, M, MI355_EPI_ACCUM, m->x, m->ldx, MI355_F32);
+    p.alpha = m->residual_mult;
+    return mi355_product_run(p, l.out, s);
+}
+
 }  // namespace
+
+bool mi355_product_wide(const mi355_proj& w, int M, int R) {
+    const int K = (w.K + 127) / 128 * 128;
+    return M > 8 || mi355_linear_max_rows(MI355_W_BF16, K, R, 0) < M || (M > 2 && K > 12288);
+}
+
+int mi355_product_run(const mi355_product& p, const mi355_proj& w, hipStream_t s) {
+    if (p.dtype == MI355_F32) {
+        MI355_CHECK_ARG(p.epi == MI355_EPI_STORE && p.alpha == 1.f && p.y_dtype == MI355_F32, MI355_E_ARG, "product: f32 operands are stored as they are");
+        return mi355_linear_dense(p.x, p.ldx, w.w, nullptr, p.y, p.ldy, p.M, w.N, w.K, MI355_F32, s);
+    }
+    mi355_linear_args a;
+    memset(&a, 0, sizeof(a));
+    a.fmt = MI355_W_BF16;
+    a.R = is_pair_epi(p.epi) ? 2 : 1;
+    a.w = w.w;
+    a.N = w.N;
+    a.K = (w.K + 127) / 128 * 128;  // (the stream and the operand are padded with zeros)
+    a.x = p.x;
+    a.x_dtype = MI355_BF16;
+    a.M = p.M;
+    a.ldx = p.ldx;
+    a.epi = p.epi;
+    a.alpha = p.alpha;
+    a.limit = p.limit;
+    a.y = p.y;
+    a.y_dtype = p.y_dtype;
+    a.ldy = p.ldy;
+    a.slice_rows = p.slice_rows;
+    a.slice_stride = p.slice_stride;
+    MI355_CHECK_ARG(p.ldx >= a.K && p.ldx % 8 == 0, MI355_E_SHAPE, "product: rows of pitch %lld hold no operand of %d columns", (long long)p.ldx, a.K);
+    if (p.slice_rows != 0 || mi355_product_wide(w, p.M, a.R)) return mi355_linear_gemm(&a, p.ws, (size_t)p.ws_bytes, s);
+    return mi355_linear_fast(&a, s);
+}
 
 extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq_batch* b, const int32_t* tokens, const int32_t* want,
                                     int n_want, float* logits, int run_end, mi355_stream_t stream) {
@@ -210,6 +472,15 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
     MI355_CHECK_ARG(m->residual_mult != 0.f && m->logit_scale != 0.f, MI355_E_ARG, "hybrid_forward: residual_mult or logit_scale is 0");
     MI355_CHECK_ARG(m->norm_add == 0.f || (m->norm_add == 1.f && m->dtype == MI355_BF16), MI355_E_ARG, "hybrid_forward: norm_add is 0, or 1 in bf16 models");
     MI355_CHECK_ARG(n_want == 0 || run_end < m->n_runs || (logits && m->final_norm), MI355_E_ARG, "hybrid_forward: nowhere to write logits");
+    MI355_CHECK_ARG(m->norm_groups == 0 || (m->norm_groups > 0 && m->width % m->norm_groups == 0 && m->norm_add == 0.f && m->ld_n >= (m->width + 127) / 128 * 128 &&
+                                            m->ld_n % 8 == 0), MI355_E_SHAPE, "hybrid_forward: bad norm groups %d of width %d", m->norm_groups, m->width);
+    for (int r = 0; r < m->n_runs; ++r) {
+        const mi355_hybrid_layer& l = m->layers[r];
+        MI355_CHECK_ARG(!l.parallel || (m->norm_groups > 0 && l.cat && l.ld_cat >= l.out.K && (l.mlp == MI355_MLP_NONE || l.mlp == MI355_MLP_CLAMPGLU) &&
+                                        l.n_mix <= 5 && (l.n_mix == 0 || (l.mu && l.shift && m->mix))),
+                        MI355_E_ARG, "hybrid_forward: bad parallel layer (run %d)", r);
+        MI355_CHECK_ARG(l.parallel || l.mlp != MI355_MLP_CLAMPGLU, MI355_E_ARG, "hybrid_forward: a clamped gated feed-forward belongs to a parallel layer (run %d)", r);
+    }
     hipStream_t s = (hipStream_t)stream;
     hipLaunchKernelGGL(embed_rows_kernel, dim3(M), dim3(256), 0, s, tokens, m->embed, m->dtype, m->x, m->width, m->ldx, m->vocab);
     MI355_LAUNCH_CHECK();
@@ -217,14 +488,19 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
     for (int r = 0; r < runs; ++r) {
         const mi355_hybrid_layer& l = m->layers[r];
         const int64_t ldp = l.in.N;
-        if (int rc = linear(m, l.in, m->x, m->ldx, l.norm1, kStore, m->proj, ldp, m->dtype, M, s)) return rc;
+        void* const y = l.parallel ? l.cat : m->att;
+        const int64_t ldy = l.parallel ? l.ld_cat : m->ld_att;
+        if (l.parallel) {
+            if (int rc = norm_groups(m, l.norm1, &l, b, nullptr, M, s)) return rc;
+            if (int rc = parallel_in(m, l, M, s)) return rc;
+        } else if (int rc = linear(m, l.in, m->x, m->ldx, l.norm1, kStore, m->proj, ldp, m->dtype, M, s)) return rc;
         if (l.mixer == MI355_MIX_ATTENTION) {
             mi355_window_attn_args a = l.attn;
             a.proj = m->proj;
             a.ld = ldp;
             a.dtype = m->dtype;
-            a.y = m->att;
-            a.ldy = m->ld_att;
+            a.y = y;
+            a.ldy = ldy;
             a.partials = m->partials;
             a.partials_bytes = m->partials_bytes;
             if (int rc = mi355_window_attention(&a, b, stream)) return rc;
@@ -238,16 +514,30 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
                 a.y = m->att;
                 if (int rc = mi355_window_cache_write(&a, b, stream)) return rc;
             }
+        } else if (l.mixer == MI355_MIX_LATENT) {
+            mi355_latent_args a = l.latent;
+            a.proj = m->proj;
+            a.ld = ldp;
+            a.dtype = m->dtype;
+            a.y = y;
+            a.ldy = ldy;
+            a.gemm_ws = m->gemm_ws;
+            a.gemm_ws_bytes = m->gemm_ws_bytes;
+            if (int rc = mi355_latent_attention(&a, b, stream)) return rc;
         } else {
             mi355_recurrent_args a = l.rec;
             a.proj = m->proj;
             a.ld = ldp;
             a.dtype = m->dtype;
-            a.y = m->att;
-            a.ldy = m->ld_att;
+            a.y = y;
+            a.ldy = ldy;
             a.scratch = m->rec_scratch;
             a.scratch_bytes = m->rec_scratch_bytes;
             if (int rc = mi355_recurrent(&a, b, stream)) return rc;
+        }
+        if (l.parallel) {
+            if (int rc = parallel_out(m, l, M, s)) return rc;
+            continue;
         }
         if (int rc = linear(m, l.out, m->att, m->ld_att, nullptr, kResidual, m->x, m->ldx, MI355_F32, M, s)) return rc;
         if (l.mlp == MI355_MLP_EXPERTS) {
@@ -271,6 +561,13 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
         }
     }
     if (run_end < m->n_runs || n_want == 0) return 0;
+    if (m->norm_groups > 0) {
+        if (int rc = norm_groups(m, m->final_norm, nullptr, b, want, n_want, s)) return rc;
+        mi355_product p = product_of(m, m->dtype == MI355_F32 ? (void*)m->xn : (void*)m->xb, m->ld_n, n_want, MI355_EPI_STORE, logits, m->ld_logits, MI355_F32);
+        MI355_CHECK_ARG(m->dtype == MI355_BF16 || m->logit_scale == 1.f, MI355_E_ARG, "hybrid_forward: no logit_scale behind a norm in groups in f32 models");
+        p.alpha = m->logit_scale;
+        return mi355_product_run(p, m->head, s);
+    }
     const float* xh = m->x;
     if (want != nullptr) {
         hipLaunchKernelGGL(gather_rows_kernel, dim3(n_want), dim3(256), 0, s, m->x, want, m->xw, m->ldx);
@@ -284,7 +581,11 @@ extern "C" int mi355_hybrid_reset_slots(const mi355_hybrid_model* m, const int32
     MI355_CHECK_ARG(m && slots && n > 0 && m->layers, MI355_E_ARG, "hybrid_reset_slots: bad argument");
     for (int r = 0; r < m->n_runs; ++r) {
         const mi355_hybrid_layer& l = m->layers[r];
-        if (l.mixer == MI355_MIX_ATTENTION) continue;  // (a ring row is written before it can be seen)
+        if (l.mixer == MI355_MIX_ATTENTION || l.mixer == MI355_MIX_LATENT) continue;  // (a cache row is written before it can be seen)
+        if (l.n_mix > 0) {
+            hipLaunchKernelGGL(zero_slots_kernel, dim3(n, 4), dim3(256), 0, (hipStream_t)stream, slots, l.shift, (int64_t)m->width);
+            MI355_LAUNCH_CHECK();
+        }
         const int64_t per = (int64_t)l.rec.heads * l.rec.dim * l.rec.vdim;
         hipLaunchKernelGGL(zero_slots_kernel, dim3(n, per > 65536 ? 64 : 4), dim3(256), 0, (hipStream_t)stream, slots, l.rec.state, per);
         MI355_LAUNCH_CHECK();

@@ -97,6 +97,9 @@ __device__ __forceinline__ void conv_rows16(const mi355_recurrent_args& a, const
     }
 }
 
+// log of a WKV key channel's decay, exp(-exp(z)): below -104 the decay is 0 in f32, and sums of many stay finite
+__device__ __forceinline__ float wkv_log_decay(float z) { return fmaxf(-expf(z), -104.f); }
+
 struct RecParams {
     mi355_recurrent_args a;
     mi355_seq_batch b;

@@ -1,4 +1,5 @@
-// Linear recurrences with a matrix state per head: the gated delta rule (with its short convolutions) and gated linear attention.
+// Linear recurrences with a matrix state per head: the gated delta rule (with its short convolutions), gated linear attention, and WKV time
+// mixing (the state in front of a token, and the token itself with a bonus per key channel).
 //
 //   rec_rows_kernel       one workgroup per (head, sequence) walks its rows one by one with the state in registers: decode steps
 //                         (convolution, gates, state update, output norm and gate in ONE launch) and short portions
@@ -25,10 +26,11 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
     const int cols = p.slices * 64;
     float* q = (float*)smem;           // [parts * RMAX], zero past dim
     float* k = q + p.parts * RMAX;
-    float* al = k + p.parts * RMAX;    // GLA: per-channel decay
-    float* pa = al + p.parts * RMAX;   // [parts][cols] partial S^T k (DELTA)
+    float* al = k + p.parts * RMAX;    // GLA, WKV: per-channel decay
+    float* uk = al + p.parts * RMAX;   // WKV: u k
+    float* pa = uk + p.parts * RMAX;   // [parts][cols] partial S^T k (DELTA)
     float* pb = pa + p.parts * cols;   // [parts][cols] partial S^T q
-    float* lr = pb + p.parts * cols;   // [kMaxRank] low-rank row (GLA)
+    float* lr = pb + p.parts * cols;   // [kMaxRank] low-rank row (GLA, WKV)
 
     const T* rows = (const T*)a.proj + (int64_t)p.b.row0[seq] * a.ld;
     const int ring_ld = 2 * a.kv_heads * dim + a.heads * vdim;
@@ -43,7 +45,7 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
         const int i = part * RMAX + r;
         S[r] = (col_ok && i < dim) ? state[(int64_t)i * vdim + col] : 0.f;
     }
-    for (int i = tid; i < p.parts * RMAX; i += nt) q[i] = k[i] = al[i] = 0.f;
+    for (int i = tid; i < p.parts * RMAX; i += nt) q[i] = k[i] = al[i] = uk[i] = 0.f;
     __syncthreads();
 
     for (int t = 0; t < cnt; ++t) {
@@ -51,7 +53,7 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
         // ---- the row's q, k (and decays) into LDS
         // (what needs no LDS is requested here, in front of the barriers: one memory latency instead of one per use)
         const bool out_ok = part == 0 && col_ok;
-        const float gate = out_ok ? silu_f32(to_f32<T>(row[a.off_g + head * vdim + col])) * a.head_norm[col] : 0.f;
+        const float gate = out_ok ? silu_f32(to_f32<T>(row[a.off_g + head * vdim + col])) * a.head_norm[head * a.norm_ld + col] : 0.f;
         float g = 1.f, beta = 1.f, v = 0.f;
         if constexpr (KIND == MI355_REC_DELTA) {
             const float dt = softplus_f32(to_f32<T>(row[a.off_a + head]) + a.dt_bias[head]);
@@ -80,16 +82,21 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
             }
         } else {
             if (col_ok) v = to_f32<T>(row[a.off_v + head * vdim + col]);
-            for (int r = tid; r < a.rank; r += nt) lr[r] = to_f32<T>(row[a.off_a + r]);
+            for (int r = tid; r < a.rank; r += nt) {
+                const float lv = to_f32<T>(row[a.off_a + r]);
+                lr[r] = KIND == MI355_REC_WKV ? tanhf(lv) : lv;
+            }
             __syncthreads();
             for (int d = tid; d < dim; d += nt) {
                 const int c = head * dim + d;
                 float z = a.a2_bias[c];
 #pragma unroll 8
                 for (int r = 0; r < a.rank; ++r) z += a.a2[(int64_t)c * a.rank + r] * lr[r];
-                al[d] = expf(-softplus_f32(-z) * a.inv_tau);
+                al[d] = expf(KIND == MI355_REC_WKV ? wkv_log_decay(z) : -softplus_f32(-z) * a.inv_tau);
                 q[d] = to_f32<T>(row[a.off_q + c]) * a.q_scale;
-                k[d] = to_f32<T>(row[a.off_k + c]);
+                const float kv = to_f32<T>(row[a.off_k + c]);
+                k[d] = kv;
+                if constexpr (KIND == MI355_REC_WKV) uk[d] = a.bonus[c] * kv;
             }
         }
         __syncthreads();
@@ -113,6 +120,14 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
             for (int r = 0; r < RMAX; ++r) {
                 S[r] += kp[r] * u;
                 o += S[r] * qp[r];
+            }
+        } else if constexpr (KIND == MI355_REC_WKV) {
+            const float* ap = al + part * RMAX;
+            const float* up = uk + part * RMAX;
+#pragma unroll
+            for (int r = 0; r < RMAX; ++r) {
+                o += (S[r] + up[r] * v) * qp[r];
+                S[r] = ap[r] * S[r] + kp[r] * v;
             }
         } else {
             const float* ap = al + part * RMAX;
@@ -168,7 +183,7 @@ __global__ __launch_bounds__(256) void conv_ring_kernel(const RecParams p) {
 
 template <typename T, int KIND, int RMAX>
 int launch_rows(const RecParams& p, hipStream_t s) {
-    const size_t lds = ((size_t)3 * p.parts * RMAX + (size_t)2 * p.parts * p.slices * 64 + kMaxRank) * 4;
+    const size_t lds = ((size_t)4 * p.parts * RMAX + (size_t)2 * p.parts * p.slices * 64 + kMaxRank) * 4;
     hipLaunchKernelGGL((rec_rows_kernel<T, KIND, RMAX>), dim3(p.a.heads, p.b.seqs), dim3(64 * p.parts * p.slices), lds, s, p);
     MI355_LAUNCH_CHECK();
     return 0;
@@ -203,7 +218,9 @@ int run(const RecParams& p, hipStream_t s) {
     const bool chunks = p.a.path == 2 || (p.a.path == 0 && fit && p.b.max_count > 8);
     if (chunks) {
         if (int rc = mi355_recurrent_chunks(p, s)) return rc;
-    } else if (int rc = p.a.kind == MI355_REC_DELTA ? run_rows<T, MI355_REC_DELTA>(p, s) : run_rows<T, MI355_REC_GLA>(p, s)) {
+    } else if (int rc = p.a.kind == MI355_REC_DELTA ? run_rows<T, MI355_REC_DELTA>(p, s)
+                        : p.a.kind == MI355_REC_WKV ? run_rows<T, MI355_REC_WKV>(p, s)
+                                                    : run_rows<T, MI355_REC_GLA>(p, s)) {
         return rc;
     }
     if (p.a.kind == MI355_REC_DELTA && (chunks || p.b.max_count > 1)) {
@@ -220,7 +237,7 @@ extern "C" int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_ba
     MI355_CHECK_ARG(b->row0 && b->count && b->slot && b->pos, MI355_E_ARG, "recurrent: null batch");
     MI355_CHECK_ARG(b->rows > 0 && b->seqs > 0 && b->seqs <= 65535 && b->seqs <= b->rows && b->max_count > 0, MI355_E_SHAPE,
                     "recurrent: bad batch (%d rows, %d sequences)", b->rows, b->seqs);
-    MI355_CHECK_ARG(a->kind == MI355_REC_DELTA || a->kind == MI355_REC_GLA, MI355_E_ARG, "recurrent: bad kind %d", a->kind);
+    MI355_CHECK_ARG(a->kind >= MI355_REC_DELTA && a->kind <= MI355_REC_WKV, MI355_E_ARG, "recurrent: bad kind %d", a->kind);
     MI355_CHECK_ARG(a->dtype == MI355_F32 || a->dtype == MI355_BF16, MI355_E_DTYPE, "recurrent: dtype must be f32 or bf16");
     MI355_CHECK_ARG(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim > 0 && a->vdim > 0, MI355_E_SHAPE,
                     "recurrent: bad heads %d / %d or sizes %d / %d", a->heads, a->kv_heads, a->dim, a->vdim);
@@ -230,10 +247,11 @@ extern "C" int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_ba
     else
         MI355_CHECK_ARG(a->rank > 0 && a->rank <= kMaxRank && a->a2 && a->a2_bias && a->kv_heads == a->heads, MI355_E_ARG,
                         "recurrent: gated linear attention needs its decay projection (rank 1..%d)", kMaxRank);
+    MI355_CHECK_ARG(a->kind != MI355_REC_WKV || a->bonus, MI355_E_ARG, "recurrent: WKV needs its bonus");
     RecParams p;
     p.a = *a;
     p.b = *b;
-    if (a->kind == MI355_REC_GLA) p.a.taps = 1;
+    if (a->kind != MI355_REC_DELTA) p.a.taps = 1;
     p.parts = p.slices = 1;
     return a->dtype == MI355_F32 ? run<float>(p, (hipStream_t)stream) : run<bf16_t>(p, (hipStream_t)stream);
 }

@@ -7,11 +7,12 @@
 //          O = diag(e^G) Q S_0 + P U,                      P_ij = e^(G_i - G_j) q_i . k_j         (j <= i)
 //          S = e^(G_end) S_0 + K^T diag(e^(G_end - G)) U
 //   gla    U = V,  e^(G_i - G_j) acts per key channel inside the products,  O = (Q e^G) S_0 + P V,  S = diag(e^(G_end)) S_0 + (K e^(G_end - G))^T V
+//   wkv    as gla, but row i reads the state in front of it: e^(G_(i-1) - G_j) and Q e^(G_(i-1)), and P_ii = sum q_i u k_i
 //
 // Every exponent is <= 0.  Launches of a step (each over all chunks at once but the scan):
 //   delta_qk_kernel    convolutions, unit norms; Q, K^T, K K^T, Q K^T per key head
 //   delta_head_kernel  decays, T = (I + A)^-1 by 16 x 16 blocks, U0 = T diag(beta) V, W = T diag(beta e^G) K, P per head
-//   gla_prep_kernel    decays, Q e^G, (K e^(G_end - G))^T, P (off-diagonal 16 x 16 blocks anchored at the row block's first row), V^T
+//   gla_prep_kernel    gla, wkv: decays, Q e^G, (K e^(G_end - G))^T, P (off-diagonal 16 x 16 blocks anchored at the row block's first row), V^T
 //   scan_kernel        one workgroup per (sequence, head, 16 columns): U = U0 - W S_0, S; the state in accumulator registers
 //   chunk_out_kernel   O, output norm, gate
 //
@@ -300,10 +301,10 @@ __global__ __launch_bounds__(256) void delta_head_kernel(const ChunkParams p) {
     }
 }
 
-// ------------------------------------------------------------------------------------ gla: per head
+// ------------------------------------------------------------------------------------ gla, wkv: per head
 // 256 threads; key channels in slices of 64.  LDS: q, k, G [64 rows][68], low-rank rows [64][rank], sums
 constexpr int kCh = 64;
-template <typename T>
+template <typename T, int KIND>
 __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
     const mi355_recurrent_args& a = p.r.a;
     extern __shared__ __attribute__((aligned(16))) float sm[];
@@ -317,7 +318,8 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
     float* k = q + kC * kP;
     float* G = k + kC * kP;
     float* seg = G + kC * kP;       // [4][64]
-    float* lr = seg + 4 * kCh;      // [rank][64]
+    float* us = seg + 4 * kCh;      // [64] wkv: bonus
+    float* lr = us + kCh;           // [rank][64]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c16 = lane & 15, g = lane >> 4;
     const T* rows = (const T*)a.proj + (int64_t)(p.r.b.row0[seq] + t0) * a.ld;
@@ -325,7 +327,8 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
     const int64_t hi = (int64_t)(chunk_base(p, seq) + chunk) * a.heads + head;
     for (int i = tid; i < kC * rank; i += 256) {
         const int t = i / rank, r = i - t * rank;
-        lr[r * kC + t] = t < n ? to_f32<T>(rows[(int64_t)t * a.ld + a.off_a + r]) : 0.f;
+        const float lv = t < n ? to_f32<T>(rows[(int64_t)t * a.ld + a.off_a + r]) : 0.f;
+        lr[r * kC + t] = KIND == MI355_REC_WKV ? tanhf(lv) : lv;
     }
     float* oq = p.s.q + hi * kC * DP;
     float* okt = p.s.kt + hi * DP * kC;
@@ -365,14 +368,22 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
 #pragma unroll
             for (int e = 0; e < 16; ++e) {
                 const int t = sb * 16 + e;
-                s += ok && t < n ? -softplus_f32(-z[e]) * a.inv_tau : 0.f;
+                s += !(ok && t < n) ? 0.f : KIND == MI355_REC_WKV ? wkv_log_decay(z[e]) : -softplus_f32(-z[e]) * a.inv_tau;
                 G[t * kP + c] = s;   // sums from the block's first row on
                 q[t * kP + c] = ok && t < n ? to_f32<T>(qv[e]) * a.q_scale : 0.f;
                 k[t * kP + c] = ok && t < n ? to_f32<T>(kv[e]) : 0.f;
             }
             seg[sb * kCh + c] = s;
+            if constexpr (KIND == MI355_REC_WKV) {
+                if (sb == 0) us[c] = ok ? a.bonus[head * dim + ch] : 0.f;
+            }
         }
         __syncthreads();
+        // what row i's query sees of the decays since its block's first row: up to its own row, or (wkv) to the row in front of it
+        auto q_sum = [&](int i, int c) {
+            if constexpr (KIND == MI355_REC_WKV) return (i & 15) == 0 ? zero4() : *(const f32x4*)(G + (i - 1) * kP + c);
+            return *(const f32x4*)(G + i * kP + c);
+        };
         // ---- diagonal blocks: wave = block, lane group g and c16 = column j, rows 4 rr + g
 #pragma unroll 2
         for (int c = 0; c < kCh; c += 4) {
@@ -381,9 +392,16 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
 #pragma unroll
             for (int rr = 0; rr < 4; ++rr) {
                 const int i = wave * 16 + rr * 4 + g;
-                const f32x4 qi = *(const f32x4*)(q + i * kP + c), gi = *(const f32x4*)(G + i * kP + c);
+                const f32x4 qi = *(const f32x4*)(q + i * kP + c), gi = q_sum(i, c);
+                if constexpr (KIND == MI355_REC_WKV) {
+                    const bool own = i == j;
+                    const f32x4 u4 = *(const f32x4*)(us + c);
 #pragma unroll
-                for (int e = 0; e < 4; ++e) dg[rr] += qi[e] * kj[e] * exp_f32(fminf(gi[e] - gj[e], 0.f));  // (j > i: dropped at the end)
+                    for (int e = 0; e < 4; ++e) dg[rr] += qi[e] * kj[e] * (own ? u4[e] : exp_f32(fminf(gi[e] - gj[e], 0.f)));
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) dg[rr] += qi[e] * kj[e] * exp_f32(fminf(gi[e] - gj[e], 0.f));  // (j > i: dropped at the end)
+                }
             }
         }
         // ---- off-diagonal blocks (I, J): q_i e^(G_i - start of I) against k_j e^(start of I - G_j)
@@ -394,7 +412,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
                 f32x4 gap = *(const f32x4*)(seg + J * kCh + c) - *(const f32x4*)(G + j * kP + c);  // from j to the end of block J
                 for (int m = J + 1; m < wave; ++m) gap += *(const f32x4*)(seg + m * kCh + c);
                 f32x4 av = *(const f32x4*)(q + i * kP + c), bv = *(const f32x4*)(k + j * kP + c);
-                const f32x4 gi = *(const f32x4*)(G + i * kP + c);
+                const f32x4 gi = q_sum(i, c);
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     av[e] *= exp_f32(gi[e]);
@@ -414,7 +432,8 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const ChunkParams p) {
 #pragma unroll
                 for (int e = 0; e < 16; ++e) {
                     const int t = wave * 16 + e;
-                    oq[t * DP + c0 + c] = q[t * kP + c] * exp_f32(before + G[t * kP + c]);
+                    const float own = KIND == MI355_REC_WKV ? (e == 0 ? 0.f : G[(t - 1) * kP + c]) : G[t * kP + c];
+                    oq[t * DP + c0 + c] = q[t * kP + c] * exp_f32(before + own);
                 }
             }
         }
@@ -649,7 +668,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
                 const int n = (wave + 4 * v) * 16 + c16;
                 if (n >= a.vdim) continue;
                 const float gate = silu_f32(to_f32<T>(rows[(int64_t)t * a.ld + a.off_g + head * a.vdim + n]));
-                y[(int64_t)t * a.ldy + head * a.vdim + n] = from_f32<T>(o[rb][v][r] * rinv * a.head_norm[n] * gate);
+                y[(int64_t)t * a.ldy + head * a.vdim + n] = from_f32<T>(o[rb][v][r] * rinv * a.head_norm[head * a.norm_ld + n] * gate);
             }
         }
 }
@@ -710,9 +729,14 @@ int run_group(const ChunkParams& p, int seqs, hipStream_t s) {
         if (int rc = launch_scan<MI355_REC_DELTA>(p, seqs, s)) return rc;
         return launch_out<T, MI355_REC_DELTA>(p, heads, s);
     }
-    const size_t lds = ((size_t)3 * kC * kP + 4 * kCh + (size_t)kC * a.rank) * 4;
-    if (int rc = set_lds(gla_prep_kernel<T>, lds)) return rc;
-    hipLaunchKernelGGL(gla_prep_kernel<T>, heads, dim3(256), lds, s, p);
+    const size_t lds = ((size_t)3 * kC * kP + 5 * kCh + (size_t)kC * a.rank) * 4;
+    if (a.kind == MI355_REC_WKV) {
+        if (int rc = set_lds(gla_prep_kernel<T, MI355_REC_WKV>, lds)) return rc;
+        hipLaunchKernelGGL((gla_prep_kernel<T, MI355_REC_WKV>), heads, dim3(256), lds, s, p);
+    } else {
+        if (int rc = set_lds(gla_prep_kernel<T, MI355_REC_GLA>, lds)) return rc;
+        hipLaunchKernelGGL((gla_prep_kernel<T, MI355_REC_GLA>), heads, dim3(256), lds, s, p);
+    }
     MI355_LAUNCH_CHECK();
     if (int rc = launch_scan<MI355_REC_GLA>(p, seqs, s)) return rc;
     return launch_out<T, MI355_REC_GLA>(p, heads, s);

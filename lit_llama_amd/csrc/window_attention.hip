@@ -1,12 +1,13 @@
-// Causal attention over a sliding window: grouped key / value heads, different key and value sizes, interleaved rotation of the first
-// rot_dims dimensions, queries and keys over their root mean square, first rows that stay visible, a sink in the softmax sum, sigmoid gates
-// per head or per value.  A slot's cache is, per key head, `kept` rows for the first positions and a ring for the others.  A layer lends
+// Causal attention over a sliding window or a chunk: grouped key / value heads, different key and value sizes, interleaved rotation of
+// rot_dims dimensions, queries, keys and values over their root mean square, first rows that stay visible, a factor and a distance bias per
+// head, a sink in the softmax sum, sigmoid gates per head or per value.  A slot's cache is, per key head, `kept` rows for the first positions and a ring for the others.  A layer lends
 // its keys and values to later ones, which read its cache (and, in a prompt step, its prepared rows).
 //
 //   window_rows_kernel    one workgroup per (row, key head, split of the keys): decode steps of any size (q and the row's own k are
 //                         normalised and rotated here, the cache row is written here: one launch per layer), f32 models, odd head sizes
 //   window_tiles_kernel   128 queries of one head per workgroup on the matrix cores (bf16 prompt steps)
-//   prepare_keys_kernel   prompt steps: k rows normalised and rotated in front of either kernel, in place or (a lender's) to kv_rows
+//   prepare_keys_kernel   prompt steps: k rows normalised and rotated, v rows normalised in front of either kernel, in place or (a lender's)
+//                         to kv_rows
 //   ring_write_kernel     prompt steps: the first and the last rows of every portion enter the cache, behind either kernel (which reads
 //                         the rows of earlier portions from it) and, of a lender, behind its last borrower
 //
@@ -25,6 +26,8 @@ constexpr double kInvTwoPi = 0.15915494309189533577;
 
 // row of position p in a slot's cache
 __device__ __forceinline__ int cache_row(const mi355_window_attn_args& a, int p) { return p < a.kept ? p : a.kept + (p - a.kept) % a.ring; }
+// first position of the window or chunk of the row at position p
+__device__ __forceinline__ int first_seen(const mi355_window_attn_args& a, int p) { return a.chunked ? p - p % a.window : p - a.window + 1; }
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 // turn of (u, v) by pos * inv_freq: the angle is reduced in f64, so far positions keep f32 accuracy
@@ -91,8 +94,9 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     const int dim = a.dim, vdim = a.vdim;
     float* q = (float*)smem;                      // [HT][dim], scaled
     float* kn = q + (HT * dim + 3) / 4 * 4;                     // [dim]: the row's own key, as the ring stores it
-    float* sc = kn + (dim + 3) / 4 * 4;           // [kKeys][HT]
-    float* stat = sc + HT * kKeys;                // [3][HT]: maximum, sum, correction
+    float* vn = kn + (dim + 3) / 4 * 4;           // [vdim, padded to VE]: the row's own value over its root mean square (unit_v)
+    float* sc = vn + (vdim + 7) / 8 * 8;          // [kKeys][HT]
+    float* stat = sc + HT * kKeys;                // [4][HT]: maximum, sum, correction, slope of the distance bias
     float* red = stat + 4 * HT;                   // [key lanes][HT][columns]: at most kRowThreads HT VE
     __shared__ int s_seq;
 
@@ -118,7 +122,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     // Numbers from g_cur on are rows of the step (a prompt's), those before lie in the cache, in three runs: first positions, ring, ring
     // behind its wrap
     const int n_first = min(a.keep, pos + 1);
-    const int w0 = max(pos - a.window + 1, n_first);
+    const int w0 = max(first_seen(a, pos), n_first);
     const int n_keys = n_first + pos - w0 + 1;
     const int w_shift = w0 - n_first;                              // position of number g >= n_first, minus g
     const int w_row = w0 < a.kept ? w0 : a.kept + (w0 - a.kept) % a.ring;
@@ -145,7 +149,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
         for (int i = 0; i < kHeld; ++i)
 #pragma unroll
             for (int e = 0; e < 2; ++e) v[i][e] = at(2 * (lane + 32 * i) + e);
-        float f = key ? 1.f : a.scale;
+        float f = key ? 1.f : a.head_scale != nullptr ? a.scale * a.head_scale[h0 + h] : a.scale;
         if (a.unit_qk) {
 #pragma unroll
             for (int i = 0; i < kHeld; ++i) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1];
@@ -153,9 +157,9 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             f /= sqrtf(group_sum(ss, 32) / (float)dim + a.unit_eps);
         }
         auto put = [&](int pi, float u, float w) {
-            if (2 * pi < a.rot_dims) {
+            if (const int ri = pi - a.rot_at / 2; ri >= 0 && 2 * ri < a.rot_dims) {
                 float c, s;
-                pair_cos_sin(pos, a.inv_freq[pi], c, s);
+                pair_cos_sin(pos, a.inv_freq[ri], c, s);
                 const float r = u * c - w * s;
                 w = w * c + u * s;
                 u = r;
@@ -182,12 +186,26 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     if (owner && ht == 0) {
         T* vw = vcache + row_of(n_keys - 1) * (unsigned)vdim;
         const T* vs = prow + a.off_v + (int64_t)kvh * vdim;
-        for (int d = tid; d < vdim; d += kRowThreads) vw[d] = vs[d];
+        if (!a.unit_v)
+            for (int d = tid; d < vdim; d += kRowThreads) vw[d] = vs[d];
+    }
+    if (owner && a.unit_v && tid < 64) {
+        T* vw = vcache + row_of(n_keys - 1) * (unsigned)vdim;
+        const T* vs = prow + a.off_v + (int64_t)kvh * vdim;
+        float ss = 0.f;
+        for (int d = tid; d < vdim; d += 64) ss += to_f32<T>(vs[d]) * to_f32<T>(vs[d]);
+        const float r = 1.0f / sqrtf(group_sum(ss, 64) / (float)vdim + a.unit_eps);
+        for (int d = tid; d < (vdim + 7) / 8 * 8; d += 64) {
+            const T o = from_f32<T>(d < vdim ? to_f32<T>(vs[d]) * r : 0.f);
+            vn[d] = to_f32<T>(o);
+            if (ht == 0 && d < vdim) vw[d] = o;
+        }
     }
     if (tid < HT) {  // the sink is a key without a value: a score of its own in the first split
         const bool sink = a.sink != nullptr && split == 0 && tid < nh;
         stat[tid] = sink ? a.sink[h0 + tid] : -INFINITY;
         stat[HT + tid] = sink ? 1.f : 0.f;
+        stat[3 * HT + tid] = a.slope != nullptr && tid < nh ? a.slope[h0 + tid] : 0.f;
     }
     __syncthreads();
 
@@ -217,7 +235,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             for (int d = l16 * VE; d < dim; d += 16 * VE) {
                 float kv[4][VE];
 #pragma unroll
-                for (int u = 0; u < 4; ++u) load_vec<T, VE>(src[u] + d, kv[u]);
+                for (int u = 0; u < 4; ++u) load_vec(src[u] + d, kv[u]);
 #pragma unroll
                 for (int h = 0; h < HT; ++h)
                     if (h < nh) {
@@ -235,9 +253,11 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
 #pragma unroll
                 for (int h = 0; h < HT; ++h) dot[u][h] = group_sum(dot[u][h], 16);
                 if (l16 == 0 && kk < nk && !(owner && kb + kk == n_keys - 1)) {
+                    const int g = kb + kk;
+                    const float dist = (float)(pos - (g < n_first ? g : g + w_shift));
 #pragma unroll
                     for (int h = 0; h < HT; ++h)
-                        if (h < nh) sc[kk * HT + h] = dot[u][h];
+                        if (h < nh) sc[kk * HT + h] = dot[u][h] - stat[3 * HT + h] * dist;
                 }
             }
         }
@@ -279,11 +299,11 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
 #pragma unroll
                 for (int e = 0; e < VE; ++e) acc[h][e] *= corr;
             }
-            auto add = [&](int kk, const T* src) {
+            auto add = [&](int kk, auto src) {
                 float v[VE], w[HT];
 #pragma unroll
                 for (int h = 0; h < HT; ++h) w[h] = sc[kk * HT + h];
-                load_vec<T, VE>(src + col * VE, v);
+                load_vec(src + col * VE, v);
 #pragma unroll
                 for (int h = 0; h < HT; ++h)
                     if (h < nh) {
@@ -292,7 +312,10 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
                     }
             };
             const int nv = owner && kb + nk == n_keys ? nk - 1 : nk;  // (the own value is not in the cache yet)
-            if (nv < nk && kl == 0) add(nk - 1, prow + a.off_v + (int64_t)kvh * vdim);
+            if (nv < nk && kl == 0) {
+                if (a.unit_v) add(nk - 1, (const float*)vn);
+                else add(nk - 1, prow + a.off_v + (int64_t)kvh * vdim);
+            }
 #pragma unroll 4
             for (int kk = kl; kk < nv; kk += n_kl) {
                 const int g = kb + kk;
@@ -371,14 +394,21 @@ __global__ __launch_bounds__(256) void prepare_keys_kernel(const WinParams p) {
     const int seq = blockIdx.y, it = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     const int i = it / a.kv_heads, g = it - i * a.kv_heads;
     if (i >= p.b.count[seq]) return;
-    const int pos = p.b.pos[seq] + i, half = a.rot_dims / 2;
+    const int pos = p.b.pos[seq] + i, half = a.rot_dims / 2, rot0 = a.rot_at / 2;
     const int64_t row = p.b.row0[seq] + i;
     const T* src = (const T*)a.proj + row * a.ld;
     const bool moved = a.role == MI355_KV_LENDS;
     const T *k = src + a.off_k + (int64_t)g * a.dim, *v = src + a.off_v + (int64_t)g * a.vdim;
     T *o = (T*)p.krows + row * p.ld_rows + (int64_t)g * a.dim, *vo = (T*)p.vrows + row * p.ld_rows + (int64_t)g * a.vdim;
-    if (moved)
+    if (a.unit_v) {
+        float ss = 0.f;
+        for (int d = lane; d < a.vdim; d += 64) ss += to_f32<T>(v[d]) * to_f32<T>(v[d]);
+        const float r = 1.0f / sqrtf(group_sum(ss, 64) / (float)a.vdim + a.unit_eps);
+        for (int d = lane; d < a.vdim; d += 64) vo[d] = from_f32<T>(to_f32<T>(v[d]) * r);
+    } else if (moved) {
         for (int d = lane; d < a.vdim; d += 64) vo[d] = v[d];
+    }
+    if (!moved && a.rot_dims == 0 && !a.unit_qk) return;
     const int pairs = (a.dim + 1) / 2;  // (an odd size: the last pair is one value)
     const int p0 = lane < pairs ? lane : pairs - 1;
     const float k0 = to_f32<T>(k[2 * p0]), k1 = 2 * p0 + 1 < a.dim ? to_f32<T>(k[2 * p0 + 1]) : 0.f;
@@ -394,9 +424,9 @@ __global__ __launch_bounds__(256) void prepare_keys_kernel(const WinParams p) {
     for (int pi = lane; pi < pairs; pi += 64) {
         const bool two = 2 * pi + 1 < a.dim;
         float u = (pi == lane ? k0 : to_f32<T>(k[2 * pi])) * rms, w = (pi == lane ? k1 : two ? to_f32<T>(k[2 * pi + 1]) : 0.f) * rms;
-        if (pi < half) {
+        if (pi >= rot0 && pi - rot0 < half) {
             float c, s;
-            pair_cos_sin(pos, a.inv_freq[pi], c, s);
+            pair_cos_sin(pos, a.inv_freq[pi - rot0], c, s);
             const float r = u * c - w * s;
             w = w * c + u * s;
             u = r;
@@ -460,18 +490,20 @@ __device__ __forceinline__ float sigmoid_fast(float z) {  // (in front of a roun
 }
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 
-template <int D>  // both head sizes padded to D (a multiple of 32)
-constexpr int tiles_lds() { return 2 * (kBK * D * 2 + D * kVtRow); }
+template <int D, int DV>  // key and value sizes padded to D and DV (multiples of 32)
+constexpr int tiles_lds() { return 2 * (kBK * D * 2 + DV * kVtRow); }
 
-template <int D>
+template <int D, int DV>
 __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(const WinParams p) {
     const mi355_window_attn_args& a = p.a;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     constexpr int kCols = D / 8;                       // 16-B columns of a key row
     constexpr int kKItems = kBK * kCols / 256;         // K chunks per thread
-    constexpr int kVItems = (16 * kCols + 255) / 256;  // V items per thread: (run of 4 keys, column)
-    constexpr int kKTile = kBK * D * 2, kVTile = D * kVtRow;
-    constexpr int kSwz = kCols < 16 ? kCols - 1 : 15;
+    constexpr int kVCols = DV / 8;
+    constexpr int kVItems = (16 * kVCols + 255) / 256;  // V items per thread: (run of 4 keys, column)
+    constexpr int kKTile = kBK * D * 2, kVTile = DV * kVtRow;
+    constexpr bool kPow2 = (kCols & (kCols - 1)) == 0;
+    constexpr int kSwz = !kPow2 ? 7 : kCols < 16 ? kCols - 1 : 15;  // (the swizzled column stays in the row: whole groups of 8)
     const int seq = blockIdx.z;
     const int cnt = p.b.count[seq];
     // an XCD (block index mod 8) takes the query blocks of neighbouring heads: their key head stays in its L2
@@ -494,16 +526,17 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const bf16_t* proj = (const bf16_t*)a.proj;
     const int q_first = pos0 + qb * kBQ, q_last = pos0 + min(qb * kBQ + kBQ, cnt) - 1;
     // key steps: those of the first `keep` positions that lie in front of the window, then the window's
-    const int kb0 = max(0, q_first - a.window + 1) / kBK, kb1 = q_last / kBK + 1;
+    const int kb0 = max(0, first_seen(a, q_first)) / kBK, kb1 = q_last / kBK + 1;
     const int n_first = min((a.keep + kBK - 1) / kBK, kb0);
     // the wave's own range, for the masks
     const int w_first = min(pos0 + qb * kBQ + wave * 32, pos0 + cnt - 1), w_last = min(w_first + 31, pos0 + cnt - 1);
+    const int q_lo = first_seen(a, q_pos), w_first_lo = first_seen(a, w_first), w_last_lo = first_seen(a, w_last);
 
     // ---- Q^T operands: q[16 ks + 8 hh .. + 8), rotated, scaled to the exp2 domain, rounded once
     bf16x8 bq[D / 16];
     {
         const bf16_t* src = proj + (int64_t)(row0 + q_row) * a.ld + a.off_q + (int64_t)h * a.dim;
-        float qs = a.scale * 1.44269504088896340736f;
+        float qs = (a.head_scale != nullptr ? a.scale * a.head_scale[h] : a.scale) * 1.44269504088896340736f;
         if (a.unit_qk) {  // lanes c and c + 32 hold the row between them
             float ss = 0.f;
 #pragma unroll
@@ -511,7 +544,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                 const int d0 = 16 * ks + 8 * hh;
                 if (d0 < a.dim) {
                     float v[8];
-                    load_vec<bf16_t, 8>(src + d0, v);
+                    load_vec(src + d0, v);
 #pragma unroll
                     for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
                 }
@@ -525,13 +558,13 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             u32x4 o = {0u, 0u, 0u, 0u};
             if (d0 < a.dim) {  // (dim % 8 == 0)
                 float v[8];
-                load_vec<bf16_t, 8>(src + d0, v);
+                load_vec(src + d0, v);
 #pragma unroll
                 for (int e = 0; e < 8; e += 2) {
                     float u = v[e], w = v[e + 1];
-                    if (d0 + e < a.rot_dims) {
+                    if (const int rd = d0 + e - a.rot_at; rd >= 0 && rd < a.rot_dims) {
                         float cs, sn;
-                        pair_cos_sin(q_pos, a.inv_freq[(d0 + e) >> 1], cs, sn);
+                        pair_cos_sin(q_pos, a.inv_freq[rd >> 1], cs, sn);
                         const float r = u * cs - w * sn;
                         w = w * cs + u * sn;
                         u = r;
@@ -545,20 +578,25 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const int64_t slot_head = (int64_t)p.b.slot[seq] * a.kv_heads + kvh;
     const bf16_t* kcache = (const bf16_t*)a.kring + slot_head * (a.kept + a.ring) * a.dim;
     const bf16_t* vcache = (const bf16_t*)a.vring + slot_head * (a.kept + a.ring) * a.vdim;
-    const bf16_t* kcur = (const bf16_t*)p.krows + (int64_t)row0 * p.ld_rows + (int64_t)kvh * a.dim;
-    const bf16_t* vcur = (const bf16_t*)p.vrows + (int64_t)row0 * p.ld_rows + (int64_t)kvh * a.vdim;
+    // rows of the step, from position k_pos0 on; role MI355_KV_ROWS: every position's, the last kdim .. dim of a key from the common tail
+    const bool all = a.role == MI355_KV_ROWS;
+    const int64_t k_row0 = all ? seq * a.rows_per_seq : row0;
+    const int k_pos0 = all ? 0 : pos0, kdim = a.dim - a.tail_dims;
+    const bf16_t* kcur = (const bf16_t*)p.krows + k_row0 * p.ld_rows + (int64_t)kvh * kdim;
+    const bf16_t* vcur = (const bf16_t*)p.vrows + k_row0 * p.ld_rows + (int64_t)kvh * a.vdim;
+    const bf16_t* tail = (const bf16_t*)a.key_tail + (int64_t)p.b.slot[seq] * a.tail_slot - kdim;  // (read from column kdim on)
     const int p_last = pos0 + cnt - 1;
     u32x4 kreg[kKItems], vreg[kVItems][4];
     const u32x4 zero4 = {0u, 0u, 0u, 0u};
     const int t_key = threadIdx.x / kCols, t_col = threadIdx.x % kCols, t_run = threadIdx.x & 15, t_vcol = threadIdx.x >> 4;
     const bool k_in = t_col * 8 < a.dim;
     auto load_tile = [&](int kb) {
-        if (kb * kBK >= pos0 && kb * kBK + kBK - 1 <= p_last) {  // all of the step's own rows: one multiply per thread
+        if (kPow2 && a.tail_dims == 0 && kb * kBK >= k_pos0 && kb * kBK + kBK - 1 <= p_last) {  // all of the step's own rows: one multiply per thread
             const unsigned ld = (unsigned)p.ld_rows;
-            const unsigned ko = (unsigned)(kb * kBK + t_key - pos0) * ld + t_col * 8;
+            const unsigned ko = (unsigned)(kb * kBK + t_key - k_pos0) * ld + t_col * 8;
 #pragma unroll
             for (int i = 0; i < kKItems; ++i) kreg[i] = *(const u32x4*)(kcur + (k_in ? ko + (unsigned)i * (256 / kCols) * ld : 0u));
-            const unsigned vo = (unsigned)(kb * kBK + t_run * 4 - pos0) * ld;
+            const unsigned vo = (unsigned)(kb * kBK + t_run * 4 - k_pos0) * ld;
 #pragma unroll
             for (int i = 0; i < kVItems; ++i) {
                 const int col = t_vcol + 16 * i;
@@ -570,7 +608,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
 #pragma unroll
                 for (int i = 0; i < kKItems; ++i) kreg[i] = zero4;
             }
-            if (D != a.vdim) {
+            if (DV != a.vdim) {
 #pragma unroll
                 for (int i = 0; i < kVItems; ++i)
                     if ((t_vcol + 16 * i) * 8 >= a.vdim) {
@@ -586,7 +624,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             const int kp = kb * kBK + key;
             kreg[i] = zero4;
             if (col * 8 < a.dim && kp <= p_last) {
-                const bf16_t* src = kp >= pos0 ? kcur + (int64_t)(kp - pos0) * p.ld_rows : kcache + (int64_t)cache_row(a, kp) * a.dim;
+                const bf16_t* src = col * 8 >= kdim ? tail + (int64_t)kp * a.ld_tail
+                                    : kp >= k_pos0 ? kcur + (int64_t)(kp - k_pos0) * p.ld_rows
+                                                   : kcache + (int64_t)cache_row(a, kp) * a.dim;
                 kreg[i] = *(const u32x4*)(src + col * 8);
             }
         }
@@ -597,8 +637,8 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             for (int r = 0; r < 4; ++r) {
                 const int kp = kb * kBK + run * 4 + r;
                 vreg[i][r] = zero4;
-                if (col < kCols && col * 8 < a.vdim && kp <= p_last) {
-                    const bf16_t* src = kp >= pos0 ? vcur + (int64_t)(kp - pos0) * p.ld_rows : vcache + (int64_t)cache_row(a, kp) * a.vdim;
+                if (col < kVCols && col * 8 < a.vdim && kp <= p_last) {
+                    const bf16_t* src = kp >= k_pos0 ? vcur + (int64_t)(kp - k_pos0) * p.ld_rows : vcache + (int64_t)cache_row(a, kp) * a.vdim;
                     vreg[i][r] = *(const u32x4*)(src + col * 8);
                 }
             }
@@ -615,7 +655,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
 #pragma unroll
         for (int i = 0; i < kVItems; ++i) {
             const int it = i * 256 + threadIdx.x, run = it & 15, col = it >> 4;
-            if (col >= kCols) continue;
+            if (col >= kVCols) continue;
             const int G = run >> 2, r = run & 3;
             const int pbyte = (G * 16 + 4 * ((r & 1) * 2 + (r >> 1))) * 2;
 #pragma unroll
@@ -633,11 +673,12 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             }
         }
     };
-    f32x16 acc[D / 32];
+    f32x16 acc[DV / 32];
 #pragma unroll
-    for (int dt = 0; dt < D / 32; ++dt)
+    for (int dt = 0; dt < DV / 32; ++dt)
 #pragma unroll
         for (int i = 0; i < 16; ++i) acc[dt][i] = 0.f;
+    const float slope2 = a.slope != nullptr ? a.slope[h] * 1.44269504088896340736f : 0.f;
     float m_run = -1.0e30f, l_run = 0.f;
     if (a.sink != nullptr) {  // a key without a value; one of the two lanes of a query counts it
         m_run = a.sink[h] * 1.44269504088896340736f;
@@ -654,7 +695,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
         const char* kt = smem + buf * kKTile;
         const char* vt = smem + 2 * kKTile + buf * kVTile;
         // a wave none of whose queries sees this step leaves it out (it still stages the next tile)
-        const bool seen = kb * kBK <= w_last && (kb * kBK + kBK - 1 > w_first - a.window || kb * kBK < a.keep);
+        const bool seen = kb * kBK <= w_last && (kb * kBK + kBK - 1 >= w_first_lo || kb * kBK < a.keep);
         if (seen) {
             f32x16 st[2];
 #pragma unroll
@@ -669,13 +710,20 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                     const bf16x8 ka = *(const bf16x8*)(kt + key * (D * 2) + (((2 * ks + hh) ^ (key & kSwz)) << 4));
                     st[t2] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka, bq[ks], st[t2], 0, 0, 0);
                 }
-            if (kb * kBK + kBK - 1 > w_first || kb * kBK <= w_last - a.window) {  // wave-uniform: the step touches an edge
+            if (slope2 != 0.f) {  // (log2 e slope (i - j) is taken off)
+                const float at = slope2 * (float)(kb * kBK + 4 * hh - q_pos);
+#pragma unroll
+                for (int t2 = 0; t2 < 2; ++t2)
+#pragma unroll
+                    for (int i = 0; i < 16; ++i) st[t2][i] += at + slope2 * (float)(t2 * 32 + (i & 3) + 8 * (i >> 2));
+            }
+            if (kb * kBK + kBK - 1 > w_first || kb * kBK < w_last_lo) {  // wave-uniform: the step touches an edge
 #pragma unroll
                 for (int t2 = 0; t2 < 2; ++t2)
 #pragma unroll
                     for (int i = 0; i < 16; ++i) {
                         const int kp = kb * kBK + t2 * 32 + (i & 3) + 8 * (i >> 2) + 4 * hh;
-                        st[t2][i] = (kp <= q_pos && (kp > q_pos - a.window || kp < a.keep)) ? st[t2][i] : -1.0e30f;
+                        st[t2][i] = (kp <= q_pos && (kp >= q_lo || kp < a.keep)) ? st[t2][i] : -1.0e30f;
                     }
             }
             // (inline assembly gets no wait states behind the matrix instruction that wrote its operands: 20 here cover the longest)
@@ -693,7 +741,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                 l_run *= corr;
                 m_run = m_new;
 #pragma unroll
-                for (int dt = 0; dt < D / 32; ++dt)
+                for (int dt = 0; dt < DV / 32; ++dt)
 #pragma unroll
                     for (int i = 0; i < 16; ++i) acc[dt][i] *= corr;
             }
@@ -712,7 +760,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             for (int sg = 0; sg < 4; ++sg) {
                 const bf16x8 pf = __builtin_bit_cast(bf16x8, pb[sg >> 1][sg & 1]);
 #pragma unroll
-                for (int dt = 0; dt < D / 32; ++dt) {
+                for (int dt = 0; dt < DV / 32; ++dt) {
                     const bf16x8 va = *(const bf16x8*)(vt + (dt * 32 + c) * kVtRow + sg * 32 + hh * 16);
                     acc[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(va, pf, acc[dt], 0, 0, 0);
                 }
@@ -730,7 +778,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
         const bool each = a.off_g >= 0 && a.gate_values;
         bf16_t* y = (bf16_t*)a.y + (int64_t)(row0 + q_row) * a.ldy + (int64_t)h * a.vdim;
 #pragma unroll
-        for (int dt = 0; dt < D / 32; ++dt)
+        for (int dt = 0; dt < DV / 32; ++dt)
 #pragma unroll
             for (int g = 0; g < 4; ++g) {
                 const int d = dt * 32 + 8 * g + 4 * hh;
@@ -753,12 +801,13 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     }
 }
 
-template <int D>
+template <int D, int DV>
 int launch_tiles(const WinParams& p, hipStream_t s) {
-    static hipError_t e = hipFuncSetAttribute((const void*)window_tiles_kernel<D>, hipFuncAttributeMaxDynamicSharedMemorySize, tiles_lds<D>());
+    constexpr int lds = tiles_lds<D, DV>();
+    static hipError_t e = hipFuncSetAttribute((const void*)window_tiles_kernel<D, DV>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     MI355_CHECK_ARG(e == hipSuccess, (int)e, "window_attention: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
     const int q_blocks = (p.b.max_count + kBQ - 1) / kBQ;
-    hipLaunchKernelGGL(window_tiles_kernel<D>, dim3((q_blocks * p.a.heads + 7) / 8 * 8, 1, p.b.seqs), dim3(256), tiles_lds<D>(), s, p);
+    hipLaunchKernelGGL((window_tiles_kernel<D, DV>), dim3((q_blocks * p.a.heads + 7) / 8 * 8, 1, p.b.seqs), dim3(256), lds, s, p);
     MI355_LAUNCH_CHECK();
     return 0;
 }
@@ -777,16 +826,17 @@ bool tiles_fit(const WinParams& p) {
 
 int run_tiles(const WinParams& p, hipStream_t s) {
     const int d = p.a.dim > p.a.vdim ? p.a.dim : p.a.vdim;
-    if (d <= 32) return launch_tiles<32>(p, s);
-    if (d <= 64) return launch_tiles<64>(p, s);
-    if (d <= 128) return launch_tiles<128>(p, s);
-    return launch_tiles<256>(p, s);
+    if (d <= 32) return launch_tiles<32, 32>(p, s);
+    if (d <= 64) return launch_tiles<64, 64>(p, s);
+    if (d <= 128) return launch_tiles<128, 128>(p, s);
+    if (p.a.dim <= 192 && p.a.vdim <= 128) return launch_tiles<192, 128>(p, s);
+    return launch_tiles<256, 256>(p, s);
 }
 
 template <typename T, int HT, int VE, bool FRESH>
 int launch_rows_step(const WinParams& p, int rows, hipStream_t s) {
     const size_t red = (size_t)kRowThreads * HT * VE;
-    const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + 8 + (size_t)HT * kKeys + 4 * HT + red) * 4;
+    const size_t lds = ((size_t)HT * p.a.dim + p.a.dim + p.a.vdim + 16 + (size_t)HT * kKeys + 4 * HT + red) * 4;
     MI355_CHECK_ARG(lds <= 160 * 1024 - 64, MI355_E_SHAPE, "window_attention: head size %d does not fit LDS", p.a.dim);
     if (lds > 64 * 1024) {
         static hipError_t e = hipFuncSetAttribute((const void*)window_rows_kernel<T, HT, VE, FRESH>, hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -853,35 +903,40 @@ int run(WinParams p, hipStream_t s) {
         }
         return 0;
     }
-    if (a.role == MI355_KV_LENDS || (a.role == MI355_KV_OWN && (a.rot_dims > 0 || a.unit_qk))) {
+    if (a.role == MI355_KV_LENDS || (a.role == MI355_KV_OWN && (a.rot_dims > 0 || a.unit_qk || a.unit_v))) {
         hipLaunchKernelGGL(prepare_keys_kernel<T>, dim3((unsigned)(((int64_t)p.b.max_count * a.kv_heads + 3) / 4), p.b.seqs), dim3(256), 0, s, p);
         MI355_LAUNCH_CHECK();
     }
     p.n_split = 1;
     // (a handful of rows per sequence would leave most of a 128-query tile empty)
-    const bool tiles = a.path == 2 || (a.path == 0 && p.b.max_count > 8);
+    const bool tiles = a.path == 2 || a.role == MI355_KV_ROWS || (a.path == 0 && p.b.max_count > 8);
     if (tiles && tiles_fit(p)) {
         if (int rc = run_tiles(p, s)) return rc;
     } else {
-        MI355_CHECK_ARG(a.path != 2, MI355_E_SHAPE, "window_attention: the tile kernel takes bf16 heads of up to 256, multiples of 8");
+        MI355_CHECK_ARG(a.path != 2 && a.role != MI355_KV_ROWS, MI355_E_SHAPE, "window_attention: the tile kernel takes bf16 heads of up to 256, multiples of 8");
         if (int rc = run_rows<T>(p, s)) return rc;
     }
     return a.role == MI355_KV_OWN ? run_cache_write<T>(p, s) : 0;
 }
 
 int make_params(const mi355_window_attn_args* a, const mi355_seq_batch* b, WinParams& p) {
-    MI355_CHECK_ARG(a && b && a->proj && a->kring && a->vring && a->y, MI355_E_ARG, "window_attention: null argument");
+    MI355_CHECK_ARG(a && b && a->proj && a->y && (a->role == MI355_KV_ROWS || (a->kring && a->vring)), MI355_E_ARG, "window_attention: null argument");
     MI355_CHECK_ARG(b->row0 && b->count && b->slot && b->pos, MI355_E_ARG, "window_attention: null batch");
     MI355_CHECK_ARG(b->rows > 0 && b->rows <= 65535 && b->seqs > 0 && b->seqs <= b->rows && b->max_count > 0, MI355_E_SHAPE,
                     "window_attention: bad batch (%d rows, %d sequences)", b->rows, b->seqs);
     MI355_CHECK_ARG(a->dtype == MI355_F32 || a->dtype == MI355_BF16, MI355_E_DTYPE, "window_attention: dtype must be f32 or bf16");
     MI355_CHECK_ARG(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim > 0 && a->vdim > 0, MI355_E_SHAPE,
                     "window_attention: bad heads %d / %d or sizes %d / %d", a->heads, a->kv_heads, a->dim, a->vdim);
-    MI355_CHECK_ARG(a->window > 0 && a->ring > 0 && a->rot_dims >= 0 && a->rot_dims % 2 == 0 && a->rot_dims <= a->dim &&
+    MI355_CHECK_ARG(a->window > 0 && a->ring > 0 && a->rot_dims >= 0 && a->rot_dims % 2 == 0 && a->rot_at >= 0 && a->rot_at % 2 == 0 && a->rot_at + a->rot_dims <= a->dim &&
                         (a->rot_dims == 0 || a->inv_freq),
                     MI355_E_SHAPE, "window_attention: bad window %d, ring %d or rotation %d", a->window, a->ring, a->rot_dims);
     MI355_CHECK_ARG(a->keep >= 0 && a->keep <= a->kept, MI355_E_SHAPE, "window_attention: %d first rows visible, %d cached", a->keep, a->kept);
-    MI355_CHECK_ARG(a->role >= MI355_KV_OWN && a->role <= MI355_KV_BORROWS && (a->role == MI355_KV_OWN || a->kv_rows), MI355_E_ARG,
+    MI355_CHECK_ARG(a->role == MI355_KV_ROWS ? b->max_count > 1 && a->rows_per_seq > 0 && a->tail_dims >= 0 && a->tail_dims < a->dim && a->tail_dims % 8 == 0 &&
+                                                   a->off_v_rows % 8 == 0 && (a->tail_dims == 0 || (a->key_tail && a->ld_tail % 8 == 0 && a->tail_slot % 8 == 0 &&
+                                                                                                    (uintptr_t)a->key_tail % 16 == 0))
+                                             : a->tail_dims == 0,
+                    MI355_E_ARG, "window_attention: bad rows of all positions");
+    MI355_CHECK_ARG(a->role >= MI355_KV_OWN && a->role <= MI355_KV_ROWS && (a->role == MI355_KV_OWN || a->kv_rows), MI355_E_ARG,
                     "window_attention: a lender and its borrowers share kv_rows");
     p.a = *a;
     p.b = *b;
@@ -893,12 +948,16 @@ int make_params(const mi355_window_attn_args* a, const mi355_seq_batch* b, WinPa
         p.krows = (const char*)a->proj + (int64_t)a->off_k * size;
         p.vrows = (const char*)a->proj + (int64_t)a->off_v * size;
         p.ld_rows = a->ld;
+    } else if (a->role == MI355_KV_ROWS) {
+        p.krows = a->kv_rows;
+        p.vrows = (const char*)a->kv_rows + (int64_t)a->off_v_rows * size;
+        p.ld_rows = a->ld_rows;
     } else {
         p.krows = a->kv_rows;
         p.vrows = (const char*)a->kv_rows + (int64_t)a->kv_heads * a->dim * size;
         p.ld_rows = (int64_t)a->kv_heads * (a->dim + a->vdim);
     }
-    MI355_CHECK_ARG((uint64_t)b->max_count * (uint64_t)p.ld_rows < 0xFFFFFFFFull && (uint64_t)b->max_count * (uint64_t)a->ld < 0xFFFFFFFFull &&
+    MI355_CHECK_ARG((uint64_t)(a->role == MI355_KV_ROWS ? a->rows_per_seq : b->max_count) * (uint64_t)p.ld_rows < 0xFFFFFFFFull && (uint64_t)b->max_count * (uint64_t)a->ld < 0xFFFFFFFFull &&
                         (uint64_t)(a->kept + (int64_t)a->ring) * (a->dim > a->vdim ? a->dim : a->vdim) < 0xFFFFFFFFull,
                     MI355_E_SHAPE, "window_attention: %d rows of pitch %lld or a cache of %d + %d rows exceed 32-bit offsets", b->max_count,
                     (long long)a->ld, a->kept, a->ring);

@@ -1,5 +1,6 @@
-"""Layered hybrid decoders: a list of layers, each with its own mixer (window attention, gated delta rule, gated linear attention) and an
-optional feed-forward (squared ReLU, gated GELU, mixture of experts), some of them run several times in a row.
+"""Layered hybrid decoders: a list of layers, each with its own mixer (window or chunk attention, latent attention, gated delta rule, gated
+linear attention, WKV time mixing) and an optional feed-forward (squared ReLU, gated GELU, clamped gate, mixture of experts), behind or beside
+the mixer; some layers run several times in a row, some use another layer's weights.
 
 `HybridConfig` reads a parsed config.json; `HybridLM` holds the weights under their checkpoint names and hands the arithmetic to
 `hybrid_engine.HybridEngine` (csrc/hybrid.hip and the kernels it calls).  A design is an entry in DESIGNS: which mixers and feed-forwards it
@@ -21,7 +22,7 @@ from . import _native as nat
 class MixerSpec:
     """Sizes and constants of one layer's mixer; which fields count depends on `type`."""
 
-    type: str                      # attention | delta | gla
+    type: str                      # attention | latent | delta | gla | wkv
     heads: int
     kv_heads: int
     dim: int                       # query / key size of a head
@@ -37,22 +38,32 @@ class MixerSpec:
     kv_from: Optional[int] = None  # the layer whose keys and values are read
     taps: int = 0                  # delta: convolution taps
     tau: float = 1.0               # gla
+    chunked: bool = False          # `window` counts chunks from position 0
+    temp: bool = False             # a learned factor per head of the scores
+    bias: bool = False             # a distance bias, its slopes from the number of heads
+    unit_v: bool = False           # v over its root mean square
+    gated: bool = True             # attention with a sigmoid gate
+    rot_dim: int = 0               # latent: rotated query / key size of a head, next to dim
+    q_rank: int = 0
+    kv_rank: int = 0
 
 
 @dataclass
 class MlpSpec:
-    kind: str                      # relu2 | geglu | experts
+    kind: str                      # relu2 | geglu | experts | clampglu
     ff: int                        # hidden size (of one expert)
     experts: int = 0
     top: int = 0
     scale: float = 1.0             # the chosen experts' weights sum to this
     ff_shared: int = 0             # of the expert that every token runs, 0: none
+    limit: float = 0.0             # clampglu: bound of both halves
 
 
 @dataclass
 class LayerSpec:
     mixer: MixerSpec
     mlp: Optional[MlpSpec] = None
+    weights_of: Optional[int] = None  # the layer whose tensors it uses
 
     @property
     def ff(self) -> int:
@@ -96,6 +107,37 @@ def _gla(m: dict) -> MixerSpec:
     return MixerSpec("gla", m["heads"], m["heads"], m["dim"], m["vdim"], tau=float(m["tau"]))
 
 
+def _chunk_attention(m: dict) -> MixerSpec:
+    """Attention inside chunks of the sequence: no rotation, a distance bias and a learned factor per head, unit values, no gate."""
+    _only(m, ("heads", "kv_heads", "dim", "vdim", "scale", "mask"), "attention mixer")
+    mask = m.get("mask") or {}
+    _only(mask, ("size",), "mask")
+    size = mask.get("size")
+    return MixerSpec("attention", m["heads"], m["kv_heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=int(size or 1 << 30),
+                     chunked=size is not None, temp=True, bias=True, unit_v=True, gated=False)
+
+
+def _latent_attention(m: dict) -> MixerSpec:
+    """Queries, keys and values through latents; a rotated part of every query and one rotated key part that the heads share; sinks."""
+    _only(m, ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "rot", "scale"), "latent attention mixer")
+    rot = m["rot"]
+    _only(rot, ("base", "dims"), "rotation")
+    if int(rot["dims"]) != int(m["rot_dim"]) or int(m["rot_dim"]) % 2:
+        raise ValueError(f"latent attention rotates its {m['rot_dim']} rotated dimensions, not {rot['dims']}")
+    return MixerSpec("latent", m["heads"], m["heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=1 << 30, rot_dims=int(rot["dims"]),
+                     rot_base=float(rot["base"]), sink=True, gated=False, rot_dim=int(m["rot_dim"]), q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]))
+
+
+def _wkv(m: dict) -> MixerSpec:
+    _only(m, ("heads", "dim"), "wkv mixer")
+    return MixerSpec("wkv", m["heads"], m["heads"], m["dim"], m["dim"])
+
+
+def _clamped(d: dict) -> MlpSpec:
+    _only(d, ("kind", "ff", "limit"), "feed-forward")
+    return MlpSpec("clampglu", int(d["ff"]), limit=float(d["limit"]))
+
+
 def _plain(kind: str) -> Callable[[dict], MlpSpec]:
     def read(d: dict) -> MlpSpec:
         _only(d, ("kind", "ff"), "feed-forward")
@@ -124,11 +166,13 @@ class Design:
     keys: Tuple[str, ...]          # of the configuration, next to the common ones
     norm_add: float = 0.0          # an RMSNorm's scale is norm_add + its weight
     tied: bool = False             # the logits are products with the embedding table
+    parallel: bool = False         # mixer and feed-forward read one norm, x += mixer(h) + ff(h); norms in groups
 
 
 DESIGNS = {
     "Sekulorn": Design({"attention": _attention, "delta": _delta, "gla": _gla}, {"dense": _plain("relu2")}, ("loop", "residual_mult")),
     "Kovalorn": Design({"attention": _sink_attention}, {"dense": _plain("geglu"), "moe": _experts}, ("logit_scale",), norm_add=1.0, tied=True),
+    "Kudazen": Design({"attention": _chunk_attention, "latent_attention": _latent_attention, "wkv": _wkv}, {"dense": _clamped}, (), tied=True, parallel=True),
 }
 
 
@@ -140,6 +184,7 @@ class HybridConfig:
     eps: float
     residual_mult: float = 1.0
     logit_scale: float = 1.0
+    norm_groups: int = 0                    # equal parts of a row that are normalised by themselves (parallel layers)
     loop: Tuple[int, int, int] = (0, 0, 1)  # layers start .. stop - 1 run `times` times in a row
     architecture: str = "Sekulorn"
     block_size: int = 1 << 24               # (positions are not tabulated: nothing limits a sequence but its cache)
@@ -152,10 +197,13 @@ class HybridConfig:
             raise ValueError(f"unknown design {name!r} (known: {sorted(DESIGNS)})")
         design = DESIGNS[name]
         _only(d, ("architecture", "vocab", "width", "layers", "norm", *design.keys), "configuration")
-        _only(d["norm"], ("eps",), "norm")
+        _only(d["norm"], ("eps", "groups") if design.parallel else ("eps",), "norm")
+        groups = int(d["norm"].get("groups") or 1) if design.parallel else 0
+        if groups and (groups < 0 or int(d["width"]) % groups):
+            raise ValueError(f"norm: {groups} groups of a row of {d['width']}")
         layers: List[LayerSpec] = []
         for e in d["layers"]:
-            _only(e, ("type", "mixer", "mlp"), "layer")
+            _only(e, ("type", "mixer", "mlp", "weights_of") if design.parallel else ("type", "mixer", "mlp"), "layer")
             if e["type"] not in design.mixers:
                 raise ValueError(f"unknown mixer {e['type']!r} (known: {sorted(design.mixers)})")
             mlp = e.get("mlp")
@@ -170,7 +218,14 @@ class HybridConfig:
                     raise ValueError(f"layer {len(layers)}: layer {spec.kv_from} in front of it has no keys of its own")
                 if (own.kv_heads, own.dim, own.vdim) != (spec.kv_heads, spec.dim, spec.vdim):
                     raise ValueError(f"layer {len(layers)}: the keys and values of layer {spec.kv_from} have other sizes")
-            layers.append(LayerSpec(spec, design.mlps[mlp["kind"]](mlp) if mlp is not None else None))
+            layers.append(LayerSpec(spec, design.mlps[mlp["kind"]](mlp) if mlp is not None else None, e.get("weights_of")))
+        for i, l in enumerate(layers):
+            if l.weights_of is not None:
+                own = layers[l.weights_of] if 0 <= l.weights_of < len(layers) else None
+                if own is None or own.weights_of is not None:
+                    raise ValueError(f"layer {i}: layer {l.weights_of} has no tensors of its own")
+                if (own.mixer, own.mlp) != (l.mixer, l.mlp):
+                    raise ValueError(f"layer {i} differs from layer {l.weights_of}, whose weights it uses")
         loop = d.get("loop")
         if loop is not None:
             _only(loop, ("start", "stop", "times"), "loop")
@@ -178,7 +233,7 @@ class HybridConfig:
             if not (0 <= span[0] <= span[1] <= len(layers) and span[2] >= 1):
                 raise ValueError(f"bad loop {span} over {len(layers)} layers")
         return cls(int(d["vocab"]), int(d["width"]), layers, float(d["norm"]["eps"]), float(d.get("residual_mult", 1.0)),
-                   float(d.get("logit_scale", 1.0)), span if loop is not None else (0, 0, 1), name, raw=d)
+                   float(d.get("logit_scale", 1.0)), groups, span if loop is not None else (0, 0, 1), name, raw=d)
 
     @property
     def design(self) -> Design:
@@ -207,12 +262,16 @@ class HybridConfig:
 def projections(m: MixerSpec) -> Tuple[str, ...]:
     """The pieces of a mixer's stacked input projection, in the order of their columns."""
     if m.type == "attention":
-        return ("q", "g") if m.kv_from is not None else ("q", "k", "v", "g")
+        return ("q", *(("k", "v") if m.kv_from is None else ()), *(("g",) if m.gated else ()))
+    if m.type == "latent":
+        return ("dq", "dkv")
+    if m.type == "wkv":
+        return ("r", "k", "v", "g", "w1")  # (each reads a mix of its own)
     return ("q", "k", "v", "g", "a", "b") if m.type == "delta" else ("q", "k", "v", "g", "a1")
 
 
 def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[int, ...]]:
-    """name -> shape of every tensor of a checkpoint; rank[i]: the low-rank size of gla layer i (only its tensors know it)."""
+    """name -> shape of every tensor of a checkpoint; rank[i]: the low-rank size of gla or wkv layer i (only its tensors know it)."""
     W = cfg.width
     out = {"embed": (cfg.vocab_size, W)}
 
@@ -220,6 +279,8 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
         out.update({p + "gate": (ff, W), p + "up": (ff, W), p + "down": (W, ff)})
 
     for i, l in enumerate(cfg.layers):
+        if l.weights_of is not None:
+            continue
         p, m = f"l{i}.", l.mixer
         hv, gk = m.heads * m.vdim, m.kv_heads * m.dim
         out[p + "norm1"] = (W,)
@@ -230,7 +291,18 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
                 out.update({x + "k": (gk, W), x + "v": (m.kv_heads * m.vdim, W)})
             if m.sink:
                 out[x + "sink"] = (m.heads,)
-            out[x + "g"] = (hv if m.gate_values else m.heads, W)
+            if m.gated:
+                out[x + "g"] = (hv if m.gate_values else m.heads, W)
+            if m.temp:
+                out[x + "temp"] = (m.heads,)
+        elif m.type == "latent":
+            out.update({x + "dq": (m.q_rank, W), x + "dq.norm": (m.q_rank,), x + "uq": (m.heads * (m.dim + m.rot_dim), m.q_rank),
+                        x + "dkv": (m.kv_rank + m.rot_dim, W), x + "dkv.norm": (m.kv_rank,), x + "uk": (gk, m.kv_rank), x + "uv": (hv, m.kv_rank),
+                        x + "sink": (m.heads,)})
+        elif m.type == "wkv":
+            out.update({x + f"mu.{s}": (W,) for s in "rkvgw"})
+            out.update({x + s: (hv, W) for s in "rkvg"})
+            out.update({x + "w1": (rank[i], W), x + "w2": (hv, rank[i]), x + "w0": (hv,), x + "u": (m.heads, m.dim), x + "norm": (hv,)})
         else:
             out.update({x + "q": (gk, W), x + "k": (gk, W), x + "v": (hv, W), x + "g": (hv, W), x + "norm": (m.vdim,)})
         if m.type == "delta":
@@ -241,10 +313,11 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
         out[x + "o"] = (W, hv)
         f = l.mlp
         if f is not None:
-            out[p + "norm2"] = (W,)
+            if not cfg.design.parallel:
+                out[p + "norm2"] = (W,)
             if f.kind == "relu2":
                 out.update({p + "mlp.up": (f.ff, W), p + "mlp.down": (W, f.ff)})
-            elif f.kind == "geglu":
+            elif f.kind in ("geglu", "clampglu"):
                 gated(p + "mlp.", f.ff)
             else:
                 out[p + "mlp.router"] = (f.experts, W)
@@ -277,7 +350,8 @@ class HybridLM(nn.Module):
 
     def load_state_dict(self, sd, strict: bool = True):
         """`sd`: name -> tensor (lazy tensors of checkpoint.lazy_load included).  Names and shapes must be the configuration's."""
-        rank = {i: sd[f"l{i}.mix.a1"].shape[0] for i, l in enumerate(self.config.layers) if l.mixer.type == "gla" and f"l{i}.mix.a1" in sd}
+        low = {"gla": "a1", "wkv": "w1"}
+        rank = {i: sd[n].shape[0] for i, l in enumerate(self.config.layers) for n in (f"l{i}.mix.{low.get(l.mixer.type)}",) if n in sd}
         shapes = tensor_shapes(self.config, {**{i: 0 for i in range(len(self.config.layers))}, **rank})
         missing, extra = sorted(set(shapes) - set(sd)), sorted(set(sd) - set(shapes))
         if missing or (strict and extra):

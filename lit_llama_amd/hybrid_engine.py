@@ -18,13 +18,15 @@ import torch
 from . import _native as nat
 from . import ops
 from ._native import ExpertsArgs, HybridLayer, HybridModel, Proj, SeqBatch, check, lib, ptr
-from .hybrid import HybridLM, MlpSpec, projections
+from .hybrid import HybridLM, LayerSpec, MixerSpec, MlpSpec, projections
 from .state import SlotManager, grown
 
-MIX = {"attention": 0, "delta": 1, "gla": 2}
-MLP = {"relu2": 1, "geglu": 2, "experts": 3}
+MIX = {"attention": 0, "delta": 1, "gla": 2, "wkv": 3, "latent": 4}
+MLP = {"relu2": 1, "geglu": 2, "experts": 3, "clampglu": 4}
 KV_OWN, KV_LENDS, KV_BORROWS = 0, 1, 2
-REC_DELTA, REC_GLA = 0, 1
+REC_DELTA, REC_GLA, REC_WKV = 0, 1, 2
+REC = {MIX["delta"]: REC_DELTA, MIX["gla"]: REC_GLA, MIX["wkv"]: REC_WKV}
+LATENT_RECORDS = 64 << 20  # bytes of softmax records of a latent attention's key splits
 
 
 class Entry(NamedTuple):
@@ -38,6 +40,10 @@ class Entry(NamedTuple):
 
 def _pad16(n: int) -> int:
     return (n + 15) // 16 * 16
+
+
+def _pad128(n: int) -> int:
+    return (n + 127) // 128 * 128
 
 
 class HybridEngine:
@@ -114,8 +120,12 @@ class HybridEngine:
         self.weight_bytes = 0
         self._expert_bytes: Dict[int, float] = {}
         self.norm_dtype = nat.dtype_code(self.dtype)
-        layers = []
+        layers: List[Optional[HybridLayer]] = []
+        self._cats: Dict[tuple, int] = {}
         for i, spec in enumerate(cfg.layers):
+            if spec.weights_of is not None:
+                layers.append(None)
+                continue
             m, p = spec.mixer, f"l{i}."
             x = p + "mix."
             L = HybridLayer()
@@ -128,9 +138,15 @@ class HybridEngine:
                 off[name] = sum(q.shape[0] for q in parts)
                 pad = _pad16(w.shape[0]) - w.shape[0]
                 parts.append(torch.cat([w, w.new_zeros((pad, w.shape[1]))]) if pad else w)
-            setattr(L, "in", self._proj(torch.cat(parts)))
-            L.out = self._proj(T[x + "o"])
-            if spec.mlp is not None:
+            if m.type == "wkv":
+                self._token_shift(L, x, parts, off)
+            else:
+                setattr(L, "in", self._proj(torch.cat(parts)))
+            if cfg.design.parallel:
+                self._parallel(L, p, spec)
+            else:
+                L.out = self._proj(T[x + "o"])
+            if spec.mlp is not None and not cfg.design.parallel:
                 L.norm2 = self._norm(p + "norm2")
                 if spec.mlp.kind == "experts":
                     L.moe = self._experts(i, spec.mlp)
@@ -140,24 +156,32 @@ class HybridEngine:
             if m.type == "attention":
                 a = L.attn
                 a.heads, a.kv_heads, a.dim, a.vdim = m.heads, m.kv_heads, m.dim, m.vdim
-                a.off_q, a.off_k, a.off_v, a.off_g = off["q"], off.get("k", 0), off.get("v", 0), off["g"]
+                a.off_q, a.off_k, a.off_v, a.off_g = off["q"], off.get("k", 0), off.get("v", 0), off.get("g", -1)
                 a.scale, a.window, a.rot_dims, a.keep = m.scale, m.window, m.rot_dims, m.keep
                 a.gate_values, a.unit_qk, a.unit_eps = int(m.gate_values), int(m.unit_qk), cfg.eps
+                a.chunked, a.unit_v = int(m.chunked), int(m.unit_v)
                 if m.sink:
                     a.sink = self._f32(T[x + "sink"])
+                if m.temp:
+                    a.head_scale = self._f32(T[x + "temp"])
+                if m.bias:
+                    a.slope = self._f32(torch.tensor([2.0 ** (-8.0 * (h + 1) / m.heads) for h in range(m.heads)], dtype=torch.float64, device=self.device))
                 if m.rot_dims:
-                    f = torch.tensor([m.rot_base ** (-2.0 * j / m.rot_dims) for j in range(m.rot_dims // 2)], dtype=torch.float64,
-                                     device=self.device)
-                    self._keep.append(f)
-                    a.inv_freq = ptr(f)
+                    a.inv_freq = self._inv_freq(m)
+            elif m.type == "latent":
+                self._latent(L, x, m, off)
             else:
                 r = L.rec
-                r.kind = REC_DELTA if m.type == "delta" else REC_GLA
+                r.kind = REC[L.mixer]
                 r.heads, r.kv_heads, r.dim, r.vdim = m.heads, m.kv_heads, m.dim, m.vdim
-                r.off_q, r.off_k, r.off_v, r.off_g = off["q"], off["k"], off["v"], off["g"]
+                r.off_q, r.off_k, r.off_v, r.off_g = off["r" if m.type == "wkv" else "q"], off["k"], off["v"], off["g"]
                 r.q_scale, r.eps, r.unit_eps = m.dim ** -0.5, cfg.eps, 1e-6
                 r.head_norm = self._f32(T[x + "norm"])
-                if m.type == "delta":
+                if m.type == "wkv":
+                    r.q_scale, r.norm_ld, r.bonus = 1.0, m.vdim, self._f32(T[x + "u"])
+                    r.off_a, r.rank = off["w1"], T[x + "w1"].shape[0]
+                    r.a2, r.a2_bias = self._f32(T[x + "w2"]), self._f32(T[x + "w0"])
+                elif m.type == "delta":
                     r.off_a, r.off_b, r.taps = off["a"], off["b"], m.taps
                     r.conv_q, r.conv_k, r.conv_v = (self._f32(T[x + n + ".conv"]) for n in "qkv")
                     r.a_log, r.dt_bias = self._f32(T[x + "A_log"]), self._f32(T[x + "dt_bias"])
@@ -165,6 +189,7 @@ class HybridEngine:
                     r.off_a, r.rank, r.inv_tau = off["a1"], T[x + "a1"].shape[0], 1.0 / m.tau
                     r.a2, r.a2_bias = self._f32(T[x + "a2"]), self._f32(T[x + "a2.b"])
             layers.append(L)
+        layers = [layers[spec.weights_of if l is None else i] for i, (l, spec) in enumerate(zip(layers, cfg.layers))]
         runs = cfg.runs()
         self.run_layers = runs
         self.layers = (HybridLayer * max(1, len(runs)))()
@@ -173,7 +198,7 @@ class HybridEngine:
             self.layers[r].kv_lender = self.layers[r].kv_last = -1
         # a lender's cache covers the windows and the first tokens of all that read it
         self.lenders = cfg.lenders()
-        self.spans = [(l.attn.window, l.attn.keep) for l in self.layers[: len(runs)]]
+        self.spans = [(1 << 30, 0) if l.mixer == MIX["latent"] else (l.attn.window, l.attn.keep) for l in self.layers[: len(runs)]]
         for r, j in enumerate(self.lenders):
             if j is not None:
                 self.layers[r].kv_lender, self.layers[j].kv_last = j, r
@@ -183,12 +208,101 @@ class HybridEngine:
         M.n_runs, M.dtype, M.norm_dtype = len(runs), nat.dtype_code(self.dtype), self.norm_dtype
         M.width, M.ldx, M.vocab, M.max_rows = cfg.width, _pad16(cfg.width), cfg.vocab_size, self.max_rows
         M.eps, M.residual_mult, M.logit_scale = cfg.eps, cfg.residual_mult, cfg.logit_scale
+        M.norm_groups, M.ld_n = cfg.norm_groups, _pad128(cfg.width)
         M.norm_add = cfg.design.norm_add if self.dtype == torch.bfloat16 else 0.0
         M.embed, M.final_norm = ptr(T["embed"]), self._norm("final.norm")
         M.head = self._proj(T["embed" if cfg.design.tied else "head"])
         M.ld_logits = M.head.N
         M.layers = self.layers
         self.n_logits = cfg.vocab_size
+
+    def _inv_freq(self, m: MixerSpec) -> int:
+        f = torch.tensor([m.rot_base ** (-2.0 * j / m.rot_dims) for j in range(m.rot_dims // 2)], dtype=torch.float64, device=self.device)
+        self._keep.append(f)
+        return ptr(f)
+
+    def _token_shift(self, L: HybridLayer, x: str, parts: List[torch.Tensor], off: Dict[str, int]) -> None:
+        """Input projections that read a mix of their own each; bf16: those of one size as one stream, where its parts are whole tiles."""
+        T, names = self.weights, projections(MixerSpec("wkv", 1, 1, 1, 1))
+        L.n_mix = len(names)
+        L.mu = self._f32(torch.stack([T[f"{x}mu.{s[0]}"] for s in names]))
+        n = sum(1 for w in parts if w.shape == parts[0].shape)
+        stack = self.dtype == torch.bfloat16 and all(w.shape == parts[0].shape for w in parts[:n]) and n > 1
+        if stack:
+            L.mix_w[0] = self._proj(torch.cat(parts[:n]))
+            L.mix_stacked = n
+        for i, (s, w) in enumerate(zip(names, parts)):
+            L.mix_at[i] = off[s]
+            if not stack or i >= n:
+                L.mix_w[i] = self._proj(w)
+        setattr(L, "in", Proj(None, sum(w.shape[0] for w in parts), self.cfg.width))
+
+    def _parallel(self, L: HybridLayer, p: str, spec: LayerSpec) -> None:
+        """Feed-forward beside the mixer: its gate / up pair, and one output weight over the row [mixer | hidden]."""
+        T = self.weights
+        o = T[p + "mix.o"]
+        pad = lambda w: torch.nn.functional.pad(w, (0, _pad16(w.shape[1]) - w.shape[1]))
+        L.parallel, L.hid_at = 1, _pad16(o.shape[1])
+        if spec.mlp is not None:
+            L.up = self._proj(T[p + "mlp.gate"], T[p + "mlp.up"])
+            L.limit = spec.mlp.limit
+            o = torch.cat([pad(o), pad(T[p + "mlp.down"])], 1)
+        L.out = self._proj(o)
+        L.ld_cat = _pad128(L.out.K)
+        key = (T[p + "mix.o"].shape[1], L.out.K)  # layers of one layout share their rows: what no layer writes stays zero
+        if key not in self._cats:
+            self._cats[key] = ptr(self._buf(self.max_rows * L.ld_cat, self.dtype))
+        L.cat = self._cats[key]
+
+    def _latent(self, L: HybridLayer, x: str, m: MixerSpec, off: Dict[str, int]) -> None:
+        T, a = self.weights, L.latent
+        a.heads, a.dim, a.rot_dim, a.vdim, a.q_rank, a.kv_rank = m.heads, m.dim, m.rot_dim, m.vdim, m.q_rank, m.kv_rank
+        a.off_q, a.off_c, a.scale, a.eps = off["dq"], off["dkv"], m.scale, self.cfg.eps
+        a.q_norm, a.c_norm, a.sink = (self._f32(T[x + n]) for n in ("dq.norm", "dkv.norm", "sink"))
+        a.inv_freq = self._inv_freq(m)
+        a.uq = self._proj(T[x + "uq"])
+        uk, uv = T[x + "uk"], T[x + "uv"]
+        a.uk_t = self._own(uk.view(m.heads, m.dim, m.kv_rank).transpose(1, 2).contiguous())
+        a.uv = self._own(uv.contiguous())
+        if self.dtype == torch.bfloat16:
+            before = self.weight_bytes  # (a second form of the same weights, for prompts)
+            rows = lambda w: torch.nn.functional.pad(w, (0, 0, 0, _pad16(w.shape[0]) - w.shape[0]))
+            a.expand = self._proj(torch.cat([rows(uk), rows(uv)]))
+            self.weight_bytes = before
+
+    def _latent_scratch(self) -> None:
+        """Rows of a step and of a sequence's expanded keys and values, shared by the latent attentions of all runs."""
+        ls = [l.latent for l in list(self.layers)[: self.m.n_runs] if l.mixer == MIX["latent"]]
+        if not ls:
+            return
+        R, f32 = self.max_rows, self.dtype == torch.float32
+        cq = self._buf(R * max(_pad128(a.q_rank) for a in ls), self.dtype)
+        q = self._buf(R * max(a.uq.N for a in ls), self.dtype)
+        qa = self._buf(R * max(a.heads * (a.kv_rank + a.rot_dim) for a in ls), self.dtype)
+        n = max(LATENT_RECORDS, max(a.heads * (a.kv_rank + 4) * 4 for a in ls))
+        rec = self._buf(n // 4, torch.float32)
+        for r in range(self.m.n_runs):
+            a = self.layers[r].latent
+            if self.layers[r].mixer == MIX["latent"]:
+                a.cq, a.q, a.qa, a.partials, a.partials_bytes = ptr(cq), ptr(q), ptr(qa), ptr(rec), n
+
+    def _expand_scratch(self) -> None:
+        """bf16: room for the keys and values of every position of a sequence (grows with the longest one)."""
+        ls = [l.latent for l in list(self.layers)[: self.m.n_runs] if l.mixer == MIX["latent"]]
+        rows = max(self.max_rows, self.max_len)
+        if not ls or self.dtype == torch.float32 or rows <= getattr(self, "_expand_rows", 0):
+            return
+        new = lambda n, dtype=self.dtype: torch.zeros(n, dtype=dtype, device=self.device)
+        ws = int(lib().mi355_linear_gemm_workspace_bytes(rows, max(_pad128(a.kv_rank) for a in ls)))
+        self._expand = [new(rows * max(_pad128(a.kv_rank) for a in ls)), new(rows * max(a.expand.N for a in ls))]
+        if ws > self.m.gemm_ws_bytes:
+            self._expand.append(new(ws, torch.uint8))
+            self.m.gemm_ws, self.m.gemm_ws_bytes = ptr(self._expand[2]), ws
+        for r in range(self.m.n_runs):
+            if self.layers[r].mixer == MIX["latent"]:
+                a = self.layers[r].latent
+                a.rows_c, a.kv_rows, a.expand_rows = ptr(self._expand[0]), ptr(self._expand[1]), rows
+        self._expand_rows = rows
 
     def _buf(self, n: int, dtype: torch.dtype) -> torch.Tensor:
         t = torch.zeros(max(1, n), dtype=dtype, device=self.device)
@@ -204,19 +318,21 @@ class HybridEngine:
         M.proj = ptr(self._buf(R * max([getattr(l, "in").N for l in ls], default=16), self.dtype))
         M.att = ptr(self._buf(R * M.ld_att, self.dtype))
         f32 = self.dtype == torch.float32
-        M.hid = ptr(self._buf(R * max([l.up.N * (3 if f32 and l.mlp == MLP["geglu"] else 1) for l in ls], default=16), self.dtype))
+        M.hid = ptr(self._buf(R * max([l.up.N * (3 if f32 and l.mlp in (MLP["geglu"], MLP["clampglu"]) else 1) for l in ls], default=16), self.dtype))
         if self.dtype == torch.float32:
-            M.xn, M.tmp = ptr(self._buf(R * M.ldx, torch.float32)), ptr(self._buf(R * M.ldx, torch.float32))
+            M.xn, M.tmp = ptr(self._buf(R * M.ld_n, torch.float32)), ptr(self._buf(R * M.ldx, torch.float32))
         else:
-            K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down)])  # (K = 0: not there)
-            n = int(lib().mi355_linear_gemm_workspace_bytes(R, K))
+            K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down, l.latent.uq)])  # (K = 0: not there)
+            n = int(lib().mi355_linear_gemm_workspace_bytes(R, _pad128(K)))
             M.gemm_ws, M.gemm_ws_bytes = ptr(self._buf(n, torch.uint8)), n
-            M.xb = ptr(self._buf(R * M.ldx, torch.bfloat16))
+            M.xb = ptr(self._buf(R * M.ld_n, torch.bfloat16))
+        M.mix = ptr(self._buf(R * M.ld_n * max([l.n_mix for l in ls], default=0), self.dtype))
+        self._latent_scratch()
         # a split attention step keeps one record per (row, head, split); one split takes none
         n = max([512 * (l.attn.vdim + 2) * max(8, l.attn.heads // l.attn.kv_heads) for l in ls if l.mixer == 0], default=0)
         M.partials, M.partials_bytes = ptr(self._buf(n, torch.float32)), n * 4
         n = max([int(lib().mi355_recurrent_scratch_bytes(l.rec.kind, R, 64, l.rec.heads, l.rec.kv_heads, l.rec.dim, l.rec.vdim))
-                 for l in ls if l.mixer != 0], default=0)
+                 for l in ls if l.mixer in REC], default=0)
         M.rec_scratch, M.rec_scratch_bytes = ptr(self._buf(n, torch.uint8)), n
         n = 0
         for l in ls:
@@ -254,12 +370,15 @@ class HybridEngine:
     def _set_len(self, n: int) -> None:
         """Rings hold min(window, longest sequence) rows (behind the first tokens').  Growing them re-lays the rings, so no sequence may be live unless every ring
         already spans its window."""
-        need = any(l.mixer == 0 and self._ring(r, n) != self._ring(r, self.max_len) for r, l in enumerate(list(self.layers)[: self.m.n_runs]))
+        need = any(l.mixer in (MIX["attention"], MIX["latent"]) and self._ring(r, n) != self._ring(r, self.max_len) for r, l in enumerate(list(self.layers)[: self.m.n_runs]))
         if need and self.slots.live == 1 and self._single is not None:
             self.reset_cache()  # (what is live is a sequence that generate() or forward() left behind)
         if need and self.max_len and self.slots.live:
             raise nat.NativeError(f"hybrid engine: sequences are live at cache length {self.max_len}; {n} needs a larger one")
         self.max_len = n
+        with torch.cuda.device(self.device), torch.cuda.stream(self.stream):
+            self._destroy_graphs()  # (captured launches hold the scratch)
+            self._expand_scratch()
         if need and self.slots.capacity:
             self.pools = [None] * self.m.n_runs
             with torch.cuda.stream(self.stream):
@@ -287,6 +406,12 @@ class HybridEngine:
                 v = grown(old[1], (n, a.kv_heads, a.kept + a.ring, a.vdim), self.dtype, dev)
                 a.kring, a.vring = ptr(k), ptr(v)
                 self.pools[r] = (k, v)
+            elif l.mixer == MIX["latent"]:
+                a = l.latent
+                a.cache_rows = self._ring(r, self.max_len or 1)
+                c = grown(old[0], (n, a.cache_rows, a.kv_rank + a.rot_dim), self.dtype, dev)
+                a.cache = ptr(c)
+                self.pools[r] = (c, None)
             else:
                 e = l.rec
                 st = grown(old[0], (n, e.heads, e.dim, e.vdim), torch.float32, dev)
@@ -294,6 +419,9 @@ class HybridEngine:
                 if e.kind == REC_DELTA:
                     cv = grown(old[1], (n, e.taps, 2 * e.kv_heads * e.dim + e.heads * e.vdim), self.dtype, dev)
                     e.conv_ring = ptr(cv)
+                if l.n_mix:
+                    cv = grown(old[1], (n, self.cfg.width), torch.float32, dev)
+                    l.shift = ptr(cv)
                 e.state = ptr(st)
                 self.pools[r] = (st, cv)
 
@@ -327,9 +455,9 @@ class HybridEngine:
         self.stream.synchronize()  # (`t` may go)
 
     # ---- steps -----------------------------------------------------------------------------------------
-    def _batch(self, rows: int, seqs: int, max_count: int) -> SeqBatch:
+    def _batch(self, rows: int, seqs: int, max_count: int, max_end: int = 0) -> SeqBatch:
         b = SeqBatch()
-        b.rows, b.seqs, b.max_count = rows, seqs, max_count
+        b.rows, b.seqs, b.max_count, b.max_end = rows, seqs, max_count, max_end
         b.row0, b.count, b.slot, b.pos = (ptr(self.meta[i]) for i in (1, 2, 3, 4))
         return b
 
@@ -349,7 +477,7 @@ class HybridEngine:
             most = max(most, n)
         self.meta.copy_(h, non_blocking=True)
         self._meta_sent.record(self.stream)
-        return self._batch(rows, len(entries), most), n_want
+        return self._batch(rows, len(entries), most, max(e.pos + len(e.tokens) for e in entries)), n_want
 
     def _cut(self, entries: Sequence[Entry]) -> List[List[Entry]]:
         """Sub-steps of at most max_rows rows and max_logits_rows wanted rows; a long portion continues in the next one."""

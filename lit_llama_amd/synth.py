@@ -323,7 +323,20 @@ def experts_bench_config(width: int, n_layer: int, vocab: int = 32000, window: i
     return {"architecture": "Kovalorn", "layers": layers, "norm": {"eps": 1e-5}, "logit_scale": 0.25, "vocab": vocab, "width": width}
 
 
-HYBRID_BENCH = {"Sekulorn": hybrid_bench_config, "Kovalorn": experts_bench_config}
+def parallel_bench_config(width: int, n_layer: int, vocab: int = 32000, chunk: int = 2048) -> dict:
+    """A Kudazen configuration of a LLaMA's width and feed-forward: chunk attention | latent | wkv | latent layers in turn, heads of 128 (64 more
+    rotated dimensions in the latent layers, latents of 512, queries through 3/8 of the width)."""
+    heads = width // 128
+    hidden = LLaMAConfig(n_embd=width, n_head=heads).n_hidden
+    latent = ("latent_attention", {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": width * 3 // 8, "kv_rank": 512,
+                                   "rot": {"base": 1e4, "dims": 64}, "scale": 192 ** -0.5})
+    mixers = [("attention", {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": chunk}}),
+              latent, ("wkv", {"heads": heads, "dim": 128}), latent]
+    layers = [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": hidden, "limit": 7.0}} for t, m in (mixers[i % 4] for i in range(n_layer))]
+    return {"architecture": "Kudazen", "layers": layers, "norm": {"eps": 1e-5, "groups": 2}, "vocab": vocab, "width": width}
+
+
+HYBRID_BENCH = {"Sekulorn": hybrid_bench_config, "Kovalorn": experts_bench_config, "Kudazen": parallel_bench_config}
 
 
 def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: torch.dtype = torch.bfloat16, rank: int = 16):
@@ -342,6 +355,14 @@ def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: tor
             t = 1.0 - cfg.design.norm_add + 0.1 * t
         elif leaf.endswith("sink"):
             t = t + 1.0
+        elif leaf.endswith("temp"):
+            t = 1.0 + 0.2 * t
+        elif leaf.startswith("mix.mu."):
+            t = torch.sigmoid(t)
+        elif leaf.endswith("mix.w0"):
+            t = 0.5 * t - 2.5
+        elif leaf.endswith("mix.u"):
+            t = 0.5 * t
         elif leaf.endswith(".conv"):
             t = t * 0.2
             t[:, -1] += 0.7
