@@ -25,7 +25,7 @@
 
 #include <hip/hip_ext.h>
 
-#include "common.h"
+#include "product.h"
 
 #ifndef MI355_GEMV_AND_OR
 #define MI355_GEMV_AND_OR 1
@@ -426,8 +426,9 @@ constexpr int kGrpLoadsMax = 12; // GRP = (scale, zero) pairs per thread, matrix
                                  // = 128 groups had kept — with groupsize 64 (172) — off the engine altogether
 constexpr int kGrpLoadsMid = 4;
 
-template <int FMT, int R, int P, int EPI, int VMODE, bool MULTI, int GRP = 0>
-__global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const GemvParams p) {
+// workgroup `bid` of `nb` over the tiles of p
+template <int FMT, int R, int P, int EPI, int VMODE, bool MULTI, int GRP>
+__device__ __forceinline__ void gemv_body(const GemvParams& p, const int bid, const int nb) {
     static_assert(!GRP || FMT == MI355_W_Q4, "grouped scales are a Q4 feature");
     const int M = MULTI ? p.M : 1;
     constexpr bool NT = true;  // weights are read once: non-temporal
@@ -455,7 +456,7 @@ __global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const 
     uint32_t* szl = (uint32_t*)(xs + (((size_t)M * p.xs_stride + 15) & ~(size_t)15));
 #define MI355_STAMP(i)                                                                          \
     do {                                                                                        \
-        if (p.dbg != nullptr && threadIdx.x == 0) p.dbg[blockIdx.x * 8 + (i)] = wall_clock64(); \
+        if (p.dbg != nullptr && threadIdx.x == 0) p.dbg[bid * 8 + (i)] = wall_clock64(); \
     } while (0)
     MI355_STAMP(0);
 
@@ -464,7 +465,6 @@ __global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const 
     // runtime values cost ~60 instructions of every launch's prologue)
     const int nu = p.u_q + (wave < p.u_r ? 1 : 0);
     const int u0 = wave * p.u_q + (wave < p.u_r ? wave : p.u_r);
-    const int bid = blockIdx.x, nb = gridDim.x;
     const int my_tiles = p.t_q + (bid < p.t_r ? 1 : 0);
     const int nu_pad = p.nu_pad;
     const int total = my_tiles * nu_pad;
@@ -804,6 +804,32 @@ __global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const 
     MI355_STAMP(5);
 #undef MI355_ISSUE
 #undef MI355_STAMP
+}
+
+template <int FMT, int R, int P, int EPI, int VMODE, bool MULTI, int GRP = 0>
+__global__ __launch_bounds__((kMaxThreads<FMT, P, GRP>)) void gemv_kernel(const GemvParams p) {
+    gemv_body<FMT, R, P, EPI, VMODE, MULTI, GRP>(p, blockIdx.x, gridDim.x);
+}
+
+// Several products of one input width in one launch, each with an operand of its own: consecutive workgroups per product
+struct GemvJobs {
+    struct Job {
+        const uint8_t* w;
+        const void* x;
+        void* y;
+        int N, n_tiles, t_q, t_r, first, grid;
+        unsigned w_bytes;
+    } job[8];
+    int n;
+};
+template <int VMODE, bool MULTI>
+__global__ __launch_bounds__((kMaxThreads<MI355_W_BF16, 2>)) void gemv_jobs_kernel(const GemvParams base, const GemvJobs jobs) {
+    int j = 0;
+    while (j + 1 < jobs.n && (int)blockIdx.x >= jobs.job[j + 1].first) ++j;
+    const GemvJobs::Job& b = jobs.job[j];
+    GemvParams p = base;
+    p.w = b.w, p.x = b.x, p.y = b.y, p.N = b.N, p.n_tiles = b.n_tiles, p.t_q = b.t_q, p.t_r = b.t_r, p.w_bytes = b.w_bytes;
+    gemv_body<MI355_W_BF16, 1, 2, MI355_EPI_STORE, VMODE, MULTI, 0>(p, blockIdx.x - b.first, b.grid);
 }
 
 // ------------------------------------------------------------------------------------ repack kernels
@@ -1153,7 +1179,9 @@ extern "C" int mi355_u8_repack(const uint8_t* q0, const uint8_t* q1, int64_t str
     return 0;
 }
 
-extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stream) {
+namespace {
+// checks, and the launch of one product
+int gemv_prepare(const mi355_linear_args* a, GemvParams& p, int& grid, int& waves, size_t& lds) {
     MI355_CHECK_ARG(a != nullptr, MI355_E_ARG, "linear_fast: null args");
     MI355_CHECK_ARG(a->fmt == MI355_W_Q4 || a->fmt == MI355_W_BF16, MI355_E_ARG,
                     "linear_fast: fmt %d not handled here (int8 goes through mi355_linear_int8)", a->fmt);
@@ -1183,7 +1211,6 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
                     "linear_fast: scales/zeros dtype must be f32 or bf16");
     MI355_CHECK_ARG(a->ldx >= a->K || a->M == 1 || a->attn_partials, MI355_E_SHAPE, "linear_fast: ldx < K");
 
-    GemvParams p;
     p.w = (const uint8_t*)a->w;
     p.x = a->x;
     p.norm_scale = a->norm_scale;
@@ -1212,7 +1239,7 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
     p.relu2 = (a->flags & MI355_LF_RELU2) ? 1 : 0;
     p.norm_add = (a->flags & MI355_LF_NORM_ONE) ? 1.f : 0.f;
     MI355_CHECK_ARG(!p.relu2 || a->epi == MI355_EPI_STORE, MI355_E_ARG, "linear_fast: RELU2 belongs to the STORE epilogue");
-    int waves = a->waves > 0 ? a->waves : 8;
+    waves = a->waves > 0 ? a->waves : 8;
     if (waves > 16) waves = 16;
     if ((a->fmt != MI355_W_Q4 || (a->group_cols > 0 && a->group_cols < a->K)) && waves > 8) waves = 8;  // see kMaxThreads
     if (waves < 4) waves = 4;  // the combine step needs 256 owner threads
@@ -1264,12 +1291,12 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
         MI355_CHECK_ARG((int64_t)a->N * p.n_groups * 2 < 0x7FFFFFF0ll, MI355_E_SHAPE, "linear_fast: scale table too large");
     }
     const int RS = a->R + ((a->fmt == MI355_W_Q4 && p.n_groups == 0) ? 1 : 0);
-    const size_t lds = kLdsHeader + (size_t)2 * waves * RS * 1024 + (((size_t)a->M * p.xs_stride + 15) & ~(size_t)15) +
+    lds = kLdsHeader + (size_t)2 * waves * RS * 1024 + (((size_t)a->M * p.xs_stride + 15) & ~(size_t)15) +
                        (size_t)2 * a->R * 16 * p.n_groups * 4;
     MI355_CHECK_ARG(lds <= (size_t)kMaxLds, MI355_E_SHAPE,
                     "linear_fast: M=%d x K=%d activations do not fit LDS (%zu B > %d B); chunk M", a->M, a->K, lds,
                     kMaxLds);
-    int grid = a->grid;
+    grid = a->grid;
     if (grid <= 0) {
         const int cus = mi355_num_cus() > 0 ? mi355_num_cus() : 256;
         grid = cus * 2;
@@ -1283,6 +1310,61 @@ extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stre
     }
     p.t_q = p.n_tiles / grid;
     p.t_r = p.n_tiles % grid;
+    return 0;
+}
+
+template <int VMODE>
+int launch_jobs(const GemvParams& p, const GemvJobs& jobs, int grid, int waves, size_t lds, hipStream_t s) {
+    static std::once_flag once;
+    static hipError_t e = hipSuccess;
+    std::call_once(once, [] {
+        e = hipFuncSetAttribute((const void*)gemv_jobs_kernel<VMODE, false>, hipFuncAttributeMaxDynamicSharedMemorySize, kMaxLds);
+        if (e == hipSuccess) e = hipFuncSetAttribute((const void*)gemv_jobs_kernel<VMODE, true>, hipFuncAttributeMaxDynamicSharedMemorySize, kMaxLds);
+    });
+    MI355_CHECK_ARG(e == hipSuccess, (int)e, "linear_fast_jobs: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
+    if (p.M > 1) hipLaunchKernelGGL((gemv_jobs_kernel<VMODE, true>), dim3(grid), dim3(waves * 64), lds, s, p, jobs);
+    else hipLaunchKernelGGL((gemv_jobs_kernel<VMODE, false>), dim3(grid), dim3(waves * 64), lds, s, p, jobs);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+}  // namespace
+
+int mi355_linear_fast_jobs(const mi355_linear_args* a, int count, mi355_stream_t stream) {
+    GemvJobs jobs;
+    MI355_CHECK_ARG(a != nullptr && count >= 1 && count <= (int)(sizeof(jobs.job) / sizeof(jobs.job[0])), MI355_E_ARG, "linear_fast_jobs: %d products", count);
+    GemvParams p;
+    int waves = 0, tiles = 0;
+    size_t lds = 0;
+    for (int i = 0; i < count; ++i) tiles += (a[i].N + 15) / 16;
+    const int room = 2 * (mi355_num_cus() > 0 ? mi355_num_cus() : 256);
+    jobs.n = count;
+    int first = 0;
+    for (int i = 0; i < count; ++i) {
+        mi355_linear_args b = a[i];
+        MI355_CHECK_ARG(b.fmt == MI355_W_BF16 && b.R == 1 && b.epi == MI355_EPI_STORE && b.K == a->K && b.M == a->M && b.ldx == a->ldx && b.ldy == a->ldy &&
+                            b.y_dtype == a->y_dtype && b.x_dtype == MI355_BF16 && b.norm_scale == nullptr && b.bias == nullptr && b.attn_partials == nullptr &&
+                            b.flags == 0 && b.alpha == a->alpha,
+                        MI355_E_ARG, "linear_fast_jobs: products of one shape but for N");
+        const int n = (b.N + 15) / 16;
+        b.grid = tiles <= room ? n : (int)((int64_t)room * n / tiles);  // (workgroups in proportion to the tiles)
+        if (b.grid < 1) b.grid = 1;
+        GemvParams q;
+        int grid, w;
+        size_t l;
+        if (int rc = gemv_prepare(&b, q, grid, w, l)) return rc;
+        if (i == 0) p = q, waves = w, lds = l;
+        else if (q.vec_mode != p.vec_mode) p.vec_mode = 0;
+        jobs.job[i] = {q.w, q.x, q.y, q.N, q.n_tiles, q.t_q, q.t_r, first, grid, q.w_bytes};
+        first += grid;
+    }
+    return p.vec_mode == 2 ? launch_jobs<2>(p, jobs, first, waves, lds, (hipStream_t)stream) : launch_jobs<0>(p, jobs, first, waves, lds, (hipStream_t)stream);
+}
+
+extern "C" int mi355_linear_fast(const mi355_linear_args* a, mi355_stream_t stream) {
+    GemvParams p;
+    int grid, waves;
+    size_t lds;
+    if (int rc = gemv_prepare(a, p, grid, waves, lds)) return rc;
     hipStream_t s = (hipStream_t)stream;
     if (a->fmt == MI355_W_Q4) {
         return a->R == 1 ? dispatch_p<MI355_W_Q4, 1>(p, a->prefetch, grid, waves, lds, s)

@@ -84,9 +84,9 @@ struct NormParams {
     const float* x;
     int64_t ldx;
     const int32_t* want;    // rows of x, or NULL: row m
-    int width, groups, size, scale_dtype;
+    int width, groups, size;
     float eps;
-    const void* scale;
+    const void* scale;      // of the model's dtype
     void* h;                // [rows, ldh]
     int64_t ldh;
     int n_mix;
@@ -108,20 +108,32 @@ __device__ __forceinline__ void put4(T* p, f32x4 v) {
     }
 }
 
-// one row per workgroup; V elements per load (4: groups of whole vectors).  Dynamic LDS: 2 groups floats of 1 / rms + 2 max(8, groups) sums
-template <typename T, int V>
+template <typename T>
+__device__ __forceinline__ f32x4 get4(const T* p) {
+    if constexpr (sizeof(T) == 4) {
+        return *(const f32x4*)p;
+    } else {
+        const u32x2 r = *(const u32x2*)p;
+        return f32x4{__uint_as_float(r[0] << 16), __uint_as_float(r[0] & 0xffff0000u), __uint_as_float(r[1] << 16), __uint_as_float(r[1] & 0xffff0000u)};
+    }
+}
+
+// One row per workgroup, and with MIX a second one: the row before, or, in the workgroup of a portion's first row, the portion's last one (it
+// enters the state there).  H > 0: rows of up to 2048 H values whose groups are whole runs of 256 (a wave's load), held in registers;
+// H = 0: any width.  Dynamic LDS: sums of squares [2][max(runs, 8, groups)], 1 / rms [2][groups]
+template <typename T, bool MIX, int H>
 __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ int s_seq;
     const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int parts = p.groups < 8 ? 8 / p.groups : 1;      // waves per group
-    float* rinv = sm;                                       // [2][groups]
-    float* sums = sm + 2 * p.groups;                        // [2][groups * parts]
+    const int per = H > 0 ? p.size / 256 : p.groups < 8 ? 8 / p.groups : 1;  // sums per group
+    const int n_sums = p.groups * per;
+    float* sums = sm;                     // [2][n_sums]
+    float* rinv = sm + 2 * n_sums;        // [2][groups]
     const float* row = p.x + (int64_t)(p.want != nullptr ? p.want[m] : m) * p.ldx;
-    // a second row: the one before, or, in the workgroup of a portion's first row, the portion's last one (it enters the state there)
-    const float* other = nullptr;
-    int seq = 0, i = 0, cnt = 0;
-    if (p.n_mix > 0) {
+    const float* other = row;
+    int seq = 0, i = 0;
+    if constexpr (MIX) {
         if (p.b.max_count == 1) {
             seq = m;
         } else {
@@ -129,70 +141,117 @@ __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
                 if (m >= p.b.row0[s] && m < p.b.row0[s] + p.b.count[s]) s_seq = s;
             __syncthreads();
             seq = s_seq;
+            i = m - p.b.row0[seq];
+            other = i > 0 ? row - p.ldx : row + (int64_t)(p.b.count[seq] - 1) * p.ldx;
         }
-        i = m - p.b.row0[seq], cnt = p.b.count[seq];
-        other = i > 0 ? row - p.ldx : cnt > 1 ? row + (int64_t)(cnt - 1) * p.ldx : nullptr;
     }
-    const int seg = (p.size / V + parts - 1) / parts;       // vectors of a wave's part of a group
-    for (int q = wave; q < p.groups * parts; q += 8) {
-        const int gr = q / parts, v0 = (q - gr * parts) * seg, v1 = min(p.size / V, v0 + seg);
-        const int64_t at = (int64_t)gr * p.size;
-        float s0 = 0.f, s1 = 0.f;
-#pragma unroll 4
-        for (int v = v0 + lane; v < v1; v += 64) {
-            if constexpr (V == 4) {
-                const f32x4 a = *(const f32x4*)(row + at + 4 * v);
-                s0 += (a[0] * a[0] + a[1] * a[1]) + (a[2] * a[2] + a[3] * a[3]);
-                if (other != nullptr) {
-                    const f32x4 c = *(const f32x4*)(other + at + 4 * v);
-                    s1 += (c[0] * c[0] + c[1] * c[1]) + (c[2] * c[2] + c[3] * c[3]);
-                }
-            } else {
-                s0 += row[at + v] * row[at + v];
-                if (other != nullptr) s1 += other[at + v] * other[at + v];
+    constexpr int HH = H > 0 ? H : 1;
+    f32x4 a[HH], o[HH], sc[HH];
+    if constexpr (H > 0) {
+#pragma unroll
+        for (int j = 0; j < H; ++j) {
+            const int k = 4 * (tid + 512 * j);
+            const bool in = k < p.width;
+            a[j] = in ? *(const f32x4*)(row + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+            if constexpr (MIX) o[j] = in ? *(const f32x4*)(other + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+#pragma unroll
+        for (int j = 0; j < H; ++j) {
+            const int k = 4 * (tid + 512 * j);
+            sc[j] = k < p.width ? get4((const T*)p.scale + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+#pragma unroll
+        for (int j = 0; j < H; ++j) {
+            const float s0 = group_sum((a[j][0] * a[j][0] + a[j][1] * a[j][1]) + (a[j][2] * a[j][2] + a[j][3] * a[j][3]), 64);
+            const int q = wave + 8 * j;
+            if (lane == 0 && q < n_sums) sums[q] = s0;
+            if constexpr (MIX) {
+                const float s1 = group_sum((o[j][0] * o[j][0] + o[j][1] * o[j][1]) + (o[j][2] * o[j][2] + o[j][3] * o[j][3]), 64);
+                if (lane == 0 && q < n_sums) sums[n_sums + q] = s1;
             }
         }
-        s0 = group_sum(s0, 64);
-        s1 = group_sum(s1, 64);
-        if (lane == 0) sums[q] = s0, sums[p.groups * parts + q] = s1;
+    } else {
+        const int seg = (p.size + per - 1) / per;
+        for (int q = wave; q < n_sums; q += 8) {
+            const int gr = q / per, v0 = (q - gr * per) * seg, v1 = min(p.size, v0 + seg);
+            const int64_t at = (int64_t)gr * p.size;
+            float s0 = 0.f, s1 = 0.f;
+            for (int v = v0 + lane; v < v1; v += 64) {
+                s0 += row[at + v] * row[at + v];
+                if constexpr (MIX) s1 += other[at + v] * other[at + v];
+            }
+            s0 = group_sum(s0, 64);
+            s1 = group_sum(s1, 64);
+            if (lane == 0) {
+                sums[q] = s0;
+                if constexpr (MIX) sums[n_sums + q] = s1;
+            }
+        }
     }
     __syncthreads();
-    for (int q = tid; q < 2 * p.groups; q += 512) {
+    for (int q = tid; q < (MIX ? 2 : 1) * p.groups; q += 512) {
         float s = 0.f;
-        for (int j = 0; j < parts; ++j) s += sums[q * parts + j];
+        for (int j = 0; j < per; ++j) s += sums[q * per + j];
         rinv[q] = 1.0f / sqrtf(s / (float)p.size + p.eps);
     }
     __syncthreads();
     T* h = (T*)p.h + (int64_t)m * p.ldh;
-    float* state = p.n_mix > 0 ? p.shift + (int64_t)p.b.slot[seq] * p.width : nullptr;
-    const bool first = p.n_mix > 0 && i == 0, begun = first && p.b.pos[seq] > 0;
-    for (int v = tid; v < p.width / V; v += 512) {
-        const int k = v * V, gr = k / p.size;
-        const float r0 = rinv[gr], r1 = rinv[p.groups + gr];
-        float sc[V], a[V], o[V];
+    float* state = MIX ? p.shift + (int64_t)p.b.slot[seq] * p.width : nullptr;
+    const bool first = MIX && i == 0, begun = first && p.b.pos[seq] > 0;
+    if constexpr (H > 0) {
 #pragma unroll
-        for (int e = 0; e < V; ++e) {
-            sc[e] = ld_as_f32(p.scale, k + e, p.scale_dtype);
-            a[e] = row[k + e] * r0 * sc[e];
-            o[e] = other != nullptr ? other[k + e] * r1 * sc[e] : a[e];
-        }
-        if constexpr (V == 4) put4(h + k, f32x4{a[0], a[1], a[2], a[3]});
-        else st_from_f32(h, k, sizeof(T) == 4 ? MI355_F32 : MI355_BF16, a[0]);
-        if (p.n_mix == 0) continue;
-        float d[V];
+        for (int j = 0; j < H; ++j) {
+            const int k = 4 * (tid + 512 * j);
+            if (k >= p.width) continue;
+            const int gr = (wave + 8 * j) / per;
+            const f32x4 v = a[j] * rinv[gr] * sc[j];
+            put4(h + k, v);
+            if constexpr (MIX) {
+                f32x4 mu[5], d = o[j] * rinv[p.groups + gr] * sc[j];
 #pragma unroll
-        for (int e = 0; e < V; ++e) {
-            const float before = !first ? o[e] : begun ? state[k + e] : 0.f;
-            if (first) state[k + e] = o[e];  // (the portion's last row; of one row, itself)
-            d[e] = before - a[e];
+                for (int s = 0; s < 5; ++s)
+                    if (s < p.n_mix) mu[s] = *(const f32x4*)(p.mu + (int64_t)s * p.width + k);
+                if (first) {  // (d: the portion's last row; of one row, itself)
+                    const f32x4 old = begun ? *(const f32x4*)(state + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+                    *(f32x4*)(state + k) = d;
+                    d = old;
+                }
+                d = d - v;
+#pragma unroll
+                for (int s = 0; s < 5; ++s)
+                    if (s < p.n_mix) put4((T*)p.mix + s * p.mix_stride + (int64_t)m * p.ldh + k, v + d * mu[s]);
+            }
         }
-        for (int s = 0; s < p.n_mix; ++s) {
-            T* x = (T*)p.mix + s * p.mix_stride + (int64_t)m * p.ldh + k;
-            const float* mu = p.mu + (int64_t)s * p.width + k;
-            if constexpr (V == 4) put4(x, f32x4{a[0] + d[0] * mu[0], a[1] + d[1] * mu[1], a[2] + d[2] * mu[2], a[3] + d[3] * mu[3]});
-            else st_from_f32(x, 0, sizeof(T) == 4 ? MI355_F32 : MI355_BF16, a[0] + d[0] * mu[0]);
+    } else {
+        for (int k = tid; k < p.width; k += 512) {
+            const int gr = k / p.size;
+            const float scale = ld_as_f32(p.scale, k, sizeof(T) == 4 ? MI355_F32 : MI355_BF16);
+            const float v = row[k] * rinv[gr] * scale;
+            st_from_f32(h, k, sizeof(T) == 4 ? MI355_F32 : MI355_BF16, v);
+            if constexpr (MIX) {
+                float d = other[k] * rinv[p.groups + gr] * scale;
+                if (first) {
+                    const float old = begun ? state[k] : 0.f;
+                    state[k] = d;
+                    d = old;
+                }
+                d -= v;
+                for (int s = 0; s < p.n_mix; ++s)
+                    st_from_f32((T*)p.mix + s * p.mix_stride + (int64_t)m * p.ldh, k, sizeof(T) == 4 ? MI355_F32 : MI355_BF16,
+                                v + d * p.mu[(int64_t)s * p.width + k]);
+            }
         }
     }
+}
+
+template <typename T, bool MIX>
+void launch_norm(const NormParams& p, int rows, hipStream_t s) {
+    const bool whole = p.size % 256 == 0 && p.width <= 8192;
+    const int sums = whole ? p.width / 256 : p.groups < 8 ? 8 : p.groups;
+    const size_t lds = (size_t)2 * (sums + p.groups) * 4;
+    if (whole && p.width <= 4096) hipLaunchKernelGGL((norm_groups_kernel<T, MIX, 2>), dim3(rows), dim3(512), lds, s, p);
+    else if (whole) hipLaunchKernelGGL((norm_groups_kernel<T, MIX, 4>), dim3(rows), dim3(512), lds, s, p);
+    else hipLaunchKernelGGL((norm_groups_kernel<T, MIX, 0>), dim3(rows), dim3(512), lds, s, p);
 }
 
 // rows [gate | up] of 2 n values -> the clamped gated unit
@@ -330,22 +389,15 @@ int norm_groups(const mi355_hybrid_model* m, const void* scale, const mi355_hybr
     const bool f32 = m->dtype == MI355_F32;
     p.x = m->x, p.ldx = m->ldx, p.want = want;
     p.width = m->width, p.groups = m->norm_groups, p.size = m->width / m->norm_groups;
-    p.eps = m->eps, p.scale = scale, p.scale_dtype = m->norm_dtype;
+    p.eps = m->eps, p.scale = scale;
     p.h = f32 ? (void*)m->xn : (void*)m->xb, p.ldh = m->ld_n;
     if (l != nullptr && l->n_mix > 0) {
         p.n_mix = l->n_mix, p.mu = l->mu, p.shift = l->shift;
         p.mix = m->mix, p.mix_stride = (int64_t)m->max_rows * m->ld_n;
         p.b = *b;
     }
-    const size_t lds = (size_t)(2 * p.groups + 2 * (p.groups < 8 ? 8 : p.groups)) * 4;
-    const bool vec = p.size % 4 == 0;
-    if (f32) {
-        if (vec) hipLaunchKernelGGL((norm_groups_kernel<float, 4>), dim3(rows), dim3(512), lds, s, p);
-        else hipLaunchKernelGGL((norm_groups_kernel<float, 1>), dim3(rows), dim3(512), lds, s, p);
-    } else {
-        if (vec) hipLaunchKernelGGL((norm_groups_kernel<bf16_t, 4>), dim3(rows), dim3(512), lds, s, p);
-        else hipLaunchKernelGGL((norm_groups_kernel<bf16_t, 1>), dim3(rows), dim3(512), lds, s, p);
-    }
+    if (f32) p.n_mix > 0 ? launch_norm<float, true>(p, rows, s) : launch_norm<float, false>(p, rows, s);
+    else p.n_mix > 0 ? launch_norm<bf16_t, true>(p, rows, s) : launch_norm<bf16_t, false>(p, rows, s);
     MI355_LAUNCH_CHECK();
     return 0;
 }
@@ -369,6 +421,21 @@ int parallel_in(const mi355_hybrid_model* m, const mi355_hybrid_layer& l, int M,
     const size_t size = dtype_size(m->dtype);
     const int64_t stride = (int64_t)m->max_rows * m->ld_n;
     int i = 0;
+    if (!f32 && l.mix_stacked > 1 && !mi355_product_wide(l.mix_w[0], M, 1)) {  // a few rows: every mix's product in one launch
+        mi355_linear_args a[5];
+        for (; i < l.n_mix; ++i) {
+            const bool part = i < l.mix_stacked;
+            const mi355_proj& w = l.mix_w[part ? 0 : i];
+            const int N = part ? w.N / l.mix_stacked : w.N, K = (w.K + 127) / 128 * 128;
+            memset(&a[i], 0, sizeof(a[i]));
+            a[i].fmt = MI355_W_BF16, a[i].R = 1, a[i].N = N, a[i].K = K;
+            a[i].w = (const char*)w.w + (part ? (int64_t)i * N * K * 2 : 0);
+            a[i].x = (const char*)m->mix + i * stride * 2, a[i].x_dtype = MI355_BF16, a[i].M = M, a[i].ldx = m->ld_n;
+            a[i].epi = MI355_EPI_STORE, a[i].alpha = 1.f;
+            a[i].y = (char*)m->proj + l.mix_at[i] * 2, a[i].y_dtype = MI355_BF16, a[i].ldy = ldp;
+        }
+        return mi355_linear_fast_jobs(a, l.n_mix, s);
+    }
     if (l.mix_stacked > 1) {  // parts of equal size, one stream
         const mi355_proj& w = l.mix_w[0];
         mi355_proj part = w;
@@ -472,7 +539,7 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
     MI355_CHECK_ARG(m->residual_mult != 0.f && m->logit_scale != 0.f, MI355_E_ARG, "hybrid_forward: residual_mult or logit_scale is 0");
     MI355_CHECK_ARG(m->norm_add == 0.f || (m->norm_add == 1.f && m->dtype == MI355_BF16), MI355_E_ARG, "hybrid_forward: norm_add is 0, or 1 in bf16 models");
     MI355_CHECK_ARG(n_want == 0 || run_end < m->n_runs || (logits && m->final_norm), MI355_E_ARG, "hybrid_forward: nowhere to write logits");
-    MI355_CHECK_ARG(m->norm_groups == 0 || (m->norm_groups > 0 && m->width % m->norm_groups == 0 && m->norm_add == 0.f && m->ld_n >= (m->width + 127) / 128 * 128 &&
+    MI355_CHECK_ARG(m->norm_groups == 0 || (m->norm_groups > 0 && m->width % m->norm_groups == 0 && m->norm_add == 0.f && m->norm_dtype == m->dtype && m->ld_n >= (m->width + 127) / 128 * 128 &&
                                             m->ld_n % 8 == 0), MI355_E_SHAPE, "hybrid_forward: bad norm groups %d of width %d", m->norm_groups, m->width);
     for (int r = 0; r < m->n_runs; ++r) {
         const mi355_hybrid_layer& l = m->layers[r];

@@ -280,21 +280,29 @@ __global__ __launch_bounds__(512) void latent_mfma_kernel(const LatParams p) {
     const bf16_t* cache = (const bf16_t*)a.cache + (int64_t)p.b.slot[seq] * a.cache_rows * p.ld_c;
     const int cols = DK / 8, items = kStep * cols;
     u32x4 reg[kTileItems<RB>];
-    auto load = [&](int kb) {
+    int key_of[kTileItems<RB>], at[kTileItems<RB>];  // a thread's chunks of a step: key, place in the LDS tile
+    {
+        const int dk = 512 / cols, dc = 512 - dk * cols;
+        int key = tid / cols, col = tid - key * cols;
 #pragma unroll
         for (int i = 0; i < kTileItems<RB>; ++i) {
-            const int it = tid + 512 * i;
-            const int key = it / cols, col = it - key * cols;
-            reg[i] = it < items && kb + key < end ? *(const u32x4*)(cache + (int64_t)(kb + key) * p.ld_c + col * 8) : u32x4{0u, 0u, 0u, 0u};
+            const bool in = tid + 512 * i < items;
+            key_of[i] = in ? key : 0x3fffffff;
+            at[i] = in ? key * P + col * 8 : 0;
+            key += dk, col += dc;
+            if (col >= cols) ++key, col -= cols;
         }
+    }
+    auto load = [&](int kb) {
+        const bf16_t* src = cache + (int64_t)kb * p.ld_c;
+#pragma unroll
+        for (int i = 0; i < kTileItems<RB>; ++i)  // (an LDS row is P elements, a cache row ld_c)
+            reg[i] = key_of[i] < end - kb ? *(const u32x4*)(src + (at[i] - key_of[i] * (P - p.ld_c))) : u32x4{0u, 0u, 0u, 0u};
     };
     auto store = [&]() {
 #pragma unroll
-        for (int i = 0; i < kTileItems<RB>; ++i) {
-            const int it = tid + 512 * i;
-            const int key = it / cols, col = it - key * cols;
-            if (it < items) *(u32x4*)(ks + key * P + col * 8) = reg[i];
-        }
+        for (int i = 0; i < kTileItems<RB>; ++i)
+            if (key_of[i] < kStep) *(u32x4*)(ks + at[i]) = reg[i];
     };
     if (begin < end) load(begin);
     for (int it = tid; it < 16 * NH * cols; it += 512) {
@@ -458,15 +466,15 @@ __global__ __launch_bounds__(256) void latent_out_rows_kernel(const LatParams p)
     }
 }
 
-// grid (heads, 64-value blocks, 16-row tiles), 256 threads; kv_rank % 8 == 0, vdim % 4 == 0.  LDS: [16][pad32(kv_rank) + 8] bf16
-__global__ __launch_bounds__(256) void latent_out_mfma_kernel(const LatParams p, int rows) {
+// grid (heads, 64-value blocks, tiles of `tile` <= 16 rows), 256 threads; kv_rank % 8 == 0, vdim % 4 == 0.  LDS: [16][pad32(kv_rank) + 8] bf16
+__global__ __launch_bounds__(256) void latent_out_mfma_kernel(const LatParams p, int rows, int tile) {
     const mi355_latent_args& a = p.a;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     __shared__ float wgt[16][kMaxSplit];
-    const int h = blockIdx.x, t0 = p.row0 + blockIdx.z * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int h = blockIdx.x, t0 = p.row0 + blockIdx.z * tile, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
     const int end = p.row0 + rows, R = a.kv_rank, Rp = pad32(R), P = Rp + 8, ld = R + kRec;
     bf16_t* os = (bf16_t*)smem;
-    const int n = min(16, end - t0);
+    const int n = min(tile, end - t0);
     for (int t = wave; t < n; t += 4) {
         float w;
         const float inv = split_weight(record(p, t0 + t, h, 0), ld, p.n_split, lane, w);
@@ -474,12 +482,12 @@ __global__ __launch_bounds__(256) void latent_out_mfma_kernel(const LatParams p,
     }
     __syncthreads();
     const int quads = Rp / 4;
-    for (int it = tid; it < 16 * quads; it += 256) {
+    for (int it = tid; it < n * quads; it += 256) {  // (rows past n: whatever stands there, in columns of the product that nobody stores)
         const int t = it / quads, r = (it - t * quads) * 4;
         f32x4 o = {0.f, 0.f, 0.f, 0.f};
-        if (t < n && r < R) {
+        if (r < R) {
             const float* rec = record(p, t0 + t, h, 0) + kRec + r;
-#pragma unroll 8
+#pragma unroll 16
             for (int s = 0; s < p.n_split; ++s) o += wgt[t][s] * *(const f32x4*)(rec + (int64_t)s * ld);
         }
         u32x2 b;
@@ -577,8 +585,9 @@ int run_latents(LatParams p, bool mfma, hipStream_t s) {
                 if (a.kv_rank <= 256) rc = nh == 2 ? launch_mfma<2, 1>(p, m, s) : launch_mfma<1, 1>(p, m, s);
                 else rc = nh == 2 ? launch_mfma<2, 2>(p, m, s) : launch_mfma<1, 2>(p, m, s);
                 if (rc) return rc;
-                hipLaunchKernelGGL(latent_out_mfma_kernel, dim3(a.heads, (a.vdim + 63) / 64, (m + 15) / 16), dim3(256),
-                                   (size_t)16 * (pad32(a.kv_rank) + 8) * 2, s, p, m);
+                const int tile = m >= 64 ? 16 : m >= 32 ? 8 : 4;  // (the records are the bytes: enough workgroups to read them)
+                hipLaunchKernelGGL(latent_out_mfma_kernel, dim3(a.heads, (a.vdim + 63) / 64, (m + tile - 1) / tile), dim3(256),
+                                   (size_t)16 * (pad32(a.kv_rank) + 8) * 2, s, p, m, tile);
                 MI355_LAUNCH_CHECK();
                 continue;
             }

@@ -21,5 +21,7 @@ struct mi355_product {
 // The weight-streaming kernel up to 8 rows, the tiled product above it (and where its LDS has no room for the operand); f32: the exact
 // generic kernel.  hybrid.hip
 int mi355_product_run(const mi355_product& p, const mi355_proj& w, hipStream_t s);
+// mi355_linear_fast of up to 8 products in one launch (bf16 operands without norm, STORE; they differ in w, x, y and N alone).  gemv.hip
+int mi355_linear_fast_jobs(const mi355_linear_args* a, int count, mi355_stream_t stream);
 // does a product of M rows take the tiled kernel?
 bool mi355_product_wide(const mi355_proj& w, int M, int R);

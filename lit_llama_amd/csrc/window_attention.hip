@@ -490,11 +490,15 @@ __device__ __forceinline__ float sigmoid_fast(float z) {  // (in front of a roun
 }
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 
-template <int D, int DV>  // key and value sizes padded to D and DV (multiples of 32)
-constexpr int tiles_lds() { return 2 * (kBK * D * 2 + DV * kVtRow); }
+// key and value sizes padded to D and DV (multiples of 32).  Wide keys in front of narrow values (D 192) go global -> LDS without registers
+// in between, and the values keep one tile: two workgroups fit a CU
+template <int D>
+constexpr bool kDmaKeys = D == 192;
+template <int D, int DV>
+constexpr int tiles_lds() { return 2 * kBK * D * 2 + (kDmaKeys<D> ? 1 : 2) * DV * kVtRow; }
 
 template <int D, int DV>
-__global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(const WinParams p) {
+__global__ __launch_bounds__(256, D <= 192 ? 2 : 1) void window_tiles_kernel(const WinParams p) {
     const mi355_window_attn_args& a = p.a;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     constexpr int kCols = D / 8;                       // 16-B columns of a key row
@@ -586,16 +590,42 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     const bf16_t* vcur = (const bf16_t*)p.vrows + k_row0 * p.ld_rows + (int64_t)kvh * a.vdim;
     const bf16_t* tail = (const bf16_t*)a.key_tail + (int64_t)p.b.slot[seq] * a.tail_slot - kdim;  // (read from column kdim on)
     const int p_last = pos0 + cnt - 1;
-    u32x4 kreg[kKItems], vreg[kVItems][4];
+    u32x4 kreg[kDmaKeys<D> ? 1 : kKItems], vreg[kVItems][4];
     const u32x4 zero4 = {0u, 0u, 0u, 0u};
     const int t_key = threadIdx.x / kCols, t_col = threadIdx.x % kCols, t_run = threadIdx.x & 15, t_vcol = threadIdx.x >> 4;
     const bool k_in = t_col * 8 < a.dim;
+    constexpr bool kDma = kDmaKeys<D>;
+    constexpr int kVTiles = kDma ? 1 : 2;
+    // kDma: a thread's chunks of a step, one after the other in LDS (chunk = (key, slot); slot s of a key holds column s ^ (key & kSwz))
+    int dkey[kDma ? kKItems : 1], dcol[kDma ? kKItems : 1];
+    if constexpr (kDma) {
+#pragma unroll
+        for (int i = 0; i < kKItems; ++i) {
+            const int it = i * 256 + threadIdx.x;
+            dkey[i] = it / kCols;
+            dcol[i] = ((it % kCols) ^ (dkey[i] & kSwz)) * 8;
+            if (dcol[i] >= a.dim) dcol[i] = 0;  // (the query has zeros there: any finite key will do)
+        }
+    }
+    auto dma_keys = [&](int kb, int buf) {
+#pragma unroll
+        for (int i = 0; i < kKItems; ++i) {
+            const int kp = min(kb * kBK + dkey[kDma ? i : 0], p_last), col = dcol[kDma ? i : 0];
+            const bf16_t* src = (col >= kdim ? tail + (unsigned)kp * (unsigned)a.ld_tail
+                                 : kp >= k_pos0 ? kcur + (unsigned)(kp - k_pos0) * (unsigned)p.ld_rows
+                                                : kcache + (unsigned)cache_row(a, kp) * (unsigned)a.dim) + col;
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
+                                             (__attribute__((address_space(3))) void*)(smem + buf * kKTile + (i * 256 + wave * 64) * 16), 16, 0, 0);
+        }
+    };
     auto load_tile = [&](int kb) {
-        if (kPow2 && a.tail_dims == 0 && kb * kBK >= k_pos0 && kb * kBK + kBK - 1 <= p_last) {  // all of the step's own rows: one multiply per thread
+        if ((kDma || a.tail_dims == 0) && kb * kBK >= k_pos0 && kb * kBK + kBK - 1 <= p_last) {  // all of the step's own rows: one multiply per thread
             const unsigned ld = (unsigned)p.ld_rows;
             const unsigned ko = (unsigned)(kb * kBK + t_key - k_pos0) * ld + t_col * 8;
+            if constexpr (!kDma) {
 #pragma unroll
-            for (int i = 0; i < kKItems; ++i) kreg[i] = *(const u32x4*)(kcur + (k_in ? ko + (unsigned)i * (256 / kCols) * ld : 0u));
+                for (int i = 0; i < kKItems; ++i) kreg[i] = *(const u32x4*)(kcur + (k_in ? ko + (unsigned)i * (256 / kCols) * ld : 0u));
+            }
             const unsigned vo = (unsigned)(kb * kBK + t_run * 4 - k_pos0) * ld;
 #pragma unroll
             for (int i = 0; i < kVItems; ++i) {
@@ -604,7 +634,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
 #pragma unroll
                 for (int r = 0; r < 4; ++r) vreg[i][r] = *(const u32x4*)(vcur + (o + (unsigned)r * ld));
             }
-            if (!k_in) {
+            if (!kDma && !k_in) {
 #pragma unroll
                 for (int i = 0; i < kKItems; ++i) kreg[i] = zero4;
             }
@@ -619,7 +649,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
             return;
         }
 #pragma unroll
-        for (int i = 0; i < kKItems; ++i) {
+        for (int i = 0; i < (kDma ? 0 : kKItems); ++i) {
             const int it = i * 256 + threadIdx.x, key = it / kCols, col = it % kCols;
             const int kp = kb * kBK + key;
             kreg[i] = zero4;
@@ -646,9 +676,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     };
     auto store_tile = [&](int buf) {
         char* kt = smem + buf * kKTile;
-        char* vt = smem + 2 * kKTile + buf * kVTile;
+        char* vt = smem + 2 * kKTile + (buf & (kVTiles - 1)) * kVTile;
 #pragma unroll
-        for (int i = 0; i < kKItems; ++i) {
+        for (int i = 0; i < (kDma ? 0 : kKItems); ++i) {
             const int it = i * 256 + threadIdx.x, key = it / kCols, col = it % kCols;
             *(u32x4*)(kt + key * (D * 2) + ((col ^ (key & kSwz)) << 4)) = kreg[i];
         }
@@ -686,14 +716,18 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
     }
     int kb = n_first > 0 ? 0 : kb0, buf = 0;
 
+    if constexpr (kDma) dma_keys(kb, 0);
     load_tile(kb);
     store_tile(0);
-    __syncthreads();
+    __syncthreads();  // (also waits for the keys on their way to LDS)
     for (; kb < kb1; buf ^= 1) {
         const int next = kb + 1 == n_first ? kb0 : kb + 1;
-        if (next < kb1) load_tile(next);
+        if (next < kb1) {
+            if constexpr (kDma) dma_keys(next, buf ^ 1);
+            load_tile(next);
+        }
         const char* kt = smem + buf * kKTile;
-        const char* vt = smem + 2 * kKTile + buf * kVTile;
+        const char* vt = smem + 2 * kKTile + (buf & (kVTiles - 1)) * kVTile;
         // a wave none of whose queries sees this step leaves it out (it still stages the next tile)
         const bool seen = kb * kBK <= w_last && (kb * kBK + kBK - 1 >= w_first_lo || kb * kBK < a.keep);
         if (seen) {
@@ -766,6 +800,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_tiles_kernel(con
                 }
             }
         }
+        if constexpr (kDma) __syncthreads();  // (every wave is done with the step's values)
         if (next < kb1) store_tile(buf ^ 1);
         __syncthreads();
         kb = next;
@@ -932,6 +967,7 @@ int make_params(const mi355_window_attn_args* a, const mi355_seq_batch* b, WinPa
                     MI355_E_SHAPE, "window_attention: bad window %d, ring %d or rotation %d", a->window, a->ring, a->rot_dims);
     MI355_CHECK_ARG(a->keep >= 0 && a->keep <= a->kept, MI355_E_SHAPE, "window_attention: %d first rows visible, %d cached", a->keep, a->kept);
     MI355_CHECK_ARG(a->role == MI355_KV_ROWS ? b->max_count > 1 && a->rows_per_seq > 0 && a->tail_dims >= 0 && a->tail_dims < a->dim && a->tail_dims % 8 == 0 &&
+                                                   (uint64_t)a->rows_per_seq * (uint64_t)a->ld_tail < 0xFFFFFFFFull &&
                                                    a->off_v_rows % 8 == 0 && (a->tail_dims == 0 || (a->key_tail && a->ld_tail % 8 == 0 && a->tail_slot % 8 == 0 &&
                                                                                                     (uintptr_t)a->key_tail % 16 == 0))
                                              : a->tail_dims == 0,
