@@ -869,7 +869,7 @@ typedef struct mi355_hybrid_model {
     float* xw;             /* [max_rows, ldx] rows whose logits are wanted */
     float* xn;             /* [max_rows, ld_n] f32 models: normalised rows */
     uint16_t* xb;          /* [max_rows, ld_n] bf16 models: normalised rows of a wide product or of a parallel layer */
-    void* mix;             /* [5][max_rows][ld_n] of dtype: the shifted mixes of a parallel layer */
+    void* mix;             /* [5][max_rows * ld_n + 1152] of dtype: the shifted mixes of a parallel layer */
     void* proj;            /* [max_rows, widest in.N] of dtype */
     void* att;             /* [max_rows, widest out.K padded to 16] of dtype */
     void* hid;             /* [max_rows, widest up.N (f32 pairs: 3 up.N)] of dtype */

@@ -118,11 +118,12 @@ __device__ __forceinline__ f32x4 get4(const T* p) {
     }
 }
 
-// One row per workgroup, and with MIX a second one: the row before, or, in the workgroup of a portion's first row, the portion's last one (it
-// enters the state there).  H > 0: rows of up to 2048 H values whose groups are whole runs of 256 (a wave's load), held in registers;
-// H = 0: any width.  Dynamic LDS: sums of squares [2][max(runs, 8, groups)], 1 / rms [2][groups]
+// One row per workgroup.  H > 0: rows of up to 2048 H values whose groups are whole runs of 256 (a wave's load), held in registers; H = 0: any
+// width, and with MIX a second row: the row before, or, in the workgroup of a portion's first row, the portion's last one (it enters the
+// state there).  Dynamic LDS: sums of squares [2][max(runs, 8, groups)], 1 / rms [2][groups]
 template <typename T, bool MIX, int H>
 __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
+    static_assert(!MIX || H == 0, "rows with mixes in registers: norm_mix_kernel");
     extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ int s_seq;
     const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -134,9 +135,8 @@ __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
     const float* other = row;
     int seq = 0, i = 0;
     if constexpr (MIX) {
-        if (p.b.max_count == 1) {
-            seq = m;
-        } else {
+        seq = m;
+        if (p.b.max_count > 1) {
             for (int s = tid; s < p.b.seqs; s += 512)
                 if (m >= p.b.row0[s] && m < p.b.row0[s] + p.b.count[s]) s_seq = s;
             __syncthreads();
@@ -146,14 +146,12 @@ __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
         }
     }
     constexpr int HH = H > 0 ? H : 1;
-    f32x4 a[HH], o[HH], sc[HH];
+    f32x4 a[HH], sc[HH];
     if constexpr (H > 0) {
 #pragma unroll
         for (int j = 0; j < H; ++j) {
             const int k = 4 * (tid + 512 * j);
-            const bool in = k < p.width;
-            a[j] = in ? *(const f32x4*)(row + k) : f32x4{0.f, 0.f, 0.f, 0.f};
-            if constexpr (MIX) o[j] = in ? *(const f32x4*)(other + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+            a[j] = k < p.width ? *(const f32x4*)(row + k) : f32x4{0.f, 0.f, 0.f, 0.f};
         }
 #pragma unroll
         for (int j = 0; j < H; ++j) {
@@ -163,12 +161,7 @@ __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
 #pragma unroll
         for (int j = 0; j < H; ++j) {
             const float s0 = group_sum((a[j][0] * a[j][0] + a[j][1] * a[j][1]) + (a[j][2] * a[j][2] + a[j][3] * a[j][3]), 64);
-            const int q = wave + 8 * j;
-            if (lane == 0 && q < n_sums) sums[q] = s0;
-            if constexpr (MIX) {
-                const float s1 = group_sum((o[j][0] * o[j][0] + o[j][1] * o[j][1]) + (o[j][2] * o[j][2] + o[j][3] * o[j][3]), 64);
-                if (lane == 0 && q < n_sums) sums[n_sums + q] = s1;
-            }
+            if (lane == 0 && wave + 8 * j < n_sums) sums[wave + 8 * j] = s0;
         }
     } else {
         const int seg = (p.size + per - 1) / per;
@@ -196,33 +189,15 @@ __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
     }
     __syncthreads();
     T* h = (T*)p.h + (int64_t)m * p.ldh;
-    float* state = MIX ? p.shift + (int64_t)p.b.slot[seq] * p.width : nullptr;
-    const bool first = MIX && i == 0, begun = first && p.b.pos[seq] > 0;
     if constexpr (H > 0) {
 #pragma unroll
         for (int j = 0; j < H; ++j) {
             const int k = 4 * (tid + 512 * j);
-            if (k >= p.width) continue;
-            const int gr = (wave + 8 * j) / per;
-            const f32x4 v = a[j] * rinv[gr] * sc[j];
-            put4(h + k, v);
-            if constexpr (MIX) {
-                f32x4 mu[5], d = o[j] * rinv[p.groups + gr] * sc[j];
-#pragma unroll
-                for (int s = 0; s < 5; ++s)
-                    if (s < p.n_mix) mu[s] = *(const f32x4*)(p.mu + (int64_t)s * p.width + k);
-                if (first) {  // (d: the portion's last row; of one row, itself)
-                    const f32x4 old = begun ? *(const f32x4*)(state + k) : f32x4{0.f, 0.f, 0.f, 0.f};
-                    *(f32x4*)(state + k) = d;
-                    d = old;
-                }
-                d = d - v;
-#pragma unroll
-                for (int s = 0; s < 5; ++s)
-                    if (s < p.n_mix) put4((T*)p.mix + s * p.mix_stride + (int64_t)m * p.ldh + k, v + d * mu[s]);
-            }
+            if (k < p.width) put4(h + k, a[j] * rinv[(wave + 8 * j) / per] * sc[j]);
         }
     } else {
+        float* state = MIX ? p.shift + (int64_t)p.b.slot[seq] * p.width : nullptr;
+        const bool first = MIX && i == 0, begun = first && p.b.pos[seq] > 0;
         for (int k = tid; k < p.width; k += 512) {
             const int gr = k / p.size;
             const float scale = ld_as_f32(p.scale, k, sizeof(T) == 4 ? MI355_F32 : MI355_BF16);
@@ -230,7 +205,7 @@ __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
             st_from_f32(h, k, sizeof(T) == 4 ? MI355_F32 : MI355_BF16, v);
             if constexpr (MIX) {
                 float d = other[k] * rinv[p.groups + gr] * scale;
-                if (first) {
+                if (first) {  // (d: the portion's last row; of one row, itself)
                     const float old = begun ? state[k] : 0.f;
                     state[k] = d;
                     d = old;
@@ -244,14 +219,123 @@ __global__ __launch_bounds__(512) void norm_groups_kernel(const NormParams p) {
     }
 }
 
+// The same with the mixes, for rows of up to 2048 H values, `per_wg` consecutive rows per workgroup: the factors stay in registers, and a row is
+// the next one's predecessor.  Dynamic LDS: sums of squares [2 (turns)][width / 256], 1 / rms [2][groups]
+constexpr int kMixRows = 4;
+template <typename T, int H>
+__global__ __launch_bounds__(512) void norm_mix_kernel(const NormParams p, int rows, int per_wg) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    __shared__ int s_seq[kMixRows];
+    const int m0 = blockIdx.x * per_wg, n = min(per_wg, rows - m0), tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int per = p.size / 256, n_sums = p.groups * per;
+    int turn = 0;
+    f32x4 sc[H], mu[5][H], raw[H], h[H], before[H];
+    auto request = [&](const float* row) {
+#pragma unroll
+        for (int j = 0; j < H; ++j) {
+            const int k = 4 * (tid + 512 * j);
+            raw[j] = k < p.width ? *(const f32x4*)(row + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+    };
+    // raw -> out = norm(raw)
+    auto norm = [&](f32x4 (&out)[H]) {
+        float* sums = sm + turn * n_sums;
+        float* rinv = sm + 2 * n_sums + turn * p.groups;
+        turn ^= 1;
+#pragma unroll
+        for (int j = 0; j < H; ++j) {
+            out[j] = raw[j] * sc[j];
+            const float s = group_sum((raw[j][0] * raw[j][0] + raw[j][1] * raw[j][1]) + (raw[j][2] * raw[j][2] + raw[j][3] * raw[j][3]), 64);
+            if (lane == 0 && wave + 8 * j < n_sums) sums[wave + 8 * j] = s;
+        }
+        __syncthreads();
+        for (int q = tid; q < p.groups; q += 512) {
+            float s = 0.f;
+            for (int j = 0; j < per; ++j) s += sums[q * per + j];
+            rinv[q] = 1.0f / sqrtf(s / (float)p.size + p.eps);
+        }
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < H; ++j)
+            if (4 * (tid + 512 * j) < p.width) out[j] *= rinv[(wave + 8 * j) / per];
+    };
+    const float* row = p.x + (int64_t)m0 * p.ldx;
+    request(m0 > 0 ? row - p.ldx : row);  // (the row before, in case it belongs to the same portion)
+#pragma unroll
+    for (int j = 0; j < H; ++j) {
+        const int k = 4 * (tid + 512 * j);
+        const bool in = k < p.width;
+        sc[j] = in ? get4((const T*)p.scale + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < 5; ++s) mu[s][j] = in && s < p.n_mix ? *(const f32x4*)(p.mu + (int64_t)s * p.width + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    if (p.b.max_count == 1) {
+        if (tid < n) s_seq[tid] = m0 + tid;
+    } else {
+        for (int s = tid; s < p.b.seqs; s += 512) {
+            const int r0 = p.b.row0[s], r1 = r0 + p.b.count[s];
+            for (int m = max(r0, m0); m < min(r1, m0 + n); ++m) s_seq[m - m0] = s;
+        }
+    }
+    __syncthreads();
+    if (p.b.row0[s_seq[0]] < m0) norm(before);
+    request(row);
+    for (int r = 0; r < n; ++r) {
+        const int seq = s_seq[r], i = m0 + r - p.b.row0[seq], cnt = p.b.count[seq];
+        norm(h);
+        if (i == 0) {  // what the state holds is this row's predecessor; the portion's last row replaces it
+            float* state = p.shift + (int64_t)p.b.slot[seq] * p.width;
+            const bool begun = p.b.pos[seq] > 0;
+            f32x4 last[H];
+            if (cnt > 1) {
+                request(row + (int64_t)(r + cnt - 1) * p.ldx);
+                norm(last);
+            }
+#pragma unroll
+            for (int j = 0; j < H; ++j) {
+                const int k = 4 * (tid + 512 * j);
+                if (k >= p.width) continue;
+                before[j] = begun ? *(const f32x4*)(state + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+                *(f32x4*)(state + k) = cnt > 1 ? last[j] : h[j];
+            }
+        }
+        if (r + 1 < n) request(row + (int64_t)(r + 1) * p.ldx);
+        const int64_t at = (int64_t)(m0 + r) * p.ldh;
+#pragma unroll
+        for (int j = 0; j < H; ++j) {
+            const int k = 4 * (tid + 512 * j);
+            if (k >= p.width) continue;
+            put4((T*)p.h + at + k, h[j]);
+            const f32x4 d = before[j] - h[j];
+#pragma unroll
+            for (int s = 0; s < 5; ++s)
+                if (s < p.n_mix) put4((T*)p.mix + s * p.mix_stride + at + k, h[j] + d * mu[s][j]);
+            before[j] = h[j];
+        }
+    }
+}
+
 template <typename T, bool MIX>
 void launch_norm(const NormParams& p, int rows, hipStream_t s) {
     const bool whole = p.size % 256 == 0 && p.width <= 8192;
     const int sums = whole ? p.width / 256 : p.groups < 8 ? 8 : p.groups;
     const size_t lds = (size_t)2 * (sums + p.groups) * 4;
-    if (whole && p.width <= 4096) hipLaunchKernelGGL((norm_groups_kernel<T, MIX, 2>), dim3(rows), dim3(512), lds, s, p);
-    else if (whole) hipLaunchKernelGGL((norm_groups_kernel<T, MIX, 4>), dim3(rows), dim3(512), lds, s, p);
-    else hipLaunchKernelGGL((norm_groups_kernel<T, MIX, 0>), dim3(rows), dim3(512), lds, s, p);
+    if constexpr (MIX) {
+        if (whole) {
+            const int per_wg = p.b.max_count == 1 ? 1 : kMixRows;
+            if (p.width <= 4096) hipLaunchKernelGGL((norm_mix_kernel<T, 2>), dim3((rows + per_wg - 1) / per_wg), dim3(512), lds, s, p, rows, per_wg);
+            else hipLaunchKernelGGL((norm_mix_kernel<T, 4>), dim3((rows + per_wg - 1) / per_wg), dim3(512), lds, s, p, rows, per_wg);
+            return;
+        }
+    }
+    if constexpr (!MIX) {
+        if (whole) {
+            if (p.width <= 4096) hipLaunchKernelGGL((norm_groups_kernel<T, false, 2>), dim3(rows), dim3(512), lds, s, p);
+            else hipLaunchKernelGGL((norm_groups_kernel<T, false, 4>), dim3(rows), dim3(512), lds, s, p);
+            return;
+        }
+    }
+    hipLaunchKernelGGL((norm_groups_kernel<T, MIX, 0>), dim3(rows), dim3(512), lds, s, p);
 }
 
 // rows [gate | up] of 2 n values -> the clamped gated unit
@@ -382,6 +466,9 @@ int linear(const mi355_hybrid_model* m, const mi355_proj& w, const void* x, int6
     return mi355_linear_fast(&a, s);
 }
 
+// between the mixes of a row: not a power of two, so that a row's mixes lie on different memory channels
+int64_t mix_stride(const mi355_hybrid_model* m) { return (int64_t)m->max_rows * m->ld_n + 1152; }
+
 int norm_groups(const mi355_hybrid_model* m, const void* scale, const mi355_hybrid_layer* l, const mi355_seq_batch* b, const int32_t* want, int rows,
                 hipStream_t s) {
     NormParams p;
@@ -393,7 +480,7 @@ int norm_groups(const mi355_hybrid_model* m, const void* scale, const mi355_hybr
     p.h = f32 ? (void*)m->xn : (void*)m->xb, p.ldh = m->ld_n;
     if (l != nullptr && l->n_mix > 0) {
         p.n_mix = l->n_mix, p.mu = l->mu, p.shift = l->shift;
-        p.mix = m->mix, p.mix_stride = (int64_t)m->max_rows * m->ld_n;
+        p.mix = m->mix, p.mix_stride = mix_stride(m);
         p.b = *b;
     }
     if (f32) p.n_mix > 0 ? launch_norm<float, true>(p, rows, s) : launch_norm<float, false>(p, rows, s);
@@ -419,7 +506,7 @@ int parallel_in(const mi355_hybrid_model* m, const mi355_hybrid_layer& l, int M,
     const int64_t ldp = l.in.N;
     if (l.n_mix == 0) return mi355_product_run(product_of(m, f32 ? (void*)m->xn : (void*)m->xb, m->ld_n, M, MI355_EPI_STORE, m->proj, ldp, m->dtype), l.in, s);
     const size_t size = dtype_size(m->dtype);
-    const int64_t stride = (int64_t)m->max_rows * m->ld_n;
+    const int64_t stride = mix_stride(m);
     int i = 0;
     if (!f32 && l.mix_stacked > 1 && !mi355_product_wide(l.mix_w[0], M, 1)) {  // a few rows: every mix's product in one launch
         mi355_linear_args a[5];

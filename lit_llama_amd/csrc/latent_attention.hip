@@ -62,33 +62,88 @@ __device__ __forceinline__ int seq_of(const LatParams& p, int row, int* shared) 
     return *shared;
 }
 
-// grid (rows), 256 threads
-template <typename T>
+// grid (rows), 256 threads; V = 8: bf16 rows of whole 16-B vectors
+template <typename T, int V>
 __global__ __launch_bounds__(256) void latent_prep_kernel(const LatParams p) {
     const mi355_latent_args& a = p.a;
     __shared__ float red[32];
     __shared__ int s_seq;
-    const int row = blockIdx.x, seq = seq_of(p, row, &s_seq), tid = threadIdx.x;
-    const int pos = p.b.pos[seq] + row - p.b.row0[seq];
+    const int row = blockIdx.x, tid = threadIdx.x;
     const T* src = (const T*)a.proj + (int64_t)row * a.ld;
     const T *cq = src + a.off_q, *c = src + a.off_c, *tail = c + a.kv_rank;
-    float sq = 0.f, sc = 0.f;
-    for (int k = tid; k < a.q_rank; k += 256) sq += to_f32<T>(cq[k]) * to_f32<T>(cq[k]);
-    for (int k = tid; k < a.kv_rank; k += 256) sc += to_f32<T>(c[k]) * to_f32<T>(c[k]);
+    T* oq = (T*)a.cq + (int64_t)row * p.ld_cq;
+    // vectors of V values, the query latent's in front of c's; a thread's first two stay in registers
+    constexpr int kHeld = 2;
+    const int nq = a.q_rank / V, nv = nq + a.kv_rank / V;
+    float x[kHeld][V], sq = 0.f, sc = 0.f;
+    auto get = [&](int v, float (&f)[V]) {
+        const T* at = v < nq ? cq + v * V : c + (v - nq) * V;
+        if constexpr (V == 8) {
+            const u32x4 r = *(const u32x4*)at;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) f[2 * e] = __uint_as_float(r[e] << 16), f[2 * e + 1] = __uint_as_float(r[e] & 0xffff0000u);
+        } else {
+            f[0] = to_f32<T>(at[0]);
+        }
+    };
+    auto add = [&](int v, const float (&f)[V]) {
+        float t = 0.f;
+#pragma unroll
+        for (int e = 0; e < V; ++e) t += f[e] * f[e];
+        if (v < nq) sq += t;
+        else sc += t;
+    };
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i)
+        if (tid + 256 * i < nv) get(tid + 256 * i, x[i]);
+    float u0 = 0.f, w0 = 0.f;
+    if (tid < a.rot_dim / 2) u0 = to_f32<T>(tail[2 * tid]), w0 = to_f32<T>(tail[2 * tid + 1]);
+    // (the row is on its way while its sequence is looked up)
+    const int seq = seq_of(p, row, &s_seq);
+    const int pos = p.b.pos[seq] + row - p.b.row0[seq];
+    T* o = (T*)a.cache + ((int64_t)p.b.slot[seq] * a.cache_rows + pos) * p.ld_c;
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i)
+        if (tid + 256 * i < nv) add(tid + 256 * i, x[i]);
+    for (int v = tid + 256 * kHeld; v < nv; v += 256) {
+        float f[V];
+        get(v, f);
+        add(v, f);
+    }
     sq = group_sum(sq, 64);
     sc = group_sum(sc, 64);
     if ((tid & 63) == 0) red[tid >> 6] = sq, red[4 + (tid >> 6)] = sc;
     __syncthreads();
     const float rq = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.q_rank + a.eps);
     const float rc = 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)a.kv_rank + a.eps);
-    T* oq = (T*)a.cq + (int64_t)row * p.ld_cq;
-    for (int k = tid; k < a.q_rank; k += 256) oq[k] = from_f32<T>(to_f32<T>(cq[k]) * rq * a.q_norm[k]);
+    auto put = [&](int v, const float (&f)[V]) {
+        const bool isq = v < nq;
+        const int k = (isq ? v : v - nq) * V;
+        const float* w = (isq ? a.q_norm : a.c_norm) + k;
+        const float r = isq ? rq : rc;
+        T* at = (isq ? oq : o) + k;
+        if constexpr (V == 8) {
+            u32x4 b;
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                b[e] = (uint32_t)f32_to_bf16(f[2 * e] * r * w[2 * e]) | ((uint32_t)f32_to_bf16(f[2 * e + 1] * r * w[2 * e + 1]) << 16);
+            *(u32x4*)at = b;
+        } else {
+            at[0] = from_f32<T>(f[0] * r * w[0]);
+        }
+    };
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i)
+        if (tid + 256 * i < nv) put(tid + 256 * i, x[i]);
+    for (int v = tid + 256 * kHeld; v < nv; v += 256) {
+        float f[V];
+        get(v, f);
+        put(v, f);
+    }
     for (int k = a.q_rank + tid; k < p.ld_cq; k += 256) oq[k] = from_f32<T>(0.f);
-    T* o = (T*)a.cache + ((int64_t)p.b.slot[seq] * a.cache_rows + pos) * p.ld_c;
-    for (int k = tid; k < a.kv_rank; k += 256) o[k] = from_f32<T>(to_f32<T>(c[k]) * rc * a.c_norm[k]);
     o += a.kv_rank;
     for (int i = tid; i < a.rot_dim / 2; i += 256) {
-        float u = to_f32<T>(tail[2 * i]), w = to_f32<T>(tail[2 * i + 1]);
+        float u = i == tid ? u0 : to_f32<T>(tail[2 * i]), w = i == tid ? w0 : to_f32<T>(tail[2 * i + 1]);
         turn(pos, a.inv_freq[i], u, w);
         o[2 * i] = from_f32<T>(u);
         o[2 * i + 1] = from_f32<T>(w);
@@ -664,8 +719,11 @@ extern "C" int mi355_latent_attention(const mi355_latent_args* a, const mi355_se
     p.ld_qh = a->dim + a->rot_dim;
     p.rows_per_seq = 0;
     const bool f32 = a->dtype == MI355_F32;
-    if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(b->rows), dim3(256), 0, s, p);
-    else hipLaunchKernelGGL(latent_prep_kernel<bf16_t>, dim3(b->rows), dim3(256), 0, s, p);
+    const bool vec = vec_sizes(*a) && a->q_rank % 8 == 0 && a->ld % 8 == 0 && a->off_q % 8 == 0 && a->off_c % 8 == 0 && (uintptr_t)a->proj % 16 == 0 &&
+                     (uintptr_t)a->cq % 16 == 0;
+    if (f32) hipLaunchKernelGGL((latent_prep_kernel<float, 1>), dim3(b->rows), dim3(256), 0, s, p);
+    else if (vec) hipLaunchKernelGGL((latent_prep_kernel<bf16_t, 8>), dim3(b->rows), dim3(256), 0, s, p);
+    else hipLaunchKernelGGL((latent_prep_kernel<bf16_t, 1>), dim3(b->rows), dim3(256), 0, s, p);
     MI355_LAUNCH_CHECK();
     mi355_product q;
     memset(&q, 0, sizeof(q));

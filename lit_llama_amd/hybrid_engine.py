@@ -326,7 +326,7 @@ class HybridEngine:
             n = int(lib().mi355_linear_gemm_workspace_bytes(R, _pad128(K)))
             M.gemm_ws, M.gemm_ws_bytes = ptr(self._buf(n, torch.uint8)), n
             M.xb = ptr(self._buf(R * M.ld_n, torch.bfloat16))
-        M.mix = ptr(self._buf(R * M.ld_n * max([l.n_mix for l in ls], default=0), self.dtype))
+        M.mix = ptr(self._buf((R * M.ld_n + 1152) * max([l.n_mix for l in ls], default=0), self.dtype))
         self._latent_scratch()
         # a split attention step keeps one record per (row, head, split); one split takes none
         n = max([512 * (l.attn.vdim + 2) * max(8, l.attn.heads // l.attn.kv_heads) for l in ls if l.mixer == 0], default=0)
