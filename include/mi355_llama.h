@@ -729,6 +729,28 @@ int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_batch* b, mi3
 /* scratch bytes a chunked prompt step of `rows` rows in `seqs` sequences takes; 0: the shape runs row by row */
 size_t mi355_recurrent_scratch_bytes(int kind, int rows, int seqs, int heads, int kv_heads, int dim, int vdim);
 
+/* h = norm(x): every one of `groups` equal parts of a row over its own root mean square, times scale; and, with n_mix > 0, the token shift's
+ * mixes: mix i of a row is h + (h' - h) mu[i], h' = h of the row before in its sequence: `shift` of the slot in front of a portion (0 at
+ * position 0), which the portion's last h replaces. */
+typedef struct mi355_norm_args {
+    int32_t dtype;         /* of scale, h and mix */
+    int32_t rows, width, groups;
+    const float* x;        /* [.., ldx] */
+    int64_t ldx;
+    const int32_t* want;   /* row of x per row of h (no mixes), or NULL: the same */
+    float eps;
+    int32_t n_mix;         /* 0 .. 5 */
+    const void* scale;     /* [width] */
+    void* h;               /* [rows, ldh] */
+    int64_t ldh;
+    const float* mu;       /* [n_mix][width] */
+    float* shift;          /* [slots][width] */
+    void* mix;             /* [n_mix][rows, ldh], mix_stride elements apart */
+    int64_t mix_stride;
+} mi355_norm_args;
+
+int mi355_norm_groups(const mi355_norm_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
+
 /* A weight of a hybrid model: BF16 stream (mi355_bf16_repack, R = 1) of a bf16 model, row-major f32 of an f32 model */
 typedef struct mi355_proj {
     const void* w;

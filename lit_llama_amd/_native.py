@@ -201,6 +201,14 @@ class LatentArgs(C.Structure):
     ]
 
 
+class NormArgs(C.Structure):
+    _fields_ = [
+        ("dtype", c_int32), ("rows", c_int32), ("width", c_int32), ("groups", c_int32), ("x", c_void_p), ("ldx", c_int64), ("want", c_void_p),
+        ("eps", c_float), ("n_mix", c_int32), ("scale", c_void_p), ("h", c_void_p), ("ldh", c_int64), ("mu", c_void_p), ("shift", c_void_p),
+        ("mix", c_void_p), ("mix_stride", c_int64),
+    ]
+
+
 class HybridLayer(C.Structure):
     _fields_ = [
         ("mixer", c_int32), ("mlp", c_int32), ("norm1", c_void_p), ("norm2", c_void_p),
@@ -293,6 +301,7 @@ PROTOTYPES = {
     "mi355_window_attention": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_window_cache_write": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_latent_attention": (c_int, [C.POINTER(LatentArgs), C.POINTER(SeqBatch), c_void_p]),
+    "mi355_norm_groups": (c_int, [C.POINTER(NormArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_experts": (c_int, [C.POINTER(ExpertsArgs), c_void_p]),
     "mi355_experts_scratch_bytes": (c_size_t, [C.POINTER(ExpertsArgs)]),
     "mi355_recurrent": (c_int, [C.POINTER(RecurrentArgs), C.POINTER(SeqBatch), c_void_p]),
@@ -306,7 +315,7 @@ PROTOTYPES = {
 }
 
 ABI_STRUCTS = [LinearArgs, AttnArgs, Int8Args, Weight, Layer, Model, FusedStepArgs, TpComm,
-               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel, ExpertsArgs, LatentArgs]
+               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel, ExpertsArgs, LatentArgs, NormArgs]
 
 _lib: Optional[C.CDLL] = None
 

@@ -38,6 +38,7 @@ extern "C" int mi355_sizeof(int which) {
         case 13: return (int)sizeof(mi355_hybrid_model);
         case 14: return (int)sizeof(mi355_experts_args);
         case 15: return (int)sizeof(mi355_latent_args);
+        case 16: return (int)sizeof(mi355_norm_args);
         default: return -1;
     }
 }

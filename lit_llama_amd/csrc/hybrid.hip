@@ -80,20 +80,8 @@ __global__ __launch_bounds__(512) void norm_rows_kernel(const float* x, int64_t 
 }
 
 // ---- parallel layers: h = norm(x) in groups, and the mixes h + (h' - h) mu of the token shift (h' = the row before)
-struct NormParams {
-    const float* x;
-    int64_t ldx;
-    const int32_t* want;    // rows of x, or NULL: row m
-    int width, groups, size;
-    float eps;
-    const void* scale;      // of the model's dtype
-    void* h;                // [rows, ldh]
-    int64_t ldh;
-    int n_mix;
-    const float* mu;        // [n_mix][width]
-    float* shift;           // [slots][width]
-    void* mix;              // [n_mix], mix_stride apart, as h
-    int64_t mix_stride;
+struct NormParams : mi355_norm_args {
+    int size;               // of a group
     mi355_seq_batch b;
 };
 
@@ -471,22 +459,17 @@ int64_t mix_stride(const mi355_hybrid_model* m) { return (int64_t)m->max_rows * 
 
 int norm_groups(const mi355_hybrid_model* m, const void* scale, const mi355_hybrid_layer* l, const mi355_seq_batch* b, const int32_t* want, int rows,
                 hipStream_t s) {
-    NormParams p;
-    memset(&p, 0, sizeof(p));
-    const bool f32 = m->dtype == MI355_F32;
-    p.x = m->x, p.ldx = m->ldx, p.want = want;
-    p.width = m->width, p.groups = m->norm_groups, p.size = m->width / m->norm_groups;
-    p.eps = m->eps, p.scale = scale;
-    p.h = f32 ? (void*)m->xn : (void*)m->xb, p.ldh = m->ld_n;
+    mi355_norm_args a;
+    memset(&a, 0, sizeof(a));
+    a.dtype = m->dtype, a.rows = rows, a.width = m->width, a.groups = m->norm_groups;
+    a.x = m->x, a.ldx = m->ldx, a.want = want;
+    a.eps = m->eps, a.scale = scale;
+    a.h = m->dtype == MI355_F32 ? (void*)m->xn : (void*)m->xb, a.ldh = m->ld_n;
     if (l != nullptr && l->n_mix > 0) {
-        p.n_mix = l->n_mix, p.mu = l->mu, p.shift = l->shift;
-        p.mix = m->mix, p.mix_stride = mix_stride(m);
-        p.b = *b;
+        a.n_mix = l->n_mix, a.mu = l->mu, a.shift = l->shift;
+        a.mix = m->mix, a.mix_stride = mix_stride(m);
     }
-    if (f32) p.n_mix > 0 ? launch_norm<float, true>(p, rows, s) : launch_norm<float, false>(p, rows, s);
-    else p.n_mix > 0 ? launch_norm<bf16_t, true>(p, rows, s) : launch_norm<bf16_t, false>(p, rows, s);
-    MI355_LAUNCH_CHECK();
-    return 0;
+    return mi355_norm_groups(&a, b, (mi355_stream_t)s);
 }
 
 mi355_product product_of(const mi355_hybrid_model* m, const void* x, int64_t ldx, int M, int epi, void* y, int64_t ldy, int y_dtype) {
@@ -580,6 +563,32 @@ int parallel_out(const mi355_hybrid_model* m, const mi355_hybrid_layer& l, int M
 }
 
 }  // namespace
+
+extern "C" int mi355_norm_groups(const mi355_norm_args* a, const mi355_seq_batch* b, mi355_stream_t stream) {
+    MI355_CHECK_ARG(a && a->x && a->scale && a->h, MI355_E_ARG, "norm_groups: null argument");
+    MI355_CHECK_ARG(a->dtype == MI355_F32 || a->dtype == MI355_BF16, MI355_E_DTYPE, "norm_groups: dtype must be f32 or bf16");
+    MI355_CHECK_ARG(a->rows > 0 && a->width > 0 && a->groups > 0 && a->groups <= 4096 && a->width % a->groups == 0 && a->ldx >= a->width && a->ldh >= a->width,
+                    MI355_E_SHAPE, "norm_groups: %d groups of a row of %d", a->groups, a->width);
+    MI355_CHECK_ARG((uintptr_t)a->x % 16 == 0 && a->ldx % 4 == 0 && (uintptr_t)a->h % 16 == 0 && a->ldh % 8 == 0 && (uintptr_t)a->scale % 16 == 0, MI355_E_SHAPE,
+                    "norm_groups: rows and scale start at multiples of 16 bytes");
+    NormParams p;
+    memset(&p, 0, sizeof(p));
+    (mi355_norm_args&)p = *a;
+    p.size = a->width / a->groups;
+    if (a->n_mix > 0) {
+        MI355_CHECK_ARG(b && b->row0 && b->count && b->slot && b->pos && b->rows == a->rows && b->max_count > 0 && a->want == nullptr, MI355_E_ARG,
+                        "norm_groups: mixes need the batch of their rows");
+        MI355_CHECK_ARG(a->n_mix <= 5 && a->mu && a->shift && a->mix && a->mix_stride % 8 == 0 && (uintptr_t)a->mix % 16 == 0 && (uintptr_t)a->mu % 16 == 0 &&
+                            (uintptr_t)a->shift % 16 == 0,
+                        MI355_E_ARG, "norm_groups: bad mixes");
+        p.b = *b;
+    }
+    hipStream_t s = (hipStream_t)stream;
+    if (a->dtype == MI355_F32) a->n_mix > 0 ? launch_norm<float, true>(p, a->rows, s) : launch_norm<float, false>(p, a->rows, s);
+    else a->n_mix > 0 ? launch_norm<bf16_t, true>(p, a->rows, s) : launch_norm<bf16_t, false>(p, a->rows, s);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
 
 bool mi355_product_wide(const mi355_proj& w, int M, int R) {
     const int K = (w.K + 127) / 128 * 128;

@@ -614,7 +614,7 @@ class PackedBatch:
         self.meta = torch.tensor([row0, list(counts), list(slots), list(pos)], dtype=torch.int32, device=device)
         self.rows = sum(counts)
         b = self.c = nat.SeqBatch()
-        b.rows, b.seqs, b.max_count = self.rows, len(counts), max(counts)
+        b.rows, b.seqs, b.max_count, b.max_end = self.rows, len(counts), max(counts), max(p + n for p, n in zip(pos, counts))
         b.row0, b.count, b.slot, b.pos = (ptr(self.meta[i]) for i in range(4))
 
 
@@ -622,12 +622,22 @@ def window_attention(proj: torch.Tensor, batch: PackedBatch, kring: torch.Tensor
                      off_q: int, off_k: int, off_v: int, off_g: int = -1, inv_freq: Optional[torch.Tensor] = None, path: int = 0,
                      partials: Optional[torch.Tensor] = None, keep: int = 0, kept: int = 0, gate_values: bool = False,
                      unit_eps: Optional[float] = None, sink: Optional[torch.Tensor] = None, role: str = "own",
-                     kv_rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     kv_rows: Optional[torch.Tensor] = None, chunked: bool = False, head_scale: Optional[torch.Tensor] = None,
+                     slope: Optional[torch.Tensor] = None, unit_v_eps: Optional[float] = None) -> torch.Tensor:
     """mi355_window_attention: proj [rows, ld] (k prepared in place by prompt steps), rings [slots, kv_heads, kept + ring, dim | vdim]
     (written).  `unit_eps`: q and k over their root mean square.  `role` own | lends | borrows: a lender fills `kv_rows` in a prompt step and
-    its cache is written by `window_cache_write`; a borrower has neither key nor value columns."""
+    its cache is written by `window_cache_write`; a borrower has neither key nor value columns.  `chunked`: the window is a chunk of the
+    sequence; `head_scale`, `slope`: per head a factor of the scores and what is taken off per position of distance; `unit_v_eps`: v over its
+    root mean square."""
     y, a = _window_args(proj, batch, kring, vring, heads, scale, window, off_q, off_k, off_v, off_g, inv_freq, path, partials, keep, kept,
                         gate_values, unit_eps, sink, role, kv_rows)
+    a.chunked = int(chunked)
+    for t in (head_scale, slope):
+        assert t is None or (t.dtype == torch.float32 and t.numel() == heads and t.is_contiguous())
+    a.head_scale, a.slope = ptr(head_scale), ptr(slope)
+    if unit_v_eps is not None:
+        assert unit_eps is None or unit_eps == unit_v_eps
+        a.unit_v, a.unit_eps = 1, unit_v_eps
     check(lib().mi355_window_attention(C.byref(a), C.byref(batch.c), stream_ptr()), "mi355_window_attention")
     return y
 
@@ -703,14 +713,14 @@ def experts(x: torch.Tensor, norm: torch.Tensor, router: torch.Tensor, weights, 
 
 def recurrent(kind: str, proj: torch.Tensor, batch: PackedBatch, state: torch.Tensor, *, off: dict, kv_heads: int, head_norm: torch.Tensor,
               eps: float, conv_ring: Optional[torch.Tensor] = None, conv=None, a_log=None, dt_bias=None, a2=None, a2_bias=None,
-              tau: float = 1.0, path: int = 0) -> torch.Tensor:
-    """mi355_recurrent: `kind` delta | gla, state [slots, heads, dim, vdim] f32 (updated), `off`: first columns of q, k, v, g, a (and b);
+              tau: float = 1.0, path: int = 0, bonus: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """mi355_recurrent: `kind` delta | gla | wkv (`off` q: r, a: the decay's low-rank input; head_norm per channel), state [slots, heads, dim, vdim] f32 (updated), `off`: first columns of q, k, v, g, a (and b);
     `conv`: the (q, k, v) taps of the delta rule, f32 [channels, taps]."""
     require_gpu(proj, "recurrent")
     _, H, dim, vdim = state.shape
     y = torch.zeros((batch.rows, H * vdim), dtype=proj.dtype, device=proj.device)
     r = nat.RecurrentArgs()
-    r.kind, r.dtype = (0 if kind == "delta" else 1), dtype_code(proj.dtype)
+    r.kind, r.dtype = ("delta", "gla", "wkv").index(kind), dtype_code(proj.dtype)
     r.proj, r.ld = ptr(proj), proj.shape[1]
     r.heads, r.kv_heads, r.dim, r.vdim = H, kv_heads, dim, vdim
     r.off_q, r.off_k, r.off_v, r.off_g, r.off_a = (off[n] for n in "qkvga")
@@ -723,8 +733,76 @@ def recurrent(kind: str, proj: torch.Tensor, batch: PackedBatch, state: torch.Te
         r.a_log, r.dt_bias, r.conv_ring = ptr(a_log), ptr(dt_bias), ptr(conv_ring)
     else:
         r.rank, r.inv_tau, r.a2, r.a2_bias = a2.shape[1], 1.0 / tau, ptr(a2), ptr(a2_bias)
+        if kind == "wkv":
+            assert bonus.dtype == torch.float32 and bonus.numel() == H * dim and head_norm.numel() == H * vdim
+            r.q_scale, r.norm_ld, r.bonus = 1.0, vdim, ptr(bonus)
     need = int(lib().mi355_recurrent_scratch_bytes(r.kind, batch.rows, batch.c.seqs, H, kv_heads, dim, vdim))
     scratch = torch.empty(max(need, 4), dtype=torch.uint8, device=proj.device)
     r.scratch, r.scratch_bytes = ptr(scratch), need
     check(lib().mi355_recurrent(C.byref(r), C.byref(batch.c), stream_ptr()), "mi355_recurrent")
     return y
+
+
+def norm_groups(x: torch.Tensor, scale: torch.Tensor, groups: int, eps: float, *, want: Optional[torch.Tensor] = None, batch: Optional[PackedBatch] = None,
+                mu: Optional[torch.Tensor] = None, shift: Optional[torch.Tensor] = None):
+    """mi355_norm_groups: x [rows, width] f32 -> h of scale's dtype; with `mu` [n, width] (h, mixes [n, rows, width]), `shift` [slots, width]
+    updated."""
+    require_gpu(x, "norm_groups")
+    W = x.shape[1]
+    rows = x.shape[0] if want is None else want.numel()
+    ldx, ldh = (W + 15) // 16 * 16, (W + 127) // 128 * 128
+    xp = torch.zeros((x.shape[0], ldx), dtype=torch.float32, device=x.device)
+    xp[:, :W] = x
+    n = 0 if mu is None else mu.shape[0]
+    out = torch.zeros((1 + n, rows, ldh), dtype=scale.dtype, device=x.device)
+    a = nat.NormArgs()
+    a.dtype, a.rows, a.width, a.groups, a.x, a.ldx, a.want = dtype_code(scale.dtype), rows, W, groups, ptr(xp), ldx, ptr(want)
+    a.eps, a.scale, a.h, a.ldh, a.n_mix = eps, ptr(scale), ptr(out), ldh, n
+    if n:
+        assert mu.dtype == shift.dtype == torch.float32 and mu.is_contiguous() and shift.is_contiguous() and shift.shape[1] == W and batch.rows == rows
+        a.mu, a.shift, a.mix, a.mix_stride = ptr(mu), ptr(shift), ptr(out[1]), rows * ldh
+    check(lib().mi355_norm_groups(C.byref(a), C.byref(batch.c) if batch is not None else None, stream_ptr()), "mi355_norm_groups")
+    assert not out[:, :, W:].any()
+    return (out[0, :, :W], out[1:, :, :W]) if n else out[0, :, :W]
+
+
+def latent_attention(proj: torch.Tensor, batch: PackedBatch, cache: torch.Tensor, w, *, heads: int, dim: int, rot_dim: int, vdim: int, off_q: int,
+                     off_c: int, scale: float, eps: float, inv_freq: torch.Tensor, path: int = 0, partials_bytes: int = 1 << 24,
+                     expand_rows: Optional[int] = None) -> torch.Tensor:
+    """mi355_latent_attention: proj [rows, ld] with the query latent at off_q and [latent | rotated key part] at off_c, cache [slots, positions,
+    kv_rank + rot_dim] (written); `w`: uq, uk, uv of proj's dtype, q_norm, c_norm, sink f32.  The scratch is full of NaNs."""
+    require_gpu(proj, "latent_attention")
+    rows, dt, dev = batch.rows, proj.dtype, proj.device
+    R, rq = w["uk"].shape[1], w["uq"].shape[1]
+    pad = lambda n, m: (n + m - 1) // m * m
+    nan = lambda n, t=dt: torch.full((max(1, n),), float("nan"), dtype=t, device=dev)
+    assert proj.is_contiguous() and cache.dtype == dt and cache.is_contiguous() and cache.shape[2] == R + rot_dim
+    assert inv_freq.dtype == torch.float64 and inv_freq.numel() == rot_dim // 2 and all(w[n].dtype == torch.float32 for n in ("q_norm", "c_norm", "sink"))
+    keep = []
+
+    def proj_of(t):
+        t = torch.nn.functional.pad(t, (0, 0, 0, pad(t.shape[0], 16) - t.shape[0]))
+        keep.append(repack_bf16(t, None, 1) if dt == torch.bfloat16 else t.contiguous())
+        return nat.Proj(ptr(keep[-1]), t.shape[0], t.shape[1])
+
+    a = nat.LatentArgs()
+    a.proj, a.ld, a.dtype, a.heads, a.dim, a.rot_dim, a.vdim, a.q_rank, a.kv_rank = ptr(proj), proj.shape[1], dtype_code(dt), heads, dim, rot_dim, vdim, rq, R
+    a.off_q, a.off_c, a.scale, a.eps, a.cache_rows, a.path = off_q, off_c, scale, eps, cache.shape[1], path
+    a.q_norm, a.c_norm, a.inv_freq, a.sink, a.cache = ptr(w["q_norm"]), ptr(w["c_norm"]), ptr(inv_freq), ptr(w["sink"]), ptr(cache)
+    a.uq = proj_of(w["uq"])
+    keep += [w["uk"].view(heads, dim, R).transpose(1, 2).contiguous(), w["uv"].contiguous()]
+    a.uk_t, a.uv = ptr(keep[-2]), ptr(keep[-1])
+    y = torch.zeros((rows, pad(heads * vdim, 4)), dtype=dt, device=dev)
+    a.y, a.ldy = ptr(y), y.shape[1]
+    bufs = [nan(rows * pad(rq, 128)), nan(rows * a.uq.N), nan(rows * heads * (R + rot_dim)), nan(partials_bytes // 4, torch.float32)]
+    a.cq, a.q, a.qa, a.partials, a.partials_bytes = (*(ptr(b) for b in bufs), partials_bytes)
+    if dt == torch.bfloat16:
+        rows16 = lambda t: torch.nn.functional.pad(t, (0, 0, 0, pad(t.shape[0], 16) - t.shape[0]))
+        a.expand = proj_of(torch.cat([rows16(w["uk"]), rows16(w["uv"])]))
+        E = expand_rows or max(1, batch.c.max_end) * batch.c.seqs
+        bufs += [nan(E * pad(R, 128)), nan(E * a.expand.N)]
+        ws = int(lib().mi355_linear_gemm_workspace_bytes(max(E, rows), max(pad(R, 128), pad(rq, 128))))
+        bufs.append(torch.empty(ws, dtype=torch.uint8, device=dev))
+        a.rows_c, a.kv_rows, a.expand_rows, a.gemm_ws, a.gemm_ws_bytes = ptr(bufs[4]), ptr(bufs[5]), E, ptr(bufs[6]), ws
+    check(lib().mi355_latent_attention(C.byref(a), C.byref(batch.c), stream_ptr()), "mi355_latent_attention")
+    return y[:, :heads * vdim]

@@ -50,7 +50,8 @@ def test_every_field_of_every_struct_sits_where_the_header_puts_it(tmp_path):
              ("mi355_model", nat.Model), ("mi355_fused_step_args", nat.FusedStepArgs), ("mi355_tp_comm", nat.TpComm),
              ("mi355_seq_batch", nat.SeqBatch), ("mi355_window_attn_args", nat.WindowAttnArgs), ("mi355_recurrent_args", nat.RecurrentArgs),
              ("mi355_proj", nat.Proj), ("mi355_hybrid_layer", nat.HybridLayer), ("mi355_hybrid_model", nat.HybridModel),
-             ("mi355_experts_args", nat.ExpertsArgs), ("mi355_latent_args", nat.LatentArgs)]
+             ("mi355_experts_args", nat.ExpertsArgs), ("mi355_latent_args", nat.LatentArgs),
+             ("mi355_norm_args", nat.NormArgs)]
     src = ["#include <stdio.h>", "#include <stddef.h>", '#include "mi355_llama.h"', "int main(void) {"]
     for cname, st in pairs:
         src.append(f'printf("{cname} %zu\\n", sizeof({cname}));')
