@@ -600,7 +600,8 @@ bool mfma_fits(const mi355_latent_args& a) {
 }
 bool tiles_fit(const mi355_latent_args& a, const mi355_seq_batch& b) {
     return vec_sizes(a) && a.dim + a.rot_dim <= 256 && a.vdim <= 256 && a.expand.w && a.rows_c && a.kv_rows && b.max_end > 0 &&
-           b.max_end <= a.expand_rows && (uintptr_t)a.rows_c % 16 == 0 && (uintptr_t)a.kv_rows % 16 == 0;
+           b.max_end <= a.expand_rows && (uint64_t)b.max_end * a.expand.N < 0xFFFFFFFFull && (uint64_t)b.max_end * (a.kv_rank + a.rot_dim) < 0xFFFFFFFFull &&
+           (uint64_t)b.max_count * a.uq.N < 0xFFFFFFFFull && (uintptr_t)a.rows_c % 16 == 0 && (uintptr_t)a.kv_rows % 16 == 0;
 }
 
 template <int NH, int RB>

@@ -323,7 +323,7 @@ def experts_bench_config(width: int, n_layer: int, vocab: int = 32000, window: i
     return {"architecture": "Kovalorn", "layers": layers, "norm": {"eps": 1e-5}, "logit_scale": 0.25, "vocab": vocab, "width": width}
 
 
-def parallel_bench_config(width: int, n_layer: int, vocab: int = 32000, chunk: int = 2048) -> dict:
+def parallel_bench_config(width: int, n_layer: int, vocab: int = 32000, chunk: int = 4096) -> dict:
     """A Kudazen configuration of a LLaMA's width and feed-forward: chunk attention | latent | wkv | latent layers in turn, heads of 128 (64 more
     rotated dimensions in the latent layers, latents of 512, queries through 3/8 of the width)."""
     heads = width // 128
