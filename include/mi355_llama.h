@@ -114,7 +114,7 @@ typedef struct mi355_linear_args {
     const void* zeros2;
     int32_t sz_dtype;
     int32_t epi;        /* MI355_EPI_* */
-    const void* bias;   /* [N] of sz_dtype or NULL (STORE/ACCUM only) */
+    const void* bias;   /* [N] of sz_dtype or NULL (STORE/ACCUM only; mi355_linear_gemm: f32, BF16 STORE) */
     void* y;            /* [M, ldy] */
     int32_t y_dtype;
     int32_t group_cols; /* Q4, mi355_linear_fast: input columns per (scale, zero) pair ("groupsize", quantization.py:284-333
@@ -680,6 +680,12 @@ typedef struct mi355_window_attn_args {
     int32_t tail_dims;     /* MI355_KV_ROWS: the last tail_dims dimensions of every key are those of key_tail, the same for all heads */
     const void* key_tail;  /* position p of slot t at t * tail_slot + p * ld_tail */
     int64_t ld_tail, tail_slot;
+    const float* q_norm;   /* [dim]: factors of a unit query's / key's dimensions in front of the rotation (unit_qk), or NULL */
+    const float* k_norm;
+    float softcap;         /* != 0: a score s becomes softcap tanh(s / softcap) */
+    float v_mix;           /* v_first: values are (1 - v_mix) v + v_mix v_first, and cached so */
+    const void* v_first;   /* [rows, ld_v_first] of dtype: key head g's value of the same row at column g * vdim, or NULL */
+    int64_t ld_v_first;
 } mi355_window_attn_args;
 
 int mi355_window_attention(const mi355_window_attn_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
@@ -691,18 +697,20 @@ int mi355_window_cache_write(const mi355_window_attn_args* a, const mi355_seq_ba
  *                         S += k u^T, o = S^T q with g = exp(-exp(A_log) softplus(a + dt_bias)), beta = sigmoid(b)
  *   kind MI355_REC_GLA    S = diag(alpha) S + k v^T, o = S^T q with alpha = sigmoid(a2 a1 + a2_bias)^(1 / tau) per key channel
  *   kind MI355_REC_WKV    o = (S + diag(u) k v^T)^T q, then S = diag(w) S + k v^T with w = exp(-exp(a2 tanh(a1) + a2_bias)) per key channel
- * then per head o / rms(o) * head_norm * silu(g). */
-enum { MI355_REC_DELTA = 0, MI355_REC_GLA = 1, MI355_REC_WKV = 2 };
+ * then per head o / rms(o) * head_norm * silu(g).
+ *   kind MI355_REC_SSD    state-space duality: short causal convolutions (with a bias) + SiLU on q, k, v; t = softplus(a + dt_bias),
+ *                         S = exp(-exp(A_log) t) S + t k v^T, o = S^T q + skip v; then o * silu(g), stored in f32 without a norm. */
+enum { MI355_REC_DELTA = 0, MI355_REC_GLA = 1, MI355_REC_WKV = 2, MI355_REC_SSD = 3 };
 typedef struct mi355_recurrent_args {
     int32_t kind;
-    int32_t dtype;         /* of proj, conv_ring and y */
+    int32_t dtype;         /* of proj, conv_ring and y (SSD: y is f32) */
     const void* proj;      /* [rows, ld] */
     int64_t ld;
     int32_t heads, kv_heads, dim, vdim;
-    int32_t off_q, off_k, off_v, off_g, off_a, off_b; /* off_a: DELTA decay input [heads], GLA / WKV low-rank input [rank]; off_b: DELTA only */
+    int32_t off_q, off_k, off_v, off_g, off_a, off_b; /* off_a: DELTA / SSD decay input [heads], GLA / WKV low-rank input [rank]; off_b: DELTA only */
     float q_scale;         /* factor of q */
     float eps;             /* of the output norm */
-    int32_t taps;          /* DELTA: convolution taps */
+    int32_t taps;          /* DELTA, SSD: convolution taps */
     int32_t rank;          /* GLA, WKV */
     float inv_tau;         /* GLA */
     float unit_eps;        /* DELTA */
@@ -723,6 +731,10 @@ typedef struct mi355_recurrent_args {
     int32_t path;          /* 0: by shape; 1: row by row; 2: chunks */
     int32_t norm_ld;       /* 0: the heads share head_norm */
     const float* bonus;    /* WKV: u [heads * dim] */
+    const float* conv_bq;  /* SSD: biases of the convolutions, or NULL: none */
+    const float* conv_bk;
+    const float* conv_bv;
+    const float* skip;     /* SSD: [heads] */
 } mi355_recurrent_args;
 
 int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
@@ -755,7 +767,40 @@ int mi355_norm_groups(const mi355_norm_args* a, const mi355_seq_batch* b, mi355_
 typedef struct mi355_proj {
     const void* w;
     int32_t N, K;
+    const float* bias;     /* [N], or NULL (products that are stored) */
 } mi355_proj;
+
+/* What stands between two sublayers whose result is normalised before it joins the stream, one pass over every row:
+ *   u = the sublayer's row t, or the embedding of tokens;  u = u * sigmoid(gate);  u = u / rms(u) * (norm_add + post)
+ *   x = x + u (an embedding: x = u);  stream_out = x;  x = sum over j < n_stream of average[j] stream[j] + average[n_stream] x
+ *   h = x / rms(x) * (norm_add + next)
+ * Every step but the sum is left out where its operand is NULL (n_stream 0: no average). */
+typedef struct mi355_join_args {
+    int32_t dtype;         /* of the norms, embed and h */
+    int32_t rows, width;
+    float eps, norm_add;
+    int32_t n_stream;
+    const int32_t* tokens; /* [rows]: rows of embed [vocab, width] in place of t */
+    const void* embed;
+    int32_t vocab;
+    int32_t gate_dtype;
+    const float* t;        /* [rows, ldt] */
+    int64_t ldt;
+    const void* gate;      /* [rows, ld_gate] of gate_dtype */
+    int64_t ld_gate;
+    const void* post;      /* [width] */
+    float* x;              /* [rows, ldx] */
+    int64_t ldx;
+    const float* stream;   /* stream[j] at j * stream_stride, rows of pitch ldx */
+    int64_t stream_stride;
+    float* stream_out;     /* [rows, ldx] */
+    const float* average;  /* [n_stream + 1] */
+    const void* next;      /* [width] */
+    void* h;               /* [rows, ldh] */
+    int64_t ldh;
+} mi355_join_args;
+
+int mi355_join_rows(const mi355_join_args* a, mi355_stream_t stream);
 
 /* Causal attention whose keys and values are products with one latent row per position: q = uq (c_q / rms(c_q) * q_norm), per head
  * [dim | rot_dim rotated]; c = c / rms(c) * c_norm; k = [uk c | the rotated tail, shared by all heads], v = uv c; scores (q . k) * scale,
@@ -798,10 +843,17 @@ typedef struct mi355_latent_args {
 
 int mi355_latent_attention(const mi355_latent_args* a, const mi355_seq_batch* b, mi355_stream_t stream);
 
-/* Mixture of experts behind an RMSNorm: x += alpha (sum over the `top` experts with the largest s_e = sigmoid(router_e . h) of
- * s_e / (their sum + 1e-20) * scale * expert_e(h)  +  shared(h)),  expert(h) = down (silu(gate h) * (up h)).
+/* Mixture of experts behind an RMSNorm: x += alpha (sum over the `top` chosen experts of their weight * expert_e(h)  +  shared(h)).
+ * score SIGMOID: s_e = sigmoid(router_e . h), the largest are chosen, weights s_e / (their sum + 1e-20) * scale;  score SOFTMAX: s = softmax over
+ * all router outputs, the largest s_e + correction_e are chosen, weights s_e * scale.  keep_groups > 0: the outputs form `groups` equal runs, and
+ * only those of the keep_groups runs with the largest (corrected) score in them can be chosen.  The last `identity` outputs are experts that
+ * give h itself.  act SILU_GATE: expert(h) = down (silu(gate h) * (up h));  RELU2: down relu(up h)^2 (no shared expert).
  * dtype BF16: streams (mi355_bf16_repack; gate and up a pair stream) in 16-bit products with f32 sums; F32: row-major f32.  The experts'
- * weights lie one behind the other (f32: gate, up, next expert). */
+ * weights lie one behind the other (f32: gate, up, next expert).
+ * `h` given: rows that are normalised already; `logits` given (with h): what the router makes of them.  `out` given: the rows of the sum are
+ * stored there, x is left alone. */
+enum { MI355_SCORE_SIGMOID = 0, MI355_SCORE_SOFTMAX = 1 };
+enum { MI355_ACT_SILU_GATE = 0, MI355_ACT_RELU2 = 1 };
 typedef struct mi355_experts_args {
     int32_t dtype;
     int32_t rows;
@@ -815,7 +867,7 @@ typedef struct mi355_experts_args {
     float norm_add;
     float eps;
     float alpha;
-    const void* router;    /* [experts, width] */
+    const void* router;    /* [experts + identity, width] */
     const void* up;
     const void* down;
     const void* shared_up;
@@ -825,15 +877,26 @@ typedef struct mi355_experts_args {
     void* scratch;         /* mi355_experts_scratch_bytes, 256-byte aligned */
     uint64_t scratch_bytes;
     int32_t path;          /* bf16; 0: by shape; 1: every row by itself; 2: sorted by expert */
+    int32_t score;         /* MI355_SCORE_* */
+    int32_t act;           /* MI355_ACT_* */
+    int32_t identity;
+    int32_t groups, keep_groups;
     int32_t reserved0;
+    const float* correction; /* [experts + identity], or NULL */
+    const void* h;         /* [rows, ldh] of dtype (bf16: zero from width to a multiple of 128), or NULL */
+    int64_t ldh;
+    const float* logits;   /* [rows, ld_logits], or NULL */
+    int64_t ld_logits;
+    float* out;            /* [rows, ld_out], ld_out >= width padded to 16 (bf16: zeros in the padding), or NULL */
+    int64_t ld_out;
 } mi355_experts_args;
 
 int mi355_experts(const mi355_experts_args* a, mi355_stream_t stream);
-/* scratch bytes of a step (dtype, rows, width, experts, top, ff, ff_shared are read) */
+/* scratch bytes of a step (dtype, rows, width, experts, top, ff, ff_shared, act are read) */
 size_t mi355_experts_scratch_bytes(const mi355_experts_args* a);
 
 
-enum { MI355_MIX_ATTENTION = 0, MI355_MIX_DELTA = 1, MI355_MIX_GLA = 2, MI355_MIX_WKV = 3, MI355_MIX_LATENT = 4 };
+enum { MI355_MIX_ATTENTION = 0, MI355_MIX_DELTA = 1, MI355_MIX_GLA = 2, MI355_MIX_WKV = 3, MI355_MIX_LATENT = 4, MI355_MIX_SSD = 5 };
 /* feed-forwards: down relu(up h)^2; down (gelu_tanh(gate h) * (up h)), `up` the pair (BF16 pair stream, or f32 gate rows then up rows;
  * up.N = the hidden size); mixture of experts; down (g sigmoid(1.702 g) (u + 1)) with g = min(gate h, limit), u = clamp(up h, -limit, limit) */
 enum { MI355_MLP_NONE = 0, MI355_MLP_RELU2 = 1, MI355_MLP_GEGLU = 2, MI355_MLP_EXPERTS = 3, MI355_MLP_CLAMPGLU = 4 };
@@ -866,6 +929,19 @@ typedef struct mi355_hybrid_layer {
     mi355_proj mix_w[5];
     int32_t mix_at[5];     /* its first column of proj */
     int32_t mix_stacked;   /* bf16: the first mix_stacked weights are one stream of equal parts, mix_w[0] */
+    /* A SANDWICH layer: x += post1(g1 mixer(h)), x += post2(g2 ff(h)), h the norm of x, g = sigmoid of gate columns that read h too; then x becomes
+     * the average of the stream so far.  The mixer's gate columns stand in `in`, the feed-forward's in `side` (f32 products), the router's
+     * logits behind them; the mixer's output row is `cat`, as of a parallel layer. */
+    int32_t sandwich;
+    int32_t gate_at;       /* first column of `in` */
+    int32_t logits_at;     /* first column of `side` */
+    int32_t out_groups;    /* SSD: equal parts of the output row that are normalised by themselves */
+    const void* post1;     /* [width] */
+    const void* post2;
+    mi355_proj side;
+    const float* average;  /* [run + 2]: weights of the embedding output and of every run's result up to this one */
+    const void* out_norm;  /* SSD: [heads * vdim] of dtype */
+    void* proj_rows;       /* [max_rows, in.N]: a projection buffer of this layer's own (later layers read its values), or NULL */
 } mi355_hybrid_layer;
 
 typedef struct mi355_hybrid_model {
@@ -895,7 +971,7 @@ typedef struct mi355_hybrid_model {
     void* proj;            /* [max_rows, widest in.N] of dtype */
     void* att;             /* [max_rows, widest out.K padded to 16] of dtype */
     void* hid;             /* [max_rows, widest up.N (f32 pairs: 3 up.N)] of dtype */
-    float* tmp;            /* [max_rows, ldx] f32 models: a product in front of its residual */
+    float* tmp;            /* [max_rows, ldx] f32 models, sandwich layers: a product in front of its residual */
     int64_t ld_att;
     void* gemm_ws;
     uint64_t gemm_ws_bytes;
@@ -905,6 +981,12 @@ typedef struct mi355_hybrid_model {
     uint64_t rec_scratch_bytes;
     void* moe_scratch;
     uint64_t moe_scratch_bytes;
+    const void* embed_norm; /* sandwich layers: [width], the embedding's own norm */
+    float* stream;         /* [n_runs + 1][max_rows, ldx]: the embedding output and every run's result */
+    float* side;           /* [max_rows, ld_side]: products of `side` */
+    int64_t ld_side;
+    float* mixed;          /* [max_rows, ld_mixed]: SSD outputs in front of their norm */
+    int64_t ld_mixed;
 } mi355_hybrid_model;
 
 /* embedding, every layer run, and the logits (f32 [n_want, ld_logits]) of the rows want[0 .. n_want) (device; NULL: all rows).

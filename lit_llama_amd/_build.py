@@ -19,7 +19,7 @@ CORE_LIB = PKG / "libmi355core.so"
 OBJ_DIR = PKG / "csrc" / "_obj"
 # what a layered hybrid model runs on; linked alone into CORE_LIB where only such a model is served
 CORE_SOURCES = ["generic.hip", "gemv.hip", "gemm.hip", "sample.hip", "graph.hip", "window_attention.hip", "recurrent.hip",
-                "recurrent_chunks.hip", "latent_attention.hip", "experts.hip", "hybrid.hip"]
+                "recurrent_chunks.hip", "latent_attention.hip", "experts.hip", "join.hip", "hybrid.hip"]
 SOURCES = CORE_SOURCES + ["int8.hip", "int8_gemm.hip", "attention.hip", "engine.hip", "gptq.hip", "fused_step.hip", "fused_step_ring.hip",
                           "fused_step_wide.hip", "tp_comm.hip", "flash_prefill.hip"]
 ARCH = "gfx950"

@@ -159,6 +159,7 @@ class WindowAttnArgs(C.Structure):
         ("role", c_int32), ("chunked", c_int32), ("kv_rows", c_void_p),
         ("head_scale", c_void_p), ("slope", c_void_p), ("unit_v", c_int32), ("rot_at", c_int32), ("rows_per_seq", c_int64), ("ld_rows", c_int64),
         ("off_v_rows", c_int32), ("tail_dims", c_int32), ("key_tail", c_void_p), ("ld_tail", c_int64), ("tail_slot", c_int64),
+        ("q_norm", c_void_p), ("k_norm", c_void_p), ("softcap", c_float), ("v_mix", c_float), ("v_first", c_void_p), ("ld_v_first", c_int64),
     ]
 
 
@@ -172,6 +173,7 @@ class RecurrentArgs(C.Structure):
         ("a2", c_void_p), ("a2_bias", c_void_p), ("head_norm", c_void_p), ("state", c_void_p), ("conv_ring", c_void_p),
         ("y", c_void_p), ("ldy", c_int64), ("scratch", c_void_p), ("scratch_bytes", C.c_uint64),
         ("path", c_int32), ("norm_ld", c_int32), ("bonus", c_void_p),
+        ("conv_bq", c_void_p), ("conv_bk", c_void_p), ("conv_bv", c_void_p), ("skip", c_void_p),
     ]
 
 
@@ -181,12 +183,23 @@ class ExpertsArgs(C.Structure):
         ("ff", c_int32), ("ff_shared", c_int32), ("scale", c_float),
         ("norm", c_void_p), ("norm_dtype", c_int32), ("norm_add", c_float), ("eps", c_float), ("alpha", c_float),
         ("router", c_void_p), ("up", c_void_p), ("down", c_void_p), ("shared_up", c_void_p), ("shared_down", c_void_p),
-        ("x", c_void_p), ("ldx", c_int64), ("scratch", c_void_p), ("scratch_bytes", C.c_uint64), ("path", c_int32), ("reserved0", c_int32),
+        ("x", c_void_p), ("ldx", c_int64), ("scratch", c_void_p), ("scratch_bytes", C.c_uint64), ("path", c_int32),
+        ("score", c_int32), ("act", c_int32), ("identity", c_int32), ("groups", c_int32), ("keep_groups", c_int32), ("reserved0", c_int32),
+        ("correction", c_void_p), ("h", c_void_p), ("ldh", c_int64), ("logits", c_void_p), ("ld_logits", c_int64), ("out", c_void_p), ("ld_out", c_int64),
     ]
 
 
 class Proj(C.Structure):
-    _fields_ = [("w", c_void_p), ("N", c_int32), ("K", c_int32)]
+    _fields_ = [("w", c_void_p), ("N", c_int32), ("K", c_int32), ("bias", c_void_p)]
+
+
+class JoinArgs(C.Structure):
+    _fields_ = [
+        ("dtype", c_int32), ("rows", c_int32), ("width", c_int32), ("eps", c_float), ("norm_add", c_float), ("n_stream", c_int32),
+        ("tokens", c_void_p), ("embed", c_void_p), ("vocab", c_int32), ("gate_dtype", c_int32), ("t", c_void_p), ("ldt", c_int64),
+        ("gate", c_void_p), ("ld_gate", c_int64), ("post", c_void_p), ("x", c_void_p), ("ldx", c_int64), ("stream", c_void_p),
+        ("stream_stride", c_int64), ("stream_out", c_void_p), ("average", c_void_p), ("next", c_void_p), ("h", c_void_p), ("ldh", c_int64),
+    ]
 
 
 class LatentArgs(C.Structure):
@@ -216,6 +229,8 @@ class HybridLayer(C.Structure):
         ("attn", WindowAttnArgs), ("rec", RecurrentArgs), ("moe", ExpertsArgs), ("kv_lender", c_int32), ("kv_last", c_int32),
         ("latent", LatentArgs), ("parallel", c_int32), ("hid_at", c_int32), ("cat", c_void_p), ("ld_cat", c_int64), ("limit", c_float),
         ("n_mix", c_int32), ("mu", c_void_p), ("shift", c_void_p), ("mix_w", Proj * 5), ("mix_at", c_int32 * 5), ("mix_stacked", c_int32),
+        ("sandwich", c_int32), ("gate_at", c_int32), ("logits_at", c_int32), ("out_groups", c_int32), ("post1", c_void_p), ("post2", c_void_p),
+        ("side", Proj), ("average", c_void_p), ("out_norm", c_void_p), ("proj_rows", c_void_p),
     ]
 
 
@@ -230,6 +245,7 @@ class HybridModel(C.Structure):
         ("tmp", c_void_p), ("ld_att", c_int64), ("gemm_ws", c_void_p), ("gemm_ws_bytes", C.c_uint64),
         ("partials", c_void_p), ("partials_bytes", C.c_uint64), ("rec_scratch", c_void_p), ("rec_scratch_bytes", C.c_uint64),
         ("moe_scratch", c_void_p), ("moe_scratch_bytes", C.c_uint64),
+        ("embed_norm", c_void_p), ("stream", c_void_p), ("side", c_void_p), ("ld_side", c_int64), ("mixed", c_void_p), ("ld_mixed", c_int64),
     ]
 
 
@@ -302,6 +318,7 @@ PROTOTYPES = {
     "mi355_window_cache_write": (c_int, [C.POINTER(WindowAttnArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_latent_attention": (c_int, [C.POINTER(LatentArgs), C.POINTER(SeqBatch), c_void_p]),
     "mi355_norm_groups": (c_int, [C.POINTER(NormArgs), C.POINTER(SeqBatch), c_void_p]),
+    "mi355_join_rows": (c_int, [C.POINTER(JoinArgs), c_void_p]),
     "mi355_experts": (c_int, [C.POINTER(ExpertsArgs), c_void_p]),
     "mi355_experts_scratch_bytes": (c_size_t, [C.POINTER(ExpertsArgs)]),
     "mi355_recurrent": (c_int, [C.POINTER(RecurrentArgs), C.POINTER(SeqBatch), c_void_p]),
@@ -315,7 +332,7 @@ PROTOTYPES = {
 }
 
 ABI_STRUCTS = [LinearArgs, AttnArgs, Int8Args, Weight, Layer, Model, FusedStepArgs, TpComm,
-               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel, ExpertsArgs, LatentArgs, NormArgs]
+               SeqBatch, WindowAttnArgs, RecurrentArgs, Proj, HybridLayer, HybridModel, ExpertsArgs, LatentArgs, NormArgs, JoinArgs]
 
 _lib: Optional[C.CDLL] = None
 

@@ -169,6 +169,28 @@ __device__ __forceinline__ float group_sum(float v, int lpr) {
     return v;
 }
 
+// four values of a row as f32
+template <typename T>
+__device__ __forceinline__ void put4(T* p, f32x4 v) {
+    if constexpr (sizeof(T) == 4) {
+        *(f32x4*)p = v;
+    } else {
+        typedef __attribute__((ext_vector_type(2))) __bf16 bf2;
+        const bf2 a = {(__bf16)v[0], (__bf16)v[1]}, b = {(__bf16)v[2], (__bf16)v[3]};
+        *(u32x2*)p = u32x2{__builtin_bit_cast(uint32_t, a), __builtin_bit_cast(uint32_t, b)};
+    }
+}
+
+template <typename T>
+__device__ __forceinline__ f32x4 get4(const T* p) {
+    if constexpr (sizeof(T) == 4) {
+        return *(const f32x4*)p;
+    } else {
+        const u32x2 r = *(const u32x2*)p;
+        return f32x4{__uint_as_float(r[0] << 16), __uint_as_float(r[0] & 0xffff0000u), __uint_as_float(r[1] << 16), __uint_as_float(r[1] & 0xffff0000u)};
+    }
+}
+
 // max(v, 0)^2
 __device__ __forceinline__ float relu2_f32(float v) {
     const float r = fmaxf(v, 0.f);

@@ -1,7 +1,9 @@
-// Mixture of experts: sigmoid router over the normalised row, the `top` largest scores, their experts' gated feed-forwards (SiLU) summed by
-// weight, and an optional shared expert that every row runs; the sum joins the residual stream.
+// Mixture of experts: a router over the normalised row (sigmoids, or a softmax with corrected choices inside the best groups), the `top` chosen
+// experts' feed-forwards (gated SiLU, or squared ReLU) summed by weight, experts that are the row itself, and an optional shared expert that every
+// row runs; the sum joins the residual stream or is stored.
 //
 //   route_rows_kernel    RMSNorm, router and choice of 1 to 16 rows per workgroup (router weights bf16 on the matrix cores, f32 sums)
+//   choose_rows_kernel   the choice alone, where norm and router are another launch's: a wave per row
 //   few rows (decode):   up_rows_kernel, down_rows_kernel: a workgroup per (row tile, chosen expert, row) / (row tile, row), every weight
 //                        piece read once per row that chose its expert; three launches in all
 //   many rows:           plan_kernel sorts the (row, choice) pairs by expert and cuts them into tiles; grouped_kernel multiplies a tile of up
@@ -34,7 +36,9 @@ struct Tile {      // up to BM rows of one expert
 struct Params {
     mi355_experts_args a;
     int kp, fp, fsp, np;        // width and the experts' ff in whole units of 128, width in whole tiles of 16
-    bf16_t* xn;                 // [rows][kp] normalised rows (f32 models: float [rows][width])
+    int outputs;                // of the router: experts, then those that are the row itself
+    bf16_t* xn;                 // [rows][ldxn] normalised rows (f32 models: float)
+    int64_t ldxn;
     int32_t* ids;               // [rows][top]
     float* weights;             // [rows][top]
     bf16_t* hid;                // [rows * top][fp] (f32 models: float [rows * top][ff])
@@ -59,9 +63,58 @@ __device__ __forceinline__ float wave_top(float v) {
     return fmaxf(v, lane_xor32(v));
 }
 
-// one wave: the `top` largest of z[0 .. E) (LDS, overwritten; lowest index first among equals), their sigmoids scaled to sum to `scale`
-__device__ __forceinline__ void choose(float* z, int E, int top, float scale, int32_t* ids, float* weights) {
-    const int lane = threadIdx.x & 63;
+// a wave's own LDS writes are in place before it reads them
+__device__ __forceinline__ void wave_lds_sync() {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// floats of LDS that choose() takes per row next to the logits
+__host__ __device__ __forceinline__ int choose_floats(const mi355_experts_args& a, int E) {
+    return a.score == MI355_SCORE_SIGMOID ? 0 : E + (a.keep_groups > 0 ? a.groups : 0);
+}
+
+// One wave: a row's experts and weights from its logits z[0 .. E) (LDS, overwritten; lowest index first among equals); `more`: choose_floats
+__device__ __forceinline__ void choose(const mi355_experts_args& a, float* z, float* more, int E, int32_t* ids, float* weights) {
+    const int lane = threadIdx.x & 63, top = a.top;
+    float* s = more;         // SOFTMAX: scores, without the correction
+    if (a.score == MI355_SCORE_SOFTMAX) {
+        float m = -INFINITY;
+        for (int e = lane; e < E; e += 64) m = fmaxf(m, z[e]);
+        m = wave_top(m);
+        float total = 0.f;
+        for (int e = lane; e < E; e += 64) {
+            const float v = expf(z[e] - m);
+            s[e] = v;
+            total += v;
+        }
+        total = group_sum(total, 64);
+        for (int e = lane; e < E; e += 64) {
+            const float v = s[e] / total;
+            s[e] = v;
+            z[e] = a.correction != nullptr ? v + a.correction[e] : v;
+        }
+        if (a.keep_groups > 0) {
+            float* best = more + E;  // per group
+            const int size = E / a.groups;
+            wave_lds_sync();
+            for (int g = lane; g < a.groups; g += 64) {
+                float v = -INFINITY;
+                for (int e = g * size; e < (g + 1) * size; ++e) v = fmaxf(v, z[e]);
+                best[g] = v;
+            }
+            wave_lds_sync();
+            for (int e = lane; e < E; e += 64) {
+                const int g = e / size;
+                const float mine = best[g];
+                int ahead = 0;
+                for (int o = 0; o < a.groups; ++o) ahead += best[o] > mine || (best[o] == mine && o < g);
+                if (ahead >= a.keep_groups) z[e] = -INFINITY;
+            }
+        }
+        wave_lds_sync();
+    }
     float best = -INFINITY;
     int bi = lane < E ? lane : E - 1;  // (rows of NaNs)
     auto scan = [&] {
@@ -79,22 +132,42 @@ __device__ __forceinline__ void choose(float* z, int E, int top, float scale, in
         unsigned long long at = __ballot(best == v);
         if (at == 0) at = 1;
         int i = __builtin_amdgcn_readlane(bi, __builtin_ctzll(at));
-        for (unsigned long long more = at & (at - 1); more != 0; more &= more - 1) i = min(i, __builtin_amdgcn_readlane(bi, __builtin_ctzll(more)));
+        for (unsigned long long more_at = at & (at - 1); more_at != 0; more_at &= more_at - 1) i = min(i, __builtin_amdgcn_readlane(bi, __builtin_ctzll(more_at)));
         if (lane == k) mine = v, my_id = i;
         if (lane == (i & 63)) {
             z[i] = -INFINITY;
             scan();
         }
     }
-    const float s = lane < top ? 1.0f / (1.0f + expf(-mine)) : 0.f;
-    const float total = group_sum(s, 64);
+    if (a.score == MI355_SCORE_SOFTMAX) {
+        if (lane < top) {
+            ids[lane] = my_id;
+            weights[lane] = s[my_id] * a.scale;
+        }
+        return;
+    }
+    const float sg = lane < top ? 1.0f / (1.0f + expf(-mine)) : 0.f;
+    const float total = group_sum(sg, 64);
     if (lane < top) {
         ids[lane] = my_id;
-        weights[lane] = s / (total + 1e-20f) * scale;
+        weights[lane] = sg / (total + 1e-20f) * a.scale;
     }
 }
 
-// grid ceil(rows / R), 512 threads; R = 1, 2, 4, 8, 16.  LDS: partial logits [8 waves][tiles of a pass][256], logits [R][experts + 1]
+// grid ceil(rows / 4), 256 threads.  LDS: per wave the logits and choose_floats
+__global__ __launch_bounds__(256) void choose_rows_kernel(const Params p) {
+    const mi355_experts_args& a = p.a;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, row = blockIdx.x * 4 + wave, E = p.outputs;
+    if (row >= a.rows) return;
+    float* z = (float*)smem + wave * (E + choose_floats(a, E));
+    const float* from = a.logits + (int64_t)row * a.ld_logits;
+    for (int e = lane; e < E; e += 64) z[e] = from[e];
+    wave_lds_sync();
+    choose(a, z, z + E, E, p.ids + (int64_t)row * a.top, p.weights + (int64_t)row * a.top);
+}
+
+// grid ceil(rows / R), 512 threads; R = 1, 2, 4, 8, 16.  LDS: partial logits [8 waves][tiles of a pass][256], logits [R][outputs + 1], choose_floats [R]
 constexpr int kRouteTiles = 2;
 template <int R>
 __global__ __launch_bounds__(512) void route_rows_kernel(const Params p) {
@@ -105,7 +178,7 @@ __global__ __launch_bounds__(512) void route_rows_kernel(const Params p) {
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int g = lane >> 4, c = lane & 15;
     const int row0 = blockIdx.x * R;
-    const int W = a.width, E = a.experts, tiles = (E + 15) / 16, pass = tiles < kRouteTiles ? tiles : kRouteTiles;
+    const int W = a.width, E = p.outputs, tiles = (E + 15) / 16, pass = tiles < kRouteTiles ? tiles : kRouteTiles;
     float* part = (float*)smem;
     float* z = part + 8 * pass * 256;
     // a wave's first router weights are requested ahead of the norm, the next unit's ahead of a unit's products (past the last tile or unit:
@@ -126,7 +199,7 @@ __global__ __launch_bounds__(512) void route_rows_kernel(const Params p) {
         const int row = row0 + wave / kPer + 8 * i, share = wave % kPer;
         const bool live = row < a.rows;
         const float* x = a.x + (int64_t)(live ? row : row0) * a.ldx;
-        bf16_t* o = p.xn + (int64_t)row * p.kp;
+        bf16_t* o = p.xn + (int64_t)row * p.ldxn;
         const bool vec = W % 4 == 0 && a.norm_dtype == MI355_BF16;
         constexpr int kHeld = 16 / kPer, kStep = 64 * kPer;  // (rows of 4096; what lies behind is read twice)
         f32x4 v[kHeld];
@@ -180,7 +253,7 @@ __global__ __launch_bounds__(512) void route_rows_kernel(const Params p) {
     }
     __syncthreads();
     const int row = min(row0 + c % R, a.rows - 1);
-    const bf16_t* xr = p.xn + (int64_t)row * p.kp + 32 * g;
+    const bf16_t* xr = p.xn + (int64_t)row * p.ldxn + 32 * g;
     for (int t0 = 0; t0 < tiles; t0 += pass) {
         f32x4 acc[kRouteTiles];
 #pragma unroll
@@ -218,10 +291,10 @@ __global__ __launch_bounds__(512) void route_rows_kernel(const Params p) {
         __syncthreads();
     }
     for (int r = wave; r < R && row0 + r < a.rows; r += 8)
-        choose(z + r * (E + 1), E, a.top, a.scale, p.ids + (int64_t)(row0 + r) * a.top, p.weights + (int64_t)(row0 + r) * a.top);
+        choose(a, z + r * (E + 1), z + R * (E + 1) + r * choose_floats(a, E), E, p.ids + (int64_t)(row0 + r) * a.top, p.weights + (int64_t)(row0 + r) * a.top);
 }
 
-// f32 models: one row per workgroup.  LDS: the normalised row, the logits
+// f32 models: one row per workgroup.  LDS: the normalised row, the logits, choose_floats
 __global__ __launch_bounds__(256) void exact_route_kernel(const Params p) {
     const mi355_experts_args& a = p.a;
     extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -232,10 +305,10 @@ __global__ __launch_bounds__(256) void exact_route_kernel(const Params p) {
     float ss = 0.f;
     for (int k = threadIdx.x; k < a.width; k += 256) ss += x[k] * x[k];
     const float rinv = 1.0f / sqrtf(block_sum(ss, red) / (float)a.width + a.eps);
-    float* o = (float*)p.xn + (int64_t)row * a.width;
+    float* o = (float*)p.xn + (int64_t)row * p.ldxn;
     for (int k = threadIdx.x; k < a.width; k += 256) o[k] = h[k] = x[k] * rinv * (a.norm_add + ld_as_f32(a.norm, k, a.norm_dtype));
     __syncthreads();
-    for (int e = wave; e < a.experts; e += 4) {
+    for (int e = wave; e < p.outputs; e += 4) {
         const float* w = (const float*)a.router + (int64_t)e * a.width;
         float s = 0.f;
         for (int k = lane; k < a.width; k += 64) s += w[k] * h[k];
@@ -243,7 +316,13 @@ __global__ __launch_bounds__(256) void exact_route_kernel(const Params p) {
         if (lane == 0) z[e] = s;
     }
     __syncthreads();
-    if (wave == 0) choose(z, a.experts, a.top, a.scale, p.ids + (int64_t)row * a.top, p.weights + (int64_t)row * a.top);
+    if (wave == 0) choose(a, z, z + p.outputs, p.outputs, p.ids + (int64_t)row * a.top, p.weights + (int64_t)row * a.top);
+}
+
+// column n of a row's sum
+__device__ __forceinline__ void put_sum(const mi355_experts_args& a, int row, int n, float v) {
+    if (a.out != nullptr) a.out[(int64_t)row * a.ld_out + n] = a.alpha * v;
+    else a.x[(int64_t)row * a.ldx + n] += a.alpha * v;
 }
 
 // ------------------------------------------------------------------------------------ f32 experts: a wave per output
@@ -255,8 +334,17 @@ __global__ __launch_bounds__(256) void exact_up_kernel(const Params p) {
     const int ff = shared ? a.ff_shared : a.ff;
     if (n >= ff) return;
     const int64_t slot = (int64_t)row * a.top + k;
-    const float* w = shared ? (const float*)a.shared_up : (const float*)a.up + (int64_t)p.ids[slot] * 2 * a.ff * a.width;
-    const float *wg = w + (int64_t)n * a.width, *wu = wg + (int64_t)ff * a.width, *h = (const float*)p.xn + (int64_t)row * a.width;
+    if (!shared && p.ids[slot] >= a.experts) return;  // (the row itself)
+    const float* w = shared ? (const float*)a.shared_up : (const float*)a.up + (int64_t)p.ids[slot] * (a.act == MI355_ACT_RELU2 ? 1 : 2) * a.ff * a.width;
+    if (a.act == MI355_ACT_RELU2) {
+        const float *wu = w + (int64_t)n * a.width, *h = (const float*)p.xn + (int64_t)row * p.ldxn;
+        float s = 0.f;
+        for (int j = lane; j < a.width; j += 64) s += wu[j] * h[j];
+        s = group_sum(s, 64);
+        if (lane == 0) ((float*)p.hid + slot * ff)[n] = relu2_f32(s);
+        return;
+    }
+    const float *wg = w + (int64_t)n * a.width, *wu = wg + (int64_t)ff * a.width, *h = (const float*)p.xn + (int64_t)row * p.ldxn;
     float sg = 0.f, su = 0.f;
     for (int j = lane; j < a.width; j += 64) sg += wg[j] * h[j], su += wu[j] * h[j];
     sg = group_sum(sg, 64), su = group_sum(su, 64);
@@ -273,61 +361,74 @@ __global__ __launch_bounds__(256) void exact_down_kernel(const Params p) {
         const bool shared = k == a.top;
         const int ff = shared ? a.ff_shared : a.ff;
         const int64_t slot = (int64_t)row * a.top + k;
+        if (!shared && p.ids[slot] >= a.experts) {
+            total += p.weights[slot] * ((const float*)p.xn)[(int64_t)row * p.ldxn + n];
+            continue;
+        }
         const float* w = (shared ? (const float*)a.shared_down : (const float*)a.down + (int64_t)p.ids[slot] * a.width * a.ff) + (int64_t)n * ff;
         const float* h = shared ? (const float*)p.hid_s + (int64_t)row * ff : (const float*)p.hid + slot * ff;
         float s = 0.f;
         for (int j = lane; j < ff; j += 64) s += w[j] * h[j];
         total += (shared ? 1.f : p.weights[slot]) * group_sum(s, 64);
     }
-    if (lane == 0) a.x[(int64_t)row * a.ldx + n] += a.alpha * total;
+    if (lane == 0) put_sum(a, row, n, total);
 }
 
 // ------------------------------------------------------------------------------------ few rows
 // grid (widest fp / 16, choices (+ 1), rows), 512 threads: 16 hidden columns of one choice; the waves share the units of K.  Every column of
-// the matrix instruction carries the same row
+// the matrix instruction carries the same row.  R: matrices of the stream (2: gate and up, 1: squared ReLU)
+template <int R>
 __global__ __launch_bounds__(512) void up_rows_kernel(const Params p) {
     const mi355_experts_args& a = p.a;
-    __shared__ float part[8][2][16];
+    __shared__ float part[8][R][16];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
     const int tile = blockIdx.x, k = blockIdx.y, row = blockIdx.z;
     const bool shared = k == a.top;
     const int fp = shared ? p.fsp : p.fp, ff = shared ? a.ff_shared : a.ff, units = p.kp / 128;
     if (tile * 16 >= fp) return;
     const int64_t slot = (int64_t)row * a.top + k;
-    const uint8_t* w = shared ? (const uint8_t*)a.shared_up : (const uint8_t*)a.up + p.ids[slot] * p.up_bytes;
-    w += (int64_t)tile * units * 8192 + lane * 16;
-    const bf16_t* x = p.xn + (int64_t)row * p.kp + 32 * g;
-    f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    const int id = shared ? 0 : p.ids[slot];
+    if (id >= a.experts) return;  // (the row itself)
+    const uint8_t* w = shared ? (const uint8_t*)a.shared_up : (const uint8_t*)a.up + id * p.up_bytes;
+    w += (int64_t)tile * units * R * 4096 + lane * 16;
+    const bf16_t* x = p.xn + (int64_t)row * p.ldxn + 32 * g;
+    f32x4 acc[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (tile * 16 < ff) {
 #pragma unroll 2
         for (int u = wave; u < units; u += 8) {
-            u32x4 q[2][4];
+            u32x4 q[R][4];
             bf16x8 b[4];
 #pragma unroll
-            for (int r = 0; r < 2; ++r)
+            for (int r = 0; r < R; ++r)
 #pragma unroll
-                for (int d = 0; d < 4; ++d) q[r][d] = *(const u32x4*)(w + (int64_t)u * 8192 + r * 4096 + d * 1024);
+                for (int d = 0; d < 4; ++d) q[r][d] = *(const u32x4*)(w + (int64_t)u * R * 4096 + r * 4096 + d * 1024);
 #pragma unroll
             for (int d = 0; d < 4; ++d) b[d] = *(const bf16x8*)(x + u * 128 + 8 * d);
 #pragma unroll
             for (int d = 0; d < 4; ++d)
 #pragma unroll
-                for (int r = 0; r < 2; ++r)
+                for (int r = 0; r < R; ++r)
                     acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, q[r][d]), b[d], acc[r], 0, 0, 0);
         }
     }
     if (c == 0) {
 #pragma unroll
-        for (int r = 0; r < 2; ++r)
+        for (int r = 0; r < R; ++r)
 #pragma unroll
             for (int i = 0; i < 4; ++i) part[wave][r][4 * g + i] = acc[r][i];
     }
     __syncthreads();
     if (threadIdx.x < 16) {
-        float s[2] = {0.f, 0.f};
+        float s[R];
 #pragma unroll
-        for (int w8 = 0; w8 < 8; ++w8) s[0] += part[w8][0][threadIdx.x], s[1] += part[w8][1][threadIdx.x];
-        (shared ? p.hid_s + (int64_t)row * fp : p.hid + slot * fp)[tile * 16 + threadIdx.x] = bf16_hw(silu_mul(s[0], s[1]));
+        for (int r = 0; r < R; ++r) {
+            s[r] = 0.f;
+#pragma unroll
+            for (int w8 = 0; w8 < 8; ++w8) s[r] += part[w8][r][threadIdx.x];
+        }
+        (shared ? p.hid_s + (int64_t)row * fp : p.hid + slot * fp)[tile * 16 + threadIdx.x] = bf16_hw(R == 2 ? silu_mul(s[0], s[R - 1]) : relu2_f32(s[0]));
     }
 }
 
@@ -337,13 +438,24 @@ __global__ __launch_bounds__(512) void down_rows_kernel(const Params p) {
     __shared__ float part[8][16];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
     const int tile = blockIdx.x, row = blockIdx.y;
-    const int units = p.fp / 128, units_s = p.fsp / 128, routed = a.top * units, items = routed + units_s;
+    __shared__ int real[kMaxTop], n_real;
     const int64_t slot0 = (int64_t)row * a.top;
+    if (a.identity > 0) {  // the choices that have weights
+        if (threadIdx.x < 64) {
+            const bool has = lane < a.top && p.ids[slot0 + min(lane, a.top - 1)] < a.experts;
+            const unsigned long long all = __ballot(has);
+            if (has) real[__popcll(all & ((1ull << lane) - 1))] = lane;
+            if (lane == 0) n_real = __popcll(all);
+        }
+        __syncthreads();
+    }
+    const int units = p.fp / 128, units_s = p.fsp / 128, routed = (a.identity > 0 ? n_real : a.top) * units, items = routed + units_s;
     f32x4 total = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 2
     for (int i = wave; i < items; i += 8) {
         const bool shared = i >= routed;
-        const int k = shared ? a.top : i / units, u = shared ? i - routed : i - k * units;
+        const int at = shared ? a.top : i / units, u = shared ? i - routed : i - at * units;
+        const int k = a.identity > 0 && !shared ? real[at] : at;
         const uint8_t* w = shared ? (const uint8_t*)a.shared_down + ((int64_t)tile * units_s + u) * 4096
                                   : (const uint8_t*)a.down + p.ids[slot0 + k] * p.down_bytes + ((int64_t)tile * units + u) * 4096;
         const bf16_t* h = (shared ? p.hid_s + (int64_t)row * p.fsp : p.hid + (slot0 + k) * p.fp) + u * 128 + 32 * g;
@@ -365,7 +477,9 @@ __global__ __launch_bounds__(512) void down_rows_kernel(const Params p) {
         float s = 0.f;
 #pragma unroll
         for (int w8 = 0; w8 < 8; ++w8) s += part[w8][threadIdx.x];
-        a.x[(int64_t)row * a.ldx + n] += a.alpha * s;
+        for (int k = 0; a.identity > 0 && k < a.top; ++k)
+            if (p.ids[slot0 + k] >= a.experts) s += p.weights[slot0 + k] * bf16_to_f32(p.xn[(int64_t)row * p.ldxn + n]);
+        put_sum(a, row, n, s);
     }
 }
 
@@ -377,7 +491,8 @@ __global__ __launch_bounds__(1024) void plan_kernel(const Params p, int bm) {
     const int tid = threadIdx.x, pairs = a.rows * a.top;
     count[tid] = 0;
     __syncthreads();
-    for (int i = tid; i < pairs; i += 1024) atomicAdd(&count[p.ids[i]], 1);
+    for (int i = tid; i < pairs; i += 1024)  // (experts that are the row itself have nothing to multiply)
+        if (p.ids[i] < a.experts) atomicAdd(&count[p.ids[i]], 1);
     __syncthreads();
     const int n = count[tid], t = (n + bm - 1) / bm;
     rows_to[tid] = n;
@@ -399,6 +514,10 @@ __global__ __launch_bounds__(1024) void plan_kernel(const Params p, int bm) {
     count[tid] = m0;
     __syncthreads();
     for (int i = tid; i < pairs; i += 1024) {
+        if (p.ids[i] >= a.experts) {
+            p.place[i] = -1;
+            continue;
+        }
         const int at = atomicAdd(&count[p.ids[i]], 1);
         p.perm[at] = i / a.top;
         p.place[i] = at;
@@ -422,11 +541,13 @@ struct Grouped {
     int64_t ldy, ldy_s;
 };
 
-// UP: pair stream, rows gathered by p.perm, SiLU(gate) up stored; else rows as sorted, plain sums stored.  A workgroup: BM rows x kWaves pairs
-// of row tiles (UP: one tile of both matrices).  Operands of the next unit: rows by LDS-DMA, weights into the registers the unit before left
-template <bool UP, int BM, int kWaves>
+// UP: rows gathered by p.perm, the activation stored (kUpPair: pair stream, SiLU(gate) up; kUpOne: squared ReLU); kDown: rows as sorted, plain sums
+// stored.  A workgroup: BM rows x kWaves pairs of row tiles (kUpPair: one tile of both matrices).  Operands of the next unit: rows by LDS-DMA, weights into the registers the unit before left
+enum { kDown = 0, kUpPair = 1, kUpOne = 2 };
+template <int UP, int BM, int kWaves>
 __global__ __launch_bounds__(64 * kWaves) void grouped_kernel(const Params p, const Grouped q) {
-    constexpr int kTT = BM / 16, kThreads = 64 * kWaves, kChunks = BM * 16 / kThreads, kPer = UP ? kWaves : kWaves * kTPW;
+    constexpr bool kPair = UP == kUpPair;
+    constexpr int kTT = BM / 16, kThreads = 64 * kWaves, kChunks = BM * 16 / kThreads, kPer = kPair ? kWaves : kWaves * kTPW;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
     const int n_e = *p.n_tiles, n_s = p.a.ff_shared > 0 ? (p.a.rows + BM - 1) / BM : 0;
@@ -459,10 +580,10 @@ __global__ __launch_bounds__(64 * kWaves) void grouped_kernel(const Params p, co
     const int64_t ldx = shared ? q.ldx_s : q.ldx;
     int tile[kTPW];
 #pragma unroll
-    for (int t = 0; t < kTPW; ++t) tile[t] = UP ? nb * kWaves + wave : nb * kPer + kTPW * wave + t;
+    for (int t = 0; t < kTPW; ++t) tile[t] = kPair ? nb * kWaves + wave : nb * kPer + kTPW * wave + t;
     auto wload = [&](int t, int u, int d, u32x4& dst) {
         const bool ok = tile[t] < real && u < units;
-        const unsigned off = (unsigned)((tile[t] * units + u) * (UP ? 2 : 1) + (UP ? t : 0)) * 4096u + d * 1024u;
+        const unsigned off = (unsigned)((tile[t] * units + u) * (kPair ? 2 : 1) + (kPair ? t : 0)) * 4096u + d * 1024u;
         dst = __builtin_bit_cast(u32x4, __builtin_amdgcn_raw_buffer_load_b128(ok ? rw : none, lane * 16, ok ? off : 0u, 0));
     };
     unsigned xoff[kChunks];
@@ -471,7 +592,7 @@ __global__ __launch_bounds__(64 * kWaves) void grouped_kernel(const Params p, co
         const int ch = i * kThreads + threadIdx.x, tok = ch >> 4, slot = ch & 15;
         xoff[i] = 0xFFFFFFF0u;
         if (tok < rows) {
-            const int row = UP && !shared ? p.perm[m0 + tok] : m0 + tok;
+            const int row = UP != kDown && !shared ? p.perm[m0 + tok] : m0 + tok;
             xoff[i] = (unsigned)((int64_t)row * ldx * 2) + (unsigned)((slot ^ swz(tok)) * 16);
         }
     }
@@ -524,7 +645,13 @@ __global__ __launch_bounds__(64 * kWaves) void grouped_kernel(const Params p, co
         const int tok = tt * 16 + c;
         if (tok >= rows) continue;
         bf16_t* dst = y + (int64_t)(m0 + tok) * ldy + 4 * g;
-        if constexpr (UP) {
+        if constexpr (UP == kUpOne) {
+#pragma unroll
+            for (int t = 0; t < kTPW; ++t)
+                if (tile[t] < tiles)
+                    *(u32x2*)(dst + tile[t] * 16) = u32x2{pack2(relu2_f32(acc[t][tt][0]), relu2_f32(acc[t][tt][1])),
+                                                          pack2(relu2_f32(acc[t][tt][2]), relu2_f32(acc[t][tt][3]))};
+        } else if constexpr (kPair) {
             if (tile[0] < tiles)
                 *(u32x2*)(dst + tile[0] * 16) = u32x2{pack2(silu_mul(acc[0][tt][0], acc[1][tt][0]), silu_mul(acc[0][tt][1], acc[1][tt][1])),
                                                       pack2(silu_mul(acc[0][tt][2], acc[1][tt][2]), silu_mul(acc[0][tt][3], acc[1][tt][3]))};
@@ -536,7 +663,7 @@ __global__ __launch_bounds__(64 * kWaves) void grouped_kernel(const Params p, co
     }
 }
 
-// grid rows: x[row] += alpha (sum of the chosen experts' rows by weight + the shared expert's)
+// grid rows: alpha (sum of the chosen experts' rows by weight + the shared expert's)
 __global__ __launch_bounds__(256) void combine_kernel(const Params p) {
     const mi355_experts_args& a = p.a;
     __shared__ float wgt[kMaxTop];
@@ -558,12 +685,12 @@ __global__ __launch_bounds__(256) void combine_kernel(const Params p) {
             for (int e = 0; e < 4; ++e) s[2 * e] += f * __uint_as_float(r[e] << 16), s[2 * e + 1] += f * __uint_as_float(r[e] & 0xffff0000u);
         };
 #pragma unroll 4
-        for (int k = 0; k < a.top; ++k) add(p.out + (int64_t)at[k] * p.np, wgt[k]);
+        for (int k = 0; k < a.top; ++k) add(at[k] >= 0 ? p.out + (int64_t)at[k] * p.np : p.xn + (int64_t)row * p.ldxn, wgt[k]);
         if (a.ff_shared > 0) add(p.out_s + (int64_t)row * p.np, 1.f);
-        f32x4* o = (f32x4*)(x + 8 * j);  // (columns width .. np are zeros plus zeros)
+        f32x4* o = (f32x4*)((a.out != nullptr ? a.out + (int64_t)row * a.ld_out : x) + 8 * j);  // (columns width .. np are zeros plus zeros)
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
-            f32x4 v = o[h];
+            f32x4 v = a.out != nullptr ? f32x4{0.f, 0.f, 0.f, 0.f} : o[h];
 #pragma unroll
             for (int e = 0; e < 4; ++e) v[e] += a.alpha * s[4 * h + e];
             o[h] = v;
@@ -584,7 +711,9 @@ size_t lay_out(Params& p, char* base) {
         return r;
     };
     const size_t rows = a.rows, pairs = rows * a.top;
-    p.xn = (bf16_t*)take(exact ? rows * a.width * 4 : rows * p.kp * 2);
+    p.outputs = a.experts + a.identity;
+    p.ldxn = a.h != nullptr ? a.ldh : exact ? a.width : p.kp;
+    p.xn = a.h != nullptr ? (bf16_t*)a.h : (bf16_t*)take(exact ? rows * a.width * 4 : rows * p.kp * 2);
     p.hid = (bf16_t*)take(exact ? pairs * a.ff * 4 : pairs * p.fp * 2);
     p.hid_s = (bf16_t*)take(exact ? rows * a.ff_shared * 4 : rows * p.fsp * 2);
     p.ids = (int32_t*)take(pairs * 4);
@@ -600,9 +729,9 @@ size_t lay_out(Params& p, char* base) {
     return at;
 }
 
-template <bool UP, int BM, int kWaves>
+template <int UP, int BM, int kWaves>
 int launch_grouped(const Params& p, const Grouped& q, hipStream_t s) {
-    constexpr int kPer = UP ? kWaves : kWaves * kTPW, kLds = 2 * BM * 256;
+    constexpr int kPer = UP == kUpPair ? kWaves : kWaves * kTPW, kLds = 2 * BM * 256;
     static hipError_t e = hipFuncSetAttribute((const void*)grouped_kernel<UP, BM, kWaves>, hipFuncAttributeMaxDynamicSharedMemorySize, kLds);
     MI355_CHECK_ARG(e == hipSuccess, (int)e, "experts: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
     const int64_t pairs = (int64_t)p.a.rows * p.a.top;
@@ -615,7 +744,7 @@ int launch_grouped(const Params& p, const Grouped& q, hipStream_t s) {
     return 0;
 }
 
-template <bool UP>
+template <int UP>
 int run_grouped(const Params& p, const Grouped& q, int bm, hipStream_t s) {
     if (bm == 128) return launch_grouped<UP, 128, 8>(p, q, s);
     if (bm == 64) return launch_grouped<UP, 64, 8>(p, q, s);
@@ -634,9 +763,9 @@ int run_many(Params& p, hipStream_t s) {
     q.units = q.units_s = p.kp / 128;
     q.real = (a.ff + 15) / 16, q.real_s = (a.ff_shared + 15) / 16, q.tiles = p.fp / 16, q.tiles_s = p.fsp / 16;
     q.bytes_s = (unsigned)((size_t)q.real_s * q.units * 8192);
-    q.x = q.x_s = p.xn, q.ldx = q.ldx_s = p.kp, q.xbytes = q.xbytes_s = (unsigned)((size_t)a.rows * p.kp * 2);
+    q.x = q.x_s = p.xn, q.ldx = q.ldx_s = p.ldxn, q.xbytes = q.xbytes_s = (unsigned)((size_t)a.rows * p.ldxn * 2);
     q.y = p.hid, q.ldy = p.fp, q.y_s = p.hid_s, q.ldy_s = p.fsp;
-    if (int rc = run_grouped<true>(p, q, bm, s)) return rc;
+    if (int rc = a.act == MI355_ACT_RELU2 ? run_grouped<kUpOne>(p, q, bm, s) : run_grouped<kUpPair>(p, q, bm, s)) return rc;
     q.w = (const uint8_t*)a.down, q.w_s = (const uint8_t*)a.shared_down, q.group_bytes = p.down_bytes;
     q.units = p.fp / 128, q.units_s = p.fsp / 128;
     q.real = q.tiles = p.np / 16;
@@ -645,7 +774,7 @@ int run_many(Params& p, hipStream_t s) {
     q.x = p.hid, q.ldx = p.fp, q.xbytes = (unsigned)((size_t)pairs * p.fp * 2);
     q.x_s = p.hid_s, q.ldx_s = p.fsp, q.xbytes_s = (unsigned)((size_t)a.rows * p.fsp * 2);
     q.y = p.out, q.y_s = p.out_s, q.ldy = q.ldy_s = p.np;
-    if (int rc = run_grouped<false>(p, q, bm, s)) return rc;
+    if (int rc = run_grouped<kDown>(p, q, bm, s)) return rc;
     hipLaunchKernelGGL(combine_kernel, dim3(a.rows), dim3(256), 0, s, p);
     MI355_LAUNCH_CHECK();
     return 0;
@@ -654,8 +783,9 @@ int run_many(Params& p, hipStream_t s) {
 template <int R>
 int launch_route(const Params& p, hipStream_t s) {
     const mi355_experts_args& a = p.a;
-    const int tiles = (a.experts + 15) / 16, pass = tiles < kRouteTiles ? tiles : kRouteTiles;
-    const size_t lds = ((size_t)8 * pass * 256 + R * (a.experts + 1)) * 4;
+    const int tiles = (p.outputs + 15) / 16, pass = tiles < kRouteTiles ? tiles : kRouteTiles;
+    const size_t lds = ((size_t)8 * pass * 256 + R * (p.outputs + 1 + choose_floats(a, p.outputs))) * 4;
+    MI355_CHECK_ARG(lds <= 144 * 1024, MI355_E_SHAPE, "experts: the choice of %d rows does not fit LDS", R);
     static hipError_t e = hipFuncSetAttribute((const void*)route_rows_kernel<R>, hipFuncAttributeMaxDynamicSharedMemorySize, 144 * 1024);
     MI355_CHECK_ARG(e == hipSuccess, (int)e, "experts: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
     hipLaunchKernelGGL(route_rows_kernel<R>, dim3((a.rows + R - 1) / R), dim3(512), lds, s, p);
@@ -663,9 +793,17 @@ int launch_route(const Params& p, hipStream_t s) {
     return 0;
 }
 
+int run_choose(const Params& p, hipStream_t s) {
+    const size_t lds = (size_t)4 * (p.outputs + choose_floats(p.a, p.outputs)) * 4;  // (at most 48 KB)
+    hipLaunchKernelGGL(choose_rows_kernel, dim3((p.a.rows + 3) / 4), dim3(256), lds, s, p);
+    MI355_LAUNCH_CHECK();
+    return 0;
+}
+
 // rows per workgroup: as few as give every CU one workgroup
 int run_route(const Params& p, hipStream_t s) {
     const int rows = p.a.rows;
+    if (p.a.logits != nullptr) return run_choose(p, s);
     if (rows <= 256) return launch_route<1>(p, s);
     if (rows <= 512) return launch_route<2>(p, s);
     if (rows <= 1024) return launch_route<4>(p, s);
@@ -676,7 +814,8 @@ int run_route(const Params& p, hipStream_t s) {
 int run_few(const Params& p, hipStream_t s) {
     const mi355_experts_args& a = p.a;
     const int shared = a.ff_shared > 0, widest = p.fp > p.fsp ? p.fp : p.fsp;
-    hipLaunchKernelGGL(up_rows_kernel, dim3(widest / 16, a.top + shared, a.rows), dim3(512), 0, s, p);
+    if (a.act == MI355_ACT_RELU2) hipLaunchKernelGGL(up_rows_kernel<1>, dim3(widest / 16, a.top + shared, a.rows), dim3(512), 0, s, p);
+    else hipLaunchKernelGGL(up_rows_kernel<2>, dim3(widest / 16, a.top + shared, a.rows), dim3(512), 0, s, p);
     MI355_LAUNCH_CHECK();
     hipLaunchKernelGGL(down_rows_kernel, dim3(p.np / 16, a.rows), dim3(512), 0, s, p);
     MI355_LAUNCH_CHECK();
@@ -686,12 +825,16 @@ int run_few(const Params& p, hipStream_t s) {
 int run_exact(const Params& p, hipStream_t s) {
     const mi355_experts_args& a = p.a;
     const int shared = a.ff_shared > 0, widest = a.ff > a.ff_shared ? a.ff : a.ff_shared;
-    const size_t lds = ((size_t)a.width + a.experts) * 4;
-    MI355_CHECK_ARG(lds <= 150 * 1024, MI355_E_SHAPE, "experts: rows of %d do not fit LDS", a.width);
-    static hipError_t e = hipFuncSetAttribute((const void*)exact_route_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024);
-    MI355_CHECK_ARG(e == hipSuccess, (int)e, "experts: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
-    hipLaunchKernelGGL(exact_route_kernel, dim3(a.rows), dim3(256), lds, s, p);
-    MI355_LAUNCH_CHECK();
+    if (a.logits != nullptr) {
+        if (int rc = run_choose(p, s)) return rc;
+    } else {
+        const size_t lds = ((size_t)a.width + p.outputs + choose_floats(a, p.outputs)) * 4;
+        MI355_CHECK_ARG(lds <= 150 * 1024, MI355_E_SHAPE, "experts: rows of %d do not fit LDS", a.width);
+        static hipError_t e = hipFuncSetAttribute((const void*)exact_route_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024);
+        MI355_CHECK_ARG(e == hipSuccess, (int)e, "experts: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
+        hipLaunchKernelGGL(exact_route_kernel, dim3(a.rows), dim3(256), lds, s, p);
+        MI355_LAUNCH_CHECK();
+    }
     hipLaunchKernelGGL(exact_up_kernel, dim3((widest + 3) / 4, a.top + shared, a.rows), dim3(256), 0, s, p);
     MI355_LAUNCH_CHECK();
     hipLaunchKernelGGL(exact_down_kernel, dim3((a.width + 3) / 4, a.rows), dim3(256), 0, s, p);
@@ -710,13 +853,26 @@ extern "C" size_t mi355_experts_scratch_bytes(const mi355_experts_args* a) {
 }
 
 extern "C" int mi355_experts(const mi355_experts_args* a, mi355_stream_t stream) {
-    MI355_CHECK_ARG(a && a->x && a->norm && a->router && a->up && a->down && a->scratch, MI355_E_ARG, "experts: null argument");
+    MI355_CHECK_ARG(a && a->up && a->down && a->scratch && (a->x || a->out), MI355_E_ARG, "experts: null argument");
+    MI355_CHECK_ARG(a->logits ? a->h != nullptr : a->router != nullptr, MI355_E_ARG, "experts: logits come with the rows they were made of, or from a router");
+    MI355_CHECK_ARG(a->h ? a->logits != nullptr : a->x != nullptr && a->norm != nullptr, MI355_E_ARG, "experts: rows come with their logits, or are normalised here");
     MI355_CHECK_ARG(a->dtype == MI355_F32 || a->dtype == MI355_BF16, MI355_E_DTYPE, "experts: dtype must be f32 or bf16");
-    MI355_CHECK_ARG(a->rows > 0 && a->rows <= 65535 && a->width > 0 && a->ff > 0 && a->ff_shared >= 0 && a->ldx >= pad_to(a->width, 16) && a->ldx % 4 == 0,
-                    MI355_E_SHAPE, "experts: bad shape (%d rows of %d, ff %d / %d)", a->rows, a->width, a->ff, a->ff_shared);
-    MI355_CHECK_ARG(a->ff_shared == 0 || (a->shared_up && a->shared_down), MI355_E_ARG, "experts: null shared expert");
-    MI355_CHECK_ARG(a->experts > 0 && a->experts <= kMaxExperts && a->top > 0 && a->top <= a->experts && a->top <= kMaxTop, MI355_E_SHAPE,
-                    "experts: %d of %d (at most %d of %d)", a->top, a->experts, kMaxTop, kMaxExperts);
+    MI355_CHECK_ARG(a->rows > 0 && a->rows <= 65535 && a->width > 0 && a->ff > 0 && a->ff_shared >= 0, MI355_E_SHAPE, "experts: bad shape (%d rows of %d, ff %d / %d)",
+                    a->rows, a->width, a->ff, a->ff_shared);
+    MI355_CHECK_ARG(a->x == nullptr || (a->ldx >= pad_to(a->width, 16) && a->ldx % 4 == 0), MI355_E_SHAPE, "experts: bad pitch of x");
+    MI355_CHECK_ARG(a->out == nullptr || (a->ld_out >= pad_to(a->width, 16) && a->ld_out % 4 == 0 && (uintptr_t)a->out % 16 == 0), MI355_E_SHAPE, "experts: bad rows of the sum");
+    MI355_CHECK_ARG(a->h == nullptr || (a->dtype == MI355_F32 ? a->ldh >= a->width : a->ldh >= pad_to(a->width, 128) && a->ldh % 8 == 0 && (uintptr_t)a->h % 16 == 0),
+                    MI355_E_SHAPE, "experts: bad normalised rows");
+    MI355_CHECK_ARG(a->ff_shared == 0 || (a->shared_up && a->shared_down && a->act == MI355_ACT_SILU_GATE), MI355_E_ARG, "experts: bad shared expert");
+    MI355_CHECK_ARG(a->experts > 0 && a->identity >= 0 && a->experts <= kMaxExperts && a->identity <= kMaxExperts - a->experts && a->top > 0 &&
+                        a->top <= a->experts + a->identity && a->top <= kMaxTop,
+                    MI355_E_SHAPE, "experts: %d of %d + %d (at most %d of %d)", a->top, a->experts, a->identity, kMaxTop, kMaxExperts);
+    MI355_CHECK_ARG((a->score == MI355_SCORE_SIGMOID && a->correction == nullptr && a->keep_groups == 0) || a->score == MI355_SCORE_SOFTMAX, MI355_E_ARG,
+                    "experts: corrections and groups belong to softmax scores");
+    MI355_CHECK_ARG(a->act == MI355_ACT_SILU_GATE || a->act == MI355_ACT_RELU2, MI355_E_ARG, "experts: bad activation %d", a->act);
+    MI355_CHECK_ARG(a->keep_groups == 0 || (a->keep_groups > 0 && a->groups >= a->keep_groups && (a->experts + a->identity) % a->groups == 0 &&
+                                            (int64_t)a->keep_groups * ((a->experts + a->identity) / a->groups) >= a->top),
+                    MI355_E_SHAPE, "experts: %d of %d groups of %d outputs", a->keep_groups, a->groups, a->experts + a->identity);
     MI355_CHECK_ARG((uintptr_t)a->x % 16 == 0 && (uintptr_t)a->norm % 8 == 0 && (uintptr_t)a->scratch % 256 == 0, MI355_E_ARG, "experts: unaligned operand");
     Params p;
     memset(&p, 0, sizeof(p));
@@ -725,11 +881,11 @@ extern "C" int mi355_experts(const mi355_experts_args* a, mi355_stream_t stream)
     MI355_CHECK_ARG(a->scratch_bytes >= need, MI355_E_SHAPE, "experts: scratch of %llu bytes, %zu needed", (unsigned long long)a->scratch_bytes, need);
     hipStream_t s = (hipStream_t)stream;
     if (a->dtype == MI355_F32) return run_exact(p, s);
-    p.up_bytes = (int64_t)((a->ff + 15) / 16) * (p.kp / 128) * 8192;
+    p.up_bytes = (int64_t)((a->ff + 15) / 16) * (p.kp / 128) * (a->act == MI355_ACT_RELU2 ? 4096 : 8192);
     p.down_bytes = (int64_t)(p.np / 16) * (p.fp / 128) * 4096;
     const int64_t pairs = (int64_t)a->rows * a->top;
     MI355_CHECK_ARG(p.up_bytes < 0xFFFFFFF0ll && p.down_bytes < 0xFFFFFFF0ll && pairs * p.fp * 2 < 0xFFFFFFF0ll && (int64_t)a->rows * p.fsp * 2 < 0xFFFFFFF0ll &&
-                        (int64_t)a->rows * p.kp * 2 < 0xFFFFFFF0ll && (int64_t)((a->ff_shared + 15) / 16) * p.kp * 64 < 0xFFFFFFF0ll &&
+                        (int64_t)a->rows * p.ldxn * 2 < 0xFFFFFFF0ll && (int64_t)((a->ff_shared + 15) / 16) * p.kp * 64 < 0xFFFFFFF0ll &&
                         (int64_t)p.np * p.fsp * 2 < 0xFFFFFFF0ll,
                     MI355_E_SHAPE, "experts: an operand exceeds 4 GiB");
     if (int rc = run_route(p, s)) return rc;

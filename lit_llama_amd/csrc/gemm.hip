@@ -118,6 +118,7 @@ struct GemmParams {
     int relu2;             // STORE: max(y, 0)^2
     float alpha;           // factor of the product where rinv is NULL (an operand that needed no staging)
     float limit;           // CLAMPGLU
+    const float* bias;     // STORE: [N], or NULL
     int slice_blocks;      // != 0: row blocks [i slice_blocks, (i + 1) slice_blocks) read the operand at xb + i slice_stride
     int64_t slice_stride;
     // grouped scales (GRP kernels): gtab[group 0..n_groups][r][tab_ld rows] = bf16 scale | bf16 zero << 16 (row n_groups
@@ -264,7 +265,7 @@ __global__ __launch_bounds__(256) void group_table_kernel(const bf16_t* s0, cons
 // y[m][n] (+)= sum over the K-slices, in slice order (deterministic)
 template <int EPI>
 __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, int ksplit, int M, int N, void* y, int y_dtype,
-                                                            int64_t ldy, int relu2, float limit) {
+                                                            int64_t ldy, int relu2, float limit, const float* bias) {
     const int64_t n4 = N >> 2;
     for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < (int64_t)M * n4; i += (int64_t)gridDim.x * blockDim.x) {
         const int m = (int)(i / n4), n = (int)(i - (int64_t)m * n4) * 4;
@@ -285,6 +286,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, i
             float* dst = (float*)y + (int64_t)m * ldy + n;
             if constexpr (EPI == MI355_EPI_ACCUM) o = *(const f32x4*)dst;
             for (int s = 0; s < ksplit; ++s) o += *(const f32x4*)(part + ((int64_t)s * M + m) * N + n);
+            if (EPI == MI355_EPI_STORE && bias != nullptr) o += *(const f32x4*)(bias + n);
             if (EPI == MI355_EPI_STORE && relu2) o = f32x4{relu2_f32(o[0]), relu2_f32(o[1]), relu2_f32(o[2]), relu2_f32(o[3])};
             *(f32x4*)dst = o;
         } else {
@@ -294,6 +296,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* part, i
                 for (int r = 0; r < 4; ++r) o[r] = bf16_to_f32(dst[r]);
             }
             for (int s = 0; s < ksplit; ++s) o += *(const f32x4*)(part + ((int64_t)s * M + m) * N + n);
+            if (EPI == MI355_EPI_STORE && bias != nullptr) o += *(const f32x4*)(bias + n);
             if (EPI == MI355_EPI_STORE && relu2) o = f32x4{relu2_f32(o[0]), relu2_f32(o[1]), relu2_f32(o[2]), relu2_f32(o[3])};
             u32x2 pk;
             pk[0] = (uint32_t)bf16_hw(o[0]) | ((uint32_t)bf16_hw(o[1]) << 16);
@@ -915,6 +918,13 @@ __global__ __launch_bounds__(64 * kWaves, (FMT == MI355_W_BF16 && kWaves == 8 &&
                         continue;
                     }
                 }
+                if constexpr (!FUSE && EPI == MI355_EPI_STORE && FMT == MI355_W_BF16) {
+                    if (p.bias != nullptr) {
+                        const f32x4 b = *(const f32x4*)(p.bias + n);
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) v[t][r] += b[r];
+                    }
+                }
                 if (p.y_dtype == MI355_F32) {
                     float* dst = (float*)p.y + (int64_t)m * p.ldy + n;
                     f32x4 o = {v[t][0], v[t][1], v[t][2], v[t][3]};
@@ -1030,7 +1040,8 @@ int launch_gemm_w(const GemmParams& p, hipStream_t s) {  // p.n_tiles: 16-row ti
     if (q.ksplit > 1) {
         const int64_t n = (int64_t)p.M * (p.N >> 2);
         const int grid = (int)((n + 255) / 256 < 2048 ? (n + 255) / 256 : 2048);
-        hipLaunchKernelGGL(splitk_reduce_kernel<EPI>, dim3(grid), dim3(256), 0, s, q.part, q.ksplit, p.M, p.N, p.y, p.y_dtype, p.ldy, p.relu2, p.limit);
+        hipLaunchKernelGGL(splitk_reduce_kernel<EPI>, dim3(grid), dim3(256), 0, s, q.part, q.ksplit, p.M, p.N, p.y, p.y_dtype, p.ldy, p.relu2, p.limit,
+                           p.bias);
         MI355_LAUNCH_CHECK();
     }
     return 0;
@@ -1188,7 +1199,9 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
         MI355_CHECK_ARG(a->sz_dtype == MI355_BF16, MI355_E_DTYPE, "linear_gemm: grouped scales / zeros must be bf16");
     }
     MI355_CHECK_ARG(a->M >= 1 && a->N > 0 && a->K > 0, MI355_E_SHAPE, "linear_gemm: bad shape M=%d N=%d K=%d", a->M, a->N, a->K);
-    MI355_CHECK_ARG(a->attn_partials == nullptr && a->bias == nullptr, MI355_E_ARG, "linear_gemm: no bias / attention prologue");
+    MI355_CHECK_ARG(a->attn_partials == nullptr, MI355_E_ARG, "linear_gemm: no attention prologue");
+    MI355_CHECK_ARG(a->bias == nullptr || (!q4 && f == nullptr && a->epi == MI355_EPI_STORE && a->sz_dtype == MI355_F32 && (uintptr_t)a->bias % 16 == 0), MI355_E_ARG,
+                    "linear_gemm: an f32 bias goes with the STORE epilogue of the BF16 stream");
     const bool swiglu = is_pair_epi(a->epi);
     MI355_CHECK_ARG(a->epi >= MI355_EPI_STORE && a->epi <= MI355_EPI_CLAMPGLU, MI355_E_ARG, "linear_gemm: bad epi");
     MI355_CHECK_ARG((a->epi != MI355_EPI_GEGLU && a->epi != MI355_EPI_CLAMPGLU) || (!q4 && f == nullptr), MI355_E_ARG, "linear_gemm: GEGLU and CLAMPGLU take the BF16 pair stream");
@@ -1303,6 +1316,7 @@ int mi355_linear_gemm_fused(const mi355_linear_args* a, const mi355_gemm_fuse* f
     p.rinv = direct ? nullptr : rinv;
     p.alpha = a->alpha == 0.f ? 1.f : a->alpha;
     p.limit = a->limit;
+    p.bias = (const float*)a->bias;
     MI355_CHECK_ARG(a->slice_rows == 0 || (direct && a->epi == MI355_EPI_STORE && a->slice_rows > 0 && a->slice_rows % 256 == 0 &&
                                            a->N % a->slice_rows == 0 && a->slice_stride % 8 == 0),
                     MI355_E_ARG, "linear_gemm: operand slices take whole row blocks of a bf16 operand and the STORE epilogue");

@@ -39,6 +39,7 @@ extern "C" int mi355_sizeof(int which) {
         case 14: return (int)sizeof(mi355_experts_args);
         case 15: return (int)sizeof(mi355_latent_args);
         case 16: return (int)sizeof(mi355_norm_args);
+        case 17: return (int)sizeof(mi355_join_args);
         default: return -1;
     }
 }

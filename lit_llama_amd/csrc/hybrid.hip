@@ -2,7 +2,7 @@
 // linears (gemv.hip for a few rows, gemm.hip above, the exact f32 kernel for f32 models), mixers (window_attention.hip, recurrent.hip) and
 // experts (experts.hip).  RMSNorm rides in the consuming linear and the residual sum in the producing one; the residual stream is f32.
 // A parallel layer normalises its row once (by groups, with the token shift of its mixer), and its mixer's output and hidden row leave
-// through one product.
+// through one product.  A sandwich layer's sublayers read rows that the pass behind the sublayer in front (join.hip) has normalised.
 #include "product.h"
 
 namespace {
@@ -84,27 +84,6 @@ struct NormParams : mi355_norm_args {
     int size;               // of a group
     mi355_seq_batch b;
 };
-
-template <typename T>
-__device__ __forceinline__ void put4(T* p, f32x4 v) {
-    if constexpr (sizeof(T) == 4) {
-        *(f32x4*)p = v;
-    } else {
-        typedef __attribute__((ext_vector_type(2))) __bf16 bf2;
-        const bf2 a = {(__bf16)v[0], (__bf16)v[1]}, b = {(__bf16)v[2], (__bf16)v[3]};
-        *(u32x2*)p = u32x2{__builtin_bit_cast(uint32_t, a), __builtin_bit_cast(uint32_t, b)};
-    }
-}
-
-template <typename T>
-__device__ __forceinline__ f32x4 get4(const T* p) {
-    if constexpr (sizeof(T) == 4) {
-        return *(const f32x4*)p;
-    } else {
-        const u32x2 r = *(const u32x2*)p;
-        return f32x4{__uint_as_float(r[0] << 16), __uint_as_float(r[0] & 0xffff0000u), __uint_as_float(r[1] << 16), __uint_as_float(r[1] & 0xffff0000u)};
-    }
-}
 
 // One row per workgroup.  H > 0: rows of up to 2048 H values whose groups are whole runs of 256 (a wave's load), held in registers; H = 0: any
 // width, and with MIX a second row: the row before, or, in the workgroup of a portion's first row, the portion's last one (it enters the
@@ -532,6 +511,55 @@ int parallel_in(const mi355_hybrid_model* m, const mi355_hybrid_layer& l, int M,
     return 0;
 }
 
+// the pass between two sublayers: the result `t` behind its gate and norm joins the stream; `next`: the norm of what reads it
+mi355_join_args join_of(const mi355_hybrid_model* m, int M, const void* next) {
+    mi355_join_args a;
+    memset(&a, 0, sizeof(a));
+    a.dtype = m->dtype, a.rows = M, a.width = m->width, a.eps = m->eps, a.norm_add = m->norm_add;
+    a.t = m->tmp, a.ldt = m->ldx;
+    a.x = m->x, a.ldx = m->ldx;
+    a.next = next, a.h = m->dtype == MI355_F32 ? (void*)m->xn : (void*)m->xb, a.ldh = m->ld_n;
+    return a;
+}
+
+// the average behind layer run r, and the norm in front of run r + 1 (none behind the last: the head has its own)
+void average_of(const mi355_hybrid_model* m, int r, mi355_join_args& a) {
+    const int64_t stride = (int64_t)m->max_rows * m->ldx;
+    a.stream = m->stream, a.stream_stride = stride, a.stream_out = m->stream + (r + 1) * stride;
+    a.n_stream = r + 1, a.average = m->layers[r].average;
+    a.next = r + 1 < m->n_runs ? m->layers[r + 1].norm1 : nullptr;
+}
+
+// the sublayers of a sandwich layer behind its mixer: gate columns at `gate` of rows of pitch ldp
+int sandwich_out(const mi355_hybrid_model* m, int r, const void* gate, int64_t ldp, int M, hipStream_t s) {
+    const mi355_hybrid_layer& l = m->layers[r];
+    if (l.out_norm != nullptr) {  // state-space outputs in groups
+        mi355_norm_args n;
+        memset(&n, 0, sizeof(n));
+        n.dtype = m->dtype, n.rows = M, n.width = l.out.K, n.groups = l.out_groups;
+        n.x = m->mixed, n.ldx = m->ld_mixed, n.eps = m->eps, n.scale = l.out_norm, n.h = l.cat, n.ldh = l.ld_cat;
+        if (int rc = mi355_norm_groups(&n, nullptr, (mi355_stream_t)s)) return rc;
+    }
+    if (int rc = mi355_product_run(product_of(m, l.cat, l.ld_cat, M, MI355_EPI_STORE, m->tmp, m->ldx, MI355_F32), l.out, s)) return rc;
+    mi355_join_args a = join_of(m, M, l.norm2);
+    a.gate = (const char*)gate + (int64_t)l.gate_at * dtype_size(m->dtype), a.ld_gate = ldp, a.gate_dtype = m->dtype, a.post = l.post1;
+    if (l.mlp == MI355_MLP_NONE) average_of(m, r, a);
+    if (int rc = mi355_join_rows(&a, (mi355_stream_t)s)) return rc;
+    if (l.mlp == MI355_MLP_NONE) return 0;
+    const void* h = a.h;
+    if (int rc = mi355_product_run(product_of(m, h, m->ld_n, M, MI355_EPI_STORE, m->side, m->ld_side, MI355_F32), l.side, s)) return rc;
+    mi355_experts_args e = l.moe;
+    e.dtype = m->dtype, e.rows = M, e.eps = m->eps, e.alpha = 1.f;
+    e.h = h, e.ldh = m->ld_n, e.logits = m->side + l.logits_at, e.ld_logits = m->ld_side;
+    e.out = m->tmp, e.ld_out = m->ldx;
+    e.scratch = m->moe_scratch, e.scratch_bytes = m->moe_scratch_bytes;
+    if (int rc = mi355_experts(&e, (mi355_stream_t)s)) return rc;
+    a = join_of(m, M, nullptr);
+    a.gate = m->side, a.ld_gate = m->ld_side, a.gate_dtype = MI355_F32, a.post = l.post2;
+    average_of(m, r, a);
+    return mi355_join_rows(&a, (mi355_stream_t)s);
+}
+
 // hidden row into `cat`, then x += out [mixer | hidden]
 int parallel_out(const mi355_hybrid_model* m, const mi355_hybrid_layer& l, int M, hipStream_t s) {
     const bool f32 = m->dtype == MI355_F32;
@@ -598,10 +626,13 @@ bool mi355_product_wide(const mi355_proj& w, int M, int R) {
 int mi355_product_run(const mi355_product& p, const mi355_proj& w, hipStream_t s) {
     if (p.dtype == MI355_F32) {
         MI355_CHECK_ARG(p.epi == MI355_EPI_STORE && p.alpha == 1.f && p.y_dtype == MI355_F32, MI355_E_ARG, "product: f32 operands are stored as they are");
-        return mi355_linear_dense(p.x, p.ldx, w.w, nullptr, p.y, p.ldy, p.M, w.N, w.K, MI355_F32, s);
+        return mi355_linear_dense(p.x, p.ldx, w.w, w.bias, p.y, p.ldy, p.M, w.N, w.K, MI355_F32, s);
     }
+    MI355_CHECK_ARG(w.bias == nullptr || p.epi == MI355_EPI_STORE, MI355_E_ARG, "product: a bias belongs to what is stored");
     mi355_linear_args a;
     memset(&a, 0, sizeof(a));
+    a.bias = w.bias;
+    a.sz_dtype = MI355_F32;
     a.fmt = MI355_W_BF16;
     a.R = is_pair_epi(p.epi) ? 2 : 1;
     a.w = w.w;
@@ -642,24 +673,40 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
         MI355_CHECK_ARG(!l.parallel || (m->norm_groups > 0 && l.cat && l.ld_cat >= l.out.K && (l.mlp == MI355_MLP_NONE || l.mlp == MI355_MLP_CLAMPGLU) &&
                                         l.n_mix <= 5 && (l.n_mix == 0 || (l.mu && l.shift && m->mix))),
                         MI355_E_ARG, "hybrid_forward: bad parallel layer (run %d)", r);
+        MI355_CHECK_ARG(!l.sandwich || (!l.parallel && m->norm_groups == 0 && m->embed_norm && m->stream && m->tmp && l.cat && l.ld_cat >= l.out.K && l.post1 && l.average &&
+                                        (l.mlp == MI355_MLP_NONE || (l.mlp == MI355_MLP_EXPERTS && l.norm2 && l.post2 && m->side && m->ld_side >= l.side.N)) &&
+                                        (l.mixer == MI355_MIX_ATTENTION || (l.mixer == MI355_MIX_SSD && m->mixed && m->ld_mixed >= l.out.K && l.out_norm)) &&
+                                        m->residual_mult == 1.f && l.sandwich == m->layers[0].sandwich),
+                        MI355_E_ARG, "hybrid_forward: bad sandwich layer (run %d)", r);
+        MI355_CHECK_ARG(l.sandwich || l.mixer != MI355_MIX_SSD, MI355_E_ARG, "hybrid_forward: a state-space mixer belongs to a sandwich layer (run %d)", r);
         MI355_CHECK_ARG(l.parallel || l.mlp != MI355_MLP_CLAMPGLU, MI355_E_ARG, "hybrid_forward: a clamped gated feed-forward belongs to a parallel layer (run %d)", r);
     }
     hipStream_t s = (hipStream_t)stream;
-    hipLaunchKernelGGL(embed_rows_kernel, dim3(M), dim3(256), 0, s, tokens, m->embed, m->dtype, m->x, m->width, m->ldx, m->vocab);
-    MI355_LAUNCH_CHECK();
+    if (m->embed_norm != nullptr && m->n_runs > 0) {
+        mi355_join_args a = join_of(m, M, m->layers[0].norm1);
+        a.tokens = tokens, a.embed = m->embed, a.vocab = m->vocab, a.post = m->embed_norm, a.stream_out = m->stream;
+        if (int rc = mi355_join_rows(&a, stream)) return rc;
+    } else {
+        hipLaunchKernelGGL(embed_rows_kernel, dim3(M), dim3(256), 0, s, tokens, m->embed, m->dtype, m->x, m->width, m->ldx, m->vocab);
+        MI355_LAUNCH_CHECK();
+    }
     const int runs = run_end < m->n_runs ? run_end : m->n_runs;
     for (int r = 0; r < runs; ++r) {
         const mi355_hybrid_layer& l = m->layers[r];
         const int64_t ldp = l.in.N;
-        void* const y = l.parallel ? l.cat : m->att;
-        const int64_t ldy = l.parallel ? l.ld_cat : m->ld_att;
-        if (l.parallel) {
+        void* const y = l.mixer == MI355_MIX_SSD ? m->mixed : l.cat != nullptr ? l.cat : m->att;
+        const int64_t ldy = l.mixer == MI355_MIX_SSD ? m->ld_mixed : l.cat != nullptr ? l.ld_cat : m->ld_att;
+        void* const proj = l.proj_rows != nullptr ? l.proj_rows : m->proj;
+        if (l.sandwich) {
+            const mi355_product in = product_of(m, m->dtype == MI355_F32 ? (void*)m->xn : (void*)m->xb, m->ld_n, M, MI355_EPI_STORE, proj, ldp, m->dtype);
+            if (int rc = mi355_product_run(in, l.in, s)) return rc;
+        } else if (l.parallel) {
             if (int rc = norm_groups(m, l.norm1, &l, b, nullptr, M, s)) return rc;
             if (int rc = parallel_in(m, l, M, s)) return rc;
         } else if (int rc = linear(m, l.in, m->x, m->ldx, l.norm1, kStore, m->proj, ldp, m->dtype, M, s)) return rc;
         if (l.mixer == MI355_MIX_ATTENTION) {
             mi355_window_attn_args a = l.attn;
-            a.proj = m->proj;
+            a.proj = proj;
             a.ld = ldp;
             a.dtype = m->dtype;
             a.y = y;
@@ -689,7 +736,7 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
             if (int rc = mi355_latent_attention(&a, b, stream)) return rc;
         } else {
             mi355_recurrent_args a = l.rec;
-            a.proj = m->proj;
+            a.proj = proj;
             a.ld = ldp;
             a.dtype = m->dtype;
             a.y = y;
@@ -697,6 +744,10 @@ extern "C" int mi355_hybrid_forward(const mi355_hybrid_model* m, const mi355_seq
             a.scratch = m->rec_scratch;
             a.scratch_bytes = m->rec_scratch_bytes;
             if (int rc = mi355_recurrent(&a, b, stream)) return rc;
+        }
+        if (l.sandwich) {
+            if (int rc = sandwich_out(m, r, proj, ldp, M, s)) return rc;
+            continue;
         }
         if (l.parallel) {
             if (int rc = parallel_out(m, l, M, s)) return rc;

@@ -1,5 +1,7 @@
 // Shared by the row-by-row and the chunked kernels of the linear recurrences (not part of the C ABI).
 #pragma once
+#include <type_traits>
+
 #include "common.h"
 
 constexpr int kMaxRank = 256;  // of the low-rank decay projection
@@ -45,8 +47,8 @@ __device__ __forceinline__ const T* conv_input(const mi355_recurrent_args& a, co
 // portion that starts at position pos0
 template <typename T>
 __device__ __forceinline__ float conv_at(const mi355_recurrent_args& a, const T* rows, const T* ring, int ring_ld, int off, int cr,
-                                         const float* w, int i, int pos0) {
-    float v = 0.f;
+                                         const float* w, int i, int pos0, float bias = 0.f) {
+    float v = bias;
     for (int j0 = 0; j0 < a.taps; j0 += 4) {
         T x[4];
         float wj[4];
@@ -67,10 +69,10 @@ __device__ __forceinline__ float conv_at(const mi355_recurrent_args& a, const T*
 // the same for 16 rows i .. i + 15 of one channel (rows past n give 0)
 template <typename T>
 __device__ __forceinline__ void conv_rows16(const mi355_recurrent_args& a, const T* rows, const T* ring, int ring_ld, int off, int cr,
-                                            const float* w, int i, int n, int pos0, float (&out)[16]) {
+                                            const float* w, int i, int n, int pos0, float (&out)[16], float bias = 0.f) {
     if (a.taps > kTaps) {
 #pragma unroll
-        for (int t = 0; t < 16; ++t) out[t] = i + t < n ? conv_at<T>(a, rows, ring, ring_ld, off, cr, w, i + t, pos0) : 0.f;
+        for (int t = 0; t < 16; ++t) out[t] = i + t < n ? conv_at<T>(a, rows, ring, ring_ld, off, cr, w, i + t, pos0, bias) : 0.f;
         return;
     }
     T raw[16 + kTaps - 1];
@@ -90,7 +92,7 @@ __device__ __forceinline__ void conv_rows16(const mi355_recurrent_args& a, const
     for (int j = 0; j < kTaps; ++j) wj[j] = j < a.taps ? wj[j] : 0.f;
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
-        float v = 0.f;
+        float v = bias;
 #pragma unroll
         for (int j = 0; j < kTaps; ++j) v += wj[j] * x[kTaps - 1 + t - j];
         out[t] = i + t < n ? silu_f32(v) : 0.f;
@@ -99,6 +101,14 @@ __device__ __forceinline__ void conv_rows16(const mi355_recurrent_args& a, const
 
 // log of a WKV key channel's decay, exp(-exp(z)): below -104 the decay is 0 in f32, and sums of many stay finite
 __device__ __forceinline__ float wkv_log_decay(float z) { return fmaxf(-expf(z), -104.f); }
+
+// kinds with short convolutions on q, k and v
+__host__ __device__ constexpr bool has_conv(int kind) { return kind == MI355_REC_DELTA || kind == MI355_REC_SSD; }
+// bias of convolution channel c
+__device__ __forceinline__ float conv_bias(const float* b, int c) { return b != nullptr ? b[c] : 0.f; }
+// how a kind stores its outputs
+template <int KIND, typename T>
+using out_t = std::conditional_t<KIND == MI355_REC_SSD, float, T>;
 
 struct RecParams {
     mi355_recurrent_args a;

@@ -1,5 +1,6 @@
-// Linear recurrences with a matrix state per head: the gated delta rule (with its short convolutions), gated linear attention, and WKV time
-// mixing (the state in front of a token, and the token itself with a bonus per key channel).
+// Linear recurrences with a matrix state per head: the gated delta rule (with its short convolutions), gated linear attention, WKV time
+// mixing (the state in front of a token, and the token itself with a bonus per key channel), and state-space duality (short convolutions, one
+// decay and one step size per head, keys and queries shared by a group of heads).
 //
 //   rec_rows_kernel       one workgroup per (head, sequence) walks its rows one by one with the state in registers: decode steps
 //                         (convolution, gates, state update, output norm and gate in ONE launch) and short portions
@@ -53,7 +54,8 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
         // ---- the row's q, k (and decays) into LDS
         // (what needs no LDS is requested here, in front of the barriers: one memory latency instead of one per use)
         const bool out_ok = part == 0 && col_ok;
-        const float gate = out_ok ? silu_f32(to_f32<T>(row[a.off_g + head * vdim + col])) * a.head_norm[head * a.norm_ld + col] : 0.f;
+        float gate = out_ok ? silu_f32(to_f32<T>(row[a.off_g + head * vdim + col])) : 0.f;
+        if constexpr (KIND != MI355_REC_SSD) gate *= out_ok ? a.head_norm[head * a.norm_ld + col] : 0.f;
         float g = 1.f, beta = 1.f, v = 0.f;
         if constexpr (KIND == MI355_REC_DELTA) {
             const float dt = softplus_f32(to_f32<T>(row[a.off_a + head]) + a.dt_bias[head]);
@@ -79,6 +81,21 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
             for (int d = tid; d < dim; d += nt) {
                 q[d] *= iq;
                 k[d] *= ik;
+            }
+        } else if constexpr (KIND == MI355_REC_SSD) {
+            const float dt = softplus_f32(to_f32<T>(row[a.off_a + head]) + a.dt_bias[head]);
+            g = expf(-expf(a.a_log[head]) * dt);
+            if (col_ok) {
+                const int c = head * vdim + col;
+                v = conv_at<T>(a, rows, ring, ring_ld, a.off_v + c, 2 * a.kv_heads * dim + c, a.conv_v + (int64_t)c * a.taps, t, pos0, conv_bias(a.conv_bv, c));
+            }
+            for (int i = tid; i < 2 * dim; i += nt) {
+                const bool key = i >= dim;
+                const int d = key ? i - dim : i, c = kvh * dim + d;
+                const float y = conv_at<T>(a, rows, ring, ring_ld, (key ? a.off_k : a.off_q) + c, (key ? a.kv_heads * dim : 0) + c,
+                                           (key ? a.conv_k : a.conv_q) + (int64_t)c * a.taps, t, pos0, conv_bias(key ? a.conv_bk : a.conv_bq, c));
+                if (key) k[d] = y * dt;
+                else q[d] = y;
             }
         } else {
             if (col_ok) v = to_f32<T>(row[a.off_v + head * vdim + col]);
@@ -121,6 +138,12 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
                 S[r] += kp[r] * u;
                 o += S[r] * qp[r];
             }
+        } else if constexpr (KIND == MI355_REC_SSD) {
+#pragma unroll
+            for (int r = 0; r < RMAX; ++r) {
+                S[r] = g * S[r] + kp[r] * v;
+                o += S[r] * qp[r];
+            }
         } else if constexpr (KIND == MI355_REC_WKV) {
             const float* ap = al + part * RMAX;
             const float* up = uk + part * RMAX;
@@ -142,10 +165,14 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
         // ---- output norm over vdim, gate (part 0 holds the columns)
         o = 0.f;
         for (int j = 0; j < p.parts; ++j) o += pb[j * cols + col];
-        const float ss = block_sum(out_ok ? o * o : 0.f, red);
-        if (out_ok) {
-            const float rinv = 1.0f / sqrtf(ss / (float)vdim + a.eps);
-            ((T*)a.y)[(int64_t)(p.b.row0[seq] + t) * a.ldy + head * vdim + col] = from_f32<T>(o * rinv * gate);
+        if constexpr (KIND == MI355_REC_SSD) {
+            if (out_ok) ((float*)a.y)[(int64_t)(p.b.row0[seq] + t) * a.ldy + head * vdim + col] = (o + a.skip[head] * v) * gate;
+        } else {
+            const float ss = block_sum(out_ok ? o * o : 0.f, red);
+            if (out_ok) {
+                const float rinv = 1.0f / sqrtf(ss / (float)vdim + a.eps);
+                ((T*)a.y)[(int64_t)(p.b.row0[seq] + t) * a.ldy + head * vdim + col] = from_f32<T>(o * rinv * gate);
+            }
         }
         __syncthreads();
     }
@@ -155,7 +182,7 @@ __global__ __launch_bounds__(1024) void rec_rows_kernel(const RecParams p) {
         if (col_ok && i < dim) state[(int64_t)i * vdim + col] = S[r];
     }
     // ---- a decode step's own inputs enter the ring here (row pos0 % taps held position pos0 - taps: nobody reads it any more)
-    if constexpr (KIND == MI355_REC_DELTA) {
+    if constexpr (has_conv(KIND)) {
         if (p.b.max_count == 1) {
             T* dst = ring + (int64_t)(pos0 % a.taps) * ring_ld;
             if (head % (a.heads / a.kv_heads) == 0)
@@ -220,10 +247,11 @@ int run(const RecParams& p, hipStream_t s) {
         if (int rc = mi355_recurrent_chunks(p, s)) return rc;
     } else if (int rc = p.a.kind == MI355_REC_DELTA ? run_rows<T, MI355_REC_DELTA>(p, s)
                         : p.a.kind == MI355_REC_WKV ? run_rows<T, MI355_REC_WKV>(p, s)
+                        : p.a.kind == MI355_REC_SSD ? run_rows<T, MI355_REC_SSD>(p, s)
                                                     : run_rows<T, MI355_REC_GLA>(p, s)) {
         return rc;
     }
-    if (p.a.kind == MI355_REC_DELTA && (chunks || p.b.max_count > 1)) {
+    if (has_conv(p.a.kind) && (chunks || p.b.max_count > 1)) {
         hipLaunchKernelGGL(conv_ring_kernel<T>, dim3(p.a.taps < p.b.max_count ? p.a.taps : p.b.max_count, p.b.seqs, 16), dim3(256), 0, s, p);
         MI355_LAUNCH_CHECK();
     }
@@ -233,25 +261,26 @@ int run(const RecParams& p, hipStream_t s) {
 }  // namespace
 
 extern "C" int mi355_recurrent(const mi355_recurrent_args* a, const mi355_seq_batch* b, mi355_stream_t stream) {
-    MI355_CHECK_ARG(a && b && a->proj && a->state && a->y && a->head_norm, MI355_E_ARG, "recurrent: null argument");
+    MI355_CHECK_ARG(a && b && a->proj && a->state && a->y && (a->head_norm || a->kind == MI355_REC_SSD), MI355_E_ARG, "recurrent: null argument");
     MI355_CHECK_ARG(b->row0 && b->count && b->slot && b->pos, MI355_E_ARG, "recurrent: null batch");
     MI355_CHECK_ARG(b->rows > 0 && b->seqs > 0 && b->seqs <= 65535 && b->seqs <= b->rows && b->max_count > 0, MI355_E_SHAPE,
                     "recurrent: bad batch (%d rows, %d sequences)", b->rows, b->seqs);
-    MI355_CHECK_ARG(a->kind >= MI355_REC_DELTA && a->kind <= MI355_REC_WKV, MI355_E_ARG, "recurrent: bad kind %d", a->kind);
+    MI355_CHECK_ARG(a->kind >= MI355_REC_DELTA && a->kind <= MI355_REC_SSD, MI355_E_ARG, "recurrent: bad kind %d", a->kind);
     MI355_CHECK_ARG(a->dtype == MI355_F32 || a->dtype == MI355_BF16, MI355_E_DTYPE, "recurrent: dtype must be f32 or bf16");
     MI355_CHECK_ARG(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim > 0 && a->vdim > 0, MI355_E_SHAPE,
                     "recurrent: bad heads %d / %d or sizes %d / %d", a->heads, a->kv_heads, a->dim, a->vdim);
-    if (a->kind == MI355_REC_DELTA)
+    if (has_conv(a->kind))
         MI355_CHECK_ARG(a->taps > 0 && a->conv_q && a->conv_k && a->conv_v && a->conv_ring && a->a_log && a->dt_bias, MI355_E_ARG,
-                        "recurrent: the delta rule needs its convolutions and decays");
+                        "recurrent: the delta rule and state-space duality need their convolutions and decays");
     else
         MI355_CHECK_ARG(a->rank > 0 && a->rank <= kMaxRank && a->a2 && a->a2_bias && a->kv_heads == a->heads, MI355_E_ARG,
                         "recurrent: gated linear attention needs its decay projection (rank 1..%d)", kMaxRank);
     MI355_CHECK_ARG(a->kind != MI355_REC_WKV || a->bonus, MI355_E_ARG, "recurrent: WKV needs its bonus");
+    MI355_CHECK_ARG(a->kind != MI355_REC_SSD || a->skip, MI355_E_ARG, "recurrent: state-space duality needs its skip factors");
     RecParams p;
     p.a = *a;
     p.b = *b;
-    if (a->kind != MI355_REC_DELTA) p.a.taps = 1;
+    if (!has_conv(a->kind)) p.a.taps = 1;
     p.parts = p.slices = 1;
     return a->dtype == MI355_F32 ? run<float>(p, (hipStream_t)stream) : run<bf16_t>(p, (hipStream_t)stream);
 }

@@ -7,11 +7,14 @@
 //          O = diag(e^G) Q S_0 + P U,                      P_ij = e^(G_i - G_j) q_i . k_j         (j <= i)
 //          S = e^(G_end) S_0 + K^T diag(e^(G_end - G)) U
 //   gla    U = V,  e^(G_i - G_j) acts per key channel inside the products,  O = (Q e^G) S_0 + P V,  S = diag(e^(G_end)) S_0 + (K e^(G_end - G))^T V
+//   ssd    as delta with U = V and A = 0 (no unit norms):  P_ij = e^(G_i - G_j) dt_j q_i . k_j (+ skip on the diagonal),
+//          S = e^(G_end) S_0 + K^T diag(e^(G_end - G) dt) V
 //   wkv    as gla, but row i reads the state in front of it: e^(G_(i-1) - G_j) and Q e^(G_(i-1)), and P_ii = sum q_i u k_i
 //
 // Every exponent is <= 0.  Launches of a step (each over all chunks at once but the scan):
-//   delta_qk_kernel    convolutions, unit norms; Q, K^T, K K^T, Q K^T per key head
+//   delta_qk_kernel    delta, ssd: convolutions, unit norms (delta); Q, K^T, K K^T (delta), Q K^T per key head
 //   delta_head_kernel  decays, T = (I + A)^-1 by 16 x 16 blocks, U0 = T diag(beta) V, W = T diag(beta e^G) K, P per head
+//   ssd_head_kernel    decays, V^T with its convolution, P per head
 //   gla_prep_kernel    gla, wkv: decays, Q e^G, (K e^(G_end - G))^T, P (off-diagonal 16 x 16 blocks anchored at the row block's first row), V^T
 //   scan_kernel        one workgroup per (sequence, head, 16 columns): U = U0 - W S_0, S; the state in accumulator registers
 //   chunk_out_kernel   O, output norm, gate
@@ -40,17 +43,17 @@ __device__ __forceinline__ void lds_barrier() {
 
 // ---------------------------------------------------------------- scratch, per packed chunk (padded sizes DP, VP: multiples of 16)
 struct Scratch {
-    float* q;     // [NC][GQ][64][DP]        delta: unit q * q_scale; gla: q e^G * q_scale
-    float* kt;    // [NC][GQ][DP][64]        delta: unit k; gla: k e^(G_end - G)
+    float* q;     // [NC][GQ][64][DP]        delta: unit q * q_scale; ssd: q; gla: q e^G * q_scale
+    float* kt;    // [NC][GQ][DP][64]        delta: unit k; ssd: k; gla: k e^(G_end - G)
     float* kk;    // [NC][G][64][64]         delta: k_i . k_j
-    float* qk;    // [NC][G][64][64]         delta: q_i . k_j
+    float* qk;    // [NC][G][64][64]         delta, ssd: q_i . k_j
     float* P;     // [NC][H][64][64]
     float* W;     // [NC][H][64][DP]         delta
     float* ut;    // [NC][H][VP][64]         U^T (delta: U0^T until the scan)
     float* st;    // [NC][H][VP][DP]         S_0^T
-    float* gam;   // [NC][H][DP]             e^(G_end) (delta: element 0)
-    float* eg;    // [NC][H][64]             delta: e^G
-    float* ed;    // [NC][H][64]             delta: e^(G_end - G)
+    float* gam;   // [NC][H][DP]             e^(G_end) (delta, ssd: element 0)
+    float* eg;    // [NC][H][64]             delta, ssd: e^G
+    float* ed;    // [NC][H][64]             delta: e^(G_end - G); ssd: e^(G_end - G) dt
 };
 
 struct ChunkParams {
@@ -72,9 +75,9 @@ __device__ __forceinline__ bool head_chunk(const ChunkParams& p, int& head, int&
     return head < p.r.a.heads;
 }
 
-// ------------------------------------------------------------------------------------ delta: q, k per key head
+// ------------------------------------------------------------------------------------ delta, ssd: q, k per key head
 // grid (chunks, kv_heads, seqs), 256 threads.  LDS: k, q [64][DP + 4]
-template <typename T>
+template <typename T, int KIND>
 __global__ __launch_bounds__(256) void delta_qk_kernel(const ChunkParams p) {
     const mi355_recurrent_args& a = p.r.a;
     extern __shared__ __attribute__((aligned(16))) float sm[];
@@ -95,7 +98,8 @@ __global__ __launch_bounds__(256) void delta_qk_kernel(const ChunkParams p) {
         if (d < dim) {
             const int c = kvh * dim + d;
             conv_rows16<T>(a, rows, ring, ring_ld, (is_k ? a.off_k : a.off_q) + c, is_k * a.kv_heads * dim + c,
-                           (is_k ? a.conv_k : a.conv_q) + (int64_t)c * a.taps, t0 + t, cnt, pos0, y);
+                           (is_k ? a.conv_k : a.conv_q) + (int64_t)c * a.taps, t0 + t, cnt, pos0, y,
+                           KIND == MI355_REC_SSD ? conv_bias(is_k ? a.conv_bk : a.conv_bq, c) : 0.f);
         } else {
 #pragma unroll
             for (int e = 0; e < 16; ++e) y[e] = 0.f;
@@ -105,7 +109,7 @@ __global__ __launch_bounds__(256) void delta_qk_kernel(const ChunkParams p) {
         for (int e = 0; e < 16; ++e) dst[e * ld] = y[e];
     }
     __syncthreads();
-    for (int t = wave; t < kC; t += 4) {  // unit vectors: a wave per row
+    for (int t = KIND == MI355_REC_DELTA ? wave : kC; t < kC; t += 4) {  // unit vectors: a wave per row
         float sq = 0.f, sk = 0.f;
         for (int d = lane; d < dim; d += 64) {
             sq += q[t * ld + d] * q[t * ld + d];
@@ -139,12 +143,12 @@ __global__ __launch_bounds__(256) void delta_qk_kernel(const ChunkParams p) {
         f32x4 akk = zero4(), aqk = zero4();
         for (int d = 4 * g; d < DP; d += 16) {
             const f32x4 b = *(const f32x4*)(k + (cb * 16 + c16) * ld + d);
-            akk = mfma4(*(const f32x4*)(k + (wave * 16 + c16) * ld + d), b, akk);
+            if constexpr (KIND == MI355_REC_DELTA) akk = mfma4(*(const f32x4*)(k + (wave * 16 + c16) * ld + d), b, akk);
             aqk = mfma4(*(const f32x4*)(q + (wave * 16 + c16) * ld + d), b, aqk);
         }
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            okk[(wave * 16 + 4 * g + r) * kC + cb * 16 + c16] = akk[r];
+            if constexpr (KIND == MI355_REC_DELTA) okk[(wave * 16 + 4 * g + r) * kC + cb * 16 + c16] = akk[r];
             oqk[(wave * 16 + 4 * g + r) * kC + cb * 16 + c16] = aqk[r];
         }
     }
@@ -298,6 +302,72 @@ __global__ __launch_bounds__(256) void delta_head_kernel(const ChunkParams p) {
             if (kb <= wave) acc = mfma4(ta[kb], *(const f32x4*)(kt + (nb * 16 + c16) * kC + kb * 16 + 4 * g) * bgv[kb], acc);
 #pragma unroll
         for (int r = 0; r < 4; ++r) oW[(wave * 16 + 4 * g + r) * DP + nb * 16 + c16] = acc[r];
+    }
+}
+
+// ------------------------------------------------------------------------------------ ssd: per head
+// 256 threads
+template <typename T>
+__global__ __launch_bounds__(256) void ssd_head_kernel(const ChunkParams p) {
+    const mi355_recurrent_args& a = p.r.a;
+    __shared__ double gcum[kC];
+    __shared__ float step[kC];
+    int head, chunk;
+    if (!head_chunk(p, head, chunk)) return;
+    const int seq = p.seq0 + blockIdx.y, t0 = chunk * kC;
+    const int cnt = p.r.b.count[seq];
+    if (t0 >= cnt) return;
+    const int DP = p.DP, VP = p.VP, tid = threadIdx.x, lane = tid & 63;
+    const int kvh = head / (a.heads / a.kv_heads);
+    const int pos0 = p.r.b.pos[seq];
+    const T* rows = (const T*)a.proj + (int64_t)p.r.b.row0[seq] * a.ld;
+    const int ring_ld = 2 * a.kv_heads * a.dim + a.heads * a.vdim;
+    const T* ring = (const T*)a.conv_ring + (int64_t)p.r.b.slot[seq] * a.taps * ring_ld;
+    const int64_t ci = chunk_base(p, seq) + chunk;
+    const int64_t gi = ci * p.GQ + kvh, hi = ci * a.heads + head;
+    if (tid < kC) {
+        float dt = 0.f, lg = 0.f;
+        if (t0 + tid < cnt) {
+            dt = softplus_f32(to_f32<T>(rows[(int64_t)(t0 + tid) * a.ld + a.off_a + head]) + a.dt_bias[head]);
+            lg = -expf(a.a_log[head]) * dt;
+        }
+        double s = lg;  // inclusive sum over the wave; f64, so that differences of far sums keep f32 accuracy
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const double v = __shfl_up(s, o, 64);
+            if (lane >= o) s += v;
+        }
+        gcum[tid] = s;
+        step[tid] = dt;
+        const double end = __shfl(s, 63, 64);
+        p.s.eg[hi * kC + tid] = expf((float)s);
+        p.s.ed[hi * kC + tid] = expf((float)(end - s)) * dt;
+        if (tid == 63) p.s.gam[hi * DP] = expf((float)end);
+    }
+    float* out = p.s.ut + hi * VP * kC;
+    for (int i = tid; i < 4 * VP; i += 256) {
+        const int d = i % VP, t = (i / VP) * 16;
+        float y[16];
+        if (d < a.vdim) {
+            const int c = head * a.vdim + d;
+            conv_rows16<T>(a, rows, ring, ring_ld, a.off_v + c, 2 * a.kv_heads * a.dim + c, a.conv_v + (int64_t)c * a.taps, t0 + t, cnt, pos0, y,
+                           conv_bias(a.conv_bv, c));
+        } else {
+#pragma unroll
+            for (int e = 0; e < 16; ++e) y[e] = 0.f;
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) *(f32x4*)(out + d * kC + t + 4 * e) = f32x4{y[4 * e], y[4 * e + 1], y[4 * e + 2], y[4 * e + 3]};
+    }
+    __syncthreads();
+    const float* qk = p.s.qk + gi * kC * kC;
+    float* oP = p.s.P + hi * kC * kC;
+    const float skip = a.skip[head];
+#pragma unroll 8
+    for (int n = 0; n < kC * kC / 256; ++n) {
+        const int i = n * 256 + tid, r = i >> 6, c = i & 63;
+        const float qv = qk[i];  // (above the diagonal blocks: unwritten scratch, dropped)
+        oP[i] = c <= r ? exp_f32((float)(gcum[r] - gcum[c])) * step[c] * qv + (c == r ? skip : 0.f) : 0.f;
     }
 }
 
@@ -489,7 +559,8 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c16 = lane & 15, g = lane >> 4;
     const int n_chunks = (p.r.b.count[seq] + kC - 1) / kC;
-    const int kvh = KIND == MI355_REC_DELTA ? head / (a.heads / a.kv_heads) : head;
+    constexpr bool kScalar = has_conv(KIND);  // one decay per head
+    const int kvh = kScalar ? head / (a.heads / a.kv_heads) : head;
     float* state = a.state + ((int64_t)p.r.b.slot[seq] * a.heads + head) * a.dim * a.vdim;
     const int64_t cb = chunk_base(p, seq);
     const int n_tiles = DP / 16;
@@ -505,7 +576,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
         }
     // a chunk's operands of this wave: two sets, the next chunk's requested when a chunk begins
     struct Ops {
-        f32x4 w[KIND == MI355_REC_DELTA ? 4 * NT : 1], k[NT][4], u, d, g[NT], v[4];
+        f32x4 w[KIND == MI355_REC_DELTA ? 4 * NT : 1], k[NT][4], u, d, g[NT], v[4], e[KIND == MI355_REC_SSD ? 4 : 1];
     };
     auto load = [&](int ch, Ops& x) {
         const int64_t hi = (cb + ch) * a.heads + head, gi = (cb + ch) * p.GQ + kvh;
@@ -516,6 +587,13 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
             for (int b = 0; b < 4 * NT; ++b) x.w[b] = *(const f32x4*)(W + min(b, n_tiles - 1) * 16 + 4 * g);
             x.u = *(const f32x4*)(ut + wave * 16 + 4 * g);
             x.d = *(const f32x4*)(p.s.ed + hi * kC + wave * 16 + 4 * g);
+            const float gm = p.s.gam[hi * DP];
+            x.g[0] = f32x4{gm, gm, gm, gm};
+        } else if constexpr (KIND == MI355_REC_SSD) {
+#pragma unroll
+            for (int b = 0; b < 4; ++b) x.v[b] = *(const f32x4*)(ut + b * 16 + 4 * g);
+#pragma unroll
+            for (int b = 0; b < 4; ++b) x.e[b] = *(const f32x4*)(p.s.ed + hi * kC + b * 16 + 4 * g);
             const float gm = p.s.gam[hi * DP];
             x.g[0] = f32x4{gm, gm, gm, gm};
         } else {
@@ -562,8 +640,12 @@ __global__ __launch_bounds__(256) void scan_kernel(const ChunkParams p) {
 #pragma unroll
             for (int b = 0; b < 4; ++b) x.v[b] = *(const f32x4*)(ul + c16 * kP + b * 16 + 4 * g);
         }
+        if constexpr (KIND == MI355_REC_SSD) {
 #pragma unroll
-        for (int t = 0; t < NT; ++t) S[t] *= x.g[KIND == MI355_REC_DELTA ? 0 : t];
+            for (int b = 0; b < 4; ++b) x.v[b] *= x.e[b];
+        }
+#pragma unroll
+        for (int t = 0; t < NT; ++t) S[t] *= x.g[kScalar ? 0 : t];
 #pragma unroll
         for (int b = 0; b < 4; ++b)
 #pragma unroll
@@ -598,7 +680,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
     const int DP = p.DP, VP = p.VP;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int c16 = lane & 15, g = lane >> 4;
-    const int kvh = KIND == MI355_REC_DELTA ? head / (a.heads / a.kv_heads) : head;
+    const int kvh = has_conv(KIND) ? head / (a.heads / a.kv_heads) : head;
     const int64_t ci = chunk_base(p, seq) + chunk, hi = ci * a.heads + head;
     const float* q = p.s.q + (ci * p.GQ + kvh) * kC * DP;
     const float* st = p.s.st + hi * VP * DP;
@@ -621,7 +703,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
             for (int v = 0; v < NV; ++v) o[rb][v] = mfma4(qv, b[v], o[rb][v]);
         }
     }
-    if constexpr (KIND == MI355_REC_DELTA) {
+    if constexpr (has_conv(KIND)) {
 #pragma unroll
         for (int rb = 0; rb < 4; ++rb) {
             const f32x4 e = *(const f32x4*)(p.s.eg + hi * kC + rb * 16 + 4 * g);
@@ -642,7 +724,8 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
             for (int v = 0; v < NV; ++v) o[rb][v] = mfma4(pv, b[v], o[rb][v]);
         }
     }
-    // ---- output norm over the head's columns, gate
+    // ---- output norm over the head's columns (ssd: none), gate
+    if constexpr (KIND != MI355_REC_SSD) {
 #pragma unroll
     for (int rb = 0; rb < 4; ++rb)
 #pragma unroll
@@ -654,21 +737,23 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
             if (c16 == 0) ssq[wave][rb * 16 + 4 * g + r] = s;
         }
     __syncthreads();
+    }
     const T* rows = (const T*)a.proj + (int64_t)(p.r.b.row0[seq] + t0) * a.ld;
-    T* y = (T*)a.y + (int64_t)(p.r.b.row0[seq] + t0) * a.ldy;
+    out_t<KIND, T>* y = (out_t<KIND, T>*)a.y + (int64_t)(p.r.b.row0[seq] + t0) * a.ldy;
 #pragma unroll
     for (int rb = 0; rb < 4; ++rb)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int t = rb * 16 + 4 * g + r;
             if (t0 + t >= cnt) continue;
-            const float rinv = 1.0f / sqrtf((ssq[0][t] + ssq[1][t] + ssq[2][t] + ssq[3][t]) / (float)a.vdim + a.eps);
+            const float rinv = KIND == MI355_REC_SSD ? 1.f : 1.0f / sqrtf((ssq[0][t] + ssq[1][t] + ssq[2][t] + ssq[3][t]) / (float)a.vdim + a.eps);
 #pragma unroll
             for (int v = 0; v < NV; ++v) {
                 const int n = (wave + 4 * v) * 16 + c16;
                 if (n >= a.vdim) continue;
                 const float gate = silu_f32(to_f32<T>(rows[(int64_t)t * a.ld + a.off_g + head * a.vdim + n]));
-                y[(int64_t)t * a.ldy + head * a.vdim + n] = from_f32<T>(o[rb][v][r] * rinv * a.head_norm[head * a.norm_ld + n] * gate);
+                const float w = KIND == MI355_REC_SSD ? gate : rinv * a.head_norm[head * a.norm_ld + n] * gate;
+                y[(int64_t)t * a.ldy + head * a.vdim + n] = from_f32<out_t<KIND, T>>(o[rb][v][r] * w);
             }
         }
 }
@@ -677,9 +762,10 @@ inline int pad16(int n) { return (n + 15) / 16 * 16; }
 
 // floats per packed chunk
 size_t chunk_floats(int kind, int heads, int kv_heads, int dim, int vdim) {
-    const size_t DP = pad16(dim), VP = pad16(vdim), H = heads, G = kind == MI355_REC_DELTA ? kv_heads : heads;
+    const size_t DP = pad16(dim), VP = pad16(vdim), H = heads, G = has_conv(kind) ? kv_heads : heads;
     size_t n = 2 * G * kC * DP + H * kC * kC + H * VP * kC + H * VP * DP + H * DP;
-    if (kind == MI355_REC_DELTA) n += 2 * G * kC * kC + H * kC * DP + 2 * H * kC;
+    if (has_conv(kind)) n += G * kC * kC + 2 * H * kC;
+    if (kind == MI355_REC_DELTA) n += G * kC * kC + H * kC * DP;
     return n;
 }
 
@@ -719,8 +805,8 @@ int run_group(const ChunkParams& p, int seqs, hipStream_t s) {
     const dim3 heads((a.heads + 7) / 8 * 8 * chunks, seqs);
     if (a.kind == MI355_REC_DELTA) {
         const size_t lds1 = (size_t)2 * kC * (p.DP + 4) * 4;
-        if (int rc = set_lds(delta_qk_kernel<T>, lds1)) return rc;
-        hipLaunchKernelGGL(delta_qk_kernel<T>, dim3(chunks, a.kv_heads, seqs), dim3(256), lds1, s, p);
+        if (int rc = set_lds(delta_qk_kernel<T, MI355_REC_DELTA>, lds1)) return rc;
+        hipLaunchKernelGGL((delta_qk_kernel<T, MI355_REC_DELTA>), dim3(chunks, a.kv_heads, seqs), dim3(256), lds1, s, p);
         MI355_LAUNCH_CHECK();
         const size_t lds2 = ((size_t)2 * kC * kP + (size_t)kC * kX + (size_t)p.VP * kP) * 4;
         if (int rc = set_lds(delta_head_kernel<T>, lds2)) return rc;
@@ -728,6 +814,16 @@ int run_group(const ChunkParams& p, int seqs, hipStream_t s) {
         MI355_LAUNCH_CHECK();
         if (int rc = launch_scan<MI355_REC_DELTA>(p, seqs, s)) return rc;
         return launch_out<T, MI355_REC_DELTA>(p, heads, s);
+    }
+    if (a.kind == MI355_REC_SSD) {
+        const size_t lds = (size_t)2 * kC * (p.DP + 4) * 4;
+        if (int rc = set_lds(delta_qk_kernel<T, MI355_REC_SSD>, lds)) return rc;
+        hipLaunchKernelGGL((delta_qk_kernel<T, MI355_REC_SSD>), dim3(chunks, a.kv_heads, seqs), dim3(256), lds, s, p);
+        MI355_LAUNCH_CHECK();
+        hipLaunchKernelGGL(ssd_head_kernel<T>, heads, dim3(256), 0, s, p);
+        MI355_LAUNCH_CHECK();
+        if (int rc = launch_scan<MI355_REC_SSD>(p, seqs, s)) return rc;
+        return launch_out<T, MI355_REC_SSD>(p, heads, s);
     }
     const size_t lds = ((size_t)3 * kC * kP + 5 * kCh + (size_t)kC * a.rank) * 4;
     if (a.kind == MI355_REC_WKV) {
@@ -755,7 +851,7 @@ int mi355_recurrent_chunks(const RecParams& r, hipStream_t s) {
     p.r = r;
     p.DP = pad16(a.dim);
     p.VP = pad16(a.vdim);
-    p.GQ = a.kind == MI355_REC_DELTA ? a.kv_heads : a.heads;
+    p.GQ = has_conv(a.kind) ? a.kv_heads : a.heads;
     const size_t per = chunk_floats(a.kind, a.heads, a.kv_heads, a.dim, a.vdim);
     // packed chunks of n sequences: at most rows / 64 + n (chunk_base)
     const size_t cap = a.scratch_bytes / (per * 4);
@@ -767,18 +863,18 @@ int mi355_recurrent_chunks(const RecParams& r, hipStream_t s) {
         f += n * cap;
         return q;
     };
-    const bool delta = a.kind == MI355_REC_DELTA;
+    const bool delta = a.kind == MI355_REC_DELTA, conv = has_conv(a.kind);
     p.s.q = take(G * kC * DP);
     p.s.kt = take(G * kC * DP);
     p.s.kk = delta ? take(G * kC * kC) : nullptr;
-    p.s.qk = delta ? take(G * kC * kC) : nullptr;
+    p.s.qk = conv ? take(G * kC * kC) : nullptr;
     p.s.P = take(H * kC * kC);
     p.s.W = delta ? take(H * kC * DP) : nullptr;
     p.s.ut = take(H * VP * kC);
     p.s.st = take(H * VP * DP);
     p.s.gam = take(H * DP);
-    p.s.eg = delta ? take(H * kC) : nullptr;
-    p.s.ed = delta ? take(H * kC) : nullptr;
+    p.s.eg = conv ? take(H * kC) : nullptr;
+    p.s.ed = conv ? take(H * kC) : nullptr;
     for (int s0 = 0; s0 < r.b.seqs; s0 += (int)most) {
         const int n = (size_t)(r.b.seqs - s0) < most ? r.b.seqs - s0 : (int)most;
         p.seq0 = s0;

@@ -1,6 +1,7 @@
 // Causal attention over a sliding window or a chunk: grouped key / value heads, different key and value sizes, interleaved rotation of
-// rot_dims dimensions, queries, keys and values over their root mean square, first rows that stay visible, a factor and a distance bias per
-// head, a sink in the softmax sum, sigmoid gates per head or per value.  A slot's cache is, per key head, `kept` rows for the first positions and a ring for the others.  A layer lends
+// rot_dims dimensions, queries, keys and values over their root mean square (and by factors per dimension), first rows that stay visible, a factor
+// and a distance bias per head, bounded scores, a sink in the softmax sum, sigmoid gates per head or per value, values mixed with those of an
+// earlier layer.  A slot's cache is, per key head, `kept` rows for the first positions and a ring for the others.  A layer lends
 // its keys and values to later ones, which read its cache (and, in a prompt step, its prepared rows).
 //
 //   window_rows_kernel    one workgroup per (row, key head, split of the keys): decode steps of any size (q and the row's own k are
@@ -29,6 +30,10 @@ __device__ __forceinline__ int cache_row(const mi355_window_attn_args& a, int p)
 // first position of the window or chunk of the row at position p
 __device__ __forceinline__ int first_seen(const mi355_window_attn_args& a, int p) { return a.chunked ? p - p % a.window : p - a.window + 1; }
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float cap_score(float s, float cap) { return cap != 0.f ? cap * tanhf(s / cap) : s; }
+// element d of key head g's value of `row`, as it is cached (without its norm): with v_first mixed, in f32
+template <typename T>
+__device__ __forceinline__ float mixed_value(const mi355_window_attn_args& a, int64_t row, int g, int d, float v);
 
 // turn of (u, v) by pos * inv_freq: the angle is reduced in f64, so far positions keep f32 accuracy
 __device__ __forceinline__ void pair_cos_sin(int pos, double inv_freq, float& c, float& s) {
@@ -49,6 +54,11 @@ template <>
 __device__ __forceinline__ float from_f32<float>(float v) { return v; }
 template <>
 __device__ __forceinline__ bf16_t from_f32<bf16_t>(float v) { return f32_to_bf16(v); }
+
+template <typename T>
+__device__ __forceinline__ float mixed_value(const mi355_window_attn_args& a, int64_t row, int g, int d, float v) {
+    return a.v_first == nullptr ? v : (1.0f - a.v_mix) * v + a.v_mix * to_f32<T>(((const T*)a.v_first)[row * a.ld_v_first + g * a.vdim + d]);
+}
 
 template <typename T, int N>
 __device__ __forceinline__ void load_vec(const T* p, float (&o)[N]) {
@@ -94,7 +104,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     const int dim = a.dim, vdim = a.vdim;
     float* q = (float*)smem;                      // [HT][dim], scaled
     float* kn = q + (HT * dim + 3) / 4 * 4;                     // [dim]: the row's own key, as the ring stores it
-    float* vn = kn + (dim + 3) / 4 * 4;           // [vdim, padded to VE]: the row's own value over its root mean square (unit_v)
+    float* vn = kn + (dim + 3) / 4 * 4;           // [vdim, padded to VE]: the row's own value where it is mixed or over its root mean square
     float* sc = vn + (vdim + 7) / 8 * 8;          // [kKeys][HT]
     float* stat = sc + HT * kKeys;                // [4][HT]: maximum, sum, correction, slope of the distance bias
     float* red = stat + 4 * HT;                   // [key lanes][HT][columns]: at most kRowThreads HT VE
@@ -134,6 +144,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     const int step = (n_keys + p.n_split - 1) / p.n_split;
     const int k_begin = split * step, k_end = min(n_keys, k_begin + step);
     const bool owner = FRESH && p.own && k_begin < n_keys && k_end == n_keys;  // this split holds the row's own key
+    const bool made_v = a.unit_v || a.v_first != nullptr;                      // ... whose value is not the projection's
 
     // 32 lanes per head, a pair of values each: over the root mean square, rotated, scaled; a decode step's own key likewise (number nh)
     T* kw = kcache + row_of(n_keys - 1) * (unsigned)dim;
@@ -156,7 +167,12 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             for (int d = 64 * kHeld + lane; d < dim; d += 32) ss += at(d) * at(d);
             f /= sqrtf(group_sum(ss, 32) / (float)dim + a.unit_eps);
         }
+        const float* by = key ? a.k_norm : a.q_norm;
         auto put = [&](int pi, float u, float w) {
+            if (by != nullptr) {
+                u *= by[2 * pi];
+                if (2 * pi + 1 < dim) w *= by[2 * pi + 1];
+            }
             if (const int ri = pi - a.rot_at / 2; ri >= 0 && 2 * ri < a.rot_dims) {
                 float c, s;
                 pair_cos_sin(pos, a.inv_freq[ri], c, s);
@@ -186,17 +202,21 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
     if (owner && ht == 0) {
         T* vw = vcache + row_of(n_keys - 1) * (unsigned)vdim;
         const T* vs = prow + a.off_v + (int64_t)kvh * vdim;
-        if (!a.unit_v)
+        if (!made_v)
             for (int d = tid; d < vdim; d += kRowThreads) vw[d] = vs[d];
     }
-    if (owner && a.unit_v && tid < 64) {
+    if (owner && made_v && tid < 64) {
         T* vw = vcache + row_of(n_keys - 1) * (unsigned)vdim;
         const T* vs = prow + a.off_v + (int64_t)kvh * vdim;
-        float ss = 0.f;
-        for (int d = tid; d < vdim; d += 64) ss += to_f32<T>(vs[d]) * to_f32<T>(vs[d]);
-        const float r = 1.0f / sqrtf(group_sum(ss, 64) / (float)vdim + a.unit_eps);
+        float r = 1.f;
+        auto value = [&](int d) { return mixed_value<T>(a, row, kvh, d, to_f32<T>(vs[d])); };
+        if (a.unit_v) {
+            float ss = 0.f;
+            for (int d = tid; d < vdim; d += 64) ss += value(d) * value(d);
+            r = 1.0f / sqrtf(group_sum(ss, 64) / (float)vdim + a.unit_eps);
+        }
         for (int d = tid; d < (vdim + 7) / 8 * 8; d += 64) {
-            const T o = from_f32<T>(d < vdim ? to_f32<T>(vs[d]) * r : 0.f);
+            const T o = from_f32<T>(d < vdim ? value(d) * r : 0.f);
             vn[d] = to_f32<T>(o);
             if (ht == 0 && d < vdim) vw[d] = o;
         }
@@ -257,7 +277,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
                     const float dist = (float)(pos - (g < n_first ? g : g + w_shift));
 #pragma unroll
                     for (int h = 0; h < HT; ++h)
-                        if (h < nh) sc[kk * HT + h] = dot[u][h] - stat[3 * HT + h] * dist;
+                        if (h < nh) sc[kk * HT + h] = cap_score(dot[u][h], a.softcap) - stat[3 * HT + h] * dist;
                 }
             }
         }
@@ -266,7 +286,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             float s = 0.f;
             for (int d = l16; d < dim; d += 16) s += kn[d] * q[h * dim + d];
             s = group_sum(s, 16);
-            if (l16 == 0) sc[(n_keys - 1 - kb) * HT + h] = s;
+            if (l16 == 0) sc[(n_keys - 1 - kb) * HT + h] = cap_score(s, a.softcap);
         }
         __syncthreads();
         // ---- running maximum and sum: one wave per head
@@ -313,7 +333,7 @@ __global__ __launch_bounds__(kRowThreads, HT <= 4 ? 4 : 2) void window_rows_kern
             };
             const int nv = owner && kb + nk == n_keys ? nk - 1 : nk;  // (the own value is not in the cache yet)
             if (nv < nk && kl == 0) {
-                if (a.unit_v) add(nk - 1, (const float*)vn);
+                if (made_v) add(nk - 1, (const float*)vn);
                 else add(nk - 1, prow + a.off_v + (int64_t)kvh * vdim);
             }
 #pragma unroll 4
@@ -400,11 +420,15 @@ __global__ __launch_bounds__(256) void prepare_keys_kernel(const WinParams p) {
     const bool moved = a.role == MI355_KV_LENDS;
     const T *k = src + a.off_k + (int64_t)g * a.dim, *v = src + a.off_v + (int64_t)g * a.vdim;
     T *o = (T*)p.krows + row * p.ld_rows + (int64_t)g * a.dim, *vo = (T*)p.vrows + row * p.ld_rows + (int64_t)g * a.vdim;
-    if (a.unit_v) {
-        float ss = 0.f;
-        for (int d = lane; d < a.vdim; d += 64) ss += to_f32<T>(v[d]) * to_f32<T>(v[d]);
-        const float r = 1.0f / sqrtf(group_sum(ss, 64) / (float)a.vdim + a.unit_eps);
-        for (int d = lane; d < a.vdim; d += 64) vo[d] = from_f32<T>(to_f32<T>(v[d]) * r);
+    if (a.unit_v || a.v_first != nullptr) {
+        auto value = [&](int d) { return mixed_value<T>(a, row, g, d, to_f32<T>(v[d])); };
+        float r = 1.f;
+        if (a.unit_v) {
+            float ss = 0.f;
+            for (int d = lane; d < a.vdim; d += 64) ss += value(d) * value(d);
+            r = 1.0f / sqrtf(group_sum(ss, 64) / (float)a.vdim + a.unit_eps);
+        }
+        for (int d = lane; d < a.vdim; d += 64) vo[d] = from_f32<T>(value(d) * r);
     } else if (moved) {
         for (int d = lane; d < a.vdim; d += 64) vo[d] = v[d];
     }
@@ -424,6 +448,10 @@ __global__ __launch_bounds__(256) void prepare_keys_kernel(const WinParams p) {
     for (int pi = lane; pi < pairs; pi += 64) {
         const bool two = 2 * pi + 1 < a.dim;
         float u = (pi == lane ? k0 : to_f32<T>(k[2 * pi])) * rms, w = (pi == lane ? k1 : two ? to_f32<T>(k[2 * pi + 1]) : 0.f) * rms;
+        if (a.k_norm != nullptr) {
+            u *= a.k_norm[2 * pi];
+            if (two) w *= a.k_norm[2 * pi + 1];
+        }
         if (pi >= rot0 && pi - rot0 < half) {
             float c, s;
             pair_cos_sin(pos, a.inv_freq[pi - rot0], c, s);
@@ -540,7 +568,8 @@ __global__ __launch_bounds__(256, D <= 192 ? 2 : 1) void window_tiles_kernel(con
     bf16x8 bq[D / 16];
     {
         const bf16_t* src = proj + (int64_t)(row0 + q_row) * a.ld + a.off_q + (int64_t)h * a.dim;
-        float qs = (a.head_scale != nullptr ? a.scale * a.head_scale[h] : a.scale) * 1.44269504088896340736f;
+        // (bounded scores: to twice the argument of the tanh in that domain)
+        float qs = (a.head_scale != nullptr ? a.scale * a.head_scale[h] : a.scale) * 1.44269504088896340736f * (a.softcap != 0.f ? 2.0f / a.softcap : 1.0f);
         if (a.unit_qk) {  // lanes c and c + 32 hold the row between them
             float ss = 0.f;
 #pragma unroll
@@ -566,6 +595,7 @@ __global__ __launch_bounds__(256, D <= 192 ? 2 : 1) void window_tiles_kernel(con
 #pragma unroll
                 for (int e = 0; e < 8; e += 2) {
                     float u = v[e], w = v[e + 1];
+                    if (a.q_norm != nullptr) u *= a.q_norm[d0 + e], w *= a.q_norm[d0 + e + 1];
                     if (const int rd = d0 + e - a.rot_at; rd >= 0 && rd < a.rot_dims) {
                         float cs, sn;
                         pair_cos_sin(q_pos, a.inv_freq[rd >> 1], cs, sn);
@@ -708,6 +738,7 @@ __global__ __launch_bounds__(256, D <= 192 ? 2 : 1) void window_tiles_kernel(con
     for (int dt = 0; dt < DV / 32; ++dt)
 #pragma unroll
         for (int i = 0; i < 16; ++i) acc[dt][i] = 0.f;
+    const float cap2 = a.softcap * 1.44269504088896340736f;
     const float slope2 = a.slope != nullptr ? a.slope[h] * 1.44269504088896340736f : 0.f;
     float m_run = -1.0e30f, l_run = 0.f;
     if (a.sink != nullptr) {  // a key without a value; one of the two lanes of a query counts it
@@ -744,6 +775,12 @@ __global__ __launch_bounds__(256, D <= 192 ? 2 : 1) void window_tiles_kernel(con
                     const bf16x8 ka = *(const bf16x8*)(kt + key * (D * 2) + (((2 * ks + hh) ^ (key & kSwz)) << 4));
                     st[t2] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka, bq[ks], st[t2], 0, 0, 0);
                 }
+            if (cap2 != 0.f) {  // cap tanh(s / cap), tanh(x) = 1 - 2 / (1 + e^2x)
+#pragma unroll
+                for (int t2 = 0; t2 < 2; ++t2)
+#pragma unroll
+                    for (int i = 0; i < 16; ++i) st[t2][i] = cap2 - 2.0f * cap2 * __builtin_amdgcn_rcpf(1.0f + exp2_fast(st[t2][i]));
+            }
             if (slope2 != 0.f) {  // (log2 e slope (i - j) is taken off)
                 const float at = slope2 * (float)(kb * kBK + 4 * hh - q_pos);
 #pragma unroll
@@ -938,7 +975,7 @@ int run(WinParams p, hipStream_t s) {
         }
         return 0;
     }
-    if (a.role == MI355_KV_LENDS || (a.role == MI355_KV_OWN && (a.rot_dims > 0 || a.unit_qk || a.unit_v))) {
+    if (a.role == MI355_KV_LENDS || (a.role == MI355_KV_OWN && (a.rot_dims > 0 || a.unit_qk || a.unit_v || a.v_first != nullptr))) {
         hipLaunchKernelGGL(prepare_keys_kernel<T>, dim3((unsigned)(((int64_t)p.b.max_count * a.kv_heads + 3) / 4), p.b.seqs), dim3(256), 0, s, p);
         MI355_LAUNCH_CHECK();
     }
@@ -965,6 +1002,9 @@ int make_params(const mi355_window_attn_args* a, const mi355_seq_batch* b, WinPa
     MI355_CHECK_ARG(a->window > 0 && a->ring > 0 && a->rot_dims >= 0 && a->rot_dims % 2 == 0 && a->rot_at >= 0 && a->rot_at % 2 == 0 && a->rot_at + a->rot_dims <= a->dim &&
                         (a->rot_dims == 0 || a->inv_freq),
                     MI355_E_SHAPE, "window_attention: bad window %d, ring %d or rotation %d", a->window, a->ring, a->rot_dims);
+    MI355_CHECK_ARG(a->unit_qk || (a->q_norm == nullptr && a->k_norm == nullptr), MI355_E_ARG, "window_attention: factors per dimension follow a norm");
+    MI355_CHECK_ARG(a->softcap >= 0.f && (a->v_first == nullptr || (a->ld_v_first >= (int64_t)a->kv_heads * a->vdim && (a->role == MI355_KV_OWN || a->role == MI355_KV_LENDS))),
+                    MI355_E_ARG, "window_attention: bad softcap %g or first values", a->softcap);
     MI355_CHECK_ARG(a->keep >= 0 && a->keep <= a->kept, MI355_E_SHAPE, "window_attention: %d first rows visible, %d cached", a->keep, a->kept);
     MI355_CHECK_ARG(a->role == MI355_KV_ROWS ? b->max_count > 1 && a->rows_per_seq > 0 && a->tail_dims >= 0 && a->tail_dims < a->dim && a->tail_dims % 8 == 0 &&
                                                    (uint64_t)a->rows_per_seq * (uint64_t)a->ld_tail < 0xFFFFFFFFull &&

@@ -1,6 +1,6 @@
 """Layered hybrid decoders: a list of layers, each with its own mixer (window or chunk attention, latent attention, gated delta rule, gated
-linear attention, WKV time mixing) and an optional feed-forward (squared ReLU, gated GELU, clamped gate, mixture of experts), behind or beside
-the mixer; some layers run several times in a row, some use another layer's weights.
+linear attention, WKV time mixing, state-space duality) and an optional feed-forward (squared ReLU, gated GELU, clamped gate, mixture of
+experts), behind or beside the mixer, or between norms of its own; some layers run several times in a row, some use another layer's weights.
 
 `HybridConfig` reads a parsed config.json; `HybridLM` holds the weights under their checkpoint names and hands the arithmetic to
 `hybrid_engine.HybridEngine` (csrc/hybrid.hip and the kernels it calls).  A design is an entry in DESIGNS: which mixers and feed-forwards it
@@ -22,7 +22,7 @@ from . import _native as nat
 class MixerSpec:
     """Sizes and constants of one layer's mixer; which fields count depends on `type`."""
 
-    type: str                      # attention | latent | delta | gla | wkv
+    type: str                      # attention | latent | delta | gla | wkv | ssd
     heads: int
     kv_heads: int
     dim: int                       # query / key size of a head
@@ -36,7 +36,7 @@ class MixerSpec:
     sink: bool = False             # a learned term in every softmax sum
     gate_values: bool = False      # a gate per value, not per head
     kv_from: Optional[int] = None  # the layer whose keys and values are read
-    taps: int = 0                  # delta: convolution taps
+    taps: int = 0                  # delta, ssd: convolution taps
     tau: float = 1.0               # gla
     chunked: bool = False          # `window` counts chunks from position 0
     temp: bool = False             # a learned factor per head of the scores
@@ -46,6 +46,13 @@ class MixerSpec:
     rot_dim: int = 0               # latent: rotated query / key size of a head, next to dim
     q_rank: int = 0
     kv_rank: int = 0
+    rot_halves: bool = False       # dimension i turns with i + rot_dims / 2, not with its neighbour
+    rot_scaling: Optional[Tuple[float, float, float, float]] = None  # factor, low, high, original length: slow turns are slowed down further
+    qk_norm: bool = False          # factors per dimension behind unit_qk
+    biased: bool = False           # q, k and v have biases
+    softcap: float = 0.0           # bound of the scores, 0: none
+    v_mix: bool = False            # v is mixed with that of the first such layer
+    norm_groups: int = 1           # ssd: parts of the output that are normalised by themselves
 
 
 @dataclass
@@ -57,6 +64,11 @@ class MlpSpec:
     scale: float = 1.0             # the chosen experts' weights sum to this
     ff_shared: int = 0             # of the expert that every token runs, 0: none
     limit: float = 0.0             # clampglu: bound of both halves
+    act: str = "silu_gate"         # experts: silu_gate | relu2
+    score: str = "sigmoid"         # experts: sigmoid (renormalised) | softmax (with a correction of the choice)
+    groups: int = 0                # experts are chosen from the best `keep_groups` of `groups` equal runs, 0: from all
+    keep_groups: int = 0
+    identity: int = 0              # router outputs behind the experts' that stand for the row itself
 
 
 @dataclass
@@ -133,6 +145,55 @@ def _wkv(m: dict) -> MixerSpec:
     return MixerSpec("wkv", m["heads"], m["heads"], m["dim"], m["dim"])
 
 
+def _halves(m: dict, extra: Tuple[str, ...], scaled: bool, **kw) -> MixerSpec:
+    """Attention over every earlier row: biased projections, rotation by halves, values mixed with the first such layer's, no gate."""
+    _only(m, ("heads", "kv_heads", "dim", "vdim", "rot", "scale", "v_mix", *extra), "attention mixer")
+    rot = m.get("rot") or {"base": 1.0, "dims": 0}
+    _only(rot, ("base", "dims", "scaling") if scaled else ("base", "dims"), "rotation")
+    if int(rot["dims"]) % 2 or int(rot["dims"]) > int(m["dim"]):
+        raise ValueError(f"rotation of {rot['dims']} of {m['dim']} dimensions")
+    scaling = rot.get("scaling")
+    if scaling is not None:
+        _only(scaling, ("factor", "low", "high", "original"), "rotation scaling")
+        scaling = tuple(float(scaling[n]) for n in ("factor", "low", "high", "original"))
+    return MixerSpec("attention", m["heads"], m["kv_heads"], m["dim"], m["vdim"], scale=float(m["scale"]), window=1 << 30, rot_dims=int(rot["dims"]),
+                     rot_base=float(rot["base"]), rot_halves=True, rot_scaling=scaling, biased=True, gated=False, v_mix=bool(m.get("v_mix")), **kw)
+
+
+def _normed_attention(m: dict) -> MixerSpec:
+    """Queries and keys over their root mean square, times a factor per dimension."""
+    return _halves(m, (), False, unit_qk=True, qk_norm=True)
+
+
+def _capped_attention(m: dict) -> MixerSpec:
+    """Bounded scores, slow rotations slowed down."""
+    return _halves(m, ("softcap",), True, softcap=float(m.get("softcap") or 0.0))
+
+
+def _ssd(m: dict) -> MixerSpec:
+    _only(m, ("heads", "groups", "state", "vdim", "conv", "norm_groups"), "state-space mixer")
+    spec = MixerSpec("ssd", m["heads"], m["groups"], m["state"], m["vdim"], taps=int(m["conv"]), norm_groups=int(m["norm_groups"]))
+    if spec.norm_groups < 1 or spec.heads * spec.vdim % spec.norm_groups:
+        raise ValueError(f"state-space mixer: {spec.norm_groups} groups of {spec.heads * spec.vdim} outputs")
+    return spec
+
+
+def _grouped_experts(d: dict) -> MlpSpec:
+    """Softmax scores with corrected choices inside the best groups, squared-ReLU experts, the last router outputs the row itself."""
+    _only(d, ("kind", "expert", "router"), "feed-forward")
+    _only(d["expert"], ("ff",), "expert")
+    r = d["router"]
+    _only(r, ("experts", "top", "groups", "identity"), "router")
+    g = r.get("groups") or {"count": 1, "keep": 1}
+    _only(g, ("count", "keep"), "router groups")
+    spec = MlpSpec("experts", int(d["expert"]["ff"]), int(r["experts"]), int(r["top"]), act="relu2", score="softmax", groups=int(g["count"]),
+                   keep_groups=int(g["keep"]), identity=int(r.get("identity") or 0))
+    total = spec.experts + spec.identity
+    if not (spec.groups >= 1 and total % spec.groups == 0 and 1 <= spec.keep_groups <= spec.groups and 1 <= spec.top <= spec.keep_groups * (total // spec.groups)):
+        raise ValueError(f"router: {spec.top} of {total} outputs in {spec.keep_groups} of {spec.groups} groups")
+    return spec
+
+
 def _clamped(d: dict) -> MlpSpec:
     _only(d, ("kind", "ff", "limit"), "feed-forward")
     return MlpSpec("clampglu", int(d["ff"]), limit=float(d["limit"]))
@@ -167,12 +228,15 @@ class Design:
     norm_add: float = 0.0          # an RMSNorm's scale is norm_add + its weight
     tied: bool = False             # the logits are products with the embedding table
     parallel: bool = False         # mixer and feed-forward read one norm, x += mixer(h) + ff(h); norms in groups
+    sandwich: bool = False         # x += post(gate(h) * sublayer(h)), then x becomes an average over depth; the embedding has a norm
 
 
 DESIGNS = {
     "Sekulorn": Design({"attention": _attention, "delta": _delta, "gla": _gla}, {"dense": _plain("relu2")}, ("loop", "residual_mult")),
     "Kovalorn": Design({"attention": _sink_attention}, {"dense": _plain("geglu"), "moe": _experts}, ("logit_scale",), norm_add=1.0, tied=True),
     "Kudazen": Design({"attention": _chunk_attention, "latent_attention": _latent_attention, "wkv": _wkv}, {"dense": _clamped}, (), tied=True, parallel=True),
+    "Gurolix": Design({"mamba2": _ssd, "attention": _normed_attention, "attention_2": _capped_attention}, {"moe": _grouped_experts}, (), norm_add=1.0,
+                      sandwich=True),
 }
 
 
@@ -226,6 +290,10 @@ class HybridConfig:
                     raise ValueError(f"layer {i}: layer {l.weights_of} has no tensors of its own")
                 if (own.mixer, own.mlp) != (l.mixer, l.mlp):
                     raise ValueError(f"layer {i} differs from layer {l.weights_of}, whose weights it uses")
+        mixed = [(i, l.mixer) for i, l in enumerate(layers) if l.mixer.v_mix]
+        for i, m in mixed:
+            if (m.kv_heads, m.vdim) != (mixed[0][1].kv_heads, mixed[0][1].vdim):
+                raise ValueError(f"layer {i} mixes values of other sizes than layer {mixed[0][0]}'s")
         loop = d.get("loop")
         if loop is not None:
             _only(loop, ("start", "stop", "times"), "loop")
@@ -248,6 +316,10 @@ class HybridConfig:
         a, b, times = self.loop
         return [*range(a), *(list(range(a, b)) * times), *range(b, len(self.layers))]
 
+    def first_values(self) -> Optional[int]:
+        """The layer whose values the others that mix them read."""
+        return next((i for i, l in enumerate(self.layers) if l.mixer.v_mix), None)
+
     def lenders(self) -> List[Optional[int]]:
         """Per run, the run whose keys and values it reads (the last one of its lender so far), None: its own."""
         last: Dict[int, int] = {}
@@ -267,6 +339,8 @@ def projections(m: MixerSpec) -> Tuple[str, ...]:
         return ("dq", "dkv")
     if m.type == "wkv":
         return ("r", "k", "v", "g", "w1")  # (each reads a mix of its own)
+    if m.type == "ssd":
+        return ("z", "x", "B", "C", "dt")  # (the rows of one tensor, `in`)
     return ("q", "k", "v", "g", "a", "b") if m.type == "delta" else ("q", "k", "v", "g", "a1")
 
 
@@ -274,6 +348,9 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
     """name -> shape of every tensor of a checkpoint; rank[i]: the low-rank size of gla or wkv layer i (only its tensors know it)."""
     W = cfg.width
     out = {"embed": (cfg.vocab_size, W)}
+    sandwich = cfg.design.sandwich
+    if sandwich:
+        out["embed.norm"] = (W,)
 
     def gated(p: str, ff: int) -> None:
         out.update({p + "gate": (ff, W), p + "up": (ff, W), p + "down": (W, ff)})
@@ -295,6 +372,16 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
                 out[x + "g"] = (hv if m.gate_values else m.heads, W)
             if m.temp:
                 out[x + "temp"] = (m.heads,)
+            if m.biased:
+                out.update({x + "q.b": (m.heads * m.dim,), x + "k.b": (gk,), x + "v.b": (m.kv_heads * m.vdim,)})
+            if m.qk_norm:
+                out.update({x + "q.norm": (m.dim,), x + "k.norm": (m.dim,)})
+            if m.v_mix:
+                out[x + "vmix"] = ()
+        elif m.type == "ssd":
+            n = hv + 2 * gk
+            out.update({x + "in": (hv + n + m.heads, W), x + "conv": (n, m.taps), x + "conv.b": (n,), x + "dt_bias": (m.heads,), x + "A_log": (m.heads,),
+                        x + "D": (m.heads,), x + "norm": (hv,)})
         elif m.type == "latent":
             out.update({x + "dq": (m.q_rank, W), x + "dq.norm": (m.q_rank,), x + "uq": (m.heads * (m.dim + m.rot_dim), m.q_rank),
                         x + "dkv": (m.kv_rank + m.rot_dim, W), x + "dkv.norm": (m.kv_rank,), x + "uk": (gk, m.kv_rank), x + "uv": (hv, m.kv_rank),
@@ -312,6 +399,10 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
             out.update({x + "a1": (rank[i], W), x + "a2": (gk, rank[i]), x + "a2.b": (gk,)})
         out[x + "o"] = (W, hv)
         f = l.mlp
+        if sandwich:
+            out.update({p + "norm1b": (W,), p + "rg1": (W, W), p + "rg1.b": (W,), p + "dwa": (i + 2,)})
+            if f is not None:
+                out.update({p + "norm2b": (W,), p + "rg2": (W, W), p + "rg2.b": (W,)})
         if f is not None:
             if not cfg.design.parallel:
                 out[p + "norm2"] = (W,)
@@ -320,9 +411,14 @@ def tensor_shapes(cfg: HybridConfig, rank: Dict[int, int]) -> Dict[str, Tuple[in
             elif f.kind in ("geglu", "clampglu"):
                 gated(p + "mlp.", f.ff)
             else:
-                out[p + "mlp.router"] = (f.experts, W)
+                out[p + "mlp.router"] = (f.experts + f.identity, W)
+                if f.score == "softmax":
+                    out[p + "mlp.correction"] = (f.experts + f.identity,)
                 for e in range(f.experts):
-                    gated(f"{p}mlp.e{e}.", f.ff)
+                    if f.act == "relu2":
+                        out.update({f"{p}mlp.e{e}.up": (f.ff, W), f"{p}mlp.e{e}.down": (W, f.ff)})
+                    else:
+                        gated(f"{p}mlp.e{e}.", f.ff)
                 if f.ff_shared:
                     gated(p + "mlp.shared.", f.ff_shared)
     out["final.norm"] = (W,)

@@ -9,9 +9,10 @@ from __future__ import annotations
 
 import ctypes as C
 import gc
+import math
 import os
 import weakref
-from typing import Dict, List, NamedTuple, Optional, Sequence
+from typing import Dict, List, NamedTuple, Optional, Sequence, Tuple
 
 import torch
 
@@ -21,11 +22,13 @@ from ._native import ExpertsArgs, HybridLayer, HybridModel, Proj, SeqBatch, chec
 from .hybrid import HybridLM, LayerSpec, MixerSpec, MlpSpec, projections
 from .state import SlotManager, grown
 
-MIX = {"attention": 0, "delta": 1, "gla": 2, "wkv": 3, "latent": 4}
+MIX = {"attention": 0, "delta": 1, "gla": 2, "wkv": 3, "latent": 4, "ssd": 5}
 MLP = {"relu2": 1, "geglu": 2, "experts": 3, "clampglu": 4}
 KV_OWN, KV_LENDS, KV_BORROWS = 0, 1, 2
-REC_DELTA, REC_GLA, REC_WKV = 0, 1, 2
-REC = {MIX["delta"]: REC_DELTA, MIX["gla"]: REC_GLA, MIX["wkv"]: REC_WKV}
+REC_DELTA, REC_GLA, REC_WKV, REC_SSD = 0, 1, 2, 3
+REC = {MIX["delta"]: REC_DELTA, MIX["gla"]: REC_GLA, MIX["wkv"]: REC_WKV, MIX["ssd"]: REC_SSD}
+SCORE = {"sigmoid": 0, "softmax": 1}
+ACT = {"silu_gate": 0, "relu2": 1}
 LATENT_RECORDS = 64 << 20  # bytes of softmax records of a latent attention's key splits
 
 
@@ -44,6 +47,18 @@ def _pad16(n: int) -> int:
 
 def _pad128(n: int) -> int:
     return (n + 127) // 128 * 128
+
+
+def _slowed(f: float, factor: float, low: float, high: float, original: float) -> float:
+    """A rotation's turns per position for longer contexts: those with more than `high` full turns in the original length stay, those with fewer
+    than `low` are divided by `factor`, in between the two are mixed."""
+    turns = original * f / (2 * math.pi)
+    if turns > high:
+        return f
+    if turns < low:
+        return f / factor
+    keep = (turns - low) / (high - low)
+    return (1 - keep) * f / factor + keep * f
 
 
 class HybridEngine:
@@ -81,13 +96,15 @@ class HybridEngine:
             return ops.repack_bf16(w, pair, 1 if pair is None else 2)
         return (w if pair is None else torch.cat([w, pair])).contiguous()
 
-    def _proj(self, w: torch.Tensor, pair: Optional[torch.Tensor] = None) -> Proj:
+    def _proj(self, w: torch.Tensor, pair: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> Proj:
         """A weight [N, K] with its rows padded to a multiple of 16 (zero rows: the padding columns of every buffer stay zero)."""
         N, K = w.shape
+        if bias is not None:
+            bias = torch.nn.functional.pad(bias.float(), (0, _pad16(N) - N))
         n = _pad16(N)
         if n != N:
             w, pair = (t if t is None else torch.cat([t, t.new_zeros((n - N, K))]) for t in (w, pair))
-        return Proj(self._own(self._stream(w, pair)), n, K)
+        return Proj(self._own(self._stream(w, pair)), n, K, None if bias is None else self._f32(bias))
 
     def _norm(self, name: str) -> int:
         """A norm's weight; f32 models hold what is multiplied by, bf16 models the stored weight (their kernels add norm_add)."""
@@ -99,8 +116,15 @@ class HybridEngine:
         T, a = self.weights, ExpertsArgs()
         a.dtype, a.width, a.experts, a.top = nat.dtype_code(self.dtype), self.cfg.width, f.experts, f.top
         a.ff, a.ff_shared, a.scale = f.ff, f.ff_shared, f.scale
-        a.router = self._own(self._stream(T[p + "router"]))
-        up = [self._stream(T[f"{p}e{e}.gate"], T[f"{p}e{e}.up"]) for e in range(f.experts)]
+        a.score, a.act, a.identity, a.groups, a.keep_groups = SCORE[f.score], ACT[f.act], f.identity, f.groups, f.keep_groups
+        if f.score == "softmax":
+            a.correction = self._f32(T[p + "correction"])
+        if not self.cfg.design.sandwich:
+            a.router = self._own(self._stream(T[p + "router"]))
+        if f.act == "relu2":
+            up = [self._stream(T[f"{p}e{e}.up"]) for e in range(f.experts)]
+        else:
+            up = [self._stream(T[f"{p}e{e}.gate"], T[f"{p}e{e}.up"]) for e in range(f.experts)]
         before = self.weight_bytes
         a.up = self._own(torch.stack(up))
         a.down = self._own(torch.stack([self._stream(T[f"{p}e{e}.down"]) for e in range(f.experts)]))
@@ -133,18 +157,20 @@ class HybridEngine:
             L.norm1 = self._norm(p + "norm1")
             # one stacked projection, every piece padded to 16 columns
             off, parts = {}, []
-            for name in projections(m):
-                w = T[x + name]
+            weights, biases = self._pieces(x, m)
+            for name, w in zip(projections(m), weights):
                 off[name] = sum(q.shape[0] for q in parts)
                 pad = _pad16(w.shape[0]) - w.shape[0]
                 parts.append(torch.cat([w, w.new_zeros((pad, w.shape[1]))]) if pad else w)
             if m.type == "wkv":
                 self._token_shift(L, x, parts, off)
+            elif cfg.design.sandwich:
+                self._sandwich(L, p, spec, parts, biases)
             else:
                 setattr(L, "in", self._proj(torch.cat(parts)))
             if cfg.design.parallel:
                 self._parallel(L, p, spec)
-            else:
+            elif not cfg.design.sandwich:
                 L.out = self._proj(T[x + "o"])
             if spec.mlp is not None and not cfg.design.parallel:
                 L.norm2 = self._norm(p + "norm2")
@@ -168,16 +194,26 @@ class HybridEngine:
                     a.slope = self._f32(torch.tensor([2.0 ** (-8.0 * (h + 1) / m.heads) for h in range(m.heads)], dtype=torch.float64, device=self.device))
                 if m.rot_dims:
                     a.inv_freq = self._inv_freq(m)
+                a.softcap = m.softcap
+                if m.qk_norm:
+                    turn = self._turned(m)
+                    a.q_norm, a.k_norm = (self._f32(T[x + n][turn]) for n in ("q.norm", "k.norm"))
+                if m.v_mix and i != cfg.first_values():
+                    a.v_mix = float(T[x + "vmix"])
             elif m.type == "latent":
                 self._latent(L, x, m, off)
             else:
                 r = L.rec
                 r.kind = REC[L.mixer]
                 r.heads, r.kv_heads, r.dim, r.vdim = m.heads, m.kv_heads, m.dim, m.vdim
-                r.off_q, r.off_k, r.off_v, r.off_g = off["r" if m.type == "wkv" else "q"], off["k"], off["v"], off["g"]
+                names = {"wkv": "rkvg", "ssd": "CBxz"}.get(m.type, "qkvg")
+                r.off_q, r.off_k, r.off_v, r.off_g = (off[n] for n in names)
                 r.q_scale, r.eps, r.unit_eps = m.dim ** -0.5, cfg.eps, 1e-6
-                r.head_norm = self._f32(T[x + "norm"])
-                if m.type == "wkv":
+                if m.type != "ssd":
+                    r.head_norm = self._f32(T[x + "norm"])
+                if m.type == "ssd":
+                    self._state_space(r, x, m, off)
+                elif m.type == "wkv":
                     r.q_scale, r.norm_ld, r.bonus = 1.0, m.vdim, self._f32(T[x + "u"])
                     r.off_a, r.rank = off["w1"], T[x + "w1"].shape[0]
                     r.a2, r.a2_bias = self._f32(T[x + "w2"]), self._f32(T[x + "w0"])
@@ -204,6 +240,16 @@ class HybridEngine:
                 self.layers[r].kv_lender, self.layers[j].kv_last = j, r
                 self.layers[r].attn.role, self.layers[j].attn.role = KV_BORROWS, KV_LENDS
                 self.spans[j] = tuple(map(max, self.spans[j], self.spans[r]))
+        first = cfg.first_values()
+        if first is not None and first in runs:  # (its projections outlive the layer: the others read its values from them)
+            lender, own = self.layers[runs.index(first)], getattr(layers[first], "in")
+            self._first_rows = self._buf(self.max_rows * own.N, self.dtype)
+            lender.proj_rows = ptr(self._first_rows)
+            for r, i in enumerate(runs):
+                if cfg.layers[i].mixer.v_mix and i != first:
+                    a = self.layers[r].attn
+                    a.v_first = lender.proj_rows + lender.attn.off_v * self._first_rows.element_size()
+                    a.ld_v_first = own.N
         M = self.m = HybridModel()
         M.n_runs, M.dtype, M.norm_dtype = len(runs), nat.dtype_code(self.dtype), self.norm_dtype
         M.width, M.ldx, M.vocab, M.max_rows = cfg.width, _pad16(cfg.width), cfg.vocab_size, self.max_rows
@@ -214,12 +260,75 @@ class HybridEngine:
         M.head = self._proj(T["embed" if cfg.design.tied else "head"])
         M.ld_logits = M.head.N
         M.layers = self.layers
+        if cfg.design.sandwich:
+            M.embed_norm = self._norm("embed.norm")
         self.n_logits = cfg.vocab_size
 
     def _inv_freq(self, m: MixerSpec) -> int:
-        f = torch.tensor([m.rot_base ** (-2.0 * j / m.rot_dims) for j in range(m.rot_dims // 2)], dtype=torch.float64, device=self.device)
-        self._keep.append(f)
-        return ptr(f)
+        f = [m.rot_base ** (-2.0 * j / m.rot_dims) for j in range(m.rot_dims // 2)]
+        if m.rot_scaling is not None:
+            f = [_slowed(v, *m.rot_scaling) for v in f]
+        t = torch.tensor(f, dtype=torch.float64, device=self.device)
+        self._keep.append(t)
+        return ptr(t)
+
+    def _turned(self, m: MixerSpec) -> torch.Tensor:
+        """Dimensions of a head in the kernels' order: the kernels turn neighbours, so the two halves are dealt out in turn.  Products of
+        queries and keys do not see the order."""
+        half = torch.arange(m.rot_dims // 2, device=self.device)
+        return torch.cat([torch.stack([half, half + m.rot_dims // 2], 1).flatten(), torch.arange(m.rot_dims, m.dim, device=self.device)])
+
+    def _pieces(self, x: str, m: MixerSpec) -> Tuple[List[torch.Tensor], Optional[List[torch.Tensor]]]:
+        """Weights and biases of a mixer's input projections, in the order of `projections`."""
+        T = self.weights
+        if m.type == "ssd":
+            hv, gk = m.heads * m.vdim, m.kv_heads * m.dim
+            return list(T[x + "in"].split([hv, hv, gk, gk, m.heads])), None
+        ws = [T[x + n] for n in projections(m)]
+        bs = [T[x + n + ".b"] for n in projections(m)] if m.biased else None
+        if m.type == "attention" and m.rot_halves and m.rot_dims:
+            turn = self._turned(m)
+            for j, n in enumerate(projections(m)):
+                if n in ("q", "k"):
+                    ws[j] = ws[j].view(-1, m.dim, ws[j].shape[1])[:, turn].reshape(ws[j].shape)
+                    if bs is not None:
+                        bs[j] = bs[j].view(-1, m.dim)[:, turn].reshape(-1)
+        return ws, bs
+
+    def _state_space(self, r, x: str, m: MixerSpec, off: Dict[str, int]) -> None:
+        T = self.weights
+        hv, gk = m.heads * m.vdim, m.kv_heads * m.dim
+        r.q_scale, r.off_a, r.taps = 1.0, off["dt"], m.taps
+        r.conv_v, r.conv_k, r.conv_q = (self._f32(t) for t in T[x + "conv"].split([hv, gk, gk]))
+        r.conv_bv, r.conv_bk, r.conv_bq = (self._f32(t) for t in T[x + "conv.b"].split([hv, gk, gk]))
+        r.a_log, r.dt_bias, r.skip = (self._f32(T[x + n]) for n in ("A_log", "dt_bias", "D"))
+
+    def _sandwich(self, L: HybridLayer, p: str, spec: LayerSpec, parts: List[torch.Tensor], biases: Optional[List[torch.Tensor]]) -> None:
+        """Sublayers between norms: the mixer's gate is one more piece of its input projection; the feed-forward's stands in a product with the router."""
+        T, W = self.weights, self.cfg.width
+        n = sum(w.shape[0] for w in parts)
+        bias = torch.zeros(n, device=self.device)
+        at = 0
+        for w, b in zip(parts, biases or ()):
+            bias[at:at + b.shape[0]] = b.float()
+            at += w.shape[0]
+        L.sandwich, L.gate_at = 1, n
+        setattr(L, "in", self._proj(torch.cat([*parts, T[p + "rg1"]]), bias=torch.cat([bias, T[p + "rg1.b"].float()])))
+        L.out = self._proj(T[p + "mix.o"])
+        L.ld_cat = _pad128(L.out.K)
+        key = (L.out.K, L.out.K)  # rows of one length share their buffer: the padding behind them stays zero
+        if key not in self._cats:
+            self._cats[key] = ptr(self._buf(self.max_rows * L.ld_cat, self.dtype))
+        L.cat = self._cats[key]
+        L.post1, L.average = self._norm(p + "norm1b"), self._f32(T[p + "dwa"])
+        if spec.mixer.type == "ssd":
+            L.out_norm, L.out_groups = ptr(T[p + "mix.norm"]), spec.mixer.norm_groups
+        if spec.mlp is not None:
+            pad = _pad16(W) - W
+            gate = torch.nn.functional.pad(T[p + "rg2"], (0, 0, 0, pad))
+            L.side = self._proj(torch.cat([gate, T[p + "mlp.router"]]),
+                                bias=torch.cat([T[p + "rg2.b"].float(), torch.zeros(pad + T[p + "mlp.router"].shape[0], device=self.device)]))
+            L.logits_at, L.post2 = W + pad, self._norm(p + "norm2b")
 
     def _token_shift(self, L: HybridLayer, x: str, parts: List[torch.Tensor], off: Dict[str, int]) -> None:
         """Input projections that read a mix of their own each; bf16: those of one size as one stream, where its parts are whole tiles."""
@@ -319,10 +428,19 @@ class HybridEngine:
         M.att = ptr(self._buf(R * M.ld_att, self.dtype))
         f32 = self.dtype == torch.float32
         M.hid = ptr(self._buf(R * max([l.up.N * (3 if f32 and l.mlp in (MLP["geglu"], MLP["clampglu"]) else 1) for l in ls], default=16), self.dtype))
-        if self.dtype == torch.float32:
-            M.xn, M.tmp = ptr(self._buf(R * M.ld_n, torch.float32)), ptr(self._buf(R * M.ldx, torch.float32))
+        sandwich = cfg.design.sandwich
+        if f32 or sandwich:
+            M.tmp = ptr(self._buf(R * M.ldx, torch.float32))
+        if sandwich:
+            M.stream = ptr(self._buf((M.n_runs + 1) * R * M.ldx, torch.float32))
+            M.ld_side = max([l.side.N for l in ls], default=16)
+            M.side = ptr(self._buf(R * M.ld_side, torch.float32))
+            M.ld_mixed = max([_pad16(l.out.K) for l in ls if l.mixer == MIX["ssd"]], default=16)
+            M.mixed = ptr(self._buf(R * M.ld_mixed if any(l.mixer == MIX["ssd"] for l in ls) else 1, torch.float32))
+        if f32:
+            M.xn = ptr(self._buf(R * M.ld_n, torch.float32))
         else:
-            K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down, l.latent.uq)])  # (K = 0: not there)
+            K = max([M.head.K] + [q.K for l in ls for q in (getattr(l, "in"), l.out, l.up, l.down, l.latent.uq, l.side)])  # (K = 0: not there)
             n = int(lib().mi355_linear_gemm_workspace_bytes(R, _pad128(K)))
             M.gemm_ws, M.gemm_ws_bytes = ptr(self._buf(n, torch.uint8)), n
             M.xb = ptr(self._buf(R * M.ld_n, torch.bfloat16))
@@ -416,7 +534,7 @@ class HybridEngine:
                 e = l.rec
                 st = grown(old[0], (n, e.heads, e.dim, e.vdim), torch.float32, dev)
                 cv = None
-                if e.kind == REC_DELTA:
+                if e.kind in (REC_DELTA, REC_SSD):
                     cv = grown(old[1], (n, e.taps, 2 * e.kv_heads * e.dim + e.heads * e.vdim), self.dtype, dev)
                     e.conv_ring = ptr(cv)
                 if l.n_mix:

@@ -29,7 +29,7 @@ def _llama(config: dict, dtype: torch.dtype, device, quantize: Optional[str] = N
         return LLaMA(LLaMAConfig(**kw)).eval()
 
 
-FAMILIES: Dict[str, Callable] = {"LLaMA": _llama, "Sekulorn": _hybrid, "Kovalorn": _hybrid, "Kudazen": _hybrid}
+FAMILIES: Dict[str, Callable] = {"LLaMA": _llama, "Sekulorn": _hybrid, "Kovalorn": _hybrid, "Kudazen": _hybrid, "Gurolix": _hybrid}
 
 
 def build_model(config: dict, dtype: torch.dtype = torch.bfloat16, device="cuda", **kw):
