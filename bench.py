@@ -72,7 +72,7 @@ def parse():
                     help="instead of the headline workload: prompt and decode rates of a layered hybrid model (Sekulorn design) of these "
                          "widths beside an unquantised LLaMA of the same width and layer count (random weights)")
     ap.add_argument("--hybrid-designs", default="Sekulorn", metavar="NAME[,NAME]",
-                    help="the designs of --hybrid (Sekulorn, Kovalorn, Kudazen: width, layers and weights that a token uses per layer are the same)")
+                    help="the designs of --hybrid (Sekulorn, Kovalorn, Kudazen, Gurolix: width, layers and weights that a token uses per layer are the same)")
     ap.add_argument("--hybrid-layers", type=int, default=8)
     ap.add_argument("--hybrid-batches", default="1,16,64")
     ap.add_argument("--hybrid-only", default="both", choices=["both", "hybrid", "llama"], help="(profiling) one side of --hybrid")

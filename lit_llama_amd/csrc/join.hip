@@ -11,14 +11,24 @@ constexpr int kThreads = 512;
 __device__ __forceinline__ float sigmoid_fast(float v) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(v * -1.44269504088896340736f)); }
 __device__ __forceinline__ float square_sum(f32x4 v) { return (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
 
+// sum over the workgroup (DPP steps and one LDS pass); `red`: 8 floats that nobody else uses
+__device__ __forceinline__ float sum_all(float v, float* red) {
+    v = group_sum(v, 64);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float s = 0.f;
+    for (int w = 0; w < (int)(blockDim.x >> 6); ++w) s += red[w];
+    return s;
+}
+
 // One row per workgroup, four consecutive values per thread, H times; the row stays in registers
 template <typename T, int H>
 __global__ __launch_bounds__(kThreads) void join_kernel(const mi355_join_args p) {
-    __shared__ float red[32];
+    __shared__ float red[2][kThreads / 64];
     const int m = blockIdx.x, nt = blockDim.x, W = p.width;
     const T* emb = p.embed != nullptr ? (const T*)p.embed + (int64_t)min(max(p.tokens[m], 0), p.vocab - 1) * W : nullptr;
     const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-    f32x4 u[H], x[H], g[H], post[H], next[H];
+    f32x4 u[H], x[H], g[H], post[H], next[H], before[H];
     auto at = [&](int i) { return 4 * ((int)threadIdx.x + nt * i); };
     // (every request of the row in front of the first sum)
 #pragma unroll
@@ -34,6 +44,15 @@ __global__ __launch_bounds__(kThreads) void join_kernel(const mi355_join_args p)
         post[i] = in && p.post != nullptr ? get4((const T*)p.post + k) + p.norm_add : zero;
         next[i] = in && p.next != nullptr ? get4((const T*)p.next + k) + p.norm_add : zero;
     }
+#pragma unroll
+    for (int i = 0; i < H; ++i) before[i] = zero;
+#pragma unroll(H > 2 ? 2 : 4)
+    for (int j = 0; j < p.n_stream; ++j) {
+        const float w = p.average[j];
+        const float* row = p.stream + j * p.stream_stride + (int64_t)m * p.ldx;
+#pragma unroll
+        for (int i = 0; i < H; ++i) before[i] += w * (at(i) < W ? *(const f32x4*)(row + at(i)) : zero);
+    }
     if (p.gate != nullptr) {
 #pragma unroll
         for (int i = 0; i < H; ++i)
@@ -44,7 +63,7 @@ __global__ __launch_bounds__(kThreads) void join_kernel(const mi355_join_args p)
         float ss = 0.f;
 #pragma unroll
         for (int i = 0; i < H; ++i) ss += square_sum(u[i]);
-        const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)W + p.eps);
+        const float r = 1.0f / sqrtf(sum_all(ss, red[0]) / (float)W + p.eps);
 #pragma unroll
         for (int i = 0; i < H; ++i) u[i] = u[i] * r * post[i];
     }
@@ -58,14 +77,7 @@ __global__ __launch_bounds__(kThreads) void join_kernel(const mi355_join_args p)
     if (p.n_stream > 0) {
         const float own = p.average[p.n_stream];
 #pragma unroll
-        for (int i = 0; i < H; ++i) x[i] *= own;
-#pragma unroll 4
-        for (int j = 0; j < p.n_stream; ++j) {
-            const float w = p.average[j];
-            const float* row = p.stream + j * p.stream_stride + (int64_t)m * p.ldx;
-#pragma unroll
-            for (int i = 0; i < H; ++i) x[i] += w * (at(i) < W ? *(const f32x4*)(row + at(i)) : zero);
-        }
+        for (int i = 0; i < H; ++i) x[i] = before[i] + own * x[i];
     }
 #pragma unroll
     for (int i = 0; i < H; ++i)
@@ -74,7 +86,7 @@ __global__ __launch_bounds__(kThreads) void join_kernel(const mi355_join_args p)
         float ss = 0.f;
 #pragma unroll
         for (int i = 0; i < H; ++i) ss += at(i) < W ? square_sum(x[i]) : 0.f;
-        const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)W + p.eps);
+        const float r = 1.0f / sqrtf(sum_all(ss, red[1]) / (float)W + p.eps);
 #pragma unroll
         for (int i = 0; i < H; ++i)
             if (at(i) < W) put4((T*)p.h + (int64_t)m * p.ldh + at(i), x[i] * r * next[i]);

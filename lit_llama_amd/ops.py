@@ -623,12 +623,15 @@ def window_attention(proj: torch.Tensor, batch: PackedBatch, kring: torch.Tensor
                      partials: Optional[torch.Tensor] = None, keep: int = 0, kept: int = 0, gate_values: bool = False,
                      unit_eps: Optional[float] = None, sink: Optional[torch.Tensor] = None, role: str = "own",
                      kv_rows: Optional[torch.Tensor] = None, chunked: bool = False, head_scale: Optional[torch.Tensor] = None,
-                     slope: Optional[torch.Tensor] = None, unit_v_eps: Optional[float] = None) -> torch.Tensor:
+                     slope: Optional[torch.Tensor] = None, unit_v_eps: Optional[float] = None, q_norm: Optional[torch.Tensor] = None,
+                     k_norm: Optional[torch.Tensor] = None, softcap: float = 0.0, v_first: Optional[torch.Tensor] = None,
+                     v_mix: float = 0.0) -> torch.Tensor:
     """mi355_window_attention: proj [rows, ld] (k prepared in place by prompt steps), rings [slots, kv_heads, kept + ring, dim | vdim]
     (written).  `unit_eps`: q and k over their root mean square.  `role` own | lends | borrows: a lender fills `kv_rows` in a prompt step and
     its cache is written by `window_cache_write`; a borrower has neither key nor value columns.  `chunked`: the window is a chunk of the
     sequence; `head_scale`, `slope`: per head a factor of the scores and what is taken off per position of distance; `unit_v_eps`: v over its
-    root mean square."""
+    root mean square; `q_norm`, `k_norm` [dim] f32: factors behind unit_eps; `softcap`: bound of the scores; `v_first` [rows, kv_heads * vdim]:
+    values that count v_mix."""
     y, a = _window_args(proj, batch, kring, vring, heads, scale, window, off_q, off_k, off_v, off_g, inv_freq, path, partials, keep, kept,
                         gate_values, unit_eps, sink, role, kv_rows)
     a.chunked = int(chunked)
@@ -638,6 +641,12 @@ def window_attention(proj: torch.Tensor, batch: PackedBatch, kring: torch.Tensor
     if unit_v_eps is not None:
         assert unit_eps is None or unit_eps == unit_v_eps
         a.unit_v, a.unit_eps = 1, unit_v_eps
+    for t in (q_norm, k_norm):
+        assert t is None or (t.dtype == torch.float32 and t.numel() == a.dim and t.is_contiguous())
+    a.q_norm, a.k_norm, a.softcap, a.v_mix = ptr(q_norm), ptr(k_norm), softcap, v_mix
+    if v_first is not None:
+        assert v_first.dtype == proj.dtype and v_first.shape == (batch.rows, a.kv_heads * a.vdim) and v_first.stride(1) == 1
+        a.v_first, a.ld_v_first = ptr(v_first), v_first.stride(0)
     check(lib().mi355_window_attention(C.byref(a), C.byref(batch.c), stream_ptr()), "mi355_window_attention")
     return y
 
@@ -682,55 +691,115 @@ def _window_args(proj, batch, kring, vring, heads, scale, window, off_q, off_k, 
     return y, a
 
 
-def experts(x: torch.Tensor, norm: torch.Tensor, router: torch.Tensor, weights, shared=None, *, top: int, scale: float, eps: float,
-            norm_add: float = 0.0, alpha: float = 1.0, path: int = 0) -> torch.Tensor:
-    """mi355_experts: x [rows, width] f32 -> x + alpha (experts + shared expert of its RMSNorm).  `weights`: per expert (gate, up, down), `shared`
-    the same or None, all of one dtype (bf16, f32) like `norm` and `router`."""
-    require_gpu(x, "experts")
-    rows, W = x.shape
-    dt = router.dtype
+def experts(x: Optional[torch.Tensor], norm: Optional[torch.Tensor], router: Optional[torch.Tensor], weights, shared=None, *, top: int, scale: float = 1.0,
+            eps: float = 0.0, norm_add: float = 0.0, alpha: float = 1.0, path: int = 0, score: str = "sigmoid", correction: Optional[torch.Tensor] = None,
+            groups: int = 0, keep_groups: int = 0, identity: int = 0, h: Optional[torch.Tensor] = None,
+            logits: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """mi355_experts: x [rows, width] f32 -> x + alpha (experts + shared expert of its RMSNorm).  `weights`: per expert (gate, up, down) or, squared ReLU,
+    (up, down), `shared` (gate, up, down) or None, all of one dtype (bf16, f32) like `norm` and `router`.  `score` sigmoid | softmax, the latter with a
+    `correction` of the choice (f32), a choice from the best `keep_groups` of `groups`, and `identity` outputs that are the row itself.  With `h`
+    [rows, width] (of that dtype) and its `logits` f32 in place of x, norm and router: alpha (experts) alone."""
+    first = x if h is None else h
+    require_gpu(first, "experts")
+    rows, W = first.shape
+    dt = weights[0][0].dtype
+    one = len(weights[0]) == 2
     ld = (W + 15) // 16 * 16
-    out = torch.zeros((rows, ld), dtype=torch.float32, device=x.device)
-    out[:, :W] = x
     stream = (lambda w, w1=None: repack_bf16(w, w1, 1 if w1 is None else 2)) if dt == torch.bfloat16 else (
         lambda w, w1=None: (w if w1 is None else torch.cat([w, w1])).contiguous())
-    keep = [norm.contiguous(), stream(router), torch.stack([stream(g, u) for g, u, _ in weights]), torch.stack([stream(d) for _, _, d in weights])]
+    keep = [torch.stack([stream(*w[:-1]) for w in weights]), torch.stack([stream(w[-1]) for w in weights])]
     a = nat.ExpertsArgs()
-    a.dtype, a.rows, a.width, a.experts, a.top = dtype_code(dt), rows, W, router.shape[0], top
+    a.dtype, a.rows, a.width, a.experts, a.top = dtype_code(dt), rows, W, len(weights), top
     a.ff, a.scale, a.eps, a.norm_add, a.alpha, a.path = weights[0][0].shape[0], scale, eps, norm_add, alpha, path
-    a.norm, a.norm_dtype = ptr(keep[0]), dtype_code(norm.dtype)
-    a.router, a.up, a.down = (ptr(t) for t in keep[1:4])
+    a.score, a.act, a.identity, a.groups, a.keep_groups = ("sigmoid", "softmax").index(score), int(one), identity, groups, keep_groups
+    a.up, a.down = (ptr(t) for t in keep)
+    if correction is not None:
+        assert correction.dtype == torch.float32 and correction.numel() == len(weights) + identity
+        a.correction = ptr(correction)
+    if h is None:
+        out = torch.zeros((rows, ld), dtype=torch.float32, device=first.device)
+        out[:, :W] = x
+        keep += [norm.contiguous(), stream(router)]
+        a.norm, a.norm_dtype, a.router = ptr(keep[2]), dtype_code(norm.dtype), ptr(keep[3])
+        a.x, a.ldx = ptr(out), ld
+    else:
+        assert h.dtype == dt and logits.dtype == torch.float32 and logits.shape == (rows, len(weights) + identity) and logits.stride(1) == 1
+        out = torch.full((rows, ld), float("nan"), dtype=torch.float32, device=first.device)
+        keep.append(torch.nn.functional.pad(h, (0, (W + 127) // 128 * 128 - W)))
+        a.h, a.ldh, a.logits, a.ld_logits, a.out, a.ld_out = ptr(keep[2]), keep[2].shape[1], ptr(logits), logits.stride(0), ptr(out), ld
     if shared is not None:
         keep += [stream(shared[0], shared[1]), stream(shared[2])]
-        a.ff_shared, a.shared_up, a.shared_down = shared[0].shape[0], ptr(keep[4]), ptr(keep[5])
-    a.x, a.ldx = ptr(out), ld
+        a.ff_shared, a.shared_up, a.shared_down = shared[0].shape[0], ptr(keep[-2]), ptr(keep[-1])
     n = int(lib().mi355_experts_scratch_bytes(C.byref(a)))
-    scratch = torch.full((n,), 255, dtype=torch.uint8, device=x.device)  # (NaNs in every format: nothing may read what no kernel wrote)
+    scratch = torch.full((n,), 255, dtype=torch.uint8, device=first.device)  # (NaNs in every format: nothing may read what no kernel wrote)
     a.scratch, a.scratch_bytes = ptr(scratch), n
     check(lib().mi355_experts(C.byref(a), stream_ptr()), "mi355_experts")
     return out[:, :W]
 
 
-def recurrent(kind: str, proj: torch.Tensor, batch: PackedBatch, state: torch.Tensor, *, off: dict, kv_heads: int, head_norm: torch.Tensor,
-              eps: float, conv_ring: Optional[torch.Tensor] = None, conv=None, a_log=None, dt_bias=None, a2=None, a2_bias=None,
-              tau: float = 1.0, path: int = 0, bonus: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """mi355_recurrent: `kind` delta | gla | wkv (`off` q: r, a: the decay's low-rank input; head_norm per channel), state [slots, heads, dim, vdim] f32 (updated), `off`: first columns of q, k, v, g, a (and b);
+def join_rows(x: Optional[torch.Tensor], t: Optional[torch.Tensor] = None, *, eps: float, tokens: Optional[torch.Tensor] = None,
+              embed: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, post: Optional[torch.Tensor] = None,
+              stream: Optional[torch.Tensor] = None, average: Optional[torch.Tensor] = None, next: Optional[torch.Tensor] = None,
+              norm_add: float = 0.0, dtype: torch.dtype = torch.bfloat16):
+    """mi355_join_rows: the sublayer rows t [rows, width] f32 (or the rows `tokens` of `embed`) behind their gate logits and norm join x f32; with `stream`
+    [n, rows, width] and `average` [n + 1] f32 their weighted average goes on.  Returns (x, the sum in front of the average, h = x behind the norm
+    `next` or None)."""
+    rows, W = (tokens.numel(), embed.shape[1]) if embed is not None else t.shape
+    dev = (embed if embed is not None else t).device
+    ldx, ldh = (W + 15) // 16 * 16, (W + 127) // 128 * 128
+    pad = lambda v: torch.nn.functional.pad(v.float(), (0, ldx - W)).contiguous()
+    xp = pad(x) if x is not None else torch.full((rows, ldx), float("nan"), dtype=torch.float32, device=dev)
+    keep = [xp]
+    a = nat.JoinArgs()
+    a.dtype, a.rows, a.width, a.eps, a.norm_add, a.x, a.ldx = dtype_code(dtype), rows, W, eps, norm_add, ptr(xp), ldx
+    if embed is not None:
+        assert embed.dtype == dtype and embed.is_contiguous() and tokens.dtype == torch.int32
+        a.tokens, a.embed, a.vocab = ptr(tokens), ptr(embed), embed.shape[0]
+    else:
+        keep.append(pad(t))
+        a.t, a.ldt = ptr(keep[-1]), ldx
+    if gate is not None:
+        keep.append(torch.nn.functional.pad(gate, (0, ldx - W)).contiguous())
+        a.gate, a.ld_gate, a.gate_dtype = ptr(keep[-1]), ldx, dtype_code(gate.dtype)
+    assert all(n is None or n.dtype == dtype for n in (post, next))
+    a.post, a.next = ptr(post), ptr(next)
+    out = torch.full_like(xp, float("nan"))
+    a.stream_out = ptr(out)
+    if average is not None:
+        keep.append(torch.stack([pad(v) for v in stream]))
+        a.stream, a.stream_stride, a.n_stream, a.average = ptr(keep[-1]), rows * ldx, len(stream), ptr(average)
+        assert average.dtype == torch.float32 and average.numel() == len(stream) + 1
+    h = torch.zeros((rows, ldh), dtype=dtype, device=dev)
+    a.h, a.ldh = ptr(h), ldh
+    check(lib().mi355_join_rows(C.byref(a), stream_ptr()), "mi355_join_rows")
+    assert not h[:, W:].any()
+    return xp[:, :W], out[:, :W], None if next is None else h[:, :W]
+
+
+def recurrent(kind: str, proj: torch.Tensor, batch: PackedBatch, state: torch.Tensor, *, off: dict, kv_heads: int, head_norm: Optional[torch.Tensor] = None,
+              eps: float = 0.0, conv_ring: Optional[torch.Tensor] = None, conv=None, a_log=None, dt_bias=None, a2=None, a2_bias=None,
+              tau: float = 1.0, path: int = 0, bonus: Optional[torch.Tensor] = None, conv_bias=None, skip: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """mi355_recurrent: `kind` delta | gla | wkv | ssd (f32 outputs, no head_norm; `conv_bias` like `conv`) (`off` q: r, a: the decay's low-rank input; head_norm per channel), state [slots, heads, dim, vdim] f32 (updated), `off`: first columns of q, k, v, g, a (and b);
     `conv`: the (q, k, v) taps of the delta rule, f32 [channels, taps]."""
     require_gpu(proj, "recurrent")
     _, H, dim, vdim = state.shape
-    y = torch.zeros((batch.rows, H * vdim), dtype=proj.dtype, device=proj.device)
+    y = torch.zeros((batch.rows, H * vdim), dtype=torch.float32 if kind == "ssd" else proj.dtype, device=proj.device)
     r = nat.RecurrentArgs()
-    r.kind, r.dtype = ("delta", "gla", "wkv").index(kind), dtype_code(proj.dtype)
+    r.kind, r.dtype = ("delta", "gla", "wkv", "ssd").index(kind), dtype_code(proj.dtype)
     r.proj, r.ld = ptr(proj), proj.shape[1]
     r.heads, r.kv_heads, r.dim, r.vdim = H, kv_heads, dim, vdim
     r.off_q, r.off_k, r.off_v, r.off_g, r.off_a = (off[n] for n in "qkvga")
     r.q_scale, r.eps, r.unit_eps, r.path = dim ** -0.5, eps, 1e-6, path
     r.head_norm, r.state, r.y, r.ldy = ptr(head_norm), ptr(state), ptr(y), y.shape[1]
-    if kind == "delta":
+    if kind in ("delta", "ssd"):
         assert conv_ring.dtype == proj.dtype and conv_ring.shape[2] == 2 * kv_heads * dim + H * vdim
-        r.off_b, r.taps = off["b"], conv[0].shape[1]
+        r.off_b, r.taps = off.get("b", 0), conv[0].shape[1]
         r.conv_q, r.conv_k, r.conv_v = (ptr(t) for t in conv)
         r.a_log, r.dt_bias, r.conv_ring = ptr(a_log), ptr(dt_bias), ptr(conv_ring)
+        if kind == "ssd":
+            r.q_scale, r.skip = 1.0, ptr(skip)
+            if conv_bias is not None:
+                r.conv_bq, r.conv_bk, r.conv_bv = (ptr(t) for t in conv_bias)
     else:
         r.rank, r.inv_tau, r.a2, r.a2_bias = a2.shape[1], 1.0 / tau, ptr(a2), ptr(a2_bias)
         if kind == "wkv":

@@ -336,7 +336,24 @@ def parallel_bench_config(width: int, n_layer: int, vocab: int = 32000, chunk: i
     return {"architecture": "Kudazen", "layers": layers, "norm": {"eps": 1e-5, "groups": 2}, "vocab": vocab, "width": width}
 
 
-HYBRID_BENCH = {"Sekulorn": hybrid_bench_config, "Kovalorn": experts_bench_config, "Kudazen": parallel_bench_config}
+def sandwich_bench_config(width: int, n_layer: int, vocab: int = 32000, experts: int = 32, identity: int = 8, top: int = 8) -> dict:
+    """A Gurolix configuration whose tokens use about as many weights per layer as a LLaMA of the same width: state-space layers (twice the width, heads
+    of 64, states of 128, 8 groups) in turn with attention layers of both kinds (heads of 128, grouped by 4), experts of an eighth of the LLaMA's hidden
+    size."""
+    heads = width // 128
+    hidden = LLaMAConfig(n_embd=width, n_head=heads).n_hidden
+    ssd = ("mamba2", {"heads": 2 * width // 64, "groups": 8, "state": 128, "vdim": 64, "conv": 4, "norm_groups": 8})
+    att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "v_mix": True}
+    scaling = {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}
+    mixers = [ssd, ("attention", {**att, "rot": {"base": 1e4, "dims": 128}}), ssd,
+              ("attention_2", {**att, "rot": {"base": 5e5, "dims": 128, "scaling": scaling}, "softcap": 30.0})]
+    moe = {"kind": "moe", "expert": {"ff": (hidden // 8 + 127) // 128 * 128},
+           "router": {"experts": experts, "identity": identity, "top": top, "groups": {"count": 4, "keep": 2}}}
+    return {"architecture": "Gurolix", "layers": [{"type": t, "mixer": m, "mlp": moe} for t, m in (mixers[i % 4] for i in range(n_layer))],
+            "norm": {"eps": 1e-5}, "vocab": vocab, "width": width}
+
+
+HYBRID_BENCH = {"Sekulorn": hybrid_bench_config, "Kovalorn": experts_bench_config, "Kudazen": parallel_bench_config, "Gurolix": sandwich_bench_config}
 
 
 def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: torch.dtype = torch.bfloat16, rank: int = 16):
@@ -351,7 +368,9 @@ def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: tor
     for name, shape in tensor_shapes(cfg, ranks).items():
         leaf = name.split(".", 1)[-1]
         t = torch.randn(shape, generator=gen, device=device, dtype=torch.float32)
-        if leaf in ("norm1", "norm2", "norm") or leaf.endswith(".norm"):
+        if leaf.startswith("mix.") and leaf.endswith(".norm") and cfg.design.sandwich:
+            t = 1.0 + 0.1 * t  # (the mixers' own norms are factors)
+        elif leaf in ("norm1", "norm2", "norm", "norm1b", "norm2b") or leaf.endswith(".norm"):
             t = 1.0 - cfg.design.norm_add + 0.1 * t
         elif leaf.endswith("sink"):
             t = t + 1.0
@@ -368,6 +387,15 @@ def make_hybrid_state_dict(config: dict, seed: int = 0, device="cpu", dtype: tor
             t[:, -1] += 0.7
         elif leaf.endswith("A_log"):
             t = t * 0.3 - 2.0
+        elif leaf.endswith("vmix"):
+            t = 0.5 + 0.2 * t
+        elif leaf == "dwa":  # (mostly the layer's own result)
+            t = 0.3 * t * shape[-1] ** -0.5
+            t[-1] += 1.0
+        elif leaf.endswith(("mix.D", "correction")):
+            t = 0.3 * t + 1.0 if leaf.endswith("mix.D") else 0.03 * t
+        elif leaf in ("rg1.b", "rg2.b", "mix.q.b", "mix.k.b", "mix.v.b", "mix.conv.b"):
+            t = 0.5 * t
         elif leaf.endswith(("dt_bias", "a2.b")):
             t = t * 0.5 + (2.0 if leaf.endswith("a2.b") else 0.0)
         elif name != "embed":

@@ -1,0 +1,174 @@
+"""Host side of the Gurolix design: configuration, registry, weight names, order of dimensions; and the plain restatement in oracle/gurolix.py
+checked against closed forms of its mechanisms."""
+import copy
+import json
+import math
+
+import pytest
+import torch
+
+from lit_llama_amd import registry, synth
+from lit_llama_amd.hybrid import HybridConfig, HybridLM, projections, tensor_shapes
+from oracle import gurolix as O
+
+MOE = {"kind": "moe", "expert": {"ff": 20}, "router": {"experts": 5, "top": 3, "identity": 3, "groups": {"count": 4, "keep": 2}}}
+SCALING = {"factor": 5.0, "low": 0.5, "high": 3.0, "original": 70}
+CONFIG = {
+    "architecture": "Gurolix", "vocab": 90, "width": 36, "norm": {"eps": 3e-4},
+    "layers": [
+        {"type": "attention", "mixer": {"heads": 4, "kv_heads": 2, "dim": 12, "vdim": 10, "rot": {"base": 500.0, "dims": 8}, "scale": 0.3, "v_mix": True}, "mlp": MOE},
+        {"type": "mamba2", "mixer": {"heads": 6, "groups": 3, "state": 8, "vdim": 7, "conv": 5, "norm_groups": 2}, "mlp": None},
+        {"type": "attention_2", "mixer": {"heads": 3, "kv_heads": 1, "dim": 6, "vdim": 9, "rot": {"base": 80.0, "dims": 6, "scaling": SCALING}, "scale": 0.4,
+                                          "softcap": 2.5}, "mlp": {**MOE, "router": {"experts": 4, "top": 2}}},
+        {"type": "attention_2", "mixer": {"heads": 2, "kv_heads": 2, "dim": 14, "vdim": 10, "rot": {"base": 80.0, "dims": 4}, "scale": 0.4, "softcap": 9.0,
+                                          "v_mix": True}, "mlp": None},
+    ],
+}
+
+
+def test_configuration_reads_every_constant():
+    c = HybridConfig.from_dict(CONFIG)
+    a, s, b, d = (x.mixer for x in c.layers)
+    assert (c.vocab_size, c.width, c.eps, c.norm_groups, c.residual_mult, c.logit_scale) == (90, 36, 3e-4, 0, 1.0, 1.0)
+    assert (a.heads, a.kv_heads, a.dim, a.vdim, a.scale, a.rot_dims, a.rot_base, a.window) == (4, 2, 12, 10, 0.3, 8, 500.0, 1 << 30)
+    assert a.unit_qk and a.qk_norm and a.biased and a.rot_halves and a.v_mix and not a.gated and a.softcap == 0 and a.rot_scaling is None
+    assert (s.heads, s.kv_heads, s.dim, s.vdim, s.taps, s.norm_groups) == (6, 3, 8, 7, 5, 2)
+    assert not b.unit_qk and not b.qk_norm and b.biased and b.softcap == 2.5 and b.rot_scaling == (5.0, 0.5, 3.0, 70.0) and not b.v_mix and d.v_mix
+    f, g = c.layers[0].mlp, c.layers[2].mlp
+    assert (f.ff, f.experts, f.identity, f.top, f.groups, f.keep_groups, f.scale, f.act, f.score) == (20, 5, 3, 3, 4, 2, 1.0, "relu2", "softmax")
+    assert (g.experts, g.identity, g.top, g.groups, g.keep_groups) == (4, 0, 2, 1, 1) and c.layers[1].mlp is None
+    assert c.design.sandwich and not c.design.parallel and not c.design.tied and c.design.norm_add == 1.0
+    assert c.first_values() == 0 and projections(a) == ("q", "k", "v") and projections(s) == ("z", "x", "B", "C", "dt")
+
+
+@pytest.mark.parametrize("path,value", [
+    (("layers", 0, "type"), "gla"), (("layers", 0, "mixer", "softcap"), 3.0), (("layers", 0, "mixer", "mask"), {"size": 4}), (("layers", 0, "mixer", "rot", "dims"), 5),
+    (("layers", 0, "mixer", "rot", "dims"), 14), (("layers", 0, "mixer", "rot", "scaling"), SCALING), (("layers", 0, "mixer", "kv_heads"), 3),
+    (("layers", 1, "mixer", "groups"), 4), (("layers", 1, "mixer", "norm_groups"), 5), (("layers", 1, "mixer", "kv_heads"), 3), (("layers", 0, "mlp", "kind"), "dense"),
+    (("layers", 0, "mlp", "shared"), {"ff": 3}), (("layers", 0, "mlp", "router", "scale"), 2.0), (("layers", 0, "mlp", "router", "top"), 5),
+    (("layers", 0, "mlp", "router", "groups", "count"), 3), (("layers", 0, "mlp", "router", "groups", "keep"), 5), (("layers", 3, "mixer", "vdim"), 9),
+    (("layers", 2, "weights_of"), 0), (("norm", "groups"), 2), (("loop",), {"start": 0, "stop": 2, "times": 2})])
+def test_what_the_framework_does_not_know_is_refused(path, value):
+    c = copy.deepcopy(CONFIG)
+    at = c
+    for k in path[:-1]:
+        at = at[k]
+    at[path[-1]] = value
+    with pytest.raises(ValueError):
+        HybridConfig.from_dict(c)
+
+
+def test_folder_loads_and_is_checked(tmp_path):
+    from safetensors.torch import save_file
+
+    sd = synth.make_hybrid_state_dict(CONFIG)
+    assert {"embed.norm", "l0.norm1b", "l0.norm2b", "l0.rg2.b", "l0.mix.q.norm", "l0.mix.v.b", "l0.mix.vmix", "l1.mix.conv.b", "l1.mix.D", "l0.mlp.e4.down", "head"} <= set(sd)
+    assert not {"l1.norm2", "l1.rg2", "l2.mix.q.norm", "l2.mix.vmix", "l0.mlp.e5.up", "l0.mlp.e0.gate"} & set(sd)
+    assert sd["l1.mix.in"].shape == (42 + 42 + 24 + 24 + 6, 36) and sd["l1.mix.conv"].shape == (90, 5) and sd["l0.mlp.router"].shape == (8, 36)
+    assert sd["l0.mix.vmix"].shape == () and [tuple(sd[f"l{i}.dwa"].shape) for i in range(4)] == [(2,), (3,), (4,), (5,)]
+    assert set(tensor_shapes(HybridConfig.from_dict(CONFIG), {})) == set(sd)
+    (tmp_path / "config.json").write_text(json.dumps(CONFIG))
+    save_file(sd, str(tmp_path / "model.safetensors"))
+    m = registry.load_model(tmp_path, torch.float32, "cpu")
+    assert isinstance(m, HybridLM) and all(torch.equal(m.tensors[n], t.float()) for n, t in sd.items())
+    for bad in ("missing", "extra", "shape"):
+        d = dict(sd)
+        if bad == "missing":
+            del d["l0.mlp.correction"]
+        elif bad == "extra":
+            d["l1.norm2"] = torch.zeros(36)
+        else:
+            d["l2.dwa"] = torch.zeros(3)
+        with pytest.raises(ValueError):
+            registry.build_model(CONFIG, device="cpu").load_state_dict(d)
+
+
+def test_slowed_rotations_match_the_restatement():
+    from lit_llama_amd.hybrid_engine import _slowed
+
+    rot = {"base": 80.0, "dims": 12, "scaling": SCALING}
+    plain = [80.0 ** (-2 * i / 12) for i in range(6)]
+    got = [_slowed(f, 5.0, 0.5, 3.0, 70.0) for f in plain]
+    assert torch.allclose(torch.tensor(got, dtype=torch.float64), O.frequencies(rot))
+    assert got[0] == plain[0] and abs(got[-1] - plain[-1] / 5) < 1e-12  # fast ones stay, slow ones are divided
+    assert any(f / 5 < g < f for f, g in zip(plain, got))
+
+
+# ---------------------------------------------------------------------------------------- the restatement itself
+def test_oracle_rotation_pairs_halves():
+    x = torch.zeros((4, 1, 6)).double()
+    x[:, 0, 1] = 1.0  # turns with dimension 1 + 2
+    f = O.frequencies({"base": 9.0, "dims": 4})
+    assert torch.allclose(f, torch.tensor([1.0, 1 / 3]).double())
+    y = O.rotate_halves(x, {"base": 9.0, "dims": 4})[:, 0]
+    t = torch.arange(4).double() / 3
+    assert torch.allclose(y[:, 1], torch.cos(t)) and torch.allclose(y[:, 3], torch.sin(t)) and not y[:, [0, 2, 4, 5]].any()
+
+
+def test_oracle_bounded_scores():
+    q = torch.ones((3, 1, 1)).double()
+    k = torch.tensor([1e6, -1e6, 0.0]).double().view(3, 1, 1)
+    v = torch.tensor([1.0, 2.0, 4.0]).double().view(3, 1, 1)
+    out = O.attend(q, k, v, 1.0, math.log(2))[:, 0, 0]  # scores log 2, -log 2, 0
+    assert torch.allclose(out, torch.tensor([1.0, (2 + 1) / 2.5, (2 + 1 + 4) / 3.5]).double())
+    assert torch.allclose(O.attend(q, 0 * k, v, 1.0, None)[:, 0, 0], torch.tensor([1.0, 1.5, 7 / 3]).double())
+
+
+def test_oracle_state_space_is_a_weighted_sum_of_the_past():
+    gen = torch.Generator().manual_seed(3)
+    rnd = lambda *s: torch.randn(s, dtype=torch.float64, generator=gen)
+    x, B, Cq, dt, a_log, D = rnd(7, 4, 3), rnd(7, 2, 5), rnd(7, 2, 5), rnd(7, 4).exp(), rnd(4), rnd(4)
+    out = O.state_space(x, B, Cq, dt, a_log, D)
+    want = torch.zeros_like(out)
+    for h in range(4):
+        for t in range(7):
+            for j in range(t + 1):
+                decay = torch.exp(-torch.exp(a_log[h]) * dt[j + 1:t + 1, h].sum())
+                want[t, h] += decay * dt[j, h] * (Cq[t, h // 2] @ B[j, h // 2]) * x[j, h]
+            want[t, h] += D[h] * x[t, h]
+    assert torch.allclose(out, want)
+
+
+def test_oracle_convolution_has_its_current_row_last():
+    x = torch.arange(1, 6).double().view(5, 1)
+    taps, bias = torch.tensor([[100.0, 10.0, 1.0]]).double(), torch.tensor([0.5]).double()
+    assert torch.allclose(O.short_conv(x, taps, bias)[:, 0], torch.tensor([1.5, 12.5, 123.5, 234.5, 345.5]).double())
+
+
+def test_oracle_router():
+    z = torch.tensor([0.0, 1.0, 2.0, 3.0, 2.5, -1.0]).double()
+    s = torch.softmax(z, -1)
+    none = torch.zeros(6).double()
+    ids, w = O.route(z, none, 3, 1, 1)
+    assert ids == [3, 4, 2] and torch.allclose(w, s[[3, 4, 2]])
+    assert O.route(z, none, 2, 3, 1)[0] == [3, 2] and O.route(z, none, 4, 3, 2)[0] == [3, 4, 2, 5]
+    ids, w = O.route(z, none - torch.tensor([0, 0, 0, 2.0, 2.0, 0]), 2, 3, 1)  # the correction moves the choice, not the weight
+    assert ids == [2, 3] and torch.allclose(w, s[[2, 3]])
+
+
+def test_oracle_experts_that_are_the_row():
+    h = torch.tensor([[1.0, -2.0]]).double()
+    w = {"router": torch.zeros((3, 2)).double(), "correction": torch.tensor([1.0, 0.0, 2.0]).double(), "e0.up": torch.tensor([[1.0, 0.0], [0.0, 1.0]]).double(),
+         "e0.down": torch.tensor([[1.0, 1.0], [5.0, 1.0]]).double(), "e1.up": torch.zeros((2, 2)).double(), "e1.down": torch.zeros((2, 2)).double()}
+    out = O.experts_ff(w, "", {"router": {"experts": 2, "identity": 1, "top": 2}}, h)
+    assert torch.allclose(out, torch.tensor([[1.0 + 1.0, 5.0 - 2.0]]).double() / 3)
+
+
+def test_oracle_depth_average_and_gate():
+    xs = [torch.full((2, 3), v).double() for v in (1.0, 10.0, 100.0)]
+    assert torch.allclose(O.depth_average(torch.tensor([3.0, 2.0, 1.0]).double(), xs), torch.full((2, 3), 123.0).double())
+    y, h = torch.ones((1, 2)).double(), torch.tensor([[2.0, 0.0]]).double()
+    out = O.gated_result(y, h, torch.tensor([[1.0, 0.0], [0.0, 1.0]]).double(), torch.tensor([0.0, math.log(3)]).double())
+    assert torch.allclose(out, torch.tensor([[1 / (1 + math.exp(-2)), 0.75]]).double())
+
+
+def test_oracle_is_causal_and_mixes_the_first_values():
+    sd = synth.make_hybrid_state_dict(CONFIG)
+    toks = torch.randint(0, 90, (20,), generator=torch.Generator().manual_seed(0)).tolist()
+    a, trail = O.forward(CONFIG, sd, toks)
+    b, _ = O.forward(CONFIG, sd, toks[:11])
+    assert torch.allclose(a[:11], b) and trail.shape == (4, 20, 36)
+    other = {**sd, "l0.mix.vmix": sd["l0.mix.vmix"] + 1}  # (the first layer's factor is not used)
+    assert torch.equal(O.forward(CONFIG, other, toks)[0], a)
+    other = {**sd, "l3.mix.vmix": sd["l3.mix.vmix"] + 1}
+    assert not torch.allclose(O.forward(CONFIG, other, toks)[0], a)
