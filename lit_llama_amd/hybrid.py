@@ -449,7 +449,10 @@ class HybridLM(nn.Module):
         low = {"gla": "a1", "wkv": "w1"}
         rank = {i: sd[n].shape[0] for i, l in enumerate(self.config.layers) for n in (f"l{i}.mix.{low.get(l.mixer.type)}",) if n in sd}
         shapes = tensor_shapes(self.config, {**{i: 0 for i in range(len(self.config.layers))}, **rank})
-        missing, extra = sorted(set(shapes) - set(sd)), sorted(set(sd) - set(shapes))
+        first = self.config.first_values()
+        idle = {f"l{i}.mix.vmix" for i, l in enumerate(self.config.layers) if l.mixer.type == "attention" and (not l.mixer.v_mix or i == first)}
+        shapes = {n: s for n, s in shapes.items() if n not in idle or n in sd}  # (nobody reads these factors: they may be there or not)
+        missing, extra = sorted(set(shapes) - set(sd)), sorted(set(sd) - set(shapes) - idle)
         if missing or (strict and extra):
             raise ValueError(f"checkpoint and configuration differ: missing {missing[:5]}, unexpected {extra[:5]}")
         self._engine = None

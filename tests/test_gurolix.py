@@ -71,10 +71,14 @@ def test_folder_loads_and_is_checked(tmp_path):
     save_file(sd, str(tmp_path / "model.safetensors"))
     m = registry.load_model(tmp_path, torch.float32, "cpu")
     assert isinstance(m, HybridLM) and all(torch.equal(m.tensors[n], t.float()) for n, t in sd.items())
-    for bad in ("missing", "extra", "shape"):
+    spare = {**{n: t for n, t in sd.items() if n != "l0.mix.vmix"}, "l2.mix.vmix": torch.tensor(0.5)}  # (factors that nobody reads may be there or not)
+    registry.build_model(CONFIG, device="cpu").load_state_dict(spare)
+    for bad in ("missing", "missing factor", "extra", "shape"):
         d = dict(sd)
         if bad == "missing":
             del d["l0.mlp.correction"]
+        elif bad == "missing factor":
+            del d["l3.mix.vmix"]
         elif bad == "extra":
             d["l1.norm2"] = torch.zeros(36)
         else:
