@@ -727,16 +727,16 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const ChunkParams p) {
     // ---- output norm over the head's columns (ssd: none), gate
     if constexpr (KIND != MI355_REC_SSD) {
 #pragma unroll
-    for (int rb = 0; rb < 4; ++rb)
+        for (int rb = 0; rb < 4; ++rb)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            float s = 0.f;
+            for (int r = 0; r < 4; ++r) {
+                float s = 0.f;
 #pragma unroll
-            for (int v = 0; v < NV; ++v) s += o[rb][v][r] * o[rb][v][r];
-            s = group_sum(s, 16);
-            if (c16 == 0) ssq[wave][rb * 16 + 4 * g + r] = s;
-        }
-    __syncthreads();
+                for (int v = 0; v < NV; ++v) s += o[rb][v][r] * o[rb][v][r];
+                s = group_sum(s, 16);
+                if (c16 == 0) ssq[wave][rb * 16 + 4 * g + r] = s;
+            }
+        __syncthreads();
     }
     const T* rows = (const T*)a.proj + (int64_t)(p.r.b.row0[seq] + t0) * a.ld;
     out_t<KIND, T>* y = (out_t<KIND, T>*)a.y + (int64_t)(p.r.b.row0[seq] + t0) * a.ldy;

@@ -464,9 +464,12 @@ def build(config, dtype, dev, seed=1):
     from lit_llama_amd.registry import build_model
 
     sd = synth.make_hybrid_state_dict(config, seed=seed)
+    gen = torch.Generator().manual_seed(seed)
     for n in sd:
         if n.endswith("router"):
             sd[n] = (sd[n].float() * 2).to(sd[n].dtype)
+        if n.endswith("correction") and dtype == torch.bfloat16:  # no choice is a rounding apart: every row goes where the restatement sends it
+            sd[n] = (2.0 * torch.randperm(len(sd[n]), generator=gen) - len(sd[n])).to(sd[n].dtype)
     m = build_model(config, dtype, dev)
     m.load_state_dict(sd)
     return m, sd
@@ -477,11 +480,11 @@ def tokens_of(n, vocab=211, seed=0):
 
 
 def close(got, ref, dtype):
-    """float32: every value; bfloat16: rows by their own size (a router may take the other of two experts a rounding apart, which a few rows see)."""
+    """float32: every value; bfloat16: rows (a norm behind a small result multiplies the rounding of a few)."""
     if dtype == torch.float32:
         return rel(got, ref) < 1e-4
     err = (got.double().cpu() - ref).pow(2).mean(-1).sqrt() / ref.pow(2).mean().sqrt()
-    return float(torch.quantile(err, 0.75)) < 0.04 and float(err.mean()) < 0.06
+    return float(torch.quantile(err, 0.97)) < 0.04 and float(err.mean()) < 0.015 and float(err.max()) < 0.3
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
